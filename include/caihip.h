@@ -40,6 +40,7 @@ extern "C" {
 #define CAI_Q4_K   12
 #define CAI_Q5_K   13
 #define CAI_Q6_K   14  /* 210-byte super-blocks (neural/neuralgguf.pas:639-717); resident as aligned ql|qh records + planes of scales and d */
+#define CAI_BF16   30  /* bfloat16 rows, resident with rows padded to 64 columns */
 #define CAI_I8ROW  100  /* per-row symmetric int8 + fp32 row scale (neural/neuralvolume.pas:926-987) */
 
 /* ---- activation opcodes fused into the linear layer (neural/neural.cl:114-146) ---- */
@@ -52,6 +53,10 @@ extern "C" {
 #define CAI_X_DEVICE 1  /* input pointer is device memory (a producer's resident buffer; cf. pExternalVBs, neural/neuralopencl.pas:946) */
 #define CAI_Y_DEVICE 2  /* output pointer is device memory (no read-back; cf. ResultBuffer, neural/neuralopencl.pas:383-388) */
 #define CAI_MATRIX_CORES 4  /* cai_qgemm only: take the matrix-core kernels even for a matrix small enough that the dispatcher would keep it on the vector units */
+
+/* ---- number formats of a layered decoder ---- */
+#define CAI_DTYPE_BF16 0  /* matrix products and the activations between them in bfloat16, sums, norms, states and the residual in 32-bit */
+#define CAI_DTYPE_F32  1  /* everything in 32-bit */
 
 /* ---- KV cache element types ---- */
 #define CAI_KV_F32 0
@@ -279,6 +284,16 @@ int cai_decoder_timeline(cai_decoder_t d, int32_t token, uint64_t* stamps_out, i
  * within tolerance.  last_logits (host, [vocab]) and argmax may be NULL. */
 int cai_decoder_prefill(cai_decoder_t d, int seq, const int32_t* tokens, int n, int pos0,
                         float* last_logits, int32_t* argmax);
+/* One engine step over any mixture of prompt portions and single tokens: entry e feeds counts[e] tokens of sequence seqs[e] (each
+ * sequence at most once) from where that sequence stands; `tokens` holds them one entry after the other.  want (one byte per
+ * token, may be NULL) marks the tokens whose logits come back: logits [wanted][vocab] and argmax [wanted], both host, both may be
+ * NULL, in token order; cai_decoder_candidates and cai_decoder_hidden_state then address the wanted rows by that order.  A layered
+ * decoder runs all entries as one batch; the others batch single tokens of sequences 0 .. n - 1 and take other entries in turn
+ * (and keep only the last pass's rows for cai_decoder_candidates). */
+int cai_decoder_step_batch(cai_decoder_t d, int n_entries, const int32_t* seqs, const int32_t* counts, const int32_t* tokens,
+                           const uint8_t* want, float* logits, int32_t* argmax);
+/* Tokens a sequence can still take before the cache (the shared page pool of a layered decoder) is full. */
+int cai_decoder_room(cai_decoder_t d, int seq, int* tokens_out);
 /* Session management (neural/neuraldecode.pas:5714-5843): always safe after a failed step. */
 /* ---- distribution pipeline ahead of the samplers, on the device ----
  * The non-greedy branch of TChatEngine.GenerateFromIds (neural/neuralchatengine.pas:1374-1396, 1495-1501): RowSoftMax ->
@@ -364,6 +379,11 @@ int cai_gguf_load_qw(cai_gguf_t g, const char* name, const char* bias_name, cai_
  * the decode kernels rotate (neural/neuralgguf.pas:428-438 composed with neural/neuralpretrained.pas:14792-14812
  * is the identity). */
 int cai_decoder_load_gguf(const char* path, int max_ctx, int max_batch, int kv_dtype, cai_decoder_t* out);
+/* Model registry: `path` is a folder with config.json and model.safetensors, loaded by the builder registered under the
+ * configuration's "architecture" (Samanex), or a GGUF file (cai_decoder_load_gguf).  max_tokens is the size of the cache pool:
+ * the tokens all live sequences may hold together, each count rounded up to whole pages of 64 (a GGUF decoder keeps max_tokens
+ * rows for every sequence); max_seq the sequences (state slots).  dtype: CAI_DTYPE_BF16 or CAI_DTYPE_F32. */
+int cai_decoder_load(const char* path, int max_tokens, int max_seq, int dtype, cai_decoder_t* out);
 
 #ifdef __cplusplus
 }

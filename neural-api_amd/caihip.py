@@ -6,7 +6,8 @@ import numpy as np
 
 from . import lib_path
 
-F32, F16, Q4_0, Q8_0, Q4_K, Q6_K, I8ROW = 0, 1, 2, 8, 12, 14, 100
+F32, F16, Q4_0, Q8_0, Q4_K, Q6_K, BF16, I8ROW = 0, 1, 2, 8, 12, 14, 30, 100
+DTYPE_BF16, DTYPE_F32 = 0, 1
 Q4_1, Q5_0, Q5_1, Q2_K, Q3_K, Q5_K = 3, 6, 7, 10, 11, 13
 ACT_NONE, ACT_RELU, ACT_SIGMOID, ACT_TANH = 0, 1, 2, 3
 ROPE_NONE, ROPE_LINEAR, ROPE_LLAMA3, ROPE_NTK, ROPE_YARN = 0, 1, 2, 3, 4
@@ -23,7 +24,7 @@ cai_rmsnorm cai_rope cai_swiglu cai_argmax cai_argmax_noalloc cai_router_topk
 cai_kv_create cai_kv_destroy cai_kv_reset cai_kv_truncate cai_kv_len cai_kv_snapshot cai_kv_restore cai_kv_snap_destroy cai_kv_export_layer cai_kv_import_layer cai_kv_set_eviction cai_kv_rows cai_attn_decode
 cai_decoder_create cai_decoder_destroy cai_decoder_set_weight cai_decoder_set_vector cai_decoder_step cai_decoder_hidden_state cai_decoder_step_window cai_prompt_lookup_draft cai_decoder_generate_lookup cai_decoder_generate cai_decoder_profile cai_decoder_timeline
 cai_decoder_prefill cai_decoder_reset cai_decoder_truncate cai_decoder_len cai_decoder_set_eviction cai_decoder_cache_rows cai_decoder_set_kv_dtype cai_decoder_set_rope_scaling cai_decoder_set_rope_freq_factors cai_decoder_set_rope_out_scale cai_sample_candidates cai_decoder_candidates cai_decoder_snapshot cai_decoder_restore cai_decoder_fork
-cai_decoder_weight_bytes cai_decoder_get_config cai_decoder_load_gguf
+cai_decoder_weight_bytes cai_decoder_get_config cai_decoder_load_gguf cai_decoder_load cai_decoder_step_batch cai_decoder_room
 cai_gguf_open cai_gguf_close cai_gguf_info cai_gguf_meta_int cai_gguf_meta_float cai_gguf_meta_str cai_gguf_meta_array_count
 cai_gguf_meta_array_str cai_gguf_find_tensor cai_gguf_tensor_info cai_gguf_tensor_data cai_gguf_load_qw""".split()
 
@@ -127,6 +128,9 @@ def load():
         L.cai_decoder_weight_bytes.argtypes = [vp, C.POINTER(i64)]
         L.cai_decoder_get_config.argtypes = [vp, C.POINTER(DecoderConfig)]
         L.cai_decoder_load_gguf.argtypes = [C.c_char_p, i32, i32, i32, C.POINTER(vp)]
+        L.cai_decoder_load.argtypes = [C.c_char_p, i32, i32, i32, C.POINTER(vp)]
+        L.cai_decoder_step_batch.argtypes = [vp, i32, vp, vp, vp, vp, vp, vp]
+        L.cai_decoder_room.argtypes = [vp, i32, C.POINTER(i32)]
         L.cai_gguf_open.argtypes = [C.c_char_p, C.POINTER(vp)]
         L.cai_gguf_close.argtypes = [vp]
         L.cai_gguf_info.argtypes = [vp, C.POINTER(i32), C.POINTER(i32), C.POINTER(i64), C.POINTER(i64), C.POINTER(i64)]
@@ -404,6 +408,16 @@ class Decoder:
         check(load().cai_decoder_get_config(self.h, C.byref(self.cfg)))
         return self
 
+    @classmethod
+    def load(cls, path, max_tokens, max_seq=1, dtype=DTYPE_BF16):
+        """a model folder (config.json, model.safetensors) or a GGUF file through the library's registry (cai_decoder_load)"""
+        self = cls.__new__(cls)
+        self.h = C.c_void_p(); self.weights = []
+        check(load().cai_decoder_load(os.fsencode(path), max_tokens, max_seq, dtype, C.byref(self.h)))
+        self.cfg = DecoderConfig()
+        check(load().cai_decoder_get_config(self.h, C.byref(self.cfg)))
+        return self
+
     def __init__(self, spec, max_batch=1, kv_dtype=KV_F32, max_ctx=None):
         c = spec["cfg"]
         self.cfg = DecoderConfig(n_layers=c["n_layers"], d_model=c["d_model"], n_q_heads=c["n_q_heads"], n_kv_heads=c["n_kv_heads"],
@@ -429,6 +443,31 @@ class Decoder:
         am = np.empty(nb, np.int32)
         check(load().cai_decoder_step(self.h, _ptr(tokens), _ptr(pos), nb, _ptr(lg), _ptr(am)))
         return am, lg
+
+    def step_batch(self, entries, want_logits=True):
+        """one engine step: entries = [(sequence, tokens, places whose logits are wanted)]; returns (argmax, logits) of the wanted
+        rows in the order of the entries, each entry's places ascending"""
+        seqs = np.array([e[0] for e in entries], np.int32)
+        counts = np.array([len(e[1]) for e in entries], np.int32)
+        tokens = np.concatenate([np.asarray(e[1], np.int32) for e in entries])
+        want = np.zeros(tokens.size, np.uint8)
+        r0 = 0
+        for e, n in zip(entries, counts):
+            for w in e[2]:
+                if not 0 <= w < n:
+                    raise ValueError("place %d of an entry of %d tokens" % (w, n))
+                want[r0 + w] = 1
+            r0 += int(n)
+        k = int(want.sum())
+        lg = np.empty((k, self.cfg.vocab), np.float32) if want_logits else None
+        am = np.empty(k, np.int32)
+        check(load().cai_decoder_step_batch(self.h, len(entries), _ptr(seqs), _ptr(counts), _ptr(tokens), _ptr(want), _ptr(lg), _ptr(am)))
+        return am, lg
+
+    def room(self, seq=0):
+        n = C.c_int32()
+        check(load().cai_decoder_room(self.h, seq, C.byref(n)))
+        return n.value
 
     def generate(self, first_token, pos, n):
         out = np.empty(n, np.int32)

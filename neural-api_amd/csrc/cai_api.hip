@@ -1,5 +1,5 @@
 // Library lifetime, error reporting, device buffers and resident weight matrices.
-#include "cai_internal.hpp"
+#include "cai_layered.hpp"
 
 #include <stdarg.h>
 #include <string.h>
@@ -62,13 +62,13 @@ int ensure_stage(void** p, size_t* cap, size_t need)
 
 int64_t block_elems(int qt)
 {
-  switch (qt) { case CAI_F32: case CAI_F16: case CAI_I8ROW: return 1; case CAI_Q4_0: case CAI_Q8_0: return 32; case CAI_Q4_K: case CAI_Q6_K: return 256; }
+  switch (qt) { case CAI_F32: case CAI_F16: case CAI_BF16: case CAI_I8ROW: return 1; case CAI_Q4_0: case CAI_Q8_0: return 32; case CAI_Q4_K: case CAI_Q6_K: return 256; }
   if (raw_block_type(qt)) return raw_block_elems(qt);
   return -1;
 }
 int64_t block_bytes(int qt)
 {
-  switch (qt) { case CAI_F32: return 4; case CAI_F16: return 2; case CAI_I8ROW: return 1; case CAI_Q4_0: return 18; case CAI_Q8_0: return 34; case CAI_Q4_K: return 144; case CAI_Q6_K: return 210; }
+  switch (qt) { case CAI_F32: return 4; case CAI_F16: case CAI_BF16: return 2; case CAI_I8ROW: return 1; case CAI_Q4_0: return 18; case CAI_Q8_0: return 34; case CAI_Q4_K: return 144; case CAI_Q6_K: return 210; }
   if (raw_block_type(qt)) return raw_block_bytes(qt);
   return -1;
 }
@@ -115,7 +115,7 @@ extern "C" int cai_shutdown(void)
   if (c.stage_in) (void)hipFree(c.stage_in);
   if (c.stage_out) (void)hipFree(c.stage_out);
   if (c.stage_sample) (void)hipFree(c.stage_sample);
-  nb_release(); ra_release(); prefill_release();
+  nb_release(); ra_release(); prefill_release(); bf16_release();
   if (c.d_small) (void)hipFree(c.d_small);
   if (c.h_small) (void)hipHostFree(c.h_small);
   if (c.tl.buf) (void)hipFree(c.tl.buf);
@@ -258,6 +258,14 @@ extern "C" int cai_qw_create(int qtype, int64_t rows, int64_t cols, const void* 
     if (e == hipSuccess) { launch_split_q6k((const uint8_t*)raw, n_blocks, w->data, w->aux, (uint16_t*)(w->aux + n_blocks * 16)); e = hipStreamSynchronize(c.stream); }
     (void)hipFree(raw);
     if (e != hipSuccess) return fail(hip_fail(e, "cai_qw_create upload", __FILE__, __LINE__));
+  } else if (qtype == CAI_BF16) {
+    w->ld = (cols + LIN_PAD - 1) / LIN_PAD * LIN_PAD;
+    w->data_bytes = rows * w->ld * 2;
+    hipError_t e = hipMalloc((void**)&w->data, (size_t)w->data_bytes);
+    if (e == hipSuccess && w->ld != cols) e = hipMemsetAsync(w->data, 0, (size_t)w->data_bytes, c.stream);
+    if (e == hipSuccess) e = hipMemcpy2DAsync(w->data, (size_t)w->ld * 2, blocks, (size_t)cols * 2, (size_t)cols * 2, (size_t)rows, hipMemcpyDefault, c.stream);
+    if (e == hipSuccess) e = hipStreamSynchronize(c.stream);
+    if (e != hipSuccess) return fail(hip_fail(e, "cai_qw_create upload", __FILE__, __LINE__));
   } else {
     w->data_bytes = raw_bytes;
     hipError_t e = hipMalloc((void**)&w->data, (size_t)raw_bytes);
@@ -346,7 +354,8 @@ extern "C" int cai_qgemv(cai_qw_t w, const float* x, int n_b, float* y, int act,
   if (!(flags & CAI_Y_DEVICE)) { if ((rc = ensure_stage(&c.stage_out, &c.stage_out_cap, yb))) return rc; dy = (float*)c.stage_out; }
   // A batch on a matrix too large for the cache: the VALU kernel would be compute-bound, the matrix-core kernel streams
   // the weights once for the batch.  Small matrices stay on the single-launch kernel (three launches cost more there).
-  if (n_b >= 2 && act == CAI_ACT_NONE && nb_supported(w) && w->data_bytes >= ((int64_t)16 << 20)) {
+  if (w->qtype == CAI_BF16) { if ((rc = bf16_linear_f32(w, dx, w->cols, n_b, dy, w->rows, act))) return rc; }
+  else if (n_b >= 2 && act == CAI_ACT_NONE && nb_supported(w) && w->data_bytes >= ((int64_t)16 << 20)) {
     if ((rc = nb_linear(w, dx, w->cols, nullptr, 0.0f, n_b, dy, w->rows, nullptr))) return rc;
   } else if ((rc = launch_gemv(w, 0, w->rows, dx, n_b, dy, w->rows, act, nullptr))) return rc;
   CAI_HIP(hipGetLastError());

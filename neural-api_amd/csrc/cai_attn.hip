@@ -2026,6 +2026,7 @@ extern "C" int cai_kv_snap_destroy(cai_kv_snap_t s)
 {
   CAI_ENTER();
   if (!s) return CAI_OK;
+  if (s->net) net_snap_free(s->net);
   if (s->k) (void)hipFree(s->k);
   if (s->v) (void)hipFree(s->v);
   if (s->ks) (void)hipFree(s->ks);

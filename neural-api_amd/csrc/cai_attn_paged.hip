@@ -1,0 +1,444 @@
+// Sliding-window grouped-query attention over a paged key/value pool: key and value widths of their own, optional per-head RMS
+// norm of queries and keys, an explicit score scale, no rotation.
+//
+// Two forms: one work-group per (row, key/value head, slice of keys) for decoded tokens, short portions and the all-32-bit mode,
+// and a matrix-core form for prompts, whose key tile is one page.  Scores, soft-max and weights are 32-bit in both; the
+// matrix-core form hands its float weights to the value product as three bfloat16 parts that add up to all 24 bits.
+#include "cai_layered.hpp"
+#include "cai_gemv_common.hpp"
+
+#include <algorithm>
+
+namespace cai {
+
+constexpr int SLICE = 256;                 // keys per work-group of the row form
+
+template <typename T> __device__ __forceinline__ float round_to(float v) { return (float)(T)v; }
+template <typename T> __device__ __forceinline__ void load8(const T* p, float* v)
+{
+  if constexpr (sizeof(T) == 2) {
+    const u32x4 u = *reinterpret_cast<const u32x4*>(p);
+#pragma unroll
+    for (int j = 0; j < 4; j++) { v[2 * j] = bf16_lo(u[j]); v[2 * j + 1] = bf16_hi(u[j]); }
+  } else {
+    const f32x4 a = *reinterpret_cast<const f32x4*>(p), c = *reinterpret_cast<const f32x4*>(p + 4);
+#pragma unroll
+    for (int j = 0; j < 4; j++) { v[j] = a[j]; v[4 + j] = c[j]; }
+  }
+}
+template <typename T> __device__ __forceinline__ T* kv_page(const KvView& kv, int slot, int key)
+{
+  return reinterpret_cast<T*>(kv.base) + (int64_t)kv.table[slot * kv.ring + (key / PAGE_TOKENS) % kv.ring] * kv.page_elems;
+}
+
+// RMS norm of a head of `dim` values by one wave: lane holds x[lane + 64 i]
+__device__ __forceinline__ void head_norm(const float* x, const float* gain, int dim, float eps, int lane, float* v)
+{
+  float s = 0.0f;
+#pragma unroll
+  for (int i = 0; i < 4; i++) { const int c = lane + 64 * i; v[i] = c < dim ? x[c] : 0.0f; s = fmaf(v[i], v[i], s); }
+  if (!gain) return;
+  s = wave_sum(s);
+  const float inv = 1.0f / sqrtf(__builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, s), 63)) / (float)dim + eps);
+#pragma unroll
+  for (int i = 0; i < 4; i++) { const int c = lane + 64 * i; if (c < dim) v[i] *= inv * gain[c]; }
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void attn_prep_kernel(const AttnDims d, const KvView kv, const AttnIn in, const StepRows r, T* qbuf)
+{
+  const int row = blockIdx.x, lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+  const int pos = r.pos[row], slot = r.slot[row], tp = pos % PAGE_TOKENS;
+  const float* p = in.proj + row * in.ldp;
+  T* page = kv_page<T>(kv, slot, pos);
+  for (int u = wave; u < d.heads + d.kv_heads; u += 4) {
+    const bool is_q = u < d.heads; const int hh = is_q ? u : u - d.heads;
+    float v[4];
+    head_norm(p + (is_q ? in.oq : in.ok) + hh * d.dim, is_q ? in.qn : in.kn, d.dim, d.eps, lane, v);
+    T* dst = is_q ? qbuf + ((int64_t)row * d.heads + hh) * d.dim_p : page + ((int64_t)hh * PAGE_TOKENS + tp) * d.dim_p;
+#pragma unroll
+    for (int i = 0; i < 4; i++) { const int c = lane + 64 * i; if (c < d.dim_p) dst[c] = (T)v[i]; }
+  }
+  for (int c = threadIdx.x; c < d.kv_heads * d.vdim_p; c += 256) {
+    const int hh = c / d.vdim_p, i = c % d.vdim_p;
+    page[kv.v_off + ((int64_t)hh * PAGE_TOKENS + tp) * d.vdim_p + i] = (T)(i < d.vdim ? p[in.ov + hh * d.vdim + i] : 0.0f);
+  }
+}
+
+// ------------------------------------------------------------------------------------------
+// Row form.  blockIdx: x slice, y = key/value head x group of HT query heads, z row.  SINGLE: the row is its entry's only one;
+// queries, the new key and the new value come from the projections and the new key/value are appended on the way.
+// part (more than one slice): per (row, head, slice) vdim_p weighted sums, the maximum and the normaliser.
+// ------------------------------------------------------------------------------------------
+template <typename T, int HT, bool SINGLE>
+__global__ __launch_bounds__(256) void attn_rows_kernel(const AttnDims d, const KvView kv, const AttnIn in, const StepRows r, const T* qbuf, T* out, const int64_t ldo, float* part)
+{
+  __shared__ float sq[HT][256], nk[256], nv[256];
+  __shared__ float sc[HT][SLICE];
+  __shared__ float red[4][HT][256];
+  __shared__ float smax[HT], ssum[HT];
+  const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int hg = d.heads / d.kv_heads, hblk = (hg + HT - 1) / HT;
+  const int row = blockIdx.z, g = blockIdx.y / hblk, h0 = g * hg + blockIdx.y % hblk * HT, nh = min(HT, (g + 1) * hg - h0);
+  const int pos = r.pos[row], slot = r.slot[row];
+  const int lo = max(0, pos - d.window + 1), k0 = lo + blockIdx.x * SLICE, nkeys = min(SLICE, pos + 1 - k0);
+  const int n_sl = gridDim.x;
+  if (nkeys <= 0) {                        // (part is only read up to the slices in use)
+    return;
+  }
+  const bool own_new = SINGLE && k0 + nkeys == pos + 1;
+  if (SINGLE) {
+    const float* p = in.proj + row * in.ldp;
+    for (int u = wave; u < nh + (own_new ? 1 : 0); u += 4) {
+      float v[4];
+      const bool is_q = u < nh;
+      head_norm(is_q ? p + in.oq + (h0 + u) * d.dim : p + in.ok + g * d.dim, is_q ? in.qn : in.kn, d.dim, d.eps, lane, v);
+      float* dst = is_q ? sq[u] : nk;
+#pragma unroll
+      for (int i = 0; i < 4; i++) dst[lane + 64 * i] = is_q ? v[i] : round_to<T>(v[i]);
+    }
+    if (own_new) for (int c = tid; c < 256; c += 256) nv[c] = c < d.vdim ? round_to<T>(p[in.ov + g * d.vdim + c]) : 0.0f;
+  } else {
+    for (int i = tid; i < nh * 256; i += 256) {
+      const int hh = i >> 8, c = i & 255;
+      sq[hh][c] = c < d.dim_p ? (float)qbuf[((int64_t)row * d.heads + h0 + hh) * d.dim_p + c] : 0.0f;
+    }
+  }
+  __syncthreads();
+  if (own_new && blockIdx.y % hblk == 0) {
+    T* page = kv_page<T>(kv, slot, pos);
+    const int tp = pos % PAGE_TOKENS;
+    for (int c = tid; c < d.dim_p; c += 256) page[((int64_t)g * PAGE_TOKENS + tp) * d.dim_p + c] = (T)nk[c];
+    for (int c = tid; c < d.vdim_p; c += 256) page[kv.v_off + ((int64_t)g * PAGE_TOKENS + tp) * d.vdim_p + c] = (T)nv[c];
+  }
+  // scores: sixteen lanes a key, eight elements a lane and turn
+  const int l16 = lane & 15;
+  for (int kb = wave * 4 + (lane >> 4); kb < ((nkeys + 63) & ~63); kb += 64) {      // four keys of each lane group at a time: their loads are in flight together
+    float kx[4][2][8];
+#pragma unroll
+    for (int u = 0; u < 4; u++) {
+      const int kk = min(kb + 16 * u, nkeys - 1), key = k0 + kk;
+      const bool fresh = SINGLE && key == pos;
+      const T* kp = kv_page<T>(kv, slot, key) + ((int64_t)g * PAGE_TOKENS + key % PAGE_TOKENS) * d.dim_p;
+#pragma unroll
+      for (int t = 0; t < 2; t++) {
+        const int c = l16 * 8 + t * 128;
+        if (t && d.dim_p <= 128) continue;
+        if (fresh) {
+#pragma unroll
+          for (int i = 0; i < 8; i++) kx[u][t][i] = nk[c + i];
+        } else if (c < d.dim_p) load8<T>(kp + c, kx[u][t]);
+        else {
+#pragma unroll
+          for (int i = 0; i < 8; i++) kx[u][t][i] = 0.0f;
+        }
+      }
+    }
+#pragma unroll
+    for (int hh = 0; hh < HT; hh++) {
+      if (hh >= nh) break;
+      float s[4] = {0.0f, 0.0f, 0.0f, 0.0f};
+#pragma unroll
+      for (int t = 0; t < 2; t++) {
+        if (t && d.dim_p <= 128) continue;
+        float q[8];
+        *reinterpret_cast<f32x4*>(q) = *reinterpret_cast<const f32x4*>(&sq[hh][l16 * 8 + t * 128]);
+        *reinterpret_cast<f32x4*>(q + 4) = *reinterpret_cast<const f32x4*>(&sq[hh][l16 * 8 + t * 128 + 4]);
+#pragma unroll
+        for (int u = 0; u < 4; u++)
+#pragma unroll
+          for (int i = 0; i < 8; i++) s[u] = fmaf(q[i], kx[u][t][i], s[u]);
+      }
+#pragma unroll
+      for (int u = 0; u < 4; u++) {
+        s[u] += __shfl_xor(s[u], 8); s[u] += __shfl_xor(s[u], 4); s[u] += __shfl_xor(s[u], 2); s[u] += __shfl_xor(s[u], 1);
+        const int kk = kb + 16 * u;
+        if (l16 == 0) sc[hh][kk] = s[u] * d.scale;
+      }
+    }
+  }
+  __syncthreads();
+  // soft-max over the slice, a wave per head
+  for (int hh = wave; hh < nh; hh += 4) {
+    float v[SLICE / 64], m = -INFINITY;
+#pragma unroll
+    for (int i = 0; i < SLICE / 64; i++) { v[i] = lane + 64 * i < nkeys ? sc[hh][lane + 64 * i] : -INFINITY; m = fmaxf(m, v[i]); }
+#pragma unroll
+    for (int o = 32; o; o >>= 1) m = fmaxf(m, __shfl_xor(m, o));
+    float s = 0.0f;
+#pragma unroll
+    for (int i = 0; i < SLICE / 64; i++) { v[i] = expf(v[i] - m); s += v[i]; sc[hh][lane + 64 * i] = v[i]; }
+#pragma unroll
+    for (int o = 32; o; o >>= 1) s += __shfl_xor(s, o);
+    if (lane == 0) { smax[hh] = m; ssum[hh] = s; }
+  }
+  __syncthreads();
+  // weighted values: CB lanes along the columns (eight each), the rest of the work-group along the keys
+  const int chunks = d.vdim_p / 8;
+  int cb_log = 0; while ((1 << cb_log) < chunks) cb_log++;
+  const int cbl = 1 << cb_log, cc = tid & (cbl - 1), kg = tid >> cb_log, nkg = 256 >> cb_log;
+  float acc[HT][8];
+#pragma unroll
+  for (int hh = 0; hh < HT; hh++)
+#pragma unroll
+    for (int i = 0; i < 8; i++) acc[hh][i] = 0.0f;
+  if (cc < chunks) {
+    for (int kb = kg; kb < nkeys; kb += nkg * 4) {
+      float vx[4][8];
+#pragma unroll
+      for (int u = 0; u < 4; u++) {
+        const int key = k0 + min(kb + nkg * u, nkeys - 1);
+        if (SINGLE && key == pos) {
+#pragma unroll
+          for (int i = 0; i < 8; i++) vx[u][i] = nv[cc * 8 + i];
+        } else load8<T>(kv_page<T>(kv, slot, key) + kv.v_off + ((int64_t)g * PAGE_TOKENS + key % PAGE_TOKENS) * d.vdim_p + cc * 8, vx[u]);
+      }
+#pragma unroll
+      for (int hh = 0; hh < HT; hh++) {
+        if (hh >= nh) break;
+#pragma unroll
+        for (int u = 0; u < 4; u++) {
+          const int kk = kb + nkg * u;
+          const float p = kk < nkeys ? sc[hh][kk] : 0.0f;
+#pragma unroll
+          for (int i = 0; i < 8; i++) acc[hh][i] = fmaf(p, vx[u][i], acc[hh][i]);
+        }
+      }
+    }
+  }
+#pragma unroll
+  for (int hh = 0; hh < HT; hh++) {
+    if (hh >= nh) break;
+    for (int o = cbl; o < 64; o <<= 1)
+#pragma unroll
+      for (int i = 0; i < 8; i++) acc[hh][i] += __shfl_xor(acc[hh][i], o);
+    if (lane < cbl && cc < chunks) {
+      *reinterpret_cast<f32x4*>(&red[wave][hh][cc * 8]) = f32x4{acc[hh][0], acc[hh][1], acc[hh][2], acc[hh][3]};
+      *reinterpret_cast<f32x4*>(&red[wave][hh][cc * 8 + 4]) = f32x4{acc[hh][4], acc[hh][5], acc[hh][6], acc[hh][7]};
+    }
+  }
+  __syncthreads();
+  for (int i = tid; i < nh * d.vdim_p; i += 256) {
+    const int hh = i / d.vdim_p, c = i % d.vdim_p;
+    const float s = red[0][hh][c] + red[1][hh][c] + red[2][hh][c] + red[3][hh][c];
+    if (n_sl == 1) { if (c < d.vdim) out[row * ldo + (h0 + hh) * d.vdim + c] = (T)(s / ssum[hh]); }
+    else part[(((int64_t)row * d.heads + h0 + hh) * n_sl + blockIdx.x) * (d.vdim_p + 2) + c] = s;
+  }
+  if (n_sl > 1 && tid < nh) {
+    float* q = part + (((int64_t)row * d.heads + h0 + tid) * n_sl + blockIdx.x) * (d.vdim_p + 2) + d.vdim_p;
+    q[0] = smax[tid]; q[1] = ssum[tid];
+  }
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void attn_rows_merge_kernel(const AttnDims d, const StepRows r, const int n_sl, const float* part, T* out, const int64_t ldo)
+{
+  const int h = blockIdx.x, row = blockIdx.y, pos = r.pos[row];
+  const int used = (min(d.window, pos + 1) + SLICE - 1) / SLICE, st = d.vdim_p + 2;
+  const float* p = part + ((int64_t)row * d.heads + h) * n_sl * st;
+  float m = -INFINITY, l = 0.0f;
+  for (int s = 0; s < used; s++) m = fmaxf(m, p[s * st + d.vdim_p]);
+  for (int s = 0; s < used; s++) l += p[s * st + d.vdim_p + 1] * expf(p[s * st + d.vdim_p] - m);
+  const int c = threadIdx.x;
+  if (c >= d.vdim) return;
+  float o = 0.0f;
+  for (int s = 0; s < used; s++) o = fmaf(p[s * st + c], expf(p[s * st + d.vdim_p] - m), o);
+  out[row * ldo + h * d.vdim + c] = (T)(o / l);
+}
+
+// ------------------------------------------------------------------------------------------
+// Prompt form: 64 query rows of one entry and one head per work-group, a wave per 16 rows; a key tile is a page.
+// S^T = K Q^T puts a query in a lane column, so its soft-max state is per lane; the score registers are the B operand of
+// O^T = V^T P^T as they are: key slot (lane group g, j) of a 32-key step is key 4 g + j of its first 16 keys for j < 4 and
+// 4 g + j - 4 of its second 16 otherwise, and V^T is read from LDS in that order.
+// ------------------------------------------------------------------------------------------
+template <int KQ, int VQ>                  // key width in 32s, value width in 16s
+__global__ __launch_bounds__(256) void attn_prompt_paged_kernel(const AttnDims d, const KvView kv, const bf16_t* qbuf, const StepRows r, const int32_t* tiles, bf16_t* out, const int64_t ldo)
+{
+  constexpr int KST = KQ * 32 + 8, VST = PAGE_TOKENS + 4;
+  __shared__ __align__(16) uint16_t sk[PAGE_TOKENS * KST];
+  __shared__ __align__(16) uint16_t sv[VQ * 16 * VST];
+  const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), fr = lane & 15, fg = lane >> 4;
+  const int32_t* en = r.ent + 4 * tiles[2 * blockIdx.x];
+  const int slot = en[0], row0 = en[1], n = en[2], pos0 = en[3], t0 = tiles[2 * blockIdx.x + 1];
+  const int h = blockIdx.y, g = h / (d.heads / d.kv_heads);
+  const int qi = t0 + wave * 16 + fr, qr = min(qi, n - 1), qpos = pos0 + qr;
+  u32x4 fq[KQ];
+#pragma unroll
+  for (int k = 0; k < KQ; k++) {
+    const int c = k * 32 + fg * 8;
+    fq[k] = u32x4{0, 0, 0, 0};
+    if (c < d.dim_p) fq[k] = *reinterpret_cast<const u32x4*>(qbuf + ((int64_t)(row0 + qr) * d.heads + h) * d.dim_p + c);
+  }
+  f32x4 o[VQ];
+#pragma unroll
+  for (int v = 0; v < VQ; v++) o[v] = f32x4{0.0f, 0.0f, 0.0f, 0.0f};
+  float m = -INFINITY, l = 0.0f;
+  const int first = max(0, pos0 + t0 - d.window + 1) / PAGE_TOKENS, last = (pos0 + min(t0 + ATTN_TILE, n) - 1) / PAGE_TOKENS;
+  const int wlo = max(0, pos0 + min(t0 + wave * 16, n - 1) - d.window + 1), whi = pos0 + min(t0 + wave * 16 + 15, n - 1);   // keys this wave's rows see
+  constexpr int KC = PAGE_TOKENS * KQ * 4 / 256, VC = PAGE_TOKENS / 2 * VQ * 2 / 256;   // 16-byte key chunks / value chunk pairs per thread
+  u32x4 rk[KC], rv[VC][2];
+  auto fetch = [&](int pg) {
+    const bf16_t* page = kv_page<bf16_t>(kv, slot, pg * PAGE_TOKENS);
+#pragma unroll
+    for (int i = 0; i < KC; i++) {
+      const int e = tid + 256 * i, t = e / (KQ * 4), c = e % (KQ * 4) * 8;
+      rk[i] = u32x4{0, 0, 0, 0};
+      if (c < d.dim_p) rk[i] = *reinterpret_cast<const u32x4*>(page + ((int64_t)g * PAGE_TOKENS + t) * d.dim_p + c);
+    }
+#pragma unroll
+    for (int i = 0; i < VC; i++) {
+      const int e = tid + 256 * i, t = e / (VQ * 2) * 2, c = e % (VQ * 2) * 8;
+      rv[i][0] = rv[i][1] = u32x4{0, 0, 0, 0};
+      if (c < d.vdim_p) {
+        const bf16_t* vp = page + kv.v_off + ((int64_t)g * PAGE_TOKENS + t) * d.vdim_p + c;
+        rv[i][0] = *reinterpret_cast<const u32x4*>(vp); rv[i][1] = *reinterpret_cast<const u32x4*>(vp + d.vdim_p);
+      }
+    }
+  };
+  const int end = pos0 + n;                // keys at and past it are not written yet: their page rows may hold anything
+  fetch(first);
+  for (int pg = first; pg <= last; pg++) {
+    __syncthreads();
+#pragma unroll
+    for (int i = 0; i < KC; i++) {
+      const int e = tid + 256 * i, t = e / (KQ * 4), c = e % (KQ * 4) * 8;
+      *reinterpret_cast<u32x4*>(sk + t * KST + c) = rk[i];
+    }
+#pragma unroll
+    for (int i = 0; i < VC; i++) {
+      const int e = tid + 256 * i, t = e / (VQ * 2) * 2, c = e % (VQ * 2) * 8;
+      const bool k0 = pg * PAGE_TOKENS + t < end, k1 = pg * PAGE_TOKENS + t + 1 < end;
+#pragma unroll
+      for (int j = 0; j < 4; j++) {
+        const uint32_t a = k0 ? rv[i][0][j] : 0, b = k1 ? rv[i][1][j] : 0;
+        *reinterpret_cast<uint32_t*>(sv + (c + 2 * j) * VST + t) = (a & 0xffffu) | (b << 16);
+        *reinterpret_cast<uint32_t*>(sv + (c + 2 * j + 1) * VST + t) = (a >> 16) | (b & 0xffff0000u);
+      }
+    }
+    __syncthreads();
+    if (pg < last) fetch(pg + 1);
+    if (pg * PAGE_TOKENS > whi || pg * PAGE_TOKENS + PAGE_TOKENS - 1 < wlo) continue;    // (the whole wave: its rows see nothing of this page)
+    f32x4 s[4];
+#pragma unroll
+    for (int t = 0; t < 4; t++) {
+      s[t] = f32x4{0.0f, 0.0f, 0.0f, 0.0f};
+#pragma unroll
+      for (int k = 0; k < KQ; k++) {
+        const u32x4 a = *reinterpret_cast<const u32x4*>(sk + (t * 16 + fr) * KST + k * 32 + fg * 8);
+        s[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, a), __builtin_bit_cast(bf16x8, fq[k]), s[t], 0, 0, 0);
+      }
+    }
+    float mt = -INFINITY;
+#pragma unroll
+    for (int t = 0; t < 4; t++)
+#pragma unroll
+      for (int i = 0; i < 4; i++) {
+        const int back = qpos - (pg * PAGE_TOKENS + t * 16 + fg * 4 + i);
+        s[t][i] = back >= 0 && back < d.window ? s[t][i] * d.scale : -INFINITY;
+        mt = fmaxf(mt, s[t][i]);
+      }
+    mt = fmaxf(mt, __shfl_xor(mt, 16)); mt = fmaxf(mt, __shfl_xor(mt, 32));
+    const float mn = fmaxf(m, mt), mr = mn == -INFINITY ? 0.0f : mn, al = expf(m - mr);
+    m = mn; l *= al;
+#pragma unroll
+    for (int v = 0; v < VQ; v++) o[v] *= al;
+    // weights in three bfloat16 parts: p = p0 + p1 + p2 exactly
+    uint16_t w[3][16];
+#pragma unroll
+    for (int t = 0; t < 4; t++)
+#pragma unroll
+      for (int i = 0; i < 4; i++) {
+        const float p = expf(s[t][i] - mr);
+        l += p;
+        const float a = __builtin_bit_cast(float, __builtin_bit_cast(uint32_t, p) & 0xffff0000u), pr = p - a;
+        const float b = __builtin_bit_cast(float, __builtin_bit_cast(uint32_t, pr) & 0xffff0000u);
+        w[0][t * 4 + i] = (uint16_t)(__builtin_bit_cast(uint32_t, a) >> 16);
+        w[1][t * 4 + i] = (uint16_t)(__builtin_bit_cast(uint32_t, b) >> 16);
+        w[2][t * 4 + i] = bf16_bits(pr - b);
+      }
+#pragma unroll
+    for (int hp = 0; hp < 2; hp++) {
+      u32x4 fp[3];
+#pragma unroll
+      for (int q = 0; q < 3; q++)
+#pragma unroll
+        for (int j = 0; j < 4; j++) fp[q][j] = w[q][hp * 8 + 2 * j] | (uint32_t)w[q][hp * 8 + 2 * j + 1] << 16;
+#pragma unroll
+      for (int v = 0; v < VQ; v++) {
+        const uint16_t* vr = sv + (v * 16 + fr) * VST + hp * 32 + fg * 4;
+        const uint2 lo2 = *reinterpret_cast<const uint2*>(vr), hi2 = *reinterpret_cast<const uint2*>(vr + 16);
+        const u32x4 a = {lo2.x, lo2.y, hi2.x, hi2.y};
+#pragma unroll
+        for (int q = 0; q < 3; q++) o[v] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, a), __builtin_bit_cast(bf16x8, fp[q]), o[v], 0, 0, 0);
+      }
+    }
+  }
+  l += __shfl_xor(l, 16); l += __shfl_xor(l, 32);
+  if (qi < n) {
+    const float inv = 1.0f / l;
+#pragma unroll
+    for (int v = 0; v < VQ; v++)
+#pragma unroll
+      for (int i = 0; i < 4; i++) {
+        const int c = v * 16 + fg * 4 + i;
+        if (c < d.vdim) out[(int64_t)(row0 + qi) * ldo + h * d.vdim + c] = (bf16_t)(o[v][i] * inv);
+      }
+  }
+}
+
+int attn_paged_prep(const AttnDims& d, const KvView& kv, int act_t, const AttnIn& in, const StepRows& r, void* qbuf)
+{
+  if (act_t == ACT_T_BF16) hipLaunchKernelGGL(attn_prep_kernel<bf16_t>, dim3(r.n_rows), dim3(256), 0, ctx().stream, d, kv, in, r, (bf16_t*)qbuf);
+  else hipLaunchKernelGGL(attn_prep_kernel<float>, dim3(r.n_rows), dim3(256), 0, ctx().stream, d, kv, in, r, (float*)qbuf);
+  CAI_HIP(hipGetLastError());
+  return CAI_OK;
+}
+
+static int n_slices(const AttnDims& d) { return (d.window + SLICE - 1) / SLICE; }
+size_t attn_paged_part_floats(const AttnDims& d, int n_rows)
+{
+  const int ns = n_slices(d);
+  return ns > 1 ? (size_t)n_rows * d.heads * ns * (d.vdim_p + 2) : 0;
+}
+
+template <typename T, int HT>
+static void run_rows(const AttnDims& d, const KvView& kv, const AttnIn& in, const StepRows& r, const T* qbuf, T* out, int64_t ldo, float* part, bool single)
+{
+  const int hg = d.heads / d.kv_heads, ns = n_slices(d);
+  const dim3 grid(ns, d.kv_heads * ((hg + HT - 1) / HT), r.n_rows);
+  if (single) hipLaunchKernelGGL((attn_rows_kernel<T, HT, true>), grid, dim3(256), 0, ctx().stream, d, kv, in, r, qbuf, out, ldo, part);
+  else hipLaunchKernelGGL((attn_rows_kernel<T, HT, false>), grid, dim3(256), 0, ctx().stream, d, kv, in, r, qbuf, out, ldo, part);
+  if (ns > 1) hipLaunchKernelGGL(attn_rows_merge_kernel<T>, dim3(d.heads, r.n_rows), dim3(256), 0, ctx().stream, d, r, ns, part, out, ldo);
+}
+template <typename T>
+static void run_rows_t(const AttnDims& d, const KvView& kv, const AttnIn& in, const StepRows& r, const void* qbuf, void* out, int64_t ldo, float* part, bool single)
+{
+  const int hg = d.heads / d.kv_heads;
+  if (hg == 1) run_rows<T, 1>(d, kv, in, r, (const T*)qbuf, (T*)out, ldo, part, single);
+  else if (hg == 2) run_rows<T, 2>(d, kv, in, r, (const T*)qbuf, (T*)out, ldo, part, single);
+  else run_rows<T, 4>(d, kv, in, r, (const T*)qbuf, (T*)out, ldo, part, single);
+}
+int attn_paged_rows(const AttnDims& d, const KvView& kv, int act_t, const void* qbuf, const StepRows& r, void* out, int64_t ldo, float* part, bool single, const AttnIn& in)
+{
+  if (act_t == ACT_T_BF16) run_rows_t<bf16_t>(d, kv, in, r, qbuf, out, ldo, part, single);
+  else run_rows_t<float>(d, kv, in, r, qbuf, out, ldo, part, single);
+  CAI_HIP(hipGetLastError());
+  return CAI_OK;
+}
+
+bool attn_paged_prompt_ok(const AttnDims& d, int act_t) { return act_t == ACT_T_BF16 && d.dim <= 256 && d.vdim <= 256; }
+
+int attn_paged_prompt(const AttnDims& d, const KvView& kv, const void* qbuf, const StepRows& r, const int32_t* tiles, int n_tiles, void* out, int64_t ldo)
+{
+  const dim3 grid(n_tiles, d.heads), blk(256);
+#define PROMPT(K, V) hipLaunchKernelGGL((attn_prompt_paged_kernel<K, V>), grid, blk, 0, ctx().stream, d, kv, (const bf16_t*)qbuf, r, tiles, (bf16_t*)out, ldo)
+#define PROMPT_V(K) do { if (d.vdim <= 64) PROMPT(K, 4); else if (d.vdim <= 128) PROMPT(K, 8); else PROMPT(K, 16); } while (0)
+  if (d.dim <= 64) PROMPT_V(2); else if (d.dim <= 128) PROMPT_V(4); else PROMPT_V(8);
+#undef PROMPT_V
+#undef PROMPT
+  CAI_HIP(hipGetLastError());
+  return CAI_OK;
+}
+
+}  // namespace cai

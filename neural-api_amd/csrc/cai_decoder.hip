@@ -7,13 +7,14 @@
 //   (append + cached GQA) -> o-proj -> Sum -> TokenRMSNorm -> gate|up -> SwiGLU -> down -> Sum }
 //   -> final TokenRMSNorm -> vocab projection -> ArgMaxRow.
 // MoE blocks (neural/neuralpretrained.pas:15331-15388): router -> softmax -> top-k gate -> expert banks.
-#include "cai_internal.hpp"
+#include "cai_layered.hpp"
 
 #include <algorithm>
 #include <map>
 
 struct cai_decoder_s {
   cai_decoder_config cfg{};
+  cai::LayeredNet* net = nullptr;    // a layered decoder: everything below but cfg is unused, the calls go to the net
   struct Layer { cai_qw_s* w[9] = {nullptr}; float* v[5] = {nullptr}; };
   std::vector<Layer> layers;
   cai_qw_s* embed = nullptr; cai_qw_s* head = nullptr;
@@ -555,9 +556,35 @@ static int lookup_draft(const int32_t* ctx_tok, int n_ctx, int match_len, int nu
   return 0;
 }
 
+int decoder_from_net(LayeredNet* n, int max_tokens, int max_seq, cai_decoder_s** out)
+{
+  cai_decoder_s* d = new cai_decoder_s();
+  d->net = n;
+  const NetSpec& s = net_spec(n);
+  cai_decoder_config& c = d->cfg;
+  c.n_layers = net_n_runs(n); c.d_model = s.width; c.vocab = s.vocab; c.max_ctx = max_tokens; c.eps = s.eps; c.max_batch = max_seq;
+  *out = d;
+  return CAI_OK;
+}
+
+static int len_of(cai_decoder_s* d, int seq) { return d->net ? net_len(d->net, seq) : d->kv.len_at(seq, 0); }
+
+// `n` consecutive tokens of one sequence of a layered decoder; logits and arg-max of every row, or of the last one only
+static int net_rows_of(cai_decoder_s* d, int seq, const int32_t* tokens, int n, bool all, float* logits, int32_t* argmax)
+{
+  std::vector<uint8_t> want((size_t)n, all ? 1 : 0);
+  want[(size_t)n - 1] = 1;
+  return net_step(d->net, 1, &seq, &n, tokens, want.data(), logits, argmax);
+}
+constexpr int NET_PROMPT_ROWS = 4096;      // rows per step of a prompt fed through cai_decoder_prefill
+
 }  // namespace cai
 
 using namespace cai;
+
+// what a layered decoder has no use for
+#define NOT_LAYERED(d, name) \
+  do { if ((d)->net) return set_error(CAI_ERR_UNSUPPORTED, name ": not available for a layered decoder"); } while (0)
 
 extern "C" int cai_decoder_create(const cai_decoder_config* cfg, cai_decoder_t* out)
 {
@@ -623,6 +650,7 @@ extern "C" int cai_decoder_destroy(cai_decoder_t d)
 {
   CAI_ENTER();
   if (!d) return CAI_OK;
+  if (d->net) { net_destroy(d->net); delete d; return CAI_OK; }
   if (ctx().ready) (void)hipStreamSynchronize(ctx().stream);
   invalidate_graphs(d);
   kv_free(&d->kv);
@@ -651,6 +679,8 @@ extern "C" int cai_decoder_set_weight(cai_decoder_t d, int layer, int slot, cai_
 {
   CAI_ENTER();
   CAI_REQUIRE(d && w, "cai_decoder_set_weight: null argument");
+  NOT_LAYERED(d, "cai_decoder_set_weight");
+  CAI_REQUIRE(w->qtype != CAI_BF16, "cai_decoder_set_weight: bfloat16 matrices belong to layered decoders");
   const cai_decoder_config& c = d->cfg;
   const int qw = d->qw(), kw = d->kw();
   int64_t rows = -1, cols = -1;
@@ -682,6 +712,7 @@ extern "C" int cai_decoder_set_vector(cai_decoder_t d, int layer, int slot, cons
   CAI_ENTER();
   CAI_READY();
   CAI_REQUIRE(d && v, "cai_decoder_set_vector: null argument");
+  NOT_LAYERED(d, "cai_decoder_set_vector");
   const cai_decoder_config& c = d->cfg;
   int want = c.d_model;
   if (slot == CAI_V_Q_NORM) want = d->qw(); else if (slot == CAI_V_K_NORM) want = d->kw();
@@ -707,6 +738,15 @@ extern "C" int cai_decoder_step(cai_decoder_t d, const int32_t* tokens, const in
   CAI_REQUIRE(d && tokens && pos, "cai_decoder_step: null argument");
   const cai_decoder_config& c = d->cfg;
   CAI_REQUIRE(n_b >= 1 && n_b <= c.max_batch, "cai_decoder_step: n_b %d outside 1..%d", n_b, c.max_batch);
+  if (d->net) {
+    std::vector<int32_t> seq(n_b), one(n_b, 1);
+    for (int b = 0; b < n_b; b++) {
+      seq[b] = b;
+      if (pos[b] != net_len(d->net, b)) return set_error(CAI_ERR_STATE, "cai_decoder_step: sequence %d is at position %d, got %d", b, net_len(d->net, b), pos[b]);
+    }
+    const std::vector<uint8_t> want((size_t)n_b, 1);
+    return net_step(d->net, n_b, seq.data(), one.data(), tokens, want.data(), logits, argmax);
+  }
   int rc = check_ready(d); if (rc) return rc;
   for (int b = 0; b < n_b; b++) {
     CAI_REQUIRE(tokens[b] >= 0 && tokens[b] < c.vocab, "cai_decoder_step: token %d outside vocab %d", tokens[b], c.vocab);
@@ -741,6 +781,10 @@ extern "C" int cai_decoder_step_window(cai_decoder_t d, int seq, const int32_t* 
   const cai_decoder_config& c = d->cfg;
   CAI_REQUIRE(n >= 1 && n <= 8, "cai_decoder_step_window: width %d outside 1..8", n);
   CAI_REQUIRE(seq >= 0 && seq < c.max_batch, "cai_decoder_step_window: sequence %d of %d", seq, c.max_batch);
+  if (d->net) {
+    if (pos0 != net_len(d->net, seq)) return set_error(CAI_ERR_STATE, "cai_decoder_step_window: sequence %d is at position %d, got %d", seq, net_len(d->net, seq), pos0);
+    return net_rows_of(d, seq, tokens, n, true, logits, argmax);
+  }
   int rc = check_ready(d); if (rc) return rc;
   if (pos0 != d->kv.len_at(seq, 0)) return set_error(CAI_ERR_STATE, "cai_decoder_step_window: sequence %d is at position %d, got %d", seq, d->kv.len_at(seq, 0), pos0);
   if (d->kv.evict_cap > 0 && n > 1) return set_error(CAI_ERR_UNSUPPORTED, "cai_decoder_step_window: a session with eviction rolls its cache and cannot take back a window; step one token at a time");
@@ -779,13 +823,13 @@ extern "C" int cai_decoder_generate_lookup(cai_decoder_t d, const int32_t* conte
   CAI_READY();
   CAI_REQUIRE(d && context && tokens_out && n_ctx >= 1 && n_tokens >= 1, "cai_decoder_generate_lookup: bad argument");
   const cai_decoder_config& c = d->cfg;
-  if (d->kv.len_at(0, 0) != n_ctx - 1)
-    return set_error(CAI_ERR_STATE, "cai_decoder_generate_lookup: the cache of sequence 0 holds %d tokens, the context's first %d are expected (its last token is fed here)", d->kv.len_at(0, 0), n_ctx - 1);
-  if (d->kv.evict_cap == 0 ? n_ctx - 1 + n_tokens > c.max_ctx : n_tokens > c.max_ctx)   // (a session with eviction runs past max_ctx, like cai_decoder_generate)
+  if (len_of(d, 0) != n_ctx - 1)
+    return set_error(CAI_ERR_STATE, "cai_decoder_generate_lookup: the cache of sequence 0 holds %d tokens, the context's first %d are expected (its last token is fed here)", len_of(d, 0), n_ctx - 1);
+  if (!d->net && (d->kv.evict_cap == 0 ? n_ctx - 1 + n_tokens > c.max_ctx : n_tokens > c.max_ctx))   // (a session with eviction runs past max_ctx, like cai_decoder_generate)
     return set_error(CAI_ERR_STATE, "cai_decoder_generate_lookup: %d tokens from %d exceed max_ctx %d", n_tokens, n_ctx - 1, c.max_ctx);
   if (match_len < 1) match_len = 1;                       // (the reference clamps both the same way)
   if (num_draft < 1) num_draft = 1;
-  const bool can_draft = d->kv.evict_cap == 0;            // a rolling cache cannot take a window back
+  const bool can_draft = d->kv.evict_cap == 0 && !d->net; // a rolling cache cannot take a window back, nor can recurrent state
   std::vector<int32_t> all(context, context + n_ctx);
   all.reserve((size_t)n_ctx + n_tokens);
   int emitted = 0, passes = 0;
@@ -801,7 +845,7 @@ extern "C" int cai_decoder_generate_lookup(cai_decoder_t d, const int32_t* conte
     int acc = 0;
     all.push_back(am[0]); tokens_out[emitted++] = am[0];
     while (acc < nd && emitted < n_tokens && win[1 + acc] == am[acc]) { acc++; all.push_back(am[acc]); tokens_out[emitted++] = am[acc]; }
-    for (int l = 0; l < c.n_layers; l++) d->kv.len_at(0, l) = pos + 1 + acc;   // rows of rejected drafts are dropped
+    for (int l = 0; l < c.n_layers && !d->net; l++) d->kv.len_at(0, l) = pos + 1 + acc;   // rows of rejected drafts are dropped
   }
   if (passes_out) *passes_out = passes;
   return CAI_OK;
@@ -813,6 +857,10 @@ extern "C" int cai_decoder_generate(cai_decoder_t d, int32_t first_token, int po
   CAI_READY();
   CAI_REQUIRE(d && tokens_out && n_tokens >= 1, "cai_decoder_generate: bad argument");
   const cai_decoder_config& c = d->cfg;
+  if (d->net) {
+    if (pos != net_len(d->net, 0)) return set_error(CAI_ERR_STATE, "cai_decoder_generate: sequence 0 is at position %d, got %d", net_len(d->net, 0), pos);
+    return net_generate(d->net, 0, first_token, n_tokens, tokens_out);
+  }
   int rc = check_ready(d); if (rc) return rc;
   CAI_REQUIRE(first_token >= 0 && first_token < c.vocab, "cai_decoder_generate: token %d outside vocab %d", first_token, c.vocab);
   if (pos != d->kv.len_at(0, 0)) return set_error(CAI_ERR_STATE, "cai_decoder_generate: sequence 0 is at position %d, got %d", d->kv.len_at(0, 0), pos);
@@ -839,6 +887,7 @@ extern "C" int cai_decoder_profile(cai_decoder_t d, int32_t token, int reps, flo
   CAI_ENTER();
   CAI_READY();
   CAI_REQUIRE(d && us_per_step_out && reps >= 1 && n_classes >= 1 && n_classes <= 8, "cai_decoder_profile: bad argument");
+  NOT_LAYERED(d, "cai_decoder_profile");
   const cai_decoder_config& c = d->cfg;
   int rc = check_ready(d); if (rc) return rc;
   CAI_REQUIRE(token >= 0 && token < c.vocab, "cai_decoder_profile: token %d outside vocab %d", token, c.vocab);
@@ -910,6 +959,7 @@ extern "C" int cai_decoder_timeline(cai_decoder_t d, int32_t token, uint64_t* st
   CAI_ENTER();
   CAI_READY();
   CAI_REQUIRE(d && stamps_out && launches_out && n_launches_out && n_stamps_out && ticks_per_us_out && stamps_cap > 0 && launches_cap > 0, "cai_decoder_timeline: bad argument");
+  NOT_LAYERED(d, "cai_decoder_timeline");
   const cai_decoder_config& c = d->cfg;
   int rc = check_ready(d); if (rc) return rc;
   CAI_REQUIRE(token >= 0 && token < c.vocab, "cai_decoder_timeline: token %d outside vocab %d", token, c.vocab);
@@ -969,6 +1019,15 @@ extern "C" int cai_decoder_prefill(cai_decoder_t d, int seq, const int32_t* toke
   CAI_REQUIRE(d && tokens && n >= 1, "cai_decoder_prefill: bad argument");
   const cai_decoder_config& c = d->cfg;
   CAI_REQUIRE(seq >= 0 && seq < c.max_batch, "cai_decoder_prefill: sequence %d of %d", seq, c.max_batch);
+  if (d->net) {
+    if (pos0 != net_len(d->net, seq)) return set_error(CAI_ERR_STATE, "cai_decoder_prefill: sequence %d is at position %d, got %d", seq, net_len(d->net, seq), pos0);
+    for (int t = 0; t < n; t += NET_PROMPT_ROWS) {
+      const int m = std::min(NET_PROMPT_ROWS, n - t);
+      const int rcn = net_rows_of(d, seq, tokens + t, m, false, t + m == n ? last_logits : nullptr, t + m == n ? argmax : nullptr);
+      if (rcn) return rcn;
+    }
+    return CAI_OK;
+  }
   int rc = check_ready(d); if (rc) return rc;
   if (pos0 != d->kv.len_at(seq, 0)) return set_error(CAI_ERR_STATE, "cai_decoder_prefill: sequence %d is at position %d, got %d", seq, d->kv.len_at(seq, 0), pos0);
   if (pos0 + n > c.max_ctx && d->kv.evict_cap == 0) return set_error(CAI_ERR_STATE, "cai_decoder_prefill: %d tokens from %d exceed max_ctx %d", n, pos0, c.max_ctx);
@@ -1026,6 +1085,7 @@ extern "C" int cai_decoder_hidden_state(cai_decoder_t d, int row, float* hidden_
   CAI_READY();
   CAI_REQUIRE(d && hidden_out, "cai_decoder_hidden_state: null argument");
   CAI_REQUIRE(row >= 0 && row < 8, "cai_decoder_hidden_state: row %d outside 0..7", row);
+  if (d->net) return net_hidden(d->net, row, hidden_out);
   if (!d->final_norm) return set_error(CAI_ERR_STATE, "cai_decoder_hidden_state: final norm gain not set");
   Context& cx = ctx();
   const int dm = d->cfg.d_model;
@@ -1046,6 +1106,11 @@ extern "C" int cai_decoder_candidates(cai_decoder_t d, int row, const int32_t* h
   CAI_REQUIRE(d && tokens_out && probs_out, "cai_decoder_candidates: null argument");
   CAI_REQUIRE(row >= 0 && row < 8, "cai_decoder_candidates: row %d outside 0..7", row);   // a row of the last step (sequence) or window (position)
   CAI_REQUIRE(m >= 1 && m <= 1024, "cai_decoder_candidates: %d candidates (1..1024)", m);
+  if (d->net) {
+    const float* lg = net_logits(d->net, row);
+    if (!lg) return set_error(CAI_ERR_STATE, "cai_decoder_candidates: the last step has no logits row %d", row);
+    return run_candidates(lg, d->cfg.vocab, hist_ids, hist_counts, n_hist, repetition, frequency, presence, temperature, m, tokens_out, probs_out, count_out);
+  }
   return run_candidates(d->logits + (int64_t)row * d->cfg.vocab, d->cfg.vocab, hist_ids, hist_counts, n_hist,
                         repetition, frequency, presence, temperature, m, tokens_out, probs_out, count_out);
 }
@@ -1055,6 +1120,7 @@ extern "C" int cai_decoder_reset(cai_decoder_t d, int seq)
   CAI_ENTER();
   CAI_REQUIRE(d, "cai_decoder_reset: null decoder");
   CAI_REQUIRE(seq >= 0 && seq < d->cfg.max_batch, "cai_decoder_reset: sequence %d of %d", seq, d->cfg.max_batch);
+  if (d->net) return net_reset(d->net, seq);
   for (int l = 0; l < d->cfg.n_layers; l++) d->kv.len_at(seq, l) = 0;
   return CAI_OK;
 }
@@ -1064,6 +1130,11 @@ extern "C" int cai_decoder_truncate(cai_decoder_t d, int seq, int n)
   CAI_ENTER();
   CAI_REQUIRE(d, "cai_decoder_truncate: null decoder");
   CAI_REQUIRE(seq >= 0 && seq < d->cfg.max_batch && n >= 0, "cai_decoder_truncate: bad argument");
+  if (d->net) {
+    if (n == 0) return net_reset(d->net, seq);
+    if (n < net_len(d->net, seq)) return set_error(CAI_ERR_UNSUPPORTED, "cai_decoder_truncate: recurrent state cannot be taken back from %d tokens to %d; restore a snapshot", net_len(d->net, seq), n);
+    return CAI_OK;
+  }
   const int have = d->kv.len_at(seq, 0);
   if (have > n && d->kv.evict_cap > 0 && have > d->kv.evict_cap)
     return set_error(CAI_ERR_STATE, "cai_decoder_truncate: %d tokens streamed under eviction, the rows before %d are gone", have, have - (d->kv.evict_cap - d->kv.evict_sinks));
@@ -1075,6 +1146,7 @@ extern "C" int cai_decoder_set_eviction(cai_decoder_t d, int sink_tokens, int re
 {
   CAI_ENTER();
   CAI_REQUIRE(d, "cai_decoder_set_eviction: null decoder");
+  NOT_LAYERED(d, "cai_decoder_set_eviction");
   const int rc = kv_set_eviction(&d->kv, sink_tokens, recent_window);
   if (rc) return rc;
   (void)hipStreamSynchronize(ctx().stream);
@@ -1088,6 +1160,7 @@ extern "C" int cai_decoder_set_kv_dtype(cai_decoder_t d, int kv_dtype)
   CAI_ENTER();
   CAI_READY();
   CAI_REQUIRE(d, "cai_decoder_set_kv_dtype: null decoder");
+  NOT_LAYERED(d, "cai_decoder_set_kv_dtype");
   CAI_REQUIRE(kv_dtype == CAI_KV_F32 || kv_dtype == CAI_KV_F16 || kv_dtype == CAI_KV_I8, "cai_decoder_set_kv_dtype: type %d", kv_dtype);
   for (int n : d->kv.len)
     if (n > 0) return set_error(CAI_ERR_STATE, "cai_decoder_set_kv_dtype: the cache holds %d tokens; the storage mode only changes on an empty session", n);
@@ -1129,6 +1202,7 @@ extern "C" int cai_decoder_set_rope_scaling(cai_decoder_t d, int mode, float fac
   CAI_ENTER();
   CAI_READY();
   CAI_REQUIRE(d, "cai_decoder_set_rope_scaling: null decoder");
+  NOT_LAYERED(d, "cai_decoder_set_rope_scaling");
   std::vector<float> th;
   int rc = rope_thetas_scaled(d->cfg.rope_theta, d->cfg.head_dim, mode, factor, original_ctx, low_freq_factor, high_freq_factor, th);
   if (rc) return rc;
@@ -1142,6 +1216,7 @@ extern "C" int cai_decoder_set_rope_out_scale(cai_decoder_t d, float scale)
   CAI_ENTER();
   CAI_READY();
   CAI_REQUIRE(d, "cai_decoder_set_rope_out_scale: null decoder");
+  NOT_LAYERED(d, "cai_decoder_set_rope_out_scale");
   CAI_REQUIRE(scale > 0.0f && scale < 3.0e38f, "cai_decoder_set_rope_out_scale: scale %g", (double)scale);
   for (int n : d->kv.len)
     if (n > 0) return set_error(CAI_ERR_STATE, "cai_decoder_set_rope_out_scale: the cache holds %d tokens; set the rule on an empty session", n);
@@ -1155,6 +1230,7 @@ extern "C" int cai_decoder_set_rope_freq_factors(cai_decoder_t d, const float* f
   CAI_ENTER();
   CAI_READY();
   CAI_REQUIRE(d && factors, "cai_decoder_set_rope_freq_factors: null argument");
+  NOT_LAYERED(d, "cai_decoder_set_rope_freq_factors");
   CAI_REQUIRE(n == d->cfg.head_dim / 2, "cai_decoder_set_rope_freq_factors: %d factors for %d rotary pairs", n, d->cfg.head_dim / 2);
   std::vector<float> th(n);
   for (int k = 0; k < n; k++) {
@@ -1169,6 +1245,7 @@ extern "C" int cai_decoder_cache_rows(cai_decoder_t d, int seq, int layer, int* 
   CAI_ENTER();
   CAI_REQUIRE(d && rows_out, "cai_decoder_cache_rows: null argument");
   CAI_REQUIRE(seq >= 0 && seq < d->cfg.max_batch && layer >= 0 && layer < d->cfg.n_layers, "cai_decoder_cache_rows: sequence %d, layer %d", seq, layer);
+  if (d->net) { *rows_out = net_rows(d->net, seq); return CAI_OK; }
   *rows_out = d->kv.live(d->kv.len_at(seq, layer));
   return CAI_OK;
 }
@@ -1178,7 +1255,7 @@ extern "C" int cai_decoder_len(cai_decoder_t d, int seq, int* len_out)
   CAI_ENTER();
   CAI_REQUIRE(d && len_out, "cai_decoder_len: null argument");
   CAI_REQUIRE(seq >= 0 && seq < d->cfg.max_batch, "cai_decoder_len: sequence %d of %d", seq, d->cfg.max_batch);
-  *len_out = d->kv.len_at(seq, 0);
+  *len_out = len_of(d, seq);
   return CAI_OK;
 }
 
@@ -1188,6 +1265,14 @@ extern "C" int cai_decoder_snapshot(cai_decoder_t d, int seq, cai_kv_snap_t* out
   CAI_READY();
   CAI_REQUIRE(d && out, "cai_decoder_snapshot: null argument");
   CAI_REQUIRE(seq >= 0 && seq < d->cfg.max_batch, "cai_decoder_snapshot: sequence %d of %d", seq, d->cfg.max_batch);
+  if (d->net) {
+    NetSnap* ns = nullptr;
+    const int rc = net_snapshot(d->net, seq, &ns);
+    if (rc) return rc;
+    *out = new cai_kv_snap_s();
+    (*out)->net = ns;
+    return CAI_OK;
+  }
   return kv_snapshot(&d->kv, seq, out);
 }
 
@@ -1197,6 +1282,8 @@ extern "C" int cai_decoder_restore(cai_decoder_t d, int seq, cai_kv_snap_t snap)
   CAI_READY();
   CAI_REQUIRE(d && snap, "cai_decoder_restore: null argument");
   CAI_REQUIRE(seq >= 0 && seq < d->cfg.max_batch, "cai_decoder_restore: sequence %d of %d", seq, d->cfg.max_batch);
+  CAI_REQUIRE(!d->net == !snap->net, "cai_decoder_restore: the snapshot is of another kind of decoder");
+  if (d->net) return net_restore(d->net, seq, snap->net);
   return kv_restore(&d->kv, seq, snap);
 }
 
@@ -1207,6 +1294,7 @@ extern "C" int cai_decoder_fork(cai_decoder_t d, int src_seq, int dst_seq)
   CAI_REQUIRE(d, "cai_decoder_fork: null decoder");
   CAI_REQUIRE(src_seq >= 0 && src_seq < d->cfg.max_batch && dst_seq >= 0 && dst_seq < d->cfg.max_batch,
               "cai_decoder_fork: sequences %d -> %d of %d", src_seq, dst_seq, d->cfg.max_batch);
+  if (d->net) return net_fork(d->net, src_seq, dst_seq);
   return kv_fork(&d->kv, src_seq, dst_seq);
 }
 
@@ -1222,6 +1310,7 @@ extern "C" int cai_decoder_weight_bytes(cai_decoder_t d, int64_t* out)
 {
   CAI_ENTER();
   CAI_REQUIRE(d && out, "cai_decoder_weight_bytes: null argument");
+  if (d->net) { *out = net_weight_bytes(d->net); return CAI_OK; }
   const cai_decoder_config& c = d->cfg;
   int rc = check_ready(d); if (rc) return rc;
   int64_t b = 0;
@@ -1241,3 +1330,72 @@ extern "C" int cai_decoder_weight_bytes(cai_decoder_t d, int64_t* out)
   return CAI_OK;
 }
 
+
+// One engine step over any mixture of prompt portions and single tokens: entry e brings counts[e] tokens of sequence seqs[e].
+// A layered decoder runs them as one batch.  The other decoders take single tokens of sequences 0 .. n - 1 as one batch and
+// anything else entry by entry: a portion whose only wanted row is its last through the prompt pass, other portions in windows.
+extern "C" int cai_decoder_step_batch(cai_decoder_t d, int n_entries, const int32_t* seqs, const int32_t* counts, const int32_t* tokens,
+                                      const uint8_t* want, float* logits, int32_t* argmax)
+{
+  CAI_ENTER();
+  CAI_READY();
+  CAI_REQUIRE(d && seqs && counts && tokens && n_entries >= 1, "cai_decoder_step_batch: bad argument");
+  if (d->net) return net_step(d->net, n_entries, seqs, counts, tokens, want, logits, argmax);
+  const int V = d->cfg.vocab, B = d->cfg.max_batch;
+  bool plain = n_entries <= B;
+  std::vector<uint8_t> seen((size_t)B, 0);
+  for (int e = 0; e < n_entries; e++) {
+    CAI_REQUIRE(seqs[e] >= 0 && seqs[e] < B && !seen[seqs[e]] && counts[e] >= 1, "cai_decoder_step_batch: entry %d: sequence %d (of %d, each once), %d tokens", e, seqs[e], B, counts[e]);
+    seen[seqs[e]] = 1;
+    plain = plain && counts[e] == 1 && seqs[e] == e;
+    if (len_of(d, seqs[e]) + counts[e] > d->cfg.max_ctx && d->kv.evict_cap == 0)
+      return set_error(CAI_ERR_STATE, "cai_decoder_step_batch: sequence %d would pass max_ctx %d", seqs[e], d->cfg.max_ctx);
+  }
+  int rc, out = 0;
+  if (plain && n_entries > 1) {
+    std::vector<int32_t> pos(n_entries), am(n_entries);
+    std::vector<float> lg(logits ? (size_t)n_entries * V : 0);
+    for (int e = 0; e < n_entries; e++) pos[e] = len_of(d, e);
+    if ((rc = cai_decoder_step(d, tokens, pos.data(), n_entries, logits ? lg.data() : nullptr, am.data()))) return rc;
+    for (int e = 0; e < n_entries; e++) {
+      if (!want || !want[e]) continue;
+      if (logits) std::copy(lg.begin() + (size_t)e * V, lg.begin() + (size_t)(e + 1) * V, logits + (size_t)out * V);
+      if (argmax) argmax[out] = am[e];
+      out++;
+    }
+    return CAI_OK;
+  }
+  for (int e = 0, r0 = 0; e < n_entries; r0 += counts[e], e++) {
+    const int n = counts[e];
+    bool inner = false;
+    for (int i = 0; want && i + 1 < n; i++) inner = inner || want[r0 + i];
+    const int width = inner && d->kv.evict_cap == 0 ? 8 : inner ? 1 : n;
+    for (int t = 0; t < n; t += width) {
+      const int m = std::min(width, n - t), pos0 = len_of(d, seqs[e]);
+      std::vector<float> lg(logits ? (size_t)(inner ? m : 1) * V : 0);
+      std::vector<int32_t> am(inner ? m : 1);
+      if (inner) rc = cai_decoder_step_window(d, seqs[e], tokens + r0 + t, m, pos0, logits ? lg.data() : nullptr, am.data());
+      else rc = cai_decoder_prefill(d, seqs[e], tokens + r0, n, pos0, logits ? lg.data() : nullptr, am.data());
+      if (rc) return rc;
+      for (int i = 0; i < m; i++) {
+        if (!want || !want[r0 + t + i]) continue;
+        const int k = inner ? i : 0;
+        if (logits) std::copy(lg.begin() + (size_t)k * V, lg.begin() + (size_t)(k + 1) * V, logits + (size_t)out * V);
+        if (argmax) argmax[out] = am[k];
+        out++;
+      }
+    }
+  }
+  return CAI_OK;
+}
+
+// Tokens sequence `seq` can still take: of the shared page pool (layered decoder) or of its own rows.
+extern "C" int cai_decoder_room(cai_decoder_t d, int seq, int* tokens_out)
+{
+  CAI_ENTER();
+  CAI_REQUIRE(d && tokens_out, "cai_decoder_room: null argument");
+  CAI_REQUIRE(seq >= 0 && seq < d->cfg.max_batch, "cai_decoder_room: sequence %d of %d", seq, d->cfg.max_batch);
+  if (d->net) *tokens_out = net_room(d->net, seq);
+  else *tokens_out = d->kv.evict_cap > 0 ? 1 << 30 : d->cfg.max_ctx - len_of(d, seq);
+  return CAI_OK;
+}

@@ -694,6 +694,7 @@ int launch_gemv_multi(const MultiGemv& m, const float* x, int n_b, float* y, int
 {
   Context& c = ctx();
   const cai_qw_s* w0 = m.w[0];
+  if (w0->qtype == CAI_BF16) return set_error(CAI_ERR_UNSUPPORTED, "gemv: bfloat16 matrices have products of their own");
   GemvParams p{};
   p.n_seg = m.n; p.x = x; p.y = y; p.residual = residual; p.norm_gain = norm_gain; p.norm_eps = norm_eps;
   p.cols = (int)w0->cols; p.y_stride = (int)y_stride; p.act = act; p.half = swiglu_half;

@@ -139,6 +139,7 @@ __device__ __forceinline__ void for_strided8(const float* x, const float* g, int
 struct cai_qw_s {
   int      qtype = 0;
   int64_t  rows = 0, cols = 0;
+  int64_t  ld = 0;             // BF16 only: elements from one row to the next (cols padded with zeros to a multiple of 64)
   uint8_t* data = nullptr;     // quants plane or the raw blocks
   uint8_t* aux = nullptr;      // half scales plane (Q8_0/Q4_0), float row scales (I8ROW), or for Q6_K the int8 scales plane (16 per block) followed by the plane of d
   float*   bias = nullptr;
@@ -185,7 +186,9 @@ struct cai_kv_s {
   int& len_at(int seq, int layer) { return len[(size_t)seq * n_layers + layer]; }
 };
 
+namespace cai { struct NetSnap; void net_snap_free(NetSnap* s); }
 struct cai_kv_snap_s {
+  cai::NetSnap* net = nullptr;            // a layered decoder's pages and state (the rest is then unused)
   int n_layers = 0, kv_heads = 0, head_dim = 0, dtype = 0, rows = 0;
   int evict_sinks = 0, evict_cap = 0;     // the eviction policy the rows were laid out under
   std::vector<int> len;                   // per layer

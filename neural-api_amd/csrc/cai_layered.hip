@@ -1,0 +1,700 @@
+// The layered decoder: decoders whose layers differ in kind and size, where a stretch of layers may run several times with the
+// same weights and a cache or state of its own per pass.  Holds the paged pool and state slots (SeqPool), the plan of layer runs,
+// and the step function.  A step is any mixture of prompt portions and single tokens of different sequences; a step of single
+// tokens only is captured once per width as a graph and replayed.
+//
+// The residual stream is float.  A sublayer's epilogue adds its result and already leaves the next sublayer's normed input, so
+// between two mixers there are three products and nothing else.
+#include "cai_layered.hpp"
+
+#include <algorithm>
+#include <map>
+#include <string.h>
+
+namespace cai {
+
+// ------------------------------------------------------------------------------------------
+// pool
+// ------------------------------------------------------------------------------------------
+int SeqPool::alloc(int n_seq_, int max_tokens, int act_t_)
+{
+  n_seq = n_seq_; act_t = act_t_;
+  keep = 0;
+  for (auto& a : attn) keep = std::max(keep, a.d.window);
+  n_pages = attn.empty() ? 0 : (max_tokens + PAGE_TOKENS - 1) / PAGE_TOKENS;
+  seq.assign(n_seq, Seq());
+  const size_t es = act_t == ACT_T_BF16 ? 2 : 4;
+  auto s = ctx().stream;
+  for (auto& a : attn) {
+    a.v_off = (int64_t)a.d.kv_heads * PAGE_TOKENS * a.d.dim_p;
+    a.page_elems = a.v_off + (int64_t)a.d.kv_heads * PAGE_TOKENS * a.d.vdim_p;
+    CAI_HIP(hipMalloc(&a.base, (size_t)n_pages * a.page_elems * es));
+    CAI_HIP(hipMemsetAsync(a.base, 0, (size_t)n_pages * a.page_elems * es, s));
+  }
+  for (auto& d : delta) {
+    d.s_elems = (int64_t)d.d.heads * d.d.dim * d.d.vdim_p();
+    d.h_elems = (int64_t)d.d.taps * d.d.channels();
+    CAI_HIP(hipMalloc((void**)&d.S, (size_t)n_seq * d.s_elems * 4));
+    CAI_HIP(hipMalloc((void**)&d.hist, (size_t)n_seq * d.h_elems * 4));
+    CAI_HIP(hipMemsetAsync(d.S, 0, (size_t)n_seq * d.s_elems * 4, s));
+    CAI_HIP(hipMemsetAsync(d.hist, 0, (size_t)n_seq * d.h_elems * 4, s));
+  }
+  if (n_pages) {
+    table.assign((size_t)n_seq * n_pages, 0);
+    CAI_HIP(hipMalloc((void**)&d_table, table.size() * sizeof(int32_t)));
+    table_dirty = true;
+    for (int p = n_pages - 1; p >= 0; p--) free_pages.push_back(p);
+  }
+  CAI_HIP(hipStreamSynchronize(s));
+  return CAI_OK;
+}
+
+void SeqPool::release_all()
+{
+  for (auto& a : attn) { if (a.base) (void)hipFree(a.base); a.base = nullptr; }
+  for (auto& d : delta) { if (d.S) (void)hipFree(d.S); if (d.hist) (void)hipFree(d.hist); d.S = d.hist = nullptr; }
+  if (d_table) (void)hipFree(d_table);
+  d_table = nullptr;
+}
+
+int SeqPool::reserve(int s, int new_len)
+{
+  if (!n_pages) return CAI_OK;
+  Seq& q = seq[s];
+  const int end = (new_len + PAGE_TOKENS - 1) / PAGE_TOKENS, need = end - q.end_page;
+  if (need <= 0) return CAI_OK;
+  if (need > (int)free_pages.size())
+    return set_error(CAI_ERR_STATE, "cache pool: sequence %d needs %d more pages of %d tokens, %zu of %d are free", s, need, PAGE_TOKENS, free_pages.size(), n_pages);
+  for (; q.end_page < end; q.end_page++) {
+    table[(size_t)s * n_pages + q.end_page % n_pages] = free_pages.back();
+    free_pages.pop_back();
+  }
+  table_dirty = true;
+  return CAI_OK;
+}
+
+void SeqPool::trim(int s)
+{
+  if (!n_pages) return;
+  Seq& q = seq[s];
+  const int first = std::max(0, q.len - keep + 1) / PAGE_TOKENS;      // page of the oldest key the next token sees
+  for (; q.first_page < std::min(first, q.end_page); q.first_page++) free_pages.push_back(table[(size_t)s * n_pages + q.first_page % n_pages]);
+}
+
+void SeqPool::free_seq(int s)
+{
+  Seq& q = seq[s];
+  if (n_pages) for (int p = q.first_page; p < q.end_page; p++) free_pages.push_back(table[(size_t)s * n_pages + p % n_pages]);
+  q = Seq();
+}
+
+int SeqPool::room(int s) const
+{
+  if (!n_pages) return 1 << 30;
+  return (seq[s].end_page + (int)free_pages.size()) * PAGE_TOKENS - seq[s].len;
+}
+
+int SeqPool::upload_table()
+{
+  if (!table_dirty || !n_pages) return CAI_OK;
+  CAI_HIP(hipMemcpyAsync(d_table, table.data(), table.size() * sizeof(int32_t), hipMemcpyHostToDevice, ctx().stream));
+  CAI_HIP(hipStreamSynchronize(ctx().stream));       // (the host copy changes with the next reservation)
+  table_dirty = false;
+  return CAI_OK;
+}
+
+int SeqPool::fork(int src, int dst)
+{
+  free_seq(dst);
+  const Seq& a = seq[src];
+  Seq& b = seq[dst];
+  auto s = ctx().stream;
+  const size_t es = act_t == ACT_T_BF16 ? 2 : 4;
+  if (n_pages) {
+    if (a.end_page - a.first_page > (int)free_pages.size())
+      return set_error(CAI_ERR_STATE, "cache pool: a copy of sequence %d needs %d pages, %zu are free", src, a.end_page - a.first_page, free_pages.size());
+    b.first_page = b.end_page = a.first_page;
+    for (; b.end_page < a.end_page; b.end_page++) {
+      const int from = table[(size_t)src * n_pages + b.end_page % n_pages], to = free_pages.back();
+      free_pages.pop_back();
+      table[(size_t)dst * n_pages + b.end_page % n_pages] = to;
+      for (auto& r : attn)
+        CAI_HIP(hipMemcpyAsync((char*)r.base + (size_t)to * r.page_elems * es, (char*)r.base + (size_t)from * r.page_elems * es, (size_t)r.page_elems * es, hipMemcpyDeviceToDevice, s));
+    }
+    table_dirty = true;
+  }
+  for (auto& r : delta) {
+    CAI_HIP(hipMemcpyAsync(r.S + dst * r.s_elems, r.S + src * r.s_elems, (size_t)r.s_elems * 4, hipMemcpyDeviceToDevice, s));
+    CAI_HIP(hipMemcpyAsync(r.hist + dst * r.h_elems, r.hist + src * r.h_elems, (size_t)r.h_elems * 4, hipMemcpyDeviceToDevice, s));
+  }
+  b.len = a.len;
+  return CAI_OK;
+}
+
+KvView SeqPool::view(int run) const
+{
+  const AttnRun& a = attn[run];
+  return KvView{a.base, a.page_elems, d_table, n_pages, a.v_off};
+}
+
+// ------------------------------------------------------------------------------------------
+// small kernels of the step
+// ------------------------------------------------------------------------------------------
+template <typename AT>
+__global__ __launch_bounds__(256) void net_embed_kernel(const uint16_t* e, const int ld, const int32_t* tok, const int width, float* x, float* x0, AT* h, const int64_t ldh, const Dyt next)
+{
+  const int64_t t = blockIdx.y;
+  const uint16_t* row = e + (int64_t)tok[t] * ld;
+  for (int i = blockIdx.x * 256 + threadIdx.x; i < width; i += gridDim.x * 256) {
+    const float v = __builtin_bit_cast(float, (uint32_t)row[i] << 16);
+    x[t * width + i] = v;
+    if (x0) x0[t * width + i] = v;
+    h[t * ldh + i] = (AT)dyt(next, v, i);
+  }
+}
+
+// Two outputs side by side: each RMS-normed over the width with its own gain, half their sum through `post` onto the residual
+// stream (+ add0), then the next sublayer's input.
+template <typename AT>
+__global__ __launch_bounds__(256) void net_join_kernel(const float* yl, const float* yr, const float* gl, const float* gr, const int width, const float eps,
+                                                       float* x, const float* add0, const Dyt post, const Dyt next, AT* h, const int64_t ldh)
+{
+  __shared__ float sl[4], sr[4];
+  const int64_t t = blockIdx.x;
+  const float *a = yl + t * width, *b = yr + t * width;
+  float s = 0.0f, q = 0.0f;
+  for_strided8(a, threadIdx.x, width, 256, [&](float v, int) { s = fmaf(v, v, s); });
+  for_strided8(b, threadIdx.x, width, 256, [&](float v, int) { q = fmaf(v, v, q); });
+  for (int o = 32; o; o >>= 1) { s += __shfl_xor(s, o); q += __shfl_xor(q, o); }
+  if ((threadIdx.x & 63) == 0) { sl[threadIdx.x >> 6] = s; sr[threadIdx.x >> 6] = q; }
+  __syncthreads();
+  const float il = 1.0f / sqrtf((sl[0] + sl[1] + sl[2] + sl[3]) / (float)width + eps), ir = 1.0f / sqrtf((sr[0] + sr[1] + sr[2] + sr[3]) / (float)width + eps);
+  for (int i = threadIdx.x; i < width; i += 256) {
+    const float y = 0.5f * (a[i] * il * gl[i] + b[i] * ir * gr[i]);
+    float v = x[t * width + i] + dyt(post, y, i);
+    if (add0) v += add0[t * width + i];
+    x[t * width + i] = v;
+    h[t * ldh + i] = (AT)dyt(next, v, i);
+  }
+}
+
+template <typename AT>
+__global__ __launch_bounds__(256) void net_gather_kernel(const AT* h, const int32_t* rows, const int64_t ld, AT* out)
+{
+  const int64_t src = rows[blockIdx.x];
+  for (int64_t i = threadIdx.x; i < ld; i += 256) out[blockIdx.x * ld + i] = h[src * ld + i];
+}
+
+// greedy hand-over between two captured steps of one row
+__global__ void net_advance_kernel(int32_t* tok, int32_t* pos, const int32_t* best, int32_t* gen, int32_t* gen_idx)
+{
+  if (threadIdx.x == 0 && blockIdx.x == 0) {
+    const int32_t t = best[0]; const int i = gen_idx[0];
+    gen[i] = t; gen_idx[0] = i + 1; tok[0] = t; pos[0] += 1;
+  }
+}
+
+// ------------------------------------------------------------------------------------------
+// the net
+// ------------------------------------------------------------------------------------------
+constexpr int DEC_ROWS = 8;                // widest captured step
+constexpr int GEN_STEPS = 8;               // greedy steps per captured launch
+
+struct LayeredNet {
+  NetSpec s;
+  int act_t = ACT_T_BF16, max_seq = 1;
+  size_t es = 2;
+  SeqPool pool;
+  std::vector<NetRun> runs;
+  // widths over all layers
+  int wp = 0, ld_proj = 0, ld_mid = 0, ld_att = 0, ld_attl = 0, ld_q = 0, ld_ra = 0, ld_rg = 0;
+  int w_q = 0, w_k = 0, w_v = 0, w_g = 0, w_b = 0, w_za = 0, w_zg = 0;
+  bool has_attn = false, looped = false;
+  int cap = 0, logit_cap = 0, best_cap = 0;
+  float *x = nullptr, *x0 = nullptr, *proj = nullptr, *yl = nullptr, *yr = nullptr, *part = nullptr, *logits = nullptr;
+  void *h = nullptr, *mid = nullptr, *att = nullptr, *attl = nullptr, *qbuf = nullptr, *ra = nullptr, *rgb = nullptr, *hw = nullptr;
+  DeltaBuf db{};
+  float* am_v = nullptr; int32_t* am_i = nullptr; int32_t* best = nullptr;
+  int32_t* d_rows = nullptr; int32_t* h_rows = nullptr; size_t rows_cap = 0;
+  int32_t* d_dec = nullptr;                // fixed row arrays of captured steps: tok, pos, slot, first, last [DEC_ROWS each], ent [4 DEC_ROWS], gen_idx
+  int32_t* h_dec = nullptr;
+  int32_t* d_gen = nullptr; int gen_cap = 0;
+  std::map<int, hipGraphExec_t> graphs;
+  bool use_graph = true;
+  std::vector<int> row_of;                 // logits row of the k-th wanted row of the last step
+  bool rows_gathered = false;
+};
+
+void net_spec_free(NetSpec& s)
+{
+  for (cai_qw_s* w : s.weights) (void)cai_qw_destroy(w);
+  for (void* v : s.vectors) (void)hipFree(v);
+  s = NetSpec();
+}
+
+static void drop_graphs(LayeredNet* n)
+{
+  for (auto& g : n->graphs) if (g.second) (void)hipGraphExecDestroy(g.second);
+  n->graphs.clear();
+}
+
+static void free_rows(LayeredNet* n)
+{
+  void* p[] = {n->x, n->x0, n->proj, n->yl, n->yr, n->part, n->h, n->mid, n->att, n->attl, n->qbuf, n->ra, n->rgb, n->db.q, n->db.k, n->db.v, n->db.g, n->db.beta, n->db.o, n->db.za, n->db.zg};
+  for (void* q : p) if (q) (void)hipFree(q);
+  n->x = n->x0 = n->proj = n->yl = n->yr = n->part = nullptr;
+  n->h = n->mid = n->att = n->attl = n->qbuf = n->ra = n->rgb = nullptr;
+  n->db = DeltaBuf{};
+  n->cap = 0;
+}
+
+static int ensure_rows(LayeredNet* n, int rows)
+{
+  if (n->cap >= rows) return CAI_OK;
+  const size_t R = (size_t)std::max(rows, std::max(DEC_ROWS, n->cap + n->cap / 2));
+  CAI_HIP(hipStreamSynchronize(ctx().stream));
+  drop_graphs(n);
+  free_rows(n);
+  const int w = n->s.width;
+  auto get = [&](void** p, size_t bytes) -> int {
+    if (!bytes) return CAI_OK;
+    CAI_HIP(hipMalloc(p, bytes));
+    CAI_HIP(hipMemsetAsync(*p, 0, bytes, ctx().stream));
+    return CAI_OK;
+  };
+  size_t part = 0;
+  for (auto& a : n->pool.attn) part = std::max(part, attn_paged_part_floats(a.d, (int)R));
+  int rc;
+  if ((rc = get((void**)&n->x, R * w * 4)) || (rc = get((void**)&n->x0, n->looped ? R * w * 4 : 0)) || (rc = get((void**)&n->proj, R * n->ld_proj * 4)) ||
+      (rc = get((void**)&n->yl, n->has_attn ? R * w * 4 : 0)) || (rc = get((void**)&n->yr, n->has_attn ? R * w * 4 : 0)) || (rc = get((void**)&n->part, part * 4)) ||
+      (rc = get(&n->h, R * n->wp * n->es)) || (rc = get(&n->mid, R * n->ld_mid * n->es)) || (rc = get(&n->att, R * n->ld_att * n->es)) ||
+      (rc = get(&n->attl, R * n->ld_attl * n->es)) || (rc = get(&n->qbuf, R * n->ld_q * n->es)) || (rc = get(&n->ra, R * n->ld_ra * n->es)) || (rc = get(&n->rgb, R * n->ld_rg * n->es)) ||
+      (rc = get((void**)&n->db.q, R * n->w_q * 4)) || (rc = get((void**)&n->db.k, R * n->w_k * 4)) || (rc = get((void**)&n->db.v, R * n->w_v * 4)) ||
+      (rc = get((void**)&n->db.g, R * n->w_g * 4)) || (rc = get((void**)&n->db.beta, R * n->w_b * 4)) || (rc = get((void**)&n->db.o, R * n->w_v * 4)) ||
+      (rc = get((void**)&n->db.za, R * n->w_za * 4)) || (rc = get((void**)&n->db.zg, R * n->w_zg * 4))) return rc;
+  CAI_HIP(hipStreamSynchronize(ctx().stream));
+  n->cap = (int)R;
+  return CAI_OK;
+}
+
+static int ensure_logits(LayeredNet* n, int rows)
+{
+  if (n->logit_cap >= rows) return CAI_OK;
+  const size_t R = (size_t)std::max(rows, DEC_ROWS);
+  CAI_HIP(hipStreamSynchronize(ctx().stream));
+  drop_graphs(n);
+  void* p[] = {n->logits, n->hw, n->am_v, n->am_i, n->best};
+  for (void* q : p) if (q) (void)hipFree(q);
+  n->logits = nullptr; n->hw = nullptr; n->am_v = nullptr; n->am_i = nullptr; n->best = nullptr; n->logit_cap = 0;
+  const int ame = argmax_scratch_entries(n->s.vocab, (int)R);
+  CAI_HIP(hipMalloc((void**)&n->logits, R * n->s.vocab * 4));
+  CAI_HIP(hipMalloc(&n->hw, R * n->wp * n->es));
+  CAI_HIP(hipMalloc((void**)&n->am_v, (size_t)ame * 4));
+  CAI_HIP(hipMalloc((void**)&n->am_i, (size_t)ame * 4));
+  CAI_HIP(hipMalloc((void**)&n->best, R * 4));
+  n->logit_cap = (int)R;
+  return CAI_OK;
+}
+
+int net_create(NetSpec&& spec, int max_tokens, int max_seq, int act_t, LayeredNet** out)
+{
+  LayeredNet* n = new LayeredNet();
+  n->s = std::move(spec);
+  n->act_t = act_t; n->es = act_t == ACT_T_BF16 ? 2 : 4; n->max_seq = max_seq;
+  NetSpec& s = n->s;
+  const int L = (int)s.layers.size();
+  auto add_run = [&](int l, bool again) {
+    NetRun r{l, again, -1, -1};
+    const NetLayer& y = s.layers[l];
+    if (y.kind == MIX_PARALLEL) { r.attn_run = (int)n->pool.attn.size(); n->pool.attn.push_back({y.attn.d}); }
+    r.delta_run = (int)n->pool.delta.size(); n->pool.delta.push_back({y.delta.d});
+    n->runs.push_back(r);
+  };
+  for (int l = 0; l < std::min(s.loop_start, L); l++) add_run(l, false);
+  for (int p = 0; p < s.loop_times; p++)
+    for (int l = s.loop_start; l < s.loop_stop; l++) add_run(l, p > 0 && l == s.loop_start);
+  for (int l = s.loop_stop; l < L; l++) add_run(l, false);
+  n->looped = s.loop_times > 1 && s.loop_stop > s.loop_start;
+  n->wp = pad_to(s.width, LIN_PAD);
+  auto up = [](int& a, int v) { a = std::max(a, v); };
+  for (const NetLayer& y : s.layers) {
+    const DeltaDims& d = y.delta.d;
+    up(n->ld_proj, pad_to((int)y.in->rows, 4));
+    up(n->ld_att, pad_to(d.heads * d.vdim, LIN_PAD));
+    up(n->w_q, d.kv_heads * d.dim); up(n->w_k, d.kv_heads * d.dim); up(n->w_v, d.heads * d.vdim);
+    up(n->w_g, d.channel_decay ? d.heads * d.dim : d.heads); up(n->w_b, d.heads + d.kv_heads);
+    if (d.rank_a) { up(n->ld_ra, pad_to(d.rank_a, LIN_PAD)); up(n->w_za, d.channel_decay ? d.heads * d.dim : d.heads); }
+    if (d.rank_g) { up(n->ld_rg, pad_to(d.rank_g, LIN_PAD)); up(n->w_zg, d.heads * d.vdim); }
+    if (y.gateup) up(n->ld_mid, pad_to(y.ff, LIN_PAD));
+    if (y.kind == MIX_PARALLEL) {
+      n->has_attn = true;
+      up(n->ld_attl, pad_to(y.attn.d.heads * y.attn.d.vdim, LIN_PAD)); up(n->ld_q, y.attn.d.heads * y.attn.d.dim_p);
+    }
+  }
+  const char* ng = getenv("CAIHIP_NO_GRAPH");
+  n->use_graph = !(ng && ng[0] == '1');
+  int rc = n->pool.alloc(max_seq, max_tokens, act_t);
+  if (!rc) rc = ensure_rows(n, DEC_ROWS);
+  if (!rc) rc = ensure_logits(n, DEC_ROWS);
+  if (!rc) {
+    hipError_t e = hipMalloc((void**)&n->d_dec, (9 * DEC_ROWS + 1) * sizeof(int32_t));
+    if (e == hipSuccess) e = hipHostMalloc((void**)&n->h_dec, (9 * DEC_ROWS + 1) * sizeof(int32_t), hipHostMallocDefault);
+    if (e != hipSuccess) rc = hip_fail(e, "layered decoder allocation", __FILE__, __LINE__);
+  }
+  if (rc) { net_destroy(n); return rc; }
+  *out = n;
+  return CAI_OK;
+}
+
+void net_destroy(LayeredNet* n)
+{
+  if (!n) return;
+  if (ctx().ready) (void)hipStreamSynchronize(ctx().stream);
+  drop_graphs(n);
+  free_rows(n);
+  void* p[] = {n->logits, n->hw, n->am_v, n->am_i, n->best, n->d_rows, n->d_dec, n->d_gen};
+  for (void* q : p) if (q) (void)hipFree(q);
+  if (n->h_rows) (void)hipHostFree(n->h_rows);
+  if (n->h_dec) (void)hipHostFree(n->h_dec);
+  n->pool.release_all();
+  net_spec_free(n->s);
+  delete n;
+}
+
+// One step over the rows of `r`.  single: every entry is one row (the decode kernels).  want: device list of the rows whose
+// logits are produced (null: all rows, in order).
+static int enqueue_net(LayeredNet* n, const StepRows& r, bool single, const int32_t* tiles, int n_tiles, const int32_t* want, int n_want)
+{
+  const NetSpec& s = n->s;
+  const int R = r.n_rows, w = s.width, at = n->act_t;
+  auto st = ctx().stream;
+  int rc;
+  auto norm1_of = [&](size_t i) -> const Dyt& { return s.layers[n->runs[i].layer].norm1; };
+  const dim3 eg((unsigned)std::min((w + 255) / 256, 32), R);
+  if (at == ACT_T_BF16) hipLaunchKernelGGL(net_embed_kernel<bf16_t>, eg, dim3(256), 0, st, (const uint16_t*)s.embed->data, (int)s.embed->ld, r.tok, w, n->x, n->x0, (bf16_t*)n->h, (int64_t)n->wp, norm1_of(0));
+  else hipLaunchKernelGGL(net_embed_kernel<float>, eg, dim3(256), 0, st, (const uint16_t*)s.embed->data, (int)s.embed->ld, r.tok, w, n->x, n->x0, (float*)n->h, (int64_t)n->wp, norm1_of(0));
+  for (size_t i = 0; i < n->runs.size(); i++) {
+    const NetRun& run = n->runs[i];
+    const NetLayer& y = s.layers[run.layer];
+    const bool last = i + 1 == n->runs.size();
+    const Dyt& after = last ? s.final_norm : norm1_of(i + 1);
+    const float* add0 = !last && n->runs[i + 1].again ? n->x0 : nullptr;
+    { LinEpi e; e.y = n->proj; e.ldy = n->ld_proj; if ((rc = launch_lin(y.in, at, n->h, n->wp, R, e))) return rc; }
+    // the recurrent mixer
+    const NetDelta& D = y.delta;
+    const DeltaIn din{n->proj, n->ld_proj, D.oq, D.ok, D.ov, D.ob, D.oa, D.og};
+    const SeqPool::DeltaRun& ds = n->pool.delta[run.delta_run];
+    if (single) {
+      if ((rc = delta_single(D.d, din, D.w, ds, r, at, n->att, n->ld_att))) return rc;
+    } else {
+      if (D.d.rank_a) {
+        LinEpi e; e.y = n->db.za; e.ldy = D.w.a2->rows;
+        if ((rc = launch_pack_rows(n->proj, n->ld_proj, D.oa, D.d.rank_a, R, at, n->ra, n->ld_ra)) || (rc = launch_lin(D.w.a2, at, n->ra, n->ld_ra, R, e))) return rc;
+      }
+      if (D.d.rank_g) {
+        LinEpi e; e.y = n->db.zg; e.ldy = D.w.g2->rows;
+        if ((rc = launch_pack_rows(n->proj, n->ld_proj, D.og, D.d.rank_g, R, at, n->rgb, n->ld_rg)) || (rc = launch_lin(D.w.g2, at, n->rgb, n->ld_rg, R, e))) return rc;
+      }
+      if ((rc = delta_prep(D.d, din, D.w, ds, r, n->db)) || (rc = delta_scan(D.d, ds, r, n->db)) || (rc = delta_finish(D.d, din, D.w, ds, r, n->db, at, n->att, n->ld_att))) return rc;
+    }
+    LinEpi res; res.mode = EPI_RESIDUAL; res.y = n->x; res.ldy = w; res.h = n->h; res.ldh = n->wp; res.post = y.norm1b;
+    if (y.gateup) res.next = y.norm2;
+    else { res.next = after; res.add0 = add0; res.ld0 = w; }
+    if (y.kind == MIX_PARALLEL) {
+      const NetAttn& A = y.attn;
+      const AttnIn ain{n->proj, n->ld_proj, A.oq, A.ok, A.ov, A.qn, A.kn};
+      const KvView kv = n->pool.view(run.attn_run);
+      if (!single && (rc = attn_paged_prep(A.d, kv, at, ain, r, n->qbuf))) return rc;
+      if (!single && tiles && attn_paged_prompt_ok(A.d, at)) rc = attn_paged_prompt(A.d, kv, n->qbuf, r, tiles, n_tiles, n->attl, n->ld_attl);
+      else rc = attn_paged_rows(A.d, kv, at, n->qbuf, r, n->attl, n->ld_attl, n->part, single, ain);
+      if (rc) return rc;
+      LinEpi el, er; el.y = n->yl; er.y = n->yr; el.ldy = er.ldy = w;
+      if ((rc = launch_lin(A.out, at, n->attl, n->ld_attl, R, el)) || (rc = launch_lin(D.out, at, n->att, n->ld_att, R, er))) return rc;
+      if (at == ACT_T_BF16) hipLaunchKernelGGL(net_join_kernel<bf16_t>, dim3(R), dim3(256), 0, st, n->yl, n->yr, y.gain_left, y.gain_right, w, s.eps, n->x, res.add0, res.post, res.next, (bf16_t*)n->h, (int64_t)n->wp);
+      else hipLaunchKernelGGL(net_join_kernel<float>, dim3(R), dim3(256), 0, st, n->yl, n->yr, y.gain_left, y.gain_right, w, s.eps, n->x, res.add0, res.post, res.next, (float*)n->h, (int64_t)n->wp);
+    } else if ((rc = launch_lin(D.out, at, n->att, n->ld_att, R, res))) return rc;
+    if (y.gateup) {
+      LinEpi g; g.mode = EPI_GLU; g.h = n->mid; g.ldh = n->ld_mid; g.glu = y.glu;
+      if ((rc = launch_lin(y.gateup, at, n->h, n->wp, R, g))) return rc;
+      res.post = y.norm2b; res.next = after; res.add0 = add0; res.ld0 = w;
+      if ((rc = launch_lin(y.down, at, n->mid, n->ld_mid, R, res))) return rc;
+    }
+  }
+  if (n_want > 0) {
+    const void* hs = n->h;
+    if (want) {
+      if (at == ACT_T_BF16) hipLaunchKernelGGL(net_gather_kernel<bf16_t>, dim3(n_want), dim3(256), 0, st, (const bf16_t*)n->h, want, (int64_t)n->wp, (bf16_t*)n->hw);
+      else hipLaunchKernelGGL(net_gather_kernel<float>, dim3(n_want), dim3(256), 0, st, (const float*)n->h, want, (int64_t)n->wp, (float*)n->hw);
+      hs = n->hw;
+    }
+    LinEpi e; e.y = n->logits; e.ldy = s.vocab;
+    if ((rc = launch_lin(s.head, at, hs, n->wp, n_want, e))) return rc;
+    launch_argmax(n->logits, s.vocab, n_want, n->best, n->am_v, n->am_i);
+  }
+  CAI_HIP(hipGetLastError());
+  return CAI_OK;
+}
+
+static StepRows dec_rows(const LayeredNet* n, int R)
+{
+  int32_t* d = n->d_dec;
+  return StepRows{d, d + DEC_ROWS, d + 2 * DEC_ROWS, d + 3 * DEC_ROWS, d + 4 * DEC_ROWS, d + 5 * DEC_ROWS, R, R};
+}
+
+// `steps` captured steps of R single rows, with the greedy hand-over after each when gen is set (R = 1)
+static int run_captured(LayeredNet* n, int R, int steps, bool gen)
+{
+  auto st = ctx().stream;
+  const StepRows r = dec_rows(n, R);
+  auto body = [&]() -> int {
+    for (int i = 0; i < steps; i++) {
+      const int rc = enqueue_net(n, r, true, nullptr, 0, nullptr, R);
+      if (rc) return rc;
+      if (gen) hipLaunchKernelGGL(net_advance_kernel, dim3(1), dim3(64), 0, st, n->d_dec, n->d_dec + DEC_ROWS, n->best, n->d_gen, n->d_dec + 9 * DEC_ROWS);
+    }
+    return CAI_OK;
+  };
+  if (!n->use_graph) return body();
+  hipGraphExec_t& ge = n->graphs[(gen ? 1000 : 0) + steps * 16 + R];
+  if (!ge) {
+    hipGraph_t g = nullptr;
+    CAI_HIP(hipStreamBeginCapture(st, hipStreamCaptureModeThreadLocal));
+    const int rc = body();
+    const hipError_t e = hipStreamEndCapture(st, &g);
+    if (rc) { if (g) (void)hipGraphDestroy(g); return rc; }
+    if (e != hipSuccess) return hip_fail(e, "hipStreamEndCapture", __FILE__, __LINE__);
+    const hipError_t e2 = hipGraphInstantiate(&ge, g, nullptr, nullptr, 0);
+    (void)hipGraphDestroy(g);
+    if (e2 != hipSuccess) { ge = nullptr; return hip_fail(e2, "hipGraphInstantiate", __FILE__, __LINE__); }
+  }
+  CAI_HIP(hipGraphLaunch(ge, st));
+  return CAI_OK;
+}
+
+int net_step(LayeredNet* n, int n_ent, const int32_t* seq, const int32_t* count, const int32_t* tokens, const uint8_t* want, float* logits_host, int32_t* argmax_host)
+{
+  CAI_REQUIRE(n_ent >= 1 && n_ent <= n->max_seq, "engine step: %d entries for %d sequences", n_ent, n->max_seq);
+  int64_t R64 = 0; bool single = true;
+  std::vector<uint8_t> seen(n->max_seq, 0);
+  for (int e = 0; e < n_ent; e++) {
+    CAI_REQUIRE(seq[e] >= 0 && seq[e] < n->max_seq && !seen[seq[e]], "engine step: entry %d names sequence %d (of %d, each once)", e, seq[e], n->max_seq);
+    CAI_REQUIRE(count[e] >= 1, "engine step: entry %d has %d tokens", e, count[e]);
+    seen[seq[e]] = 1; R64 += count[e]; single = single && count[e] == 1;
+  }
+  CAI_REQUIRE(R64 <= (1 << 17), "engine step: %lld rows", (long long)R64);
+  const int R = (int)R64;
+  for (int i = 0; i < R; i++) CAI_REQUIRE(tokens[i] >= 0 && tokens[i] < n->s.vocab, "engine step: token %d outside vocab %d", tokens[i], n->s.vocab);
+  // pages for all entries or for none
+  if (n->pool.n_pages) {
+    int need = 0;
+    for (int e = 0; e < n_ent; e++) { const auto& q = n->pool.seq[seq[e]]; need += std::max(0, (q.len + count[e] + PAGE_TOKENS - 1) / PAGE_TOKENS - q.end_page); }
+    if (need > (int)n->pool.free_pages.size())
+      return set_error(CAI_ERR_STATE, "engine step: %d more cache pages of %d tokens needed, %zu of %d free", need, PAGE_TOKENS, n->pool.free_pages.size(), n->pool.n_pages);
+  }
+  int rc;
+  for (int e = 0; e < n_ent; e++) if ((rc = n->pool.reserve(seq[e], n->pool.seq[seq[e]].len + count[e]))) return rc;
+  if ((rc = n->pool.upload_table())) return rc;
+  auto st = ctx().stream;
+  std::vector<int32_t> wrows;
+  for (int i = 0; i < R; i++) if (want && want[i]) wrows.push_back(i);
+  const int W = (int)wrows.size();
+  n->row_of.clear();
+  if (single && R <= DEC_ROWS) {
+    int32_t* hd = n->h_dec;
+    for (int e = 0; e < R; e++) {
+      const int pos = n->pool.seq[seq[e]].len;
+      hd[e] = tokens[e]; hd[DEC_ROWS + e] = pos; hd[2 * DEC_ROWS + e] = seq[e]; hd[3 * DEC_ROWS + e] = e; hd[4 * DEC_ROWS + e] = e;
+      int32_t* en = hd + 5 * DEC_ROWS + 4 * e; en[0] = seq[e]; en[1] = e; en[2] = 1; en[3] = pos;
+    }
+    CAI_HIP(hipMemcpyAsync(n->d_dec, hd, 9 * DEC_ROWS * sizeof(int32_t), hipMemcpyHostToDevice, st));
+    if ((rc = run_captured(n, R, 1, false))) return rc;
+    n->row_of = wrows; n->rows_gathered = false;
+  } else {
+    // rows, entries, tiles of the prompt attention kernel, wanted rows
+    std::vector<int32_t> tiles;
+    bool tall = false;
+    for (int e = 0; e < n_ent; e++) { tall = tall || count[e] >= 16; for (int t = 0; t < count[e]; t += ATTN_TILE) { tiles.push_back(e); tiles.push_back(t); } }
+    const size_t need = (size_t)5 * R + 4 * n_ent + tiles.size() + W;
+    if (n->rows_cap < need) {
+      CAI_HIP(hipStreamSynchronize(st));
+      if (n->d_rows) (void)hipFree(n->d_rows);
+      if (n->h_rows) (void)hipHostFree(n->h_rows);
+      n->d_rows = nullptr; n->h_rows = nullptr; n->rows_cap = 0;
+      CAI_HIP(hipMalloc((void**)&n->d_rows, need * 2 * sizeof(int32_t)));
+      CAI_HIP(hipHostMalloc((void**)&n->h_rows, need * 2 * sizeof(int32_t), hipHostMallocDefault));
+      n->rows_cap = need * 2;
+    }
+    if ((rc = ensure_rows(n, R)) || (rc = ensure_logits(n, std::max(W, 1)))) return rc;
+    int32_t* hr = n->h_rows;
+    int32_t* ent = hr + 5 * R;
+    for (int e = 0, i = 0; e < n_ent; e++) {
+      const int pos0 = n->pool.seq[seq[e]].len, r0 = i;
+      ent[4 * e] = seq[e]; ent[4 * e + 1] = r0; ent[4 * e + 2] = count[e]; ent[4 * e + 3] = pos0;
+      for (int t = 0; t < count[e]; t++, i++) { hr[i] = tokens[i]; hr[R + i] = pos0 + t; hr[2 * R + i] = seq[e]; hr[3 * R + i] = r0; hr[4 * R + i] = r0 + count[e] - 1; }
+    }
+    int32_t* ht = ent + 4 * n_ent;
+    std::copy(tiles.begin(), tiles.end(), ht);
+    std::copy(wrows.begin(), wrows.end(), ht + tiles.size());
+    CAI_HIP(hipMemcpyAsync(n->d_rows, hr, need * sizeof(int32_t), hipMemcpyHostToDevice, st));
+    const int32_t* d = n->d_rows;
+    const StepRows r{d, d + R, d + 2 * R, d + 3 * R, d + 4 * R, d + 5 * R, R, n_ent};
+    const int32_t* dt = d + 5 * R + 4 * n_ent;
+    if ((rc = enqueue_net(n, r, false, tall ? dt : nullptr, (int)tiles.size() / 2, dt + tiles.size(), W))) return rc;
+    for (int k = 0; k < W; k++) n->row_of.push_back(k);
+    n->rows_gathered = true;
+  }
+  for (int k = 0; k < W; k++) {
+    // (consecutive logits rows come back in one copy)
+    int k2 = k; while (k2 + 1 < W && n->row_of[k2 + 1] == n->row_of[k2] + 1) k2++;
+    if (logits_host) CAI_HIP(hipMemcpyAsync(logits_host + (size_t)k * n->s.vocab, n->logits + (size_t)n->row_of[k] * n->s.vocab, (size_t)(k2 - k + 1) * n->s.vocab * 4, hipMemcpyDeviceToHost, st));
+    if (argmax_host) CAI_HIP(hipMemcpyAsync(argmax_host + k, n->best + n->row_of[k], (size_t)(k2 - k + 1) * 4, hipMemcpyDeviceToHost, st));
+    k = k2;
+  }
+  CAI_HIP(hipStreamSynchronize(st));
+  for (int e = 0; e < n_ent; e++) { n->pool.seq[seq[e]].len += count[e]; n->pool.trim(seq[e]); }
+  return CAI_OK;
+}
+
+int net_generate(LayeredNet* n, int seq, int32_t first, int n_tokens, int32_t* out_host)
+{
+  auto st = ctx().stream;
+  CAI_REQUIRE(first >= 0 && first < n->s.vocab, "greedy generation: token %d outside vocab %d", first, n->s.vocab);
+  if (n->gen_cap < n_tokens) {
+    CAI_HIP(hipStreamSynchronize(st));
+    if (n->d_gen) (void)hipFree(n->d_gen);
+    n->d_gen = nullptr; n->gen_cap = 0;
+    drop_graphs(n);
+    CAI_HIP(hipMalloc((void**)&n->d_gen, (size_t)std::max(n_tokens, 256) * 4));
+    n->gen_cap = std::max(n_tokens, 256);
+  }
+  SeqPool::Seq& q = n->pool.seq[seq];
+  int32_t* hd = n->h_dec;
+  hd[0] = first; hd[DEC_ROWS] = q.len; hd[2 * DEC_ROWS] = seq; hd[3 * DEC_ROWS] = 0; hd[4 * DEC_ROWS] = 0;
+  hd[5 * DEC_ROWS] = seq; hd[5 * DEC_ROWS + 1] = 0; hd[5 * DEC_ROWS + 2] = 1; hd[5 * DEC_ROWS + 3] = q.len; hd[9 * DEC_ROWS] = 0;
+  CAI_HIP(hipMemcpyAsync(n->d_dec, hd, (9 * DEC_ROWS + 1) * sizeof(int32_t), hipMemcpyHostToDevice, st));
+  for (int i = 0; i < n_tokens;) {
+    // as many tokens as the pool gives pages for, at most a page's worth at a time; pages behind the windows come back in between
+    int m = std::min(std::min(n_tokens - i, PAGE_TOKENS), n->pool.room(seq));
+    if (m < 1) return set_error(CAI_ERR_STATE, "greedy generation: the cache pool is out of pages after %d of %d tokens", i, n_tokens);
+    int rc = n->pool.reserve(seq, q.len + m);
+    if (rc || (rc = n->pool.upload_table())) return rc;
+    for (int k = 0; k < m;) {
+      const int steps = m - k >= GEN_STEPS ? GEN_STEPS : 1;
+      if ((rc = run_captured(n, 1, steps, true))) return rc;
+      k += steps;
+    }
+    q.len += m; i += m;
+    n->pool.trim(seq);
+  }
+  CAI_HIP(hipMemcpyAsync(out_host, n->d_gen, (size_t)n_tokens * 4, hipMemcpyDeviceToHost, st));
+  CAI_HIP(hipStreamSynchronize(st));
+  n->row_of.assign(1, 0); n->rows_gathered = false;
+  return CAI_OK;
+}
+
+int net_len(const LayeredNet* n, int seq) { return n->pool.seq[seq].len; }
+int net_room(const LayeredNet* n, int seq) { return n->pool.room(seq); }
+int net_free_tokens(const LayeredNet* n) { return n->pool.n_pages ? (int)n->pool.free_pages.size() * PAGE_TOKENS : 1 << 30; }
+int net_rows(const LayeredNet* n, int seq) { const auto& q = n->pool.seq[seq]; return n->pool.n_pages ? q.len - q.first_page * PAGE_TOKENS : 0; }
+int net_n_runs(const LayeredNet* n) { return (int)n->runs.size(); }
+int net_reset(LayeredNet* n, int seq) { n->pool.free_seq(seq); return CAI_OK; }
+const NetSpec& net_spec(const LayeredNet* n) { return n->s; }
+float* net_logits(LayeredNet* n, int row) { return row >= 0 && row < (int)n->row_of.size() ? n->logits + (size_t)n->row_of[row] * n->s.vocab : nullptr; }
+
+int net_fork(LayeredNet* n, int src, int dst)
+{
+  if (src == dst) return CAI_OK;
+  const int rc = n->pool.fork(src, dst);
+  if (rc) { n->pool.free_seq(dst); return rc; }
+  CAI_HIP(hipStreamSynchronize(ctx().stream));
+  return CAI_OK;
+}
+
+int net_hidden(LayeredNet* n, int row, float* host)
+{
+  if (row < 0 || row >= (int)n->row_of.size()) return set_error(CAI_ERR_STATE, "hidden state: row %d of the last step's %zu rows with logits", row, n->row_of.size());
+  const char* src = (const char*)(n->rows_gathered ? n->hw : n->h) + (size_t)n->row_of[row] * n->wp * n->es;
+  std::vector<uint32_t> raw(n->s.width);
+  CAI_HIP(hipMemcpyAsync(raw.data(), src, (size_t)n->s.width * n->es, hipMemcpyDeviceToHost, ctx().stream));
+  CAI_HIP(hipStreamSynchronize(ctx().stream));
+  if (n->es == 4) memcpy(host, raw.data(), (size_t)n->s.width * 4);
+  else { const uint16_t* b = (const uint16_t*)raw.data(); for (int i = 0; i < n->s.width; i++) { const uint32_t u = (uint32_t)b[i] << 16; memcpy(host + i, &u, 4); } }
+  return CAI_OK;
+}
+
+int64_t net_weight_bytes(const LayeredNet* n)
+{
+  // a layer that runs several times is streamed as often
+  auto qb = [](const cai_qw_s* w) { return w ? w->algo_bytes : 0; };
+  int64_t b = qb(n->s.head) + n->s.embed->algo_bytes / n->s.embed->rows + 2 * (int64_t)n->s.width * 4;
+  for (const NetRun& r : n->runs) {
+    const NetLayer& y = n->s.layers[r.layer];
+    b += qb(y.in) + qb(y.delta.out) + qb(y.attn.out) + qb(y.delta.w.a2) + qb(y.delta.w.g2) + qb(y.gateup) + qb(y.down) + 8 * (int64_t)n->s.width * 4;
+  }
+  return b;
+}
+
+// ------------------------------------------------------------------------------------------
+// snapshots: live pages and state of one sequence
+// ------------------------------------------------------------------------------------------
+struct NetSnap {
+  int len = 0, first_page = 0, end_page = 0, n_attn = 0, n_delta = 0; int64_t bytes = 0;
+  char* data = nullptr;
+};
+static int64_t snap_bytes(const LayeredNet* n, int pages)
+{
+  int64_t b = 0;
+  for (auto& a : n->pool.attn) b += pages * a.page_elems * (int64_t)n->es;
+  for (auto& d : n->pool.delta) b += (d.s_elems + d.h_elems) * 4;
+  return b;
+}
+// walks the pieces of a sequence in snapshot order: f(device pointer, bytes, offset)
+template <typename F> static int snap_walk(LayeredNet* n, int seq, F f)
+{
+  int64_t off = 0; int rc;
+  const auto& q = n->pool.seq[seq];
+  for (int p = q.first_page; n->pool.n_pages && p < q.end_page; p++)
+    for (auto& a : n->pool.attn) {
+      const size_t sz = (size_t)a.page_elems * n->es;
+      if ((rc = f((char*)a.base + n->pool.table[(size_t)seq * n->pool.n_pages + p % n->pool.n_pages] * sz, sz, off))) return rc;
+      off += sz;
+    }
+  for (auto& d : n->pool.delta) {
+    if ((rc = f((char*)(d.S + seq * d.s_elems), (size_t)d.s_elems * 4, off))) return rc;
+    off += d.s_elems * 4;
+    if ((rc = f((char*)(d.hist + seq * d.h_elems), (size_t)d.h_elems * 4, off))) return rc;
+    off += d.h_elems * 4;
+  }
+  return CAI_OK;
+}
+int net_snapshot(LayeredNet* n, int seq, NetSnap** out)
+{
+  const auto& q = n->pool.seq[seq];
+  NetSnap* s = new NetSnap();
+  s->len = q.len; s->first_page = q.first_page; s->end_page = q.end_page; s->n_attn = (int)n->pool.attn.size(); s->n_delta = (int)n->pool.delta.size();
+  s->bytes = snap_bytes(n, q.end_page - q.first_page);
+  if (hipMalloc((void**)&s->data, (size_t)s->bytes) != hipSuccess) { (void)hipGetLastError(); delete s; return set_error(CAI_ERR_NOMEM, "snapshot: %lld bytes", (long long)q.len); }
+  const int rc = snap_walk(n, seq, [&](char* p, size_t sz, int64_t off) -> int { CAI_HIP(hipMemcpyAsync(s->data + off, p, sz, hipMemcpyDeviceToDevice, ctx().stream)); return CAI_OK; });
+  if (rc) { net_snap_free(s); return rc; }
+  CAI_HIP(hipStreamSynchronize(ctx().stream));
+  *out = s;
+  return CAI_OK;
+}
+int net_restore(LayeredNet* n, int seq, const NetSnap* s)
+{
+  const int pages = s->end_page - s->first_page;
+  CAI_REQUIRE(s->n_attn == (int)n->pool.attn.size() && s->n_delta == (int)n->pool.delta.size() && s->bytes == snap_bytes(n, pages), "restore: the snapshot is of another model");
+  n->pool.free_seq(seq);
+  auto& q = n->pool.seq[seq];
+  q.first_page = q.end_page = s->first_page;
+  int rc = n->pool.reserve(seq, s->end_page * PAGE_TOKENS);
+  if (rc) { q = SeqPool::Seq(); return rc; }
+  q.len = s->len;
+  rc = snap_walk(n, seq, [&](char* p, size_t sz, int64_t off) -> int { CAI_HIP(hipMemcpyAsync(p, s->data + off, sz, hipMemcpyDeviceToDevice, ctx().stream)); return CAI_OK; });
+  if (rc) return rc;
+  CAI_HIP(hipStreamSynchronize(ctx().stream));
+  return CAI_OK;
+}
+void net_snap_free(NetSnap* s) { if (!s) return; if (s->data) (void)hipFree(s->data); delete s; }
+
+}  // namespace cai

@@ -1,0 +1,185 @@
+// Declarations shared by the layered-decoder translation units: 16-bit weights, paged cache and state slots, the gated delta
+// rule, windowed attention over pages (gfx950 only).
+#pragma once
+#include "cai_internal.hpp"
+
+namespace cai {
+
+typedef __bf16 bf16_t;
+typedef bf16_t bf16x8 __attribute__((ext_vector_type(8)));
+typedef float f32x4 __attribute__((ext_vector_type(4)));
+typedef uint32_t u32x4 __attribute__((ext_vector_type(4)));
+
+// Activations between two products are bfloat16 (the serving precision) or float (everything in 32-bit).
+enum { ACT_T_BF16 = 0, ACT_T_F32 = 1 };
+constexpr int LIN_PAD = 64;                 // widths of 16-bit matrices and of the activations they read are padded to this with zeros
+inline int pad_to(int n, int m) { return (n + m - 1) / m * m; }
+
+__device__ __forceinline__ float bf16_lo(uint32_t u) { return __builtin_bit_cast(float, u << 16); }
+__device__ __forceinline__ float bf16_hi(uint32_t u) { return __builtin_bit_cast(float, u & 0xffff0000u); }
+__device__ __forceinline__ uint16_t bf16_bits(float f) { return __builtin_bit_cast(uint16_t, (bf16_t)f); }
+__device__ __forceinline__ float to_f32(float v) { return v; }
+__device__ __forceinline__ float to_f32(bf16_t v) { return (float)v; }
+
+// Dynamic Tanh: y = w * tanh(alpha x) + b.  No statistics, so it lives in the epilogue of whatever produces x.  w == null: none.
+struct Dyt { const float* w = nullptr; const float* b = nullptr; float alpha = 0.0f; };
+__device__ __forceinline__ float dyt(const Dyt& t, float x, int i) { return t.w ? tanhf(t.alpha * x) * t.w[i] + t.b[i] : x; }
+
+// What a linear layer does with its finished sums.
+enum { EPI_STORE = 0, EPI_GLU = 1, EPI_RESIDUAL = 2 };
+enum { GLU_RELU = 0, GLU_SILU = 1 };
+struct LinEpi {
+  int mode = EPI_STORE;
+  float* y = nullptr; int64_t ldy = 0;              // STORE: result; RESIDUAL: the residual stream, updated in place
+  void* h = nullptr; int64_t ldh = 0;               // GLU: act(gate) * up; RESIDUAL: input of the next sublayer (null: none)
+  const float* add0 = nullptr; int64_t ld0 = 0;     // RESIDUAL: added to the stream after the sum (start of a repeated pass)
+  const float* bias = nullptr; int act = CAI_ACT_NONE;   // STORE
+  int glu = GLU_RELU;
+  Dyt post, next;                                   // RESIDUAL: x += post(sum) [+ add0]; h = next(x)
+};
+// Gated matrices interleave their rows in blocks of 16: 16 gate rows, then the 16 up rows of the same outputs.
+__host__ __device__ inline int glu_row(int j, int up) { return (j >> 4) * 32 + up * 16 + (j & 15); }
+
+// y = W x for n_tok activation rows x[t][ldx] (zero padded to LIN_PAD columns, element type act_t); W is a CAI_BF16 matrix.
+int launch_lin(const cai_qw_s* w, int act_t, const void* x, int64_t ldx, int n_tok, const LinEpi& e);
+// two products of one shape class in one launch (same padded width not required): decode rows only
+int launch_pack_rows(const float* x, int64_t ldx, int64_t col0, int cols, int n_tok, int act_t, void* out, int64_t ldo);
+int bf16_dequant_rows(const cai_qw_s* w, int64_t row0, int64_t n_rows, float* out);
+int bf16_linear_f32(const cai_qw_s* w, const float* x, int64_t ldx, int n_tok, float* y, int64_t ldy, int act);   // unpadded float rows in, float rows out
+void bf16_release();
+
+// ------------------------------------------------------------------------------------------
+// Rows of one engine step.  A step is any number of entries (portions of prompts and single tokens) concatenated; per row the
+// token, its position, the sequence slot and the first and last row of its entry; per entry slot, first row, rows, position.
+// ------------------------------------------------------------------------------------------
+struct StepRows {
+  const int32_t *tok, *pos, *slot, *first, *last;   // [n_rows] device
+  const int32_t* ent;                               // [n_ent][4] device: slot, row0, n, pos0
+  int n_rows, n_ent;
+};
+
+// ------------------------------------------------------------------------------------------
+// Paged key/value pool and recurrent-state slots.
+// One page holds PAGE_TOKENS positions of every attention run (layer x pass) of ONE sequence; the pool is sized in tokens over
+// all live sequences.  Page p of a sequence (positions p * PAGE_TOKENS ..) is table[slot][p mod ring]; pages that lie wholly
+// before every window are handed back while the sequence runs on, so a ring of as many entries as the pool has pages never
+// wraps onto a live page.  Recurrent state has one fixed place per (run, slot) and is read as zero at position 0.
+// ------------------------------------------------------------------------------------------
+constexpr int PAGE_TOKENS = 64;
+struct AttnDims {
+  int heads, kv_heads, dim, vdim, window; float scale, eps;
+  int dim_p, vdim_p;                       // row strides in the pool: padded to 8 elements (zero filled)
+};
+struct DeltaDims {
+  int heads, kv_heads, dim, vdim, taps; float eps;
+  int channel_decay;                       // decay per head and key channel instead of per head
+  int sigmoid_gate;                        // output gate sigmoid instead of silu
+  int rank_a, rank_g;                      // low-rank projections in front of decay and gate (0: direct)
+  __host__ __device__ int channels() const { return 2 * kv_heads * dim + heads * vdim; }
+  __host__ __device__ int vdim_p() const { return (vdim + 3) & ~3; }   // row stride of the state
+};
+struct KvView {                            // what a kernel needs to reach one attention run's pages
+  void* base; int64_t page_elems;          // K [kv_head][PAGE_TOKENS][dim_p] then V [kv_head][PAGE_TOKENS][vdim_p]
+  const int32_t* table; int ring;          // [slot][ring]
+  int64_t v_off;                           // elements from a page's K to its V
+};
+struct SeqPool {
+  int n_seq = 0, n_pages = 0, act_t = ACT_T_BF16, keep = 0;   // keep: the widest window (0: no attention run)
+  struct AttnRun { AttnDims d; void* base = nullptr; int64_t page_elems = 0, v_off = 0; };
+  struct DeltaRun { DeltaDims d; float* S = nullptr; float* hist = nullptr; int64_t s_elems = 0, h_elems = 0; };
+  std::vector<AttnRun> attn; std::vector<DeltaRun> delta;
+  int32_t* d_table = nullptr; std::vector<int32_t> table; bool table_dirty = false;
+  std::vector<int> free_pages;
+  struct Seq { int len = 0; int first_page = 0, end_page = 0; };   // live pages [first_page, end_page)
+  std::vector<Seq> seq;
+
+  int alloc(int n_seq, int max_tokens, int act_t);        // after attn / delta list their runs
+  void release_all();
+  int reserve(int s, int new_len);                        // pages for positions [.., new_len)
+  void trim(int s);                                       // hands back the pages no window reaches any more
+  void free_seq(int s);
+  int upload_table();
+  int room(int s) const;                                  // tokens sequence s can still take before the pool is out of pages
+  int fork(int src, int dst);
+  KvView view(int run) const;
+};
+
+// ---- windowed grouped attention over pages (cai_attn_paged.hip) ----
+// rows of proj: q at column oq ([heads][dim]), k at ok, v at ov.  Queries and keys are RMS-normed per head over dim with a
+// shared gain before the score (gain null: not).
+struct AttnIn { const float* proj; int64_t ldp; int oq, ok, ov; const float *qn, *kn; };
+int attn_paged_prep(const AttnDims& d, const KvView& kv, int act_t, const AttnIn& in, const StepRows& r, void* qbuf);     // norms + append; qbuf [row][heads][dim_p]
+int attn_paged_rows(const AttnDims& d, const KvView& kv, int act_t, const void* qbuf, const StepRows& r, void* out, int64_t ldo, float* part, bool single, const AttnIn& in);
+size_t attn_paged_part_floats(const AttnDims& d, int n_rows);
+bool attn_paged_prompt_ok(const AttnDims& d, int act_t);
+int attn_paged_prompt(const AttnDims& d, const KvView& kv, const void* qbuf, const StepRows& r, const int32_t* tiles, int n_tiles, void* out, int64_t ldo);
+constexpr int ATTN_TILE = 64;              // query rows of one entry per work-group of the prompt kernel
+
+// ---- gated delta rule (cai_delta.hip) ----
+// Columns of proj: q, k, v (before the convolution), b (write strength), a (decay logits, or their low-rank input), g likewise.
+struct DeltaIn { const float* proj; int64_t ldp; int oq, ok, ov, ob, oa, og; };
+struct DeltaW {
+  const float *cq, *ck, *cv;               // convolution taps [channels][taps]
+  const float *rate;                       // -exp(A_log) per head
+  const float *dt_bias, *norm;             // [heads] or [heads * dim]; [vdim]
+  const cai_qw_s *a2, *g2;                 // low-rank seconds (CAI_BF16), null when direct
+};
+struct DeltaBuf { float *q, *k, *v, *g, *beta, *o, *za, *zg; };   // per-row scratch of a prompt pass
+int delta_prep(const DeltaDims& d, const DeltaIn& in, const DeltaW& w, const SeqPool::DeltaRun& st, const StepRows& r, const DeltaBuf& b);
+int delta_scan(const DeltaDims& d, const SeqPool::DeltaRun& st, const StepRows& r, const DeltaBuf& b);
+int delta_finish(const DeltaDims& d, const DeltaIn& in, const DeltaW& w, const SeqPool::DeltaRun& st, const StepRows& r, const DeltaBuf& b, int act_t, void* out, int64_t ldo);
+int delta_single(const DeltaDims& d, const DeltaIn& in, const DeltaW& w, const SeqPool::DeltaRun& st, const StepRows& r, int act_t, void* out, int64_t ldo);
+
+// ------------------------------------------------------------------------------------------
+// The layered decoder (cai_layered.hip): layers of different kinds, some run several times.
+// ------------------------------------------------------------------------------------------
+struct NetLinear { cai_qw_s* w = nullptr; };
+struct NetDelta { DeltaDims d{}; DeltaW w{}; int oq = 0, ok = 0, ov = 0, ob = 0, oa = 0, og = 0; cai_qw_s* out = nullptr; };
+struct NetAttn { AttnDims d{}; const float *qn = nullptr, *kn = nullptr; int oq = 0, ok = 0, ov = 0; cai_qw_s* out = nullptr; };
+enum { MIX_DELTA = 0, MIX_PARALLEL = 1 };
+struct NetLayer {
+  int kind = MIX_DELTA;
+  cai_qw_s* in = nullptr;                  // every projection of the layer's input, stacked
+  NetDelta delta; NetAttn attn;            // PARALLEL: both
+  const float *gain_left = nullptr, *gain_right = nullptr;   // PARALLEL: gains of the two outputs' RMS norms
+  Dyt norm1, norm1b, norm2, norm2b;
+  cai_qw_s *gateup = nullptr, *down = nullptr; int ff = 0, glu = GLU_RELU;   // gateup null: no feed-forward
+};
+struct NetRun { int layer; bool again; int attn_run, delta_run; };   // again: the embedding output is added before this run
+struct LayeredNet;
+struct NetSpec {                           // filled by a loader
+  int width = 0, vocab = 0; float eps = 0.0f;
+  cai_qw_s *embed = nullptr, *head = nullptr;
+  Dyt final_norm;
+  std::vector<NetLayer> layers;
+  int loop_start = 0, loop_stop = 0, loop_times = 1;
+  std::vector<cai_qw_s*> weights;          // owned
+  std::vector<void*> vectors;              // owned device memory
+};
+void net_spec_free(NetSpec& s);
+int  net_create(NetSpec&& s, int max_tokens, int max_seq, int act_t, LayeredNet** out);
+void net_destroy(LayeredNet* n);
+// One engine step over any entries.  want[i] != 0: logits of row i are produced, in row order; *_host may be null.
+int  net_step(LayeredNet* n, int n_ent, const int32_t* seq, const int32_t* count, const int32_t* tokens, const uint8_t* want,
+              float* logits_host, int32_t* argmax_host);
+int  net_generate(LayeredNet* n, int seq, int32_t first, int n_tokens, int32_t* out_host);
+int  net_len(const LayeredNet* n, int seq);
+int  net_room(const LayeredNet* n, int seq);
+int  net_free_tokens(const LayeredNet* n);
+int  net_rows(const LayeredNet* n, int seq);
+int  net_n_runs(const LayeredNet* n);
+int  net_reset(LayeredNet* n, int seq);
+int  net_fork(LayeredNet* n, int src, int dst);
+float* net_logits(LayeredNet* n, int row);         // device row of the last step (null: no such row)
+int  net_hidden(LayeredNet* n, int row, float* host);
+const NetSpec& net_spec(const LayeredNet* n);
+int64_t net_weight_bytes(const LayeredNet* n);
+struct NetSnap;
+int  net_snapshot(LayeredNet* n, int seq, NetSnap** out);
+int  net_restore(LayeredNet* n, int seq, const NetSnap* s);
+void net_snap_free(NetSnap* s);
+
+// a decoder around a net (cai_decoder.hip), and the model registry's entry (cai_models.hip)
+int decoder_from_net(LayeredNet* n, int max_tokens, int max_seq, cai_decoder_s** out);
+
+}  // namespace cai

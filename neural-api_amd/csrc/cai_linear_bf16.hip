@@ -1,0 +1,391 @@
+// Linear layers over bfloat16 weights: a streaming matrix-vector kernel for up to eight activation rows (decode) and a
+// matrix-core kernel for more (prompts and mixed batches).
+//
+// Weights are row-major [out][padded in], the padding zero.  Activations are bfloat16 (matrix cores multiply bfloat16 with
+// 32-bit sums) or float; with float activations the weights are widened exactly and every product and sum is 32-bit (the
+// 16x16x4 float form of the matrix cores).  What follows the product runs in its epilogue on the 32-bit sums: bias and
+// activation, act(gate) * up of a gated pair, or the residual update with the Dynamic Tanh before and after it - that norm
+// has no statistics, so a sublayer needs no launch besides its products and its mixer.
+#include "cai_layered.hpp"
+#include "cai_gemv_common.hpp"
+
+#include <algorithm>
+
+namespace cai {
+
+__device__ __forceinline__ float glu_act(float g, int kind) { return kind == GLU_SILU ? silu_mul(1.0f, g) : fmaxf(g, 0.0f); }
+
+template <typename AT> __device__ __forceinline__ void put_act(void* p, int64_t i, float v)
+{
+  if constexpr (sizeof(AT) == 2) reinterpret_cast<uint16_t*>(p)[i] = bf16_bits(v);
+  else reinterpret_cast<float*>(p)[i] = v;
+}
+
+// one finished sum of STORE / RESIDUAL
+template <typename AT> __device__ __forceinline__ void epi_one(const LinEpi& e, int n, int t, float v)
+{
+  if (e.mode == EPI_STORE) {
+    if (e.bias) v += e.bias[n];
+    e.y[t * e.ldy + n] = act_apply(v, e.act);
+  } else {
+    float x = e.y[t * e.ldy + n] + dyt(e.post, v, n);
+    if (e.add0) x += e.add0[t * e.ld0 + n];
+    e.y[t * e.ldy + n] = x;
+    if (e.h) put_act<AT>(e.h, t * e.ldh + n, dyt(e.next, x, n));
+  }
+}
+
+// ------------------------------------------------------------------------------------------
+// Decode: NB activation rows.  A wave owns R weight rows (of a gated matrix R / 2 outputs) or, with ksplit > 1, every ksplit-th
+// 512-wide turn of them; the activations are staged in LDS as float in panels, the weights stream past once.
+// ------------------------------------------------------------------------------------------
+constexpr int GV_WAVES = 8;
+constexpr int GV_LDS = 16384;              // floats of staged activations
+
+template <typename AT, int NB, int R>
+__global__ __launch_bounds__(64 * GV_WAVES) void gemv_bf16(const uint16_t* __restrict__ W, const AT* __restrict__ x, int n_rows, int ldw, int64_t ldx, int ksplit, LinEpi e)
+{
+  __shared__ float xs[GV_LDS];
+  __shared__ float part[GV_WAVES][R * NB];
+  const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+  const int ks = wave % ksplit;
+  const int grp = blockIdx.x * (GV_WAVES / ksplit) + wave / ksplit;
+  constexpr int PANEL = GV_LDS / NB / 512 * 512;
+  const bool glu = e.mode == EPI_GLU;
+  const uint16_t* row[R];
+#pragma unroll
+  for (int i = 0; i < R; i++) {
+    int r = glu ? glu_row(grp * (R / 2) + i % (R / 2 > 0 ? R / 2 : 1), i / (R / 2 > 0 ? R / 2 : 1)) : grp * R + i;
+    row[i] = W + (int64_t)min(r, n_rows - 1) * ldw;
+  }
+  float acc[R][NB];
+#pragma unroll
+  for (int i = 0; i < R; i++)
+#pragma unroll
+    for (int b = 0; b < NB; b++) acc[i][b] = 0.0f;
+  for (int p0 = 0; p0 < ldw; p0 += PANEL) {
+    const int pk = min(PANEL, ldw - p0), pk512 = (pk + 511) / 512 * 512;
+    // eight weights a turn ahead of the staging: the first requests are out while the activations arrive
+    u32x4 w0[R];
+    const int k_first = ks * 512 + lane * 8;
+#pragma unroll
+    for (int i = 0; i < R; i++) w0[i] = *reinterpret_cast<const u32x4*>(row[i] + p0 + (k_first < pk ? k_first : 0));
+    if (p0) __syncthreads();
+#pragma unroll
+    for (int b = 0; b < NB; b++)
+      for (int k = threadIdx.x * 8; k < pk512; k += 64 * GV_WAVES * 8) {
+        float v[8];
+        if (k < pk) {
+          if constexpr (sizeof(AT) == 2) {
+            const u32x4 u = *reinterpret_cast<const u32x4*>(x + b * ldx + p0 + k);
+#pragma unroll
+            for (int j = 0; j < 4; j++) { v[2 * j] = bf16_lo(u[j]); v[2 * j + 1] = bf16_hi(u[j]); }
+          } else {
+            const f32x4 a = *reinterpret_cast<const f32x4*>(x + b * ldx + p0 + k), c = *reinterpret_cast<const f32x4*>(x + b * ldx + p0 + k + 4);
+#pragma unroll
+            for (int j = 0; j < 4; j++) { v[j] = a[j]; v[4 + j] = c[j]; }
+          }
+        } else {
+#pragma unroll
+          for (int j = 0; j < 8; j++) v[j] = 0.0f;
+        }
+        // a turn of 512 values is kept as two halves of 256 (four values a lane each), so that a wave's 16-byte reads are contiguous
+        float* o = xs + b * PANEL + (k >> 9) * 512 + ((k >> 3) & 63) * 4;
+        *reinterpret_cast<f32x4*>(o) = f32x4{v[0], v[1], v[2], v[3]};
+        *reinterpret_cast<f32x4*>(o + 256) = f32x4{v[4], v[5], v[6], v[7]};
+      }
+    __syncthreads();
+    for (int k0 = ks * 512; k0 < pk512; k0 += ksplit * 512) {
+      u32x4 w1[R];
+      const int kn = k0 + ksplit * 512 + lane * 8;
+#pragma unroll
+      for (int i = 0; i < R; i++) w1[i] = *reinterpret_cast<const u32x4*>(row[i] + p0 + (kn < pk ? kn : 0));
+#pragma unroll
+      for (int b = 0; b < NB; b++) {
+        const f32x4 xa = *reinterpret_cast<const f32x4*>(xs + b * PANEL + k0 + lane * 4);
+        const f32x4 xb = *reinterpret_cast<const f32x4*>(xs + b * PANEL + k0 + 256 + lane * 4);
+#pragma unroll
+        for (int i = 0; i < R; i++) {
+          float s = acc[i][b];
+          s = fmaf(bf16_lo(w0[i][0]), xa[0], s); s = fmaf(bf16_hi(w0[i][0]), xa[1], s);
+          s = fmaf(bf16_lo(w0[i][1]), xa[2], s); s = fmaf(bf16_hi(w0[i][1]), xa[3], s);
+          s = fmaf(bf16_lo(w0[i][2]), xb[0], s); s = fmaf(bf16_hi(w0[i][2]), xb[1], s);
+          s = fmaf(bf16_lo(w0[i][3]), xb[2], s); s = fmaf(bf16_hi(w0[i][3]), xb[3], s);
+          acc[i][b] = s;
+        }
+      }
+#pragma unroll
+      for (int i = 0; i < R; i++) w0[i] = w1[i];
+    }
+  }
+  float mine = 0.0f;                       // lane i * NB + b holds the sum of row i, activation b
+#pragma unroll
+  for (int i = 0; i < R; i++)
+#pragma unroll
+    for (int b = 0; b < NB; b++) {
+      const float t = wave_sum(acc[i][b]);
+      const float s = __builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, t), 63));
+      if (lane == i * NB + b) mine = s;
+    }
+  if (ksplit > 1) {
+    if (lane < R * NB) part[wave][lane] = mine;
+    __syncthreads();
+    if (ks != 0) return;
+    if (lane < R * NB) for (int j = 1; j < ksplit; j++) mine += part[wave + j][lane];
+  }
+  const int i = lane / NB, b = lane % NB;
+  if (glu) {
+    const float up = __shfl(mine, lane + R / 2 * NB);
+    const int j = grp * (R / 2) + i;
+    if (i < R / 2 && glu_row(j, 0) < n_rows) put_act<AT>(e.h, b * e.ldh + j, glu_act(mine, e.glu) * up);
+  } else if (i < R && grp * R + i < n_rows) epi_one<AT>(e, grp * R + i, b, mine);
+}
+
+// ------------------------------------------------------------------------------------------
+// Prompts: C^T tile = W tile x activations^T on the matrix cores; a lane ends with four consecutive outputs of one token.
+// Both operand tiles are 128 bytes deep per row (64 bfloat16 or 32 floats), double buffered in LDS; the 16-byte chunks of a row
+// are stored at chunk ^ (row & 7), which makes the fragment reads conflict-free.
+// ------------------------------------------------------------------------------------------
+template <typename AT, int BM, int BN, int WM, int WN>
+__global__ __launch_bounds__(64 * WM * WN) void gemm_bf16(const uint16_t* __restrict__ W, const AT* __restrict__ X, int n_rows, int ldw, int64_t ldx, int n_tok, int tiles_m, int n_tiles, LinEpi e)
+{
+  constexpr int NT = 64 * WM * WN;
+  constexpr int BK = 128 / (int)sizeof(AT);          // elements per row of a tile
+  constexpr int TM = BM / WM / 16, TN = BN / WN / 16;
+  constexpr int CA = BM * 8 / NT, CW = BN * 8 / NT;  // 16-byte chunks per thread
+  static_assert(CA >= 1 && CW >= 1 && BM * 8 % NT == 0 && BN * 8 % NT == 0 && TN % 2 == 0, "tile shape");
+  __shared__ u32x4 sx[2][BM * 8], sw[2][BN * 8];
+  // consecutive work-groups go to different XCDs: give each XCD a contiguous run of tiles, token tiles fastest, so that the
+  // work-groups of an XCD share weight rows in its L2
+  int tile;
+  {
+    const int xcd = blockIdx.x & 7, per = n_tiles >> 3, rem = n_tiles & 7;
+    tile = xcd * per + min(xcd, rem) + (blockIdx.x >> 3);
+  }
+  const int m0 = tile % tiles_m * BM, n0 = tile / tiles_m * BN;
+  const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int wm = wave / WN * (BM / WM), wn = wave % WN * (BN / WN);
+  const AT* xp[CA]; const uint16_t* wp[CW];
+#pragma unroll
+  for (int i = 0; i < CA; i++) { const int c = tid + i * NT; xp[i] = X + (int64_t)min(m0 + (c >> 3), n_tok - 1) * ldx + (c & 7) * (16 / sizeof(AT)); }
+#pragma unroll
+  for (int i = 0; i < CW; i++) { const int c = tid + i * NT; wp[i] = W + (int64_t)min(n0 + (c >> 3), n_rows - 1) * ldw + (c & 7) * (16 / sizeof(AT)); }
+  u32x4 rx[CA], rw[CW];
+  auto fetch = [&](int k) {
+#pragma unroll
+    for (int i = 0; i < CA; i++) rx[i] = *reinterpret_cast<const u32x4*>(xp[i] + k);
+#pragma unroll
+    for (int i = 0; i < CW; i++) {
+      if constexpr (sizeof(AT) == 2) rw[i] = *reinterpret_cast<const u32x4*>(wp[i] + k);
+      else {
+        const uint2 u = *reinterpret_cast<const uint2*>(wp[i] + k);
+        rw[i] = u32x4{u.x << 16, u.x & 0xffff0000u, u.y << 16, u.y & 0xffff0000u};
+      }
+    }
+  };
+  auto stash = [&](int s) {
+#pragma unroll
+    for (int i = 0; i < CA; i++) { const int c = tid + i * NT, r = c >> 3; sx[s][r * 8 + ((c & 7) ^ (r & 7))] = rx[i]; }
+#pragma unroll
+    for (int i = 0; i < CW; i++) { const int c = tid + i * NT, r = c >> 3; sw[s][r * 8 + ((c & 7) ^ (r & 7))] = rw[i]; }
+  };
+  f32x4 acc[TN][TM];
+#pragma unroll
+  for (int j = 0; j < TN; j++)
+#pragma unroll
+    for (int i = 0; i < TM; i++) acc[j][i] = f32x4{0.0f, 0.0f, 0.0f, 0.0f};
+  const int fr = lane & 15, fc = lane >> 4;
+  fetch(0); stash(0);
+  __syncthreads();
+  const int nk = ldw / BK;
+  for (int kt = 0; kt < nk; kt++) {
+    const int s = kt & 1;
+    if (kt + 1 < nk) fetch((kt + 1) * BK);
+#pragma unroll
+    for (int kk = 0; kk < 2; kk++) {
+      u32x4 fx[TM], fw[TN];
+#pragma unroll
+      for (int i = 0; i < TM; i++) { const int r = wm + i * 16 + fr; fx[i] = sx[s][r * 8 + ((kk * 4 + fc) ^ (r & 7))]; }
+#pragma unroll
+      for (int j = 0; j < TN; j++) { const int r = wn + j * 16 + fr; fw[j] = sw[s][r * 8 + ((kk * 4 + fc) ^ (r & 7))]; }
+#pragma unroll
+      for (int j = 0; j < TN; j++)
+#pragma unroll
+        for (int i = 0; i < TM; i++) {
+          if constexpr (sizeof(AT) == 2) {
+            acc[j][i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, fw[j]), __builtin_bit_cast(bf16x8, fx[i]), acc[j][i], 0, 0, 0);
+          } else {
+            // the k index a lane group contributes at step q is 4 * group + q of the 16-wide block, for both operands alike
+            const f32x4 a = __builtin_bit_cast(f32x4, fw[j]), b = __builtin_bit_cast(f32x4, fx[i]);
+#pragma unroll
+            for (int q = 0; q < 4; q++) acc[j][i] = __builtin_amdgcn_mfma_f32_16x16x4f32(a[q], b[q], acc[j][i], 0, 0, 0);
+          }
+        }
+    }
+    if (kt + 1 < nk) stash(s ^ 1);
+    __syncthreads();
+  }
+#pragma unroll
+  for (int i = 0; i < TM; i++) {
+    const int t = m0 + wm + i * 16 + fr;
+    if (t >= n_tok) continue;
+    if (e.mode == EPI_GLU) {
+#pragma unroll
+      for (int j = 0; j < TN; j += 2) {
+        const int n = n0 + wn + j * 16;                // block of 16 gate rows; its up rows are the next fragment
+        if (n >= n_rows) continue;
+        const int o = (n >> 1) + fc * 4;
+        float v[4];
+#pragma unroll
+        for (int q = 0; q < 4; q++) v[q] = glu_act(acc[j][i][q], e.glu) * acc[j + 1][i][q];
+        if constexpr (sizeof(AT) == 2)
+          *reinterpret_cast<uint2*>(reinterpret_cast<uint16_t*>(e.h) + t * e.ldh + o) = make_uint2(bf16_bits(v[0]) | (uint32_t)bf16_bits(v[1]) << 16, bf16_bits(v[2]) | (uint32_t)bf16_bits(v[3]) << 16);
+        else *reinterpret_cast<f32x4*>(reinterpret_cast<float*>(e.h) + t * e.ldh + o) = f32x4{v[0], v[1], v[2], v[3]};
+      }
+      continue;
+    }
+#pragma unroll
+    for (int j = 0; j < TN; j++) {
+      const int n = n0 + wn + j * 16 + fc * 4;
+      if (n >= n_rows) continue;
+      if (n + 3 < n_rows && (e.ldy & 3) == 0 && (e.ldh & 3) == 0 && (e.ld0 & 3) == 0) {
+        f32x4* yp = reinterpret_cast<f32x4*>(e.y + t * e.ldy + n);
+        f32x4 v = acc[j][i];
+        if (e.mode == EPI_STORE) {
+          if (e.bias || e.act != CAI_ACT_NONE) {
+#pragma unroll
+            for (int q = 0; q < 4; q++) v[q] = act_apply(e.bias ? v[q] + e.bias[n + q] : v[q], e.act);
+          }
+          *yp = v;
+        } else {
+          f32x4 x = *yp;
+#pragma unroll
+          for (int q = 0; q < 4; q++) x[q] += dyt(e.post, v[q], n + q);
+          if (e.add0) x += *reinterpret_cast<const f32x4*>(e.add0 + t * e.ld0 + n);
+          *yp = x;
+          if (e.h) {
+#pragma unroll
+            for (int q = 0; q < 4; q++) v[q] = dyt(e.next, x[q], n + q);
+            if constexpr (sizeof(AT) == 2)
+              *reinterpret_cast<uint2*>(reinterpret_cast<uint16_t*>(e.h) + t * e.ldh + n) = make_uint2(bf16_bits(v[0]) | (uint32_t)bf16_bits(v[1]) << 16, bf16_bits(v[2]) | (uint32_t)bf16_bits(v[3]) << 16);
+            else *reinterpret_cast<f32x4*>(reinterpret_cast<float*>(e.h) + t * e.ldh + n) = v;
+          }
+        }
+      } else {
+#pragma unroll
+        for (int q = 0; q < 4; q++) if (n + q < n_rows) epi_one<AT>(e, n + q, t, acc[j][i][q]);
+      }
+    }
+  }
+}
+
+template <typename AT, int BM, int BN, int WM, int WN>
+static void run_gemm(const cai_qw_s* w, const AT* x, int64_t ldx, int n_tok, const LinEpi& e)
+{
+  const int tm = (n_tok + BM - 1) / BM, tn = ((int)w->rows + BN - 1) / BN;
+  hipLaunchKernelGGL((gemm_bf16<AT, BM, BN, WM, WN>), dim3(tm * tn), dim3(64 * WM * WN), 0, ctx().stream,
+                     (const uint16_t*)w->data, x, (int)w->rows, (int)w->ld, ldx, n_tok, tm, tm * tn, e);
+}
+
+template <typename AT, int NB>
+static void run_gemv(const cai_qw_s* w, const AT* x, int64_t ldx, const LinEpi& e)
+{
+  const int rows = (int)w->rows, turns = ((int)w->ld + 511) / 512;
+  // four rows a wave once that still leaves every CU eight waves; fewer rows, then a split of the row, for small matrices
+  const int want = ctx().n_cu * 8;
+  const bool four = rows / 4 >= want;
+  const int groups = e.mode == EPI_GLU ? (four ? (rows / 2 + 1) / 2 : rows / 2) : (rows + (four ? 3 : 1)) / (four ? 4 : 2);
+  int ks = 1;
+  while (ks < GV_WAVES && ks * 2 <= turns && groups * ks * 2 <= want * 2) ks *= 2;
+  const int per = GV_WAVES / ks;
+  const dim3 grid((groups + per - 1) / per), blk(64 * GV_WAVES);
+  if (four) hipLaunchKernelGGL((gemv_bf16<AT, NB, 4>), grid, blk, 0, ctx().stream, (const uint16_t*)w->data, x, rows, (int)w->ld, ldx, ks, e);
+  else hipLaunchKernelGGL((gemv_bf16<AT, NB, 2>), grid, blk, 0, ctx().stream, (const uint16_t*)w->data, x, rows, (int)w->ld, ldx, ks, e);
+}
+
+template <typename AT>
+static int run_lin(const cai_qw_s* w, const AT* x, int64_t ldx, int n_tok, const LinEpi& e)
+{
+  if (n_tok <= 8) {
+    switch (n_tok) {
+      case 1: run_gemv<AT, 1>(w, x, ldx, e); break;
+      case 2: run_gemv<AT, 2>(w, x, ldx, e); break;
+      case 3: run_gemv<AT, 3>(w, x, ldx, e); break;
+      case 4: run_gemv<AT, 4>(w, x, ldx, e); break;
+      case 5: run_gemv<AT, 5>(w, x, ldx, e); break;
+      case 6: run_gemv<AT, 6>(w, x, ldx, e); break;
+      case 7: run_gemv<AT, 7>(w, x, ldx, e); break;
+      default: run_gemv<AT, 8>(w, x, ldx, e); break;
+    }
+    return CAI_OK;
+  }
+  auto tiles = [&](int bm, int bn) { return (int64_t)((n_tok + bm - 1) / bm) * ((w->rows + bn - 1) / bn); };
+  if (n_tok > 64 && tiles(128, 128) >= ctx().n_cu) run_gemm<AT, 128, 128, 2, 2>(w, x, ldx, n_tok, e);
+  else if (n_tok > 32 && tiles(64, 64) >= ctx().n_cu) run_gemm<AT, 64, 64, 2, 2>(w, x, ldx, n_tok, e);
+  else run_gemm<AT, 32, 64, 2, 2>(w, x, ldx, n_tok, e);
+  return CAI_OK;
+}
+
+int launch_lin(const cai_qw_s* w, int act_t, const void* x, int64_t ldx, int n_tok, const LinEpi& e)
+{
+  CAI_REQUIRE(w->qtype == CAI_BF16 && n_tok >= 1 && ldx >= w->ld, "bf16 linear layer: %lld columns need activation rows of %lld, got %lld", (long long)w->cols, (long long)w->ld, (long long)ldx);
+  CAI_REQUIRE(e.mode != EPI_GLU || w->rows % 32 == 0, "bf16 linear layer: a gated matrix needs whole blocks of 32 rows");
+  const int rc = act_t == ACT_T_BF16 ? run_lin<bf16_t>(w, (const bf16_t*)x, ldx, n_tok, e) : run_lin<float>(w, (const float*)x, ldx, n_tok, e);
+  if (rc) return rc;
+  CAI_HIP(hipGetLastError());
+  return CAI_OK;
+}
+
+// ------------------------------------------------------------------------------------------
+// float columns [col0, col0 + cols) of x -> padded activation rows of the chosen type
+// ------------------------------------------------------------------------------------------
+template <typename AT>
+__global__ __launch_bounds__(256) void pack_rows_kernel(const float* x, int64_t ldx, int64_t col0, int cols, void* out, int64_t ldo)
+{
+  const int t = blockIdx.y;
+  for (int i = blockIdx.x * 256 + threadIdx.x; i < ldo; i += gridDim.x * 256)
+    put_act<AT>(out, t * ldo + i, i < cols ? x[t * ldx + col0 + i] : 0.0f);
+}
+int launch_pack_rows(const float* x, int64_t ldx, int64_t col0, int cols, int n_tok, int act_t, void* out, int64_t ldo)
+{
+  const dim3 grid((unsigned)std::min<int64_t>((ldo + 255) / 256, 32), n_tok);
+  if (act_t == ACT_T_BF16) hipLaunchKernelGGL(pack_rows_kernel<bf16_t>, grid, dim3(256), 0, ctx().stream, x, ldx, col0, cols, out, ldo);
+  else hipLaunchKernelGGL(pack_rows_kernel<float>, grid, dim3(256), 0, ctx().stream, x, ldx, col0, cols, out, ldo);
+  CAI_HIP(hipGetLastError());
+  return CAI_OK;
+}
+
+__global__ __launch_bounds__(256) void bf16_rows_kernel(const uint16_t* w, int64_t ld, int64_t cols, int64_t row0, float* out)
+{
+  const int64_t r = blockIdx.y;
+  for (int64_t i = blockIdx.x * 256 + threadIdx.x; i < cols; i += (int64_t)gridDim.x * 256)
+    out[r * cols + i] = __builtin_bit_cast(float, (uint32_t)w[(row0 + r) * ld + i] << 16);
+}
+int bf16_dequant_rows(const cai_qw_s* w, int64_t row0, int64_t n_rows, float* out)
+{
+  for (int64_t r = 0; r < n_rows; r += 32768)
+    hipLaunchKernelGGL(bf16_rows_kernel, dim3((unsigned)std::min<int64_t>((w->cols + 255) / 256, 32), (unsigned)std::min<int64_t>(n_rows - r, 32768)), dim3(256), 0, ctx().stream,
+                       (const uint16_t*)w->data, w->ld, w->cols, row0 + r, out + r * w->cols);
+  CAI_HIP(hipGetLastError());
+  return CAI_OK;
+}
+
+// the stand-alone products (cai_qgemv, cai_qgemm) take unpadded float rows
+static float* g_pack = nullptr; static size_t g_pack_cap = 0;
+void bf16_release() { if (g_pack) (void)hipFree(g_pack); g_pack = nullptr; g_pack_cap = 0; }
+int bf16_linear_f32(const cai_qw_s* w, const float* x, int64_t ldx, int n_tok, float* y, int64_t ldy, int act)
+{
+  const size_t need = (size_t)n_tok * w->ld;
+  if (g_pack_cap < need) {
+    CAI_HIP(hipStreamSynchronize(ctx().stream));
+    bf16_release();
+    CAI_HIP(hipMalloc((void**)&g_pack, need * 4));
+    g_pack_cap = need;
+  }
+  int rc = launch_pack_rows(x, ldx, 0, (int)w->cols, n_tok, ACT_T_F32, g_pack, w->ld);
+  if (rc) return rc;
+  LinEpi e; e.y = y; e.ldy = ldy; e.bias = w->bias; e.act = act;
+  return launch_lin(w, ACT_T_F32, g_pack, w->ld, n_tok, e);
+}
+
+}  // namespace cai

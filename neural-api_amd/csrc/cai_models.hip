@@ -1,0 +1,323 @@
+// Model registry: a folder with config.json and model.safetensors is loaded by the builder registered under its
+// "architecture"; a file is a GGUF container (cai_gguf.hip).  Host code only.
+//
+// A builder reads every size from the configuration or from a tensor's shape, checks the two against each other before anything
+// is sized from them, stacks the projections that share an input into one matrix, and describes the layers to the layered
+// decoder.
+#include "cai_layered.hpp"
+#include "cai_json.hpp"
+
+#include <fcntl.h>
+#include <string.h>
+#include <sys/mman.h>
+#include <sys/stat.h>
+#include <unistd.h>
+
+#include <map>
+#include <string>
+
+namespace cai {
+
+namespace {
+
+// ------------------------------------------------------------------------------------------
+// safetensors: an 8-byte little-endian header length, the JSON header (name -> dtype, shape, data_offsets), the data
+// ------------------------------------------------------------------------------------------
+struct StTensor { std::string dtype; std::vector<int64_t> shape; const uint8_t* data = nullptr; int64_t bytes = 0, elems = 1; };
+
+struct SafeTensors {
+  void* base = MAP_FAILED; size_t size = 0;
+  std::map<std::string, StTensor> t;
+  ~SafeTensors() { if (base != MAP_FAILED) munmap(base, size); }
+
+  int open(const std::string& path)
+  {
+    const int fd = ::open(path.c_str(), O_RDONLY | O_CLOEXEC);
+    if (fd < 0) return set_error(CAI_ERR_INVALID, "safetensors: cannot open %s", path.c_str());
+    struct stat sb;
+    if (fstat(fd, &sb) || sb.st_size < 8) { close(fd); return set_error(CAI_ERR_INVALID, "safetensors: %s is too short", path.c_str()); }
+    size = (size_t)sb.st_size;
+    base = mmap(nullptr, size, PROT_READ, MAP_PRIVATE, fd, 0);
+    close(fd);
+    if (base == MAP_FAILED) return set_error(CAI_ERR_INVALID, "safetensors: cannot map %s", path.c_str());
+    const uint8_t* p = (const uint8_t*)base;
+    uint64_t hl = 0;
+    memcpy(&hl, p, 8);
+    if (hl > size - 8) return set_error(CAI_ERR_INVALID, "safetensors: header of %llu bytes in a file of %zu: %s", (unsigned long long)hl, size, path.c_str());
+    Json j; std::string err;
+    if (!JsonReader::parse((const char*)p + 8, (size_t)hl, j, err) || j.kind != Json::OBJ) return set_error(CAI_ERR_INVALID, "safetensors: %s: %s", err.c_str(), path.c_str());
+    const uint64_t data0 = 8 + hl, room = size - data0;
+    for (auto& kv : j.obj) {
+      if (kv.first == "__metadata__") continue;
+      const Json *dt = kv.second.get("dtype"), *sh = kv.second.get("shape"), *of = kv.second.get("data_offsets");
+      bool ok = dt && dt->kind == Json::STR && sh && sh->kind == Json::ARR && of && of->kind == Json::ARR && of->arr.size() == 2 && of->arr[0].is_int() && of->arr[1].is_int();
+      StTensor x;
+      if (ok) {
+        x.dtype = dt->str;
+        for (auto& d : sh->arr) {
+          ok = ok && d.is_int() && d.num >= 0 && d.num < 2147483648.0 && x.elems < ((int64_t)1 << 40);
+          if (ok) { x.shape.push_back((int64_t)d.num); x.elems *= (int64_t)d.num; }
+        }
+        const double a = of->arr[0].num, b = of->arr[1].num;
+        const int64_t es = x.dtype == "BF16" || x.dtype == "F16" ? 2 : x.dtype == "F32" || x.dtype == "I32" ? 4 : 0;
+        ok = ok && a >= 0 && b >= a && b <= (double)room && es > 0 && (int64_t)(b - a) == x.elems * es;
+        if (ok) { x.data = p + data0 + (uint64_t)a; x.bytes = (int64_t)(b - a); }
+      }
+      if (!ok) return set_error(CAI_ERR_INVALID, "safetensors: tensor \"%s\" has a bad type, shape or range: %s", kv.first.c_str(), path.c_str());
+      if (!t.emplace(kv.first, x).second) return set_error(CAI_ERR_INVALID, "safetensors: tensor \"%s\" is listed twice: %s", kv.first.c_str(), path.c_str());
+    }
+    return CAI_OK;
+  }
+};
+
+// ------------------------------------------------------------------------------------------
+// what every builder uses: checked access to configuration and tensors.  The first failure sticks in rc.
+// ------------------------------------------------------------------------------------------
+struct Builder {
+  SafeTensors st;
+  NetSpec s;
+  int rc = CAI_OK;
+
+  bool fail(const std::string& m) { if (!rc) rc = set_error(CAI_ERR_INVALID, "model: %s", m.c_str()); return false; }
+
+  int integer(const Json* o, const char* key, const std::string& where, int lo = 1, int hi = 1 << 24)
+  {
+    const Json* v = o ? o->get(key) : nullptr;
+    if (!v || !v->is_int() || v->num < lo || v->num > hi) { fail("\"" + where + key + "\" is missing or not an integer in " + std::to_string(lo) + ".." + std::to_string(hi)); return lo; }
+    return (int)v->num;
+  }
+  float number(const Json* o, const char* key, const std::string& where)
+  {
+    const Json* v = o ? o->get(key) : nullptr;
+    if (!v || v->kind != Json::NUM) { fail("\"" + where + key + "\" is missing or not a number"); return 0.0f; }
+    return (float)v->num;
+  }
+  const StTensor* tensor(const std::string& name, std::vector<int64_t> shape)
+  {
+    auto it = st.t.find(name);
+    if (it == st.t.end()) { fail("missing tensor \"" + name + "\""); return nullptr; }
+    bool ok = it->second.shape.size() == shape.size();
+    for (size_t i = 0; ok && i < shape.size(); i++) ok = shape[i] < 0 ? it->second.shape[i] > 0 : it->second.shape[i] == shape[i];
+    if (!ok) {
+      std::string a, b;
+      for (int64_t v : it->second.shape) a += (a.empty() ? "" : "x") + std::to_string(v);
+      for (int64_t v : shape) b += (b.empty() ? "" : "x") + (v < 0 ? std::string("?") : std::to_string(v));
+      fail("tensor \"" + name + "\" is [" + a + "], expected [" + b + "]");
+      return nullptr;
+    }
+    return &it->second;
+  }
+  bool floats(const std::string& name, std::vector<int64_t> shape, std::vector<float>& out)
+  {
+    const StTensor* t = tensor(name, shape);
+    if (!t) return false;
+    out.resize((size_t)t->elems);
+    if (t->dtype == "F32") memcpy(out.data(), t->data, (size_t)t->bytes);
+    else if (t->dtype == "BF16") for (int64_t i = 0; i < t->elems; i++) { uint16_t b; memcpy(&b, t->data + 2 * i, 2); const uint32_t u = (uint32_t)b << 16; memcpy(&out[i], &u, 4); }
+    else return fail("tensor \"" + name + "\" has type " + t->dtype + ", expected BF16 or F32");
+    return true;
+  }
+  float* upload(const std::vector<float>& v)
+  {
+    if (rc) return nullptr;
+    void* p = nullptr;
+    hipError_t e = hipMalloc(&p, v.size() * 4);
+    if (e == hipSuccess) { s.vectors.push_back(p); e = hipMemcpy(p, v.data(), v.size() * 4, hipMemcpyHostToDevice); }
+    if (e != hipSuccess) { rc = hip_fail(e, "model vector upload", __FILE__, __LINE__); return nullptr; }
+    return (float*)p;
+  }
+  float* vec(const std::string& name, std::vector<int64_t> shape)
+  {
+    std::vector<float> v;
+    return floats(name, shape, v) ? upload(v) : nullptr;
+  }
+  // rows of several matrices of one width, one after the other; order (may be null) gives the source row of each resident row,
+  // -1 a row of zeros
+  cai_qw_s* stack(const std::vector<std::pair<std::string, int64_t>>& parts, int64_t cols, const std::vector<int>* order = nullptr)
+  {
+    if (rc) return nullptr;
+    int64_t rows = 0;
+    std::vector<const uint8_t*> src;
+    for (auto& p : parts) {
+      const StTensor* t = tensor(p.first, {p.second, cols});
+      if (!t) return nullptr;
+      if (t->dtype != "BF16") { fail("tensor \"" + p.first + "\" has type " + t->dtype + ", expected BF16"); return nullptr; }
+      for (int64_t r = 0; r < p.second; r++) src.push_back(t->data + r * cols * 2);
+      rows += p.second;
+    }
+    if (order) {
+      std::vector<const uint8_t*> re(order->size());
+      for (size_t i = 0; i < order->size(); i++) re[i] = (*order)[i] < 0 ? nullptr : src[(size_t)(*order)[i]];
+      src.swap(re); rows = (int64_t)src.size();
+    }
+    std::vector<uint8_t> buf((size_t)(rows * cols * 2));
+    for (int64_t r = 0; r < rows; r++) { if (src[r]) memcpy(buf.data() + r * cols * 2, src[r], (size_t)cols * 2); else memset(buf.data() + r * cols * 2, 0, (size_t)cols * 2); }
+    cai_qw_t w = nullptr;
+    if ((rc = cai_qw_create(CAI_BF16, rows, cols, buf.data(), nullptr, &w))) return nullptr;
+    s.weights.push_back(w);
+    return w;
+  }
+  Dyt dyt_norm(const std::string& name, int width)
+  {
+    Dyt d;
+    std::vector<float> a;
+    if (!floats(name + ".alpha", {}, a)) return d;
+    d.alpha = a[0];
+    d.w = vec(name, {width}); d.b = vec(name + ".b", {width});
+    return d;
+  }
+};
+
+// ------------------------------------------------------------------------------------------
+// Samanex: gated-delta-rule layers and layers of a windowed attention beside a delta rule with a decay per key channel; Dynamic
+// Tanh before and after each sublayer; a stretch of layers repeated with the embedding output added in front of each repeat.
+// ------------------------------------------------------------------------------------------
+void delta_block(Builder& b, const Json* c, const std::string& where, const std::string& pre, int width, bool channel, NetDelta& D,
+                 std::vector<std::pair<std::string, int64_t>>& parts, int& at)
+{
+  DeltaDims& d = D.d;
+  d.heads = b.integer(c, "heads", where, 1, 65535); d.kv_heads = b.integer(c, "kv_heads", where, 1, 65535);
+  d.dim = b.integer(c, "dim", where, 1, 256); d.vdim = b.integer(c, "vdim", where, 1, 256); d.taps = b.integer(c, "conv", where, 1, 4096);
+  d.eps = b.s.eps; d.channel_decay = channel; d.sigmoid_gate = channel;
+  if (b.rc) return;
+  if (d.heads % d.kv_heads) { b.fail(where + "heads is not a multiple of " + where + "kv_heads"); return; }
+  const int kw = d.kv_heads * d.dim, vw = d.heads * d.vdim;
+  auto take = [&](const char* n, int rows) { const int o = at; parts.push_back({pre + n, rows}); at += rows; return o; };
+  D.oq = take("q", kw); D.ok = take("k", kw); D.ov = take("v", vw); D.ob = take("b", d.heads);
+  if (channel) {
+    const StTensor *a1 = b.tensor(pre + "a1", {-1, width}), *g1 = b.tensor(pre + "g1", {-1, width});
+    if (!a1 || !g1) return;
+    d.rank_a = (int)a1->shape[0]; d.rank_g = (int)g1->shape[0];
+    if (d.rank_a > 512 || d.rank_g > 512) { b.fail(where + "low-rank projections of more than 512 rows"); return; }
+    D.oa = take("a1", d.rank_a); D.og = take("g1", d.rank_g);
+    D.w.a2 = b.stack({{pre + "a2", (int64_t)d.heads * d.dim}}, d.rank_a);
+    D.w.g2 = b.stack({{pre + "g2", vw}}, d.rank_g);
+    D.w.dt_bias = b.vec(pre + "dt_bias", {(int64_t)d.heads * d.dim});
+  } else {
+    D.oa = take("a", d.heads); D.og = take("g", vw);
+    D.w.dt_bias = b.vec(pre + "dt_bias", {d.heads});
+  }
+  D.w.cq = b.vec(pre + "q.conv", {kw, d.taps}); D.w.ck = b.vec(pre + "k.conv", {kw, d.taps}); D.w.cv = b.vec(pre + "v.conv", {vw, d.taps});
+  std::vector<float> al;
+  if (!b.floats(pre + "A_log", {d.heads}, al)) return;
+  for (float& v : al) v = -expf(v);
+  D.w.rate = b.upload(al);
+  D.w.norm = b.vec(pre + "norm", {d.vdim});
+  D.out = b.stack({{pre + "o", width}}, vw);
+}
+
+void attn_block(Builder& b, const Json* c, const std::string& where, const std::string& pre, int width, NetAttn& A,
+                std::vector<std::pair<std::string, int64_t>>& parts, int& at)
+{
+  AttnDims& d = A.d;
+  d.heads = b.integer(c, "heads", where, 1, 65535); d.kv_heads = b.integer(c, "kv_heads", where, 1, 65535);
+  d.dim = b.integer(c, "dim", where, 1, 256); d.vdim = b.integer(c, "vdim", where, 1, 256);
+  d.window = b.integer(c ? c->get("mask") : nullptr, "size", where + "mask.", 1, 1 << 30);
+  d.scale = b.number(c, "scale", where); d.eps = b.s.eps;
+  d.dim_p = pad_to(d.dim, 8); d.vdim_p = pad_to(d.vdim, 8);
+  if (b.rc) return;
+  if (d.heads % d.kv_heads) { b.fail(where + "heads is not a multiple of " + where + "kv_heads"); return; }
+  auto take = [&](const char* n, int rows) { const int o = at; parts.push_back({pre + n, rows}); at += rows; return o; };
+  A.oq = take("q", d.heads * d.dim); A.ok = take("k", d.kv_heads * d.dim); A.ov = take("v", d.kv_heads * d.vdim);
+  A.qn = b.vec(pre + "q.norm", {d.dim}); A.kn = b.vec(pre + "k.norm", {d.dim});
+  A.out = b.stack({{pre + "o", width}}, (int64_t)d.heads * d.vdim);
+}
+
+void build_samanex(Builder& b, const Json& cfg)
+{
+  NetSpec& s = b.s;
+  s.width = b.integer(&cfg, "width", ""); s.vocab = b.integer(&cfg, "vocab", "", 1, 1 << 28);
+  s.eps = b.number(cfg.get("norm"), "eps", "norm.");
+  const Json* layers = cfg.get("layers");
+  if (!layers || layers->kind != Json::ARR || layers->arr.empty()) { b.fail("\"layers\" is missing or empty"); return; }
+  const int L = (int)layers->arr.size();
+  const Json* loop = cfg.get("loop");
+  if (loop && loop->kind != Json::NUL) {
+    s.loop_start = b.integer(loop, "start", "loop.", 0, L); s.loop_stop = b.integer(loop, "stop", "loop.", 0, L); s.loop_times = b.integer(loop, "times", "loop.", 1, 4096);
+    if (!b.rc && s.loop_stop < s.loop_start) b.fail("loop.stop lies before loop.start");
+  }
+  if (b.rc) return;
+  const int w = s.width;
+  s.embed = b.stack({{"embed", s.vocab}}, w);
+  s.head = b.stack({{"head", s.vocab}}, w);
+  s.final_norm = b.dyt_norm("final.norm", w);
+  for (int l = 0; l < L && !b.rc; l++) {
+    const Json& c = layers->arr[l];
+    const std::string p = "l" + std::to_string(l) + ".", where = "layers[" + std::to_string(l) + "].";
+    const Json *type = c.get("type"), *mix = c.get("mixer"), *mlp = c.get("mlp");
+    NetLayer y;
+    std::vector<std::pair<std::string, int64_t>> parts; int at = 0;
+    if (type && type->kind == Json::STR && type->str == "delta") {
+      y.kind = MIX_DELTA;
+      delta_block(b, mix, where + "mixer.", p + "mix.", w, false, y.delta, parts, at);
+    } else if (type && type->kind == Json::STR && type->str == "parallel") {
+      y.kind = MIX_PARALLEL;
+      attn_block(b, mix ? mix->get("left") : nullptr, where + "mixer.left.", p + "mix.left.", w, y.attn, parts, at);
+      if (!b.rc) delta_block(b, mix ? mix->get("right") : nullptr, where + "mixer.right.", p + "mix.right.", w, true, y.delta, parts, at);
+      y.gain_left = b.vec(p + "mix.left.out", {w}); y.gain_right = b.vec(p + "mix.right.out", {w});
+    } else b.fail("\"" + where + "type\" is not one of delta, parallel");
+    if (b.rc) return;
+    y.in = b.stack(parts, w);
+    y.norm1 = b.dyt_norm(p + "norm1", w); y.norm1b = b.dyt_norm(p + "norm1b", w);
+    if (mlp && mlp->kind == Json::OBJ) {
+      const Json* kind = mlp->get("kind");
+      if (!kind || kind->kind != Json::STR || kind->str != "dense") { b.fail("\"" + where + "mlp.kind\" is not dense"); return; }
+      y.ff = b.integer(mlp, "ff", where + "mlp.");
+      if (b.rc) return;
+      y.norm2 = b.dyt_norm(p + "norm2", w); y.norm2b = b.dyt_norm(p + "norm2b", w);
+      std::vector<int> order((size_t)pad_to(y.ff, 16) * 2, -1);     // gate and up rows interleaved in blocks of 16
+      for (int j = 0; j < y.ff; j++) { order[(size_t)glu_row(j, 0)] = j; order[(size_t)glu_row(j, 1)] = y.ff + j; }
+      y.gateup = b.stack({{p + "mlp.gate", y.ff}, {p + "mlp.up", y.ff}}, w, &order);
+      y.down = b.stack({{p + "mlp.down", w}}, y.ff);
+      y.glu = GLU_RELU;
+    } else if (mlp && mlp->kind != Json::NUL) b.fail("\"" + where + "mlp\" is neither an object nor null");
+    s.layers.push_back(y);
+  }
+}
+
+struct Arch { const char* name; void (*build)(Builder&, const Json&); };
+const Arch ARCHS[] = {{"Samanex", build_samanex}};
+
+bool is_dir(const char* path) { struct stat sb; return stat(path, &sb) == 0 && S_ISDIR(sb.st_mode); }
+
+int read_config(const std::string& path, Json& j)
+{
+  FILE* f = fopen(path.c_str(), "rb");
+  if (!f) return set_error(CAI_ERR_INVALID, "model: cannot open %s", path.c_str());
+  std::string text; char buf[65536]; size_t k;
+  while ((k = fread(buf, 1, sizeof buf, f)) > 0) text.append(buf, k);
+  fclose(f);
+  std::string err;
+  if (!JsonReader::parse(text.data(), text.size(), j, err) || j.kind != Json::OBJ) return set_error(CAI_ERR_INVALID, "model: %s: %s", err.c_str(), path.c_str());
+  return CAI_OK;
+}
+
+}  // namespace
+}  // namespace cai
+
+using namespace cai;
+
+extern "C" int cai_decoder_load(const char* path, int max_tokens, int max_seq, int dtype, cai_decoder_t* out)
+{
+  CAI_ENTER();
+  CAI_REQUIRE(path && out, "cai_decoder_load: null argument");
+  *out = nullptr;
+  CAI_REQUIRE(dtype == CAI_DTYPE_BF16 || dtype == CAI_DTYPE_F32, "cai_decoder_load: number format %d", dtype);
+  if (!is_dir(path)) return cai_decoder_load_gguf(path, max_tokens, max_seq, dtype == CAI_DTYPE_F32 ? CAI_KV_F32 : CAI_KV_F16, out);
+  CAI_REQUIRE(max_seq >= 1 && max_seq <= 256 && max_tokens >= 1 && max_tokens <= (1 << 26), "cai_decoder_load: %d sequences, %d tokens", max_seq, max_tokens);
+  Json cfg;
+  int rc = read_config(std::string(path) + "/config.json", cfg);
+  if (rc) return rc;
+  const Json* a = cfg.get("architecture");
+  const Arch* arch = nullptr; std::string known;
+  for (const Arch& k : ARCHS) { if (a && a->kind == Json::STR && a->str == k.name) arch = &k; known += (known.empty() ? "" : ", ") + std::string(k.name); }
+  if (!arch) return set_error(CAI_ERR_UNSUPPORTED, "model: architecture \"%s\" is not one of: %s", a && a->kind == Json::STR ? a->str.c_str() : "", known.c_str());
+  CAI_READY();
+  Builder b;
+  if ((rc = b.st.open(std::string(path) + "/model.safetensors"))) return rc;
+  arch->build(b, cfg);
+  if (b.rc) { net_spec_free(b.s); return b.rc; }
+  LayeredNet* n = nullptr;
+  if ((rc = net_create(std::move(b.s), max_tokens, max_seq, dtype == CAI_DTYPE_F32 ? ACT_T_F32 : ACT_T_BF16, &n))) return rc;
+  return decoder_from_net(n, max_tokens, max_seq, out);
+}

@@ -1,5 +1,5 @@
 // Elementwise layer math, block dequantization, embedding gather, arg-max and the MoE router for gfx950.
-#include "cai_internal.hpp"
+#include "cai_layered.hpp"
 #include "cai_blocks_raw.hpp"
 #include <string.h>
 #include <math.h>
@@ -82,6 +82,7 @@ __global__ void dequant_rows_kernel(int qtype, const uint8_t* data, const uint8_
 
 int launch_dequant_rows(const cai_qw_s* w, int64_t row0, int64_t n_rows, float* out)
 {
+  if (w->qtype == CAI_BF16) return bf16_dequant_rows(w, row0, n_rows, out);
   const int64_t n = n_rows * w->cols;
   hipLaunchKernelGGL(dequant_rows_kernel, dim3((unsigned)((n + 255) / 256)), dim3(256), 0, ctx().stream,
                      w->qtype, w->data, w->aux, qw_aux2(w), w->cols, row0, n, out);

@@ -9,7 +9,7 @@
 //   * P = sum_{k in block} q_k x_k comes out of v_mfma_f32_32x32x8_f16 with fp32 accumulation;
 //   * the block scales are applied in fp32 afterwards: Y += (d*sc) * P - (dmin*mn) * sum_{k in block} x_k
 //     (Q4_K, neural/neuralgguf.pas:472-514).
-#include "cai_internal.hpp"
+#include "cai_layered.hpp"
 #include "cai_gemv_common.hpp"
 #include <algorithm>
 
@@ -831,7 +831,8 @@ extern "C" int cai_qgemm(cai_qw_t w, const float* x, int n_tokens, float* y, int
     dx = (const float*)c.stage_in;
   }
   if (!(flags & CAI_Y_DEVICE)) { if ((rc = ensure_stage(&c.stage_out, &c.stage_out_cap, yb))) return rc; dy = (float*)c.stage_out; }
-  if ((flags & CAI_MATRIX_CORES) && nb_supported(w) && !gemm_mfma_supported(w)) rc = nb_linear(w, dx, w->cols, nullptr, 0.0f, n_tokens, dy, w->rows, nullptr);
+  if (w->qtype == CAI_BF16) rc = bf16_linear_f32(w, dx, w->cols, n_tokens, dy, w->rows, CAI_ACT_NONE);
+  else if ((flags & CAI_MATRIX_CORES) && nb_supported(w) && !gemm_mfma_supported(w)) rc = nb_linear(w, dx, w->cols, nullptr, 0.0f, n_tokens, dy, w->rows, nullptr);
   else rc = prefill_linear(w, dx, w->cols, nullptr, 0.0f, n_tokens, dy, w->rows, nullptr);
   if (rc) return rc;
   CAI_HIP(hipGetLastError());

@@ -1,0 +1,186 @@
+"""Plain, slow float64 implementation of the layered decoder designs, one function per mechanism.
+
+This is the checker of the layered decoder (tests/test_layered_*.py): numpy only, token by token where the mechanism is a
+recurrence, a full score matrix where it is an attention, and no code shared with the product library.
+"""
+import json
+import os
+import struct
+
+import numpy as np
+
+
+# ---------------------------------------------------------------- mechanisms
+def linear(w, x):
+    """rows of x through a matrix stored [out, in]"""
+    return x @ w.T
+
+
+def dynamic_tanh(x, alpha, w, b):
+    """y = w * tanh(alpha x) + b: a squashing in place of a normalisation, no statistics"""
+    return np.tanh(alpha * x) * w + b
+
+
+def rms_norm(x, eps):
+    """x over its root mean square along the last axis, eps inside the root"""
+    return x / np.sqrt((x * x).mean(-1, keepdims=True) + eps)
+
+
+def sigmoid(z):
+    return 0.5 * (1.0 + np.tanh(0.5 * z))
+
+
+def silu(z):
+    return z * sigmoid(z)
+
+
+def softplus(z):
+    return np.logaddexp(0.0, z)
+
+
+def causal_conv(x, taps_w):
+    """depthwise convolution over time, zeros before the start; taps_w[c, -1] weighs the current token"""
+    n_taps = taps_w.shape[1]
+    y = np.zeros_like(x)
+    for t in range(x.shape[0]):
+        for k in range(n_taps):
+            s = t - (n_taps - 1) + k
+            if s >= 0:
+                y[t] += taps_w[:, k] * x[s]
+    return y
+
+
+def unit(x):
+    return x / np.sqrt((x * x).sum(-1, keepdims=True) + 1e-6)
+
+
+def softmax_rows(s):
+    e = np.exp(s - s.max(-1, keepdims=True))
+    return e / e.sum(-1, keepdims=True)
+
+
+def window_attention(q, k, v, scale, window):
+    """q [T, H, d], k [T, G, d], v [T, G, dv]; query i sees the `window` tokens that end at itself"""
+    T, H, _ = q.shape
+    G = k.shape[1]
+    i, j = np.arange(T)[:, None], np.arange(T)[None, :]
+    seen = (j <= i) & (i - j < window)
+    out = np.zeros((T, H, v.shape[2]))
+    for h in range(H):
+        g = h // (H // G)
+        s = np.where(seen, (q[:, h] @ k[:, g].T) * scale, -np.inf)
+        out[:, h] = softmax_rows(s) @ v[:, g]
+    return out
+
+
+def delta_rule(q, k, v, decay, beta):
+    """Gated delta rule, token by token.  q, k [T, H, d]; v [T, H, dv]; decay [T, H, d] (one per key channel, a per-head
+    decay repeated); beta [T, H].  S [H, d, dv] starts at zero: decay the rows, write the correction, read."""
+    T, H, d = q.shape
+    S = np.zeros((H, d, v.shape[2]))
+    out = np.zeros(v.shape)
+    for t in range(T):
+        S *= decay[t][:, :, None]
+        u = beta[t][:, None] * (v[t] - np.einsum("hkv,hk->hv", S, k[t]))
+        S += k[t][:, :, None] * u[:, None, :]
+        out[t] = np.einsum("hkv,hk->hv", S, q[t])
+    return out
+
+
+# ---------------------------------------------------------------- mixers
+def delta_mixer(w, pre, c, h, eps, channel_decay):
+    T = h.shape[0]
+    H, G, d, dv = c["heads"], c["kv_heads"], c["dim"], c["vdim"]
+    act = [silu(causal_conv(linear(w[pre + n], h), w[pre + n + ".conv"])) for n in "qkv"]
+    q = unit(act[0].reshape(T, G, d)) * d ** -0.5
+    k = unit(act[1].reshape(T, G, d))
+    v = act[2].reshape(T, H, dv)
+    q, k = (np.repeat(z, H // G, axis=1) for z in (q, k))
+    beta = sigmoid(linear(w[pre + "b"], h))
+    rate = np.exp(w[pre + "A_log"])
+    if channel_decay:
+        z = linear(w[pre + "a2"], linear(w[pre + "a1"], h)) + w[pre + "dt_bias"].reshape(-1)
+        decay = np.exp(-rate[None, :, None] * softplus(z).reshape(T, H, d))
+        gate = sigmoid(linear(w[pre + "g2"], linear(w[pre + "g1"], h)))
+    else:
+        z = linear(w[pre + "a"], h) + w[pre + "dt_bias"]
+        decay = np.repeat(np.exp(-rate * softplus(z))[:, :, None], d, axis=2)
+        gate = silu(linear(w[pre + "g"], h))
+    o = delta_rule(q, k, v, decay, beta)
+    o = rms_norm(o, eps) * w[pre + "norm"] * gate.reshape(T, H, dv)
+    return linear(w[pre + "o"], o.reshape(T, H * dv))
+
+
+def attention_mixer(w, pre, c, h, eps):
+    T = h.shape[0]
+    H, G, d, dv = c["heads"], c["kv_heads"], c["dim"], c["vdim"]
+    q = rms_norm(linear(w[pre + "q"], h).reshape(T, H, d), eps) * w[pre + "q.norm"]
+    k = rms_norm(linear(w[pre + "k"], h).reshape(T, G, d), eps) * w[pre + "k.norm"]
+    v = linear(w[pre + "v"], h).reshape(T, G, dv)
+    o = window_attention(q, k, v, c["scale"], c["mask"]["size"])
+    return linear(w[pre + "o"], o.reshape(T, H * dv))
+
+
+def parallel_mixer(w, pre, c, h, eps):
+    a = attention_mixer(w, pre + "left.", c["left"], h, eps)
+    b = delta_mixer(w, pre + "right.", c["right"], h, eps, True)
+    return 0.5 * (rms_norm(a, eps) * w[pre + "left.out"] + rms_norm(b, eps) * w[pre + "right.out"])
+
+
+def relu_glu(w, pre, h):
+    return linear(w[pre + "down"], np.maximum(linear(w[pre + "gate"], h), 0.0) * linear(w[pre + "up"], h))
+
+
+# ---------------------------------------------------------------- the model
+def run_order(cfg):
+    """(layer, first layer of a repeated pass) for every layer run"""
+    n = len(cfg["layers"])
+    lp = cfg.get("loop") or {"start": 0, "stop": 0, "times": 1}
+    runs = [(i, False) for i in range(lp["start"])]
+    for p in range(lp["times"]):
+        runs += [(i, p > 0 and i == lp["start"]) for i in range(lp["start"], lp["stop"])]
+    return runs + [(i, False) for i in range(max(lp["stop"], lp["start"]), n)]
+
+
+def forward(cfg, w, tokens, layers_out=None):
+    """logits [T, vocab] of a whole prompt"""
+    eps = cfg["norm"]["eps"]
+    norm = lambda name, x: dynamic_tanh(x, w[name + ".alpha"], w[name], w[name + ".b"])
+    x = w["embed"][np.asarray(tokens)]
+    x0 = x
+    for i, again in run_order(cfg):
+        L = cfg["layers"][i]
+        p = "l%d." % i
+        if again:
+            x = x + x0
+        h = norm(p + "norm1", x)
+        y = delta_mixer(w, p + "mix.", L["mixer"], h, eps, False) if L["type"] == "delta" else parallel_mixer(w, p + "mix.", L["mixer"], h, eps)
+        x = x + norm(p + "norm1b", y)
+        if L.get("mlp"):
+            x = x + norm(p + "norm2b", relu_glu(w, p + "mlp.", norm(p + "norm2", x)))
+        if layers_out is not None:
+            layers_out.append(x.copy())
+    return linear(w["head"], norm("final.norm", x))
+
+
+# ---------------------------------------------------------------- files
+def read_model(path):
+    """(config, float64 tensors) of a folder with config.json and model.safetensors"""
+    with open(os.path.join(path, "config.json")) as f:
+        cfg = json.load(f)
+    with open(os.path.join(path, "model.safetensors"), "rb") as f:
+        (n,) = struct.unpack("<Q", f.read(8))
+        head = json.loads(f.read(n))
+        blob = f.read()
+    out = {}
+    for name, t in head.items():
+        if name == "__metadata__":
+            continue
+        a, b = t["data_offsets"]
+        raw = blob[a:b]
+        if t["dtype"] == "BF16":
+            v = (np.frombuffer(raw, "<u2").astype(np.uint32) << 16).view(np.float32)
+        else:
+            v = np.frombuffer(raw, {"F32": "<f4", "I32": "<i4", "F16": "<f2"}[t["dtype"]])
+        out[name] = v.reshape(t["shape"]).astype(np.float64)
+    return cfg, out
