@@ -289,6 +289,82 @@ def step_timeline(dec, tok, np):
     print(json.dumps({"step_timeline_us": out}))
 
 
+LAYERED_SIZES = {"w2048": dict(width=2048, ff=5632, heads=16, kv_heads=8, dim=128, n_layers=8, vocab=32768),
+                 "w4096": dict(width=4096, ff=11008, heads=32, kv_heads=16, dim=128, n_layers=8, vocab=32768)}
+
+
+def layered_bench(cai, synth, torch, only, size):
+    """Prompt (512 and 2048 tokens) and decode (batch 1, 4, 8 after a 512-token prompt) throughput of the layered decoder and of the
+    closest older model at equal size.  Times are HIP events around the library's own entry points; median of 5."""
+    import tempfile
+
+    import numpy as np
+    lib = cai.load()
+
+    def timed(f, reps=5, before=None):
+        out = []
+        for _ in range(reps):
+            if before:
+                before()
+            cai.check(lib.cai_sync()); cai.check(lib.cai_timer_start())
+            f()
+            ms = C.c_float(); cai.check(lib.cai_timer_stop(C.byref(ms)))
+            out.append(ms.value)
+        return sorted(out)[len(out) // 2]
+
+    for name, z in LAYERED_SIZES.items():
+        if size and size != name:
+            continue
+        for kind in ("samanex", "llama"):
+            if only and only != kind:
+                continue
+            rng = np.random.default_rng(1)
+            if kind == "samanex":
+                cfg = synth.layered_config(window=1024, **z)
+                with tempfile.TemporaryDirectory() as td:
+                    synth.write_layered_folder(td, cfg, 1)
+                    dec = cai.Decoder.load(td, 8 * 4096, 8, cai.DTYPE_BF16)
+                per_tok = 2.0 * sum(int(np.prod(s[0])) for n, s in synth.layered_shapes(cfg).items() if len(s[0]) == 2 and n not in ("embed", "head") and not n.endswith(".conv"))
+                label = "Samanex bf16"
+            else:
+                c = dict(n_layers=z["n_layers"], d_model=z["width"], n_q_heads=z["heads"], n_kv_heads=z["kv_heads"] // 2, head_dim=z["dim"], ffn=z["ff"], vocab=z["vocab"],
+                         max_ctx=4096, eps=1e-6, rope_theta=1e6)
+                dec = cai.Decoder(synth.random_decoder_spec(c, cai.Q8_0, cai.Q8_0, seed=1), max_batch=8, kv_dtype=cai.KV_F16)
+                qw, kw = c["n_q_heads"] * c["head_dim"], c["n_kv_heads"] * c["head_dim"]
+                per_tok = 2.0 * c["n_layers"] * (c["d_model"] * (2 * qw + 2 * kw) + 3 * c["d_model"] * c["ffn"])
+                label = "Llama Q8_0"
+            wb = dec.weight_bytes()
+            for T in (512, 2048):
+                tok = rng.integers(0, z["vocab"], T).astype(np.int32)
+                for _ in range(2):
+                    dec.reset(); dec.prefill(tok, want_logits=False)
+                ms = timed(lambda: dec.prefill(tok, want_logits=False), before=lambda: dec.reset())
+                print(json.dumps({"layered_bench": label, "size": name, "what": "prompt", "tokens": T, "ms": round(ms, 3), "tok_per_s": round(T / ms * 1e3),
+                                  "linear_TFLOP_per_s": round(per_tok * T / ms / 1e9, 1), "frac_of_bf16_peak": round(per_tok * T / ms / 1e9 / 2500.0, 4)}), flush=True)
+            tok = rng.integers(0, z["vocab"], 512).astype(np.int32)
+            for B in (1, 4, 8):
+                for b in range(8):
+                    dec.reset(b)
+                for b in range(B):
+                    dec.prefill(tok, seq=b, want_logits=False)
+                n = 64
+                pos = [512]
+
+                def run():
+                    if B == 1:
+                        dec.generate(int(tok[0]), pos[0], n)
+                    else:
+                        for i in range(n):
+                            dec.step(tok[:B], np.full(B, pos[0] + i, np.int32), want_logits=False)
+                    pos[0] += n
+                run()
+                ms = timed(run) / n
+                print(json.dumps({"layered_bench": label, "size": name, "what": "decode", "batch": B, "ms_per_step": round(ms, 4), "tok_per_s": round(B / ms * 1e3, 1),
+                                  "weight_GB_per_s": round(wb / ms / 1e6, 1), "frac_of_hbm_peak": round(wb / ms / 1e6 / HBM_PEAK_GBS, 4)}), flush=True)
+            dec.close()
+            torch.cuda.empty_cache()
+
+
 def gateup_kernel_name(qtype, cols):
     """Name of the batch-1 fused gate|up kernel the library launches for this weight type and width (rows of 17..24
     super-blocks are packed four to a wave: the fifth template argument, else 1)."""
@@ -319,6 +395,9 @@ def main():
     ap.add_argument("--gemm-sweep", action="store_true", help="isolated prompt-product sweep: Q8_0 / Q4_0 / Q4_K / Q5_K / Q6_K, four shapes, 64..2048 tokens (cai_qgemm, device pointers)")
     ap.add_argument("--step-timeline", action="store_true", help="device-side timeline of one captured batch-1 step (cai_decoder_timeline): per kernel class the gap to the previous launch, dispatch skew, staging, loop and tail times from wall-clock stamps taken inside the kernels")
     ap.add_argument("--copy-calibration", action="store_true", help="only run the 1 GiB device copy kernel 5 times (reference for traffic counters)")
+    ap.add_argument("--layered", action="store_true", help="layered decoder (Samanex, bfloat16) at two sizes with random weights beside the Llama-type decoder of the same width, feed-forward, heads and depth (Q8_0 body, half-precision cache): prompt and decode throughput, one JSON line per measurement")
+    ap.add_argument("--layered-only", choices=["", "samanex", "llama"], default="", help="with --layered: measure one of the two (for profiles)")
+    ap.add_argument("--layered-size", choices=["", "w2048", "w4096"], default="", help="with --layered: measure one size")
     args = ap.parse_args()
     if args.gpus != 1:
         print("bench.py: this build runs on ONE GPU; --gpus %d is not supported (no collectives are part of it)" % args.gpus, file=sys.stderr)
@@ -350,6 +429,9 @@ def main():
         return
     if args.gemm_sweep:
         gemm_sweep(cai, synth, torch)
+        return
+    if args.layered:
+        layered_bench(cai, synth, torch, args.layered_only, args.layered_size)
         return
     conf = CONFIGS[args.config]
     cfg = dict(conf["cfg"])

@@ -40,7 +40,7 @@ extern "C" {
 #define CAI_Q4_K   12
 #define CAI_Q5_K   13
 #define CAI_Q6_K   14  /* 210-byte super-blocks (neural/neuralgguf.pas:639-717); resident as aligned ql|qh records + planes of scales and d */
-#define CAI_BF16   30  /* bfloat16 rows, resident with rows padded to 64 columns */
+#define CAI_BF16   101  /* bfloat16 rows of a layered decoder, resident with rows padded to 64 columns (a type of this library, not the ggml id) */
 #define CAI_I8ROW  100  /* per-row symmetric int8 + fp32 row scale (neural/neuralvolume.pas:926-987) */
 
 /* ---- activation opcodes fused into the linear layer (neural/neural.cl:114-146) ---- */
@@ -67,6 +67,7 @@ extern "C" {
 typedef struct cai_qw_s*      cai_qw_t;       /* resident quantized weight matrix */
 typedef struct cai_kv_s*      cai_kv_t;       /* KV cache of one sequence, all layers */
 typedef struct cai_kv_snap_s* cai_kv_snap_t;  /* deep copy of a KV cache's live rows */
+typedef struct cai_sched_s*   cai_sched_t;    /* continuous-batching scheduler over a decoder */
 typedef struct cai_decoder_s* cai_decoder_t;  /* step-resident decoder */
 
 /* =====================================================================================
@@ -294,6 +295,20 @@ int cai_decoder_step_batch(cai_decoder_t d, int n_entries, const int32_t* seqs, 
                            const uint8_t* want, float* logits, int32_t* argmax);
 /* Tokens a sequence can still take before the cache (the shared page pool of a layered decoder) is full. */
 int cai_decoder_room(cai_decoder_t d, int seq, int* tokens_out);
+/* ---- continuous batching ----
+ * A scheduler owns the sequences of one decoder (nothing else may step it meanwhile).  Requests are admitted first come, first
+ * served when a sequence and the cache their whole length needs are free; a step feeds one token of every decoding request and
+ * prompt portions of at most `portion` tokens of the others, max_rows tokens together (0: defaults of 512 and 2048).
+ * temperature <= 0 takes the arg-max; otherwise the next token is drawn from the top_k most probable (cai_decoder_candidates) in
+ * proportion, with the request's own generator started from `seed`.  eos < 0: none; an eos token is the last one returned. */
+int cai_sched_create(cai_decoder_t d, int max_rows, int portion, cai_sched_t* out);
+int cai_sched_destroy(cai_sched_t s);
+int cai_sched_submit(cai_sched_t s, const int32_t* prompt, int n, int max_new, int eos, float temperature, int top_k, uint64_t seed, int64_t* id_out);
+int cai_sched_step(cai_sched_t s, int* live_out, int* waiting_out);   /* one engine step; either count may be NULL */
+int cai_sched_run(cai_sched_t s);                                    /* steps until nothing is live or waiting */
+/* tokens produced so far: *n_out counts them all, at most cap are copied; *done_out (may be NULL) */
+int cai_sched_result(cai_sched_t s, int64_t id, int32_t* tokens_out, int cap, int* n_out, int* done_out);
+int cai_sched_drop(cai_sched_t s, int64_t id);                       /* ends a request wherever it is and forgets it */
 /* Session management (neural/neuraldecode.pas:5714-5843): always safe after a failed step. */
 /* ---- distribution pipeline ahead of the samplers, on the device ----
  * The non-greedy branch of TChatEngine.GenerateFromIds (neural/neuralchatengine.pas:1374-1396, 1495-1501): RowSoftMax ->

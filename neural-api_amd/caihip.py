@@ -6,7 +6,7 @@ import numpy as np
 
 from . import lib_path
 
-F32, F16, Q4_0, Q8_0, Q4_K, Q6_K, BF16, I8ROW = 0, 1, 2, 8, 12, 14, 30, 100
+F32, F16, Q4_0, Q8_0, Q4_K, Q6_K, I8ROW, BF16 = 0, 1, 2, 8, 12, 14, 100, 101
 DTYPE_BF16, DTYPE_F32 = 0, 1
 Q4_1, Q5_0, Q5_1, Q2_K, Q3_K, Q5_K = 3, 6, 7, 10, 11, 13
 ACT_NONE, ACT_RELU, ACT_SIGMOID, ACT_TANH = 0, 1, 2, 3
@@ -25,6 +25,7 @@ cai_kv_create cai_kv_destroy cai_kv_reset cai_kv_truncate cai_kv_len cai_kv_snap
 cai_decoder_create cai_decoder_destroy cai_decoder_set_weight cai_decoder_set_vector cai_decoder_step cai_decoder_hidden_state cai_decoder_step_window cai_prompt_lookup_draft cai_decoder_generate_lookup cai_decoder_generate cai_decoder_profile cai_decoder_timeline
 cai_decoder_prefill cai_decoder_reset cai_decoder_truncate cai_decoder_len cai_decoder_set_eviction cai_decoder_cache_rows cai_decoder_set_kv_dtype cai_decoder_set_rope_scaling cai_decoder_set_rope_freq_factors cai_decoder_set_rope_out_scale cai_sample_candidates cai_decoder_candidates cai_decoder_snapshot cai_decoder_restore cai_decoder_fork
 cai_decoder_weight_bytes cai_decoder_get_config cai_decoder_load_gguf cai_decoder_load cai_decoder_step_batch cai_decoder_room
+cai_sched_create cai_sched_destroy cai_sched_submit cai_sched_step cai_sched_run cai_sched_result cai_sched_drop
 cai_gguf_open cai_gguf_close cai_gguf_info cai_gguf_meta_int cai_gguf_meta_float cai_gguf_meta_str cai_gguf_meta_array_count
 cai_gguf_meta_array_str cai_gguf_find_tensor cai_gguf_tensor_info cai_gguf_tensor_data cai_gguf_load_qw""".split()
 
@@ -131,6 +132,13 @@ def load():
         L.cai_decoder_load.argtypes = [C.c_char_p, i32, i32, i32, C.POINTER(vp)]
         L.cai_decoder_step_batch.argtypes = [vp, i32, vp, vp, vp, vp, vp, vp]
         L.cai_decoder_room.argtypes = [vp, i32, C.POINTER(i32)]
+        L.cai_sched_create.argtypes = [vp, i32, i32, C.POINTER(vp)]
+        L.cai_sched_destroy.argtypes = [vp]
+        L.cai_sched_submit.argtypes = [vp, vp, i32, i32, i32, f32, i32, C.c_uint64, C.POINTER(i64)]
+        L.cai_sched_step.argtypes = [vp, C.POINTER(i32), C.POINTER(i32)]
+        L.cai_sched_run.argtypes = [vp]
+        L.cai_sched_result.argtypes = [vp, i64, vp, i32, C.POINTER(i32), C.POINTER(i32)]
+        L.cai_sched_drop.argtypes = [vp, i64]
         L.cai_gguf_open.argtypes = [C.c_char_p, C.POINTER(vp)]
         L.cai_gguf_close.argtypes = [vp]
         L.cai_gguf_info.argtypes = [vp, C.POINTER(i32), C.POINTER(i32), C.POINTER(i64), C.POINTER(i64), C.POINTER(i64)]
@@ -585,6 +593,50 @@ class Decoder:
             self.h = None
             for w in self.weights:
                 w.close()
+
+    def __del__(self):
+        try:
+            self.close()
+        except Exception:
+            pass
+
+
+class Scheduler:
+    """continuous batching over a decoder's sequences (cai_sched_*)"""
+
+    def __init__(self, dec, max_rows=0, portion=0):
+        self.h = C.c_void_p(); self.dec = dec
+        check(load().cai_sched_create(dec.h, max_rows, portion, C.byref(self.h)))
+
+    def submit(self, prompt, max_new, eos=-1, temperature=0.0, top_k=0, seed=0):
+        prompt = np.ascontiguousarray(prompt, np.int32); i = C.c_int64()
+        check(load().cai_sched_submit(self.h, _ptr(prompt), prompt.size, max_new, eos, temperature, top_k, seed, C.byref(i)))
+        return i.value
+
+    def step(self):
+        """one engine step: (live, waiting) afterwards"""
+        a, b = C.c_int(), C.c_int()
+        check(load().cai_sched_step(self.h, C.byref(a), C.byref(b)))
+        return a.value, b.value
+
+    def run(self):
+        check(load().cai_sched_run(self.h))
+
+    def result(self, i):
+        """(tokens, finished)"""
+        n, done = C.c_int(), C.c_int()
+        check(load().cai_sched_result(self.h, i, None, 0, C.byref(n), C.byref(done)))
+        out = np.empty(max(n.value, 1), np.int32)
+        check(load().cai_sched_result(self.h, i, _ptr(out), n.value, C.byref(n), C.byref(done)))
+        return out[:n.value].tolist(), bool(done.value)
+
+    def drop(self, i):
+        check(load().cai_sched_drop(self.h, i))
+
+    def close(self):
+        if self.h:
+            load().cai_sched_destroy(self.h)
+            self.h = None
 
     def __del__(self):
         try:

@@ -567,6 +567,11 @@ int decoder_from_net(LayeredNet* n, int max_tokens, int max_seq, cai_decoder_s**
   return CAI_OK;
 }
 
+int  decoder_pool_pages(cai_decoder_s* d) { return d->net ? net_pool_pages(d->net) : 0; }
+int  decoder_peak_pages(cai_decoder_s* d, int64_t total, int portion) { return d->net ? net_peak_pages(d->net, total, portion) : 0; }
+bool decoder_bounded(cai_decoder_s* d) { return !d->net && d->kv.evict_cap == 0; }
+bool decoder_keeps_rows(cai_decoder_s* d) { return d->net != nullptr; }
+
 static int len_of(cai_decoder_s* d, int seq) { return d->net ? net_len(d->net, seq) : d->kv.len_at(seq, 0); }
 
 // `n` consecutive tokens of one sequence of a layered decoder; logits and arg-max of every row, or of the last one only
@@ -1084,8 +1089,8 @@ extern "C" int cai_decoder_hidden_state(cai_decoder_t d, int row, float* hidden_
   CAI_ENTER();
   CAI_READY();
   CAI_REQUIRE(d && hidden_out, "cai_decoder_hidden_state: null argument");
-  CAI_REQUIRE(row >= 0 && row < 8, "cai_decoder_hidden_state: row %d outside 0..7", row);
   if (d->net) return net_hidden(d->net, row, hidden_out);
+  CAI_REQUIRE(row >= 0 && row < 8, "cai_decoder_hidden_state: row %d outside 0..7", row);
   if (!d->final_norm) return set_error(CAI_ERR_STATE, "cai_decoder_hidden_state: final norm gain not set");
   Context& cx = ctx();
   const int dm = d->cfg.d_model;
@@ -1104,13 +1109,13 @@ extern "C" int cai_decoder_candidates(cai_decoder_t d, int row, const int32_t* h
   CAI_ENTER();
   CAI_READY();
   CAI_REQUIRE(d && tokens_out && probs_out, "cai_decoder_candidates: null argument");
-  CAI_REQUIRE(row >= 0 && row < 8, "cai_decoder_candidates: row %d outside 0..7", row);   // a row of the last step (sequence) or window (position)
   CAI_REQUIRE(m >= 1 && m <= 1024, "cai_decoder_candidates: %d candidates (1..1024)", m);
   if (d->net) {
     const float* lg = net_logits(d->net, row);
     if (!lg) return set_error(CAI_ERR_STATE, "cai_decoder_candidates: the last step has no logits row %d", row);
     return run_candidates(lg, d->cfg.vocab, hist_ids, hist_counts, n_hist, repetition, frequency, presence, temperature, m, tokens_out, probs_out, count_out);
   }
+  CAI_REQUIRE(row >= 0 && row < 8, "cai_decoder_candidates: row %d outside 0..7", row);   // a row of the last step (sequence) or window (position)
   return run_candidates(d->logits + (int64_t)row * d->cfg.vocab, d->cfg.vocab, hist_ids, hist_counts, n_hist,
                         repetition, frequency, presence, temperature, m, tokens_out, probs_out, count_out);
 }

@@ -594,7 +594,14 @@ int net_generate(LayeredNet* n, int seq, int32_t first, int n_tokens, int32_t* o
 
 int net_len(const LayeredNet* n, int seq) { return n->pool.seq[seq].len; }
 int net_room(const LayeredNet* n, int seq) { return n->pool.room(seq); }
-int net_free_tokens(const LayeredNet* n) { return n->pool.n_pages ? (int)n->pool.free_pages.size() * PAGE_TOKENS : 1 << 30; }
+int net_pool_pages(const LayeredNet* n) { return n->pool.n_pages; }
+int net_peak_pages(const LayeredNet* n, int64_t total, int portion)
+{
+  if (!n->pool.n_pages) return 0;
+  // a step's rows and the window before them, which may start and end inside a page
+  const int64_t window = ((int64_t)n->pool.keep - 1 + portion + 2 * (PAGE_TOKENS - 1)) / PAGE_TOKENS;
+  return (int)std::min<int64_t>((total + PAGE_TOKENS - 1) / PAGE_TOKENS, window);
+}
 int net_rows(const LayeredNet* n, int seq) { const auto& q = n->pool.seq[seq]; return n->pool.n_pages ? q.len - q.first_page * PAGE_TOKENS : 0; }
 int net_n_runs(const LayeredNet* n) { return (int)n->runs.size(); }
 int net_reset(LayeredNet* n, int seq) { n->pool.free_seq(seq); return CAI_OK; }

@@ -165,7 +165,8 @@ int  net_step(LayeredNet* n, int n_ent, const int32_t* seq, const int32_t* count
 int  net_generate(LayeredNet* n, int seq, int32_t first, int n_tokens, int32_t* out_host);
 int  net_len(const LayeredNet* n, int seq);
 int  net_room(const LayeredNet* n, int seq);
-int  net_free_tokens(const LayeredNet* n);
+int  net_pool_pages(const LayeredNet* n);
+int  net_peak_pages(const LayeredNet* n, int64_t total, int portion);   // most pages a sequence of `total` tokens fed in such portions holds at once
 int  net_rows(const LayeredNet* n, int seq);
 int  net_n_runs(const LayeredNet* n);
 int  net_reset(LayeredNet* n, int seq);
@@ -181,5 +182,10 @@ void net_snap_free(NetSnap* s);
 
 // a decoder around a net (cai_decoder.hip), and the model registry's entry (cai_models.hip)
 int decoder_from_net(LayeredNet* n, int max_tokens, int max_seq, cai_decoder_s** out);
+// what the scheduler asks of a decoder
+int  decoder_pool_pages(cai_decoder_s* d);          // pages all sequences share (0: every sequence has rows of its own)
+int  decoder_peak_pages(cai_decoder_s* d, int64_t total, int portion);
+bool decoder_bounded(cai_decoder_s* d);             // a sequence ends at max_ctx
+bool decoder_keeps_rows(cai_decoder_s* d);          // every wanted row of a batch step stays addressable
 
 }  // namespace cai

@@ -177,10 +177,19 @@ class TNNetStreamingDecoder {
     Check(cai_decoder_get_config(d_, &cfg_));
     logits_.resize((size_t)cfg_.vocab);
   }
+  // a model folder (config.json, model.safetensors) or a GGUF file through the library's registry: pMaxTokens cached tokens over
+  // pSequences sequences, in the number format pDType (CAI_DTYPE_BF16 / CAI_DTYPE_F32)
+  TNNetStreamingDecoder(const std::string& Model, int pMaxTokens, int pSequences, int pDType)
+  {
+    Check(cai_decoder_load(Model.c_str(), pMaxTokens, pSequences, pDType, &d_));
+    Check(cai_decoder_get_config(d_, &cfg_));
+    logits_.resize((size_t)cfg_.vocab);
+  }
   ~TNNetStreamingDecoder() { if (d_) cai_decoder_destroy(d_); }
   TNNetStreamingDecoder(const TNNetStreamingDecoder&) = delete;
   TNNetStreamingDecoder& operator=(const TNNetStreamingDecoder&) = delete;
 
+  cai_decoder_t Handle() const { return d_; }
   const cai_decoder_config& Config() const { return cfg_; }
   void Reset() { Check(cai_decoder_reset(d_, 0)); }
   // One streamed forward of a window of token ids; AbsPos is the absolute position of the FIRST token of the window.
@@ -259,6 +268,35 @@ class TNNetStreamingDecoder {
   std::vector<int32_t> argmax_rows_;
   int rows_ = 0;
   int32_t argmax_ = -1;
+};
+
+// Continuous batching over the sequences of a decoder (cai_sched_*).
+class TBatchScheduler {
+ public:
+  explicit TBatchScheduler(TNNetStreamingDecoder& Decoder, int MaxRows = 0, int Portion = 0) { Check(cai_sched_create(Decoder.Handle(), MaxRows, Portion, &s_)); }
+  ~TBatchScheduler() { if (s_) cai_sched_destroy(s_); }
+  TBatchScheduler(const TBatchScheduler&) = delete;
+  TBatchScheduler& operator=(const TBatchScheduler&) = delete;
+  int64_t Submit(const std::vector<int32_t>& Prompt, int MaxNew, int Eos = -1, float Temperature = 0.0f, int TopK = 0, uint64_t Seed = 0)
+  {
+    int64_t id = 0;
+    Check(cai_sched_submit(s_, Prompt.data(), (int)Prompt.size(), MaxNew, Eos, Temperature, TopK, Seed, &id));
+    return id;
+  }
+  bool Step() { int live = 0, waiting = 0; Check(cai_sched_step(s_, &live, &waiting)); return live + waiting > 0; }
+  void Run() { Check(cai_sched_run(s_)); }
+  std::vector<int32_t> Result(int64_t Id, bool* Done = nullptr) const
+  {
+    int n = 0, done = 0;
+    Check(cai_sched_result(s_, Id, nullptr, 0, &n, &done));
+    std::vector<int32_t> out((size_t)n);
+    Check(cai_sched_result(s_, Id, out.data(), n, &n, &done));
+    if (Done) *Done = done != 0;
+    return out;
+  }
+
+ private:
+  cai_sched_t s_ = nullptr;
 };
 
 }  // namespace caihip

@@ -20,20 +20,21 @@ const
   CAI_ERR_UNSUPPORTED = -4; CAI_ERR_STATE = -5;
 
   // ggml tensor type ids (neural/neuralgguf.pas:86-98) + per-row int8
-  CAI_F32 = 0; CAI_F16 = 1; CAI_Q4_0 = 2; CAI_Q8_0 = 8; CAI_Q4_K = 12; CAI_Q6_K = 14; CAI_I8ROW = 100;
+  CAI_F32 = 0; CAI_F16 = 1; CAI_Q4_0 = 2; CAI_Q8_0 = 8; CAI_Q4_K = 12; CAI_Q6_K = 14; CAI_I8ROW = 100; CAI_BF16 = 101;
   CAI_Q4_1 = 3; CAI_Q5_0 = 6; CAI_Q5_1 = 7; CAI_Q2_K = 10; CAI_Q3_K = 11; CAI_Q5_K = 13;
   CAI_ROPE_NONE = 0; CAI_ROPE_LINEAR = 1; CAI_ROPE_LLAMA3 = 2; CAI_ROPE_NTK = 3; CAI_ROPE_YARN = 4;
   // fused activation opcodes = csAct* of the OpenCL kernels (neural/neural.cl:114-146)
   CAI_ACT_NONE = 0; CAI_ACT_RELU = 1; CAI_ACT_SIGMOID = 2; CAI_ACT_TANH = 3;
   CAI_X_DEVICE = 1; CAI_Y_DEVICE = 2; CAI_MATRIX_CORES = 4;
+  CAI_DTYPE_BF16 = 0; CAI_DTYPE_F32 = 1;
   CAI_KV_F32 = 0; CAI_KV_F16 = 1; CAI_KV_I8 = 2;
   CAI_W_EMBED = 0; CAI_W_HEAD = 1; CAI_W_Q = 2; CAI_W_K = 3; CAI_W_V = 4; CAI_W_O = 5;
   CAI_W_GATEUP = 6; CAI_W_DOWN = 7; CAI_W_ROUTER = 8;
   CAI_V_ATTN_NORM = 0; CAI_V_MLP_NORM = 1; CAI_V_FINAL_NORM = 2; CAI_V_Q_NORM = 3; CAI_V_K_NORM = 4;
 
 type
-  TCaiQW = Pointer; TCaiKV = Pointer; TCaiKVSnap = Pointer; TCaiDecoder = Pointer; TCaiGGUF = Pointer;
-  PCaiQW = ^TCaiQW; PCaiKV = ^TCaiKV; PCaiKVSnap = ^TCaiKVSnap; PCaiDecoder = ^TCaiDecoder; PCaiGGUF = ^TCaiGGUF;
+  TCaiQW = Pointer; TCaiKV = Pointer; TCaiKVSnap = Pointer; TCaiDecoder = Pointer; TCaiGGUF = Pointer; TCaiSched = Pointer;
+  PCaiQW = ^TCaiQW; PCaiKV = ^TCaiKV; PCaiKVSnap = ^TCaiKVSnap; PCaiDecoder = ^TCaiDecoder; PCaiGGUF = ^TCaiGGUF; PCaiSched = ^TCaiSched;
 
   TCaiDecoderConfig = packed record
     n_layers, d_model, n_q_heads, n_kv_heads, head_dim, ffn, vocab, max_ctx: LongInt;
@@ -120,6 +121,18 @@ function cai_decoder_fork(d: TCaiDecoder; src_seq, dst_seq: LongInt): LongInt; c
 function cai_decoder_weight_bytes(d: TCaiDecoder; algorithmic_bytes_out: PInt64): LongInt; cdecl; external CAIHIP_LIB;
 function cai_decoder_get_config(d: TCaiDecoder; out_cfg: Pointer): LongInt; cdecl; external CAIHIP_LIB;
 function cai_decoder_load_gguf(path: PChar; max_ctx, max_batch, kv_dtype: LongInt; out_decoder: PCaiDecoder): LongInt; cdecl; external CAIHIP_LIB;
+function cai_decoder_load(path: PChar; max_tokens, max_seq, dtype: LongInt; out_decoder: PCaiDecoder): LongInt; cdecl; external CAIHIP_LIB;
+function cai_decoder_step_batch(d: TCaiDecoder; n_entries: LongInt; seqs, counts, tokens: PLongInt; want: PByte; logits: PSingle; argmax: PLongInt): LongInt; cdecl; external CAIHIP_LIB;
+function cai_decoder_room(d: TCaiDecoder; seq: LongInt; tokens_out: PLongInt): LongInt; cdecl; external CAIHIP_LIB;
+
+// continuous batching
+function cai_sched_create(d: TCaiDecoder; max_rows, portion: LongInt; out_s: PCaiSched): LongInt; cdecl; external CAIHIP_LIB;
+function cai_sched_destroy(s: TCaiSched): LongInt; cdecl; external CAIHIP_LIB;
+function cai_sched_submit(s: TCaiSched; prompt: PLongInt; n, max_new, eos: LongInt; temperature: Single; top_k: LongInt; seed: QWord; id_out: PInt64): LongInt; cdecl; external CAIHIP_LIB;
+function cai_sched_step(s: TCaiSched; live_out, waiting_out: PLongInt): LongInt; cdecl; external CAIHIP_LIB;
+function cai_sched_run(s: TCaiSched): LongInt; cdecl; external CAIHIP_LIB;
+function cai_sched_result(s: TCaiSched; id: Int64; tokens_out: PLongInt; cap: LongInt; n_out, done_out: PLongInt): LongInt; cdecl; external CAIHIP_LIB;
+function cai_sched_drop(s: TCaiSched; id: Int64): LongInt; cdecl; external CAIHIP_LIB;
 
 // GGUF container (TNNetGGUFReader, neural/neuralgguf.pas:1072-1220)
 function cai_gguf_open(path: PChar; out_gguf: PCaiGGUF): LongInt; cdecl; external CAIHIP_LIB;

@@ -212,3 +212,82 @@ def random_decoder_spec(cfg, qtype, head_qtype, seed=424242, qkv_bias=False, std
             put((l, cai.W_DOWN), cai.Q6_K if hi else qtype, d, I)
     c = {k: v for k, v in cfg.items() if k != "tied"}
     return dict(cfg=c, tensors=T, vecs=Vv)
+
+
+# ---- model folders for the layered decoder ----
+def layered_config(width, ff, heads, kv_heads, dim, n_layers, vocab, window, conv=4, every=4, loop=None):
+    """A Samanex configuration of real-model proportions: every `every`-th layer is a parallel one, the others are delta layers."""
+    rec = dict(heads=heads, kv_heads=kv_heads, dim=dim, vdim=dim, conv=conv)
+    par = dict(left=dict(heads=heads, kv_heads=max(1, kv_heads // 2), dim=dim, vdim=dim, scale=dim ** -0.5, mask=dict(size=window)), right=dict(rec, kv_heads=heads))
+    layers = [dict(type="parallel" if i % every == every - 1 else "delta", mixer=par if i % every == every - 1 else rec, mlp=dict(kind="dense", ff=ff)) for i in range(n_layers)]
+    return dict(architecture="Samanex", width=width, vocab=vocab, layers=layers, norm=dict(eps=1e-6), loop=loop or dict(start=0, stop=n_layers, times=1))
+
+
+def layered_shapes(cfg, rank=128):
+    """name -> (shape, standard deviation, mean) of every tensor of a Samanex model"""
+    w, out = cfg["width"], {}
+
+    def lin(name, rows, cols):
+        out[name] = ((rows, cols), cols ** -0.5, 0.0)
+
+    def norm(name):
+        out[name] = ((w,), 0.1, 1.0); out[name + ".b"] = ((w,), 0.05, 0.0); out[name + ".alpha"] = ((), 0.0, 0.7)
+
+    def delta(p, c, channel):
+        kw, vw = c["kv_heads"] * c["dim"], c["heads"] * c["vdim"]
+        for n, r in (("q", kw), ("k", kw), ("v", vw)):
+            lin(p + n, r, w); out[p + n + ".conv"] = ((r, c["conv"]), 0.3, 0.25)
+        lin(p + "b", c["heads"], w); out[p + "A_log"] = ((c["heads"],), 0.5, 0.0); out[p + "norm"] = ((c["vdim"],), 0.1, 1.0)
+        if channel:
+            lin(p + "a1", rank, w); lin(p + "a2", c["heads"] * c["dim"], rank); lin(p + "g1", rank, w); lin(p + "g2", vw, rank)
+        else:
+            lin(p + "a", c["heads"], w); lin(p + "g", vw, w)
+        out[p + "dt_bias"] = ((c["heads"] * c["dim"] if channel else c["heads"],), 1.0, -3.0)
+        lin(p + "o", w, vw)
+
+    out["embed"] = ((cfg["vocab"], w), 1.0, 0.0)
+    lin("head", cfg["vocab"], w); norm("final.norm")
+    for i, L in enumerate(cfg["layers"]):
+        p, m = "l%d." % i, L["mixer"]
+        norm(p + "norm1"); norm(p + "norm1b")
+        if L["type"] == "delta":
+            delta(p + "mix.", m, False)
+        else:
+            a = m["left"]
+            lin(p + "mix.left.q", a["heads"] * a["dim"], w); lin(p + "mix.left.k", a["kv_heads"] * a["dim"], w); lin(p + "mix.left.v", a["kv_heads"] * a["vdim"], w)
+            lin(p + "mix.left.o", w, a["heads"] * a["vdim"])
+            out[p + "mix.left.q.norm"] = ((a["dim"],), 0.1, 1.0); out[p + "mix.left.k.norm"] = ((a["dim"],), 0.1, 1.0)
+            delta(p + "mix.right.", m["right"], True)
+            out[p + "mix.left.out"] = ((w,), 0.1, 1.0); out[p + "mix.right.out"] = ((w,), 0.1, 1.0)
+        if L["mlp"]:
+            norm(p + "norm2"); norm(p + "norm2b")
+            lin(p + "mlp.gate", L["mlp"]["ff"], w); lin(p + "mlp.up", L["mlp"]["ff"], w); lin(p + "mlp.down", w, L["mlp"]["ff"])
+    return out
+
+
+def write_layered_folder(folder, cfg, seed=0, rank=128):
+    """config.json and model.safetensors with random bfloat16 weights (one random block, repeated from a random start)"""
+    import json
+    import os
+    import struct
+
+    import numpy as np
+    rng = np.random.default_rng(seed)
+    block = rng.standard_normal((1 << 22) + 4099, dtype=np.float32)
+    os.makedirs(folder, exist_ok=True)
+    with open(os.path.join(folder, "config.json"), "w") as f:
+        json.dump(cfg, f)
+    shapes, head, at = layered_shapes(cfg, rank), {}, 0
+    for name, (shape, _, _) in shapes.items():
+        n = 2 * int(np.prod(shape, dtype=np.int64))
+        head[name] = dict(dtype="BF16", shape=list(shape), data_offsets=[at, at + n]); at += n
+    h = json.dumps(head).encode(); h += b" " * (-len(h) % 8)
+    with open(os.path.join(folder, "model.safetensors"), "wb") as f:
+        f.write(struct.pack("<Q", len(h)) + h)
+        for name, (shape, std, mean) in shapes.items():
+            n = int(np.prod(shape, dtype=np.int64))
+            bits = ((block * np.float32(std) + np.float32(mean)).view(np.uint32) >> 16).astype(np.uint16)
+            k = int(rng.integers(0, 4096))
+            while n > 0:
+                m = min(n, bits.size - k)
+                f.write(bits[k:k + m].tobytes()); n -= m; k = 0

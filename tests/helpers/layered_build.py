@@ -1,0 +1,107 @@
+"""Small random Samanex models for the layered-decoder tests: a configuration, weights rounded to bfloat16, a model folder."""
+import json
+import os
+import struct
+
+import numpy as np
+
+
+def to_bf16(a):
+    """(bits, the rounded values as float64)"""
+    u = np.ascontiguousarray(a, np.float32).view(np.uint32).astype(np.uint64)
+    u = ((u + 0x7fff + ((u >> 16) & 1)) >> 16).astype(np.uint16)
+    return u, (u.astype(np.uint32) << 16).view(np.float32).astype(np.float64)
+
+
+def delta(heads=2, kv_heads=1, dim=20, vdim=36, conv=3):
+    return dict(heads=heads, kv_heads=kv_heads, dim=dim, vdim=vdim, conv=conv)
+
+
+def attn(heads=4, kv_heads=2, dim=24, vdim=40, window=9, scale=0.21):
+    return dict(heads=heads, kv_heads=kv_heads, dim=dim, vdim=vdim, scale=scale, mask=dict(size=window))
+
+
+def layer(mixer, ff=56):
+    """a delta layer from a delta mixer, a parallel layer from a (left, right) pair; ff None: no feed-forward"""
+    mlp = None if ff is None else dict(kind="dense", ff=ff)
+    if isinstance(mixer, tuple):
+        return dict(type="parallel", mixer=dict(left=mixer[0], right=mixer[1]), mlp=mlp)
+    return dict(type="delta", mixer=mixer, mlp=mlp)
+
+
+def config(layers, width=72, vocab=131, eps=1e-5, loop=None):
+    return dict(architecture="Samanex", width=width, vocab=vocab, layers=layers, norm=dict(eps=eps),
+                loop=loop or dict(start=0, stop=len(layers), times=1))
+
+
+def weights(cfg, seed=0, rank_a=7, rank_g=11):
+    """name -> float array before rounding"""
+    rng = np.random.default_rng(seed)
+    w, width = {}, cfg["width"]
+
+    def lin(name, rows, cols, gain=1.0):
+        w[name] = rng.standard_normal((rows, cols)) * gain / np.sqrt(cols)
+
+    def vec(name, shape, mean=0.0, spread=0.2):
+        w[name] = mean + spread * rng.standard_normal(shape)
+
+    def norm(name):
+        vec(name, width, 1.0); vec(name + ".b", width, 0.0, 0.1)
+        w[name + ".alpha"] = np.asarray(rng.uniform(0.4, 1.2))
+
+    def put_delta(p, c, channel):
+        kw, vw = c["kv_heads"] * c["dim"], c["heads"] * c["vdim"]
+        for n, r in (("q", kw), ("k", kw), ("v", vw)):
+            lin(p + n, r, width, 1.5); vec(p + n + ".conv", (r, c["conv"]), 0.3, 0.5)
+        lin(p + "b", c["heads"], width)
+        w[p + "A_log"] = rng.uniform(-2.0, 1.0, c["heads"])
+        vec(p + "norm", c["vdim"], 1.0)
+        if channel:
+            lin(p + "a1", rank_a, width); lin(p + "a2", c["heads"] * c["dim"], rank_a, 2.0)
+            lin(p + "g1", rank_g, width); lin(p + "g2", vw, rank_g, 2.0)
+            vec(p + "dt_bias", c["heads"] * c["dim"], -2.0, 1.0)
+        else:
+            lin(p + "a", c["heads"], width); lin(p + "g", vw, width)
+            vec(p + "dt_bias", c["heads"], -2.0, 1.0)
+        lin(p + "o", width, vw)
+
+    vec("embed", (cfg["vocab"], width), 0.0, 1.0)
+    lin("head", cfg["vocab"], width, 2.0)
+    norm("final.norm")
+    for i, L in enumerate(cfg["layers"]):
+        p, m = "l%d." % i, L["mixer"]
+        norm(p + "norm1"); norm(p + "norm1b")
+        if L["type"] == "delta":
+            put_delta(p + "mix.", m, False)
+        else:
+            a = m["left"]
+            lin(p + "mix.left.q", a["heads"] * a["dim"], width); lin(p + "mix.left.k", a["kv_heads"] * a["dim"], width)
+            lin(p + "mix.left.v", a["kv_heads"] * a["vdim"], width); lin(p + "mix.left.o", width, a["heads"] * a["vdim"])
+            vec(p + "mix.left.q.norm", a["dim"], 1.3); vec(p + "mix.left.k.norm", a["dim"], 1.2)
+            put_delta(p + "mix.right.", m["right"], True)
+            vec(p + "mix.left.out", width, 1.1); vec(p + "mix.right.out", width, 0.9)
+        if L["mlp"]:
+            norm(p + "norm2"); norm(p + "norm2b")
+            lin(p + "mlp.gate", L["mlp"]["ff"], width); lin(p + "mlp.up", L["mlp"]["ff"], width); lin(p + "mlp.down", width, L["mlp"]["ff"])
+    return w
+
+
+def write(folder, cfg, w):
+    """writes config.json and model.safetensors; returns the rounded weights as float64"""
+    os.makedirs(folder, exist_ok=True)
+    with open(os.path.join(folder, "config.json"), "w") as f:
+        json.dump(cfg, f)
+    head, parts, at, out = {}, [], 0, {}
+    for name, a in w.items():
+        bits, out[name] = to_bf16(a)
+        out[name] = out[name].reshape(np.shape(a))
+        raw = bits.tobytes()
+        head[name] = dict(dtype="BF16", shape=list(np.shape(a)), data_offsets=[at, at + len(raw)])
+        parts.append(raw); at += len(raw)
+    h = json.dumps(head).encode()
+    h += b" " * (-len(h) % 8)
+    with open(os.path.join(folder, "model.safetensors"), "wb") as f:
+        f.write(struct.pack("<Q", len(h)) + h)
+        for raw in parts:
+            f.write(raw)
+    return out

@@ -1,0 +1,96 @@
+"""The layered decoder's float64 checker against independent statements of the same mechanisms, and the registry's refusals."""
+import json
+import os
+
+import numpy as np
+import pytest
+
+from helpers import layered_build as B
+from helpers import layered_ref as R
+
+
+def test_delta_rule_without_decay_recalls_what_was_written():
+    # orthogonal keys, full write strength: reading with a key returns the value last written under it
+    k = np.eye(4)[None][:, [0, 1, 2, 0, 3]].transpose(1, 0, 2)
+    v = np.arange(5 * 3, dtype=float).reshape(5, 1, 3)
+    q = np.eye(4)[[0, 0, 1, 0, 2]][:, None]
+    o = R.delta_rule(q, k, v, np.ones((5, 1, 4)), np.ones((5, 1)))
+    assert np.allclose(o[:, 0], [v[0, 0], v[0, 0], v[1, 0], v[3, 0], v[2, 0]])
+
+
+def test_delta_rule_is_a_product_of_state_transitions():
+    rng = np.random.default_rng(1)
+    T, d, dv = 6, 5, 4
+    q, k, v = rng.standard_normal((T, 1, d)), R.unit(rng.standard_normal((T, 1, d))), rng.standard_normal((T, 1, dv))
+    g, b = rng.uniform(0.2, 1.0, (T, 1, d)), rng.uniform(0, 1, (T, 1))
+    S, want = np.zeros((d, dv)), []
+    for t in range(T):
+        kk = k[t, 0][:, None]
+        S = (np.eye(d) - b[t, 0] * kk @ kk.T) @ np.diag(g[t, 0]) @ S + b[t, 0] * kk @ v[t]
+        want.append(q[t, 0] @ S)
+    assert np.allclose(R.delta_rule(q, k, v, g, b)[:, 0], want)
+
+
+def test_convolution_is_causal_and_its_last_tap_is_the_current_token():
+    x = np.random.default_rng(2).standard_normal((7, 3))
+    w = np.zeros((3, 4)); w[:, 3] = [1, 0, 0]; w[:, 1] = [0, 1, 0]; w[:, 0] = [0, 0, 1]
+    y = R.causal_conv(x, w)
+    assert np.allclose(y[:, 0], x[:, 0])
+    assert np.allclose(y[2:, 1], x[:-2, 1]) and np.all(y[:2, 1] == 0)
+    assert np.allclose(y[3:, 2], x[:-3, 2]) and np.all(y[:3, 2] == 0)
+
+
+@pytest.mark.parametrize("window", [1, 3, 50])
+def test_window_attention_sees_exactly_its_window(window):
+    rng = np.random.default_rng(3)
+    T = 9
+    q, k, v = rng.standard_normal((T, 4, 6)), rng.standard_normal((T, 2, 6)), rng.standard_normal((T, 2, 5))
+    o = R.window_attention(q, k, v, 0.3, window)
+    for i in range(T):
+        lo = max(0, i - window + 1)
+        for h in range(4):
+            s = np.exp(0.3 * k[lo:i + 1, h // 2] @ q[i, h])
+            assert np.allclose(o[i, h], (s / s.sum()) @ v[lo:i + 1, h // 2])
+
+
+def test_run_order_of_repeated_layers():
+    cfg = dict(layers=[None] * 5, loop=dict(start=1, stop=3, times=3))
+    assert R.run_order(cfg) == [(0, False), (1, False), (2, False), (1, True), (2, False), (1, True), (2, False), (3, False), (4, False)]
+    assert R.run_order(dict(layers=[None] * 2)) == [(0, False), (1, False)]
+
+
+def test_checker_is_sensitive_to_what_it_checks():
+    """a window off by one, a lost state, a wrong group or a missing repeat moves the logits well beyond the tests' tolerances"""
+    cfg = B.config([B.layer(B.delta()), B.layer((B.attn(), B.delta(dim=12)))], loop=dict(start=0, stop=2, times=2))
+    w = {n: B.to_bf16(a)[1].reshape(np.shape(a)) for n, a in B.weights(cfg, 5).items()}
+    tok = np.random.default_rng(6).integers(0, cfg["vocab"], 40)
+    base = R.forward(cfg, w, tok)
+    for change in (lambda c: c["layers"][1]["mixer"]["left"]["mask"].update(size=10), lambda c: c["loop"].update(times=1),
+                   lambda c: c["layers"][1]["mixer"]["left"].update(scale=0.25), lambda c: c["norm"].update(eps=0.1)):
+        other = json.loads(json.dumps(cfg)); change(other)
+        assert np.abs(R.forward(other, w, tok) - base).max() > 2e-2
+    assert np.abs(R.forward(cfg, w, tok[1:])[-1] - base[-1]).max() > 2e-5      # a token well before every window still counts
+
+
+@pytest.mark.parametrize("text, reason", [("{", "malformed"), ("[]", ""), ('{"architecture": "Nobody"}', "Samanex"), ("{}", "Samanex"),
+                                          ('{"architecture": "Samanex"} x', "after"), ('{"architecture": "\\ud800"}', "malformed")])
+def test_registry_refuses_what_it_does_not_know(tmp_path, text, reason):
+    from helpers.device import cai
+    (tmp_path / "config.json").write_text(text)
+    with pytest.raises(cai.CaiError) as e:
+        cai.Decoder.load(str(tmp_path), 64)
+    assert reason in str(e.value)
+
+
+def test_registry_refuses_bad_arguments(tmp_path):
+    from helpers.device import cai
+    for args in ((0, 1, 0), (64, 0, 0), (64, 1, 7)):
+        with pytest.raises(cai.CaiError):
+            cai.Decoder.load(str(tmp_path), *args)
+    with pytest.raises(cai.CaiError):
+        cai.Decoder.load(str(tmp_path / "absent"), 64)
+
+
+def test_trace_runner_is_executable():
+    root = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
+    assert os.access(os.path.join(root, "bin", "trace_run"), os.X_OK)
