@@ -11,7 +11,7 @@
 
 namespace cai {
 
-constexpr int SLICE = 256;                 // keys per work-group of the row form
+constexpr int SLICE = 64;                  // keys per work-group of the row form: a slice lies in at most two pages
 
 template <typename T> __device__ __forceinline__ float round_to(float v) { return (float)(T)v; }
 template <typename T> __device__ __forceinline__ void load8(const T* p, float* v)
@@ -111,6 +111,9 @@ __global__ __launch_bounds__(256) void attn_rows_kernel(const AttnDims d, const 
     for (int c = tid; c < d.dim_p; c += 256) page[((int64_t)g * PAGE_TOKENS + tp) * d.dim_p + c] = (T)nk[c];
     for (int c = tid; c < d.vdim_p; c += 256) page[kv.v_off + ((int64_t)g * PAGE_TOKENS + tp) * d.vdim_p + c] = (T)nv[c];
   }
+  // the slice's two pages (the second may be the first again)
+  const int pk = (k0 / PAGE_TOKENS + 1) * PAGE_TOKENS;                 // first key of the second page
+  const T* pg0 = kv_page<T>(kv, slot, k0), *pg1 = kv_page<T>(kv, slot, k0 + nkeys - 1);
   // scores: sixteen lanes a key, eight elements a lane and turn
   const int l16 = lane & 15;
   for (int kb = wave * 4 + (lane >> 4); kb < ((nkeys + 63) & ~63); kb += 64) {      // four keys of each lane group at a time: their loads are in flight together
@@ -119,7 +122,7 @@ __global__ __launch_bounds__(256) void attn_rows_kernel(const AttnDims d, const 
     for (int u = 0; u < 4; u++) {
       const int kk = min(kb + 16 * u, nkeys - 1), key = k0 + kk;
       const bool fresh = SINGLE && key == pos;
-      const T* kp = kv_page<T>(kv, slot, key) + ((int64_t)g * PAGE_TOKENS + key % PAGE_TOKENS) * d.dim_p;
+      const T* kp = (key < pk ? pg0 : pg1) + ((int64_t)g * PAGE_TOKENS + key % PAGE_TOKENS) * d.dim_p;
 #pragma unroll
       for (int t = 0; t < 2; t++) {
         const int c = l16 * 8 + t * 128;
@@ -191,7 +194,7 @@ __global__ __launch_bounds__(256) void attn_rows_kernel(const AttnDims d, const 
         if (SINGLE && key == pos) {
 #pragma unroll
           for (int i = 0; i < 8; i++) vx[u][i] = nv[cc * 8 + i];
-        } else load8<T>(kv_page<T>(kv, slot, key) + kv.v_off + ((int64_t)g * PAGE_TOKENS + key % PAGE_TOKENS) * d.vdim_p + cc * 8, vx[u]);
+        } else load8<T>((key < pk ? pg0 : pg1) + kv.v_off + ((int64_t)g * PAGE_TOKENS + key % PAGE_TOKENS) * d.vdim_p + cc * 8, vx[u]);
       }
 #pragma unroll
       for (int hh = 0; hh < HT; hh++) {
@@ -233,17 +236,36 @@ __global__ __launch_bounds__(256) void attn_rows_kernel(const AttnDims d, const 
 template <typename T>
 __global__ __launch_bounds__(256) void attn_rows_merge_kernel(const AttnDims d, const StepRows r, const int n_sl, const float* part, T* out, const int64_t ldo)
 {
-  const int h = blockIdx.x, row = blockIdx.y, pos = r.pos[row];
+  __shared__ float sm[4], sl[4], sw[256];
+  const int h = blockIdx.x, row = blockIdx.y, pos = r.pos[row], tid = threadIdx.x;
   const int used = (min(d.window, pos + 1) + SLICE - 1) / SLICE, st = d.vdim_p + 2;
   const float* p = part + ((int64_t)row * d.heads + h) * n_sl * st;
   float m = -INFINITY, l = 0.0f;
-  for (int s = 0; s < used; s++) m = fmaxf(m, p[s * st + d.vdim_p]);
-  for (int s = 0; s < used; s++) l += p[s * st + d.vdim_p + 1] * expf(p[s * st + d.vdim_p] - m);
-  const int c = threadIdx.x;
-  if (c >= d.vdim) return;
-  float o = 0.0f;
-  for (int s = 0; s < used; s++) o = fmaf(p[s * st + c], expf(p[s * st + d.vdim_p] - m), o);
-  out[row * ldo + h * d.vdim + c] = (T)(o / l);
+  for (int s = tid; s < used; s += 256) m = fmaxf(m, p[s * st + d.vdim_p]);
+  for (int o = 32; o; o >>= 1) m = fmaxf(m, __shfl_xor(m, o));
+  if ((tid & 63) == 0) sm[tid >> 6] = m;
+  __syncthreads();
+  m = fmaxf(fmaxf(sm[0], sm[1]), fmaxf(sm[2], sm[3]));
+  for (int s = tid; s < used; s += 256) l += p[s * st + d.vdim_p + 1] * expf(p[s * st + d.vdim_p] - m);
+  for (int o = 32; o; o >>= 1) l += __shfl_xor(l, o);
+  if ((tid & 63) == 0) sl[tid >> 6] = l;
+  float acc = 0.0f;
+  for (int s0 = 0; s0 < used; s0 += 256) {               // a block of slice weights at a time
+    const int ns = min(256, used - s0);
+    __syncthreads();
+    if (tid < ns) sw[tid] = expf(p[(s0 + tid) * st + d.vdim_p] - m);
+    __syncthreads();
+    if (tid < d.vdim) {
+      for (int s = 0; s < ns; s += 8) {
+        float t[8];
+#pragma unroll
+        for (int u = 0; u < 8; u++) t[u] = p[(s0 + min(s + u, ns - 1)) * st + tid];
+#pragma unroll
+        for (int u = 0; u < 8; u++) if (s + u < ns) acc = fmaf(t[u], sw[s + u], acc);
+      }
+    }
+  }
+  if (tid < d.vdim) out[row * ldo + h * d.vdim + tid] = (T)(acc / (sl[0] + sl[1] + sl[2] + sl[3]));
 }
 
 // ------------------------------------------------------------------------------------------
@@ -276,6 +298,8 @@ __global__ __launch_bounds__(256) void attn_prompt_paged_kernel(const AttnDims d
   float m = -INFINITY, l = 0.0f;
   const int first = max(0, pos0 + t0 - d.window + 1) / PAGE_TOKENS, last = (pos0 + min(t0 + ATTN_TILE, n) - 1) / PAGE_TOKENS;
   const int wlo = max(0, pos0 + min(t0 + wave * 16, n - 1) - d.window + 1), whi = pos0 + min(t0 + wave * 16 + 15, n - 1);   // keys this wave's rows see
+  const int wmin = pos0 + min(t0 + wave * 16, n - 1);                 // the wave's first row
+  const float scale2 = d.scale * 1.44269504088896340736f;             // scores in base-2 logarithms
   constexpr int KC = PAGE_TOKENS * KQ * 4 / 256, VC = PAGE_TOKENS / 2 * VQ * 2 / 256;   // 16-byte key chunks / value chunk pairs per thread
   u32x4 rk[KC], rv[VC][2];
   auto fetch = [&](int pg) {
@@ -330,32 +354,39 @@ __global__ __launch_bounds__(256) void attn_prompt_paged_kernel(const AttnDims d
       }
     }
     float mt = -INFINITY;
+    if (pg * PAGE_TOKENS + PAGE_TOKENS - 1 <= wmin && pg * PAGE_TOKENS > whi - d.window) {   // every row of the wave sees the whole page
 #pragma unroll
-    for (int t = 0; t < 4; t++)
+      for (int t = 0; t < 4; t++)
 #pragma unroll
-      for (int i = 0; i < 4; i++) {
-        const int back = qpos - (pg * PAGE_TOKENS + t * 16 + fg * 4 + i);
-        s[t][i] = back >= 0 && back < d.window ? s[t][i] * d.scale : -INFINITY;
-        mt = fmaxf(mt, s[t][i]);
-      }
+        for (int i = 0; i < 4; i++) { s[t][i] *= scale2; mt = fmaxf(mt, s[t][i]); }
+    } else {
+#pragma unroll
+      for (int t = 0; t < 4; t++)
+#pragma unroll
+        for (int i = 0; i < 4; i++) {
+          const int back = qpos - (pg * PAGE_TOKENS + t * 16 + fg * 4 + i);
+          s[t][i] = back >= 0 && back < d.window ? s[t][i] * scale2 : -INFINITY;
+          mt = fmaxf(mt, s[t][i]);
+        }
+    }
     mt = fmaxf(mt, __shfl_xor(mt, 16)); mt = fmaxf(mt, __shfl_xor(mt, 32));
-    const float mn = fmaxf(m, mt), mr = mn == -INFINITY ? 0.0f : mn, al = expf(m - mr);
+    const float mn = fmaxf(m, mt), mr = mn == -INFINITY ? 0.0f : mn, al = __builtin_amdgcn_exp2f(m - mr);
     m = mn; l *= al;
 #pragma unroll
     for (int v = 0; v < VQ; v++) o[v] *= al;
-    // weights in three bfloat16 parts: p = p0 + p1 + p2 exactly
-    uint16_t w[3][16];
+    // weights in three bfloat16 parts, p = p0 + p1 + p2 exactly (upper halves of p and of what is left)
+    uint32_t w[3][16];
 #pragma unroll
     for (int t = 0; t < 4; t++)
 #pragma unroll
       for (int i = 0; i < 4; i++) {
-        const float p = expf(s[t][i] - mr);
+        const float p = __builtin_amdgcn_exp2f(s[t][i] - mr);
         l += p;
-        const float a = __builtin_bit_cast(float, __builtin_bit_cast(uint32_t, p) & 0xffff0000u), pr = p - a;
-        const float b = __builtin_bit_cast(float, __builtin_bit_cast(uint32_t, pr) & 0xffff0000u);
-        w[0][t * 4 + i] = (uint16_t)(__builtin_bit_cast(uint32_t, a) >> 16);
-        w[1][t * 4 + i] = (uint16_t)(__builtin_bit_cast(uint32_t, b) >> 16);
-        w[2][t * 4 + i] = bf16_bits(pr - b);
+        const uint32_t b0 = __builtin_bit_cast(uint32_t, p);
+        const float r1 = p - __builtin_bit_cast(float, b0 & 0xffff0000u);
+        const uint32_t b1 = __builtin_bit_cast(uint32_t, r1);
+        w[0][t * 4 + i] = b0; w[1][t * 4 + i] = b1;
+        w[2][t * 4 + i] = __builtin_bit_cast(uint32_t, r1 - __builtin_bit_cast(float, b1 & 0xffff0000u));
       }
 #pragma unroll
     for (int hp = 0; hp < 2; hp++) {
@@ -363,7 +394,7 @@ __global__ __launch_bounds__(256) void attn_prompt_paged_kernel(const AttnDims d
 #pragma unroll
       for (int q = 0; q < 3; q++)
 #pragma unroll
-        for (int j = 0; j < 4; j++) fp[q][j] = w[q][hp * 8 + 2 * j] | (uint32_t)w[q][hp * 8 + 2 * j + 1] << 16;
+        for (int j = 0; j < 4; j++) fp[q][j] = __builtin_amdgcn_perm(w[q][hp * 8 + 2 * j + 1], w[q][hp * 8 + 2 * j], 0x07060302);   // upper halves of two words
 #pragma unroll
       for (int v = 0; v < VQ; v++) {
         const uint16_t* vr = sv + (v * 16 + fr) * VST + hp * 32 + fg * 4;

@@ -46,52 +46,133 @@ __device__ __forceinline__ float conv_silu(const float* cur, int64_t ldp, int ba
 }
 
 // ------------------------------------------------------------------------------------------
-// prompt pass 1: one work-group per row; q and k unit vectors (q scaled), v, decay, write strength, q . k
+// prompt pass 1: q and k unit vectors (q scaled), v, decay (its logarithm for the chunked pass), write strength, q . k.
+// A wave owns one unit - the q and k channels of a key head, 256 channels of v, 256 decays, the write strengths - over eight
+// consecutive rows; the convolution slides over them, so each input is fetched once (TAPS = 4; other lengths look back per row).
 // ------------------------------------------------------------------------------------------
-__global__ __launch_bounds__(256) void delta_prep_kernel(const DeltaDims d, const DeltaIn in, const DeltaW w, const float* hist, const int64_t h_elems, const StepRows r, const DeltaBuf b)
-{
-  const int row = blockIdx.x, lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
-  const int pos = r.pos[row], back = row - r.first[row], C = d.channels(), kw = d.kv_heads * d.dim;
-  const float* ring = hist + r.slot[row] * h_elems;
-  const float* p = in.proj + row * in.ldp;
-  const float qs = rsqrtf((float)d.dim);
-  for (int g = wave; g < d.kv_heads; g += 4) {
-    float q[4], k[4], sq = 0.0f, sk = 0.0f, dot = 0.0f;
+constexpr int PREP_ROWS = 8;
+
+template <int TAPS>
+struct ConvWindow {                        // four channels of a lane: c = lane + 64 i
+  float w[4][TAPS], h[4][TAPS - 1];        // taps, the inputs before the current one (h[0] the latest)
+  __device__ __forceinline__ void taps(const float* cw, int c0, int lane, int n)
+  {
 #pragma unroll
-    for (int i = 0; i < 4; i++) {
-      const int c = lane + 64 * i, ch = g * d.dim + c;
-      q[i] = k[i] = 0.0f;
-      if (c < d.dim) {
-        q[i] = conv_silu(p + in.oq, in.ldp, back, pos, ring, C, 0, w.cq, d.taps, ch);
-        k[i] = conv_silu(p + in.ok, in.ldp, back, pos, ring, C, kw, w.ck, d.taps, ch);
+    for (int i = 0; i < 4; i++)
+#pragma unroll
+      for (int k = 0; k < TAPS; k++) { const int c = lane + 64 * i; w[i][k] = c < n ? cw[(c0 + c) * TAPS + k] : 0.0f; }
+  }
+  __device__ __forceinline__ void history(const float* cur, int64_t ldp, int back, int pos, const float* ring, int channels, int hc, int c0, int lane, int n)
+  {
+#pragma unroll
+    for (int i = 0; i < 4; i++)
+#pragma unroll
+      for (int j = 1; j < TAPS; j++) {
+        const int c = lane + 64 * i;
+        h[i][j - 1] = 0.0f;
+        if (c < n) {
+          if (j <= back) h[i][j - 1] = cur[c0 + c - (int64_t)j * ldp];
+          else if (j <= pos) h[i][j - 1] = ring[(int64_t)((pos - j) % TAPS) * channels + hc + c0 + c];
+        }
       }
-      sq = fmaf(q[i], q[i], sq); sk = fmaf(k[i], k[i], sk); dot = fmaf(q[i], k[i], dot);
-    }
-    const float nq = qs / sqrtf(wave_total(sq) + 1e-6f), nk = 1.0f / sqrtf(wave_total(sk) + 1e-6f);
-    dot = wave_total(dot) * nq * nk;
+  }
+  __device__ __forceinline__ float step(int i, float x)
+  {
+    float s = w[i][TAPS - 1] * x;
 #pragma unroll
+    for (int j = 1; j < TAPS; j++) s = fmaf(w[i][TAPS - 1 - j], h[i][j - 1], s);
+#pragma unroll
+    for (int j = TAPS - 2; j > 0; j--) h[i][j] = h[i][j - 1];
+    h[i][0] = x;
+    return s * sigmoid_f(s);
+  }
+};
+
+template <int TAPS>
+__global__ __launch_bounds__(256) void delta_prep_kernel(const DeltaDims d, const DeltaIn in, const DeltaW w, const float* hist, const int64_t h_elems, const StepRows r, const DeltaBuf b, const int log_decay)
+{
+  const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+  const int r0 = blockIdx.x * PREP_ROWS, r1 = min(r0 + PREP_ROWS, r.n_rows);
+  const int C = d.channels(), kw = d.kv_heads * d.dim, vw = d.heads * d.vdim, bw = d.heads + d.kv_heads;
+  const int gw = d.channel_decay ? d.heads * d.dim : d.heads;
+  const int nv = (vw + 255) / 256, ng = (gw + 255) / 256;
+  int unit = blockIdx.y * 4 + wave;
+  if (unit < d.kv_heads) {
+    const int g = unit, c0 = g * d.dim;
+    const float qs = rsqrtf((float)d.dim);
+    ConvWindow<TAPS ? TAPS : 2> wq, wk;
+    if (TAPS) { wq.taps(w.cq, c0, lane, d.dim); wk.taps(w.ck, c0, lane, d.dim); }
+    for (int row = r0; row < r1; row++) {
+      const int pos = r.pos[row], back = row - r.first[row];
+      const float* ring = hist + r.slot[row] * h_elems;
+      const float* p = in.proj + row * in.ldp;
+      if (TAPS && (row == r0 || back == 0)) {
+        wq.history(p + in.oq, in.ldp, back, pos, ring, C, 0, c0, lane, d.dim);
+        wk.history(p + in.ok, in.ldp, back, pos, ring, C, kw, c0, lane, d.dim);
+      }
+      float q[4], k[4], sq = 0.0f, sk = 0.0f, dot = 0.0f;
+#pragma unroll
+      for (int i = 0; i < 4; i++) { const int c = lane + 64 * i; q[i] = c < d.dim ? p[in.oq + c0 + c] : 0.0f; k[i] = c < d.dim ? p[in.ok + c0 + c] : 0.0f; }
+#pragma unroll
+      for (int i = 0; i < 4; i++) {
+        const int c = lane + 64 * i;
+        if (i * 64 >= d.dim) continue;
+        if (TAPS) { q[i] = wq.step(i, q[i]); k[i] = wk.step(i, k[i]); }
+        else if (c < d.dim) {
+          q[i] = conv_silu(p + in.oq, in.ldp, back, pos, ring, C, 0, w.cq, d.taps, c0 + c);
+          k[i] = conv_silu(p + in.ok, in.ldp, back, pos, ring, C, kw, w.ck, d.taps, c0 + c);
+        }
+        sq = fmaf(q[i], q[i], sq); sk = fmaf(k[i], k[i], sk); dot = fmaf(q[i], k[i], dot);
+      }
+      const float nq = qs / sqrtf(wave_total(sq) + 1e-6f), nk = 1.0f / sqrtf(wave_total(sk) + 1e-6f);
+      dot = wave_total(dot) * nq * nk;
+#pragma unroll
+      for (int i = 0; i < 4; i++) {
+        const int c = lane + 64 * i;
+        if (c < d.dim) { b.q[(int64_t)row * kw + c0 + c] = q[i] * nq; b.k[(int64_t)row * kw + c0 + c] = k[i] * nk; }
+      }
+      if (lane == 0) b.beta[(int64_t)row * bw + d.heads + g] = dot;
+    }
+    return;
+  }
+  unit -= d.kv_heads;
+  if (unit < nv) {
+    const int c0 = unit * 256, n = min(256, vw - c0);
+    ConvWindow<TAPS ? TAPS : 2> wv;
+    if (TAPS) wv.taps(w.cv, c0, lane, n);
+    for (int row = r0; row < r1; row++) {
+      const int pos = r.pos[row], back = row - r.first[row];
+      const float* ring = hist + r.slot[row] * h_elems;
+      const float* p = in.proj + row * in.ldp + in.ov;
+      if (TAPS && (row == r0 || back == 0)) wv.history(p, in.ldp, back, pos, ring, C, 2 * kw, c0, lane, n);
+#pragma unroll
+      for (int i = 0; i < 4; i++) {
+        const int c = lane + 64 * i;
+        if (TAPS) { const float v = wv.step(i, c < n ? p[c0 + c] : 0.0f); if (c < n) b.v[(int64_t)row * vw + c0 + c] = v; }
+        else if (c < n) b.v[(int64_t)row * vw + c0 + c] = conv_silu(p, in.ldp, back, pos, ring, C, 2 * kw, w.cv, d.taps, c0 + c);
+      }
+    }
+    return;
+  }
+  unit -= nv;
+  if (unit < ng) {
     for (int i = 0; i < 4; i++) {
-      const int c = lane + 64 * i;
-      if (c < d.dim) { b.q[(int64_t)row * kw + g * d.dim + c] = q[i] * nq; b.k[(int64_t)row * kw + g * d.dim + c] = k[i] * nk; }
+      const int c = unit * 256 + lane + 64 * i;
+      if (c >= gw) continue;
+      const float bias = w.dt_bias[c], rate = w.rate[d.channel_decay ? c / d.dim : c];
+#pragma unroll
+      for (int u = 0; u < PREP_ROWS; u++) {
+        const int row = min(r0 + u, r1 - 1);
+        const float z = d.rank_a ? b.za[(int64_t)row * gw + c] : in.proj[row * in.ldp + in.oa + c];
+        const float l = rate * softplus_f(z + bias);
+        b.g[(int64_t)row * gw + c] = log_decay ? l : expf(l);
+      }
     }
-    if (lane == 0) b.beta[(int64_t)row * (d.heads + d.kv_heads) + d.heads + g] = dot;
+    return;
   }
-  const int vw = d.heads * d.vdim;
-  for (int c = threadIdx.x; c < vw; c += 256)
-    b.v[(int64_t)row * vw + c] = conv_silu(p + in.ov, in.ldp, back, pos, ring, C, 2 * kw, w.cv, d.taps, c);
-  for (int h = threadIdx.x; h < d.heads; h += 256) b.beta[(int64_t)row * (d.heads + d.kv_heads) + h] = sigmoid_f(p[in.ob + h]);
-  if (d.channel_decay) {
-    const int gw = d.heads * d.dim;
-    for (int c = threadIdx.x; c < gw; c += 256) {
-      const float z = (d.rank_a ? b.za[(int64_t)row * gw + c] : p[in.oa + c]) + w.dt_bias[c];
-      b.g[(int64_t)row * gw + c] = expf(w.rate[c / d.dim] * softplus_f(z));
-    }
-  } else {
-    for (int h = threadIdx.x; h < d.heads; h += 256) {
-      const float z = (d.rank_a ? b.za[(int64_t)row * d.heads + h] : p[in.oa + h]) + w.dt_bias[h];
-      b.g[(int64_t)row * d.heads + h] = expf(w.rate[h] * softplus_f(z));
-    }
-  }
+  if (unit == ng)
+    for (int row = r0; row < r1; row++)
+      for (int h = lane; h < d.heads; h += 64) b.beta[(int64_t)row * bw + h] = sigmoid_f(in.proj[row * in.ldp + in.ob + h]);
 }
 
 // ------------------------------------------------------------------------------------------
@@ -378,9 +459,13 @@ __global__ __launch_bounds__(1024) void delta_single_kernel(const DeltaDims d, c
   }
 }
 
-int delta_prep(const DeltaDims& d, const DeltaIn& in, const DeltaW& w, const SeqPool::DeltaRun& st, const StepRows& r, const DeltaBuf& b)
+int delta_prep(const DeltaDims& d, const DeltaIn& in, const DeltaW& w, const SeqPool::DeltaRun& st, const StepRows& r, const DeltaBuf& b, bool log_decay)
 {
-  hipLaunchKernelGGL(delta_prep_kernel, dim3(r.n_rows), dim3(256), 0, ctx().stream, d, in, w, st.hist, st.h_elems, r, b);
+  const int gw = d.channel_decay ? d.heads * d.dim : d.heads;
+  const int units = d.kv_heads + (d.heads * d.vdim + 255) / 256 + (gw + 255) / 256 + 1;
+  const dim3 grid((r.n_rows + PREP_ROWS - 1) / PREP_ROWS, (units + 3) / 4);
+  if (d.taps == 4) hipLaunchKernelGGL(delta_prep_kernel<4>, grid, dim3(256), 0, ctx().stream, d, in, w, st.hist, st.h_elems, r, b, (int)log_decay);
+  else hipLaunchKernelGGL(delta_prep_kernel<0>, grid, dim3(256), 0, ctx().stream, d, in, w, st.hist, st.h_elems, r, b, (int)log_decay);
   CAI_HIP(hipGetLastError());
   return CAI_OK;
 }

@@ -156,26 +156,40 @@ __global__ __launch_bounds__(256) void net_embed_kernel(const uint16_t* e, const
 // Two outputs side by side: each RMS-normed over the width with its own gain, half their sum through `post` onto the residual
 // stream (+ add0), then the next sublayer's input.
 template <typename AT>
-__global__ __launch_bounds__(256) void net_join_kernel(const float* yl, const float* yr, const float* gl, const float* gr, const int width, const float eps,
-                                                       float* x, const float* add0, const Dyt post, const Dyt next, AT* h, const int64_t ldh)
+__global__ __launch_bounds__(1024) void net_join_kernel(const float* yl, const float* yr, const float* gl, const float* gr, const int width, const float eps,
+                                                        float* x, const float* add0, const Dyt post, const Dyt next, AT* h, const int64_t ldh)
 {
-  __shared__ float sl[4], sr[4];
+  __shared__ float sl[16], sr[16];
   const int64_t t = blockIdx.x;
+  const int tid = threadIdx.x;
   const float *a = yl + t * width, *b = yr + t * width;
+  // up to four values a thread stay in registers; wider rows are read again
+  float av[4], bv[4], xv[4];
   float s = 0.0f, q = 0.0f;
-  for_strided8(a, threadIdx.x, width, 256, [&](float v, int) { s = fmaf(v, v, s); });
-  for_strided8(b, threadIdx.x, width, 256, [&](float v, int) { q = fmaf(v, v, q); });
+#pragma unroll
+  for (int u = 0; u < 4; u++) {
+    const int i = min(tid + u * 1024, width - 1);
+    av[u] = a[i]; bv[u] = b[i]; xv[u] = x[t * width + i];
+  }
+#pragma unroll
+  for (int u = 0; u < 4; u++) if (tid + u * 1024 < width) { s = fmaf(av[u], av[u], s); q = fmaf(bv[u], bv[u], q); }
+  for (int i = tid + 4096; i < width; i += 1024) { s = fmaf(a[i], a[i], s); q = fmaf(b[i], b[i], q); }
   for (int o = 32; o; o >>= 1) { s += __shfl_xor(s, o); q += __shfl_xor(q, o); }
-  if ((threadIdx.x & 63) == 0) { sl[threadIdx.x >> 6] = s; sr[threadIdx.x >> 6] = q; }
+  if ((tid & 63) == 0) { sl[tid >> 6] = s; sr[tid >> 6] = q; }
   __syncthreads();
-  const float il = 1.0f / sqrtf((sl[0] + sl[1] + sl[2] + sl[3]) / (float)width + eps), ir = 1.0f / sqrtf((sr[0] + sr[1] + sr[2] + sr[3]) / (float)width + eps);
-  for (int i = threadIdx.x; i < width; i += 256) {
-    const float y = 0.5f * (a[i] * il * gl[i] + b[i] * ir * gr[i]);
-    float v = x[t * width + i] + dyt(post, y, i);
+  s = q = 0.0f;
+#pragma unroll
+  for (int u = 0; u < 16; u++) { s += sl[u]; q += sr[u]; }
+  const float il = 1.0f / sqrtf(s / (float)width + eps), ir = 1.0f / sqrtf(q / (float)width + eps);
+  auto put = [&](int i, float va, float vb, float vx) {
+    float v = vx + dyt(post, 0.5f * (va * il * gl[i] + vb * ir * gr[i]), i);
     if (add0) v += add0[t * width + i];
     x[t * width + i] = v;
     h[t * ldh + i] = (AT)dyt(next, v, i);
-  }
+  };
+#pragma unroll
+  for (int u = 0; u < 4; u++) if (tid + u * 1024 < width) put(tid + u * 1024, av[u], bv[u], xv[u]);
+  for (int i = tid + 4096; i < width; i += 1024) put(i, a[i], b[i], x[t * width + i]);
 }
 
 template <typename AT>
@@ -395,7 +409,7 @@ static int enqueue_net(LayeredNet* n, const StepRows& r, bool single, const int3
         LinEpi e; e.y = n->db.zg; e.ldy = D.w.g2->rows;
         if ((rc = launch_pack_rows(n->proj, n->ld_proj, D.og, D.d.rank_g, R, at, n->rgb, n->ld_rg)) || (rc = launch_lin(D.w.g2, at, n->rgb, n->ld_rg, R, e))) return rc;
       }
-      if ((rc = delta_prep(D.d, din, D.w, ds, r, n->db)) || (rc = delta_scan(D.d, ds, r, n->db)) || (rc = delta_finish(D.d, din, D.w, ds, r, n->db, at, n->att, n->ld_att))) return rc;
+      if ((rc = delta_prep(D.d, din, D.w, ds, r, n->db, false)) || (rc = delta_scan(D.d, ds, r, n->db)) || (rc = delta_finish(D.d, din, D.w, ds, r, n->db, at, n->att, n->ld_att))) return rc;
     }
     LinEpi res; res.mode = EPI_RESIDUAL; res.y = n->x; res.ldy = w; res.h = n->h; res.ldh = n->wp; res.post = y.norm1b;
     if (y.gateup) res.next = y.norm2;
@@ -410,8 +424,8 @@ static int enqueue_net(LayeredNet* n, const StepRows& r, bool single, const int3
       if (rc) return rc;
       LinEpi el, er; el.y = n->yl; er.y = n->yr; el.ldy = er.ldy = w;
       if ((rc = launch_lin(A.out, at, n->attl, n->ld_attl, R, el)) || (rc = launch_lin(D.out, at, n->att, n->ld_att, R, er))) return rc;
-      if (at == ACT_T_BF16) hipLaunchKernelGGL(net_join_kernel<bf16_t>, dim3(R), dim3(256), 0, st, n->yl, n->yr, y.gain_left, y.gain_right, w, s.eps, n->x, res.add0, res.post, res.next, (bf16_t*)n->h, (int64_t)n->wp);
-      else hipLaunchKernelGGL(net_join_kernel<float>, dim3(R), dim3(256), 0, st, n->yl, n->yr, y.gain_left, y.gain_right, w, s.eps, n->x, res.add0, res.post, res.next, (float*)n->h, (int64_t)n->wp);
+      if (at == ACT_T_BF16) hipLaunchKernelGGL(net_join_kernel<bf16_t>, dim3(R), dim3(1024), 0, st, n->yl, n->yr, y.gain_left, y.gain_right, w, s.eps, n->x, res.add0, res.post, res.next, (bf16_t*)n->h, (int64_t)n->wp);
+      else hipLaunchKernelGGL(net_join_kernel<float>, dim3(R), dim3(1024), 0, st, n->yl, n->yr, y.gain_left, y.gain_right, w, s.eps, n->x, res.add0, res.post, res.next, (float*)n->h, (int64_t)n->wp);
     } else if ((rc = launch_lin(D.out, at, n->att, n->ld_att, R, res))) return rc;
     if (y.gateup) {
       LinEpi g; g.mode = EPI_GLU; g.h = n->mid; g.ldh = n->ld_mid; g.glu = y.glu;

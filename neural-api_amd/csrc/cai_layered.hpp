@@ -125,7 +125,7 @@ struct DeltaW {
   const cai_qw_s *a2, *g2;                 // low-rank seconds (CAI_BF16), null when direct
 };
 struct DeltaBuf { float *q, *k, *v, *g, *beta, *o, *za, *zg; };   // per-row scratch of a prompt pass
-int delta_prep(const DeltaDims& d, const DeltaIn& in, const DeltaW& w, const SeqPool::DeltaRun& st, const StepRows& r, const DeltaBuf& b);
+int delta_prep(const DeltaDims& d, const DeltaIn& in, const DeltaW& w, const SeqPool::DeltaRun& st, const StepRows& r, const DeltaBuf& b, bool log_decay);
 int delta_scan(const DeltaDims& d, const SeqPool::DeltaRun& st, const StepRows& r, const DeltaBuf& b);
 int delta_finish(const DeltaDims& d, const DeltaIn& in, const DeltaW& w, const SeqPool::DeltaRun& st, const StepRows& r, const DeltaBuf& b, int act_t, void* out, int64_t ldo);
 int delta_single(const DeltaDims& d, const DeltaIn& in, const DeltaW& w, const SeqPool::DeltaRun& st, const StepRows& r, int act_t, void* out, int64_t ldo);
