@@ -46,7 +46,7 @@ __device__ __forceinline__ float conv_silu(const float* cur, int64_t ldp, int ba
 }
 
 // ------------------------------------------------------------------------------------------
-// prompt pass 1: q and k unit vectors (q scaled), v, decay (its logarithm for the chunked pass), write strength, q . k.
+// prompt pass 1: q and k unit vectors (q scaled), v, decay, write strength, q . k.
 // A wave owns one unit - the q and k channels of a key head, 256 channels of v, 256 decays, the write strengths - over eight
 // consecutive rows; the convolution slides over them, so each input is fetched once (TAPS = 4; other lengths look back per row).
 // ------------------------------------------------------------------------------------------
@@ -89,7 +89,7 @@ struct ConvWindow {                        // four channels of a lane: c = lane 
 };
 
 template <int TAPS>
-__global__ __launch_bounds__(256) void delta_prep_kernel(const DeltaDims d, const DeltaIn in, const DeltaW w, const float* hist, const int64_t h_elems, const StepRows r, const DeltaBuf b, const int log_decay)
+__global__ __launch_bounds__(256) void delta_prep_kernel(const DeltaDims d, const DeltaIn in, const DeltaW w, const float* hist, const int64_t h_elems, const StepRows r, const DeltaBuf b)
 {
   const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const int r0 = blockIdx.x * PREP_ROWS, r1 = min(r0 + PREP_ROWS, r.n_rows);
@@ -164,8 +164,7 @@ __global__ __launch_bounds__(256) void delta_prep_kernel(const DeltaDims d, cons
       for (int u = 0; u < PREP_ROWS; u++) {
         const int row = min(r0 + u, r1 - 1);
         const float z = d.rank_a ? b.za[(int64_t)row * gw + c] : in.proj[row * in.ldp + in.oa + c];
-        const float l = rate * softplus_f(z + bias);
-        b.g[(int64_t)row * gw + c] = log_decay ? l : expf(l);
+        b.g[(int64_t)row * gw + c] = expf(rate * softplus_f(z + bias));
       }
     }
     return;
@@ -176,7 +175,7 @@ __global__ __launch_bounds__(256) void delta_prep_kernel(const DeltaDims d, cons
 }
 
 // ------------------------------------------------------------------------------------------
-// prompt pass 2: the scan.  A wave owns four columns of one head's state: 16 lanes a column, RPL rows a lane (rows
+// prompt pass 2 for short portions: the scan.  A wave owns four columns of one head's state: 16 lanes a column, RPL rows a lane (rows
 // 64 j + 4 (lane & 15) + i), in registers for the whole portion.  Tokens are staged through LDS 16 at a time, the next block
 // requested before the current one is walked; the walk itself has no barrier.
 // ------------------------------------------------------------------------------------------
@@ -275,6 +274,268 @@ __global__ __launch_bounds__(256) void delta_scan_kernel(const DeltaDims d, floa
     const int rr = (j >> 2) * 64 + rg * 4 + (j & 3);
     if (rr < d.dim && col < dvp) Sg[(int64_t)rr * dvp + col] = S[j];
   }
+}
+
+// ------------------------------------------------------------------------------------------
+// prompt pass 2 for long portions: the same recurrence in chunks of 16 tokens, on the float matrix cores (32-bit throughout).
+//
+// With P_t the product of the decays of the chunk's tokens up to t, D_ts that of the tokens after s up to t, and S the state
+// before the chunk, the writes u of a chunk solve a unit lower triangular system,
+//     u_t = beta_t (v_t - S^T (P_t k_t) - sum_{s<t} A_ts u_s),   A_ts = k_t . D_ts k_s,
+// so with T = (I + diag(beta) A)^-1 diag(beta):   U = T V - (T [P k]) S =: U0 - W S.   Then
+//     o_t = S^T (P_t q_t) + sum_{s<=t} (q_t . D_ts k_s) u_s,      S <- P_16 S + sum_s (D_16,s k_s) u_s^T.
+// Everything before "S" is made for all chunks at once (first kernel); the second kernel walks the chunks of a sequence with a
+// 16-column slice of the state in registers.  Decays enter only as running products, never as quotients or differences of
+// logarithms, so strong decay costs no accuracy.
+// ------------------------------------------------------------------------------------------
+constexpr int CHUNK = DELTA_CHUNK;
+
+template <bool CH>
+__global__ __launch_bounds__(256) void delta_chunk_kernel(const DeltaDims d, const StepRows r, const DeltaBuf b, const int32_t* chunks)
+{
+  extern __shared__ float lds[];
+  __shared__ float sA[CHUNK][CHUNK + 1], sQ[CHUNK][CHUNK + 1], sP[CH ? 1 : 4][CHUNK][CHUNK + 1];
+  __shared__ f32x4 sT[CHUNK][CHUNK / 4];
+  __shared__ float sbeta[CHUNK], sg1[CHUNK], sdot[CHUNK];
+  const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), fr = lane & 15, fg = lane >> 4;
+  const int32_t* en = r.ent + 4 * chunks[2 * blockIdx.x];
+  const int t0 = chunks[2 * blockIdx.x + 1], nt = min(CHUNK, en[2] - t0), h = blockIdx.y;
+  const int64_t row0 = en[1] + t0;
+  const int g = h / (d.heads / d.kv_heads), kw = d.kv_heads * d.dim, vw = d.heads * d.vdim, gw = d.heads * d.dim, bw = d.heads + d.kv_heads;
+  const int dp = (d.dim + 15) & ~15, DS = dp + 4;
+  float *sk = lds, *sq = lds + CHUNK * DS, *sg = lds + 2 * CHUNK * DS;       // sg: channel decays, later their running products
+  for (int e = tid; e < CHUNK * dp; e += 256) {
+    const int t = e / dp, c = e - t * dp;
+    const bool ok = t < nt && c < d.dim;
+    const int64_t rw = row0 + (ok ? t : 0); const int cc = ok ? c : 0;
+    const float k = b.k[rw * kw + g * d.dim + cc], q = b.q[rw * kw + g * d.dim + cc];
+    sk[t * DS + c] = ok ? k : 0.0f; sq[t * DS + c] = ok ? q : 0.0f;
+    if (CH) { const float x = b.g[rw * gw + h * d.dim + cc]; sg[t * DS + c] = ok ? x : 1.0f; }
+  }
+  if (tid < CHUNK) {
+    const bool ok = tid < nt; const int64_t rw = row0 + (ok ? tid : 0);
+    sbeta[tid] = ok ? b.beta[rw * bw + h] : 0.0f; sdot[tid] = ok ? b.beta[rw * bw + d.heads + g] : 0.0f;
+    sg1[tid] = !CH && ok ? b.g[rw * d.heads + h] : 1.0f;
+  }
+  __syncthreads();
+  if (CH) {
+    // thread (s, 16 channel lanes): running product of the decays after s
+    const int s = tid >> 4, cl = tid & 15;
+    float a[CHUNK], o[CHUNK];
+#pragma unroll
+    for (int t = 0; t < CHUNK; t++) a[t] = o[t] = 0.0f;
+    for (int c = cl; c < dp; c += 16) {
+      const float ks = sk[s * DS + c];
+      float e = ks;
+#pragma unroll
+      for (int t = 1; t < CHUNK; t++) {
+        e = t > s ? e * sg[t * DS + c] : e;
+        a[t] = fmaf(sk[t * DS + c], e, a[t]); o[t] = fmaf(sq[t * DS + c], e, o[t]);
+      }
+    }
+#pragma unroll
+    for (int t = 0; t < CHUNK; t++) {
+      const float x = row16_total(a[t]), y = row16_total(o[t]);
+      if (cl == 0) { sA[t][s] = t > s ? x : 0.0f; sQ[t][s] = t > s ? y : t == s ? sdot[t] : 0.0f; }
+    }
+    __syncthreads();
+    // k times the decays behind it (in place of the decays), q times those up to it, the chunk's whole decay
+    for (int c = tid; c < dp; c += 256) {
+      float z = 1.0f;
+      float gr[CHUNK];
+#pragma unroll
+      for (int t = CHUNK - 1; t >= 0; t--) {
+        gr[t] = sg[t * DS + c];
+        if (t < nt && c < d.dim) b.g[(row0 + t) * gw + h * d.dim + c] = sk[t * DS + c] * z;
+        z *= gr[t];
+      }
+      float p = 1.0f;
+#pragma unroll
+      for (int t = 0; t < CHUNK; t++) {
+        p *= gr[t];
+        sg[t * DS + c] = p;
+        if (t < nt && c < d.dim) b.qt[(row0 + t) * gw + h * d.dim + c] = sq[t * DS + c] * p;
+      }
+      if (c < d.dim) b.gt[(int64_t)blockIdx.x * gw + h * d.dim + c] = p;
+    }
+  } else {
+    // K K^T and Q K^T, half of the width by each of two waves
+    f32x4 acc = {0.0f, 0.0f, 0.0f, 0.0f};
+    const float* am = wave & 1 ? sq : sk;
+    for (int kt = wave >> 1; kt < dp / 16; kt += 2) {
+      const f32x4 x = *reinterpret_cast<const f32x4*>(am + fr * DS + kt * 16 + fg * 4), y = *reinterpret_cast<const f32x4*>(sk + fr * DS + kt * 16 + fg * 4);
+#pragma unroll
+      for (int i = 0; i < 4; i++) acc = __builtin_amdgcn_mfma_f32_16x16x4f32(x[i], y[i], acc, 0, 0, 0);
+    }
+#pragma unroll
+    for (int i = 0; i < 4; i++) sP[wave][fg * 4 + i][fr] = acc[i];
+    __syncthreads();
+    const int t = tid >> 4, s = tid & 15;
+    float e = t >= s ? 1.0f : 0.0f;
+#pragma unroll
+    for (int x = 1; x < CHUNK; x++) e *= x > s && x <= t ? sg1[x] : 1.0f;
+    sA[t][s] = t > s ? e * (sP[0][t][s] + sP[2][t][s]) : 0.0f;
+    sQ[t][s] = e * (sP[1][t][s] + sP[3][t][s]);
+    if (tid < nt) {
+      float p = 1.0f, z = 1.0f;
+#pragma unroll
+      for (int x = 0; x < CHUNK; x++) { p *= x <= tid ? sg1[x] : 1.0f; z *= x > tid ? sg1[x] : 1.0f; }
+      float* o = b.gt + ((row0 + tid) * d.heads + h) * 2;
+      o[0] = p; o[1] = z;
+    }
+  }
+  __syncthreads();
+  {
+    const int t = tid >> 4, s = tid & 15;
+    if (t < nt) b.qk[((row0 + t) * d.heads + h) * CHUNK + s] = sQ[t][s];
+  }
+  if (tid < CHUNK) {                       // column tid of T by forward substitution
+    float c[CHUNK];
+#pragma unroll
+    for (int t = 0; t < CHUNK; t++) {
+      float x = t == tid ? 1.0f : 0.0f;
+#pragma unroll
+      for (int s = 0; s < t; s++) x = fmaf(-sA[t][s], c[s], x);
+      c[t] = x * sbeta[t];
+      reinterpret_cast<float*>(sT[t])[tid] = c[t];
+    }
+  }
+  if (!CH && tid >= 64 && tid < 64 + CHUNK) {            // running products for T [P k]
+    float p = 1.0f;
+    for (int x = 0; x <= tid - 64; x++) p *= sg1[x];
+    sdot[tid - 64] = p;
+  }
+  __syncthreads();
+  const f32x4 tf = sT[fr][fg];
+  for (int ct = wave; ct < dp / 16; ct += 4) {           // W = T [P k]
+    f32x4 acc = {0.0f, 0.0f, 0.0f, 0.0f};
+    const int c = ct * 16 + fr;
+#pragma unroll
+    for (int i = 0; i < 4; i++) {
+      const int s = fg * 4 + i;
+      acc = __builtin_amdgcn_mfma_f32_16x16x4f32(tf[i], sk[s * DS + c] * (CH ? sg[s * DS + c] : sdot[s]), acc, 0, 0, 0);
+    }
+#pragma unroll
+    for (int i = 0; i < 4; i++) if (fg * 4 + i < nt && c < d.dim) b.w[(row0 + fg * 4 + i) * gw + h * d.dim + c] = acc[i];
+  }
+  for (int ct = wave; ct * 16 < d.vdim; ct += 4) {       // U0 = T V, in place of V
+    f32x4 acc = {0.0f, 0.0f, 0.0f, 0.0f};
+    const int c = ct * 16 + fr;
+    float x[4];
+#pragma unroll
+    for (int i = 0; i < 4; i++) x[i] = fg * 4 + i < nt && c < d.vdim ? b.v[(row0 + fg * 4 + i) * vw + h * d.vdim + c] : 0.0f;
+#pragma unroll
+    for (int i = 0; i < 4; i++) acc = __builtin_amdgcn_mfma_f32_16x16x4f32(tf[i], x[i], acc, 0, 0, 0);
+#pragma unroll
+    for (int i = 0; i < 4; i++) if (fg * 4 + i < nt && c < d.vdim) b.v[(row0 + fg * 4 + i) * vw + h * d.vdim + c] = acc[i];
+  }
+}
+
+// The walk: one work-group per (16 value columns, head, entry); wave w holds key rows of tiles w TPW .. as matrix-core result
+// registers, which are at the same time the right operand of the products with S.
+template <int TPW, bool CH>
+__global__ __launch_bounds__(256) void delta_walk_kernel(const DeltaDims d, float* state, const int64_t s_elems, const StepRows r, const DeltaBuf b, const int32_t* chunk0)
+{
+  __shared__ f32x4 part[2][4][2][64];
+  const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), fr = lane & 15, fg = lane >> 4;
+  const int h = blockIdx.y, col = blockIdx.x * 16 + fr;
+  const int32_t* en = r.ent + 4 * blockIdx.z;
+  const int slot = en[0], row0 = en[1], n = en[2], pos0 = en[3], ch0 = chunk0[blockIdx.z];
+  const int g = h / (d.heads / d.kv_heads), kw = d.kv_heads * d.dim, vw = d.heads * d.vdim, gw = d.heads * d.dim, dvp = d.vdim_p();
+  float* Sg = state + slot * s_elems + (int64_t)h * d.dim * dvp;
+  const bool vec = (d.dim & 3) == 0;
+  f32x4 S[TPW];
+#pragma unroll
+  for (int j = 0; j < TPW; j++)
+#pragma unroll
+    for (int i = 0; i < 4; i++) {
+      const int c = (wave * TPW + j) * 16 + fg * 4 + i;
+      S[j][i] = pos0 > 0 && c < d.dim && col < d.vdim ? Sg[(int64_t)c * dvp + col] : 0.0f;
+    }
+  struct In { f32x4 w[TPW], q[TPW], k[TPW], tot[TPW], u0, qk; };
+  auto four = [&](const float* p, int c, bool ok) -> f32x4 {              // columns c .. c + 3 of a row of d.dim values
+    f32x4 x = {0.0f, 0.0f, 0.0f, 0.0f};
+    if (ok) {
+      if (vec) { if (c < d.dim) x = *reinterpret_cast<const f32x4*>(p + c); }
+      else {
+#pragma unroll
+        for (int i = 0; i < 4; i++) if (c + i < d.dim) x[i] = p[c + i];
+      }
+    }
+    return x;
+  };
+  auto fetch = [&](int t0, In& x) {
+    const int nt = min(CHUNK, n - t0);
+    const int64_t rr = row0 + t0, rt = rr + min(fr, nt - 1);
+    const bool rok = fr < nt;
+    float kz[4];
+    float p = 1.0f, tot = 1.0f;
+    if (!CH) {
+      p = b.gt[(rt * d.heads + h) * 2]; tot = b.gt[((rr + nt - 1) * d.heads + h) * 2];
+#pragma unroll
+      for (int i = 0; i < 4; i++) kz[i] = b.gt[((rr + min(fg * 4 + i, nt - 1)) * d.heads + h) * 2 + 1];
+    }
+#pragma unroll
+    for (int j = 0; j < TPW; j++) {
+      const int tile = (wave * TPW + j) * 16, c4 = tile + fg * 4, c1 = tile + fr;
+      x.w[j] = four(b.w + rt * gw + h * d.dim, c4, rok);
+      x.q[j] = CH ? four(b.qt + rt * gw + h * d.dim, c4, rok) : four(b.q + rt * kw + g * d.dim, c4, rok) * p;
+#pragma unroll
+      for (int i = 0; i < 4; i++) {
+        const int t = fg * 4 + i;
+        const bool ok = t < nt && c1 < d.dim;
+        const int64_t rw = rr + (ok ? t : 0); const int cc = ok ? c1 : 0;
+        const float k = CH ? b.g[rw * gw + h * d.dim + cc] : b.k[rw * kw + g * d.dim + cc] * kz[i];
+        x.k[j][i] = ok ? k : 0.0f;
+      }
+      x.tot[j] = CH ? four(b.gt + (int64_t)(ch0 + t0 / CHUNK) * gw + h * d.dim, c4, true) : f32x4{tot, tot, tot, tot};
+    }
+    x.u0 = f32x4{0.0f, 0.0f, 0.0f, 0.0f};
+    if (wave == 0) {
+#pragma unroll
+      for (int i = 0; i < 4; i++) if (fg * 4 + i < nt && col < d.vdim) x.u0[i] = b.v[(rr + fg * 4 + i) * vw + h * d.vdim + col];
+    }
+    x.qk = f32x4{0.0f, 0.0f, 0.0f, 0.0f};
+    if (wave == 3 && rok) x.qk = *reinterpret_cast<const f32x4*>(b.qk + (rt * d.heads + h) * CHUNK + fg * 4);
+  };
+  In cur;
+  fetch(0, cur);
+  for (int t0 = 0, it = 0; t0 < n; t0 += CHUNK, it ^= 1) {
+    In nxt;
+    if (t0 + CHUNK < n) fetch(t0 + CHUNK, nxt);
+    f32x4 u = cur.u0, o = {0.0f, 0.0f, 0.0f, 0.0f};
+#pragma unroll
+    for (int j = 0; j < TPW; j++)
+#pragma unroll
+      for (int i = 0; i < 4; i++) {
+        u = __builtin_amdgcn_mfma_f32_16x16x4f32(-cur.w[j][i], S[j][i], u, 0, 0, 0);
+        o = __builtin_amdgcn_mfma_f32_16x16x4f32(cur.q[j][i], S[j][i], o, 0, 0, 0);
+      }
+    part[it][wave][0][lane] = u; part[it][wave][1][lane] = o;
+    __syncthreads();
+    u = (part[it][0][0][lane] + part[it][1][0][lane]) + (part[it][2][0][lane] + part[it][3][0][lane]);
+#pragma unroll
+    for (int j = 0; j < TPW; j++) S[j] *= cur.tot[j];
+#pragma unroll
+    for (int i = 0; i < 4; i++)
+#pragma unroll
+      for (int j = 0; j < TPW; j++) S[j] = __builtin_amdgcn_mfma_f32_16x16x4f32(cur.k[j][i], u[i], S[j], 0, 0, 0);
+    if (wave == 3) {
+      o = (part[it][0][1][lane] + part[it][1][1][lane]) + (part[it][2][1][lane] + part[it][3][1][lane]);
+#pragma unroll
+      for (int i = 0; i < 4; i++) o = __builtin_amdgcn_mfma_f32_16x16x4f32(cur.qk[i], u[i], o, 0, 0, 0);
+#pragma unroll
+      for (int i = 0; i < 4; i++) if (t0 + fg * 4 + i < n && col < d.vdim) b.o[(int64_t)(row0 + t0 + fg * 4 + i) * vw + h * d.vdim + col] = o[i];
+    }
+    if (t0 + CHUNK < n) cur = nxt;
+  }
+#pragma unroll
+  for (int j = 0; j < TPW; j++)
+#pragma unroll
+    for (int i = 0; i < 4; i++) {
+      const int c = (wave * TPW + j) * 16 + fg * 4 + i;
+      if (c < d.dim && col < dvp) Sg[(int64_t)c * dvp + col] = S[j][i];
+    }
 }
 
 // ------------------------------------------------------------------------------------------
@@ -459,13 +720,13 @@ __global__ __launch_bounds__(1024) void delta_single_kernel(const DeltaDims d, c
   }
 }
 
-int delta_prep(const DeltaDims& d, const DeltaIn& in, const DeltaW& w, const SeqPool::DeltaRun& st, const StepRows& r, const DeltaBuf& b, bool log_decay)
+int delta_prep(const DeltaDims& d, const DeltaIn& in, const DeltaW& w, const SeqPool::DeltaRun& st, const StepRows& r, const DeltaBuf& b)
 {
   const int gw = d.channel_decay ? d.heads * d.dim : d.heads;
   const int units = d.kv_heads + (d.heads * d.vdim + 255) / 256 + (gw + 255) / 256 + 1;
   const dim3 grid((r.n_rows + PREP_ROWS - 1) / PREP_ROWS, (units + 3) / 4);
-  if (d.taps == 4) hipLaunchKernelGGL(delta_prep_kernel<4>, grid, dim3(256), 0, ctx().stream, d, in, w, st.hist, st.h_elems, r, b, (int)log_decay);
-  else hipLaunchKernelGGL(delta_prep_kernel<0>, grid, dim3(256), 0, ctx().stream, d, in, w, st.hist, st.h_elems, r, b, (int)log_decay);
+  if (d.taps == 4) hipLaunchKernelGGL(delta_prep_kernel<4>, grid, dim3(256), 0, ctx().stream, d, in, w, st.hist, st.h_elems, r, b);
+  else hipLaunchKernelGGL(delta_prep_kernel<0>, grid, dim3(256), 0, ctx().stream, d, in, w, st.hist, st.h_elems, r, b);
   CAI_HIP(hipGetLastError());
   return CAI_OK;
 }
@@ -478,6 +739,21 @@ int delta_scan(const DeltaDims& d, const SeqPool::DeltaRun& st, const StepRows& 
                        else hipLaunchKernelGGL((delta_scan_kernel<RPL, false>), grid, blk, 0, s, d, st.S, st.s_elems, r, b); } while (0)
   if (d.dim <= 64) SCAN(4); else if (d.dim <= 128) SCAN(8); else SCAN(16);
 #undef SCAN
+  CAI_HIP(hipGetLastError());
+  return CAI_OK;
+}
+
+int delta_chunked(const DeltaDims& d, const SeqPool::DeltaRun& st, const StepRows& r, const DeltaBuf& b, const int32_t* chunks, int n_chunks, const int32_t* chunk0)
+{
+  auto s = ctx().stream;
+  const size_t lds = (size_t)(d.channel_decay ? 3 : 2) * CHUNK * (((d.dim + 15) & ~15) + 4) * 4;
+  const dim3 g1(n_chunks, d.heads), g2((d.vdim + 15) / 16, d.heads, r.n_ent), blk(256);
+  if (d.channel_decay) hipLaunchKernelGGL(delta_chunk_kernel<true>, g1, blk, lds, s, d, r, b, chunks);
+  else hipLaunchKernelGGL(delta_chunk_kernel<false>, g1, blk, lds, s, d, r, b, chunks);
+#define WALK(N) do { if (d.channel_decay) hipLaunchKernelGGL((delta_walk_kernel<N, true>), g2, blk, 0, s, d, st.S, st.s_elems, r, b, chunk0); \
+                     else hipLaunchKernelGGL((delta_walk_kernel<N, false>), g2, blk, 0, s, d, st.S, st.s_elems, r, b, chunk0); } while (0)
+  if (d.dim <= 64) WALK(1); else if (d.dim <= 128) WALK(2); else WALK(4);
+#undef WALK
   CAI_HIP(hipGetLastError());
   return CAI_OK;
 }

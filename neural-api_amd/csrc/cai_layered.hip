@@ -222,7 +222,7 @@ struct LayeredNet {
   std::vector<NetRun> runs;
   // widths over all layers
   int wp = 0, ld_proj = 0, ld_mid = 0, ld_att = 0, ld_attl = 0, ld_q = 0, ld_ra = 0, ld_rg = 0;
-  int w_q = 0, w_k = 0, w_v = 0, w_g = 0, w_b = 0, w_za = 0, w_zg = 0;
+  int w_q = 0, w_k = 0, w_v = 0, w_g = 0, w_b = 0, w_za = 0, w_zg = 0, w_hd = 0, w_qt = 0, w_qk = 0, w_gt1 = 0;
   bool has_attn = false, looped = false;
   int cap = 0, logit_cap = 0, best_cap = 0;
   float *x = nullptr, *x0 = nullptr, *proj = nullptr, *yl = nullptr, *yr = nullptr, *part = nullptr, *logits = nullptr;
@@ -254,7 +254,7 @@ static void drop_graphs(LayeredNet* n)
 
 static void free_rows(LayeredNet* n)
 {
-  void* p[] = {n->x, n->x0, n->proj, n->yl, n->yr, n->part, n->h, n->mid, n->att, n->attl, n->qbuf, n->ra, n->rgb, n->db.q, n->db.k, n->db.v, n->db.g, n->db.beta, n->db.o, n->db.za, n->db.zg};
+  void* p[] = {n->x, n->x0, n->proj, n->yl, n->yr, n->part, n->h, n->mid, n->att, n->attl, n->qbuf, n->ra, n->rgb, n->db.q, n->db.k, n->db.v, n->db.g, n->db.beta, n->db.o, n->db.za, n->db.zg, n->db.w, n->db.qt, n->db.qk, n->db.gt};
   for (void* q : p) if (q) (void)hipFree(q);
   n->x = n->x0 = n->proj = n->yl = n->yr = n->part = nullptr;
   n->h = n->mid = n->att = n->attl = n->qbuf = n->ra = n->rgb = nullptr;
@@ -285,7 +285,9 @@ static int ensure_rows(LayeredNet* n, int rows)
       (rc = get(&n->attl, R * n->ld_attl * n->es)) || (rc = get(&n->qbuf, R * n->ld_q * n->es)) || (rc = get(&n->ra, R * n->ld_ra * n->es)) || (rc = get(&n->rgb, R * n->ld_rg * n->es)) ||
       (rc = get((void**)&n->db.q, R * n->w_q * 4)) || (rc = get((void**)&n->db.k, R * n->w_k * 4)) || (rc = get((void**)&n->db.v, R * n->w_v * 4)) ||
       (rc = get((void**)&n->db.g, R * n->w_g * 4)) || (rc = get((void**)&n->db.beta, R * n->w_b * 4)) || (rc = get((void**)&n->db.o, R * n->w_v * 4)) ||
-      (rc = get((void**)&n->db.za, R * n->w_za * 4)) || (rc = get((void**)&n->db.zg, R * n->w_zg * 4))) return rc;
+      (rc = get((void**)&n->db.za, R * n->w_za * 4)) || (rc = get((void**)&n->db.zg, R * n->w_zg * 4)) ||
+      (rc = get((void**)&n->db.w, R * n->w_hd * 4)) || (rc = get((void**)&n->db.qt, R * n->w_qt * 4)) || (rc = get((void**)&n->db.qk, R * n->w_qk * 4)) ||
+      (rc = get((void**)&n->db.gt, std::max(R * n->w_gt1, (R / DELTA_CHUNK + n->max_seq + 1) * n->w_qt) * 4))) return rc;
   CAI_HIP(hipStreamSynchronize(ctx().stream));
   n->cap = (int)R;
   return CAI_OK;
@@ -337,6 +339,8 @@ int net_create(NetSpec&& spec, int max_tokens, int max_seq, int act_t, LayeredNe
     up(n->ld_att, pad_to(d.heads * d.vdim, LIN_PAD));
     up(n->w_q, d.kv_heads * d.dim); up(n->w_k, d.kv_heads * d.dim); up(n->w_v, d.heads * d.vdim);
     up(n->w_g, d.channel_decay ? d.heads * d.dim : d.heads); up(n->w_b, d.heads + d.kv_heads);
+    up(n->w_hd, d.heads * d.dim); up(n->w_qk, d.heads * DELTA_CHUNK);
+    if (d.channel_decay) up(n->w_qt, d.heads * d.dim); else up(n->w_gt1, 2 * d.heads);
     if (d.rank_a) { up(n->ld_ra, pad_to(d.rank_a, LIN_PAD)); up(n->w_za, d.channel_decay ? d.heads * d.dim : d.heads); }
     if (d.rank_g) { up(n->ld_rg, pad_to(d.rank_g, LIN_PAD)); up(n->w_zg, d.heads * d.vdim); }
     if (y.gateup) up(n->ld_mid, pad_to(y.ff, LIN_PAD));
@@ -375,9 +379,12 @@ void net_destroy(LayeredNet* n)
   delete n;
 }
 
+// Work lists of a step with prompt portions (device pointers; null: the forms for short portions are taken)
+struct StepLists { const int32_t* tiles = nullptr; int n_tiles = 0; const int32_t* chunks = nullptr; int n_chunks = 0; const int32_t* chunk0 = nullptr; };
+
 // One step over the rows of `r`.  single: every entry is one row (the decode kernels).  want: device list of the rows whose
 // logits are produced (null: all rows, in order).
-static int enqueue_net(LayeredNet* n, const StepRows& r, bool single, const int32_t* tiles, int n_tiles, const int32_t* want, int n_want)
+static int enqueue_net(LayeredNet* n, const StepRows& r, bool single, const StepLists& lists, const int32_t* want, int n_want)
 {
   const NetSpec& s = n->s;
   const int R = r.n_rows, w = s.width, at = n->act_t;
@@ -409,7 +416,9 @@ static int enqueue_net(LayeredNet* n, const StepRows& r, bool single, const int3
         LinEpi e; e.y = n->db.zg; e.ldy = D.w.g2->rows;
         if ((rc = launch_pack_rows(n->proj, n->ld_proj, D.og, D.d.rank_g, R, at, n->rgb, n->ld_rg)) || (rc = launch_lin(D.w.g2, at, n->rgb, n->ld_rg, R, e))) return rc;
       }
-      if ((rc = delta_prep(D.d, din, D.w, ds, r, n->db, false)) || (rc = delta_scan(D.d, ds, r, n->db)) || (rc = delta_finish(D.d, din, D.w, ds, r, n->db, at, n->att, n->ld_att))) return rc;
+      if ((rc = delta_prep(D.d, din, D.w, ds, r, n->db)) ||
+          (rc = lists.chunks ? delta_chunked(D.d, ds, r, n->db, lists.chunks, lists.n_chunks, lists.chunk0) : delta_scan(D.d, ds, r, n->db)) ||
+          (rc = delta_finish(D.d, din, D.w, ds, r, n->db, at, n->att, n->ld_att))) return rc;
     }
     LinEpi res; res.mode = EPI_RESIDUAL; res.y = n->x; res.ldy = w; res.h = n->h; res.ldh = n->wp; res.post = y.norm1b;
     if (y.gateup) res.next = y.norm2;
@@ -419,7 +428,7 @@ static int enqueue_net(LayeredNet* n, const StepRows& r, bool single, const int3
       const AttnIn ain{n->proj, n->ld_proj, A.oq, A.ok, A.ov, A.qn, A.kn};
       const KvView kv = n->pool.view(run.attn_run);
       if (!single && (rc = attn_paged_prep(A.d, kv, at, ain, r, n->qbuf))) return rc;
-      if (!single && tiles && attn_paged_prompt_ok(A.d, at)) rc = attn_paged_prompt(A.d, kv, n->qbuf, r, tiles, n_tiles, n->attl, n->ld_attl);
+      if (!single && lists.tiles && attn_paged_prompt_ok(A.d, at)) rc = attn_paged_prompt(A.d, kv, n->qbuf, r, lists.tiles, lists.n_tiles, n->attl, n->ld_attl);
       else rc = attn_paged_rows(A.d, kv, at, n->qbuf, r, n->attl, n->ld_attl, n->part, single, ain);
       if (rc) return rc;
       LinEpi el, er; el.y = n->yl; er.y = n->yr; el.ldy = er.ldy = w;
@@ -462,7 +471,7 @@ static int run_captured(LayeredNet* n, int R, int steps, bool gen)
   const StepRows r = dec_rows(n, R);
   auto body = [&]() -> int {
     for (int i = 0; i < steps; i++) {
-      const int rc = enqueue_net(n, r, true, nullptr, 0, nullptr, R);
+      const int rc = enqueue_net(n, r, true, StepLists(), nullptr, R);
       if (rc) return rc;
       if (gen) hipLaunchKernelGGL(net_advance_kernel, dim3(1), dim3(64), 0, st, n->d_dec, n->d_dec + DEC_ROWS, n->best, n->d_gen, n->d_dec + 9 * DEC_ROWS);
     }
@@ -525,10 +534,15 @@ int net_step(LayeredNet* n, int n_ent, const int32_t* seq, const int32_t* count,
     n->row_of = wrows; n->rows_gathered = false;
   } else {
     // rows, entries, tiles of the prompt attention kernel, wanted rows
-    std::vector<int32_t> tiles;
-    bool tall = false;
-    for (int e = 0; e < n_ent; e++) { tall = tall || count[e] >= 16; for (int t = 0; t < count[e]; t += ATTN_TILE) { tiles.push_back(e); tiles.push_back(t); } }
-    const size_t need = (size_t)5 * R + 4 * n_ent + tiles.size() + W;
+    std::vector<int32_t> tiles, chunks, chunk0;
+    bool tall = false, chunked = false;
+    for (int e = 0; e < n_ent; e++) {
+      tall = tall || count[e] >= 16; chunked = chunked || count[e] >= DELTA_CHUNK_MIN;
+      chunk0.push_back((int)chunks.size() / 2);
+      for (int t = 0; t < count[e]; t += ATTN_TILE) { tiles.push_back(e); tiles.push_back(t); }
+      for (int t = 0; t < count[e]; t += DELTA_CHUNK) { chunks.push_back(e); chunks.push_back(t); }
+    }
+    const size_t need = (size_t)5 * R + 4 * n_ent + tiles.size() + chunks.size() + chunk0.size() + W;
     if (n->rows_cap < need) {
       CAI_HIP(hipStreamSynchronize(st));
       if (n->d_rows) (void)hipFree(n->d_rows);
@@ -547,13 +561,18 @@ int net_step(LayeredNet* n, int n_ent, const int32_t* seq, const int32_t* count,
       for (int t = 0; t < count[e]; t++, i++) { hr[i] = tokens[i]; hr[R + i] = pos0 + t; hr[2 * R + i] = seq[e]; hr[3 * R + i] = r0; hr[4 * R + i] = r0 + count[e] - 1; }
     }
     int32_t* ht = ent + 4 * n_ent;
-    std::copy(tiles.begin(), tiles.end(), ht);
-    std::copy(wrows.begin(), wrows.end(), ht + tiles.size());
+    ht = std::copy(tiles.begin(), tiles.end(), ht);
+    ht = std::copy(chunks.begin(), chunks.end(), ht);
+    ht = std::copy(chunk0.begin(), chunk0.end(), ht);
+    std::copy(wrows.begin(), wrows.end(), ht);
     CAI_HIP(hipMemcpyAsync(n->d_rows, hr, need * sizeof(int32_t), hipMemcpyHostToDevice, st));
     const int32_t* d = n->d_rows;
     const StepRows r{d, d + R, d + 2 * R, d + 3 * R, d + 4 * R, d + 5 * R, R, n_ent};
-    const int32_t* dt = d + 5 * R + 4 * n_ent;
-    if ((rc = enqueue_net(n, r, false, tall ? dt : nullptr, (int)tiles.size() / 2, dt + tiles.size(), W))) return rc;
+    const int32_t* dt = d + 5 * R + 4 * n_ent, *dc = dt + tiles.size(), *dc0 = dc + chunks.size();
+    StepLists lists;
+    if (tall) { lists.tiles = dt; lists.n_tiles = (int)tiles.size() / 2; }
+    if (chunked) { lists.chunks = dc; lists.n_chunks = (int)chunks.size() / 2; lists.chunk0 = dc0; }
+    if ((rc = enqueue_net(n, r, false, lists, dc0 + chunk0.size(), W))) return rc;
     for (int k = 0; k < W; k++) n->row_of.push_back(k);
     n->rows_gathered = true;
   }

@@ -124,9 +124,15 @@ struct DeltaW {
   const float *dt_bias, *norm;             // [heads] or [heads * dim]; [vdim]
   const cai_qw_s *a2, *g2;                 // low-rank seconds (CAI_BF16), null when direct
 };
-struct DeltaBuf { float *q, *k, *v, *g, *beta, *o, *za, *zg; };   // per-row scratch of a prompt pass
-int delta_prep(const DeltaDims& d, const DeltaIn& in, const DeltaW& w, const SeqPool::DeltaRun& st, const StepRows& r, const DeltaBuf& b, bool log_decay);
+struct DeltaBuf {                          // per-row scratch of a prompt pass
+  float *q, *k, *v, *g, *beta, *o, *za, *zg;
+  float *w, *qt, *qk, *gt;                 // chunked form: T [P k], P q, q D k, and the products of decays
+};
+constexpr int DELTA_CHUNK = 16;            // tokens per chunk
+constexpr int DELTA_CHUNK_MIN = 32;        // portions from here on make a step take the chunked form
+int delta_prep(const DeltaDims& d, const DeltaIn& in, const DeltaW& w, const SeqPool::DeltaRun& st, const StepRows& r, const DeltaBuf& b);
 int delta_scan(const DeltaDims& d, const SeqPool::DeltaRun& st, const StepRows& r, const DeltaBuf& b);
+int delta_chunked(const DeltaDims& d, const SeqPool::DeltaRun& st, const StepRows& r, const DeltaBuf& b, const int32_t* chunks, int n_chunks, const int32_t* chunk0);   // chunks: entry, first row in it; chunk0: first chunk of each entry
 int delta_finish(const DeltaDims& d, const DeltaIn& in, const DeltaW& w, const SeqPool::DeltaRun& st, const StepRows& r, const DeltaBuf& b, int act_t, void* out, int64_t ldo);
 int delta_single(const DeltaDims& d, const DeltaIn& in, const DeltaW& w, const SeqPool::DeltaRun& st, const StepRows& r, int act_t, void* out, int64_t ldo);
 
