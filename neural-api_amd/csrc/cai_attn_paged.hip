@@ -281,9 +281,18 @@ __global__ __launch_bounds__(256) void attn_prompt_paged_kernel(const AttnDims d
   __shared__ __align__(16) uint16_t sk[PAGE_TOKENS * KST];
   __shared__ __align__(16) uint16_t sv[VQ * 16 * VST];
   const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), fr = lane & 15, fg = lane >> 4;
-  const int32_t* en = r.ent + 4 * tiles[2 * blockIdx.x];
-  const int slot = en[0], row0 = en[1], n = en[2], pos0 = en[3], t0 = tiles[2 * blockIdx.x + 1];
-  const int h = blockIdx.y, g = h / (d.heads / d.kv_heads);
+  // with key/value heads in whole eights, everything that reads one of them runs on one XCD (consecutive work-groups go to
+  // different ones), heads of a group and neighbouring tiles next to each other
+  const int hg = d.heads / d.kv_heads;
+  int tile = blockIdx.x, h = blockIdx.y;
+  if (d.kv_heads % 8 == 0) {
+    const int id = blockIdx.x + gridDim.x * blockIdx.y, j = id >> 3;
+    h = ((id & 7) + 8 * (j / (hg * (int)gridDim.x))) * hg + j % hg;
+    tile = j / hg % gridDim.x;
+  }
+  const int32_t* en = r.ent + 4 * tiles[2 * tile];
+  const int slot = en[0], row0 = en[1], n = en[2], pos0 = en[3], t0 = tiles[2 * tile + 1];
+  const int g = h / hg;
   const int qi = t0 + wave * 16 + fr, qr = min(qi, n - 1), qpos = pos0 + qr;
   u32x4 fq[KQ];
 #pragma unroll
@@ -302,22 +311,23 @@ __global__ __launch_bounds__(256) void attn_prompt_paged_kernel(const AttnDims d
   const float scale2 = d.scale * 1.44269504088896340736f;             // scores in base-2 logarithms
   constexpr int KC = PAGE_TOKENS * KQ * 4 / 256, VC = PAGE_TOKENS / 2 * VQ * 2 / 256;   // 16-byte key chunks / value chunk pairs per thread
   u32x4 rk[KC], rv[VC][2];
+  // value chunks: eight lanes along pairs of keys, then along the columns, so that the transposing LDS writes spread over the banks
+  auto vtok = [](int e) { return ((e & 7) + (e / (VQ * 2 * 8)) * 8) * 2; };
+  auto vcol = [](int e) { return (e >> 3) % (VQ * 2) * 8; };
+  int page_no = kv.table[slot * kv.ring + first % kv.ring];
   auto fetch = [&](int pg) {
-    const bf16_t* page = kv_page<bf16_t>(kv, slot, pg * PAGE_TOKENS);
+    const bf16_t* page = reinterpret_cast<const bf16_t*>(kv.base) + (int64_t)page_no * kv.page_elems;
+    page_no = kv.table[slot * kv.ring + min(pg + 1, last) % kv.ring];      // (the next page's number, a page ahead)
 #pragma unroll
     for (int i = 0; i < KC; i++) {
       const int e = tid + 256 * i, t = e / (KQ * 4), c = e % (KQ * 4) * 8;
-      rk[i] = u32x4{0, 0, 0, 0};
-      if (c < d.dim_p) rk[i] = *reinterpret_cast<const u32x4*>(page + ((int64_t)g * PAGE_TOKENS + t) * d.dim_p + c);
+      rk[i] = *reinterpret_cast<const u32x4*>(page + (unsigned)((g * PAGE_TOKENS + t) * d.dim_p + (c < d.dim_p ? c : 0)));
     }
 #pragma unroll
     for (int i = 0; i < VC; i++) {
-      const int e = tid + 256 * i, t = e / (VQ * 2) * 2, c = e % (VQ * 2) * 8;
-      rv[i][0] = rv[i][1] = u32x4{0, 0, 0, 0};
-      if (c < d.vdim_p) {
-        const bf16_t* vp = page + kv.v_off + ((int64_t)g * PAGE_TOKENS + t) * d.vdim_p + c;
-        rv[i][0] = *reinterpret_cast<const u32x4*>(vp); rv[i][1] = *reinterpret_cast<const u32x4*>(vp + d.vdim_p);
-      }
+      const int t = vtok(tid + 256 * i), c = vcol(tid + 256 * i);
+      const bf16_t* vp = page + kv.v_off + (unsigned)((g * PAGE_TOKENS + t) * d.vdim_p + (c < d.vdim_p ? c : 0));
+      rv[i][0] = *reinterpret_cast<const u32x4*>(vp); rv[i][1] = *reinterpret_cast<const u32x4*>(vp + d.vdim_p);
     }
   };
   const int end = pos0 + n;                // keys at and past it are not written yet: their page rows may hold anything
@@ -327,12 +337,12 @@ __global__ __launch_bounds__(256) void attn_prompt_paged_kernel(const AttnDims d
 #pragma unroll
     for (int i = 0; i < KC; i++) {
       const int e = tid + 256 * i, t = e / (KQ * 4), c = e % (KQ * 4) * 8;
-      *reinterpret_cast<u32x4*>(sk + t * KST + c) = rk[i];
+      *reinterpret_cast<u32x4*>(sk + t * KST + c) = c < d.dim_p ? rk[i] : u32x4{0, 0, 0, 0};
     }
 #pragma unroll
     for (int i = 0; i < VC; i++) {
-      const int e = tid + 256 * i, t = e / (VQ * 2) * 2, c = e % (VQ * 2) * 8;
-      const bool k0 = pg * PAGE_TOKENS + t < end, k1 = pg * PAGE_TOKENS + t + 1 < end;
+      const int t = vtok(tid + 256 * i), c = vcol(tid + 256 * i);
+      const bool k0 = c < d.vdim_p && pg * PAGE_TOKENS + t < end, k1 = c < d.vdim_p && pg * PAGE_TOKENS + t + 1 < end;
 #pragma unroll
       for (int j = 0; j < 4; j++) {
         const uint32_t a = k0 ? rv[i][0][j] : 0, b = k1 ? rv[i][1][j] : 0;

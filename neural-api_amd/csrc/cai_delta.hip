@@ -433,17 +433,20 @@ __global__ __launch_bounds__(256) void delta_chunk_kernel(const DeltaDims d, con
 
 // The walk: one work-group per (16 value columns, head, entry); wave w holds key rows of tiles w TPW .. as matrix-core result
 // registers, which are at the same time the right operand of the products with S.
-template <int TPW, bool CH>
-__global__ __launch_bounds__(256) void delta_walk_kernel(const DeltaDims d, float* state, const int64_t s_elems, const StepRows r, const DeltaBuf b, const int32_t* chunk0)
+template <int NW, int TPW, bool CH, bool VEC>      // VEC: the key width is a multiple of four
+__global__ __launch_bounds__(64 * NW) void delta_walk_kernel(const DeltaDims d, float* state, const int64_t s_elems, const StepRows r, const DeltaBuf b, const int32_t* chunk0)
 {
-  __shared__ f32x4 part[2][4][2][64];
+  __shared__ f32x4 part[3][NW][2][64];
   const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), fr = lane & 15, fg = lane >> 4;
-  const int h = blockIdx.y, col = blockIdx.x * 16 + fr;
-  const int32_t* en = r.ent + 4 * blockIdx.z;
-  const int slot = en[0], row0 = en[1], n = en[2], pos0 = en[3], ch0 = chunk0[blockIdx.z];
+  // consecutive work-groups go to different XCDs; the column slices of a head read the same chunk data, so with heads in whole
+  // eights every head stays on one XCD (and in its L2)
+  const int slices = (d.vdim + 15) / 16;
+  const int h = d.heads % 8 == 0 ? (blockIdx.x & 7) + 8 * ((blockIdx.x >> 3) / slices) : blockIdx.x / slices;
+  const int col = (d.heads % 8 == 0 ? (blockIdx.x >> 3) % slices : blockIdx.x % slices) * 16 + fr;
+  const int32_t* en = r.ent + 4 * blockIdx.y;
+  const int slot = en[0], row0 = en[1], n = en[2], pos0 = en[3], ch0 = chunk0[blockIdx.y];
   const int g = h / (d.heads / d.kv_heads), kw = d.kv_heads * d.dim, vw = d.heads * d.vdim, gw = d.heads * d.dim, dvp = d.vdim_p();
   float* Sg = state + slot * s_elems + (int64_t)h * d.dim * dvp;
-  const bool vec = (d.dim & 3) == 0;
   f32x4 S[TPW];
 #pragma unroll
   for (int j = 0; j < TPW; j++)
@@ -452,82 +455,117 @@ __global__ __launch_bounds__(256) void delta_walk_kernel(const DeltaDims d, floa
       const int c = (wave * TPW + j) * 16 + fg * 4 + i;
       S[j][i] = pos0 > 0 && c < d.dim && col < d.vdim ? Sg[(int64_t)c * dvp + col] : 0.0f;
     }
-  struct In { f32x4 w[TPW], q[TPW], k[TPW], tot[TPW], u0, qk; };
-  auto four = [&](const float* p, int c, bool ok) -> f32x4 {              // columns c .. c + 3 of a row of d.dim values
-    f32x4 x = {0.0f, 0.0f, 0.0f, 0.0f};
-    if (ok) {
-      if (vec) { if (c < d.dim) x = *reinterpret_cast<const f32x4*>(p + c); }
-      else {
+  // A chunk's inputs are requested two chunks ahead and stay as they come until they are used: arithmetic on them here would wait
+  // for them here, and so would a request under a branch where the paths join.  A request is a scalar base of the chunk plus a lane
+  // offset that never changes; rows past the portion's end (of another entry, or of the slack behind the last row) and columns past
+  // the width are replaced by zeros at use.
+  struct In { f32x4 w[TPW], q[TPW], k[TPW], tot[TPW], u0, qk; float p, all, kz[4]; };
+  bool ok4[TPW][VEC ? 1 : 4], ok1[TPW];
+  unsigned lw[TPW], lq[TPW], lk[TPW], lt[TPW];
 #pragma unroll
-        for (int i = 0; i < 4; i++) if (c + i < d.dim) x[i] = p[c + i];
-      }
-    }
-    return x;
+  for (int j = 0; j < TPW; j++) {
+    const int c4 = (wave * TPW + j) * 16 + fg * 4, c1 = (wave * TPW + j) * 16 + fr;
+    ok1[j] = c1 < d.dim;
+#pragma unroll
+    for (int i = 0; i < (VEC ? 1 : 4); i++) ok4[j][i] = c4 + i < d.dim;
+    lt[j] = c4 < d.dim ? c4 : 0;
+    lw[j] = fr * gw + lt[j]; lq[j] = fr * (CH ? gw : kw) + lt[j];
+    lk[j] = fg * 4 * (CH ? gw : kw) + (ok1[j] ? c1 : 0);
+  }
+  const unsigned lv = fg * 4 * vw + min(col, d.vdim - 1), lqk = fr * d.heads * CHUNK + fg * 4, lp = fr * d.heads * 2, lz = fg * 4 * d.heads * 2 + 1;
+  auto four = [&](const float* p, unsigned c) -> f32x4 {
+    if (VEC) return *reinterpret_cast<const f32x4*>(p + c);
+    return f32x4{p[c], p[c + 1], p[c + 2], p[c + 3]};                     // (may run into the next row: replaced at use)
   };
-  auto fetch = [&](int t0, In& x) {
-    const int nt = min(CHUNK, n - t0);
-    const int64_t rr = row0 + t0, rt = rr + min(fr, nt - 1);
-    const bool rok = fr < nt;
-    float kz[4];
-    float p = 1.0f, tot = 1.0f;
-    if (!CH) {
-      p = b.gt[(rt * d.heads + h) * 2]; tot = b.gt[((rr + nt - 1) * d.heads + h) * 2];
-#pragma unroll
-      for (int i = 0; i < 4; i++) kz[i] = b.gt[((rr + min(fg * 4 + i, nt - 1)) * d.heads + h) * 2 + 1];
-    }
+  const int nc = (n + CHUNK - 1) / CHUNK;
+  auto fetch = [&](int c, In& x) {
+    const int cc = min(c, nc - 1);
+    const int64_t rr = row0 + cc * CHUNK;
+    const float *wb = b.w + rr * gw + h * d.dim, *qb = CH ? b.qt + rr * gw + h * d.dim : b.q + rr * kw + g * d.dim;
+    const float *kb = CH ? b.g + rr * gw + h * d.dim : b.k + rr * kw + g * d.dim, *tb = b.gt + (int64_t)(ch0 + cc) * gw + h * d.dim;
+    const int ks = CH ? gw : kw;
 #pragma unroll
     for (int j = 0; j < TPW; j++) {
-      const int tile = (wave * TPW + j) * 16, c4 = tile + fg * 4, c1 = tile + fr;
-      x.w[j] = four(b.w + rt * gw + h * d.dim, c4, rok);
-      x.q[j] = CH ? four(b.qt + rt * gw + h * d.dim, c4, rok) : four(b.q + rt * kw + g * d.dim, c4, rok) * p;
+      x.w[j] = four(wb, lw[j]); x.q[j] = four(qb, lq[j]);
 #pragma unroll
-      for (int i = 0; i < 4; i++) {
-        const int t = fg * 4 + i;
-        const bool ok = t < nt && c1 < d.dim;
-        const int64_t rw = rr + (ok ? t : 0); const int cc = ok ? c1 : 0;
-        const float k = CH ? b.g[rw * gw + h * d.dim + cc] : b.k[rw * kw + g * d.dim + cc] * kz[i];
-        x.k[j][i] = ok ? k : 0.0f;
-      }
-      x.tot[j] = CH ? four(b.gt + (int64_t)(ch0 + t0 / CHUNK) * gw + h * d.dim, c4, true) : f32x4{tot, tot, tot, tot};
+      for (int i = 0; i < 4; i++) x.k[j][i] = (kb + i * ks)[lk[j]];
+      if (CH) x.tot[j] = four(tb, lt[j]);
     }
-    x.u0 = f32x4{0.0f, 0.0f, 0.0f, 0.0f};
-    if (wave == 0) {
+    if (!CH) {
+      const float* pz = b.gt + (rr * d.heads + h) * 2;
+      x.p = pz[lp]; x.all = pz[(min(CHUNK, n - cc * CHUNK) - 1) * d.heads * 2];
 #pragma unroll
-      for (int i = 0; i < 4; i++) if (fg * 4 + i < nt && col < d.vdim) x.u0[i] = b.v[(rr + fg * 4 + i) * vw + h * d.vdim + col];
+      for (int i = 0; i < 4; i++) x.kz[i] = (pz + i * d.heads * 2)[lz];
     }
-    x.qk = f32x4{0.0f, 0.0f, 0.0f, 0.0f};
-    if (wave == 3 && rok) x.qk = *reinterpret_cast<const f32x4*>(b.qk + (rt * d.heads + h) * CHUNK + fg * 4);
+    const float* vb = b.v + rr * vw + h * d.vdim;
+#pragma unroll
+    for (int i = 0; i < 4; i++) x.u0[i] = (vb + i * vw)[lv];
+    x.qk = *reinterpret_cast<const f32x4*>(b.qk + (rr * d.heads + h) * CHUNK + lqk);
   };
-  In cur;
-  fetch(0, cur);
-  for (int t0 = 0, it = 0; t0 < n; t0 += CHUNK, it ^= 1) {
-    In nxt;
-    if (t0 + CHUNK < n) fetch(t0 + CHUNK, nxt);
-    f32x4 u = cur.u0, o = {0.0f, 0.0f, 0.0f, 0.0f};
+  auto total = [&](int it, int k) -> f32x4 {
+    f32x4 x[NW];
+#pragma unroll
+    for (int v = 0; v < NW; v++) x[v] = part[it][v][k][lane];
+#pragma unroll
+    for (int m = NW / 2; m; m >>= 1)
+#pragma unroll
+      for (int v = 0; v < m; v++) x[v] += x[v + m];
+    return x[0];
+  };
+  auto chunk = [&](int c, const In& x, int it) {         // (a chunk past the last one changes nothing)
+    const int nt = min(CHUNK, n - c * CHUNK);
+    const bool rok = fr < nt;
+    bool tok[4];
+#pragma unroll
+    for (int i = 0; i < 4; i++) tok[i] = fg * 4 + i < nt;
+    f32x4 u, o = {0.0f, 0.0f, 0.0f, 0.0f};
+#pragma unroll
+    for (int i = 0; i < 4; i++) u[i] = wave == 0 && tok[i] && col < d.vdim ? x.u0[i] : 0.0f;
 #pragma unroll
     for (int j = 0; j < TPW; j++)
 #pragma unroll
       for (int i = 0; i < 4; i++) {
-        u = __builtin_amdgcn_mfma_f32_16x16x4f32(-cur.w[j][i], S[j][i], u, 0, 0, 0);
-        o = __builtin_amdgcn_mfma_f32_16x16x4f32(cur.q[j][i], S[j][i], o, 0, 0, 0);
+        const bool ok = rok && ok4[j][VEC ? 0 : i];
+        const float w = ok ? x.w[j][i] : 0.0f, q = ok ? (CH ? x.q[j][i] : x.q[j][i] * x.p) : 0.0f;
+        u = __builtin_amdgcn_mfma_f32_16x16x4f32(-w, S[j][i], u, 0, 0, 0);
+        o = __builtin_amdgcn_mfma_f32_16x16x4f32(q, S[j][i], o, 0, 0, 0);
       }
     part[it][wave][0][lane] = u; part[it][wave][1][lane] = o;
     __syncthreads();
-    u = (part[it][0][0][lane] + part[it][1][0][lane]) + (part[it][2][0][lane] + part[it][3][0][lane]);
+    u = total(it, 0);
 #pragma unroll
-    for (int j = 0; j < TPW; j++) S[j] *= cur.tot[j];
+    for (int j = 0; j < TPW; j++)
+#pragma unroll
+      for (int i = 0; i < 4; i++) S[j][i] *= nt > 0 ? (CH ? x.tot[j][i] : x.all) : 1.0f;
 #pragma unroll
     for (int i = 0; i < 4; i++)
 #pragma unroll
-      for (int j = 0; j < TPW; j++) S[j] = __builtin_amdgcn_mfma_f32_16x16x4f32(cur.k[j][i], u[i], S[j], 0, 0, 0);
-    if (wave == 3) {
-      o = (part[it][0][1][lane] + part[it][1][1][lane]) + (part[it][2][1][lane] + part[it][3][1][lane]);
+      for (int j = 0; j < TPW; j++) {
+        const float k = tok[i] && ok1[j] ? (CH ? x.k[j][i] : x.k[j][i] * x.kz[i]) : 0.0f;
+        S[j] = __builtin_amdgcn_mfma_f32_16x16x4f32(k, u[i], S[j], 0, 0, 0);
+      }
+    if (wave == NW - 1) {
+      o = total(it, 1);
 #pragma unroll
-      for (int i = 0; i < 4; i++) o = __builtin_amdgcn_mfma_f32_16x16x4f32(cur.qk[i], u[i], o, 0, 0, 0);
+      for (int i = 0; i < 4; i++) o = __builtin_amdgcn_mfma_f32_16x16x4f32(rok ? x.qk[i] : 0.0f, u[i], o, 0, 0, 0);
+      float* ob = b.o + (int64_t)(row0 + c * CHUNK) * vw + h * d.vdim;
 #pragma unroll
-      for (int i = 0; i < 4; i++) if (t0 + fg * 4 + i < n && col < d.vdim) b.o[(int64_t)(row0 + t0 + fg * 4 + i) * vw + h * d.vdim + col] = o[i];
+      for (int i = 0; i < 4; i++) if (tok[i] && col < d.vdim) (ob + i * vw)[fg * 4 * vw + col] = o[i];
     }
-    if (t0 + CHUNK < n) cur = nxt;
+  };
+  // (the scheduling barriers keep a chunk's requests in front of the chunk that is worked on: they are used two chunks later)
+  In xa, xb, xc;
+  fetch(0, xa); fetch(1, xb);
+  for (int c = 0; c < nc; c += 3) {
+    fetch(c + 2, xc);
+    __builtin_amdgcn_sched_barrier(0);
+    chunk(c, xa, 0);
+    fetch(c + 3, xa);
+    __builtin_amdgcn_sched_barrier(0);
+    chunk(c + 1, xb, 1);
+    fetch(c + 4, xb);
+    __builtin_amdgcn_sched_barrier(0);
+    chunk(c + 2, xc, 2);
   }
 #pragma unroll
   for (int j = 0; j < TPW; j++)
@@ -747,13 +785,15 @@ int delta_chunked(const DeltaDims& d, const SeqPool::DeltaRun& st, const StepRow
 {
   auto s = ctx().stream;
   const size_t lds = (size_t)(d.channel_decay ? 3 : 2) * CHUNK * (((d.dim + 15) & ~15) + 4) * 4;
-  const dim3 g1(n_chunks, d.heads), g2((d.vdim + 15) / 16, d.heads, r.n_ent), blk(256);
+  const dim3 g1(n_chunks, d.heads), g2((d.vdim + 15) / 16 * d.heads, r.n_ent), blk(256);
   if (d.channel_decay) hipLaunchKernelGGL(delta_chunk_kernel<true>, g1, blk, lds, s, d, r, b, chunks);
   else hipLaunchKernelGGL(delta_chunk_kernel<false>, g1, blk, lds, s, d, r, b, chunks);
-#define WALK(N) do { if (d.channel_decay) hipLaunchKernelGGL((delta_walk_kernel<N, true>), g2, blk, 0, s, d, st.S, st.s_elems, r, b, chunk0); \
-                     else hipLaunchKernelGGL((delta_walk_kernel<N, false>), g2, blk, 0, s, d, st.S, st.s_elems, r, b, chunk0); } while (0)
-  if (d.dim <= 64) WALK(1); else if (d.dim <= 128) WALK(2); else WALK(4);
+#define WALK_V(NW, N, CH) do { if (d.dim % 4 == 0) hipLaunchKernelGGL((delta_walk_kernel<NW, N, CH, true>), g2, dim3(64 * NW), 0, s, d, st.S, st.s_elems, r, b, chunk0); \
+                               else hipLaunchKernelGGL((delta_walk_kernel<NW, N, CH, false>), g2, dim3(64 * NW), 0, s, d, st.S, st.s_elems, r, b, chunk0); } while (0)
+#define WALK(NW, N) do { if (d.channel_decay) WALK_V(NW, N, true); else WALK_V(NW, N, false); } while (0)
+  if (d.dim <= 64) WALK(4, 1); else if (d.dim <= 128) WALK(8, 1); else WALK(8, 2);
 #undef WALK
+#undef WALK_V
   CAI_HIP(hipGetLastError());
   return CAI_OK;
 }

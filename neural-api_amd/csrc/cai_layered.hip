@@ -164,13 +164,15 @@ __global__ __launch_bounds__(1024) void net_join_kernel(const float* yl, const f
   const int tid = threadIdx.x;
   const float *a = yl + t * width, *b = yr + t * width;
   // up to four values a thread stay in registers; wider rows are read again
-  float av[4], bv[4], xv[4];
+  float av[4], bv[4], xv[4], glv[4], grv[4];
   float s = 0.0f, q = 0.0f;
 #pragma unroll
   for (int u = 0; u < 4; u++) {
     const int i = min(tid + u * 1024, width - 1);
     av[u] = a[i]; bv[u] = b[i]; xv[u] = x[t * width + i];
   }
+#pragma unroll
+  for (int u = 0; u < 4; u++) { const int i = min(tid + u * 1024, width - 1); glv[u] = gl[i]; grv[u] = gr[i]; }
 #pragma unroll
   for (int u = 0; u < 4; u++) if (tid + u * 1024 < width) { s = fmaf(av[u], av[u], s); q = fmaf(bv[u], bv[u], q); }
   for (int i = tid + 4096; i < width; i += 1024) { s = fmaf(a[i], a[i], s); q = fmaf(b[i], b[i], q); }
@@ -181,15 +183,15 @@ __global__ __launch_bounds__(1024) void net_join_kernel(const float* yl, const f
 #pragma unroll
   for (int u = 0; u < 16; u++) { s += sl[u]; q += sr[u]; }
   const float il = 1.0f / sqrtf(s / (float)width + eps), ir = 1.0f / sqrtf(q / (float)width + eps);
-  auto put = [&](int i, float va, float vb, float vx) {
-    float v = vx + dyt(post, 0.5f * (va * il * gl[i] + vb * ir * gr[i]), i);
+  auto put = [&](int i, float va, float vb, float vx, float ga, float gb) {
+    float v = vx + dyt(post, 0.5f * (va * il * ga + vb * ir * gb), i);
     if (add0) v += add0[t * width + i];
     x[t * width + i] = v;
     h[t * ldh + i] = (AT)dyt(next, v, i);
   };
 #pragma unroll
-  for (int u = 0; u < 4; u++) if (tid + u * 1024 < width) put(tid + u * 1024, av[u], bv[u], xv[u]);
-  for (int i = tid + 4096; i < width; i += 1024) put(i, a[i], b[i], x[t * width + i]);
+  for (int u = 0; u < 4; u++) if (tid + u * 1024 < width) put(tid + u * 1024, av[u], bv[u], xv[u], glv[u], grv[u]);
+  for (int i = tid + 4096; i < width; i += 1024) put(i, a[i], b[i], x[t * width + i], gl[i], gr[i]);
 }
 
 template <typename AT>
@@ -276,6 +278,7 @@ static int ensure_rows(LayeredNet* n, int rows)
     CAI_HIP(hipMemsetAsync(*p, 0, bytes, ctx().stream));
     return CAI_OK;
   };
+  const size_t RS = R + DELTA_CHUNK + 1;    // the chunked walk requests whole chunks: up to 15 rows (and three values) past the last one
   size_t part = 0;
   for (auto& a : n->pool.attn) part = std::max(part, attn_paged_part_floats(a.d, (int)R));
   int rc;
@@ -283,11 +286,11 @@ static int ensure_rows(LayeredNet* n, int rows)
       (rc = get((void**)&n->yl, n->has_attn ? R * w * 4 : 0)) || (rc = get((void**)&n->yr, n->has_attn ? R * w * 4 : 0)) || (rc = get((void**)&n->part, part * 4)) ||
       (rc = get(&n->h, R * n->wp * n->es)) || (rc = get(&n->mid, R * n->ld_mid * n->es)) || (rc = get(&n->att, R * n->ld_att * n->es)) ||
       (rc = get(&n->attl, R * n->ld_attl * n->es)) || (rc = get(&n->qbuf, R * n->ld_q * n->es)) || (rc = get(&n->ra, R * n->ld_ra * n->es)) || (rc = get(&n->rgb, R * n->ld_rg * n->es)) ||
-      (rc = get((void**)&n->db.q, R * n->w_q * 4)) || (rc = get((void**)&n->db.k, R * n->w_k * 4)) || (rc = get((void**)&n->db.v, R * n->w_v * 4)) ||
-      (rc = get((void**)&n->db.g, R * n->w_g * 4)) || (rc = get((void**)&n->db.beta, R * n->w_b * 4)) || (rc = get((void**)&n->db.o, R * n->w_v * 4)) ||
+      (rc = get((void**)&n->db.q, RS * n->w_q * 4)) || (rc = get((void**)&n->db.k, RS * n->w_k * 4)) || (rc = get((void**)&n->db.v, RS * n->w_v * 4)) ||
+      (rc = get((void**)&n->db.g, RS * n->w_g * 4)) || (rc = get((void**)&n->db.beta, RS * n->w_b * 4)) || (rc = get((void**)&n->db.o, RS * n->w_v * 4)) ||
       (rc = get((void**)&n->db.za, R * n->w_za * 4)) || (rc = get((void**)&n->db.zg, R * n->w_zg * 4)) ||
-      (rc = get((void**)&n->db.w, R * n->w_hd * 4)) || (rc = get((void**)&n->db.qt, R * n->w_qt * 4)) || (rc = get((void**)&n->db.qk, R * n->w_qk * 4)) ||
-      (rc = get((void**)&n->db.gt, std::max(R * n->w_gt1, (R / DELTA_CHUNK + n->max_seq + 1) * n->w_qt) * 4))) return rc;
+      (rc = get((void**)&n->db.w, RS * n->w_hd * 4)) || (rc = get((void**)&n->db.qt, RS * n->w_qt * 4)) || (rc = get((void**)&n->db.qk, RS * n->w_qk * 4)) ||
+      (rc = get((void**)&n->db.gt, std::max(RS * n->w_gt1, (R / DELTA_CHUNK + n->max_seq + 1) * n->w_qt + 4) * 4))) return rc;
   CAI_HIP(hipStreamSynchronize(ctx().stream));
   n->cap = (int)R;
   return CAI_OK;

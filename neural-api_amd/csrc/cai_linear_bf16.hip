@@ -40,12 +40,12 @@ template <typename AT> __device__ __forceinline__ void epi_one(const LinEpi& e, 
 // 512-wide turn of them; the activations are staged in LDS as float in panels, the weights stream past once.
 // ------------------------------------------------------------------------------------------
 constexpr int GV_WAVES = 8;
-constexpr int GV_LDS = 16384;              // floats of staged activations
+constexpr int GV_LDS = 16384;              // most floats of staged activations (a launch asks for what its width needs)
 
 template <typename AT, int NB, int R>
 __global__ __launch_bounds__(64 * GV_WAVES) void gemv_bf16(const uint16_t* __restrict__ W, const AT* __restrict__ x, int n_rows, int ldw, int64_t ldx, int ksplit, LinEpi e)
 {
-  __shared__ float xs[GV_LDS];
+  extern __shared__ float xs[];            // [NB][panel]
   __shared__ float part[GV_WAVES][R * NB];
   const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const int ks = wave % ksplit;
@@ -299,8 +299,9 @@ static void run_gemv(const cai_qw_s* w, const AT* x, int64_t ldx, const LinEpi& 
   while (ks < GV_WAVES && ks * 2 <= turns && groups * ks * 2 <= want * 2) ks *= 2;
   const int per = GV_WAVES / ks;
   const dim3 grid((groups + per - 1) / per), blk(64 * GV_WAVES);
-  if (four) hipLaunchKernelGGL((gemv_bf16<AT, NB, 4>), grid, blk, 0, ctx().stream, (const uint16_t*)w->data, x, rows, (int)w->ld, ldx, ks, e);
-  else hipLaunchKernelGGL((gemv_bf16<AT, NB, 2>), grid, blk, 0, ctx().stream, (const uint16_t*)w->data, x, rows, (int)w->ld, ldx, ks, e);
+  const size_t lds = (size_t)((NB - 1) * (GV_LDS / NB / 512 * 512) + std::min(GV_LDS / NB / 512 * 512, turns * 512)) * 4;
+  if (four) hipLaunchKernelGGL((gemv_bf16<AT, NB, 4>), grid, blk, lds, ctx().stream, (const uint16_t*)w->data, x, rows, (int)w->ld, ldx, ks, e);
+  else hipLaunchKernelGGL((gemv_bf16<AT, NB, 2>), grid, blk, lds, ctx().stream, (const uint16_t*)w->data, x, rows, (int)w->ld, ldx, ks, e);
 }
 
 template <typename AT>
