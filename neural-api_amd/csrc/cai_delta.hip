@@ -431,12 +431,14 @@ __global__ __launch_bounds__(256) void delta_chunk_kernel(const DeltaDims d, con
   }
 }
 
-// The walk: one work-group per (16 value columns, head, entry); wave w holds key rows of tiles w TPW .. as matrix-core result
-// registers, which are at the same time the right operand of the products with S.
+// The walk: one work-group per (16 value columns, head, entry).  Waves 0 .. NW - 1 hold the state - wave w the key rows of tiles
+// w TPW .. as matrix-core result registers, which are at the same time the right operand of the products with S - and wave NW makes
+// the output: it contributes U0 to the sum of a chunk's writes and finishes the previous chunk's rows of o while the others are a
+// chunk further.  One barrier a chunk; the partial sums live in LDS for three chunks.
 template <int NW, int TPW, bool CH, bool VEC>      // VEC: the key width is a multiple of four
-__global__ __launch_bounds__(64 * NW) void delta_walk_kernel(const DeltaDims d, float* state, const int64_t s_elems, const StepRows r, const DeltaBuf b, const int32_t* chunk0)
+__global__ __launch_bounds__(64 * (NW + 1)) void delta_walk_kernel(const DeltaDims d, float* state, const int64_t s_elems, const StepRows r, const DeltaBuf b, const int32_t* chunk0)
 {
-  __shared__ f32x4 part[3][NW][2][64];
+  __shared__ f32x4 pu[3][NW + 1][64], po[3][NW][64];
   const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), fr = lane & 15, fg = lane >> 4;
   // consecutive work-groups go to different XCDs; the column slices of a head read the same chunk data, so with heads in whole
   // eights every head stays on one XCD (and in its L2)
@@ -446,6 +448,64 @@ __global__ __launch_bounds__(64 * NW) void delta_walk_kernel(const DeltaDims d, 
   const int32_t* en = r.ent + 4 * blockIdx.y;
   const int slot = en[0], row0 = en[1], n = en[2], pos0 = en[3], ch0 = chunk0[blockIdx.y];
   const int g = h / (d.heads / d.kv_heads), kw = d.kv_heads * d.dim, vw = d.heads * d.vdim, gw = d.heads * d.dim, dvp = d.vdim_p();
+  const int nc = (n + CHUNK - 1) / CHUNK;
+  auto total = [&](int it) -> f32x4 {                    // a chunk's writes: U0 and every wave's part of - W S
+    f32x4 x[NW];
+#pragma unroll
+    for (int v = 0; v < NW; v++) x[v] = pu[it][v][lane];
+    x[0] += pu[it][NW][lane];
+#pragma unroll
+    for (int m = NW / 2; m; m >>= 1)
+#pragma unroll
+      for (int v = 0; v < m; v++) x[v] += x[v + m];
+    return x[0];
+  };
+  if (wave == NW) {
+    const unsigned lv = fg * 4 * vw + min(col, d.vdim - 1), lqk = fr * d.heads * CHUNK + fg * 4, lo = fg * 4 * vw + col;
+    struct Out { f32x4 u0, qk; };
+    auto fetch = [&](int c, Out& x) {
+      const int64_t rr = row0 + min(c, nc - 1) * CHUNK;
+      const float* vb = b.v + rr * vw + h * d.vdim;
+#pragma unroll
+      for (int i = 0; i < 4; i++) x.u0[i] = (vb + i * vw)[lv];
+      x.qk = *reinterpret_cast<const f32x4*>(b.qk + (rr * d.heads + h) * CHUNK + lqk);
+    };
+    f32x4 qk_last = {0.0f, 0.0f, 0.0f, 0.0f};
+    auto finish = [&](int c, int it) {                   // rows of o of chunk c (parts it)
+      f32x4 o = po[it][0][lane];
+#pragma unroll
+      for (int v = 1; v < NW; v++) o += po[it][v][lane];
+      const f32x4 u = total(it);
+#pragma unroll
+      for (int i = 0; i < 4; i++) o = __builtin_amdgcn_mfma_f32_16x16x4f32(qk_last[i], u[i], o, 0, 0, 0);
+      const int nt = n - c * CHUNK;
+      if (c < 0) return;
+      float* ob = b.o + (int64_t)(row0 + c * CHUNK) * vw + h * d.vdim;
+#pragma unroll
+      for (int i = 0; i < 4; i++) if (fg * 4 + i < nt && col < d.vdim) (ob + i * vw)[lo] = o[i];
+    };
+    auto chunk = [&](int c, const Out& x, int it) {
+      const int nt = n - c * CHUNK;
+      f32x4 u;
+#pragma unroll
+      for (int i = 0; i < 4; i++) u[i] = fg * 4 + i < nt && col < d.vdim ? x.u0[i] : 0.0f;
+      pu[it][NW][lane] = u;
+      __syncthreads();
+      finish(c - 1, (it + 2) % 3);
+#pragma unroll
+      for (int i = 0; i < 4; i++) qk_last[i] = fr < nt ? x.qk[i] : 0.0f;
+    };
+    Out xa, xb, xc;
+    fetch(0, xa); fetch(1, xb);
+    for (int c = 0; c < nc; c += 3) {
+      fetch(c + 2, xc); chunk(c, xa, 0);
+      fetch(c + 3, xa); chunk(c + 1, xb, 1);
+      fetch(c + 4, xb); chunk(c + 2, xc, 2);
+    }
+    __syncthreads();
+    finish((nc + 2) / 3 * 3 - 1, 2);
+    return;
+  }
   float* Sg = state + slot * s_elems + (int64_t)h * d.dim * dvp;
   f32x4 S[TPW];
 #pragma unroll
@@ -459,7 +519,7 @@ __global__ __launch_bounds__(64 * NW) void delta_walk_kernel(const DeltaDims d, 
   // for them here, and so would a request under a branch where the paths join.  A request is a scalar base of the chunk plus a lane
   // offset that never changes; rows past the portion's end (of another entry, or of the slack behind the last row) and columns past
   // the width are replaced by zeros at use.
-  struct In { f32x4 w[TPW], q[TPW], k[TPW], tot[TPW], u0, qk; float p, all, kz[4]; };
+  struct In { f32x4 w[TPW], q[TPW], k[TPW], tot[TPW]; float p, all, kz[4]; };
   bool ok4[TPW][VEC ? 1 : 4], ok1[TPW];
   unsigned lw[TPW], lq[TPW], lk[TPW], lt[TPW];
 #pragma unroll
@@ -472,12 +532,11 @@ __global__ __launch_bounds__(64 * NW) void delta_walk_kernel(const DeltaDims d, 
     lw[j] = fr * gw + lt[j]; lq[j] = fr * (CH ? gw : kw) + lt[j];
     lk[j] = fg * 4 * (CH ? gw : kw) + (ok1[j] ? c1 : 0);
   }
-  const unsigned lv = fg * 4 * vw + min(col, d.vdim - 1), lqk = fr * d.heads * CHUNK + fg * 4, lp = fr * d.heads * 2, lz = fg * 4 * d.heads * 2 + 1;
+  const unsigned lp = fr * d.heads * 2, lz = fg * 4 * d.heads * 2 + 1;
   auto four = [&](const float* p, unsigned c) -> f32x4 {
     if (VEC) return *reinterpret_cast<const f32x4*>(p + c);
     return f32x4{p[c], p[c + 1], p[c + 2], p[c + 3]};                     // (may run into the next row: replaced at use)
   };
-  const int nc = (n + CHUNK - 1) / CHUNK;
   auto fetch = [&](int c, In& x) {
     const int cc = min(c, nc - 1);
     const int64_t rr = row0 + cc * CHUNK;
@@ -497,42 +556,27 @@ __global__ __launch_bounds__(64 * NW) void delta_walk_kernel(const DeltaDims d, 
 #pragma unroll
       for (int i = 0; i < 4; i++) x.kz[i] = (pz + i * d.heads * 2)[lz];
     }
-    const float* vb = b.v + rr * vw + h * d.vdim;
-#pragma unroll
-    for (int i = 0; i < 4; i++) x.u0[i] = (vb + i * vw)[lv];
-    x.qk = *reinterpret_cast<const f32x4*>(b.qk + (rr * d.heads + h) * CHUNK + lqk);
-  };
-  auto total = [&](int it, int k) -> f32x4 {
-    f32x4 x[NW];
-#pragma unroll
-    for (int v = 0; v < NW; v++) x[v] = part[it][v][k][lane];
-#pragma unroll
-    for (int m = NW / 2; m; m >>= 1)
-#pragma unroll
-      for (int v = 0; v < m; v++) x[v] += x[v + m];
-    return x[0];
   };
   auto chunk = [&](int c, const In& x, int it) {         // (a chunk past the last one changes nothing)
-    const int nt = min(CHUNK, n - c * CHUNK);
+    const int nt = n - c * CHUNK;
     const bool rok = fr < nt;
-    bool tok[4];
+    f32x4 u[2] = {{0.0f, 0.0f, 0.0f, 0.0f}, {0.0f, 0.0f, 0.0f, 0.0f}}, o = {0.0f, 0.0f, 0.0f, 0.0f};
 #pragma unroll
-    for (int i = 0; i < 4; i++) tok[i] = fg * 4 + i < nt;
-    f32x4 u, o = {0.0f, 0.0f, 0.0f, 0.0f};
+    for (int i = 0; i < 4; i++)
 #pragma unroll
-    for (int i = 0; i < 4; i++) u[i] = wave == 0 && tok[i] && col < d.vdim ? x.u0[i] : 0.0f;
+      for (int j = 0; j < TPW; j++)
+        u[(i * TPW + j) & 1] = __builtin_amdgcn_mfma_f32_16x16x4f32(rok && ok4[j][VEC ? 0 : i] ? -x.w[j][i] : 0.0f, S[j][i], u[(i * TPW + j) & 1], 0, 0, 0);
+    pu[it][wave][lane] = u[0] + u[1];
+    __syncthreads();
+    const f32x4 t = total(it);
 #pragma unroll
-    for (int j = 0; j < TPW; j++)
+    for (int i = 0; i < 4; i++)
 #pragma unroll
-      for (int i = 0; i < 4; i++) {
-        const bool ok = rok && ok4[j][VEC ? 0 : i];
-        const float w = ok ? x.w[j][i] : 0.0f, q = ok ? (CH ? x.q[j][i] : x.q[j][i] * x.p) : 0.0f;
-        u = __builtin_amdgcn_mfma_f32_16x16x4f32(-w, S[j][i], u, 0, 0, 0);
+      for (int j = 0; j < TPW; j++) {      // the read-out with the state before the chunk, while the sums arrive
+        const float q = rok && ok4[j][VEC ? 0 : i] ? (CH ? x.q[j][i] : x.q[j][i] * x.p) : 0.0f;
         o = __builtin_amdgcn_mfma_f32_16x16x4f32(q, S[j][i], o, 0, 0, 0);
       }
-    part[it][wave][0][lane] = u; part[it][wave][1][lane] = o;
-    __syncthreads();
-    u = total(it, 0);
+    po[it][wave][lane] = o;
 #pragma unroll
     for (int j = 0; j < TPW; j++)
 #pragma unroll
@@ -541,17 +585,9 @@ __global__ __launch_bounds__(64 * NW) void delta_walk_kernel(const DeltaDims d, 
     for (int i = 0; i < 4; i++)
 #pragma unroll
       for (int j = 0; j < TPW; j++) {
-        const float k = tok[i] && ok1[j] ? (CH ? x.k[j][i] : x.k[j][i] * x.kz[i]) : 0.0f;
-        S[j] = __builtin_amdgcn_mfma_f32_16x16x4f32(k, u[i], S[j], 0, 0, 0);
+        const float k = fg * 4 + i < nt && ok1[j] ? (CH ? x.k[j][i] : x.k[j][i] * x.kz[i]) : 0.0f;
+        S[j] = __builtin_amdgcn_mfma_f32_16x16x4f32(k, t[i], S[j], 0, 0, 0);
       }
-    if (wave == NW - 1) {
-      o = total(it, 1);
-#pragma unroll
-      for (int i = 0; i < 4; i++) o = __builtin_amdgcn_mfma_f32_16x16x4f32(rok ? x.qk[i] : 0.0f, u[i], o, 0, 0, 0);
-      float* ob = b.o + (int64_t)(row0 + c * CHUNK) * vw + h * d.vdim;
-#pragma unroll
-      for (int i = 0; i < 4; i++) if (tok[i] && col < d.vdim) (ob + i * vw)[fg * 4 * vw + col] = o[i];
-    }
   };
   // (the scheduling barriers keep a chunk's requests in front of the chunk that is worked on: they are used two chunks later)
   In xa, xb, xc;
@@ -567,6 +603,7 @@ __global__ __launch_bounds__(64 * NW) void delta_walk_kernel(const DeltaDims d, 
     __builtin_amdgcn_sched_barrier(0);
     chunk(c + 2, xc, 2);
   }
+  __syncthreads();                         // the last chunk's read-outs are there
 #pragma unroll
   for (int j = 0; j < TPW; j++)
 #pragma unroll
@@ -788,10 +825,10 @@ int delta_chunked(const DeltaDims& d, const SeqPool::DeltaRun& st, const StepRow
   const dim3 g1(n_chunks, d.heads), g2((d.vdim + 15) / 16 * d.heads, r.n_ent), blk(256);
   if (d.channel_decay) hipLaunchKernelGGL(delta_chunk_kernel<true>, g1, blk, lds, s, d, r, b, chunks);
   else hipLaunchKernelGGL(delta_chunk_kernel<false>, g1, blk, lds, s, d, r, b, chunks);
-#define WALK_V(NW, N, CH) do { if (d.dim % 4 == 0) hipLaunchKernelGGL((delta_walk_kernel<NW, N, CH, true>), g2, dim3(64 * NW), 0, s, d, st.S, st.s_elems, r, b, chunk0); \
-                               else hipLaunchKernelGGL((delta_walk_kernel<NW, N, CH, false>), g2, dim3(64 * NW), 0, s, d, st.S, st.s_elems, r, b, chunk0); } while (0)
+#define WALK_V(NW, N, CH) do { if (d.dim % 4 == 0) hipLaunchKernelGGL((delta_walk_kernel<NW, N, CH, true>), g2, dim3(64 * (NW + 1)), 0, s, d, st.S, st.s_elems, r, b, chunk0); \
+                               else hipLaunchKernelGGL((delta_walk_kernel<NW, N, CH, false>), g2, dim3(64 * (NW + 1)), 0, s, d, st.S, st.s_elems, r, b, chunk0); } while (0)
 #define WALK(NW, N) do { if (d.channel_decay) WALK_V(NW, N, true); else WALK_V(NW, N, false); } while (0)
-  if (d.dim <= 64) WALK(4, 1); else if (d.dim <= 128) WALK(8, 1); else WALK(8, 2);
+  if (d.dim <= 64) WALK(4, 1); else if (d.dim <= 128) WALK(4, 2); else WALK(8, 2);
 #undef WALK
 #undef WALK_V
   CAI_HIP(hipGetLastError());

@@ -45,7 +45,10 @@ constexpr int GV_LDS = 16384;              // most floats of staged activations 
 template <typename AT, int NB, int R>
 __global__ __launch_bounds__(64 * GV_WAVES) void gemv_bf16(const uint16_t* __restrict__ W, const AT* __restrict__ x, int n_rows, int ldw, int64_t ldx, int ksplit, LinEpi e)
 {
-  extern __shared__ float xs[];            // [NB][panel]
+  // one row: as much as its width needs (more work-groups fit a CU); several rows: a fixed array, its layout known at compile time
+  extern __shared__ float xs_dyn[];
+  __shared__ float xs_fix[NB == 1 ? 1 : GV_LDS];
+  float* const xs = NB == 1 ? xs_dyn : xs_fix;
   __shared__ float part[GV_WAVES][R * NB];
   const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const int ks = wave % ksplit;
@@ -299,7 +302,7 @@ static void run_gemv(const cai_qw_s* w, const AT* x, int64_t ldx, const LinEpi& 
   while (ks < GV_WAVES && ks * 2 <= turns && groups * ks * 2 <= want * 2) ks *= 2;
   const int per = GV_WAVES / ks;
   const dim3 grid((groups + per - 1) / per), blk(64 * GV_WAVES);
-  const size_t lds = (size_t)((NB - 1) * (GV_LDS / NB / 512 * 512) + std::min(GV_LDS / NB / 512 * 512, turns * 512)) * 4;
+  const size_t lds = NB == 1 ? (size_t)std::min(GV_LDS, turns * 512) * 4 : 0;
   if (four) hipLaunchKernelGGL((gemv_bf16<AT, NB, 4>), grid, blk, lds, ctx().stream, (const uint16_t*)w->data, x, rows, (int)w->ld, ldx, ks, e);
   else hipLaunchKernelGGL((gemv_bf16<AT, NB, 2>), grid, blk, lds, ctx().stream, (const uint16_t*)w->data, x, rows, (int)w->ld, ldx, ks, e);
 }
