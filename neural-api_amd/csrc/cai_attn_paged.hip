@@ -87,6 +87,24 @@ __global__ __launch_bounds__(256) void attn_rows_kernel(const AttnDims d, const 
     return;
   }
   const bool own_new = SINGLE && k0 + nkeys == pos + 1;
+  // The slice's keys are requested first: sixteen lanes a key, eight elements a lane and turn, four keys a lane group.  A slice lies
+  // in at most two pages; a single row's own key is not in its page yet and comes from LDS below (columns past the width meet zeros
+  // in the query).
+  const int l16 = lane & 15, kb = wave * 4 + (lane >> 4);
+  const int pk = (k0 / PAGE_TOKENS + 1) * PAGE_TOKENS;                 // first key of the second page
+  const T* pg0 = kv_page<T>(kv, slot, k0), *pg1 = kv_page<T>(kv, slot, k0 + nkeys - 1);
+  float kx[4][2][8];
+#pragma unroll
+  for (int u = 0; u < 4; u++) {
+    const int key = k0 + max(0, min(kb + 16 * u, nkeys - 1 - (own_new ? 1 : 0)));
+    const T* kp = (key < pk ? pg0 : pg1) + ((int64_t)g * PAGE_TOKENS + key % PAGE_TOKENS) * d.dim_p;
+#pragma unroll
+    for (int t = 0; t < 2; t++) {
+      if (t && d.dim_p <= 128) continue;
+      const int c = l16 * 8 + t * 128;
+      load8<T>(kp + (c < d.dim_p ? c : 0), kx[u][t]);
+    }
+  }
   if (SINGLE) {
     const float* p = in.proj + row * in.ldp;
     for (int u = wave; u < nh + (own_new ? 1 : 0); u += 4) {
@@ -111,53 +129,28 @@ __global__ __launch_bounds__(256) void attn_rows_kernel(const AttnDims d, const 
     for (int c = tid; c < d.dim_p; c += 256) page[((int64_t)g * PAGE_TOKENS + tp) * d.dim_p + c] = (T)nk[c];
     for (int c = tid; c < d.vdim_p; c += 256) page[kv.v_off + ((int64_t)g * PAGE_TOKENS + tp) * d.vdim_p + c] = (T)nv[c];
   }
-  // the slice's two pages (the second may be the first again)
-  const int pk = (k0 / PAGE_TOKENS + 1) * PAGE_TOKENS;                 // first key of the second page
-  const T* pg0 = kv_page<T>(kv, slot, k0), *pg1 = kv_page<T>(kv, slot, k0 + nkeys - 1);
-  // scores: sixteen lanes a key, eight elements a lane and turn
-  const int l16 = lane & 15;
-  for (int kb = wave * 4 + (lane >> 4); kb < ((nkeys + 63) & ~63); kb += 64) {      // four keys of each lane group at a time: their loads are in flight together
-    float kx[4][2][8];
+  // scores of a lane group's four keys
 #pragma unroll
-    for (int u = 0; u < 4; u++) {
-      const int kk = min(kb + 16 * u, nkeys - 1), key = k0 + kk;
-      const bool fresh = SINGLE && key == pos;
-      const T* kp = (key < pk ? pg0 : pg1) + ((int64_t)g * PAGE_TOKENS + key % PAGE_TOKENS) * d.dim_p;
+  for (int hh = 0; hh < HT; hh++) {
+    if (hh >= nh) break;
+    float s[4] = {0.0f, 0.0f, 0.0f, 0.0f};
 #pragma unroll
-      for (int t = 0; t < 2; t++) {
-        const int c = l16 * 8 + t * 128;
-        if (t && d.dim_p <= 128) continue;
-        if (fresh) {
+    for (int t = 0; t < 2; t++) {
+      if (t && d.dim_p <= 128) continue;
+      float q[8];
+      *reinterpret_cast<f32x4*>(q) = *reinterpret_cast<const f32x4*>(&sq[hh][l16 * 8 + t * 128]);
+      *reinterpret_cast<f32x4*>(q + 4) = *reinterpret_cast<const f32x4*>(&sq[hh][l16 * 8 + t * 128 + 4]);
 #pragma unroll
-          for (int i = 0; i < 8; i++) kx[u][t][i] = nk[c + i];
-        } else if (c < d.dim_p) load8<T>(kp + c, kx[u][t]);
-        else {
+      for (int u = 0; u < 4; u++) {
+        const bool fresh = own_new && kb + 16 * u == nkeys - 1;
 #pragma unroll
-          for (int i = 0; i < 8; i++) kx[u][t][i] = 0.0f;
-        }
+        for (int i = 0; i < 8; i++) s[u] = fmaf(q[i], fresh ? nk[l16 * 8 + t * 128 + i] : kx[u][t][i], s[u]);
       }
     }
 #pragma unroll
-    for (int hh = 0; hh < HT; hh++) {
-      if (hh >= nh) break;
-      float s[4] = {0.0f, 0.0f, 0.0f, 0.0f};
-#pragma unroll
-      for (int t = 0; t < 2; t++) {
-        if (t && d.dim_p <= 128) continue;
-        float q[8];
-        *reinterpret_cast<f32x4*>(q) = *reinterpret_cast<const f32x4*>(&sq[hh][l16 * 8 + t * 128]);
-        *reinterpret_cast<f32x4*>(q + 4) = *reinterpret_cast<const f32x4*>(&sq[hh][l16 * 8 + t * 128 + 4]);
-#pragma unroll
-        for (int u = 0; u < 4; u++)
-#pragma unroll
-          for (int i = 0; i < 8; i++) s[u] = fmaf(q[i], kx[u][t][i], s[u]);
-      }
-#pragma unroll
-      for (int u = 0; u < 4; u++) {
-        s[u] += __shfl_xor(s[u], 8); s[u] += __shfl_xor(s[u], 4); s[u] += __shfl_xor(s[u], 2); s[u] += __shfl_xor(s[u], 1);
-        const int kk = kb + 16 * u;
-        if (l16 == 0) sc[hh][kk] = s[u] * d.scale;
-      }
+    for (int u = 0; u < 4; u++) {
+      s[u] += __shfl_xor(s[u], 8); s[u] += __shfl_xor(s[u], 4); s[u] += __shfl_xor(s[u], 2); s[u] += __shfl_xor(s[u], 1);
+      if (l16 == 0) sc[hh][kb + 16 * u] = s[u] * d.scale;
     }
   }
   __syncthreads();

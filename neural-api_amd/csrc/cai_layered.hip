@@ -280,7 +280,9 @@ static int ensure_rows(LayeredNet* n, int rows)
   };
   const size_t RS = R + DELTA_CHUNK + 1;    // the chunked walk requests whole chunks: up to 15 rows (and three values) past the last one
   size_t part = 0;
-  for (auto& a : n->pool.attn) part = std::max(part, attn_paged_part_floats(a.d, (int)R));
+  // (with bfloat16 activations only steps without a prompt portion take the row form)
+  const int part_rows = n->act_t == ACT_T_F32 ? (int)R : std::min((int)R, ATTN_PROMPT_MIN * n->max_seq);
+  for (auto& a : n->pool.attn) part = std::max(part, attn_paged_part_floats(a.d, part_rows));
   int rc;
   if ((rc = get((void**)&n->x, R * w * 4)) || (rc = get((void**)&n->x0, n->looped ? R * w * 4 : 0)) || (rc = get((void**)&n->proj, R * n->ld_proj * 4)) ||
       (rc = get((void**)&n->yl, n->has_attn ? R * w * 4 : 0)) || (rc = get((void**)&n->yr, n->has_attn ? R * w * 4 : 0)) || (rc = get((void**)&n->part, part * 4)) ||
@@ -324,8 +326,12 @@ int net_create(NetSpec&& spec, int max_tokens, int max_seq, int act_t, LayeredNe
   const int L = (int)s.layers.size();
   auto add_run = [&](int l, bool again) {
     NetRun r{l, again, -1, -1};
-    const NetLayer& y = s.layers[l];
-    if (y.kind == MIX_PARALLEL) { r.attn_run = (int)n->pool.attn.size(); n->pool.attn.push_back({y.attn.d}); }
+    NetLayer& y = s.layers[l];
+    if (y.kind == MIX_PARALLEL) {
+      // (a sequence longer than the pool exists only if every window is shorter than it: a wider window sees the same keys cut down)
+      y.attn.d.window = std::min(y.attn.d.window, (max_tokens + PAGE_TOKENS - 1) / PAGE_TOKENS * PAGE_TOKENS);
+      r.attn_run = (int)n->pool.attn.size(); n->pool.attn.push_back({y.attn.d});
+    }
     r.delta_run = (int)n->pool.delta.size(); n->pool.delta.push_back({y.delta.d});
     n->runs.push_back(r);
   };
@@ -540,7 +546,7 @@ int net_step(LayeredNet* n, int n_ent, const int32_t* seq, const int32_t* count,
     std::vector<int32_t> tiles, chunks, chunk0;
     bool tall = false, chunked = false;
     for (int e = 0; e < n_ent; e++) {
-      tall = tall || count[e] >= 16; chunked = chunked || count[e] >= DELTA_CHUNK_MIN;
+      tall = tall || count[e] >= ATTN_PROMPT_MIN; chunked = chunked || count[e] >= DELTA_CHUNK_MIN;
       chunk0.push_back((int)chunks.size() / 2);
       for (int t = 0; t < count[e]; t += ATTN_TILE) { tiles.push_back(e); tiles.push_back(t); }
       for (int t = 0; t < count[e]; t += DELTA_CHUNK) { chunks.push_back(e); chunks.push_back(t); }

@@ -113,6 +113,7 @@ int attn_paged_rows(const AttnDims& d, const KvView& kv, int act_t, const void* 
 size_t attn_paged_part_floats(const AttnDims& d, int n_rows);
 bool attn_paged_prompt_ok(const AttnDims& d, int act_t);
 int attn_paged_prompt(const AttnDims& d, const KvView& kv, const void* qbuf, const StepRows& r, const int32_t* tiles, int n_tiles, void* out, int64_t ldo);
+constexpr int ATTN_PROMPT_MIN = 16;        // portions from here on make a step take the prompt kernel
 constexpr int ATTN_TILE = 64;              // query rows of one entry per work-group of the prompt kernel
 
 // ---- gated delta rule (cai_delta.hip) ----

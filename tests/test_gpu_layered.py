@@ -146,6 +146,33 @@ def test_portions_and_decoding_agree_with_the_whole(cai, model, cuts, dt):
     dec.close()
 
 
+@pytest.mark.parametrize("loop", [None, (0, 3, 2), (2, 3, 3), (0, 1, 4), (1, 1, 5), (1, 2, 1), (0, 2, 2)], ids=str)
+def test_repeated_layers(cai, tmp_path, loop):
+    """stretches at the start, in the middle, at the end, of one layer, empty and run once: each pass has cache and state of its own"""
+    cfg = B.config([B.layer(B.delta()), B.layer((B.attn(window=5), B.delta(dim=12)), ff=None), B.layer((B.attn(heads=2, window=70), B.delta()))],
+                   loop=loop and dict(start=loop[0], stop=loop[1], times=loop[2]))
+    if loop is None:
+        del cfg["loop"]
+    m = Model(tmp_path, cfg, seed=4)
+    tok = m.tokens(100, 1)
+    dec = m.open(cai, 128)
+    for cuts in ([100], [40, 1], [33, 2, 5]):
+        dec.reset()
+        check(feed(dec, tok, cuts), m.ref(tok), "f32")
+    dec.close()
+
+
+@pytest.mark.parametrize("dt", ["f32", "bf16"])
+def test_a_window_wider_than_the_pool(cai, tmp_path, dt):
+    m = Model(tmp_path, B.config([B.layer((B.attn(heads=3, kv_heads=1, dim=40, vdim=72, window=1 << 29), B.delta()))]), seed=6)
+    tok = m.tokens(384, 2)
+    dec = m.open(cai, 384, 1, dt)
+    for cuts in ([384], [300, 1]):
+        dec.reset()
+        check(feed(dec, tok, cuts), m.ref(tok), dt)
+    dec.close()
+
+
 @pytest.mark.parametrize("dt", ["f32", "bf16"])
 def test_first_tokens(cai, model, dt):
     dec = model.open(cai, 64, 1, dt)
