@@ -293,7 +293,7 @@ LAYERED_SIZES = {"w2048": dict(width=2048, ff=5632, heads=16, kv_heads=8, dim=12
                  "w4096": dict(width=4096, ff=11008, heads=32, kv_heads=16, dim=128, n_layers=8, vocab=32768)}
 
 
-def layered_bench(cai, synth, torch, only, size):
+def layered_bench(cai, synth, torch, only, size, what, prompt_len, batch):
     """Prompt (512 and 2048 tokens) and decode (batch 1, 4, 8 after a 512-token prompt) throughput of the layered decoder and of the
     closest older model at equal size.  Times are HIP events around the library's own entry points; median of 5."""
     import tempfile
@@ -334,7 +334,7 @@ def layered_bench(cai, synth, torch, only, size):
                 per_tok = 2.0 * c["n_layers"] * (c["d_model"] * (2 * qw + 2 * kw) + 3 * c["d_model"] * c["ffn"])
                 label = "Llama Q8_0"
             wb = dec.weight_bytes()
-            for T in (512, 2048):
+            for T in () if what == "decode" else (prompt_len,) if prompt_len > 0 else (512, 2048):
                 tok = rng.integers(0, z["vocab"], T).astype(np.int32)
                 for _ in range(2):
                     dec.reset(); dec.prefill(tok, want_logits=False)
@@ -342,7 +342,7 @@ def layered_bench(cai, synth, torch, only, size):
                 print(json.dumps({"layered_bench": label, "size": name, "what": "prompt", "tokens": T, "ms": round(ms, 3), "tok_per_s": round(T / ms * 1e3),
                                   "linear_TFLOP_per_s": round(per_tok * T / ms / 1e9, 1), "frac_of_bf16_peak": round(per_tok * T / ms / 1e9 / 2500.0, 4)}), flush=True)
             tok = rng.integers(0, z["vocab"], 512).astype(np.int32)
-            for B in (1, 4, 8):
+            for B in () if what == "prompt" else (batch,) if what == "decode" else (1, 4, 8):
                 for b in range(8):
                     dec.reset(b)
                 for b in range(B):
@@ -398,6 +398,7 @@ def main():
     ap.add_argument("--layered", action="store_true", help="layered decoder (Samanex, bfloat16) at two sizes with random weights beside the Llama-type decoder of the same width, feed-forward, heads and depth (Q8_0 body, half-precision cache): prompt and decode throughput, one JSON line per measurement")
     ap.add_argument("--layered-only", choices=["", "samanex", "llama"], default="", help="with --layered: measure one of the two (for profiles)")
     ap.add_argument("--layered-size", choices=["", "w2048", "w4096"], default="", help="with --layered: measure one size")
+    ap.add_argument("--layered-what", choices=["", "prompt", "decode"], default="", help="with --layered: prompts only (of --prompt tokens, if given) or decoding only (of --batch sequences)")
     args = ap.parse_args()
     if args.gpus != 1:
         print("bench.py: this build runs on ONE GPU; --gpus %d is not supported (no collectives are part of it)" % args.gpus, file=sys.stderr)
@@ -431,7 +432,7 @@ def main():
         gemm_sweep(cai, synth, torch)
         return
     if args.layered:
-        layered_bench(cai, synth, torch, args.layered_only, args.layered_size)
+        layered_bench(cai, synth, torch, args.layered_only, args.layered_size, args.layered_what, args.prompt, args.batch)
         return
     conf = CONFIGS[args.config]
     cfg = dict(conf["cfg"])
