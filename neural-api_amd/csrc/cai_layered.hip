@@ -226,7 +226,7 @@ struct LayeredNet {
   int wp = 0, ld_proj = 0, ld_mid = 0, ld_att = 0, ld_attl = 0, ld_q = 0, ld_ra = 0, ld_rg = 0;
   int w_q = 0, w_k = 0, w_v = 0, w_g = 0, w_b = 0, w_za = 0, w_zg = 0, w_hd = 0, w_qt = 0, w_qk = 0, w_gt1 = 0;
   bool has_attn = false, looped = false;
-  int cap = 0, logit_cap = 0, best_cap = 0;
+  int cap = 0, logit_cap = 0;
   float *x = nullptr, *x0 = nullptr, *proj = nullptr, *yl = nullptr, *yr = nullptr, *part = nullptr, *logits = nullptr;
   void *h = nullptr, *mid = nullptr, *att = nullptr, *attl = nullptr, *qbuf = nullptr, *ra = nullptr, *rgb = nullptr, *hw = nullptr;
   DeltaBuf db{};
@@ -722,7 +722,7 @@ int net_snapshot(LayeredNet* n, int seq, NetSnap** out)
   NetSnap* s = new NetSnap();
   s->len = q.len; s->first_page = q.first_page; s->end_page = q.end_page; s->n_attn = (int)n->pool.attn.size(); s->n_delta = (int)n->pool.delta.size();
   s->bytes = snap_bytes(n, q.end_page - q.first_page);
-  if (hipMalloc((void**)&s->data, (size_t)s->bytes) != hipSuccess) { (void)hipGetLastError(); delete s; return set_error(CAI_ERR_NOMEM, "snapshot: %lld bytes", (long long)q.len); }
+  if (hipMalloc((void**)&s->data, (size_t)s->bytes) != hipSuccess) { (void)hipGetLastError(); delete s; return set_error(CAI_ERR_NOMEM, "snapshot: out of device memory (a sequence of %d tokens)", q.len); }
   const int rc = snap_walk(n, seq, [&](char* p, size_t sz, int64_t off) -> int { CAI_HIP(hipMemcpyAsync(s->data + off, p, sz, hipMemcpyDeviceToDevice, ctx().stream)); return CAI_OK; });
   if (rc) { net_snap_free(s); return rc; }
   CAI_HIP(hipStreamSynchronize(ctx().stream));

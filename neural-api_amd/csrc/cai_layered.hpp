@@ -42,7 +42,7 @@ __host__ __device__ inline int glu_row(int j, int up) { return (j >> 4) * 32 + u
 
 // y = W x for n_tok activation rows x[t][ldx] (zero padded to LIN_PAD columns, element type act_t); W is a CAI_BF16 matrix.
 int launch_lin(const cai_qw_s* w, int act_t, const void* x, int64_t ldx, int n_tok, const LinEpi& e);
-// two products of one shape class in one launch (same padded width not required): decode rows only
+// float columns [col0, col0 + cols) of x -> rows of the chosen type, zero padded to ldo
 int launch_pack_rows(const float* x, int64_t ldx, int64_t col0, int cols, int n_tok, int act_t, void* out, int64_t ldo);
 int bf16_dequant_rows(const cai_qw_s* w, int64_t row0, int64_t n_rows, float* out);
 int bf16_linear_f32(const cai_qw_s* w, const float* x, int64_t ldx, int n_tok, float* y, int64_t ldy, int act);   // unpadded float rows in, float rows out
@@ -140,7 +140,6 @@ int delta_single(const DeltaDims& d, const DeltaIn& in, const DeltaW& w, const S
 // ------------------------------------------------------------------------------------------
 // The layered decoder (cai_layered.hip): layers of different kinds, some run several times.
 // ------------------------------------------------------------------------------------------
-struct NetLinear { cai_qw_s* w = nullptr; };
 struct NetDelta { DeltaDims d{}; DeltaW w{}; int oq = 0, ok = 0, ov = 0, ob = 0, oa = 0, og = 0; cai_qw_s* out = nullptr; };
 struct NetAttn { AttnDims d{}; const float *qn = nullptr, *kn = nullptr; int oq = 0, ok = 0, ov = 0; cai_qw_s* out = nullptr; };
 enum { MIX_DELTA = 0, MIX_PARALLEL = 1 };

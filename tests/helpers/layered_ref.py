@@ -1,12 +1,8 @@
 """Plain, slow float64 implementation of the layered decoder designs, one function per mechanism.
 
-This is the checker of the layered decoder (tests/test_layered_*.py): numpy only, token by token where the mechanism is a
+This is the oracle of the layered decoder (tests/test_layered_ref.py, tests/test_gpu_layered.py): numpy only, token by token where the mechanism is a
 recurrence, a full score matrix where it is an attention, and no code shared with the product library.
 """
-import json
-import os
-import struct
-
 import numpy as np
 
 
@@ -161,26 +157,3 @@ def forward(cfg, w, tokens, layers_out=None):
         if layers_out is not None:
             layers_out.append(x.copy())
     return linear(w["head"], norm("final.norm", x))
-
-
-# ---------------------------------------------------------------- files
-def read_model(path):
-    """(config, float64 tensors) of a folder with config.json and model.safetensors"""
-    with open(os.path.join(path, "config.json")) as f:
-        cfg = json.load(f)
-    with open(os.path.join(path, "model.safetensors"), "rb") as f:
-        (n,) = struct.unpack("<Q", f.read(8))
-        head = json.loads(f.read(n))
-        blob = f.read()
-    out = {}
-    for name, t in head.items():
-        if name == "__metadata__":
-            continue
-        a, b = t["data_offsets"]
-        raw = blob[a:b]
-        if t["dtype"] == "BF16":
-            v = (np.frombuffer(raw, "<u2").astype(np.uint32) << 16).view(np.float32)
-        else:
-            v = np.frombuffer(raw, {"F32": "<f4", "I32": "<i4", "F16": "<f2"}[t["dtype"]])
-        out[name] = v.reshape(t["shape"]).astype(np.float64)
-    return cfg, out

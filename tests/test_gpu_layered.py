@@ -1,4 +1,4 @@
-"""The layered decoder on the device against the float64 checker: every mechanism alone, prompts, decoding, portions, mixed
+"""The layered decoder on the device against the float64 oracle: every mechanism alone, prompts, decoding, portions, mixed
 batches, reused pages and slots, window edges, long decoding, greedy and sampled generation through the scheduler."""
 import json
 import os
@@ -260,7 +260,7 @@ def test_window_edges(cai, tmp_path, window, dt):
     inside, outside = keys.copy(), keys.copy()
     for p in places:
         inside[p + window - 1] = 400 + keys[p]; outside[p + window] = 400 + keys[p]
-    # the checker tells the edge apart: seen from the last place of the window, not from the next one
+    # the oracle tells the edge apart: seen from the last place of the window, not from the next one
     wider = json.loads(json.dumps(cfg)); wider["layers"][0]["mixer"]["left"]["mask"]["size"] = window + 1
     rows = [p + window for p in places if not (outside[p] >= 400)]
     apart = np.abs(R.forward(wider, m.w, outside) - m.ref(outside))[rows].max(1)
@@ -312,7 +312,7 @@ def greedy(dec, prompt, n, seq=0):
 
 
 def margin(model, prompt, out):
-    """smallest lead of the chosen token in the checker's logits along a greedy run"""
+    """smallest lead of the chosen token in the oracle's logits along a greedy run"""
     lg = model.ref(list(prompt) + out[:-1])[len(prompt) - 1:]
     top = np.sort(lg, axis=1)
     assert [int(r.argmax()) for r in lg] == out or float((top[:, -1] - top[:, -2]).min()) < 1e-3

@@ -1,4 +1,4 @@
-"""The layered decoder's float64 checker against independent statements of the same mechanisms, and the registry's refusals."""
+"""The layered decoder's float64 oracle against independent statements of the same mechanisms, and the registry's refusals."""
 import json
 import os
 
@@ -59,7 +59,7 @@ def test_run_order_of_repeated_layers():
     assert R.run_order(dict(layers=[None] * 2)) == [(0, False), (1, False)]
 
 
-def test_checker_is_sensitive_to_what_it_checks():
+def test_oracle_is_sensitive_to_what_it_checks():
     """a window off by one, a lost state, a wrong group or a missing repeat moves the logits well beyond the tests' tolerances"""
     cfg = B.config([B.layer(B.delta()), B.layer((B.attn(), B.delta(dim=12)))], loop=dict(start=0, stop=2, times=2))
     w = {n: B.to_bf16(a)[1].reshape(np.shape(a)) for n, a in B.weights(cfg, 5).items()}
