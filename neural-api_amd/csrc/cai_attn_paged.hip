@@ -1,5 +1,6 @@
-// Sliding-window grouped-query attention over a paged key/value pool: key and value widths of their own, optional per-head RMS
-// norm of queries and keys, an explicit score scale, no rotation.
+// Grouped-query attention over a paged key/value pool, in a sliding window or in fixed blocks of positions: key and value widths of
+// their own, optional per-head RMS norm of queries and keys, optional rotation of the first dimensions of a head, an explicit score
+// scale, an optional sigmoid gate on the heads' outputs.
 //
 // Two forms: one work-group per (row, key/value head, slice of keys) for decoded tokens, short portions and the all-32-bit mode,
 // and a matrix-core form for prompts, whose key tile is one page.  Scores, soft-max and weights are 32-bit in both; the
@@ -31,17 +32,37 @@ template <typename T> __device__ __forceinline__ T* kv_page(const KvView& kv, in
   return reinterpret_cast<T*>(kv.base) + (int64_t)kv.table[slot * kv.ring + (key / PAGE_TOKENS) % kv.ring] * kv.page_elems;
 }
 
-// RMS norm of a head of `dim` values by one wave: lane holds x[lane + 64 i]
-__device__ __forceinline__ void head_norm(const float* x, const float* gain, int dim, float eps, int lane, float* v)
+// A query or key head of `dim` values by one wave, lane holds x[lane + 64 i]: RMS norm (gain null: none), then the rotation at
+// position pos.  The angle is reduced in turns with double precision before sine and cosine.
+__device__ __forceinline__ void head_vector(const float* x, const float* gain, const AttnDims& d, int pos, int lane, float* v)
 {
-  float s = 0.0f;
+  float s = 0.0f, inv = 1.0f;
 #pragma unroll
-  for (int i = 0; i < 4; i++) { const int c = lane + 64 * i; v[i] = c < dim ? x[c] : 0.0f; s = fmaf(v[i], v[i], s); }
-  if (!gain) return;
-  s = wave_sum(s);
-  const float inv = 1.0f / sqrtf(__builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, s), 63)) / (float)dim + eps);
+  for (int i = 0; i < 4; i++) { const int c = lane + 64 * i; v[i] = c < d.dim ? x[c] : 0.0f; s = fmaf(v[i], v[i], s); }
+  if (gain) {
+    s = wave_sum(s);
+    inv = 1.0f / sqrtf(__builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, s), 63)) / (float)d.dim + d.eps);
 #pragma unroll
-  for (int i = 0; i < 4; i++) { const int c = lane + 64 * i; if (c < dim) v[i] *= inv * gain[c]; }
+    for (int i = 0; i < 4; i++) { const int c = lane + 64 * i; if (c < d.dim) v[i] *= inv * gain[c]; }
+  }
+  const int half = d.rot / 2;
+#pragma unroll
+  for (int i = 0; i < 4; i++) {
+    const int c = lane + 64 * i;
+    if (c >= d.rot) continue;
+    const bool lo = c < half;
+    const int j = lo ? c : c - half, other = lo ? c + half : j;
+    float o = x[other];
+    if (gain) o *= inv * gain[other];
+    const double t = (double)pos * d.turns[j];
+    float sn, cs;
+    sincospif((float)(2.0 * (t - rint(t))), &sn, &cs);
+    v[i] = lo ? v[i] * cs - o * sn : v[i] * cs + o * sn;
+  }
+}
+__device__ __forceinline__ float out_gate(const AttnIn& in, int64_t row, int c)
+{
+  return in.og < 0 ? 1.0f : 1.0f / (1.0f + expf(-in.proj[row * in.ldp + in.og + c]));
 }
 
 template <typename T>
@@ -54,7 +75,7 @@ __global__ __launch_bounds__(256) void attn_prep_kernel(const AttnDims d, const 
   for (int u = wave; u < d.heads + d.kv_heads; u += 4) {
     const bool is_q = u < d.heads; const int hh = is_q ? u : u - d.heads;
     float v[4];
-    head_norm(p + (is_q ? in.oq : in.ok) + hh * d.dim, is_q ? in.qn : in.kn, d.dim, d.eps, lane, v);
+    head_vector(p + (is_q ? in.oq : in.ok) + hh * d.dim, is_q ? in.qn : in.kn, d, pos, lane, v);
     T* dst = is_q ? qbuf + ((int64_t)row * d.heads + hh) * d.dim_p : page + ((int64_t)hh * PAGE_TOKENS + tp) * d.dim_p;
 #pragma unroll
     for (int i = 0; i < 4; i++) { const int c = lane + 64 * i; if (c < d.dim_p) dst[c] = (T)v[i]; }
@@ -81,7 +102,7 @@ __global__ __launch_bounds__(256) void attn_rows_kernel(const AttnDims d, const 
   const int hg = d.heads / d.kv_heads, hblk = (hg + HT - 1) / HT;
   const int row = blockIdx.z, g = blockIdx.y / hblk, h0 = g * hg + blockIdx.y % hblk * HT, nh = min(HT, (g + 1) * hg - h0);
   const int pos = r.pos[row], slot = r.slot[row];
-  const int lo = max(0, pos - d.window + 1), k0 = lo + blockIdx.x * SLICE, nkeys = min(SLICE, pos + 1 - k0);
+  const int lo = d.first_key(pos), k0 = lo + blockIdx.x * SLICE, nkeys = min(SLICE, pos + 1 - k0);
   const int n_sl = gridDim.x;
   if (nkeys <= 0) {                        // (part is only read up to the slices in use)
     return;
@@ -110,7 +131,7 @@ __global__ __launch_bounds__(256) void attn_rows_kernel(const AttnDims d, const 
     for (int u = wave; u < nh + (own_new ? 1 : 0); u += 4) {
       float v[4];
       const bool is_q = u < nh;
-      head_norm(is_q ? p + in.oq + (h0 + u) * d.dim : p + in.ok + g * d.dim, is_q ? in.qn : in.kn, d.dim, d.eps, lane, v);
+      head_vector(is_q ? p + in.oq + (h0 + u) * d.dim : p + in.ok + g * d.dim, is_q ? in.qn : in.kn, d, pos, lane, v);
       float* dst = is_q ? sq[u] : nk;
 #pragma unroll
       for (int i = 0; i < 4; i++) dst[lane + 64 * i] = is_q ? v[i] : round_to<T>(v[i]);
@@ -217,7 +238,7 @@ __global__ __launch_bounds__(256) void attn_rows_kernel(const AttnDims d, const 
   for (int i = tid; i < nh * d.vdim_p; i += 256) {
     const int hh = i / d.vdim_p, c = i % d.vdim_p;
     const float s = red[0][hh][c] + red[1][hh][c] + red[2][hh][c] + red[3][hh][c];
-    if (n_sl == 1) { if (c < d.vdim) out[row * ldo + (h0 + hh) * d.vdim + c] = (T)(s / ssum[hh]); }
+    if (n_sl == 1) { if (c < d.vdim) out[row * ldo + (h0 + hh) * d.vdim + c] = (T)(s / ssum[hh] * out_gate(in, row, (h0 + hh) * d.vdim + c)); }
     else part[(((int64_t)row * d.heads + h0 + hh) * n_sl + blockIdx.x) * (d.vdim_p + 2) + c] = s;
   }
   if (n_sl > 1 && tid < nh) {
@@ -227,11 +248,11 @@ __global__ __launch_bounds__(256) void attn_rows_kernel(const AttnDims d, const 
 }
 
 template <typename T>
-__global__ __launch_bounds__(256) void attn_rows_merge_kernel(const AttnDims d, const StepRows r, const int n_sl, const float* part, T* out, const int64_t ldo)
+__global__ __launch_bounds__(256) void attn_rows_merge_kernel(const AttnDims d, const AttnIn in, const StepRows r, const int n_sl, const float* part, T* out, const int64_t ldo)
 {
   __shared__ float sm[4], sl[4], sw[256];
   const int h = blockIdx.x, row = blockIdx.y, pos = r.pos[row], tid = threadIdx.x;
-  const int used = (min(d.window, pos + 1) + SLICE - 1) / SLICE, st = d.vdim_p + 2;
+  const int used = (pos - d.first_key(pos) + SLICE) / SLICE, st = d.vdim_p + 2;
   const float* p = part + ((int64_t)row * d.heads + h) * n_sl * st;
   float m = -INFINITY, l = 0.0f;
   for (int s = tid; s < used; s += 256) m = fmaxf(m, p[s * st + d.vdim_p]);
@@ -258,7 +279,7 @@ __global__ __launch_bounds__(256) void attn_rows_merge_kernel(const AttnDims d, 
       }
     }
   }
-  if (tid < d.vdim) out[row * ldo + h * d.vdim + tid] = (T)(acc / (sl[0] + sl[1] + sl[2] + sl[3]));
+  if (tid < d.vdim) out[row * ldo + h * d.vdim + tid] = (T)(acc / (sl[0] + sl[1] + sl[2] + sl[3]) * out_gate(in, row, h * d.vdim + tid));
 }
 
 // ------------------------------------------------------------------------------------------
@@ -268,7 +289,7 @@ __global__ __launch_bounds__(256) void attn_rows_merge_kernel(const AttnDims d, 
 // 4 g + j - 4 of its second 16 otherwise, and V^T is read from LDS in that order.
 // ------------------------------------------------------------------------------------------
 template <int KQ, int VQ>                  // key width in 32s, value width in 16s
-__global__ __launch_bounds__(256) void attn_prompt_paged_kernel(const AttnDims d, const KvView kv, const bf16_t* qbuf, const StepRows r, const int32_t* tiles, bf16_t* out, const int64_t ldo)
+__global__ __launch_bounds__(256) void attn_prompt_paged_kernel(const AttnDims d, const KvView kv, const AttnIn in, const bf16_t* qbuf, const StepRows r, const int32_t* tiles, bf16_t* out, const int64_t ldo)
 {
   constexpr int KST = KQ * 32 + 8, VST = PAGE_TOKENS + 4;
   __shared__ __align__(16) uint16_t sk[PAGE_TOKENS * KST];
@@ -286,7 +307,7 @@ __global__ __launch_bounds__(256) void attn_prompt_paged_kernel(const AttnDims d
   const int32_t* en = r.ent + 4 * tiles[2 * tile];
   const int slot = en[0], row0 = en[1], n = en[2], pos0 = en[3], t0 = tiles[2 * tile + 1];
   const int g = h / hg;
-  const int qi = t0 + wave * 16 + fr, qr = min(qi, n - 1), qpos = pos0 + qr;
+  const int qi = t0 + wave * 16 + fr, qr = min(qi, n - 1), qpos = pos0 + qr, qlo = d.first_key(qpos);
   u32x4 fq[KQ];
 #pragma unroll
   for (int k = 0; k < KQ; k++) {
@@ -298,9 +319,9 @@ __global__ __launch_bounds__(256) void attn_prompt_paged_kernel(const AttnDims d
 #pragma unroll
   for (int v = 0; v < VQ; v++) o[v] = f32x4{0.0f, 0.0f, 0.0f, 0.0f};
   float m = -INFINITY, l = 0.0f;
-  const int first = max(0, pos0 + t0 - d.window + 1) / PAGE_TOKENS, last = (pos0 + min(t0 + ATTN_TILE, n) - 1) / PAGE_TOKENS;
-  const int wlo = max(0, pos0 + min(t0 + wave * 16, n - 1) - d.window + 1), whi = pos0 + min(t0 + wave * 16 + 15, n - 1);   // keys this wave's rows see
-  const int wmin = pos0 + min(t0 + wave * 16, n - 1);                 // the wave's first row
+  const int first = d.first_key(pos0 + t0) / PAGE_TOKENS, last = (pos0 + min(t0 + ATTN_TILE, n) - 1) / PAGE_TOKENS;
+  const int wmin = pos0 + min(t0 + wave * 16, n - 1), whi = pos0 + min(t0 + wave * 16 + 15, n - 1);   // the wave's first and last row
+  const int wlo = d.first_key(wmin), wall = d.first_key(whi);         // first key any of its rows sees, first key all of them see
   const float scale2 = d.scale * 1.44269504088896340736f;             // scores in base-2 logarithms
   constexpr int KC = PAGE_TOKENS * KQ * 4 / 256, VC = PAGE_TOKENS / 2 * VQ * 2 / 256;   // 16-byte key chunks / value chunk pairs per thread
   u32x4 rk[KC], rv[VC][2];
@@ -357,7 +378,7 @@ __global__ __launch_bounds__(256) void attn_prompt_paged_kernel(const AttnDims d
       }
     }
     float mt = -INFINITY;
-    if (pg * PAGE_TOKENS + PAGE_TOKENS - 1 <= wmin && pg * PAGE_TOKENS > whi - d.window) {   // every row of the wave sees the whole page
+    if (pg * PAGE_TOKENS + PAGE_TOKENS - 1 <= wmin && pg * PAGE_TOKENS >= wall) {   // every row of the wave sees the whole page
 #pragma unroll
       for (int t = 0; t < 4; t++)
 #pragma unroll
@@ -367,8 +388,8 @@ __global__ __launch_bounds__(256) void attn_prompt_paged_kernel(const AttnDims d
       for (int t = 0; t < 4; t++)
 #pragma unroll
         for (int i = 0; i < 4; i++) {
-          const int back = qpos - (pg * PAGE_TOKENS + t * 16 + fg * 4 + i);
-          s[t][i] = back >= 0 && back < d.window ? s[t][i] * scale2 : -INFINITY;
+          const int key = pg * PAGE_TOKENS + t * 16 + fg * 4 + i;
+          s[t][i] = key <= qpos && key >= qlo ? s[t][i] * scale2 : -INFINITY;
           mt = fmaxf(mt, s[t][i]);
         }
     }
@@ -416,7 +437,7 @@ __global__ __launch_bounds__(256) void attn_prompt_paged_kernel(const AttnDims d
 #pragma unroll
       for (int i = 0; i < 4; i++) {
         const int c = v * 16 + fg * 4 + i;
-        if (c < d.vdim) out[(int64_t)(row0 + qi) * ldo + h * d.vdim + c] = (bf16_t)(o[v][i] * inv);
+        if (c < d.vdim) out[(int64_t)(row0 + qi) * ldo + h * d.vdim + c] = (bf16_t)(o[v][i] * inv * out_gate(in, row0 + qi, h * d.vdim + c));
       }
   }
 }
@@ -429,7 +450,7 @@ int attn_paged_prep(const AttnDims& d, const KvView& kv, int act_t, const AttnIn
   return CAI_OK;
 }
 
-static int n_slices(const AttnDims& d) { return (d.window + SLICE - 1) / SLICE; }
+static int n_slices(const AttnDims& d) { return (d.span + SLICE - 1) / SLICE; }
 size_t attn_paged_part_floats(const AttnDims& d, int n_rows)
 {
   const int ns = n_slices(d);
@@ -443,7 +464,7 @@ static void run_rows(const AttnDims& d, const KvView& kv, const AttnIn& in, cons
   const dim3 grid(ns, d.kv_heads * ((hg + HT - 1) / HT), r.n_rows);
   if (single) hipLaunchKernelGGL((attn_rows_kernel<T, HT, true>), grid, dim3(256), 0, ctx().stream, d, kv, in, r, qbuf, out, ldo, part);
   else hipLaunchKernelGGL((attn_rows_kernel<T, HT, false>), grid, dim3(256), 0, ctx().stream, d, kv, in, r, qbuf, out, ldo, part);
-  if (ns > 1) hipLaunchKernelGGL(attn_rows_merge_kernel<T>, dim3(d.heads, r.n_rows), dim3(256), 0, ctx().stream, d, r, ns, part, out, ldo);
+  if (ns > 1) hipLaunchKernelGGL(attn_rows_merge_kernel<T>, dim3(d.heads, r.n_rows), dim3(256), 0, ctx().stream, d, in, r, ns, part, out, ldo);
 }
 template <typename T>
 static void run_rows_t(const AttnDims& d, const KvView& kv, const AttnIn& in, const StepRows& r, const void* qbuf, void* out, int64_t ldo, float* part, bool single)
@@ -463,10 +484,10 @@ int attn_paged_rows(const AttnDims& d, const KvView& kv, int act_t, const void* 
 
 bool attn_paged_prompt_ok(const AttnDims& d, int act_t) { return act_t == ACT_T_BF16 && d.dim <= 256 && d.vdim <= 256; }
 
-int attn_paged_prompt(const AttnDims& d, const KvView& kv, const void* qbuf, const StepRows& r, const int32_t* tiles, int n_tiles, void* out, int64_t ldo)
+int attn_paged_prompt(const AttnDims& d, const KvView& kv, const AttnIn& in, const void* qbuf, const StepRows& r, const int32_t* tiles, int n_tiles, void* out, int64_t ldo)
 {
   const dim3 grid(n_tiles, d.heads), blk(256);
-#define PROMPT(K, V) hipLaunchKernelGGL((attn_prompt_paged_kernel<K, V>), grid, blk, 0, ctx().stream, d, kv, (const bf16_t*)qbuf, r, tiles, (bf16_t*)out, ldo)
+#define PROMPT(K, V) hipLaunchKernelGGL((attn_prompt_paged_kernel<K, V>), grid, blk, 0, ctx().stream, d, kv, in, (const bf16_t*)qbuf, r, tiles, (bf16_t*)out, ldo)
 #define PROMPT_V(K) do { if (d.vdim <= 64) PROMPT(K, 4); else if (d.vdim <= 128) PROMPT(K, 8); else PROMPT(K, 16); } while (0)
   if (d.dim <= 64) PROMPT_V(2); else if (d.dim <= 128) PROMPT_V(4); else PROMPT_V(8);
 #undef PROMPT_V

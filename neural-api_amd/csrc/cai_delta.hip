@@ -4,46 +4,10 @@
 // Per head a float state S [dim][vdim] (rows padded to four columns, the padding stays zero); one token does  S <- diag(g) S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q.
 // With S' = diag(g) S the read-out is  o = S'^T q + (q . k) u, so both products with S' are taken together and the second
 // reduction is off the dependent chain.  Everything that touches the state is 32-bit.
-//
-// A sequence's last `taps` raw inputs of every convolved channel are kept in a ring (entry position mod taps).  The ring has one
-// entry more than a token looks back, so the entry the newest token takes is never one that the same step still reads.
 #include "cai_layered.hpp"
-#include "cai_gemv_common.hpp"
+#include "cai_recurrent.hpp"
 
 namespace cai {
-
-__device__ __forceinline__ float wave_total(float v)   // the sum in every lane
-{
-  v = wave_sum(v);
-  return __builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, v), 63));
-}
-__device__ __forceinline__ float sigmoid_f(float z)
-{
-  if (z >= 0.0f) return 1.0f / (1.0f + expf(-z));
-  const float s = expf(z); return s / (1.0f + s);
-}
-__device__ __forceinline__ float softplus_f(float z) { return fmaxf(z, 0.0f) + log1pf(expf(-fabsf(z))); }
-template <int CTRL> __device__ __forceinline__ float dpp_add(float v)
-{
-  return v + __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), CTRL, 0xf, 0xf, true));
-}
-__device__ __forceinline__ float row16_total(float v)  // the sum over the lane's row of 16, in every lane of it (row rotations)
-{
-  v = dpp_add<0x128>(v); v = dpp_add<0x124>(v); v = dpp_add<0x122>(v); return dpp_add<0x121>(v);
-}
-
-// convolution + silu of channel c (column oc + c of the raw projections, ring channel hc + c) for a row `back` rows into its entry
-__device__ __forceinline__ float conv_silu(const float* cur, int64_t ldp, int back, int pos, const float* ring, int channels, int hc, const float* w, int taps, int c)
-{
-  float s = w[c * taps + taps - 1] * cur[c];
-  for (int j = 1; j < taps; j++) {
-    float x = 0.0f;
-    if (j <= back) x = cur[c - (int64_t)j * ldp];
-    else if (j <= pos) x = ring[(int64_t)((pos - j) % taps) * channels + hc + c];
-    s = fmaf(w[c * taps + taps - 1 - j], x, s);
-  }
-  return s * sigmoid_f(s);
-}
 
 // ------------------------------------------------------------------------------------------
 // prompt pass 1: q and k unit vectors (q scaled), v, decay, write strength, q . k.
@@ -51,42 +15,6 @@ __device__ __forceinline__ float conv_silu(const float* cur, int64_t ldp, int ba
 // consecutive rows; the convolution slides over them, so each input is fetched once (TAPS = 4; other lengths look back per row).
 // ------------------------------------------------------------------------------------------
 constexpr int PREP_ROWS = 8;
-
-template <int TAPS>
-struct ConvWindow {                        // four channels of a lane: c = lane + 64 i
-  float w[4][TAPS], h[4][TAPS - 1];        // taps, the inputs before the current one (h[0] the latest)
-  __device__ __forceinline__ void taps(const float* cw, int c0, int lane, int n)
-  {
-#pragma unroll
-    for (int i = 0; i < 4; i++)
-#pragma unroll
-      for (int k = 0; k < TAPS; k++) { const int c = lane + 64 * i; w[i][k] = c < n ? cw[(c0 + c) * TAPS + k] : 0.0f; }
-  }
-  __device__ __forceinline__ void history(const float* cur, int64_t ldp, int back, int pos, const float* ring, int channels, int hc, int c0, int lane, int n)
-  {
-#pragma unroll
-    for (int i = 0; i < 4; i++)
-#pragma unroll
-      for (int j = 1; j < TAPS; j++) {
-        const int c = lane + 64 * i;
-        h[i][j - 1] = 0.0f;
-        if (c < n) {
-          if (j <= back) h[i][j - 1] = cur[c0 + c - (int64_t)j * ldp];
-          else if (j <= pos) h[i][j - 1] = ring[(int64_t)((pos - j) % TAPS) * channels + hc + c0 + c];
-        }
-      }
-  }
-  __device__ __forceinline__ float step(int i, float x)
-  {
-    float s = w[i][TAPS - 1] * x;
-#pragma unroll
-    for (int j = 1; j < TAPS; j++) s = fmaf(w[i][TAPS - 1 - j], h[i][j - 1], s);
-#pragma unroll
-    for (int j = TAPS - 2; j > 0; j--) h[i][j] = h[i][j - 1];
-    h[i][0] = x;
-    return s * sigmoid_f(s);
-  }
-};
 
 template <int TAPS>
 __global__ __launch_bounds__(256) void delta_prep_kernel(const DeltaDims d, const DeltaIn in, const DeltaW w, const float* hist, const int64_t h_elems, const StepRows r, const DeltaBuf b)
@@ -795,7 +723,7 @@ __global__ __launch_bounds__(1024) void delta_single_kernel(const DeltaDims d, c
   }
 }
 
-int delta_prep(const DeltaDims& d, const DeltaIn& in, const DeltaW& w, const SeqPool::DeltaRun& st, const StepRows& r, const DeltaBuf& b)
+int delta_prep(const DeltaDims& d, const DeltaIn& in, const DeltaW& w, const SeqPool::StateRun& st, const StepRows& r, const DeltaBuf& b)
 {
   const int gw = d.channel_decay ? d.heads * d.dim : d.heads;
   const int units = d.kv_heads + (d.heads * d.vdim + 255) / 256 + (gw + 255) / 256 + 1;
@@ -806,7 +734,7 @@ int delta_prep(const DeltaDims& d, const DeltaIn& in, const DeltaW& w, const Seq
   return CAI_OK;
 }
 
-int delta_scan(const DeltaDims& d, const SeqPool::DeltaRun& st, const StepRows& r, const DeltaBuf& b)
+int delta_scan(const DeltaDims& d, const SeqPool::StateRun& st, const StepRows& r, const DeltaBuf& b)
 {
   const dim3 grid((d.vdim + 15) / 16, d.heads, r.n_ent), blk(256);
   auto s = ctx().stream;
@@ -818,7 +746,7 @@ int delta_scan(const DeltaDims& d, const SeqPool::DeltaRun& st, const StepRows& 
   return CAI_OK;
 }
 
-int delta_chunked(const DeltaDims& d, const SeqPool::DeltaRun& st, const StepRows& r, const DeltaBuf& b, const int32_t* chunks, int n_chunks, const int32_t* chunk0)
+int delta_chunked(const DeltaDims& d, const SeqPool::StateRun& st, const StepRows& r, const DeltaBuf& b, const int32_t* chunks, int n_chunks, const int32_t* chunk0)
 {
   auto s = ctx().stream;
   const size_t lds = (size_t)(d.channel_decay ? 3 : 2) * CHUNK * (((d.dim + 15) & ~15) + 4) * 4;
@@ -835,7 +763,7 @@ int delta_chunked(const DeltaDims& d, const SeqPool::DeltaRun& st, const StepRow
   return CAI_OK;
 }
 
-int delta_finish(const DeltaDims& d, const DeltaIn& in, const DeltaW& w, const SeqPool::DeltaRun& st, const StepRows& r, const DeltaBuf& b, int act_t, void* out, int64_t ldo)
+int delta_finish(const DeltaDims& d, const DeltaIn& in, const DeltaW& w, const SeqPool::StateRun& st, const StepRows& r, const DeltaBuf& b, int act_t, void* out, int64_t ldo)
 {
   if (act_t == ACT_T_BF16) hipLaunchKernelGGL(delta_finish_kernel<bf16_t>, dim3(r.n_rows), dim3(256), 0, ctx().stream, d, in, w, st.hist, st.h_elems, r, b, (bf16_t*)out, ldo);
   else hipLaunchKernelGGL(delta_finish_kernel<float>, dim3(r.n_rows), dim3(256), 0, ctx().stream, d, in, w, st.hist, st.h_elems, r, b, (float*)out, ldo);
@@ -843,7 +771,7 @@ int delta_finish(const DeltaDims& d, const DeltaIn& in, const DeltaW& w, const S
   return CAI_OK;
 }
 
-int delta_single(const DeltaDims& d, const DeltaIn& in, const DeltaW& w, const SeqPool::DeltaRun& st, const StepRows& r, int act_t, void* out, int64_t ldo)
+int delta_single(const DeltaDims& d, const DeltaIn& in, const DeltaW& w, const SeqPool::StateRun& st, const StepRows& r, int act_t, void* out, int64_t ldo)
 {
   const int ct_log = d.vdim > 64 ? 5 : d.vdim > 32 ? 4 : 3, rgs = 1024 >> ct_log, rpt = (d.dim + rgs - 1) / rgs;
   const dim3 grid(d.heads, r.n_rows), blk(1024);

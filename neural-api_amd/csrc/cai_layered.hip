@@ -4,7 +4,7 @@
 // tokens only is captured once per width as a graph and replayed.
 //
 // The residual stream is float.  A sublayer's epilogue adds its result and already leaves the next sublayer's normed input, so
-// between two mixers there are three products and nothing else.
+// between two mixers with a dense feed-forward there are three products and nothing else.
 #include "cai_layered.hpp"
 
 #include <algorithm>
@@ -31,9 +31,7 @@ int SeqPool::alloc(int n_seq_, int max_tokens, int act_t_)
     CAI_HIP(hipMalloc(&a.base, (size_t)n_pages * a.page_elems * es));
     CAI_HIP(hipMemsetAsync(a.base, 0, (size_t)n_pages * a.page_elems * es, s));
   }
-  for (auto& d : delta) {
-    d.s_elems = (int64_t)d.d.heads * d.d.dim * d.d.vdim_p();
-    d.h_elems = (int64_t)d.d.taps * d.d.channels();
+  for (auto& d : state) {
     CAI_HIP(hipMalloc((void**)&d.S, (size_t)n_seq * d.s_elems * 4));
     CAI_HIP(hipMalloc((void**)&d.hist, (size_t)n_seq * d.h_elems * 4));
     CAI_HIP(hipMemsetAsync(d.S, 0, (size_t)n_seq * d.s_elems * 4, s));
@@ -52,7 +50,7 @@ int SeqPool::alloc(int n_seq_, int max_tokens, int act_t_)
 void SeqPool::release_all()
 {
   for (auto& a : attn) { if (a.base) (void)hipFree(a.base); a.base = nullptr; }
-  for (auto& d : delta) { if (d.S) (void)hipFree(d.S); if (d.hist) (void)hipFree(d.hist); d.S = d.hist = nullptr; }
+  for (auto& d : state) { if (d.S) (void)hipFree(d.S); if (d.hist) (void)hipFree(d.hist); d.S = d.hist = nullptr; }
   if (d_table) (void)hipFree(d_table);
   d_table = nullptr;
 }
@@ -77,7 +75,9 @@ void SeqPool::trim(int s)
 {
   if (!n_pages) return;
   Seq& q = seq[s];
-  const int first = std::max(0, q.len - keep + 1) / PAGE_TOKENS;      // page of the oldest key the next token sees
+  int oldest = q.len;                                                 // the oldest key the next token sees
+  for (auto& a : attn) oldest = std::min(oldest, a.d.first_key(q.len));
+  const int first = oldest / PAGE_TOKENS;
   for (; q.first_page < std::min(first, q.end_page); q.first_page++) free_pages.push_back(table[(size_t)s * n_pages + q.first_page % n_pages]);
 }
 
@@ -123,7 +123,7 @@ int SeqPool::fork(int src, int dst)
     }
     table_dirty = true;
   }
-  for (auto& r : delta) {
+  for (auto& r : state) {
     CAI_HIP(hipMemcpyAsync(r.S + dst * r.s_elems, r.S + src * r.s_elems, (size_t)r.s_elems * 4, hipMemcpyDeviceToDevice, s));
     CAI_HIP(hipMemcpyAsync(r.hist + dst * r.h_elems, r.hist + src * r.h_elems, (size_t)r.h_elems * 4, hipMemcpyDeviceToDevice, s));
   }
@@ -141,7 +141,7 @@ KvView SeqPool::view(int run) const
 // small kernels of the step
 // ------------------------------------------------------------------------------------------
 template <typename AT>
-__global__ __launch_bounds__(256) void net_embed_kernel(const uint16_t* e, const int ld, const int32_t* tok, const int width, float* x, float* x0, AT* h, const int64_t ldh, const Dyt next)
+__global__ __launch_bounds__(256) void net_embed_kernel(const uint16_t* e, const int ld, const int32_t* tok, const int width, float* x, float* x0, AT* h, const int64_t ldh, const Dyt next, AT* cat, const int64_t ldc)
 {
   const int64_t t = blockIdx.y;
   const uint16_t* row = e + (int64_t)tok[t] * ld;
@@ -150,6 +150,7 @@ __global__ __launch_bounds__(256) void net_embed_kernel(const uint16_t* e, const
     x[t * width + i] = v;
     if (x0) x0[t * width + i] = v;
     h[t * ldh + i] = (AT)dyt(next, v, i);
+    if (cat) cat[t * ldc + i] = (AT)v;
   }
 }
 
@@ -225,11 +226,17 @@ struct LayeredNet {
   // widths over all layers
   int wp = 0, ld_proj = 0, ld_mid = 0, ld_att = 0, ld_attl = 0, ld_q = 0, ld_ra = 0, ld_rg = 0;
   int w_q = 0, w_k = 0, w_v = 0, w_g = 0, w_b = 0, w_za = 0, w_zg = 0, w_hd = 0, w_qt = 0, w_qk = 0, w_gt1 = 0;
-  bool has_attn = false, looped = false;
+  int ld_cat = 0, ld_ys = 0;
+  int64_t w_cb = 0, w_sx = 0, w_sb = 0, w_sdt = 0, w_sy = 0;                       // state-space scratch, elements per row (cb: per chunk)
+  int64_t w_ez = 0, w_ep = 0, w_emid = 0, w_emid_s = 0, w_etiles = 0;              // experts: scores, pairs, activations of a row's pairs, of the shared expert, most tiles of experts
+  bool has_parallel = false, looped = false;
   int cap = 0, logit_cap = 0;
   float *x = nullptr, *x0 = nullptr, *proj = nullptr, *yl = nullptr, *yr = nullptr, *part = nullptr, *logits = nullptr;
   void *h = nullptr, *mid = nullptr, *att = nullptr, *attl = nullptr, *qbuf = nullptr, *ra = nullptr, *rgb = nullptr, *hw = nullptr;
+  void* cat = nullptr;                     // [stream; embedding] in front of a pass
   DeltaBuf db{};
+  SsdBuf sb{};
+  ExpertBuf eb{};
   float* am_v = nullptr; int32_t* am_i = nullptr; int32_t* best = nullptr;
   int32_t* d_rows = nullptr; int32_t* h_rows = nullptr; size_t rows_cap = 0;
   int32_t* d_dec = nullptr;                // fixed row arrays of captured steps: tok, pos, slot, first, last [DEC_ROWS each], ent [4 DEC_ROWS], gen_idx
@@ -256,11 +263,13 @@ static void drop_graphs(LayeredNet* n)
 
 static void free_rows(LayeredNet* n)
 {
-  void* p[] = {n->x, n->x0, n->proj, n->yl, n->yr, n->part, n->h, n->mid, n->att, n->attl, n->qbuf, n->ra, n->rgb, n->db.q, n->db.k, n->db.v, n->db.g, n->db.beta, n->db.o, n->db.za, n->db.zg, n->db.w, n->db.qt, n->db.qk, n->db.gt};
+  void* p[] = {n->x, n->x0, n->proj, n->yl, n->yr, n->part, n->h, n->mid, n->att, n->attl, n->qbuf, n->ra, n->rgb, n->db.q, n->db.k, n->db.v, n->db.g, n->db.beta, n->db.o, n->db.za, n->db.zg, n->db.w, n->db.qt, n->db.qk, n->db.gt, n->cat,
+               n->sb.x, n->sb.B, n->sb.C, n->sb.dt, n->sb.cb, n->sb.y, n->eb.z, n->eb.wgt, n->eb.y, n->eb.ys, n->eb.sel, n->eb.order, n->eb.tiles, n->eb.n_tiles, n->eb.mid, n->eb.mid_s};
   for (void* q : p) if (q) (void)hipFree(q);
   n->x = n->x0 = n->proj = n->yl = n->yr = n->part = nullptr;
   n->h = n->mid = n->att = n->attl = n->qbuf = n->ra = n->rgb = nullptr;
-  n->db = DeltaBuf{};
+  n->cat = nullptr;
+  n->db = DeltaBuf{}; n->sb = SsdBuf{}; n->eb = ExpertBuf{};
   n->cap = 0;
 }
 
@@ -285,14 +294,21 @@ static int ensure_rows(LayeredNet* n, int rows)
   for (auto& a : n->pool.attn) part = std::max(part, attn_paged_part_floats(a.d, part_rows));
   int rc;
   if ((rc = get((void**)&n->x, R * w * 4)) || (rc = get((void**)&n->x0, n->looped ? R * w * 4 : 0)) || (rc = get((void**)&n->proj, R * n->ld_proj * 4)) ||
-      (rc = get((void**)&n->yl, n->has_attn ? R * w * 4 : 0)) || (rc = get((void**)&n->yr, n->has_attn ? R * w * 4 : 0)) || (rc = get((void**)&n->part, part * 4)) ||
+      (rc = get((void**)&n->yl, n->has_parallel ? R * w * 4 : 0)) || (rc = get((void**)&n->yr, n->has_parallel ? R * w * 4 : 0)) || (rc = get((void**)&n->part, part * 4)) ||
       (rc = get(&n->h, R * n->wp * n->es)) || (rc = get(&n->mid, R * n->ld_mid * n->es)) || (rc = get(&n->att, R * n->ld_att * n->es)) ||
       (rc = get(&n->attl, R * n->ld_attl * n->es)) || (rc = get(&n->qbuf, R * n->ld_q * n->es)) || (rc = get(&n->ra, R * n->ld_ra * n->es)) || (rc = get(&n->rgb, R * n->ld_rg * n->es)) ||
       (rc = get((void**)&n->db.q, RS * n->w_q * 4)) || (rc = get((void**)&n->db.k, RS * n->w_k * 4)) || (rc = get((void**)&n->db.v, RS * n->w_v * 4)) ||
       (rc = get((void**)&n->db.g, RS * n->w_g * 4)) || (rc = get((void**)&n->db.beta, RS * n->w_b * 4)) || (rc = get((void**)&n->db.o, RS * n->w_v * 4)) ||
       (rc = get((void**)&n->db.za, R * n->w_za * 4)) || (rc = get((void**)&n->db.zg, R * n->w_zg * 4)) ||
       (rc = get((void**)&n->db.w, RS * n->w_hd * 4)) || (rc = get((void**)&n->db.qt, RS * n->w_qt * 4)) || (rc = get((void**)&n->db.qk, RS * n->w_qk * 4)) ||
-      (rc = get((void**)&n->db.gt, std::max(RS * n->w_gt1, (R / DELTA_CHUNK + n->max_seq + 1) * n->w_qt + 4) * 4))) return rc;
+      (rc = get((void**)&n->db.gt, std::max(RS * n->w_gt1, (R / DELTA_CHUNK + n->max_seq + 1) * n->w_qt + 4) * 4)) ||
+      (rc = get(&n->cat, R * n->ld_cat * n->es)) ||
+      (rc = get((void**)&n->sb.x, R * n->w_sx * 4)) || (rc = get((void**)&n->sb.B, R * n->w_sb * 4)) || (rc = get((void**)&n->sb.C, R * n->w_sb * 4)) ||
+      (rc = get((void**)&n->sb.dt, R * n->w_sdt * 4)) || (rc = get((void**)&n->sb.cb, (R / SSD_CHUNK + n->max_seq + 1) * n->w_cb * 4)) || (rc = get((void**)&n->sb.y, R * n->w_sy * 4)) ||
+      (rc = get((void**)&n->eb.z, R * n->w_ez * 4)) || (rc = get((void**)&n->eb.sel, R * n->w_ep * 4)) || (rc = get((void**)&n->eb.wgt, R * n->w_ep * 4)) ||
+      (rc = get((void**)&n->eb.order, R * n->w_ep * 4)) || (rc = get((void**)&n->eb.y, R * n->w_ep * w * 4)) || (rc = get((void**)&n->eb.ys, R * n->ld_ys * 4)) ||
+      (rc = get((void**)&n->eb.tiles, n->w_ep ? ((R * n->w_ep + BANK_TILE - 1) / BANK_TILE + n->w_etiles) * 12 : 0)) || (rc = get((void**)&n->eb.n_tiles, n->w_ep ? 4 : 0)) ||
+      (rc = get(&n->eb.mid, R * n->w_emid * n->es)) || (rc = get(&n->eb.mid_s, R * n->w_emid_s * n->es))) return rc;
   CAI_HIP(hipStreamSynchronize(ctx().stream));
   n->cap = (int)R;
   return CAI_OK;
@@ -324,38 +340,57 @@ int net_create(NetSpec&& spec, int max_tokens, int max_seq, int act_t, LayeredNe
   n->act_t = act_t; n->es = act_t == ACT_T_BF16 ? 2 : 4; n->max_seq = max_seq;
   NetSpec& s = n->s;
   const int L = (int)s.layers.size();
-  auto add_run = [&](int l, bool again) {
-    NetRun r{l, again, -1, -1};
+  auto add_run = [&](int l, bool first, int pass) {
+    NetRun r{l, first && !s.loop_in && pass > 0, first && s.loop_in, -1, -1};
     NetLayer& y = s.layers[l];
-    if (y.kind == MIX_PARALLEL) {
+    if (y.has_attn()) {
       // (a sequence longer than the pool exists only if every window is shorter than it: a wider window sees the same keys cut down)
-      y.attn.d.window = std::min(y.attn.d.window, (max_tokens + PAGE_TOKENS - 1) / PAGE_TOKENS * PAGE_TOKENS);
-      r.attn_run = (int)n->pool.attn.size(); n->pool.attn.push_back({y.attn.d});
+      AttnDims& d = y.attn.d;
+      d.span = std::min(d.window, (max_tokens + PAGE_TOKENS - 1) / PAGE_TOKENS * PAGE_TOKENS);
+      if (!d.chunked) d.window = d.span;
+      r.attn_run = (int)n->pool.attn.size(); n->pool.attn.push_back({d});
     }
-    r.delta_run = (int)n->pool.delta.size(); n->pool.delta.push_back({y.delta.d});
+    if (y.has_delta() || y.kind == MIX_SSD) {
+      const DeltaDims& d = y.delta.d; const SsdDims& m = y.ssd.d;
+      SeqPool::StateRun st;
+      if (y.kind == MIX_SSD) { st.s_elems = (int64_t)m.heads * m.state * m.vdim_p(); st.h_elems = (int64_t)m.taps * m.channels(); }
+      else { st.s_elems = (int64_t)d.heads * d.dim * d.vdim_p(); st.h_elems = (int64_t)d.taps * d.channels(); }
+      r.state_run = (int)n->pool.state.size(); n->pool.state.push_back(st);
+    }
     n->runs.push_back(r);
   };
-  for (int l = 0; l < std::min(s.loop_start, L); l++) add_run(l, false);
+  for (int l = 0; l < std::min(s.loop_start, L); l++) add_run(l, false, 0);
   for (int p = 0; p < s.loop_times; p++)
-    for (int l = s.loop_start; l < s.loop_stop; l++) add_run(l, p > 0 && l == s.loop_start);
-  for (int l = s.loop_stop; l < L; l++) add_run(l, false);
-  n->looped = s.loop_times > 1 && s.loop_stop > s.loop_start;
+    for (int l = s.loop_start; l < s.loop_stop; l++) add_run(l, l == s.loop_start, p);
+  for (int l = s.loop_stop; l < L; l++) add_run(l, false, 0);
+  n->looped = !s.loop_in && s.loop_times > 1 && s.loop_stop > s.loop_start;
   n->wp = pad_to(s.width, LIN_PAD);
-  auto up = [](int& a, int v) { a = std::max(a, v); };
+  if (s.loop_in) n->ld_cat = pad_to(2 * s.width, LIN_PAD);
+  auto up = [](auto& a, int64_t v) { if (v > a) a = v; };
   for (const NetLayer& y : s.layers) {
-    const DeltaDims& d = y.delta.d;
     up(n->ld_proj, pad_to((int)y.in->rows, 4));
-    up(n->ld_att, pad_to(d.heads * d.vdim, LIN_PAD));
-    up(n->w_q, d.kv_heads * d.dim); up(n->w_k, d.kv_heads * d.dim); up(n->w_v, d.heads * d.vdim);
-    up(n->w_g, d.channel_decay ? d.heads * d.dim : d.heads); up(n->w_b, d.heads + d.kv_heads);
-    up(n->w_hd, d.heads * d.dim); up(n->w_qk, d.heads * DELTA_CHUNK);
-    if (d.channel_decay) up(n->w_qt, d.heads * d.dim); else up(n->w_gt1, 2 * d.heads);
-    if (d.rank_a) { up(n->ld_ra, pad_to(d.rank_a, LIN_PAD)); up(n->w_za, d.channel_decay ? d.heads * d.dim : d.heads); }
-    if (d.rank_g) { up(n->ld_rg, pad_to(d.rank_g, LIN_PAD)); up(n->w_zg, d.heads * d.vdim); }
+    if (y.has_delta()) {
+      const DeltaDims& d = y.delta.d;
+      up(n->ld_att, pad_to(d.heads * d.vdim, LIN_PAD));
+      up(n->w_q, d.kv_heads * d.dim); up(n->w_k, d.kv_heads * d.dim); up(n->w_v, d.heads * d.vdim);
+      up(n->w_g, d.channel_decay ? d.heads * d.dim : d.heads); up(n->w_b, d.heads + d.kv_heads);
+      up(n->w_hd, d.heads * d.dim); up(n->w_qk, d.heads * DELTA_CHUNK);
+      if (d.channel_decay) up(n->w_qt, d.heads * d.dim); else up(n->w_gt1, 2 * d.heads);
+      if (d.rank_a) { up(n->ld_ra, pad_to(d.rank_a, LIN_PAD)); up(n->w_za, d.channel_decay ? d.heads * d.dim : d.heads); }
+      if (d.rank_g) { up(n->ld_rg, pad_to(d.rank_g, LIN_PAD)); up(n->w_zg, d.heads * d.vdim); }
+    }
     if (y.gateup) up(n->ld_mid, pad_to(y.ff, LIN_PAD));
-    if (y.kind == MIX_PARALLEL) {
-      n->has_attn = true;
-      up(n->ld_attl, pad_to(y.attn.d.heads * y.attn.d.vdim, LIN_PAD)); up(n->ld_q, y.attn.d.heads * y.attn.d.dim_p);
+    if (y.has_attn()) { up(n->ld_attl, pad_to(y.attn.d.heads * y.attn.d.vdim, LIN_PAD)); up(n->ld_q, y.attn.d.heads * y.attn.d.dim_p); }
+    if (y.kind == MIX_PARALLEL) n->has_parallel = true;
+    if (y.kind == MIX_SSD) {
+      const SsdDims& d = y.ssd.d;
+      up(n->ld_att, pad_to(d.inner(), LIN_PAD));
+      up(n->w_sx, d.heads * d.xp()); up(n->w_sb, d.groups * d.np()); up(n->w_sdt, d.heads); up(n->w_sy, d.inner()); up(n->w_cb, d.groups * SSD_CHUNK * SSD_CHUNK);
+    }
+    if (y.experts.n) {
+      const NetExperts& x = y.experts;
+      up(n->w_ez, x.n); up(n->w_ep, x.top); up(n->w_etiles, x.n); up(n->w_emid, std::max(x.active(), x.top * x.mid_p())); up(n->w_emid_s, x.shared_p());
+      if (x.ff_shared) up(n->ld_ys, s.width);
     }
   }
   const char* ng = getenv("CAIHIP_NO_GRAPH");
@@ -388,8 +423,11 @@ void net_destroy(LayeredNet* n)
   delete n;
 }
 
-// Work lists of a step with prompt portions (device pointers; null: the forms for short portions are taken)
-struct StepLists { const int32_t* tiles = nullptr; int n_tiles = 0; const int32_t* chunks = nullptr; int n_chunks = 0; const int32_t* chunk0 = nullptr; };
+// Work lists of a step with prompt portions (device pointers): tiles of 64 rows and of DELTA_CHUNK rows (entry, first row in it), and
+// the first tile of each entry.  tall: some portion is long enough for the prompt attention kernel; chunks null: none is long enough
+// for the chunked delta rule.
+static_assert(ATTN_TILE == SSD_CHUNK, "one list of tiles serves the prompt attention and the state-space walk");
+struct StepLists { const int32_t *tiles = nullptr, *tile0 = nullptr; int n_tiles = 0; bool tall = false; const int32_t* chunks = nullptr; int n_chunks = 0; const int32_t* chunk0 = nullptr; };
 
 // One step over the rows of `r`.  single: every entry is one row (the decode kernels).  want: device list of the rows whose
 // logits are produced (null: all rows, in order).
@@ -401,56 +439,84 @@ static int enqueue_net(LayeredNet* n, const StepRows& r, bool single, const Step
   int rc;
   auto norm1_of = [&](size_t i) -> const Dyt& { return s.layers[n->runs[i].layer].norm1; };
   const dim3 eg((unsigned)std::min((w + 255) / 256, 32), R);
-  if (at == ACT_T_BF16) hipLaunchKernelGGL(net_embed_kernel<bf16_t>, eg, dim3(256), 0, st, (const uint16_t*)s.embed->data, (int)s.embed->ld, r.tok, w, n->x, n->x0, (bf16_t*)n->h, (int64_t)n->wp, norm1_of(0));
-  else hipLaunchKernelGGL(net_embed_kernel<float>, eg, dim3(256), 0, st, (const uint16_t*)s.embed->data, (int)s.embed->ld, r.tok, w, n->x, n->x0, (float*)n->h, (int64_t)n->wp, norm1_of(0));
+  // where the stream goes after the last sublayer before run i: the norm of what follows, or as it is in front of loop_in
+  auto lead_to = [&](size_t i, LinEpi& e) {
+    if (i < n->runs.size() && n->runs[i].enter) { e.next = Dyt(); e.h = n->cat; e.ldh = n->ld_cat; return; }
+    e.next = i < n->runs.size() ? norm1_of(i) : s.final_norm; e.h = n->h; e.ldh = n->wp;
+    if (i < n->runs.size() && n->runs[i].again) { e.add0 = n->x0; e.ld0 = w; }
+  };
+  LinEpi first; lead_to(0, first);
+#define EMBED(T) hipLaunchKernelGGL(net_embed_kernel<T>, eg, dim3(256), 0, st, (const uint16_t*)s.embed->data, (int)s.embed->ld, r.tok, w, n->x, n->x0, (T*)first.h, first.ldh, first.next, s.loop_in ? (T*)n->cat + w : nullptr, (int64_t)n->ld_cat)
+  if (at == ACT_T_BF16) EMBED(bf16_t); else EMBED(float);
+#undef EMBED
   for (size_t i = 0; i < n->runs.size(); i++) {
     const NetRun& run = n->runs[i];
     const NetLayer& y = s.layers[run.layer];
-    const bool last = i + 1 == n->runs.size();
-    const Dyt& after = last ? s.final_norm : norm1_of(i + 1);
-    const float* add0 = !last && n->runs[i + 1].again ? n->x0 : nullptr;
-    { LinEpi e; e.y = n->proj; e.ldy = n->ld_proj; if ((rc = launch_lin(y.in, at, n->h, n->wp, R, e))) return rc; }
-    // the recurrent mixer
-    const NetDelta& D = y.delta;
-    const DeltaIn din{n->proj, n->ld_proj, D.oq, D.ok, D.ov, D.ob, D.oa, D.og};
-    const SeqPool::DeltaRun& ds = n->pool.delta[run.delta_run];
-    if (single) {
-      if ((rc = delta_single(D.d, din, D.w, ds, r, at, n->att, n->ld_att))) return rc;
-    } else {
-      if (D.d.rank_a) {
-        LinEpi e; e.y = n->db.za; e.ldy = D.w.a2->rows;
-        if ((rc = launch_pack_rows(n->proj, n->ld_proj, D.oa, D.d.rank_a, R, at, n->ra, n->ld_ra)) || (rc = launch_lin(D.w.a2, at, n->ra, n->ld_ra, R, e))) return rc;
-      }
-      if (D.d.rank_g) {
-        LinEpi e; e.y = n->db.zg; e.ldy = D.w.g2->rows;
-        if ((rc = launch_pack_rows(n->proj, n->ld_proj, D.og, D.d.rank_g, R, at, n->rgb, n->ld_rg)) || (rc = launch_lin(D.w.g2, at, n->rgb, n->ld_rg, R, e))) return rc;
-      }
-      if ((rc = delta_prep(D.d, din, D.w, ds, r, n->db)) ||
-          (rc = lists.chunks ? delta_chunked(D.d, ds, r, n->db, lists.chunks, lists.n_chunks, lists.chunk0) : delta_scan(D.d, ds, r, n->db)) ||
-          (rc = delta_finish(D.d, din, D.w, ds, r, n->db, at, n->att, n->ld_att))) return rc;
+    if (run.enter) {
+      LinEpi e; e.mode = EPI_RESIDUAL; e.fresh = true; e.y = n->x; e.ldy = w; e.h = n->h; e.ldh = n->wp; e.next = y.norm1;
+      if ((rc = launch_lin(s.loop_in, at, n->cat, n->ld_cat, R, e))) return rc;
     }
-    LinEpi res; res.mode = EPI_RESIDUAL; res.y = n->x; res.ldy = w; res.h = n->h; res.ldh = n->wp; res.post = y.norm1b;
-    if (y.gateup) res.next = y.norm2;
-    else { res.next = after; res.add0 = add0; res.ld0 = w; }
-    if (y.kind == MIX_PARALLEL) {
+    { LinEpi e; e.y = n->proj; e.ldy = n->ld_proj; e.bias = y.in_b; if ((rc = launch_lin(y.in, at, n->h, n->wp, R, e))) return rc; }
+    LinEpi res; res.mode = EPI_RESIDUAL; res.y = n->x; res.ldy = w; res.post = y.norm1b;
+    if (y.has_mlp()) { res.next = y.norm2; res.h = n->h; res.ldh = n->wp; }
+    else lead_to(i + 1, res);
+    if (y.has_delta()) {
+      const NetDelta& D = y.delta;
+      const DeltaIn din{n->proj, n->ld_proj, D.oq, D.ok, D.ov, D.ob, D.oa, D.og};
+      const SeqPool::StateRun& ds = n->pool.state[run.state_run];
+      if (single) {
+        if ((rc = delta_single(D.d, din, D.w, ds, r, at, n->att, n->ld_att))) return rc;
+      } else {
+        if (D.d.rank_a) {
+          LinEpi e; e.y = n->db.za; e.ldy = D.w.a2->rows;
+          if ((rc = launch_pack_rows(n->proj, n->ld_proj, D.oa, D.d.rank_a, R, at, n->ra, n->ld_ra)) || (rc = launch_lin(D.w.a2, at, n->ra, n->ld_ra, R, e))) return rc;
+        }
+        if (D.d.rank_g) {
+          LinEpi e; e.y = n->db.zg; e.ldy = D.w.g2->rows;
+          if ((rc = launch_pack_rows(n->proj, n->ld_proj, D.og, D.d.rank_g, R, at, n->rgb, n->ld_rg)) || (rc = launch_lin(D.w.g2, at, n->rgb, n->ld_rg, R, e))) return rc;
+        }
+        if ((rc = delta_prep(D.d, din, D.w, ds, r, n->db)) ||
+            (rc = lists.chunks ? delta_chunked(D.d, ds, r, n->db, lists.chunks, lists.n_chunks, lists.chunk0) : delta_scan(D.d, ds, r, n->db)) ||
+            (rc = delta_finish(D.d, din, D.w, ds, r, n->db, at, n->att, n->ld_att))) return rc;
+      }
+    }
+    if (y.kind == MIX_SSD) {
+      const NetSsd& M = y.ssd;
+      const SsdIn sin{n->proj, n->ld_proj, M.oz, M.ox, M.odt};
+      const SeqPool::StateRun& ss = n->pool.state[run.state_run];
+      if (single) rc = ssd_single(M.d, sin, M.w, ss, r, n->sb);
+      else if (!(rc = ssd_prep(M.d, sin, M.w, ss, r, n->sb))) rc = ssd_walk(M.d, M.w, ss, r, n->sb, lists.tiles, lists.n_tiles, lists.tile0);
+      if (rc || (rc = ssd_finish(M.d, sin, M.w, ss, r, n->sb, single, at, n->att, n->ld_att))) return rc;
+    }
+    if (y.has_attn()) {
       const NetAttn& A = y.attn;
-      const AttnIn ain{n->proj, n->ld_proj, A.oq, A.ok, A.ov, A.qn, A.kn};
+      const AttnIn ain{n->proj, n->ld_proj, A.oq, A.ok, A.ov, A.og, A.qn, A.kn};
       const KvView kv = n->pool.view(run.attn_run);
       if (!single && (rc = attn_paged_prep(A.d, kv, at, ain, r, n->qbuf))) return rc;
-      if (!single && lists.tiles && attn_paged_prompt_ok(A.d, at)) rc = attn_paged_prompt(A.d, kv, n->qbuf, r, lists.tiles, lists.n_tiles, n->attl, n->ld_attl);
+      if (!single && lists.tall && attn_paged_prompt_ok(A.d, at)) rc = attn_paged_prompt(A.d, kv, ain, n->qbuf, r, lists.tiles, lists.n_tiles, n->attl, n->ld_attl);
       else rc = attn_paged_rows(A.d, kv, at, n->qbuf, r, n->attl, n->ld_attl, n->part, single, ain);
       if (rc) return rc;
-      LinEpi el, er; el.y = n->yl; er.y = n->yr; el.ldy = er.ldy = w;
-      if ((rc = launch_lin(A.out, at, n->attl, n->ld_attl, R, el)) || (rc = launch_lin(D.out, at, n->att, n->ld_att, R, er))) return rc;
-      if (at == ACT_T_BF16) hipLaunchKernelGGL(net_join_kernel<bf16_t>, dim3(R), dim3(1024), 0, st, n->yl, n->yr, y.gain_left, y.gain_right, w, s.eps, n->x, res.add0, res.post, res.next, (bf16_t*)n->h, (int64_t)n->wp);
-      else hipLaunchKernelGGL(net_join_kernel<float>, dim3(R), dim3(1024), 0, st, n->yl, n->yr, y.gain_left, y.gain_right, w, s.eps, n->x, res.add0, res.post, res.next, (float*)n->h, (int64_t)n->wp);
-    } else if ((rc = launch_lin(D.out, at, n->att, n->ld_att, R, res))) return rc;
-    if (y.gateup) {
-      LinEpi g; g.mode = EPI_GLU; g.h = n->mid; g.ldh = n->ld_mid; g.glu = y.glu;
-      if ((rc = launch_lin(y.gateup, at, n->h, n->wp, R, g))) return rc;
-      res.post = y.norm2b; res.next = after; res.add0 = add0; res.ld0 = w;
-      if ((rc = launch_lin(y.down, at, n->mid, n->ld_mid, R, res))) return rc;
     }
+    if (y.kind == MIX_PARALLEL) {
+      LinEpi el, er; el.y = n->yl; er.y = n->yr; el.ldy = er.ldy = w;
+      if ((rc = launch_lin(y.attn.out, at, n->attl, n->ld_attl, R, el)) || (rc = launch_lin(y.delta.out, at, n->att, n->ld_att, R, er))) return rc;
+#define JOIN(T) hipLaunchKernelGGL(net_join_kernel<T>, dim3(R), dim3(1024), 0, st, n->yl, n->yr, y.gain_left, y.gain_right, w, s.eps, n->x, res.add0, res.post, res.next, (T*)res.h, res.ldh)
+      if (at == ACT_T_BF16) JOIN(bf16_t); else JOIN(float);
+#undef JOIN
+    } else if (y.kind == MIX_ATTN) {
+      res.bias = y.attn.out_b;
+      if ((rc = launch_lin(y.attn.out, at, n->attl, n->ld_attl, R, res))) return rc;
+      res.bias = nullptr;
+    } else if ((rc = launch_lin(y.kind == MIX_SSD ? y.ssd.out : y.delta.out, at, n->att, n->ld_att, R, res))) return rc;
+    if (!y.has_mlp()) continue;
+    res.post = y.norm2b;
+    lead_to(i + 1, res);
+    if (y.experts.n) {
+      if ((rc = experts_run(y.experts, w, at, n->h, n->wp, R, n->eb, res))) return rc;
+      continue;
+    }
+    LinEpi g; g.mode = EPI_GLU; g.h = n->mid; g.ldh = n->ld_mid; g.glu = y.glu;
+    if ((rc = launch_lin(y.gateup, at, n->h, n->wp, R, g)) || (rc = launch_lin(y.down, at, n->mid, n->ld_mid, R, res))) return rc;
   }
   if (n_want > 0) {
     const void* hs = n->h;
@@ -543,15 +609,15 @@ int net_step(LayeredNet* n, int n_ent, const int32_t* seq, const int32_t* count,
     n->row_of = wrows; n->rows_gathered = false;
   } else {
     // rows, entries, tiles of the prompt attention kernel, wanted rows
-    std::vector<int32_t> tiles, chunks, chunk0;
+    std::vector<int32_t> tiles, tile0, chunks, chunk0;
     bool tall = false, chunked = false;
     for (int e = 0; e < n_ent; e++) {
       tall = tall || count[e] >= ATTN_PROMPT_MIN; chunked = chunked || count[e] >= DELTA_CHUNK_MIN;
-      chunk0.push_back((int)chunks.size() / 2);
+      chunk0.push_back((int)chunks.size() / 2); tile0.push_back((int)tiles.size() / 2);
       for (int t = 0; t < count[e]; t += ATTN_TILE) { tiles.push_back(e); tiles.push_back(t); }
       for (int t = 0; t < count[e]; t += DELTA_CHUNK) { chunks.push_back(e); chunks.push_back(t); }
     }
-    const size_t need = (size_t)5 * R + 4 * n_ent + tiles.size() + chunks.size() + chunk0.size() + W;
+    const size_t need = (size_t)5 * R + 4 * n_ent + tiles.size() + tile0.size() + chunks.size() + chunk0.size() + W;
     if (n->rows_cap < need) {
       CAI_HIP(hipStreamSynchronize(st));
       if (n->d_rows) (void)hipFree(n->d_rows);
@@ -571,15 +637,16 @@ int net_step(LayeredNet* n, int n_ent, const int32_t* seq, const int32_t* count,
     }
     int32_t* ht = ent + 4 * n_ent;
     ht = std::copy(tiles.begin(), tiles.end(), ht);
+    ht = std::copy(tile0.begin(), tile0.end(), ht);
     ht = std::copy(chunks.begin(), chunks.end(), ht);
     ht = std::copy(chunk0.begin(), chunk0.end(), ht);
     std::copy(wrows.begin(), wrows.end(), ht);
     CAI_HIP(hipMemcpyAsync(n->d_rows, hr, need * sizeof(int32_t), hipMemcpyHostToDevice, st));
     const int32_t* d = n->d_rows;
     const StepRows r{d, d + R, d + 2 * R, d + 3 * R, d + 4 * R, d + 5 * R, R, n_ent};
-    const int32_t* dt = d + 5 * R + 4 * n_ent, *dc = dt + tiles.size(), *dc0 = dc + chunks.size();
+    const int32_t* dt = d + 5 * R + 4 * n_ent, *dt0 = dt + tiles.size(), *dc = dt0 + tile0.size(), *dc0 = dc + chunks.size();
     StepLists lists;
-    if (tall) { lists.tiles = dt; lists.n_tiles = (int)tiles.size() / 2; }
+    lists.tiles = dt; lists.n_tiles = (int)tiles.size() / 2; lists.tile0 = dt0; lists.tall = tall;
     if (chunked) { lists.chunks = dc; lists.n_chunks = (int)chunks.size() / 2; lists.chunk0 = dc0; }
     if ((rc = enqueue_net(n, r, false, lists, dc0 + chunk0.size(), W))) return rc;
     for (int k = 0; k < W; k++) n->row_of.push_back(k);
@@ -678,7 +745,10 @@ int64_t net_weight_bytes(const LayeredNet* n)
   int64_t b = qb(n->s.head) + n->s.embed->algo_bytes / n->s.embed->rows + 2 * (int64_t)n->s.width * 4;
   for (const NetRun& r : n->runs) {
     const NetLayer& y = n->s.layers[r.layer];
-    b += qb(y.in) + qb(y.delta.out) + qb(y.attn.out) + qb(y.delta.w.a2) + qb(y.delta.w.g2) + qb(y.gateup) + qb(y.down) + 8 * (int64_t)n->s.width * 4;
+    const NetExperts& x = y.experts;
+    b += qb(y.in) + qb(y.delta.out) + qb(y.attn.out) + qb(y.ssd.out) + qb(y.delta.w.a2) + qb(y.delta.w.g2) + qb(y.gateup) + qb(y.down) + 8 * (int64_t)n->s.width * 4;
+    if (r.enter) b += qb(n->s.loop_in);
+    if (x.n) b += qb(x.router) + qb(x.s_gateup) + qb(x.s_down) + (qb(x.gateup) + qb(x.down)) / x.n * x.top;   // (of one token)
   }
   return b;
 }
@@ -687,14 +757,14 @@ int64_t net_weight_bytes(const LayeredNet* n)
 // snapshots: live pages and state of one sequence
 // ------------------------------------------------------------------------------------------
 struct NetSnap {
-  int len = 0, first_page = 0, end_page = 0, n_attn = 0, n_delta = 0; int64_t bytes = 0;
+  int len = 0, first_page = 0, end_page = 0, n_attn = 0, n_state = 0; int64_t bytes = 0;
   char* data = nullptr;
 };
 static int64_t snap_bytes(const LayeredNet* n, int pages)
 {
   int64_t b = 0;
   for (auto& a : n->pool.attn) b += pages * a.page_elems * (int64_t)n->es;
-  for (auto& d : n->pool.delta) b += (d.s_elems + d.h_elems) * 4;
+  for (auto& d : n->pool.state) b += (d.s_elems + d.h_elems) * 4;
   return b;
 }
 // walks the pieces of a sequence in snapshot order: f(device pointer, bytes, offset)
@@ -708,7 +778,7 @@ template <typename F> static int snap_walk(LayeredNet* n, int seq, F f)
       if ((rc = f((char*)a.base + n->pool.table[(size_t)seq * n->pool.n_pages + p % n->pool.n_pages] * sz, sz, off))) return rc;
       off += sz;
     }
-  for (auto& d : n->pool.delta) {
+  for (auto& d : n->pool.state) {
     if ((rc = f((char*)(d.S + seq * d.s_elems), (size_t)d.s_elems * 4, off))) return rc;
     off += d.s_elems * 4;
     if ((rc = f((char*)(d.hist + seq * d.h_elems), (size_t)d.h_elems * 4, off))) return rc;
@@ -720,7 +790,7 @@ int net_snapshot(LayeredNet* n, int seq, NetSnap** out)
 {
   const auto& q = n->pool.seq[seq];
   NetSnap* s = new NetSnap();
-  s->len = q.len; s->first_page = q.first_page; s->end_page = q.end_page; s->n_attn = (int)n->pool.attn.size(); s->n_delta = (int)n->pool.delta.size();
+  s->len = q.len; s->first_page = q.first_page; s->end_page = q.end_page; s->n_attn = (int)n->pool.attn.size(); s->n_state = (int)n->pool.state.size();
   s->bytes = snap_bytes(n, q.end_page - q.first_page);
   if (hipMalloc((void**)&s->data, (size_t)s->bytes) != hipSuccess) { (void)hipGetLastError(); delete s; return set_error(CAI_ERR_NOMEM, "snapshot: out of device memory (a sequence of %d tokens)", q.len); }
   const int rc = snap_walk(n, seq, [&](char* p, size_t sz, int64_t off) -> int { CAI_HIP(hipMemcpyAsync(s->data + off, p, sz, hipMemcpyDeviceToDevice, ctx().stream)); return CAI_OK; });
@@ -732,7 +802,7 @@ int net_snapshot(LayeredNet* n, int seq, NetSnap** out)
 int net_restore(LayeredNet* n, int seq, const NetSnap* s)
 {
   const int pages = s->end_page - s->first_page;
-  CAI_REQUIRE(s->n_attn == (int)n->pool.attn.size() && s->n_delta == (int)n->pool.delta.size() && s->bytes == snap_bytes(n, pages), "restore: the snapshot is of another model");
+  CAI_REQUIRE(s->n_attn == (int)n->pool.attn.size() && s->n_state == (int)n->pool.state.size() && s->bytes == snap_bytes(n, pages), "restore: the snapshot is of another model");
   n->pool.free_seq(seq);
   auto& q = n->pool.seq[seq];
   q.first_page = q.end_page = s->first_page;

@@ -1,5 +1,5 @@
-// Declarations shared by the layered-decoder translation units: 16-bit weights, paged cache and state slots, the gated delta
-// rule, windowed attention over pages (gfx950 only).
+// Declarations shared by the layered-decoder translation units: 16-bit weights, paged cache and state slots, recurrent mixers (the
+// gated delta rule, state-space duality), attention over pages, mixtures of experts (gfx950 only).
 #pragma once
 #include "cai_internal.hpp"
 
@@ -27,14 +27,17 @@ __device__ __forceinline__ float dyt(const Dyt& t, float x, int i) { return t.w 
 
 // What a linear layer does with its finished sums.
 enum { EPI_STORE = 0, EPI_GLU = 1, EPI_RESIDUAL = 2 };
-enum { GLU_RELU = 0, GLU_SILU = 1 };
+// Gated pairs: relu(g) u;  silu(g) u;  gelu(g) u, tanh form;  with g = min(gate, limit) and u = clamp(up, -limit, limit):
+// g sigmoid(1.702 g) (u + 1)
+enum { GLU_RELU = 0, GLU_SILU = 1, GLU_GELU_TANH = 2, GLU_CLAMPED = 3 };
 struct LinEpi {
   int mode = EPI_STORE;
   float* y = nullptr; int64_t ldy = 0;              // STORE: result; RESIDUAL: the residual stream, updated in place
   void* h = nullptr; int64_t ldh = 0;               // GLU: act(gate) * up; RESIDUAL: input of the next sublayer (null: none)
   const float* add0 = nullptr; int64_t ld0 = 0;     // RESIDUAL: added to the stream after the sum (start of a repeated pass)
-  const float* bias = nullptr; int act = CAI_ACT_NONE;   // STORE
-  int glu = GLU_RELU;
+  const float* bias = nullptr; int act = CAI_ACT_NONE;   // STORE: act(sum + bias); RESIDUAL: the sum includes it
+  int glu = GLU_RELU; float limit = 0.0f;
+  bool fresh = false;                               // RESIDUAL: x = post(sum) instead of x += post(sum)
   Dyt post, next;                                   // RESIDUAL: x += post(sum) [+ add0]; h = next(x)
 };
 // Gated matrices interleave their rows in blocks of 16: 16 gate rows, then the 16 up rows of the same outputs.
@@ -42,6 +45,12 @@ __host__ __device__ inline int glu_row(int j, int up) { return (j >> 4) * 32 + u
 
 // y = W x for n_tok activation rows x[t][ldx] (zero padded to LIN_PAD columns, element type act_t); W is a CAI_BF16 matrix.
 int launch_lin(const cai_qw_s* w, int act_t, const void* x, int64_t ldx, int n_tok, const LinEpi& e);
+// The same over a bank of equal matrices stacked in w (mat_rows rows each): work lists of (matrix, first place, places) over an order
+// of activation rows.  Place p reads activation row order[p] / div (div 0: row p) and writes row p of e.h, scaled by
+// scale[order[p]] (GLU), or row order[p] of e.y (STORE).
+constexpr int BANK_TILE = 64;
+struct BankList { const int32_t *tiles, *n_tiles, *order; const float* scale; int div, max_tiles; };   // tiles [.][3], n_tiles on the device
+int launch_lin_bank(const cai_qw_s* w, int mat_rows, int act_t, const void* x, int64_t ldx, const BankList& l, const LinEpi& e);
 // float columns [col0, col0 + cols) of x -> rows of the chosen type, zero padded to ldo
 int launch_pack_rows(const float* x, int64_t ldx, int64_t col0, int cols, int n_tok, int act_t, void* out, int64_t ldo);
 int bf16_dequant_rows(const cai_qw_s* w, int64_t row0, int64_t n_rows, float* out);
@@ -69,6 +78,10 @@ constexpr int PAGE_TOKENS = 64;
 struct AttnDims {
   int heads, kv_heads, dim, vdim, window; float scale, eps;
   int dim_p, vdim_p;                       // row strides in the pool: padded to 8 elements (zero filled)
+  int chunked;                             // window is the size of fixed blocks of positions: a token sees its own block up to itself
+  int rot; const double* turns;            // the first rot dimensions turn, i with i + rot / 2, by turns[i] full turns a position (0: none)
+  int span;                                // most keys a token sees
+  __host__ __device__ int first_key(int pos) const { return chunked ? pos / window * window : pos >= window ? pos - window + 1 : 0; }
 };
 struct DeltaDims {
   int heads, kv_heads, dim, vdim, taps; float eps;
@@ -78,22 +91,31 @@ struct DeltaDims {
   __host__ __device__ int channels() const { return 2 * kv_heads * dim + heads * vdim; }
   __host__ __device__ int vdim_p() const { return (vdim + 3) & ~3; }   // row stride of the state
 };
+// State-space duality: heads of [state][vdim], groups of heads that share B and C; one convolution over x | B | C.
+struct SsdDims {
+  int heads, vdim, state, groups, taps, norm_groups; float eps;
+  __host__ __device__ int inner() const { return heads * vdim; }
+  __host__ __device__ int channels() const { return heads * vdim + 2 * groups * state; }
+  __host__ __device__ int vdim_p() const { return (vdim + 3) & ~3; }   // row stride of the state
+  __host__ __device__ int np() const { return (state + 15) & ~15; }    // strides of the prompt buffers (zero filled)
+  __host__ __device__ int xp() const { return (vdim + 15) & ~15; }
+};
 struct KvView {                            // what a kernel needs to reach one attention run's pages
   void* base; int64_t page_elems;          // K [kv_head][PAGE_TOKENS][dim_p] then V [kv_head][PAGE_TOKENS][vdim_p]
   const int32_t* table; int ring;          // [slot][ring]
   int64_t v_off;                           // elements from a page's K to its V
 };
 struct SeqPool {
-  int n_seq = 0, n_pages = 0, act_t = ACT_T_BF16, keep = 0;   // keep: the widest window (0: no attention run)
+  int n_seq = 0, n_pages = 0, act_t = ACT_T_BF16, keep = 0;   // keep: the widest window or block (0: no attention run)
   struct AttnRun { AttnDims d; void* base = nullptr; int64_t page_elems = 0, v_off = 0; };
-  struct DeltaRun { DeltaDims d; float* S = nullptr; float* hist = nullptr; int64_t s_elems = 0, h_elems = 0; };
-  std::vector<AttnRun> attn; std::vector<DeltaRun> delta;
+  struct StateRun { int64_t s_elems = 0, h_elems = 0; float* S = nullptr; float* hist = nullptr; };   // state and convolution inputs of one sequence
+  std::vector<AttnRun> attn; std::vector<StateRun> state;
   int32_t* d_table = nullptr; std::vector<int32_t> table; bool table_dirty = false;
   std::vector<int> free_pages;
   struct Seq { int len = 0; int first_page = 0, end_page = 0; };   // live pages [first_page, end_page)
   std::vector<Seq> seq;
 
-  int alloc(int n_seq, int max_tokens, int act_t);        // after attn / delta list their runs
+  int alloc(int n_seq, int max_tokens, int act_t);        // after attn / state list their runs
   void release_all();
   int reserve(int s, int new_len);                        // pages for positions [.., new_len)
   void trim(int s);                                       // hands back the pages no window reaches any more
@@ -104,15 +126,16 @@ struct SeqPool {
   KvView view(int run) const;
 };
 
-// ---- windowed grouped attention over pages (cai_attn_paged.hip) ----
+// ---- grouped attention over pages, in a sliding window or in fixed blocks (cai_attn_paged.hip) ----
 // rows of proj: q at column oq ([heads][dim]), k at ok, v at ov.  Queries and keys are RMS-normed per head over dim with a
-// shared gain before the score (gain null: not).
-struct AttnIn { const float* proj; int64_t ldp; int oq, ok, ov; const float *qn, *kn; };
+// shared gain before the rotation and the score (gain null: not).  og >= 0: the heads' outputs are multiplied by the sigmoid of
+// the columns from og on ([heads][vdim]).
+struct AttnIn { const float* proj; int64_t ldp; int oq, ok, ov, og; const float *qn, *kn; };
 int attn_paged_prep(const AttnDims& d, const KvView& kv, int act_t, const AttnIn& in, const StepRows& r, void* qbuf);     // norms + append; qbuf [row][heads][dim_p]
 int attn_paged_rows(const AttnDims& d, const KvView& kv, int act_t, const void* qbuf, const StepRows& r, void* out, int64_t ldo, float* part, bool single, const AttnIn& in);
 size_t attn_paged_part_floats(const AttnDims& d, int n_rows);
 bool attn_paged_prompt_ok(const AttnDims& d, int act_t);
-int attn_paged_prompt(const AttnDims& d, const KvView& kv, const void* qbuf, const StepRows& r, const int32_t* tiles, int n_tiles, void* out, int64_t ldo);
+int attn_paged_prompt(const AttnDims& d, const KvView& kv, const AttnIn& in, const void* qbuf, const StepRows& r, const int32_t* tiles, int n_tiles, void* out, int64_t ldo);
 constexpr int ATTN_PROMPT_MIN = 16;        // portions from here on make a step take the prompt kernel
 constexpr int ATTN_TILE = 64;              // query rows of one entry per work-group of the prompt kernel
 
@@ -131,31 +154,71 @@ struct DeltaBuf {                          // per-row scratch of a prompt pass
 };
 constexpr int DELTA_CHUNK = 16;            // tokens per chunk
 constexpr int DELTA_CHUNK_MIN = 32;        // portions from here on make a step take the chunked form
-int delta_prep(const DeltaDims& d, const DeltaIn& in, const DeltaW& w, const SeqPool::DeltaRun& st, const StepRows& r, const DeltaBuf& b);
-int delta_scan(const DeltaDims& d, const SeqPool::DeltaRun& st, const StepRows& r, const DeltaBuf& b);
-int delta_chunked(const DeltaDims& d, const SeqPool::DeltaRun& st, const StepRows& r, const DeltaBuf& b, const int32_t* chunks, int n_chunks, const int32_t* chunk0);   // chunks: entry, first row in it; chunk0: first chunk of each entry
-int delta_finish(const DeltaDims& d, const DeltaIn& in, const DeltaW& w, const SeqPool::DeltaRun& st, const StepRows& r, const DeltaBuf& b, int act_t, void* out, int64_t ldo);
-int delta_single(const DeltaDims& d, const DeltaIn& in, const DeltaW& w, const SeqPool::DeltaRun& st, const StepRows& r, int act_t, void* out, int64_t ldo);
+int delta_prep(const DeltaDims& d, const DeltaIn& in, const DeltaW& w, const SeqPool::StateRun& st, const StepRows& r, const DeltaBuf& b);
+int delta_scan(const DeltaDims& d, const SeqPool::StateRun& st, const StepRows& r, const DeltaBuf& b);
+int delta_chunked(const DeltaDims& d, const SeqPool::StateRun& st, const StepRows& r, const DeltaBuf& b, const int32_t* chunks, int n_chunks, const int32_t* chunk0);   // chunks: entry, first row in it; chunk0: first chunk of each entry
+int delta_finish(const DeltaDims& d, const DeltaIn& in, const DeltaW& w, const SeqPool::StateRun& st, const StepRows& r, const DeltaBuf& b, int act_t, void* out, int64_t ldo);
+int delta_single(const DeltaDims& d, const DeltaIn& in, const DeltaW& w, const SeqPool::StateRun& st, const StepRows& r, int act_t, void* out, int64_t ldo);
+
+// ---- state-space duality (cai_ssd.hip) ----
+// Columns of proj: z, x | B | C (before the convolution), dt.
+struct SsdIn { const float* proj; int64_t ldp; int oz, ox, odt; };
+struct SsdW { const float *conv, *conv_b, *dt_bias, *rate, *D, *norm; };   // taps [channels][taps]; rate = -exp(A_log)
+struct SsdBuf { float *x, *B, *C, *dt, *cb, *y; };                          // per-row scratch; cb: C B^T of every chunk and group
+constexpr int SSD_CHUNK = 64;
+int ssd_prep(const SsdDims& d, const SsdIn& in, const SsdW& w, const SeqPool::StateRun& st, const StepRows& r, const SsdBuf& b);
+int ssd_walk(const SsdDims& d, const SsdW& w, const SeqPool::StateRun& st, const StepRows& r, const SsdBuf& b, const int32_t* chunks, int n_chunks, const int32_t* chunk0);
+int ssd_single(const SsdDims& d, const SsdIn& in, const SsdW& w, const SeqPool::StateRun& st, const StepRows& r, const SsdBuf& b);
+int ssd_finish(const SsdDims& d, const SsdIn& in, const SsdW& w, const SeqPool::StateRun& st, const StepRows& r, const SsdBuf& b, bool single, int act_t, void* out, int64_t ldo);
+
+// ---- mixtures of experts over bfloat16 weights (cai_experts.hip) ----
+// Soft-max scores over all experts; the `top` largest of score + correction are chosen; their weights are the scores over their sum,
+// times scale.  A shared expert may run for every token beside them.
+struct NetExperts {
+  int n = 0, top = 0, ff = 0, ff_shared = 0, glu = GLU_CLAMPED, glu_shared = GLU_CLAMPED;   // ff_shared 0: no shared expert
+  float scale = 1.0f, limit = 0.0f, limit_shared = 0.0f;
+  cai_qw_s *router = nullptr, *gateup = nullptr, *down = nullptr, *s_gateup = nullptr, *s_down = nullptr;   // gateup, down: banks
+  const float* correction = nullptr;       // [n], may be null
+  int gu_rows() const { return pad_to(ff, 16) * 2; }
+  int mid_p() const { return pad_to(ff, LIN_PAD); }
+  int shared_p() const { return ff_shared ? pad_to(ff_shared, LIN_PAD) : 0; }
+  int active() const { return top * mid_p() + shared_p(); }            // a row's gated activations, one slot after the other
+  int max_tiles(int rows) const { return (rows * top + BANK_TILE - 1) / BANK_TILE + n; }
+};
+constexpr int EXPERTS_MAX = 512, EXPERTS_TOP = 64;
+constexpr int EXPERTS_FEW = 8;             // up to so many rows take the gathering kernels
+struct ExpertBuf {
+  float *z, *wgt, *y, *ys; int32_t *sel, *order, *tiles, *n_tiles; void *mid, *mid_s;
+};
+int experts_run(const NetExperts& x, int width, int act_t, const void* h, int64_t ldh, int n_rows, const ExpertBuf& b, const LinEpi& res);   // res: the residual update
 
 // ------------------------------------------------------------------------------------------
 // The layered decoder (cai_layered.hip): layers of different kinds, some run several times.
 // ------------------------------------------------------------------------------------------
 struct NetDelta { DeltaDims d{}; DeltaW w{}; int oq = 0, ok = 0, ov = 0, ob = 0, oa = 0, og = 0; cai_qw_s* out = nullptr; };
-struct NetAttn { AttnDims d{}; const float *qn = nullptr, *kn = nullptr; int oq = 0, ok = 0, ov = 0; cai_qw_s* out = nullptr; };
-enum { MIX_DELTA = 0, MIX_PARALLEL = 1 };
+struct NetAttn { AttnDims d{}; const float *qn = nullptr, *kn = nullptr, *out_b = nullptr; int oq = 0, ok = 0, ov = 0, og = -1; cai_qw_s* out = nullptr; };
+struct NetSsd { SsdDims d{}; SsdW w{}; int oz = 0, ox = 0, odt = 0; cai_qw_s* out = nullptr; };
+enum { MIX_DELTA = 0, MIX_PARALLEL = 1, MIX_ATTN = 2, MIX_SSD = 3 };   // PARALLEL: attention and a delta rule side by side
 struct NetLayer {
   int kind = MIX_DELTA;
   cai_qw_s* in = nullptr;                  // every projection of the layer's input, stacked
-  NetDelta delta; NetAttn attn;            // PARALLEL: both
+  const float* in_b = nullptr;             // its bias (null: none)
+  NetDelta delta; NetAttn attn; NetSsd ssd;
   const float *gain_left = nullptr, *gain_right = nullptr;   // PARALLEL: gains of the two outputs' RMS norms
   Dyt norm1, norm1b, norm2, norm2b;
-  cai_qw_s *gateup = nullptr, *down = nullptr; int ff = 0, glu = GLU_RELU;   // gateup null: no feed-forward
+  cai_qw_s *gateup = nullptr, *down = nullptr; int ff = 0, glu = GLU_RELU;   // gateup null: no dense feed-forward
+  NetExperts experts;                      // n > 0: the feed-forward is a mixture
+  bool has_delta() const { return kind == MIX_DELTA || kind == MIX_PARALLEL; }
+  bool has_attn() const { return kind == MIX_ATTN || kind == MIX_PARALLEL; }
+  bool has_mlp() const { return gateup || experts.n > 0; }
 };
-struct NetRun { int layer; bool again; int attn_run, delta_run; };   // again: the embedding output is added before this run
+// again: the embedding output is added before this run; enter: the stream is replaced by loop_in [stream; embedding output] before it
+struct NetRun { int layer; bool again, enter; int attn_run, state_run; };
 struct LayeredNet;
 struct NetSpec {                           // filled by a loader
   int width = 0, vocab = 0; float eps = 0.0f;
   cai_qw_s *embed = nullptr, *head = nullptr;
+  cai_qw_s* loop_in = nullptr;             // in front of every pass of the repeated stretch (null: the embedding output is added from the second pass on)
   Dyt final_norm;
   std::vector<NetLayer> layers;
   int loop_start = 0, loop_stop = 0, loop_times = 1;

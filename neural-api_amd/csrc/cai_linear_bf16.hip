@@ -5,35 +5,13 @@
 // 32-bit sums) or float; with float activations the weights are widened exactly and every product and sum is 32-bit (the
 // 16x16x4 float form of the matrix cores).  What follows the product runs in its epilogue on the 32-bit sums: bias and
 // activation, act(gate) * up of a gated pair, or the residual update with the Dynamic Tanh before and after it - that norm
-// has no statistics, so a sublayer needs no launch besides its products and its mixer.
-#include "cai_layered.hpp"
-#include "cai_gemv_common.hpp"
+// has no statistics, so a sublayer needs no launch besides its products and its mixer.  The matrix-core kernel also runs over a
+// bank of equal matrices with a list of activation rows for each (mixtures of experts).
+#include "cai_lin_epilogue.hpp"
 
 #include <algorithm>
 
 namespace cai {
-
-__device__ __forceinline__ float glu_act(float g, int kind) { return kind == GLU_SILU ? silu_mul(1.0f, g) : fmaxf(g, 0.0f); }
-
-template <typename AT> __device__ __forceinline__ void put_act(void* p, int64_t i, float v)
-{
-  if constexpr (sizeof(AT) == 2) reinterpret_cast<uint16_t*>(p)[i] = bf16_bits(v);
-  else reinterpret_cast<float*>(p)[i] = v;
-}
-
-// one finished sum of STORE / RESIDUAL
-template <typename AT> __device__ __forceinline__ void epi_one(const LinEpi& e, int n, int t, float v)
-{
-  if (e.mode == EPI_STORE) {
-    if (e.bias) v += e.bias[n];
-    e.y[t * e.ldy + n] = act_apply(v, e.act);
-  } else {
-    float x = e.y[t * e.ldy + n] + dyt(e.post, v, n);
-    if (e.add0) x += e.add0[t * e.ld0 + n];
-    e.y[t * e.ldy + n] = x;
-    if (e.h) put_act<AT>(e.h, t * e.ldh + n, dyt(e.next, x, n));
-  }
-}
 
 // ------------------------------------------------------------------------------------------
 // Decode: NB activation rows.  A wave owns R weight rows (of a gated matrix R / 2 outputs) or, with ksplit > 1, every ksplit-th
@@ -140,7 +118,7 @@ __global__ __launch_bounds__(64 * GV_WAVES) void gemv_bf16(const uint16_t* __res
   if (glu) {
     const float up = __shfl(mine, lane + R / 2 * NB);
     const int j = grp * (R / 2) + i;
-    if (i < R / 2 && glu_row(j, 0) < n_rows) put_act<AT>(e.h, b * e.ldh + j, glu_act(mine, e.glu) * up);
+    if (i < R / 2 && glu_row(j, 0) < n_rows) put_act<AT>(e.h, b * e.ldh + j, glu_pair(e.glu, e.limit, mine, up));
   } else if (i < R && grp * R + i < n_rows) epi_one<AT>(e, grp * R + i, b, mine);
 }
 
@@ -149,8 +127,8 @@ __global__ __launch_bounds__(64 * GV_WAVES) void gemv_bf16(const uint16_t* __res
 // Both operand tiles are 128 bytes deep per row (64 bfloat16 or 32 floats), double buffered in LDS; the 16-byte chunks of a row
 // are stored at chunk ^ (row & 7), which makes the fragment reads conflict-free.
 // ------------------------------------------------------------------------------------------
-template <typename AT, int BM, int BN, int WM, int WN>
-__global__ __launch_bounds__(64 * WM * WN) void gemm_bf16(const uint16_t* __restrict__ W, const AT* __restrict__ X, int n_rows, int ldw, int64_t ldx, int n_tok, int tiles_m, int n_tiles, LinEpi e)
+template <typename AT, int BM, int BN, int WM, int WN, bool BANK>
+__global__ __launch_bounds__(64 * WM * WN) void gemm_bf16(const uint16_t* __restrict__ W, const AT* __restrict__ X, int n_rows, int ldw, int64_t ldx, int n_tok, int tiles_m, int n_tiles, LinEpi e, BankList l)
 {
   constexpr int NT = 64 * WM * WN;
   constexpr int BK = 128 / (int)sizeof(AT);          // elements per row of a tile
@@ -165,12 +143,25 @@ __global__ __launch_bounds__(64 * WM * WN) void gemm_bf16(const uint16_t* __rest
     const int xcd = blockIdx.x & 7, per = n_tiles >> 3, rem = n_tiles & 7;
     tile = xcd * per + min(xcd, rem) + (blockIdx.x >> 3);
   }
-  const int m0 = tile % tiles_m * BM, n0 = tile / tiles_m * BN;
+  int m0 = tile % tiles_m * BM;
+  const int n0 = tile / tiles_m * BN;
+  if constexpr (BANK) {                    // n_rows: of one matrix; the token tile is a run of places of the order
+    const int tm = tile % tiles_m;
+    if (tm >= *l.n_tiles) return;
+    const int32_t* tl = l.tiles + 3 * tm;
+    W += (int64_t)tl[0] * n_rows * ldw;
+    m0 = tl[1]; n_tok = m0 + tl[2];
+  }
   const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int wm = wave / WN * (BM / WM), wn = wave % WN * (BN / WN);
   const AT* xp[CA]; const uint16_t* wp[CW];
 #pragma unroll
-  for (int i = 0; i < CA; i++) { const int c = tid + i * NT; xp[i] = X + (int64_t)min(m0 + (c >> 3), n_tok - 1) * ldx + (c & 7) * (16 / sizeof(AT)); }
+  for (int i = 0; i < CA; i++) {
+    const int c = tid + i * NT;
+    int t = min(m0 + (c >> 3), n_tok - 1);
+    if constexpr (BANK) { if (l.div) t = l.order[t] / l.div; }
+    xp[i] = X + (int64_t)t * ldx + (c & 7) * (16 / sizeof(AT));
+  }
 #pragma unroll
   for (int i = 0; i < CW; i++) { const int c = tid + i * NT; wp[i] = W + (int64_t)min(n0 + (c >> 3), n_rows - 1) * ldw + (c & 7) * (16 / sizeof(AT)); }
   u32x4 rx[CA], rw[CW];
@@ -230,8 +221,13 @@ __global__ __launch_bounds__(64 * WM * WN) void gemm_bf16(const uint16_t* __rest
   }
 #pragma unroll
   for (int i = 0; i < TM; i++) {
-    const int t = m0 + wm + i * 16 + fr;
+    int t = m0 + wm + i * 16 + fr;
     if (t >= n_tok) continue;
+    float scale = 1.0f;
+    if constexpr (BANK) {
+      const int at = l.order[t];
+      if (e.mode == EPI_GLU) scale = l.scale[at]; else t = at;
+    }
     if (e.mode == EPI_GLU) {
 #pragma unroll
       for (int j = 0; j < TN; j += 2) {
@@ -240,10 +236,14 @@ __global__ __launch_bounds__(64 * WM * WN) void gemm_bf16(const uint16_t* __rest
         const int o = (n >> 1) + fc * 4;
         float v[4];
 #pragma unroll
-        for (int q = 0; q < 4; q++) v[q] = glu_act(acc[j][i][q], e.glu) * acc[j + 1][i][q];
+        for (int q = 0; q < 4; q++) v[q] = glu_pair(e.glu, e.limit, acc[j][i][q], acc[j + 1][i][q]);
+        if constexpr (BANK) {
+#pragma unroll
+          for (int q = 0; q < 4; q++) v[q] *= scale;
+        }
         if constexpr (sizeof(AT) == 2)
-          *reinterpret_cast<uint2*>(reinterpret_cast<uint16_t*>(e.h) + t * e.ldh + o) = make_uint2(bf16_bits(v[0]) | (uint32_t)bf16_bits(v[1]) << 16, bf16_bits(v[2]) | (uint32_t)bf16_bits(v[3]) << 16);
-        else *reinterpret_cast<f32x4*>(reinterpret_cast<float*>(e.h) + t * e.ldh + o) = f32x4{v[0], v[1], v[2], v[3]};
+          *reinterpret_cast<uint2*>(reinterpret_cast<uint16_t*>(e.h) + (int64_t)t * e.ldh + o) = make_uint2(bf16_bits(v[0]) | (uint32_t)bf16_bits(v[1]) << 16, bf16_bits(v[2]) | (uint32_t)bf16_bits(v[3]) << 16);
+        else *reinterpret_cast<f32x4*>(reinterpret_cast<float*>(e.h) + (int64_t)t * e.ldh + o) = f32x4{v[0], v[1], v[2], v[3]};
       }
       continue;
     }
@@ -252,7 +252,7 @@ __global__ __launch_bounds__(64 * WM * WN) void gemm_bf16(const uint16_t* __rest
       const int n = n0 + wn + j * 16 + fc * 4;
       if (n >= n_rows) continue;
       if (n + 3 < n_rows && (e.ldy & 3) == 0 && (e.ldh & 3) == 0 && (e.ld0 & 3) == 0) {
-        f32x4* yp = reinterpret_cast<f32x4*>(e.y + t * e.ldy + n);
+        f32x4* yp = reinterpret_cast<f32x4*>(e.y + (int64_t)t * e.ldy + n);
         f32x4 v = acc[j][i];
         if (e.mode == EPI_STORE) {
           if (e.bias || e.act != CAI_ACT_NONE) {
@@ -261,17 +261,19 @@ __global__ __launch_bounds__(64 * WM * WN) void gemm_bf16(const uint16_t* __rest
           }
           *yp = v;
         } else {
-          f32x4 x = *yp;
+          f32x4 x = {0.0f, 0.0f, 0.0f, 0.0f};
+          if (!e.fresh) x = *yp;
+          if (e.bias) v += f32x4{e.bias[n], e.bias[n + 1], e.bias[n + 2], e.bias[n + 3]};
 #pragma unroll
           for (int q = 0; q < 4; q++) x[q] += dyt(e.post, v[q], n + q);
-          if (e.add0) x += *reinterpret_cast<const f32x4*>(e.add0 + t * e.ld0 + n);
+          if (e.add0) x += *reinterpret_cast<const f32x4*>(e.add0 + (int64_t)t * e.ld0 + n);
           *yp = x;
           if (e.h) {
 #pragma unroll
             for (int q = 0; q < 4; q++) v[q] = dyt(e.next, x[q], n + q);
             if constexpr (sizeof(AT) == 2)
-              *reinterpret_cast<uint2*>(reinterpret_cast<uint16_t*>(e.h) + t * e.ldh + n) = make_uint2(bf16_bits(v[0]) | (uint32_t)bf16_bits(v[1]) << 16, bf16_bits(v[2]) | (uint32_t)bf16_bits(v[3]) << 16);
-            else *reinterpret_cast<f32x4*>(reinterpret_cast<float*>(e.h) + t * e.ldh + n) = v;
+              *reinterpret_cast<uint2*>(reinterpret_cast<uint16_t*>(e.h) + (int64_t)t * e.ldh + n) = make_uint2(bf16_bits(v[0]) | (uint32_t)bf16_bits(v[1]) << 16, bf16_bits(v[2]) | (uint32_t)bf16_bits(v[3]) << 16);
+            else *reinterpret_cast<f32x4*>(reinterpret_cast<float*>(e.h) + (int64_t)t * e.ldh + n) = v;
           }
         }
       } else {
@@ -286,8 +288,26 @@ template <typename AT, int BM, int BN, int WM, int WN>
 static void run_gemm(const cai_qw_s* w, const AT* x, int64_t ldx, int n_tok, const LinEpi& e)
 {
   const int tm = (n_tok + BM - 1) / BM, tn = ((int)w->rows + BN - 1) / BN;
-  hipLaunchKernelGGL((gemm_bf16<AT, BM, BN, WM, WN>), dim3(tm * tn), dim3(64 * WM * WN), 0, ctx().stream,
-                     (const uint16_t*)w->data, x, (int)w->rows, (int)w->ld, ldx, n_tok, tm, tm * tn, e);
+  hipLaunchKernelGGL((gemm_bf16<AT, BM, BN, WM, WN, false>), dim3(tm * tn), dim3(64 * WM * WN), 0, ctx().stream,
+                     (const uint16_t*)w->data, x, (int)w->rows, (int)w->ld, ldx, n_tok, tm, tm * tn, e, BankList{});
+}
+
+template <typename AT>
+static void run_bank(const cai_qw_s* w, int mat_rows, const AT* x, int64_t ldx, const BankList& l, const LinEpi& e)
+{
+  const int tm = l.max_tiles, tn = (mat_rows + 63) / 64;
+  hipLaunchKernelGGL((gemm_bf16<AT, BANK_TILE, 64, 2, 2, true>), dim3(tm * tn), dim3(256), 0, ctx().stream,
+                     (const uint16_t*)w->data, x, mat_rows, (int)w->ld, ldx, 0, tm, tm * tn, e, l);
+}
+
+int launch_lin_bank(const cai_qw_s* w, int mat_rows, int act_t, const void* x, int64_t ldx, const BankList& l, const LinEpi& e)
+{
+  CAI_REQUIRE(w->qtype == CAI_BF16 && mat_rows >= 1 && w->rows % mat_rows == 0 && ldx >= w->ld && l.max_tiles >= 1, "bf16 bank: matrices of %d rows of %lld, activation rows of %lld", mat_rows, (long long)w->rows, (long long)ldx);
+  CAI_REQUIRE(e.mode == EPI_STORE || (e.mode == EPI_GLU && mat_rows % 32 == 0), "bf16 bank: a gated matrix needs whole blocks of 32 rows");
+  if (act_t == ACT_T_BF16) run_bank<bf16_t>(w, mat_rows, (const bf16_t*)x, ldx, l, e);
+  else run_bank<float>(w, mat_rows, (const float*)x, ldx, l, e);
+  CAI_HIP(hipGetLastError());
+  return CAI_OK;
 }
 
 template <typename AT, int NB>

@@ -7,7 +7,9 @@
 #include "cai_layered.hpp"
 #include "cai_json.hpp"
 
+#include <algorithm>
 #include <fcntl.h>
+#include <math.h>
 #include <string.h>
 #include <sys/mman.h>
 #include <sys/stat.h>
@@ -117,14 +119,14 @@ struct Builder {
     else return fail("tensor \"" + name + "\" has type " + t->dtype + ", expected BF16 or F32");
     return true;
   }
-  float* upload(const std::vector<float>& v)
+  template <typename T> T* upload(const std::vector<T>& v)
   {
     if (rc) return nullptr;
     void* p = nullptr;
-    hipError_t e = hipMalloc(&p, v.size() * 4);
-    if (e == hipSuccess) { s.vectors.push_back(p); e = hipMemcpy(p, v.data(), v.size() * 4, hipMemcpyHostToDevice); }
+    hipError_t e = hipMalloc(&p, v.size() * sizeof(T));
+    if (e == hipSuccess) { s.vectors.push_back(p); e = hipMemcpy(p, v.data(), v.size() * sizeof(T), hipMemcpyHostToDevice); }
     if (e != hipSuccess) { rc = hip_fail(e, "model vector upload", __FILE__, __LINE__); return nullptr; }
-    return (float*)p;
+    return (T*)p;
   }
   float* vec(const std::string& name, std::vector<int64_t> shape)
   {
@@ -157,15 +159,48 @@ struct Builder {
     s.weights.push_back(w);
     return w;
   }
-  Dyt dyt_norm(const std::string& name, int width)
+  // mult: a constant the norm's result is multiplied by, carried in its weight and bias
+  Dyt dyt_norm(const std::string& name, int width, float mult = 1.0f)
   {
     Dyt d;
-    std::vector<float> a;
-    if (!floats(name + ".alpha", {}, a)) return d;
-    d.alpha = a[0];
-    d.w = vec(name, {width}); d.b = vec(name + ".b", {width});
+    std::vector<float> a, w, b;
+    if (!floats(name + ".alpha", {}, a) || !floats(name, {width}, w) || !floats(name + ".b", {width}, b)) return d;
+    for (float& v : w) v *= mult;
+    for (float& v : b) v *= mult;
+    d.alpha = a[0]; d.w = upload(w); d.b = upload(b);
     return d;
   }
+  // gate and up matrices of one or several feed-forwards (names end before "gate"), rows interleaved in blocks of 16, one after the other
+  cai_qw_s* gated(const std::vector<std::string>& pre, int ff, int width)
+  {
+    std::vector<std::pair<std::string, int64_t>> parts;
+    std::vector<int> order((size_t)pad_to(ff, 16) * 2 * pre.size(), -1);
+    for (size_t e = 0; e < pre.size(); e++) {
+      parts.push_back({pre[e] + "gate", ff}); parts.push_back({pre[e] + "up", ff});
+      const size_t base = e * (size_t)pad_to(ff, 16) * 2;
+      for (int j = 0; j < ff; j++) { order[base + glu_row(j, 0)] = (int)(2 * e) * ff + j; order[base + glu_row(j, 1)] = (int)(2 * e + 1) * ff + j; }
+    }
+    return stack(parts, width, &order);
+  }
+  const Json* layer_list(const Json& cfg)          // sizes every layered design has, and its list of layers
+  {
+    s.width = integer(&cfg, "width", ""); s.vocab = integer(&cfg, "vocab", "", 1, 1 << 28);
+    s.eps = number(cfg.get("norm"), "eps", "norm.");
+    const Json* layers = cfg.get("layers");
+    if (!layers || layers->kind != Json::ARR || layers->arr.empty()) { fail("\"layers\" is missing or empty"); return nullptr; }
+    const int L = (int)layers->arr.size();
+    const Json* loop = cfg.get("loop");
+    if (loop && loop->kind != Json::NUL) {
+      s.loop_start = integer(loop, "start", "loop.", 0, L); s.loop_stop = integer(loop, "stop", "loop.", 0, L); s.loop_times = integer(loop, "times", "loop.", 1, 4096);
+      if (!rc && s.loop_stop < s.loop_start) fail("loop.stop lies before loop.start");
+    }
+    if (rc) return nullptr;
+    s.embed = stack({{"embed", s.vocab}}, s.width);
+    s.head = stack({{"head", s.vocab}}, s.width);
+    s.final_norm = dyt_norm("final.norm", s.width);
+    return rc ? nullptr : layers;
+  }
+  std::string word(const Json* o, const char* key) { const Json* v = o ? o->get(key) : nullptr; return v && v->kind == Json::STR ? v->str : std::string(); }
 };
 
 // ------------------------------------------------------------------------------------------
@@ -219,28 +254,16 @@ void attn_block(Builder& b, const Json* c, const std::string& where, const std::
   if (d.heads % d.kv_heads) { b.fail(where + "heads is not a multiple of " + where + "kv_heads"); return; }
   auto take = [&](const char* n, int rows) { const int o = at; parts.push_back({pre + n, rows}); at += rows; return o; };
   A.oq = take("q", d.heads * d.dim); A.ok = take("k", d.kv_heads * d.dim); A.ov = take("v", d.kv_heads * d.vdim);
-  A.qn = b.vec(pre + "q.norm", {d.dim}); A.kn = b.vec(pre + "k.norm", {d.dim});
+  A.qn = b.vec(pre + "q.norm", {d.dim}); A.kn = b.vec(pre + "k.norm", {d.dim}); A.og = -1;
   A.out = b.stack({{pre + "o", width}}, (int64_t)d.heads * d.vdim);
 }
 
 void build_samanex(Builder& b, const Json& cfg)
 {
   NetSpec& s = b.s;
-  s.width = b.integer(&cfg, "width", ""); s.vocab = b.integer(&cfg, "vocab", "", 1, 1 << 28);
-  s.eps = b.number(cfg.get("norm"), "eps", "norm.");
-  const Json* layers = cfg.get("layers");
-  if (!layers || layers->kind != Json::ARR || layers->arr.empty()) { b.fail("\"layers\" is missing or empty"); return; }
-  const int L = (int)layers->arr.size();
-  const Json* loop = cfg.get("loop");
-  if (loop && loop->kind != Json::NUL) {
-    s.loop_start = b.integer(loop, "start", "loop.", 0, L); s.loop_stop = b.integer(loop, "stop", "loop.", 0, L); s.loop_times = b.integer(loop, "times", "loop.", 1, 4096);
-    if (!b.rc && s.loop_stop < s.loop_start) b.fail("loop.stop lies before loop.start");
-  }
-  if (b.rc) return;
-  const int w = s.width;
-  s.embed = b.stack({{"embed", s.vocab}}, w);
-  s.head = b.stack({{"head", s.vocab}}, w);
-  s.final_norm = b.dyt_norm("final.norm", w);
+  const Json* layers = b.layer_list(cfg);
+  if (!layers) return;
+  const int L = (int)layers->arr.size(), w = s.width;
   for (int l = 0; l < L && !b.rc; l++) {
     const Json& c = layers->arr[l];
     const std::string p = "l" + std::to_string(l) + ".", where = "layers[" + std::to_string(l) + "].";
@@ -265,9 +288,7 @@ void build_samanex(Builder& b, const Json& cfg)
       y.ff = b.integer(mlp, "ff", where + "mlp.");
       if (b.rc) return;
       y.norm2 = b.dyt_norm(p + "norm2", w); y.norm2b = b.dyt_norm(p + "norm2b", w);
-      std::vector<int> order((size_t)pad_to(y.ff, 16) * 2, -1);     // gate and up rows interleaved in blocks of 16
-      for (int j = 0; j < y.ff; j++) { order[(size_t)glu_row(j, 0)] = j; order[(size_t)glu_row(j, 1)] = y.ff + j; }
-      y.gateup = b.stack({{p + "mlp.gate", y.ff}, {p + "mlp.up", y.ff}}, w, &order);
+      y.gateup = b.gated({p + "mlp."}, y.ff, w);
       y.down = b.stack({{p + "mlp.down", w}}, y.ff);
       y.glu = GLU_RELU;
     } else if (mlp && mlp->kind != Json::NUL) b.fail("\"" + where + "mlp\" is neither an object nor null");
@@ -275,8 +296,124 @@ void build_samanex(Builder& b, const Json& cfg)
   }
 }
 
+// ------------------------------------------------------------------------------------------
+// Kiruvik: rotary attention in fixed blocks of positions with an output gate, and Mamba-2 layers; dense or mixture-of-experts
+// feed-forwards; Dynamic Tanh before and after each sublayer, the latter times one constant; a stretch of layers run several times,
+// a matrix over the stream and the embedding output in front of every pass.
+// ------------------------------------------------------------------------------------------
+void block_attention(Builder& b, const Json* c, const std::string& where, const std::string& pre, int width, NetLayer& y)
+{
+  NetAttn& A = y.attn; AttnDims& d = A.d;
+  d.heads = b.integer(c, "heads", where, 1, 65535); d.kv_heads = b.integer(c, "kv_heads", where, 1, 65535);
+  d.dim = b.integer(c, "dim", where, 1, 256); d.vdim = b.integer(c, "vdim", where, 1, 256);
+  const Json *mask = c ? c->get("mask") : nullptr, *rot = c ? c->get("rot") : nullptr;
+  d.window = b.integer(mask, "size", where + "mask.", 1, 1 << 30); d.chunked = 1;
+  d.rot = b.integer(rot, "dims", where + "rot.", 0, d.dim);
+  const float base = b.number(rot, "base", where + "rot.");
+  d.scale = b.number(c, "scale", where); d.eps = b.s.eps;
+  d.dim_p = pad_to(d.dim, 8); d.vdim_p = pad_to(d.vdim, 8);
+  if (b.rc) return;
+  if (d.heads % d.kv_heads) { b.fail(where + "heads is not a multiple of " + where + "kv_heads"); return; }
+  if (d.rot % 2 || !(base > 0.0f)) { b.fail(where + "rot needs an even number of dims and a base above zero"); return; }
+  if (d.rot) {
+    std::vector<double> turns((size_t)d.rot / 2);
+    for (int i = 0; i < d.rot / 2; i++) turns[i] = pow((double)rot->get("base")->num, -2.0 * i / d.rot) / (2.0 * M_PI);
+    d.turns = b.upload(turns);
+  }
+  const int qw = d.heads * d.dim, kw = d.kv_heads * d.dim, vw = d.kv_heads * d.vdim, ow = d.heads * d.vdim;
+  A.oq = 0; A.ok = qw; A.ov = qw + kw; A.og = qw + kw + vw;
+  y.in = b.stack({{pre + "q", qw}, {pre + "k", kw}, {pre + "v", vw}, {pre + "g", ow}}, width);
+  std::vector<float> bias, part;
+  for (auto& n : {std::make_pair("q.b", qw), std::make_pair("k.b", kw), std::make_pair("v.b", vw)}) {
+    if (!b.floats(pre + n.first, {n.second}, part)) return;
+    bias.insert(bias.end(), part.begin(), part.end());
+  }
+  bias.resize((size_t)A.og + ow, 0.0f);                  // (the gate has none)
+  y.in_b = b.upload(bias);
+  A.out = b.stack({{pre + "o", width}}, ow);
+  A.out_b = b.vec(pre + "o.b", {width});
+}
+
+void ssd_block(Builder& b, const Json* c, const std::string& where, const std::string& pre, int width, NetLayer& y)
+{
+  NetSsd& M = y.ssd; SsdDims& d = M.d;
+  d.heads = b.integer(c, "heads", where, 1, 65535); d.vdim = b.integer(c, "vdim", where, 1, 256); d.state = b.integer(c, "state", where, 1, 256);
+  d.groups = b.integer(c, "groups", where, 1, 65535); d.taps = b.integer(c, "conv", where, 1, 4096); d.norm_groups = b.integer(c, "norm_groups", where, 1, 65535);
+  d.eps = b.s.eps;
+  if (b.rc) return;
+  if (d.heads % d.groups) { b.fail(where + "heads is not a multiple of " + where + "groups"); return; }
+  if (d.inner() % d.norm_groups) { b.fail("heads times vdim is not a multiple of " + where + "norm_groups"); return; }
+  M.oz = 0; M.ox = d.inner(); M.odt = M.ox + d.channels();
+  y.in = b.stack({{pre + "in", (int64_t)M.odt + d.heads}}, width);
+  M.w.conv = b.vec(pre + "conv", {d.channels(), d.taps}); M.w.conv_b = b.vec(pre + "conv.b", {d.channels()});
+  M.w.dt_bias = b.vec(pre + "dt_bias", {d.heads}); M.w.D = b.vec(pre + "D", {d.heads}); M.w.norm = b.vec(pre + "norm", {d.inner()});
+  std::vector<float> al;
+  if (!b.floats(pre + "A_log", {d.heads}, al)) return;
+  for (float& v : al) v = -expf(v);
+  M.w.rate = b.upload(al);
+  M.out = b.stack({{pre + "o", width}}, d.inner());
+}
+
+void experts_block(Builder& b, const Json* c, const std::string& where, const std::string& pre, int width, NetExperts& x)
+{
+  const Json *r = c->get("router"), *e = c->get("expert"), *sh = c->get("shared");
+  const int n = b.integer(r, "experts", where + "router.", 1, EXPERTS_MAX);
+  x.top = b.integer(r, "top", where + "router.", 1, std::min(n, EXPERTS_TOP)); x.scale = b.number(r, "scale", where + "router.");
+  x.ff = b.integer(e, "ff", where + "expert."); x.limit = b.number(e, "limit", where + "expert.");
+  if (b.rc) return;
+  x.glu = x.glu_shared = GLU_CLAMPED;
+  x.router = b.stack({{pre + "router", n}}, width);
+  x.correction = b.vec(pre + "correction", {n});
+  std::vector<std::string> names; std::vector<std::pair<std::string, int64_t>> down;
+  for (int i = 0; i < n; i++) { names.push_back(pre + "e" + std::to_string(i) + "."); down.push_back({names.back() + "down", width}); }
+  x.gateup = b.gated(names, x.ff, width);
+  x.down = b.stack(down, x.ff);
+  if (sh && sh->kind != Json::NUL) {
+    x.ff_shared = b.integer(sh, "ff", where + "shared."); x.limit_shared = b.number(sh, "limit", where + "shared.");
+    if (b.rc) return;
+    x.s_gateup = b.gated({pre + "shared."}, x.ff_shared, width);
+    x.s_down = b.stack({{pre + "shared.down", width}}, x.ff_shared);
+  }
+  x.n = n;
+}
+
+void build_kiruvik(Builder& b, const Json& cfg)
+{
+  NetSpec& s = b.s;
+  const Json* layers = b.layer_list(cfg);
+  const float mult = b.number(&cfg, "residual_mult", "");
+  if (!layers || b.rc) return;
+  const int L = (int)layers->arr.size(), w = s.width;
+  if (s.loop_stop > s.loop_start) s.loop_in = b.stack({{"loop.in", w}}, 2 * w);
+  for (int l = 0; l < L && !b.rc; l++) {
+    const Json& c = layers->arr[l];
+    const std::string p = "l" + std::to_string(l) + ".", where = "layers[" + std::to_string(l) + "].", type = b.word(&c, "type");
+    const Json *mix = c.get("mixer"), *mlp = c.get("mlp");
+    NetLayer y;
+    if (type == "attention") { y.kind = MIX_ATTN; block_attention(b, mix, where + "mixer.", p + "mix.", w, y); }
+    else if (type == "mamba2") { y.kind = MIX_SSD; ssd_block(b, mix, where + "mixer.", p + "mix.", w, y); }
+    else b.fail("\"" + where + "type\" is not one of attention, mamba2");
+    if (b.rc) return;
+    y.norm1 = b.dyt_norm(p + "norm1", w); y.norm1b = b.dyt_norm(p + "norm1b", w, mult);
+    if (mlp && mlp->kind == Json::OBJ) {
+      const std::string kind = b.word(mlp, "kind");
+      if (kind == "dense") {
+        y.ff = b.integer(mlp, "ff", where + "mlp.");
+        if (b.rc) return;
+        y.gateup = b.gated({p + "mlp."}, y.ff, w);
+        y.down = b.stack({{p + "mlp.down", w}}, y.ff);
+        y.glu = GLU_GELU_TANH;
+      } else if (kind == "moe") experts_block(b, mlp, where + "mlp.", p + "mlp.", w, y.experts);
+      else b.fail("\"" + where + "mlp.kind\" is not one of dense, moe");
+      if (b.rc) return;
+      y.norm2 = b.dyt_norm(p + "norm2", w); y.norm2b = b.dyt_norm(p + "norm2b", w, mult);
+    } else if (mlp && mlp->kind != Json::NUL) b.fail("\"" + where + "mlp\" is neither an object nor null");
+    s.layers.push_back(y);
+  }
+}
+
 struct Arch { const char* name; void (*build)(Builder&, const Json&); };
-const Arch ARCHS[] = {{"Samanex", build_samanex}};
+const Arch ARCHS[] = {{"Samanex", build_samanex}, {"Kiruvik", build_kiruvik}};
 
 bool is_dir(const char* path) { struct stat sb; return stat(path, &sb) == 0 && S_ISDIR(sb.st_mode); }
 

@@ -127,7 +127,113 @@ def relu_glu(w, pre, h):
     return linear(w[pre + "down"], np.maximum(linear(w[pre + "gate"], h), 0.0) * linear(w[pre + "up"], h))
 
 
-# ---------------------------------------------------------------- the model
+# ---------------------------------------------------------------- mechanisms of Kiruvik
+def gelu_tanh(z):
+    return 0.5 * z * (1.0 + np.tanh(np.sqrt(2.0 / np.pi) * (z + 0.044715 * z ** 3)))
+
+
+def rotate_half(x, base, dims, pos0=0):
+    """x [T, heads, d]: dimension i of the first `dims` turns with dimension i + dims / 2 by position * base^(-2i/dims)"""
+    half = dims // 2
+    out = x.copy()
+    for t in range(x.shape[0]):
+        for i in range(half):
+            a = (pos0 + t) * base ** (-2.0 * i / dims)
+            u, v = x[t, :, i], x[t, :, i + half]
+            out[t, :, i] = u * np.cos(a) - v * np.sin(a)
+            out[t, :, i + half] = v * np.cos(a) + u * np.sin(a)
+    return out
+
+
+def chunk_attention(q, k, v, scale, size):
+    """as window_attention, but query i sees the keys up to itself of its own block of `size` positions"""
+    T, H, _ = q.shape
+    G = k.shape[1]
+    i, j = np.arange(T)[:, None], np.arange(T)[None, :]
+    seen = (j <= i) & (i // size == j // size)
+    out = np.zeros((T, H, v.shape[2]))
+    for h in range(H):
+        g = h // (H // G)
+        s = np.where(seen, (q[:, h] @ k[:, g].T) * scale, -np.inf)
+        out[:, h] = softmax_rows(s) @ v[:, g]
+    return out
+
+
+def ssd_recurrence(x, B, C, dt, rate, D):
+    """State-space duality, token by token.  x [T, H, P]; B, C [T, G, N]; dt [T, H]; rate, D [H].  S [H, N, P] starts at zero:
+    decay by exp(-rate dt), add dt B x^T, read with C; the input passes by with weight D."""
+    T, H, P = x.shape
+    G, N = B.shape[1:]
+    S = np.zeros((H, N, P))
+    y = np.zeros_like(x)
+    for t in range(T):
+        for h in range(H):
+            g = h // (H // G)
+            S[h] = np.exp(-rate[h] * dt[t, h]) * S[h] + dt[t, h] * np.outer(B[t, g], x[t, h])
+            y[t, h] = S[h].T @ C[t, g] + D[h] * x[t, h]
+    return y
+
+
+def group_rms_norm(x, groups, eps):
+    T, n = x.shape
+    return rms_norm(x.reshape(T, groups, n // groups), eps).reshape(T, n)
+
+
+def clamped_expert(w, pre, h, limit):
+    g = np.minimum(linear(w[pre + "gate"], h), limit)
+    u = np.clip(linear(w[pre + "up"], h), -limit, limit)
+    return linear(w[pre + "down"], g * sigmoid(1.702 * g) * (u + 1.0))
+
+
+def route(z, correction, top, scale):
+    """[T, experts] weights of one token's experts, zero where not chosen: soft-max scores, chosen with the correction added, weighted
+    without it"""
+    s = softmax_rows(z)
+    out = np.zeros_like(s)
+    for t in range(s.shape[0]):
+        chosen = np.argsort(-(s[t] + correction), kind="stable")[:top]
+        out[t, chosen] = s[t, chosen] / (s[t, chosen].sum() + 1e-20) * scale
+    return out
+
+
+def rotary_attention_mixer(w, pre, c, h):
+    T = h.shape[0]
+    H, G, d, dv = c["heads"], c["kv_heads"], c["dim"], c["vdim"]
+    q, k, v = (linear(w[pre + n], h) + w[pre + n + ".b"] for n in "qkv")
+    q = rotate_half(q.reshape(T, H, d), c["rot"]["base"], c["rot"]["dims"])
+    k = rotate_half(k.reshape(T, G, d), c["rot"]["base"], c["rot"]["dims"])
+    o = chunk_attention(q, k, v.reshape(T, G, dv), c["scale"], c["mask"]["size"]).reshape(T, H * dv)
+    o = o * sigmoid(linear(w[pre + "g"], h))
+    return linear(w[pre + "o"], o) + w[pre + "o.b"]
+
+
+def ssd_mixer(w, pre, c, h, eps):
+    T = h.shape[0]
+    H, P, N, G = c["heads"], c["vdim"], c["state"], c["groups"]
+    inner = H * P
+    z, x, B, C, dt = np.split(linear(w[pre + "in"], h), np.cumsum([inner, inner, G * N, G * N]), axis=1)
+    xbc = silu(causal_conv(np.concatenate([x, B, C], axis=1), w[pre + "conv"]) + w[pre + "conv.b"])
+    x, B, C = np.split(xbc, np.cumsum([inner, G * N]), axis=1)
+    dt = softplus(dt + w[pre + "dt_bias"])
+    y = ssd_recurrence(x.reshape(T, H, P), B.reshape(T, G, N), C.reshape(T, G, N), dt, np.exp(w[pre + "A_log"]), w[pre + "D"])
+    y = group_rms_norm(y.reshape(T, inner) * silu(z), c["norm_groups"], eps) * w[pre + "norm"]
+    return linear(w[pre + "o"], y)
+
+
+def gelu_glu(w, pre, h):
+    return linear(w[pre + "down"], gelu_tanh(linear(w[pre + "gate"], h)) * linear(w[pre + "up"], h))
+
+
+def expert_mixture(w, pre, c, h):
+    r = c["router"]
+    wt = route(linear(w[pre + "router"], h), w[pre + "correction"], r["top"], r["scale"])
+    y = clamped_expert(w, pre + "shared.", h, c["shared"]["limit"])
+    for e in range(r["experts"]):
+        y = y + wt[:, e:e + 1] * clamped_expert(w, pre + "e%d." % e, h, c["expert"]["limit"])
+    return y
+
+
+# ---------------------------------------------------------------- the models
 def run_order(cfg):
     """(layer, first layer of a repeated pass) for every layer run"""
     n = len(cfg["layers"])
@@ -140,6 +246,8 @@ def run_order(cfg):
 
 def forward(cfg, w, tokens, layers_out=None):
     """logits [T, vocab] of a whole prompt"""
+    if cfg["architecture"] == "Kiruvik":
+        return kiruvik_forward(cfg, w, tokens, layers_out)
     eps = cfg["norm"]["eps"]
     norm = lambda name, x: dynamic_tanh(x, w[name + ".alpha"], w[name], w[name + ".b"])
     x = w["embed"][np.asarray(tokens)]
@@ -154,6 +262,31 @@ def forward(cfg, w, tokens, layers_out=None):
         x = x + norm(p + "norm1b", y)
         if L.get("mlp"):
             x = x + norm(p + "norm2b", relu_glu(w, p + "mlp.", norm(p + "norm2", x)))
+        if layers_out is not None:
+            layers_out.append(x.copy())
+    return linear(w["head"], norm("final.norm", x))
+
+
+def kiruvik_forward(cfg, w, tokens, layers_out=None):
+    eps, m = cfg["norm"]["eps"], cfg["residual_mult"]
+    norm = lambda name, x: dynamic_tanh(x, w[name + ".alpha"], w[name], w[name + ".b"])
+    x = w["embed"][np.asarray(tokens)]
+    x0 = x
+    lp = cfg.get("loop")
+    n = len(cfg["layers"])
+    order = list(range(n)) if not lp else list(range(lp["start"])) + list(range(lp["start"], lp["stop"])) * lp["times"] + list(range(lp["stop"], n))
+    for r, i in enumerate(order):
+        L = cfg["layers"][i]
+        p = "l%d." % i
+        if lp and lp["start"] <= r < lp["start"] + (lp["stop"] - lp["start"]) * lp["times"] and i == lp["start"]:
+            x = linear(w["loop.in"], np.concatenate([x, x0], axis=1))
+        h = norm(p + "norm1", x)
+        y = rotary_attention_mixer(w, p + "mix.", L["mixer"], h) if L["type"] == "attention" else ssd_mixer(w, p + "mix.", L["mixer"], h, eps)
+        x = x + m * norm(p + "norm1b", y)
+        if L.get("mlp"):
+            h = norm(p + "norm2", x)
+            y = gelu_glu(w, p + "mlp.", h) if L["mlp"]["kind"] == "dense" else expert_mixture(w, p + "mlp.", L["mlp"], h)
+            x = x + m * norm(p + "norm2b", y)
         if layers_out is not None:
             layers_out.append(x.copy())
     return linear(w["head"], norm("final.norm", x))
