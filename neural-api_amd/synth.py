@@ -223,8 +223,21 @@ def layered_config(width, ff, heads, kv_heads, dim, n_layers, vocab, window, con
     return dict(architecture="Samanex", width=width, vocab=vocab, layers=layers, norm=dict(eps=1e-6), loop=loop or dict(start=0, stop=n_layers, times=1))
 
 
+def kiruvik_config(width, ff, heads, kv_heads, dim, n_layers, vocab, block, conv=4, every=4, experts=32, top=4, state=128, vdim=64, groups=1):
+    """A Kiruvik configuration of real-model proportions: every `every`-th layer is an attention, the others are Mamba-2 layers of twice
+    the width inside; dense feed-forwards and mixtures (of as many active rows: `top` experts and a shared one of half) in turn."""
+    att = dict(heads=heads, kv_heads=max(1, kv_heads // 2), dim=dim, vdim=dim, scale=dim ** -0.5, mask=dict(size=block), rot=dict(base=1e4, dims=dim))
+    ssd = dict(heads=2 * width // vdim, vdim=vdim, state=state, groups=groups, conv=conv, norm_groups=1)
+    moe = dict(kind="moe", expert=dict(ff=ff // (2 * top), limit=7.0), router=dict(experts=experts, top=top, scale=1.5), shared=dict(ff=ff // 2, limit=7.0))
+    layers = [dict(type="attention" if i % every == every - 1 else "mamba2", mixer=att if i % every == every - 1 else ssd, mlp=moe if i % 2 else dict(kind="dense", ff=ff))
+              for i in range(n_layers)]
+    return dict(architecture="Kiruvik", width=width, vocab=vocab, layers=layers, norm=dict(eps=1e-6), residual_mult=0.8, loop=dict(start=0, stop=n_layers, times=1))
+
+
 def layered_shapes(cfg, rank=128):
-    """name -> (shape, standard deviation, mean) of every tensor of a Samanex model"""
+    """name -> (shape, standard deviation, mean) of every tensor of a layered model"""
+    if cfg["architecture"] == "Kiruvik":
+        return kiruvik_shapes(cfg)
     w, out = cfg["width"], {}
 
     def lin(name, rows, cols):
@@ -263,6 +276,62 @@ def layered_shapes(cfg, rank=128):
             norm(p + "norm2"); norm(p + "norm2b")
             lin(p + "mlp.gate", L["mlp"]["ff"], w); lin(p + "mlp.up", L["mlp"]["ff"], w); lin(p + "mlp.down", w, L["mlp"]["ff"])
     return out
+
+
+def kiruvik_shapes(cfg):
+    w, out = cfg["width"], {}
+
+    def lin(name, rows, cols):
+        out[name] = ((rows, cols), cols ** -0.5, 0.0)
+
+    def norm(name):
+        out[name] = ((w,), 0.1, 1.0); out[name + ".b"] = ((w,), 0.05, 0.0); out[name + ".alpha"] = ((), 0.0, 0.7)
+
+    def glu(p, ff):
+        lin(p + "gate", ff, w); lin(p + "up", ff, w); lin(p + "down", w, ff)
+
+    out["embed"] = ((cfg["vocab"], w), 1.0, 0.0)
+    lin("head", cfg["vocab"], w); lin("loop.in", w, 2 * w); norm("final.norm")
+    for i, L in enumerate(cfg["layers"]):
+        p, m = "l%d." % i, L["mixer"]
+        norm(p + "norm1"); norm(p + "norm1b")
+        if L["type"] == "attention":
+            for n, r in (("q", m["heads"] * m["dim"]), ("k", m["kv_heads"] * m["dim"]), ("v", m["kv_heads"] * m["vdim"])):
+                lin(p + "mix." + n, r, w); out[p + "mix." + n + ".b"] = ((r,), 0.1, 0.0)
+            lin(p + "mix.g", m["heads"] * m["vdim"], w); lin(p + "mix.o", w, m["heads"] * m["vdim"]); out[p + "mix.o.b"] = ((w,), 0.1, 0.0)
+        else:
+            inner = m["heads"] * m["vdim"]; ch = inner + 2 * m["groups"] * m["state"]
+            lin(p + "mix.in", inner + ch + m["heads"], w); lin(p + "mix.o", w, inner)
+            out[p + "mix.conv"] = ((ch, m["conv"]), 0.3, 0.25); out[p + "mix.conv.b"] = ((ch,), 0.1, 0.0)
+            out[p + "mix.dt_bias"] = ((m["heads"],), 1.0, -3.0); out[p + "mix.A_log"] = ((m["heads"],), 0.5, 0.0)
+            out[p + "mix.D"] = ((m["heads"],), 0.1, 1.0); out[p + "mix.norm"] = ((inner,), 0.1, 1.0)
+        f = L["mlp"]
+        if f:
+            norm(p + "norm2"); norm(p + "norm2b")
+            if f["kind"] == "dense":
+                glu(p + "mlp.", f["ff"])
+            else:
+                lin(p + "mlp.router", f["router"]["experts"], w); out[p + "mlp.correction"] = ((f["router"]["experts"],), 0.01, 0.0)
+                for e in range(f["router"]["experts"]):
+                    glu(p + "mlp.e%d." % e, f["expert"]["ff"])
+                glu(p + "mlp.shared.", f["shared"]["ff"])
+    return out
+
+
+def layered_active_weights(cfg):
+    """linear weights one token of a prompt meets, the vocabulary left out"""
+    import numpy as np
+    total = 0
+    for name, (shape, _, _) in layered_shapes(cfg).items():
+        if len(shape) != 2 or name in ("embed", "head") or name.endswith("conv"):
+            continue
+        n = int(np.prod(shape))
+        part = name.split(".")
+        if len(part) > 2 and part[1] == "mlp" and part[2][0] == "e" and part[2][1:].isdigit():
+            r = cfg["layers"][int(part[0][1:])]["mlp"]["router"]
+            n = n * r["top"] / r["experts"]
+        total += n
+    return total
 
 
 def write_layered_folder(folder, cfg, seed=0, rank=128):

@@ -1,4 +1,4 @@
-"""Small random Samanex models for the layered-decoder tests: a configuration, weights rounded to bfloat16, a model folder."""
+"""Small random models for the layered-decoder tests: a configuration, weights rounded to bfloat16, a model folder."""
 import json
 import os
 import struct
@@ -34,8 +34,88 @@ def config(layers, width=72, vocab=131, eps=1e-5, loop=None):
                 loop=loop or dict(start=0, stop=len(layers), times=1))
 
 
+# ---------------------------------------------------------------- Kiruvik
+def rotary(heads=4, kv_heads=2, dim=24, vdim=40, block=9, scale=0.21, rot=10, base=500.0):
+    return dict(heads=heads, kv_heads=kv_heads, dim=dim, vdim=vdim, scale=scale, mask=dict(size=block), rot=dict(base=base, dims=rot))
+
+
+def ssd(heads=4, vdim=18, state=20, groups=2, conv=3, norm_groups=3):
+    return dict(heads=heads, vdim=vdim, state=state, groups=groups, conv=conv, norm_groups=norm_groups)
+
+
+def moe(experts=6, top=2, ff=20, scale=1.7, limit=0.9, shared_ff=28, shared_limit=1.3):
+    return dict(kind="moe", expert=dict(ff=ff, limit=limit), router=dict(experts=experts, top=top, scale=scale), shared=dict(ff=shared_ff, limit=shared_limit))
+
+
+def klayer(mixer, mlp=None):
+    """an attention or a state-space layer; mlp: a width (dense), a mixture, or None"""
+    return dict(type="attention" if "rot" in mixer else "mamba2", mixer=mixer, mlp=dict(kind="dense", ff=mlp) if isinstance(mlp, int) else mlp)
+
+
+def kconfig(layers, width=72, vocab=131, eps=1e-5, loop=None, mult=0.8):
+    return dict(architecture="Kiruvik", width=width, vocab=vocab, layers=layers, norm=dict(eps=eps), residual_mult=mult, loop=loop)
+
+
+def kiruvik_weights(cfg, seed=0):
+    rng = np.random.default_rng(seed)
+    w, width = {}, cfg["width"]
+
+    def lin(name, rows, cols, gain=1.0):
+        w[name] = rng.standard_normal((rows, cols)) * gain / np.sqrt(cols)
+
+    def vec(name, shape, mean=0.0, spread=0.2):
+        w[name] = mean + spread * rng.standard_normal(shape)
+
+    def norm(name):
+        vec(name, width, 1.0); vec(name + ".b", width, 0.0, 0.1)
+        w[name + ".alpha"] = np.asarray(rng.uniform(0.4, 1.2))
+
+    def glu(p, ff):
+        lin(p + "gate", ff, width, 1.5); lin(p + "up", ff, width, 1.5); lin(p + "down", width, ff)
+
+    vec("embed", (cfg["vocab"], width), 0.0, 1.0)
+    lin("head", cfg["vocab"], width, 2.0)
+    norm("final.norm")
+    if cfg["loop"] and cfg["loop"]["stop"] > cfg["loop"]["start"]:
+        lin("loop.in", width, 2 * width, 1.3)
+    for i, L in enumerate(cfg["layers"]):
+        p, m, f = "l%d." % i, L["mixer"], L["mlp"]
+        norm(p + "norm1"); norm(p + "norm1b")
+        if L["type"] == "attention":
+            for n, r in (("q", m["heads"] * m["dim"]), ("k", m["kv_heads"] * m["dim"]), ("v", m["kv_heads"] * m["vdim"])):
+                lin(p + "mix." + n, r, width, 1.5); vec(p + "mix." + n + ".b", r, 0.0, 0.4)
+            lin(p + "mix.g", m["heads"] * m["vdim"], width, 2.0)
+            lin(p + "mix.o", width, m["heads"] * m["vdim"]); vec(p + "mix.o.b", width, 0.0, 0.3)
+        else:
+            inner = m["heads"] * m["vdim"]; ch = inner + 2 * m["groups"] * m["state"]
+            lin(p + "mix.in", inner + ch + m["heads"], width, 1.5)
+            vec(p + "mix.conv", (ch, m["conv"]), 0.3, 0.5); vec(p + "mix.conv.b", ch, 0.0, 0.3)
+            vec(p + "mix.dt_bias", m["heads"], -2.0, 1.0); w[p + "mix.A_log"] = rng.uniform(-2.0, 1.0, m["heads"])
+            vec(p + "mix.D", m["heads"], 0.7, 0.5); vec(p + "mix.norm", inner, 1.0)
+            lin(p + "mix.o", width, inner)
+        if f:
+            norm(p + "norm2"); norm(p + "norm2b")
+            if f["kind"] == "dense":
+                glu(p + "mlp.", f["ff"])
+            else:
+                lin(p + "mlp.router", f["router"]["experts"], width, 2.0); vec(p + "mlp.correction", f["router"]["experts"], 0.0, 0.1)
+                for e in range(f["router"]["experts"]):
+                    glu(p + "mlp.e%d." % e, f["expert"]["ff"])
+                glu(p + "mlp.shared.", f["shared"]["ff"])
+    return w
+
+
+def steady_choice(w):
+    """corrections so far apart that they alone decide which experts run: rounding cannot change the choice"""
+    for n in w:
+        if n.endswith(".correction"):
+            w[n] = 4.0 * np.random.default_rng(len(w[n])).permutation(len(w[n]))
+
+
 def weights(cfg, seed=0, rank_a=7, rank_g=11):
     """name -> float array before rounding"""
+    if cfg["architecture"] == "Kiruvik":
+        return kiruvik_weights(cfg, seed)
     rng = np.random.default_rng(seed)
     w, width = {}, cfg["width"]
 

@@ -136,12 +136,11 @@ def rotate_half(x, base, dims, pos0=0):
     """x [T, heads, d]: dimension i of the first `dims` turns with dimension i + dims / 2 by position * base^(-2i/dims)"""
     half = dims // 2
     out = x.copy()
-    for t in range(x.shape[0]):
-        for i in range(half):
-            a = (pos0 + t) * base ** (-2.0 * i / dims)
-            u, v = x[t, :, i], x[t, :, i + half]
-            out[t, :, i] = u * np.cos(a) - v * np.sin(a)
-            out[t, :, i + half] = v * np.cos(a) + u * np.sin(a)
+    for i in range(half):
+        a = ((pos0 + np.arange(x.shape[0])) * base ** (-2.0 * i / dims))[:, None]
+        u, v = x[:, :, i], x[:, :, i + half]
+        out[:, :, i] = u * np.cos(a) - v * np.sin(a)
+        out[:, :, i + half] = v * np.cos(a) + u * np.sin(a)
     return out
 
 

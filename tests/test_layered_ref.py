@@ -72,6 +72,81 @@ def test_oracle_is_sensitive_to_what_it_checks():
     assert np.abs(R.forward(cfg, w, tok[1:])[-1] - base[-1]).max() > 2e-5      # a token well before every window still counts
 
 
+# ---------------------------------------------------------------- Kiruvik's mechanisms
+def test_rotation_turns_pairs_by_relative_position():
+    rng = np.random.default_rng(4)
+    x, y = rng.standard_normal((1, 1, 12)), rng.standard_normal((1, 1, 12))
+    rot = lambda z, p: R.rotate_half(z, 50.0, 8, p)
+    assert np.allclose(rot(x, 0), x) and np.allclose(rot(x, 9)[..., 8:], x[..., 8:])
+    assert np.allclose((rot(x, 7) * rot(y, 3)).sum(), (rot(x, 104) * rot(y, 100)).sum())       # scores depend on the distance alone
+    z = np.zeros((1, 1, 12)); z[0, 0, 1] = 1.0
+    a = 5 * 50.0 ** (-2 / 8)
+    assert np.allclose(rot(z, 5)[0, 0, [1, 5]], [np.cos(a), np.sin(a)])                         # dimension i pairs with i + dims / 2
+    many = rng.standard_normal((6, 2, 12))
+    assert np.allclose(R.rotate_half(many, 50.0, 8)[4], R.rotate_half(many[4:5], 50.0, 8, 4)[0])
+
+
+@pytest.mark.parametrize("size", [1, 3, 4, 50])
+def test_block_attention_sees_its_own_block_up_to_itself(size):
+    rng = np.random.default_rng(3)
+    T = 9
+    q, k, v = rng.standard_normal((T, 4, 6)), rng.standard_normal((T, 2, 6)), rng.standard_normal((T, 2, 5))
+    o = R.chunk_attention(q, k, v, 0.3, size)
+    for i in range(T):
+        lo = i - i % size
+        for h in range(4):
+            s = np.exp(0.3 * k[lo:i + 1, h // 2] @ q[i, h])
+            assert np.allclose(o[i, h], (s / s.sum()) @ v[lo:i + 1, h // 2])
+
+
+def test_state_space_recurrence_is_a_decayed_sum_over_the_past():
+    rng = np.random.default_rng(5)
+    T, H, P, G, N = 7, 4, 3, 2, 5
+    x, B_, C = rng.standard_normal((T, H, P)), rng.standard_normal((T, G, N)), rng.standard_normal((T, G, N))
+    dt, rate, D = rng.uniform(0.1, 1, (T, H)), rng.uniform(0.1, 2, H), rng.standard_normal(H)
+    y = R.ssd_recurrence(x, B_, C, dt, rate, D)
+    for t in range(T):
+        for h in range(H):
+            g = h // 2
+            want = D[h] * x[t, h] + sum((C[t, g] @ B_[s, g]) * np.exp(-rate[h] * dt[s + 1:t + 1, h].sum()) * dt[s, h] * x[s, h] for s in range(t + 1))
+            assert np.allclose(y[t, h], want)
+
+
+def test_routing_chooses_with_the_correction_and_weighs_without_it():
+    z = np.log(np.array([[0.4, 0.3, 0.2, 0.1]]))
+    assert np.allclose(R.route(z, np.zeros(4), 2, 3.0), [[3 * 0.4 / 0.7, 3 * 0.3 / 0.7, 0, 0]])
+    assert np.allclose(R.route(z, np.array([0, 0, 0, 0.5]), 2, 3.0), [[3 * 0.4 / 0.5, 0, 0, 3 * 0.1 / 0.5]])
+
+
+def test_clamped_expert_and_gelu():
+    one = np.eye(1)
+    w = {"gate": one, "up": one, "down": one}
+    f = lambda h, limit: R.clamped_expert(w, "", np.array([[h]]), limit)[0, 0]
+    act = lambda g, u: g / (1 + np.exp(-1.702 * g)) * (u + 1)
+    assert np.isclose(f(0.5, 2.0), act(0.5, 0.5)) and np.isclose(f(3.0, 2.0), act(2.0, 2.0)) and np.isclose(f(-3.0, 2.0), act(-3.0, -2.0))      # the gate has no lower bound
+    assert np.isclose(R.gelu_tanh(np.array(1.0)), 0.841192, atol=1e-6) and np.isclose(R.gelu_tanh(np.array(-2.0)), -0.045402, atol=1e-6)
+    x = np.arange(1.0, 7.0)[None]
+    assert np.allclose(R.group_rms_norm(x, 3, 0.0)[0, :2], x[0, :2] / np.sqrt(2.5))
+
+
+def test_kiruvik_oracle_is_sensitive_to_what_it_checks():
+    """every constant of the configuration, a lost state and a pass without its matrix move the logits well beyond the tests' tolerances"""
+    cfg = B.kconfig([B.klayer(B.ssd(), B.moe()), B.klayer(B.rotary(), 40), B.klayer(B.ssd(heads=3, norm_groups=1, groups=1))], loop=dict(start=1, stop=3, times=2))
+    w = {n: B.to_bf16(a)[1].reshape(np.shape(a)) for n, a in B.weights(cfg, 5).items()}
+    tok = np.random.default_rng(6).integers(0, cfg["vocab"], 40)
+    base = R.forward(cfg, w, tok)
+    at = lambda c, i: c["layers"][i]
+    for change in (lambda c: at(c, 1)["mixer"]["mask"].update(size=10), lambda c: c["loop"].update(times=1), lambda c: c["loop"].update(start=0), lambda c: c.update(residual_mult=0.85),
+                   lambda c: at(c, 1)["mixer"].update(scale=0.25), lambda c: at(c, 1)["mixer"]["rot"].update(base=600.0), lambda c: at(c, 1)["mixer"]["rot"].update(dims=12),
+                   lambda c: c["norm"].update(eps=0.1), lambda c: at(c, 0)["mixer"].update(norm_groups=1), lambda c: at(c, 0)["mlp"]["router"].update(top=3),
+                   lambda c: at(c, 0)["mlp"]["router"].update(scale=2.0), lambda c: at(c, 0)["mlp"]["expert"].update(limit=1.0), lambda c: at(c, 0)["mlp"]["shared"].update(limit=1.1)):
+        other = json.loads(json.dumps(cfg)); change(other)
+        assert np.abs(R.forward(other, w, tok) - base).max() > 1e-2
+    for name in ("l0.mix.conv.b", "l0.mix.D", "l0.mix.dt_bias", "l1.mix.q.b", "l1.mix.k.b", "l1.mix.v.b", "l1.mix.o.b", "l0.mlp.correction", "loop.in"):
+        other = dict(w); other[name] = w[name] * 0.5
+        assert np.abs(R.forward(cfg, other, tok) - base).max() > 1e-2, name
+
+
 @pytest.mark.parametrize("text, reason", [("{", "malformed"), ("[]", ""), ('{"architecture": "Nobody"}', "Samanex"), ("{}", "Samanex"),
                                           ('{"architecture": "Samanex"} x', "after"), ('{"architecture": "\\ud800"}', "malformed")])
 def test_registry_refuses_what_it_does_not_know(tmp_path, text, reason):
