@@ -9,36 +9,55 @@
 
 namespace cai {
 
+// maximum over a wave, and minimum of whole numbers, in every lane (a lane without a partner meets itself)
+template <int CTRL, int ROWS> __device__ __forceinline__ float dpp_max(float v)
+{
+  const int x = __builtin_bit_cast(int, v);
+  return fmaxf(v, __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(x, x, CTRL, ROWS, 0xf, false)));
+}
+template <int CTRL, int ROWS> __device__ __forceinline__ int dpp_min(int v) { return min(v, __builtin_amdgcn_update_dpp(v, v, CTRL, ROWS, 0xf, false)); }
+__device__ __forceinline__ float wave_max(float v)
+{
+  v = dpp_max<0x111, 0xf>(v); v = dpp_max<0x112, 0xf>(v); v = dpp_max<0x114, 0xf>(v); v = dpp_max<0x118, 0xf>(v); v = dpp_max<0x142, 0xa>(v); v = dpp_max<0x143, 0xc>(v);
+  return __builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, v), 63));
+}
+__device__ __forceinline__ int wave_min(int v)
+{
+  v = dpp_min<0x111, 0xf>(v); v = dpp_min<0x112, 0xf>(v); v = dpp_min<0x114, 0xf>(v); v = dpp_min<0x118, 0xf>(v); v = dpp_min<0x142, 0xa>(v); v = dpp_min<0x143, 0xc>(v);
+  return __builtin_amdgcn_readlane(v, 63);
+}
+// a finished sum over the lanes of a wave, in every lane
+__device__ __forceinline__ float lanes_total(float v)
+{
+  v = wave_sum(v);
+  return __builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, v), 63));
+}
+
 // One row's experts, by one wave: lane k < top ends with the k-th choice and its weight.  Equal choice scores: the lower index.
 __device__ __forceinline__ void route_row(const float* z, const float* correction, const int n, const int top, const float scale, const int lane, int& expert, float& weight)
 {
   constexpr int PER = EXPERTS_MAX / 64;
   float s[PER], c[PER], m = -INFINITY, sum = 0.0f;
 #pragma unroll
-  for (int i = 0; i < PER; i++) { const int e = lane + 64 * i; s[i] = e < n ? z[e] : -INFINITY; m = fmaxf(m, s[i]); }
+  for (int i = 0; i < PER; i++) { const int e = lane + 64 * i; s[i] = e < n ? z[e] : -INFINITY; c[i] = e < n && correction ? correction[e] : 0.0f; m = fmaxf(m, s[i]); }
+  m = wave_max(m);
 #pragma unroll
-  for (int o = 32; o; o >>= 1) m = fmaxf(m, __shfl_xor(m, o));
-#pragma unroll
-  for (int i = 0; i < PER; i++) { s[i] = expf(s[i] - m); sum += s[i]; }
-#pragma unroll
-  for (int o = 32; o; o >>= 1) sum += __shfl_xor(sum, o);
+  for (int i = 0; i < PER; i++) if (64 * i < n) { s[i] = expf(s[i] - m); sum += s[i]; }
+  sum = lanes_total(sum);
 #pragma unroll
   for (int i = 0; i < PER; i++) {
-    const int e = lane + 64 * i;
-    s[i] /= sum;
-    c[i] = e < n ? s[i] + (correction ? correction[e] : 0.0f) : -INFINITY;
+    if (64 * i < n) s[i] /= sum;
+    c[i] = lane + 64 * i < n ? s[i] + c[i] : -INFINITY;
   }
   expert = 0; weight = 0.0f;
   float total = 0.0f;
   for (int k = 0; k < top; k++) {
     float bv = -INFINITY, bs = 0.0f; int be = n - 1;     // (always a valid expert, also if the scores are not numbers)
 #pragma unroll
-    for (int i = 0; i < PER; i++) { const int e = lane + 64 * i; if (e < n && c[i] > bv) { bv = c[i]; be = e; bs = s[i]; } }
-#pragma unroll
-    for (int o = 32; o; o >>= 1) {
-      const float ov = __shfl_xor(bv, o), os = __shfl_xor(bs, o); const int oe = __shfl_xor(be, o);
-      if (ov > bv || (ov == bv && oe < be)) { bv = ov; be = oe; bs = os; }
-    }
+    for (int i = 0; i < PER; i++) if (64 * i < n && c[i] > bv) { bv = c[i]; be = lane + 64 * i; bs = s[i]; }
+    const float most = wave_max(bv);
+    be = wave_min(bv == most ? be : n - 1);
+    bs = __builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, bs), be & 63));
     total += bs;
     if (lane == k) { expert = be; weight = bs; }
 #pragma unroll
@@ -47,12 +66,6 @@ __device__ __forceinline__ void route_row(const float* z, const float* correctio
   weight = weight / (total + 1e-20f) * scale;
 }
 
-// a finished sum over the lanes of a wave, in every lane
-__device__ __forceinline__ float lanes_total(float v)
-{
-  v = wave_sum(v);
-  return __builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, v), 63));
-}
 // eight activations times eight weights
 template <typename AT> __device__ __forceinline__ float dot8(const AT* x, const u32x4 w, float s)
 {
@@ -69,62 +82,113 @@ template <typename AT> __device__ __forceinline__ float dot8(const AT* x, const 
 }
 
 // ------------------------------------------------------------------------------------------
-// A few rows, gate and up: blockIdx x = outputs, y = slot (the chosen experts, then the shared one), z = row.  A wave makes two outputs;
-// every wave routes its row itself, and the first work-group of a slot and row leaves the choice for the output product.
+// Up to EXPERTS_FEW rows.  The gate and up kernel takes blockIdx x = outputs, y = entry; a wave makes two outputs of every row of its
+// entry, so that a matrix is read once however many rows chose it.  The entries of one row are its choices, and every wave routes the
+// row itself; for more rows a launch before it routes them and lists the experts that were chosen.  The last entry is the shared one.
 // ------------------------------------------------------------------------------------------
+struct FewEntry { int32_t expert, n_rows; uint8_t row[EXPERTS_FEW], slot[EXPERTS_FEW]; };
+static_assert(sizeof(FewEntry) == EXPERTS_FEW_WORDS * 4, "size of a listed expert");
 struct FewGateUp {
-  const uint16_t *w, *ws; int ldw, gu_rows; int n, top, ff, ff_s; float scale, limit, limit_s; int glu, glu_s; int mid_p, active;
+  const uint16_t *w, *ws; int ldw, gu_rows; int n, top, ff, ff_s; float scale, limit, limit_s; int glu, glu_s; int mid_p, active; int n_rows;
 };
-template <typename AT>
-__global__ __launch_bounds__(256) void experts_gateup_kernel(const FewGateUp p, const float* z, const float* correction, const AT* h, const int64_t ldh, int32_t* sel, AT* mid)
+
+__global__ __launch_bounds__(64 * EXPERTS_FEW) void experts_few_kernel(const float* z, const float* correction, const int n, const int top, const float scale, const int n_rows, float* wgt, FewEntry* list, int32_t* n_list)
 {
-  const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), slot = blockIdx.y;
-  const int64_t row = blockIdx.z;
-  const bool shared = slot == p.top;
+  __shared__ __align__(4) int8_t slot_of[EXPERTS_FEW][EXPERTS_MAX];   // the choice of a row that is this expert, -1: none
+  __shared__ int wave_count[EXPERTS_FEW];
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, tid = threadIdx.x;
+  for (int i = tid; i < EXPERTS_FEW * EXPERTS_MAX / 4; i += 64 * EXPERTS_FEW) reinterpret_cast<int32_t*>(&slot_of[0][0])[i] = -1;
+  __syncthreads();
+  if (wave < n_rows) {
+    int e; float w;
+    route_row(z + (int64_t)wave * n, correction, n, top, scale, lane, e, w);
+    if (lane < top) { wgt[wave * top + lane] = w; slot_of[wave][e] = (int8_t)lane; }
+  }
+  __syncthreads();
+  // a thread per expert: the chosen ones in order
+  static_assert(64 * EXPERTS_FEW >= EXPERTS_MAX, "a thread per expert");
+  FewEntry x{tid, 0, {}, {}};
+  if (tid < n)
+#pragma unroll
+    for (int r = 0; r < EXPERTS_FEW; r++)
+      if (slot_of[r][tid] >= 0) { x.row[x.n_rows] = (uint8_t)r; x.slot[x.n_rows] = (uint8_t)slot_of[r][tid]; x.n_rows++; }
+  const uint64_t chosen = __ballot(x.n_rows > 0);
+  if (lane == 0) wave_count[wave] = __popcll(chosen);
+  __syncthreads();
+  int at = __popcll(chosen & ((1ull << lane) - 1)), total = 0;
+  for (int i = 0; i < EXPERTS_FEW; i++) { if (i < wave) at += wave_count[i]; total += wave_count[i]; }
+  if (x.n_rows) list[at] = x;
+  if (tid == 0) *n_list = total;
+}
+
+template <typename AT, int NB>
+__global__ __launch_bounds__(256) void experts_gateup_kernel(const FewGateUp p, const float* z, const float* correction, const float* wgt, const FewEntry* list, const int32_t* n_list, const AT* h, const int64_t ldh, int32_t* sel, AT* mid)
+{
+  constexpr int UNROLL = NB == 1 ? 2 : 1;
+  const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), entry = blockIdx.y;
+  const bool shared = p.ws && entry == (int)gridDim.y - 1;
   const int ff = shared ? p.ff_s : p.ff, j0 = (blockIdx.x * 4 + wave) * 2;
   if (j0 >= ff) return;
   const uint16_t* W = p.ws;
   float weight = 1.0f;
+  int nb = p.n_rows;
   if (!shared) {
-    int e; float wt;
-    route_row(z + row * p.n, correction, p.n, p.top, p.scale, lane, e, wt);
-    if (j0 == 0 && lane == slot) sel[row * p.top + slot] = e;
-    e = __shfl(e, slot); weight = __shfl(wt, slot);
-    W = p.w + (int64_t)e * p.gu_rows * p.ldw;
+    if constexpr (NB == 1) {
+      int e; float wt;
+      route_row(z, correction, p.n, p.top, p.scale, lane, e, wt);
+      if (j0 == 0 && lane == entry) sel[entry] = e;
+      W = p.w + (int64_t)__shfl(e, entry) * p.gu_rows * p.ldw; weight = __shfl(wt, entry);
+    } else {
+      if (entry >= *n_list) return;
+      W = p.w + (int64_t)list[entry].expert * p.gu_rows * p.ldw; nb = list[entry].n_rows;
+    }
   }
   const int j1 = min(j0 + 1, ff - 1);
   const uint16_t* wr[4] = {W + (int64_t)glu_row(j0, 0) * p.ldw, W + (int64_t)glu_row(j0, 1) * p.ldw, W + (int64_t)glu_row(j1, 0) * p.ldw, W + (int64_t)glu_row(j1, 1) * p.ldw};
-  const AT* x = h + row * ldh;
-  float acc[4] = {0.0f, 0.0f, 0.0f, 0.0f};
-#pragma unroll 2
+  const AT* x[NB];
+#pragma unroll
+  for (int b = 0; b < NB; b++) x[b] = h + (int64_t)(NB == 1 || b >= nb ? 0 : shared ? b : list[entry].row[b]) * ldh;
+  float acc[NB][4];
+#pragma unroll
+  for (int b = 0; b < NB; b++)
+#pragma unroll
+    for (int i = 0; i < 4; i++) acc[b][i] = 0.0f;
+#pragma unroll UNROLL
   for (int k = lane * 8; k < p.ldw; k += 512) {
     u32x4 v[4];
 #pragma unroll
     for (int i = 0; i < 4; i++) v[i] = *reinterpret_cast<const u32x4*>(wr[i] + k);
 #pragma unroll
-    for (int i = 0; i < 4; i++) acc[i] = dot8<AT>(x + k, v[i], acc[i]);
+    for (int b = 0; b < NB; b++) {
+      if (b >= nb) break;
+#pragma unroll
+      for (int i = 0; i < 4; i++) acc[b][i] = dot8<AT>(x[b] + k, v[i], acc[b][i]);
+    }
   }
 #pragma unroll
-  for (int i = 0; i < 4; i++) acc[i] = lanes_total(acc[i]);
-  if (lane < 2 && j0 + lane < ff)
-    put_act<AT>(mid, row * p.active + slot * p.mid_p + j0 + lane,
-                glu_pair(shared ? p.glu_s : p.glu, shared ? p.limit_s : p.limit, lane ? acc[2] : acc[0], lane ? acc[3] : acc[1]) * weight);
+  for (int b = 0; b < NB; b++) {
+    if (b >= nb) break;
+#pragma unroll
+    for (int i = 0; i < 4; i++) acc[b][i] = lanes_total(acc[b][i]);
+    const int row = NB == 1 ? 0 : shared ? b : list[entry].row[b], slot = NB == 1 ? entry : shared ? p.top : list[entry].slot[b];
+    if (NB > 1) weight = shared ? 1.0f : wgt[row * p.top + slot];
+    if (lane < 2 && j0 + lane < ff)
+      put_act<AT>(mid, (int64_t)row * p.active + slot * p.mid_p + j0 + lane,
+                  glu_pair(shared ? p.glu_s : p.glu, shared ? p.limit_s : p.limit, lane ? acc[b][2] : acc[b][0], lane ? acc[b][3] : acc[b][1]) * weight);
+  }
 }
 
-// ------------------------------------------------------------------------------------------
-// A few rows, output: a wave makes two outputs of a row over all its slots, then the residual update.
-// ------------------------------------------------------------------------------------------
+// The output product of one row: a wave makes two outputs over all choices, then the residual update.
 template <typename AT>
-__global__ __launch_bounds__(256) void experts_down_kernel(const uint16_t* w, const uint16_t* ws, const int ldw, const int lds, const int top, const int active, const int width, const int n_experts,
+__global__ __launch_bounds__(256) void experts_down_kernel(const uint16_t* w, const uint16_t* ws, const int ldw, const int lds, const int top, const int width, const int n_experts,
                                                            const int32_t* sel, const AT* mid, const LinEpi e)
 {
   const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
-  const int64_t row = blockIdx.y;
   const int o0 = (blockIdx.x * 4 + wave) * 2;
   if (o0 >= width) return;
   const int o1 = min(o0 + 1, width - 1);
   float acc[2] = {0.0f, 0.0f};
-  const AT* x = mid + row * active;
+  const AT* x = mid;
   auto slot = [&](const uint16_t* m, int ld) {
     const uint16_t *a = m + (int64_t)o0 * ld, *b = m + (int64_t)o1 * ld;
 #pragma unroll 2
@@ -135,26 +199,116 @@ __global__ __launch_bounds__(256) void experts_down_kernel(const uint16_t* w, co
     x += ld;
   };
 #pragma unroll 4
-  for (int s = 0; s < top; s++) slot(w + (int64_t)min(max(sel[row * top + s], 0), n_experts - 1) * width * ldw, ldw);
+  for (int s = 0; s < top; s++) slot(w + (int64_t)min(max(sel[s], 0), n_experts - 1) * width * ldw, ldw);
   if (ws) slot(ws, lds);
   const float y0 = lanes_total(acc[0]), y1 = lanes_total(acc[1]);
-  if (lane < 2 && o0 + lane < width) epi_one<AT>(e, o0 + lane, (int)row, lane ? y1 : y0);
+  if (lane < 2 && o0 + lane < width) epi_one<AT>(e, o0 + lane, 0, lane ? y1 : y0);
+}
+
+// That of several rows, an entry at a time (blockIdx as in the gate and up kernel): outputs of every choice, summed by experts_sum_kernel.
+template <typename AT, int NB>
+__global__ __launch_bounds__(256) void experts_out_kernel(const uint16_t* w, const uint16_t* ws, const int ldw, const int lds, const int top, const int active, const int width, const int n_rows,
+                                                          const FewEntry* list, const int32_t* n_list, const AT* mid, float* y, float* ys)
+{
+  const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), entry = blockIdx.y;
+  const bool shared = ws && entry == (int)gridDim.y - 1;
+  const int o0 = (blockIdx.x * 4 + wave) * 2;
+  if (o0 >= width || (!shared && entry >= *n_list)) return;
+  const int o1 = min(o0 + 1, width - 1), ld = shared ? lds : ldw, nb = shared ? n_rows : list[entry].n_rows;
+  const uint16_t* m = shared ? ws : w + (int64_t)list[entry].expert * width * ldw;
+  const uint16_t *wa = m + (int64_t)o0 * ld, *wb = m + (int64_t)o1 * ld;
+  int row[NB], slot[NB];
+  const AT* x[NB];
+  float acc[NB][2];
+#pragma unroll
+  for (int b = 0; b < NB; b++) {
+    row[b] = b >= nb ? 0 : shared ? b : list[entry].row[b]; slot[b] = b >= nb ? 0 : shared ? top : list[entry].slot[b];
+    x[b] = mid + (int64_t)row[b] * active + slot[b] * ldw;
+    acc[b][0] = acc[b][1] = 0.0f;
+  }
+  for (int k = lane * 8; k < ld; k += 512) {
+    const u32x4 va = *reinterpret_cast<const u32x4*>(wa + k), vb = *reinterpret_cast<const u32x4*>(wb + k);
+#pragma unroll
+    for (int b = 0; b < NB; b++) {
+      if (b >= nb) break;
+      acc[b][0] = dot8<AT>(x[b] + k, va, acc[b][0]); acc[b][1] = dot8<AT>(x[b] + k, vb, acc[b][1]);
+    }
+  }
+#pragma unroll
+  for (int b = 0; b < NB; b++) {
+    if (b >= nb) break;
+    const float y0 = lanes_total(acc[b][0]), y1 = lanes_total(acc[b][1]);
+    if (lane < 2 && o0 + lane < width) (shared ? ys + (int64_t)row[b] * width : y + ((int64_t)row[b] * top + slot[b]) * width)[o0 + lane] = lane ? y1 : y0;
+  }
 }
 
 // ------------------------------------------------------------------------------------------
 // More rows: routing (a wave a row), the (row, choice) pairs ordered by expert with their tiles (one work-group), grouped products
 // (cai_linear_bf16.hip), and the sum of a row's outputs with the residual update.
 // ------------------------------------------------------------------------------------------
-__global__ __launch_bounds__(256) void experts_route_kernel(const float* z, const float* correction, const int n, const int top, const float scale, const int n_rows, int32_t* sel, float* wgt)
+// Router scores of 16 rows and their choices: eight waves share the width, 16 ET experts at a time; the matrix cores multiply as in the
+// other products (bfloat16, or exactly widened weights in 32-bit), the sums meet in LDS.
+template <typename AT, int ET>
+__global__ __launch_bounds__(512) void experts_route_kernel(const uint16_t* W, const int ldw, const AT* h, const int64_t ldh, const float* correction, const int n, const int top, const float scale, const int n_rows, int32_t* sel, float* wgt)
 {
-  const int lane = threadIdx.x & 63; const int64_t row = blockIdx.x * 4 + (threadIdx.x >> 6);
-  if (row >= n_rows) return;
-  int e; float w;
-  route_row(z + row * n, correction, n, top, scale, lane, e, w);
-  if (lane < top) { sel[row * top + lane] = e; wgt[row * top + lane] = w; }
+  extern __shared__ float lds[];                         // [8][16 ET][16] sums, [16][n] scores
+  constexpr int STEP = sizeof(AT) == 2 ? 32 : 16, AHEAD = 8;
+  float* z = lds + 8 * 16 * ET * 16;
+  const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), fr = lane & 15, fg = lane >> 4, r0 = blockIdx.x * 16;
+  const AT* xp = h + (int64_t)min(r0 + fr, n_rows - 1) * ldh + fg * (STEP / 4);
+  for (int e0 = 0; e0 < n; e0 += 16 * ET) {
+    const uint16_t* wp[ET]; f32x4 acc[ET];
+#pragma unroll
+    for (int t = 0; t < ET; t++) { wp[t] = W + (int64_t)min(e0 + t * 16 + fr, n - 1) * ldw + fg * (STEP / 4); acc[t] = f32x4{0.0f, 0.0f, 0.0f, 0.0f}; }
+    for (int k0 = wave * STEP; k0 < ldw; k0 += 8 * STEP * AHEAD) {
+      u32x4 x[AHEAD], wv[AHEAD][ET];
+#pragma unroll
+      for (int a = 0; a < AHEAD; a++) {                  // (turns past the width repeat the first one and are not used)
+        const int k = k0 + a * 8 * STEP < ldw ? k0 + a * 8 * STEP : k0;
+        x[a] = *reinterpret_cast<const u32x4*>(xp + k);
+#pragma unroll
+        for (int t = 0; t < ET; t++) {
+          if constexpr (sizeof(AT) == 2) wv[a][t] = *reinterpret_cast<const u32x4*>(wp[t] + k);
+          else { const uint2 u = *reinterpret_cast<const uint2*>(wp[t] + k); wv[a][t] = u32x4{u.x << 16, u.x & 0xffff0000u, u.y << 16, u.y & 0xffff0000u}; }
+        }
+      }
+#pragma unroll
+      for (int a = 0; a < AHEAD; a++) {
+        if (k0 + a * 8 * STEP >= ldw) continue;
+#pragma unroll
+        for (int t = 0; t < ET; t++) {
+          if constexpr (sizeof(AT) == 2) acc[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, wv[a][t]), __builtin_bit_cast(bf16x8, x[a]), acc[t], 0, 0, 0);
+          else {
+            const f32x4 wf = __builtin_bit_cast(f32x4, wv[a][t]), xf = __builtin_bit_cast(f32x4, x[a]);
+#pragma unroll
+            for (int q = 0; q < 4; q++) acc[t] = __builtin_amdgcn_mfma_f32_16x16x4f32(wf[q], xf[q], acc[t], 0, 0, 0);
+          }
+        }
+      }
+    }
+    __syncthreads();
+#pragma unroll
+    for (int t = 0; t < ET; t++)
+#pragma unroll
+      for (int i = 0; i < 4; i++) lds[(wave * 16 * ET + t * 16 + fg * 4 + i) * 16 + fr] = acc[t][i];
+    __syncthreads();
+    for (int i = tid; i < 16 * 16 * ET; i += 512) {
+      const int e = i >> 4, r = i & 15;
+      float s = 0.0f;
+#pragma unroll
+      for (int v = 0; v < 8; v++) s += lds[(v * 16 * ET + e) * 16 + r];
+      if (e0 + e < n) z[r * n + e0 + e] = s;
+    }
+  }
+  __syncthreads();
+  for (int r = wave; r < 16 && r0 + r < n_rows; r += 8) {
+    int e; float w;
+    route_row(z + r * n, correction, n, top, scale, lane, e, w);
+    if (lane < top) { sel[(int64_t)(r0 + r) * top + lane] = e; wgt[(int64_t)(r0 + r) * top + lane] = w; }
+  }
 }
 
-__global__ __launch_bounds__(1024) void experts_order_kernel(const int32_t* sel, const int n, const int pairs, int32_t* order, int32_t* tiles, int32_t* n_tiles)
+__global__ __launch_bounds__(1024) void experts_order_kernel(const int32_t* sel, const int n, const int pairs, const int tile, int32_t* order, int32_t* tiles, int32_t* n_tiles)
 {
   __shared__ int count[EXPERTS_MAX], at[EXPERTS_MAX], tile0[EXPERTS_MAX];
   const int tid = threadIdx.x;
@@ -165,7 +319,7 @@ __global__ __launch_bounds__(1024) void experts_order_kernel(const int32_t* sel,
   if (tid < 64) {                          // running sums of counts and tiles over the experts, a wave
     int base = 0, tbase = 0;
     for (int e0 = 0; e0 < n; e0 += 64) {
-      const int e = e0 + tid, c = e < n ? count[e] : 0, t = (c + BANK_TILE - 1) / BANK_TILE;
+      const int e = e0 + tid, c = e < n ? count[e] : 0, t = (c + tile - 1) / tile;
       int a = c, b = t;
       for (int o = 1; o < 64; o <<= 1) { const int x = __shfl_up(a, o), y = __shfl_up(b, o); if (tid >= o) { a += x; b += y; } }
       if (e < n) { at[e] = base + a - c; tile0[e] = tbase + b - t; }
@@ -176,7 +330,7 @@ __global__ __launch_bounds__(1024) void experts_order_kernel(const int32_t* sel,
   __syncthreads();
   for (int e = tid; e < n; e += 1024) {
     int t = tile0[e];
-    for (int c = 0; c < count[e]; c += BANK_TILE, t++) { tiles[3 * t] = e; tiles[3 * t + 1] = at[e] + c; tiles[3 * t + 2] = min(BANK_TILE, count[e] - c); }
+    for (int c = 0; c < count[e]; c += tile, t++) { tiles[3 * t] = e; tiles[3 * t + 1] = at[e] + c; tiles[3 * t + 2] = min(tile, count[e] - c); }
   }
   __syncthreads();
   for (int i = tid; i < pairs; i += 1024) order[atomicAdd(&at[sel[i]], 1)] = i;
@@ -193,25 +347,49 @@ __global__ __launch_bounds__(256) void experts_sum_kernel(const float* y, const 
   }
 }
 
+template <typename AT, int NB>
+static void run_few(const NetExperts& x, int width, const AT* h, int64_t ldh, int n_rows, const ExpertBuf& b, const LinEpi& res)
+{
+  auto st = ctx().stream;
+  const uint16_t *sg = x.s_gateup ? (const uint16_t*)x.s_gateup->data : nullptr, *sd = x.s_down ? (const uint16_t*)x.s_down->data : nullptr;
+  const FewGateUp p{(const uint16_t*)x.gateup->data, sg, (int)x.gateup->ld, x.gu_rows(), x.n, x.top, x.ff, x.ff_shared,
+                    x.scale, x.limit, x.limit_shared, x.glu, x.glu_shared, x.mid_p(), x.active(), n_rows};
+  FewEntry* list = (FewEntry*)b.few;
+  if (NB > 1) hipLaunchKernelGGL(experts_few_kernel, dim3(1), dim3(64 * EXPERTS_FEW), 0, st, b.z, x.correction, x.n, x.top, x.scale, n_rows, b.wgt, list, b.n_tiles);
+  const int entries = NB == 1 ? x.top : std::min(x.n, n_rows * x.top);
+  hipLaunchKernelGGL((experts_gateup_kernel<AT, NB>), dim3((std::max(x.ff, x.ff_shared) + 7) / 8, entries + (sg ? 1 : 0)), dim3(256), 0, st, p, b.z, x.correction, b.wgt, list, b.n_tiles, h, ldh, b.sel, (AT*)b.mid);
+  const int lds = x.s_down ? (int)x.s_down->ld : 0;
+  const dim3 outs((width + 7) / 8, NB == 1 ? 1 : entries + (sd ? 1 : 0));
+  if constexpr (NB == 1)
+    hipLaunchKernelGGL(experts_down_kernel<AT>, outs, dim3(256), 0, st, (const uint16_t*)x.down->data, sd, (int)x.down->ld, lds, x.top, width, x.n, b.sel, (const AT*)b.mid, res);
+  else {
+    hipLaunchKernelGGL((experts_out_kernel<AT, NB>), outs, dim3(256), 0, st, (const uint16_t*)x.down->data, sd, (int)x.down->ld, lds, x.top, x.active(), width, n_rows, list, b.n_tiles, (const AT*)b.mid, b.y, b.ys);
+    hipLaunchKernelGGL(experts_sum_kernel<AT>, dim3(std::min((width + 255) / 256, 32), n_rows), dim3(256), 0, st, b.y, sd ? b.ys : nullptr, x.top, width, res);
+  }
+}
+
 template <typename AT>
 static int run(const NetExperts& x, int width, int act_t, const AT* h, int64_t ldh, int n_rows, const ExpertBuf& b, const LinEpi& res)
 {
   auto st = ctx().stream;
   int rc;
-  { LinEpi e; e.y = b.z; e.ldy = x.n; if ((rc = launch_lin(x.router, act_t, h, ldh, n_rows, e))) return rc; }
   if (n_rows <= EXPERTS_FEW) {
-    const FewGateUp p{(const uint16_t*)x.gateup->data, x.s_gateup ? (const uint16_t*)x.s_gateup->data : nullptr, (int)x.gateup->ld, x.gu_rows(), x.n, x.top, x.ff, x.ff_shared,
-                      x.scale, x.limit, x.limit_shared, x.glu, x.glu_shared, x.mid_p(), x.active()};
-    const int ff = std::max(x.ff, x.ff_shared);
-    hipLaunchKernelGGL(experts_gateup_kernel<AT>, dim3((ff + 7) / 8, x.top + (x.ff_shared ? 1 : 0), n_rows), dim3(256), 0, st, p, b.z, x.correction, h, ldh, b.sel, (AT*)b.mid);
-    hipLaunchKernelGGL(experts_down_kernel<AT>, dim3((width + 7) / 8, n_rows), dim3(256), 0, st, (const uint16_t*)x.down->data, x.s_down ? (const uint16_t*)x.s_down->data : nullptr,
-                       (int)x.down->ld, x.s_down ? (int)x.s_down->ld : 0, x.top, x.active(), width, x.n, b.sel, (const AT*)b.mid, res);
+    LinEpi e; e.y = b.z; e.ldy = x.n;
+    if ((rc = launch_lin(x.router, act_t, h, ldh, n_rows, e))) return rc;
+    if (n_rows == 1) run_few<AT, 1>(x, width, h, ldh, n_rows, b, res);
+    else if (n_rows == 2) run_few<AT, 2>(x, width, h, ldh, n_rows, b, res);
+    else if (n_rows <= 4) run_few<AT, 4>(x, width, h, ldh, n_rows, b, res);
+    else run_few<AT, 8>(x, width, h, ldh, n_rows, b, res);
     CAI_HIP(hipGetLastError());
     return CAI_OK;
   }
-  hipLaunchKernelGGL(experts_route_kernel, dim3((n_rows + 3) / 4), dim3(256), 0, st, b.z, x.correction, x.n, x.top, x.scale, n_rows, b.sel, b.wgt);
-  hipLaunchKernelGGL(experts_order_kernel, dim3(1), dim3(1024), 0, st, b.sel, x.n, n_rows * x.top, b.order, b.tiles, b.n_tiles);
-  BankList l{b.tiles, b.n_tiles, b.order, b.wgt, x.top, x.max_tiles(n_rows)};
+#define ROUTE(ET) hipLaunchKernelGGL((experts_route_kernel<AT, ET>), dim3((n_rows + 15) / 16), dim3(512), (8 * 16 * ET * 16 + 16 * x.n) * sizeof(float), st, \
+                                     (const uint16_t*)x.router->data, (int)x.router->ld, h, ldh, x.correction, x.n, x.top, x.scale, n_rows, b.sel, b.wgt)
+  if (x.n <= 16) ROUTE(1); else if (x.n <= 32) ROUTE(2); else ROUTE(4);
+#undef ROUTE
+  const int tile = n_rows * x.top >= x.n * 96 ? BANK_TILE_MAX : BANK_TILE;       // (by the mean number of rows of an expert)
+  hipLaunchKernelGGL(experts_order_kernel, dim3(1), dim3(1024), 0, st, b.sel, x.n, n_rows * x.top, tile, b.order, b.tiles, b.n_tiles);
+  BankList l{b.tiles, b.n_tiles, b.order, b.wgt, x.top, tile, x.max_tiles(n_rows, tile)};
   { LinEpi e; e.mode = EPI_GLU; e.h = b.mid; e.ldh = x.mid_p(); e.glu = x.glu; e.limit = x.limit; if ((rc = launch_lin_bank(x.gateup, x.gu_rows(), act_t, h, ldh, l, e))) return rc; }
   l.div = 0;
   { LinEpi e; e.y = b.y; e.ldy = width; if ((rc = launch_lin_bank(x.down, width, act_t, b.mid, x.mid_p(), l, e))) return rc; }

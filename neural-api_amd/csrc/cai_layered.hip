@@ -264,7 +264,7 @@ static void drop_graphs(LayeredNet* n)
 static void free_rows(LayeredNet* n)
 {
   void* p[] = {n->x, n->x0, n->proj, n->yl, n->yr, n->part, n->h, n->mid, n->att, n->attl, n->qbuf, n->ra, n->rgb, n->db.q, n->db.k, n->db.v, n->db.g, n->db.beta, n->db.o, n->db.za, n->db.zg, n->db.w, n->db.qt, n->db.qk, n->db.gt, n->cat,
-               n->sb.x, n->sb.B, n->sb.C, n->sb.dt, n->sb.cb, n->sb.y, n->eb.z, n->eb.wgt, n->eb.y, n->eb.ys, n->eb.sel, n->eb.order, n->eb.tiles, n->eb.n_tiles, n->eb.mid, n->eb.mid_s};
+               n->sb.x, n->sb.B, n->sb.C, n->sb.dt, n->sb.cb, n->sb.bt, n->sb.fac, n->sb.y, n->eb.z, n->eb.wgt, n->eb.y, n->eb.ys, n->eb.sel, n->eb.order, n->eb.tiles, n->eb.n_tiles, n->eb.few, n->eb.mid, n->eb.mid_s};
   for (void* q : p) if (q) (void)hipFree(q);
   n->x = n->x0 = n->proj = n->yl = n->yr = n->part = nullptr;
   n->h = n->mid = n->att = n->attl = n->qbuf = n->ra = n->rgb = nullptr;
@@ -303,9 +303,10 @@ static int ensure_rows(LayeredNet* n, int rows)
       (rc = get((void**)&n->db.w, RS * n->w_hd * 4)) || (rc = get((void**)&n->db.qt, RS * n->w_qt * 4)) || (rc = get((void**)&n->db.qk, RS * n->w_qk * 4)) ||
       (rc = get((void**)&n->db.gt, std::max(RS * n->w_gt1, (R / DELTA_CHUNK + n->max_seq + 1) * n->w_qt + 4) * 4)) ||
       (rc = get(&n->cat, R * n->ld_cat * n->es)) ||
-      (rc = get((void**)&n->sb.x, R * n->w_sx * 4)) || (rc = get((void**)&n->sb.B, R * n->w_sb * 4)) || (rc = get((void**)&n->sb.C, R * n->w_sb * 4)) ||
+      (rc = get((void**)&n->sb.x, (R + SSD_CHUNK) * n->w_sx * 4)) || (rc = get((void**)&n->sb.B, R * n->w_sb * 4)) || (rc = get((void**)&n->sb.C, (R + SSD_CHUNK) * n->w_sb * 4)) ||
       (rc = get((void**)&n->sb.dt, R * n->w_sdt * 4)) || (rc = get((void**)&n->sb.cb, (R / SSD_CHUNK + n->max_seq + 1) * n->w_cb * 4)) || (rc = get((void**)&n->sb.y, R * n->w_sy * 4)) ||
-      (rc = get((void**)&n->eb.z, R * n->w_ez * 4)) || (rc = get((void**)&n->eb.sel, R * n->w_ep * 4)) || (rc = get((void**)&n->eb.wgt, R * n->w_ep * 4)) ||
+      (rc = get((void**)&n->sb.bt, (R / SSD_CHUNK + n->max_seq + 1) * n->w_sb * SSD_CHUNK * 4)) || (rc = get((void**)&n->sb.fac, (R / SSD_CHUNK + n->max_seq + 1) * n->w_sdt * SSD_FACTORS * 4)) ||
+      (rc = get((void**)&n->eb.z, EXPERTS_FEW * n->w_ez * 4)) || (rc = get((void**)&n->eb.few, n->w_ep ? (size_t)EXPERTS_MAX * EXPERTS_FEW_WORDS * 4 : 0)) || (rc = get((void**)&n->eb.sel, R * n->w_ep * 4)) || (rc = get((void**)&n->eb.wgt, R * n->w_ep * 4)) ||
       (rc = get((void**)&n->eb.order, R * n->w_ep * 4)) || (rc = get((void**)&n->eb.y, R * n->w_ep * w * 4)) || (rc = get((void**)&n->eb.ys, R * n->ld_ys * 4)) ||
       (rc = get((void**)&n->eb.tiles, n->w_ep ? ((R * n->w_ep + BANK_TILE - 1) / BANK_TILE + n->w_etiles) * 12 : 0)) || (rc = get((void**)&n->eb.n_tiles, n->w_ep ? 4 : 0)) ||
       (rc = get(&n->eb.mid, R * n->w_emid * n->es)) || (rc = get(&n->eb.mid_s, R * n->w_emid_s * n->es))) return rc;

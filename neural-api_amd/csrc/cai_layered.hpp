@@ -48,8 +48,8 @@ int launch_lin(const cai_qw_s* w, int act_t, const void* x, int64_t ldx, int n_t
 // The same over a bank of equal matrices stacked in w (mat_rows rows each): work lists of (matrix, first place, places) over an order
 // of activation rows.  Place p reads activation row order[p] / div (div 0: row p) and writes row p of e.h, scaled by
 // scale[order[p]] (GLU), or row order[p] of e.y (STORE).
-constexpr int BANK_TILE = 64;
-struct BankList { const int32_t *tiles, *n_tiles, *order; const float* scale; int div, max_tiles; };   // tiles [.][3], n_tiles on the device
+constexpr int BANK_TILE = 64, BANK_TILE_MAX = 128;      // most places of a list entry: one of the two
+struct BankList { const int32_t *tiles, *n_tiles, *order; const float* scale; int div, tile, max_tiles; };   // tiles [.][3], n_tiles on the device
 int launch_lin_bank(const cai_qw_s* w, int mat_rows, int act_t, const void* x, int64_t ldx, const BankList& l, const LinEpi& e);
 // float columns [col0, col0 + cols) of x -> rows of the chosen type, zero padded to ldo
 int launch_pack_rows(const float* x, int64_t ldx, int64_t col0, int cols, int n_tok, int act_t, void* out, int64_t ldo);
@@ -97,7 +97,7 @@ struct SsdDims {
   __host__ __device__ int inner() const { return heads * vdim; }
   __host__ __device__ int channels() const { return heads * vdim + 2 * groups * state; }
   __host__ __device__ int vdim_p() const { return (vdim + 3) & ~3; }   // row stride of the state
-  __host__ __device__ int np() const { return (state + 15) & ~15; }    // strides of the prompt buffers (zero filled)
+  __host__ __device__ int np() const { return (state + 63) & ~63; }    // strides of the prompt buffers (zero filled)
   __host__ __device__ int xp() const { return (vdim + 15) & ~15; }
 };
 struct KvView {                            // what a kernel needs to reach one attention run's pages
@@ -164,8 +164,8 @@ int delta_single(const DeltaDims& d, const DeltaIn& in, const DeltaW& w, const S
 // Columns of proj: z, x | B | C (before the convolution), dt.
 struct SsdIn { const float* proj; int64_t ldp; int oz, ox, odt; };
 struct SsdW { const float *conv, *conv_b, *dt_bias, *rate, *D, *norm; };   // taps [channels][taps]; rate = -exp(A_log)
-struct SsdBuf { float *x, *B, *C, *dt, *cb, *y; };                          // per-row scratch; cb: C B^T of every chunk and group
-constexpr int SSD_CHUNK = 64;
+struct SsdBuf { float *x, *B, *C, *dt, *cb, *bt, *fac, *y; };               // per-row scratch; per chunk: C B^T and B^T of every group, decay factors of every head
+constexpr int SSD_CHUNK = 64, SSD_FACTORS = 4 * SSD_CHUNK + 4;
 int ssd_prep(const SsdDims& d, const SsdIn& in, const SsdW& w, const SeqPool::StateRun& st, const StepRows& r, const SsdBuf& b);
 int ssd_walk(const SsdDims& d, const SsdW& w, const SeqPool::StateRun& st, const StepRows& r, const SsdBuf& b, const int32_t* chunks, int n_chunks, const int32_t* chunk0);
 int ssd_single(const SsdDims& d, const SsdIn& in, const SsdW& w, const SeqPool::StateRun& st, const StepRows& r, const SsdBuf& b);
@@ -183,12 +183,13 @@ struct NetExperts {
   int mid_p() const { return pad_to(ff, LIN_PAD); }
   int shared_p() const { return ff_shared ? pad_to(ff_shared, LIN_PAD) : 0; }
   int active() const { return top * mid_p() + shared_p(); }            // a row's gated activations, one slot after the other
-  int max_tiles(int rows) const { return (rows * top + BANK_TILE - 1) / BANK_TILE + n; }
+  int max_tiles(int rows, int tile) const { return (rows * top + tile - 1) / tile + n; }
 };
 constexpr int EXPERTS_MAX = 512, EXPERTS_TOP = 64;
 constexpr int EXPERTS_FEW = 8;             // up to so many rows take the gathering kernels
+constexpr int EXPERTS_FEW_WORDS = 2 + EXPERTS_FEW / 2;   // words of a listed expert: itself, its rows, which rows, which of their choices
 struct ExpertBuf {
-  float *z, *wgt, *y, *ys; int32_t *sel, *order, *tiles, *n_tiles; void *mid, *mid_s;
+  float *z, *wgt, *y, *ys; int32_t *sel, *order, *tiles, *n_tiles, *few; void *mid, *mid_s;
 };
 int experts_run(const NetExperts& x, int width, int act_t, const void* h, int64_t ldh, int n_rows, const ExpertBuf& b, const LinEpi& res);   // res: the residual update
 

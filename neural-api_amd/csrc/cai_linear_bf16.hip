@@ -292,11 +292,11 @@ static void run_gemm(const cai_qw_s* w, const AT* x, int64_t ldx, int n_tok, con
                      (const uint16_t*)w->data, x, (int)w->rows, (int)w->ld, ldx, n_tok, tm, tm * tn, e, BankList{});
 }
 
-template <typename AT>
+template <typename AT, int BM, int BN>
 static void run_bank(const cai_qw_s* w, int mat_rows, const AT* x, int64_t ldx, const BankList& l, const LinEpi& e)
 {
-  const int tm = l.max_tiles, tn = (mat_rows + 63) / 64;
-  hipLaunchKernelGGL((gemm_bf16<AT, BANK_TILE, 64, 2, 2, true>), dim3(tm * tn), dim3(256), 0, ctx().stream,
+  const int tm = l.max_tiles, tn = (mat_rows + BN - 1) / BN;
+  hipLaunchKernelGGL((gemm_bf16<AT, BM, BN, 2, 2, true>), dim3(tm * tn), dim3(256), 0, ctx().stream,
                      (const uint16_t*)w->data, x, mat_rows, (int)w->ld, ldx, 0, tm, tm * tn, e, l);
 }
 
@@ -304,8 +304,12 @@ int launch_lin_bank(const cai_qw_s* w, int mat_rows, int act_t, const void* x, i
 {
   CAI_REQUIRE(w->qtype == CAI_BF16 && mat_rows >= 1 && w->rows % mat_rows == 0 && ldx >= w->ld && l.max_tiles >= 1, "bf16 bank: matrices of %d rows of %lld, activation rows of %lld", mat_rows, (long long)w->rows, (long long)ldx);
   CAI_REQUIRE(e.mode == EPI_STORE || (e.mode == EPI_GLU && mat_rows % 32 == 0), "bf16 bank: a gated matrix needs whole blocks of 32 rows");
-  if (act_t == ACT_T_BF16) run_bank<bf16_t>(w, mat_rows, (const bf16_t*)x, ldx, l, e);
-  else run_bank<float>(w, mat_rows, (const float*)x, ldx, l, e);
+  CAI_REQUIRE(l.tile == BANK_TILE || l.tile == BANK_TILE_MAX, "bf16 bank: runs of %d places", l.tile);
+  if (act_t == ACT_T_BF16) {
+    if (l.tile == BANK_TILE_MAX) run_bank<bf16_t, BANK_TILE_MAX, 128>(w, mat_rows, (const bf16_t*)x, ldx, l, e);
+    else run_bank<bf16_t, BANK_TILE, 64>(w, mat_rows, (const bf16_t*)x, ldx, l, e);
+  } else if (l.tile == BANK_TILE_MAX) run_bank<float, BANK_TILE_MAX, 128>(w, mat_rows, (const float*)x, ldx, l, e);
+  else run_bank<float, BANK_TILE, 64>(w, mat_rows, (const float*)x, ldx, l, e);
   CAI_HIP(hipGetLastError());
   return CAI_OK;
 }
