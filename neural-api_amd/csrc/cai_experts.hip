@@ -246,25 +246,26 @@ __global__ __launch_bounds__(256) void experts_out_kernel(const uint16_t* w, con
 // More rows: routing (a wave a row), the (row, choice) pairs ordered by expert with their tiles (one work-group), grouped products
 // (cai_linear_bf16.hip), and the sum of a row's outputs with the residual update.
 // ------------------------------------------------------------------------------------------
-// Router scores of 16 rows and their choices: eight waves share the width, 16 ET experts at a time; the matrix cores multiply as in the
+// Router scores of 16 rows and their choices: sixteen waves share the width, 16 ET experts at a time; the matrix cores multiply as in the
 // other products (bfloat16, or exactly widened weights in 32-bit), the sums meet in LDS.
+constexpr int ROUTE_WAVES = 16;
 template <typename AT, int ET>
-__global__ __launch_bounds__(512) void experts_route_kernel(const uint16_t* W, const int ldw, const AT* h, const int64_t ldh, const float* correction, const int n, const int top, const float scale, const int n_rows, int32_t* sel, float* wgt)
+__global__ __launch_bounds__(64 * ROUTE_WAVES) void experts_route_kernel(const uint16_t* W, const int ldw, const AT* h, const int64_t ldh, const float* correction, const int n, const int top, const float scale, const int n_rows, int32_t* sel, float* wgt)
 {
-  extern __shared__ float lds[];                         // [8][16 ET][16] sums, [16][n] scores
+  extern __shared__ float lds[];                         // [ROUTE_WAVES][16 ET][16] sums, [16][n] scores
   constexpr int STEP = sizeof(AT) == 2 ? 32 : 16, AHEAD = 8;
-  float* z = lds + 8 * 16 * ET * 16;
+  float* z = lds + ROUTE_WAVES * 16 * ET * 16;
   const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), fr = lane & 15, fg = lane >> 4, r0 = blockIdx.x * 16;
   const AT* xp = h + (int64_t)min(r0 + fr, n_rows - 1) * ldh + fg * (STEP / 4);
   for (int e0 = 0; e0 < n; e0 += 16 * ET) {
     const uint16_t* wp[ET]; f32x4 acc[ET];
 #pragma unroll
     for (int t = 0; t < ET; t++) { wp[t] = W + (int64_t)min(e0 + t * 16 + fr, n - 1) * ldw + fg * (STEP / 4); acc[t] = f32x4{0.0f, 0.0f, 0.0f, 0.0f}; }
-    for (int k0 = wave * STEP; k0 < ldw; k0 += 8 * STEP * AHEAD) {
+    for (int k0 = wave * STEP; k0 < ldw; k0 += ROUTE_WAVES * STEP * AHEAD) {
       u32x4 x[AHEAD], wv[AHEAD][ET];
 #pragma unroll
       for (int a = 0; a < AHEAD; a++) {                  // (turns past the width repeat the first one and are not used)
-        const int k = k0 + a * 8 * STEP < ldw ? k0 + a * 8 * STEP : k0;
+        const int k = k0 + a * ROUTE_WAVES * STEP < ldw ? k0 + a * ROUTE_WAVES * STEP : k0;
         x[a] = *reinterpret_cast<const u32x4*>(xp + k);
 #pragma unroll
         for (int t = 0; t < ET; t++) {
@@ -274,7 +275,7 @@ __global__ __launch_bounds__(512) void experts_route_kernel(const uint16_t* W, c
       }
 #pragma unroll
       for (int a = 0; a < AHEAD; a++) {
-        if (k0 + a * 8 * STEP >= ldw) continue;
+        if (k0 + a * ROUTE_WAVES * STEP >= ldw) continue;
 #pragma unroll
         for (int t = 0; t < ET; t++) {
           if constexpr (sizeof(AT) == 2) acc[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, wv[a][t]), __builtin_bit_cast(bf16x8, x[a]), acc[t], 0, 0, 0);
@@ -292,16 +293,16 @@ __global__ __launch_bounds__(512) void experts_route_kernel(const uint16_t* W, c
 #pragma unroll
       for (int i = 0; i < 4; i++) lds[(wave * 16 * ET + t * 16 + fg * 4 + i) * 16 + fr] = acc[t][i];
     __syncthreads();
-    for (int i = tid; i < 16 * 16 * ET; i += 512) {
+    for (int i = tid; i < 16 * 16 * ET; i += 64 * ROUTE_WAVES) {
       const int e = i >> 4, r = i & 15;
       float s = 0.0f;
 #pragma unroll
-      for (int v = 0; v < 8; v++) s += lds[(v * 16 * ET + e) * 16 + r];
+      for (int v = 0; v < ROUTE_WAVES; v++) s += lds[(v * 16 * ET + e) * 16 + r];
       if (e0 + e < n) z[r * n + e0 + e] = s;
     }
   }
   __syncthreads();
-  for (int r = wave; r < 16 && r0 + r < n_rows; r += 8) {
+  for (int r = wave; r < 16 && r0 + r < n_rows; r += ROUTE_WAVES) {
     int e; float w;
     route_row(z + r * n, correction, n, top, scale, lane, e, w);
     if (lane < top) { sel[(int64_t)(r0 + r) * top + lane] = e; wgt[(int64_t)(r0 + r) * top + lane] = w; }
@@ -383,9 +384,9 @@ static int run(const NetExperts& x, int width, int act_t, const AT* h, int64_t l
     CAI_HIP(hipGetLastError());
     return CAI_OK;
   }
-#define ROUTE(ET) hipLaunchKernelGGL((experts_route_kernel<AT, ET>), dim3((n_rows + 15) / 16), dim3(512), (8 * 16 * ET * 16 + 16 * x.n) * sizeof(float), st, \
+#define ROUTE(ET) hipLaunchKernelGGL((experts_route_kernel<AT, ET>), dim3((n_rows + 15) / 16), dim3(64 * ROUTE_WAVES), (ROUTE_WAVES * 16 * ET * 16 + 16 * x.n) * sizeof(float), st, \
                                      (const uint16_t*)x.router->data, (int)x.router->ld, h, ldh, x.correction, x.n, x.top, x.scale, n_rows, b.sel, b.wgt)
-  if (x.n <= 16) ROUTE(1); else if (x.n <= 32) ROUTE(2); else ROUTE(4);
+  if (x.n <= 16) ROUTE(1); else ROUTE(2);
 #undef ROUTE
   const int tile = n_rows * x.top >= x.n * 96 ? BANK_TILE_MAX : BANK_TILE;       // (by the mean number of rows of an expert)
   hipLaunchKernelGGL(experts_order_kernel, dim3(1), dim3(1024), 0, st, b.sel, x.n, n_rows * x.top, tile, b.order, b.tiles, b.n_tiles);
