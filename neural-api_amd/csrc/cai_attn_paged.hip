@@ -1,6 +1,8 @@
 // Grouped-query attention over a paged key/value pool, in a sliding window or in fixed blocks of positions: key and value widths of
-// their own, optional per-head RMS norm of queries and keys, optional rotation of the first dimensions of a head, an explicit score
-// scale, an optional sigmoid gate on the heads' outputs.
+// their own, optional RMS norm of queries and keys (per head or over all heads at once), optional rotation of the first dimensions of
+// a head, optional growth of the queries with the position, an explicit score scale, an optional sigmoid gate on the heads' outputs.
+// The weights are a soft-max over the keys or, each key for itself, a sigmoid of the score with a logarithmic loss over the distance.
+// A run may read the pages that an earlier run has filled.
 //
 // Two forms: one work-group per (row, key/value head, slice of keys) for decoded tokens, short portions and the all-32-bit mode,
 // and a matrix-core form for prompts, whose key tile is one page.  Scores, soft-max and weights are 32-bit in both; the
@@ -32,16 +34,45 @@ template <typename T> __device__ __forceinline__ T* kv_page(const KvView& kv, in
   return reinterpret_cast<T*>(kv.base) + (int64_t)kv.table[slot * kv.ring + (key / PAGE_TOKENS) % kv.ring] * kv.page_elems;
 }
 
-// A query or key head of `dim` values by one wave, lane holds x[lane + 64 i]: RMS norm (gain null: none), then the rotation at
-// position pos.  The angle is reduced in turns with double precision before sine and cosine.
-__device__ __forceinline__ void head_vector(const float* x, const float* gain, const AttnDims& d, int pos, int lane, float* v)
+// What all query heads (or key heads) of a row share: the RMS norm's factor under whole_norm, and the queries' growth.
+struct RowFactors { float inv_q = 1.0f, inv_k = 1.0f, temp = 1.0f; };
+// by a work-group of 256, over the columns of proj; red: LDS for 8 floats
+__device__ __forceinline__ RowFactors row_factors(const AttnDims& d, const AttnIn& in, const float* p, int pos, bool with_k, float* red)
 {
-  float s = 0.0f, inv = 1.0f;
+  RowFactors f;
+  if (d.temp_every) f.temp = 1.0f + d.temp * logf((float)((pos + 1) / d.temp_every + 1));
+  if (!d.whole_norm) return f;
+  const int tid = threadIdx.x, nq = d.heads * d.dim, nk = with_k ? d.kv_heads * d.dim : 0;
+  float q = 0.0f, k = 0.0f;
+#pragma unroll 8
+  for (int c = tid; c < nq; c += 256) { const float v = p[in.oq + c]; q = fmaf(v, v, q); }
+#pragma unroll 4
+  for (int c = tid; c < nk; c += 256) { const float v = p[in.ok + c]; k = fmaf(v, v, k); }
+  q = wave_sum(q); k = wave_sum(k);
+  if ((tid & 63) == 63) { red[tid >> 6] = q; red[4 + (tid >> 6)] = k; }
+  __syncthreads();
+  f.inv_q = 1.0f / sqrtf((red[0] + red[1] + red[2] + red[3]) / (float)nq + d.eps);
+  if (with_k) f.inv_k = 1.0f / sqrtf((red[4] + red[5] + red[6] + red[7]) / (float)nk + d.eps);
+  return f;
+}
+
+// weight of a key `far` positions before the query, from the scaled product of the two
+__device__ __forceinline__ float sigmoid_weight(const AttnDims& d, int h, float score, int far)
+{
+  return 1.0f / (1.0f + expf(-(score - d.r1[h] * logf(1.0f + d.r2[h] * (float)far) + d.bias[h])));
+}
+
+// A query or key head of `dim` values by one wave, lane holds x[lane + 64 i]: RMS norm (gain null: none) with the factor `inv` or, without
+// whole_norm, one of its own, then the rotation at position pos, then `times`.  The angle is reduced in turns with double precision
+// before sine and cosine.
+__device__ __forceinline__ void head_vector(const float* x, const float* gain, float inv, const float times, const AttnDims& d, int pos, int lane, float* v)
+{
+  float s = 0.0f;
 #pragma unroll
   for (int i = 0; i < 4; i++) { const int c = lane + 64 * i; v[i] = c < d.dim ? x[c] : 0.0f; s = fmaf(v[i], v[i], s); }
   if (gain) {
     s = wave_sum(s);
-    inv = 1.0f / sqrtf(__builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, s), 63)) / (float)d.dim + d.eps);
+    if (!d.whole_norm) inv = 1.0f / sqrtf(__builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, s), 63)) / (float)d.dim + d.eps);
 #pragma unroll
     for (int i = 0; i < 4; i++) { const int c = lane + 64 * i; if (c < d.dim) v[i] *= inv * gain[c]; }
   }
@@ -59,6 +90,8 @@ __device__ __forceinline__ void head_vector(const float* x, const float* gain, c
     sincospif((float)(2.0 * (t - rint(t))), &sn, &cs);
     v[i] = lo ? v[i] * cs - o * sn : v[i] * cs + o * sn;
   }
+#pragma unroll
+  for (int i = 0; i < 4; i++) v[i] *= times;
 }
 __device__ __forceinline__ float out_gate(const AttnIn& in, int64_t row, int c)
 {
@@ -69,18 +102,23 @@ template <typename T>
 __global__ __launch_bounds__(256) void attn_prep_kernel(const AttnDims d, const KvView kv, const AttnIn in, const StepRows r, T* qbuf)
 {
   const int row = blockIdx.x, lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
+  __shared__ float red[8];
   const int pos = r.pos[row], slot = r.slot[row], tp = pos % PAGE_TOKENS;
   const float* p = in.proj + row * in.ldp;
+  const bool append = in.ok >= 0;
+  const RowFactors f = row_factors(d, in, p, pos, append, red);
   T* page = kv_page<T>(kv, slot, pos);
-  for (int u = wave; u < d.heads + d.kv_heads; u += 4) {
+  const int by_head = d.whole_norm ? d.dim : 0;            // gains of one head after the other, or shared
+  for (int u = wave; u < d.heads + (append ? d.kv_heads : 0); u += 4) {
     const bool is_q = u < d.heads; const int hh = is_q ? u : u - d.heads;
+    const float* gain = is_q ? in.qn : in.kn;
     float v[4];
-    head_vector(p + (is_q ? in.oq : in.ok) + hh * d.dim, is_q ? in.qn : in.kn, d, pos, lane, v);
+    head_vector(p + (is_q ? in.oq : in.ok) + hh * d.dim, gain ? gain + hh * by_head : nullptr, is_q ? f.inv_q : f.inv_k, is_q ? f.temp : 1.0f, d, pos, lane, v);
     T* dst = is_q ? qbuf + ((int64_t)row * d.heads + hh) * d.dim_p : page + ((int64_t)hh * PAGE_TOKENS + tp) * d.dim_p;
 #pragma unroll
     for (int i = 0; i < 4; i++) { const int c = lane + 64 * i; if (c < d.dim_p) dst[c] = (T)v[i]; }
   }
-  for (int c = threadIdx.x; c < d.kv_heads * d.vdim_p; c += 256) {
+  if (append) for (int c = threadIdx.x; c < d.kv_heads * d.vdim_p; c += 256) {
     const int hh = c / d.vdim_p, i = c % d.vdim_p;
     page[kv.v_off + ((int64_t)hh * PAGE_TOKENS + tp) * d.vdim_p + i] = (T)(i < d.vdim ? p[in.ov + hh * d.vdim + i] : 0.0f);
   }
@@ -88,8 +126,9 @@ __global__ __launch_bounds__(256) void attn_prep_kernel(const AttnDims d, const 
 
 // ------------------------------------------------------------------------------------------
 // Row form.  blockIdx: x slice, y = key/value head x group of HT query heads, z row.  SINGLE: the row is its entry's only one;
-// queries, the new key and the new value come from the projections and the new key/value are appended on the way.
-// part (more than one slice): per (row, head, slice) vdim_p weighted sums, the maximum and the normaliser.
+// queries, the new key and the new value come from the projections and the new key/value are appended on the way (unless an earlier
+// run has filled the pages).
+// part (more than one slice): per (row, head, slice) vdim_p weighted sums, the maximum and the normaliser (of a soft-max).
 // ------------------------------------------------------------------------------------------
 template <typename T, int HT, bool SINGLE>
 __global__ __launch_bounds__(256) void attn_rows_kernel(const AttnDims d, const KvView kv, const AttnIn in, const StepRows r, const T* qbuf, T* out, const int64_t ldo, float* part)
@@ -97,7 +136,7 @@ __global__ __launch_bounds__(256) void attn_rows_kernel(const AttnDims d, const 
   __shared__ float sq[HT][256], nk[256], nv[256];
   __shared__ float sc[HT][SLICE];
   __shared__ float red[4][HT][256];
-  __shared__ float smax[HT], ssum[HT];
+  __shared__ float smax[HT], ssum[HT], rf[8];
   const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
   const int hg = d.heads / d.kv_heads, hblk = (hg + HT - 1) / HT;
   const int row = blockIdx.z, g = blockIdx.y / hblk, h0 = g * hg + blockIdx.y % hblk * HT, nh = min(HT, (g + 1) * hg - h0);
@@ -107,7 +146,7 @@ __global__ __launch_bounds__(256) void attn_rows_kernel(const AttnDims d, const 
   if (nkeys <= 0) {                        // (part is only read up to the slices in use)
     return;
   }
-  const bool own_new = SINGLE && k0 + nkeys == pos + 1;
+  const bool own_new = SINGLE && in.ok >= 0 && k0 + nkeys == pos + 1;
   // The slice's keys are requested first: sixteen lanes a key, eight elements a lane and turn, four keys a lane group.  A slice lies
   // in at most two pages; a single row's own key is not in its page yet and comes from LDS below (columns past the width meet zeros
   // in the query).
@@ -128,10 +167,13 @@ __global__ __launch_bounds__(256) void attn_rows_kernel(const AttnDims d, const 
   }
   if (SINGLE) {
     const float* p = in.proj + row * in.ldp;
+    const RowFactors f = row_factors(d, in, p, pos, own_new, rf);
     for (int u = wave; u < nh + (own_new ? 1 : 0); u += 4) {
       float v[4];
       const bool is_q = u < nh;
-      head_vector(is_q ? p + in.oq + (h0 + u) * d.dim : p + in.ok + g * d.dim, is_q ? in.qn : in.kn, d, pos, lane, v);
+      const int hh = is_q ? h0 + u : g;
+      const float* gain = is_q ? in.qn : in.kn;
+      head_vector(p + (is_q ? in.oq : in.ok) + hh * d.dim, gain && d.whole_norm ? gain + hh * d.dim : gain, is_q ? f.inv_q : f.inv_k, is_q ? f.temp : 1.0f, d, pos, lane, v);
       float* dst = is_q ? sq[u] : nk;
 #pragma unroll
       for (int i = 0; i < 4; i++) dst[lane + 64 * i] = is_q ? v[i] : round_to<T>(v[i]);
@@ -175,8 +217,17 @@ __global__ __launch_bounds__(256) void attn_rows_kernel(const AttnDims d, const 
     }
   }
   __syncthreads();
-  // soft-max over the slice, a wave per head
-  for (int hh = wave; hh < nh; hh += 4) {
+  // weights over the slice, a wave per head
+  if (d.sigmoid) {
+    for (int hh = wave; hh < nh; hh += 4) {
+#pragma unroll
+      for (int i = 0; i < SLICE / 64; i++) {
+        const int k = lane + 64 * i;
+        sc[hh][k] = k < nkeys ? sigmoid_weight(d, h0 + hh, sc[hh][k], pos - k0 - k) : 0.0f;
+      }
+      if (lane == 0) { smax[hh] = 0.0f; ssum[hh] = 1.0f; }
+    }
+  } else for (int hh = wave; hh < nh; hh += 4) {
     float v[SLICE / 64], m = -INFINITY;
 #pragma unroll
     for (int i = 0; i < SLICE / 64; i++) { v[i] = lane + 64 * i < nkeys ? sc[hh][lane + 64 * i] : -INFINITY; m = fmaxf(m, v[i]); }
@@ -205,7 +256,7 @@ __global__ __launch_bounds__(256) void attn_rows_kernel(const AttnDims d, const 
 #pragma unroll
       for (int u = 0; u < 4; u++) {
         const int key = k0 + min(kb + nkg * u, nkeys - 1);
-        if (SINGLE && key == pos) {
+        if (own_new && key == pos) {
 #pragma unroll
           for (int i = 0; i < 8; i++) vx[u][i] = nv[cc * 8 + i];
         } else load8<T>((key < pk ? pg0 : pg1) + kv.v_off + ((int64_t)g * PAGE_TOKENS + key % PAGE_TOKENS) * d.vdim_p + cc * 8, vx[u]);
@@ -255,19 +306,23 @@ __global__ __launch_bounds__(256) void attn_rows_merge_kernel(const AttnDims d, 
   const int used = (pos - d.first_key(pos) + SLICE) / SLICE, st = d.vdim_p + 2;
   const float* p = part + ((int64_t)row * d.heads + h) * n_sl * st;
   float m = -INFINITY, l = 0.0f;
-  for (int s = tid; s < used; s += 256) m = fmaxf(m, p[s * st + d.vdim_p]);
-  for (int o = 32; o; o >>= 1) m = fmaxf(m, __shfl_xor(m, o));
-  if ((tid & 63) == 0) sm[tid >> 6] = m;
-  __syncthreads();
-  m = fmaxf(fmaxf(sm[0], sm[1]), fmaxf(sm[2], sm[3]));
-  for (int s = tid; s < used; s += 256) l += p[s * st + d.vdim_p + 1] * expf(p[s * st + d.vdim_p] - m);
-  for (int o = 32; o; o >>= 1) l += __shfl_xor(l, o);
-  if ((tid & 63) == 0) sl[tid >> 6] = l;
+  if (d.sigmoid) {                         // plain sums
+    if (tid < 4) sl[tid] = 0.25f;
+  } else {
+    for (int s = tid; s < used; s += 256) m = fmaxf(m, p[s * st + d.vdim_p]);
+    for (int o = 32; o; o >>= 1) m = fmaxf(m, __shfl_xor(m, o));
+    if ((tid & 63) == 0) sm[tid >> 6] = m;
+    __syncthreads();
+    m = fmaxf(fmaxf(sm[0], sm[1]), fmaxf(sm[2], sm[3]));
+    for (int s = tid; s < used; s += 256) l += p[s * st + d.vdim_p + 1] * expf(p[s * st + d.vdim_p] - m);
+    for (int o = 32; o; o >>= 1) l += __shfl_xor(l, o);
+    if ((tid & 63) == 0) sl[tid >> 6] = l;
+  }
   float acc = 0.0f;
   for (int s0 = 0; s0 < used; s0 += 256) {               // a block of slice weights at a time
     const int ns = min(256, used - s0);
     __syncthreads();
-    if (tid < ns) sw[tid] = expf(p[(s0 + tid) * st + d.vdim_p] - m);
+    if (tid < ns) sw[tid] = d.sigmoid ? 1.0f : expf(p[(s0 + tid) * st + d.vdim_p] - m);
     __syncthreads();
     if (tid < d.vdim) {
       for (int s = 0; s < ns; s += 8) {
@@ -288,7 +343,7 @@ __global__ __launch_bounds__(256) void attn_rows_merge_kernel(const AttnDims d, 
 // O^T = V^T P^T as they are: key slot (lane group g, j) of a 32-key step is key 4 g + j of its first 16 keys for j < 4 and
 // 4 g + j - 4 of its second 16 otherwise, and V^T is read from LDS in that order.
 // ------------------------------------------------------------------------------------------
-template <int KQ, int VQ>                  // key width in 32s, value width in 16s
+template <int KQ, int VQ, bool SIG>        // key width in 32s, value width in 16s; sigmoid weights
 __global__ __launch_bounds__(256) void attn_prompt_paged_kernel(const AttnDims d, const KvView kv, const AttnIn in, const bf16_t* qbuf, const StepRows r, const int32_t* tiles, bf16_t* out, const int64_t ldo)
 {
   constexpr int KST = KQ * 32 + 8, VST = PAGE_TOKENS + 4;
@@ -321,6 +376,8 @@ __global__ __launch_bounds__(256) void attn_prompt_paged_kernel(const AttnDims d
   float m = -INFINITY, l = 0.0f;
   const int first = d.first_key(pos0 + t0) / PAGE_TOKENS, last = (pos0 + min(t0 + ATTN_TILE, n) - 1) / PAGE_TOKENS;
   const int wmin = pos0 + min(t0 + wave * 16, n - 1), whi = pos0 + min(t0 + wave * 16 + 15, n - 1);   // the wave's first and last row
+  // sigmoid weights: 1 / (1 + 2^(cs score + r1 log2(1 + r2 far) - bias log2 e))
+  const float cs = SIG ? -d.scale * 1.44269504088896340736f : 0.0f, dr1 = SIG ? d.r1[h] : 0.0f, dr2 = SIG ? d.r2[h] : 0.0f, db = SIG ? -1.44269504088896340736f * d.bias[h] : 0.0f;
   const int wlo = d.first_key(wmin), wall = d.first_key(whi);         // first key any of its rows sees, first key all of them see
   const float scale2 = d.scale * 1.44269504088896340736f;             // scores in base-2 logarithms
   constexpr int KC = PAGE_TOKENS * KQ * 4 / 256, VC = PAGE_TOKENS / 2 * VQ * 2 / 256;   // 16-byte key chunks / value chunk pairs per thread
@@ -377,8 +434,20 @@ __global__ __launch_bounds__(256) void attn_prompt_paged_kernel(const AttnDims d
         s[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8, a), __builtin_bit_cast(bf16x8, fq[k]), s[t], 0, 0, 0);
       }
     }
-    float mt = -INFINITY;
-    if (pg * PAGE_TOKENS + PAGE_TOKENS - 1 <= wmin && pg * PAGE_TOKENS >= wall) {   // every row of the wave sees the whole page
+    float mt = -INFINITY, mr = 0.0f;
+    if constexpr (SIG) {
+      const bool whole = pg * PAGE_TOKENS + PAGE_TOKENS - 1 <= wmin && pg * PAGE_TOKENS >= wall;
+#pragma unroll
+      for (int t = 0; t < 4; t++)
+#pragma unroll
+        for (int i = 0; i < 4; i++) {
+          const int key = pg * PAGE_TOKENS + t * 16 + fg * 4 + i;
+          const float far = (float)(qpos - key);
+          float z = fmaf(cs, s[t][i], fmaf(dr1, __builtin_amdgcn_logf(fmaf(dr2, whole ? far : fmaxf(far, 0.0f), 1.0f)), db));
+          if (!whole && (key > qpos || key < qlo)) z = INFINITY;
+          s[t][i] = __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(z));
+        }
+    } else if (pg * PAGE_TOKENS + PAGE_TOKENS - 1 <= wmin && pg * PAGE_TOKENS >= wall) {   // every row of the wave sees the whole page
 #pragma unroll
       for (int t = 0; t < 4; t++)
 #pragma unroll
@@ -393,19 +462,23 @@ __global__ __launch_bounds__(256) void attn_prompt_paged_kernel(const AttnDims d
           mt = fmaxf(mt, s[t][i]);
         }
     }
-    mt = fmaxf(mt, __shfl_xor(mt, 16)); mt = fmaxf(mt, __shfl_xor(mt, 32));
-    const float mn = fmaxf(m, mt), mr = mn == -INFINITY ? 0.0f : mn, al = __builtin_amdgcn_exp2f(m - mr);
-    m = mn; l *= al;
+    if constexpr (!SIG) {
+      mt = fmaxf(mt, __shfl_xor(mt, 16)); mt = fmaxf(mt, __shfl_xor(mt, 32));
+      const float mn = fmaxf(m, mt);
+      mr = mn == -INFINITY ? 0.0f : mn;
+      const float al = __builtin_amdgcn_exp2f(m - mr);
+      m = mn; l *= al;
 #pragma unroll
-    for (int v = 0; v < VQ; v++) o[v] *= al;
+      for (int v = 0; v < VQ; v++) o[v] *= al;
+    }
     // weights in three bfloat16 parts, p = p0 + p1 + p2 exactly (upper halves of p and of what is left)
     uint32_t w[3][16];
 #pragma unroll
     for (int t = 0; t < 4; t++)
 #pragma unroll
       for (int i = 0; i < 4; i++) {
-        const float p = __builtin_amdgcn_exp2f(s[t][i] - mr);
-        l += p;
+        const float p = SIG ? s[t][i] : __builtin_amdgcn_exp2f(s[t][i] - mr);
+        if constexpr (!SIG) l += p;
         const uint32_t b0 = __builtin_bit_cast(uint32_t, p);
         const float r1 = p - __builtin_bit_cast(float, b0 & 0xffff0000u);
         const uint32_t b1 = __builtin_bit_cast(uint32_t, r1);
@@ -431,7 +504,7 @@ __global__ __launch_bounds__(256) void attn_prompt_paged_kernel(const AttnDims d
   }
   l += __shfl_xor(l, 16); l += __shfl_xor(l, 32);
   if (qi < n) {
-    const float inv = 1.0f / l;
+    const float inv = SIG ? 1.0f : 1.0f / l;
 #pragma unroll
     for (int v = 0; v < VQ; v++)
 #pragma unroll
@@ -450,17 +523,19 @@ int attn_paged_prep(const AttnDims& d, const KvView& kv, int act_t, const AttnIn
   return CAI_OK;
 }
 
-static int n_slices(const AttnDims& d) { return (d.span + SLICE - 1) / SLICE; }
+static int n_slices(const AttnDims& d, int reach) { return (std::min(d.span, reach) + SLICE - 1) / SLICE; }
+constexpr size_t PART_FLOATS = 64 << 20;   // partial results of more rows than fit this are made in turns
+static size_t part_row(const AttnDims& d, int ns) { return (size_t)d.heads * ns * (d.vdim_p + 2); }
 size_t attn_paged_part_floats(const AttnDims& d, int n_rows)
 {
-  const int ns = n_slices(d);
-  return ns > 1 ? (size_t)n_rows * d.heads * ns * (d.vdim_p + 2) : 0;
+  const int ns = n_slices(d, d.span);
+  return ns > 1 ? std::max(part_row(d, ns), std::min(PART_FLOATS, (size_t)n_rows * part_row(d, ns))) : 0;
 }
 
 template <typename T, int HT>
 static void run_rows(const AttnDims& d, const KvView& kv, const AttnIn& in, const StepRows& r, const T* qbuf, T* out, int64_t ldo, float* part, bool single)
 {
-  const int hg = d.heads / d.kv_heads, ns = n_slices(d);
+  const int hg = d.heads / d.kv_heads, ns = n_slices(d, r.reach);
   const dim3 grid(ns, d.kv_heads * ((hg + HT - 1) / HT), r.n_rows);
   if (single) hipLaunchKernelGGL((attn_rows_kernel<T, HT, true>), grid, dim3(256), 0, ctx().stream, d, kv, in, r, qbuf, out, ldo, part);
   else hipLaunchKernelGGL((attn_rows_kernel<T, HT, false>), grid, dim3(256), 0, ctx().stream, d, kv, in, r, qbuf, out, ldo, part);
@@ -474,10 +549,22 @@ static void run_rows_t(const AttnDims& d, const KvView& kv, const AttnIn& in, co
   else if (hg == 2) run_rows<T, 2>(d, kv, in, r, (const T*)qbuf, (T*)out, ldo, part, single);
   else run_rows<T, 4>(d, kv, in, r, (const T*)qbuf, (T*)out, ldo, part, single);
 }
-int attn_paged_rows(const AttnDims& d, const KvView& kv, int act_t, const void* qbuf, const StepRows& r, void* out, int64_t ldo, float* part, bool single, const AttnIn& in)
+int attn_paged_rows(const AttnDims& d, const KvView& kv, int act_t, const void* qbuf, const StepRows& r, void* out, int64_t ldo, float* part, size_t part_floats, bool single, const AttnIn& in)
 {
-  if (act_t == ACT_T_BF16) run_rows_t<bf16_t>(d, kv, in, r, qbuf, out, ldo, part, single);
-  else run_rows_t<float>(d, kv, in, r, qbuf, out, ldo, part, single);
+  const int ns = n_slices(d, r.reach);
+  size_t turn = 32768;                     // rows of one launch
+  if (ns > 1) turn = std::min(turn, part_floats / part_row(d, ns));
+  CAI_REQUIRE(turn >= 1, "attention: partial results of %d slices do not fit %zu floats", ns, part_floats);
+  const size_t es = act_t == ACT_T_BF16 ? 2 : 4;
+  for (int r0 = 0; r0 < r.n_rows; r0 += (int)turn) {
+    StepRows q = r; AttnIn a = in;
+    q.pos += r0; q.slot += r0; q.n_rows = std::min((int)turn, r.n_rows - r0);
+    a.proj += r0 * in.ldp;
+    const char* qb = (const char*)qbuf + (size_t)r0 * d.heads * d.dim_p * es;
+    char* o = (char*)out + (size_t)r0 * ldo * es;
+    if (act_t == ACT_T_BF16) run_rows_t<bf16_t>(d, kv, a, q, qb, o, ldo, part, single);
+    else run_rows_t<float>(d, kv, a, q, qb, o, ldo, part, single);
+  }
   CAI_HIP(hipGetLastError());
   return CAI_OK;
 }
@@ -487,11 +574,13 @@ bool attn_paged_prompt_ok(const AttnDims& d, int act_t) { return act_t == ACT_T_
 int attn_paged_prompt(const AttnDims& d, const KvView& kv, const AttnIn& in, const void* qbuf, const StepRows& r, const int32_t* tiles, int n_tiles, void* out, int64_t ldo)
 {
   const dim3 grid(n_tiles, d.heads), blk(256);
-#define PROMPT(K, V) hipLaunchKernelGGL((attn_prompt_paged_kernel<K, V>), grid, blk, 0, ctx().stream, d, kv, in, (const bf16_t*)qbuf, r, tiles, (bf16_t*)out, ldo)
+#define PROMPT_S(K, V, S) hipLaunchKernelGGL((attn_prompt_paged_kernel<K, V, S>), grid, blk, 0, ctx().stream, d, kv, in, (const bf16_t*)qbuf, r, tiles, (bf16_t*)out, ldo)
+#define PROMPT(K, V) do { if (d.sigmoid) PROMPT_S(K, V, true); else PROMPT_S(K, V, false); } while (0)
 #define PROMPT_V(K) do { if (d.vdim <= 64) PROMPT(K, 4); else if (d.vdim <= 128) PROMPT(K, 8); else PROMPT(K, 16); } while (0)
   if (d.dim <= 64) PROMPT_V(2); else if (d.dim <= 128) PROMPT_V(4); else PROMPT_V(8);
 #undef PROMPT_V
 #undef PROMPT
+#undef PROMPT_S
   CAI_HIP(hipGetLastError());
   return CAI_OK;
 }

@@ -33,20 +33,27 @@ __device__ __forceinline__ float lanes_total(float v)
   return __builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, v), 63));
 }
 
+// How a row's experts are chosen and weighted.
+struct Routing { const float* correction; int n, top, among; float scale; };
+
 // One row's experts, by one wave: lane k < top ends with the k-th choice and its weight.  Equal choice scores: the lower index.
-__device__ __forceinline__ void route_row(const float* z, const float* correction, const int n, const int top, const float scale, const int lane, int& expert, float& weight)
+__device__ __forceinline__ void route_row(const float* z, const Routing& q, const int lane, int& expert, float& weight)
 {
+  const float* correction = q.correction;
+  const int n = q.n, top = q.top;
   constexpr int PER = EXPERTS_MAX / 64;
   float s[PER], c[PER], m = -INFINITY, sum = 0.0f;
 #pragma unroll
   for (int i = 0; i < PER; i++) { const int e = lane + 64 * i; s[i] = e < n ? z[e] : -INFINITY; c[i] = e < n && correction ? correction[e] : 0.0f; m = fmaxf(m, s[i]); }
   m = wave_max(m);
+  if (!q.among) {
 #pragma unroll
-  for (int i = 0; i < PER; i++) if (64 * i < n) { s[i] = expf(s[i] - m); sum += s[i]; }
-  sum = lanes_total(sum);
+    for (int i = 0; i < PER; i++) if (64 * i < n) { s[i] = expf(s[i] - m); sum += s[i]; }
+    sum = lanes_total(sum);
+  }
 #pragma unroll
   for (int i = 0; i < PER; i++) {
-    if (64 * i < n) s[i] /= sum;
+    if (64 * i < n && !q.among) s[i] /= sum;
     c[i] = lane + 64 * i < n ? s[i] + c[i] : -INFINITY;
   }
   expert = 0; weight = 0.0f;
@@ -58,12 +65,13 @@ __device__ __forceinline__ void route_row(const float* z, const float* correctio
     const float most = wave_max(bv);
     be = wave_min(bv == most ? be : n - 1);
     bs = __builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, bs), be & 63));
+    if (q.among) bs = expf(bs - m);        // (m is the largest logit, the first choice)
     total += bs;
     if (lane == k) { expert = be; weight = bs; }
 #pragma unroll
     for (int i = 0; i < PER; i++) if (lane + 64 * i == be) c[i] = -INFINITY;
   }
-  weight = weight / (total + 1e-20f) * scale;
+  weight = weight / (total + 1e-20f) * q.scale;
 }
 
 // eight activations times eight weights
@@ -89,11 +97,12 @@ template <typename AT> __device__ __forceinline__ float dot8(const AT* x, const 
 struct FewEntry { int32_t expert, n_rows; uint8_t row[EXPERTS_FEW], slot[EXPERTS_FEW]; };
 static_assert(sizeof(FewEntry) == EXPERTS_FEW_WORDS * 4, "size of a listed expert");
 struct FewGateUp {
-  const uint16_t *w, *ws; int ldw, gu_rows; int n, top, ff, ff_s; float scale, limit, limit_s; int glu, glu_s; int mid_p, active; int n_rows;
+  const uint16_t *w, *ws; int ldw, gu_rows; Routing q; int ff, ff_s; float limit, limit_s; int glu, glu_s; int mid_p, active; int n_rows;
 };
 
-__global__ __launch_bounds__(64 * EXPERTS_FEW) void experts_few_kernel(const float* z, const float* correction, const int n, const int top, const float scale, const int n_rows, float* wgt, FewEntry* list, int32_t* n_list)
+__global__ __launch_bounds__(64 * EXPERTS_FEW) void experts_few_kernel(const float* z, const int64_t ldz, const Routing q, const int n_rows, float* wgt, FewEntry* list, int32_t* n_list)
 {
+  const int n = q.n, top = q.top;
   __shared__ __align__(4) int8_t slot_of[EXPERTS_FEW][EXPERTS_MAX];   // the choice of a row that is this expert, -1: none
   __shared__ int wave_count[EXPERTS_FEW];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, tid = threadIdx.x;
@@ -101,7 +110,7 @@ __global__ __launch_bounds__(64 * EXPERTS_FEW) void experts_few_kernel(const flo
   __syncthreads();
   if (wave < n_rows) {
     int e; float w;
-    route_row(z + (int64_t)wave * n, correction, n, top, scale, lane, e, w);
+    route_row(z + wave * ldz, q, lane, e, w);
     if (lane < top) { wgt[wave * top + lane] = w; slot_of[wave][e] = (int8_t)lane; }
   }
   __syncthreads();
@@ -122,7 +131,7 @@ __global__ __launch_bounds__(64 * EXPERTS_FEW) void experts_few_kernel(const flo
 }
 
 template <typename AT, int NB>
-__global__ __launch_bounds__(256) void experts_gateup_kernel(const FewGateUp p, const float* z, const float* correction, const float* wgt, const FewEntry* list, const int32_t* n_list, const AT* h, const int64_t ldh, int32_t* sel, AT* mid)
+__global__ __launch_bounds__(256) void experts_gateup_kernel(const FewGateUp p, const float* z, const float* wgt, const FewEntry* list, const int32_t* n_list, const AT* h, const int64_t ldh, int32_t* sel, AT* mid)
 {
   constexpr int UNROLL = NB == 1 ? 2 : 1;
   const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), entry = blockIdx.y;
@@ -135,7 +144,7 @@ __global__ __launch_bounds__(256) void experts_gateup_kernel(const FewGateUp p, 
   if (!shared) {
     if constexpr (NB == 1) {
       int e; float wt;
-      route_row(z, correction, p.n, p.top, p.scale, lane, e, wt);
+      route_row(z, p.q, lane, e, wt);
       if (j0 == 0 && lane == entry) sel[entry] = e;
       W = p.w + (int64_t)__shfl(e, entry) * p.gu_rows * p.ldw; weight = __shfl(wt, entry);
     } else {
@@ -170,8 +179,8 @@ __global__ __launch_bounds__(256) void experts_gateup_kernel(const FewGateUp p, 
     if (b >= nb) break;
 #pragma unroll
     for (int i = 0; i < 4; i++) acc[b][i] = lanes_total(acc[b][i]);
-    const int row = NB == 1 ? 0 : shared ? b : list[entry].row[b], slot = NB == 1 ? entry : shared ? p.top : list[entry].slot[b];
-    if (NB > 1) weight = shared ? 1.0f : wgt[row * p.top + slot];
+    const int row = NB == 1 ? 0 : shared ? b : list[entry].row[b], slot = NB == 1 ? entry : shared ? p.q.top : list[entry].slot[b];
+    if (NB > 1) weight = shared ? 1.0f : wgt[row * p.q.top + slot];
     if (lane < 2 && j0 + lane < ff)
       put_act<AT>(mid, (int64_t)row * p.active + slot * p.mid_p + j0 + lane,
                   glu_pair(shared ? p.glu_s : p.glu, shared ? p.limit_s : p.limit, lane ? acc[b][2] : acc[b][0], lane ? acc[b][3] : acc[b][1]) * weight);
@@ -250,8 +259,9 @@ __global__ __launch_bounds__(256) void experts_out_kernel(const uint16_t* w, con
 // other products (bfloat16, or exactly widened weights in 32-bit), the sums meet in LDS.
 constexpr int ROUTE_WAVES = 16;
 template <typename AT, int ET>
-__global__ __launch_bounds__(64 * ROUTE_WAVES) void experts_route_kernel(const uint16_t* W, const int ldw, const AT* h, const int64_t ldh, const float* correction, const int n, const int top, const float scale, const int n_rows, int32_t* sel, float* wgt)
+__global__ __launch_bounds__(64 * ROUTE_WAVES) void experts_route_kernel(const uint16_t* W, const int ldw, const AT* h, const int64_t ldh, const Routing q, const int n_rows, int32_t* sel, float* wgt)
 {
+  const int n = q.n, top = q.top;
   extern __shared__ float lds[];                         // [ROUTE_WAVES][16 ET][16] sums, [16][n] scores
   constexpr int STEP = sizeof(AT) == 2 ? 32 : 16, AHEAD = 8;
   float* z = lds + ROUTE_WAVES * 16 * ET * 16;
@@ -304,9 +314,20 @@ __global__ __launch_bounds__(64 * ROUTE_WAVES) void experts_route_kernel(const u
   __syncthreads();
   for (int r = wave; r < 16 && r0 + r < n_rows; r += ROUTE_WAVES) {
     int e; float w;
-    route_row(z + r * n, correction, n, top, scale, lane, e, w);
+    route_row(z + r * n, q, lane, e, w);
     if (lane < top) { sel[(int64_t)(r0 + r) * top + lane] = e; wgt[(int64_t)(r0 + r) * top + lane] = w; }
   }
+}
+
+// choices of rows whose logits are there already, a wave a row
+__global__ __launch_bounds__(256) void experts_pick_kernel(const float* z, const int64_t ldz, const Routing q, const int n_rows, int32_t* sel, float* wgt)
+{
+  const int lane = threadIdx.x & 63;
+  const int64_t row = blockIdx.x * 4 + (threadIdx.x >> 6);
+  if (row >= n_rows) return;
+  int e; float w;
+  route_row(z + row * ldz, q, lane, e, w);
+  if (lane < q.top) { sel[row * q.top + lane] = e; wgt[row * q.top + lane] = w; }
 }
 
 __global__ __launch_bounds__(1024) void experts_order_kernel(const int32_t* sel, const int n, const int pairs, const int tile, int32_t* order, int32_t* tiles, int32_t* n_tiles)
@@ -348,17 +369,19 @@ __global__ __launch_bounds__(256) void experts_sum_kernel(const float* y, const 
   }
 }
 
+static Routing routing(const NetExperts& x) { return Routing{x.correction, x.n, x.top, x.route == ROUTE_AMONG, x.scale}; }
+
 template <typename AT, int NB>
-static void run_few(const NetExperts& x, int width, const AT* h, int64_t ldh, int n_rows, const ExpertBuf& b, const LinEpi& res)
+static void run_few(const NetExperts& x, int width, const AT* h, int64_t ldh, int n_rows, const float* z, int64_t ldz, const ExpertBuf& b, const LinEpi& res)
 {
   auto st = ctx().stream;
   const uint16_t *sg = x.s_gateup ? (const uint16_t*)x.s_gateup->data : nullptr, *sd = x.s_down ? (const uint16_t*)x.s_down->data : nullptr;
-  const FewGateUp p{(const uint16_t*)x.gateup->data, sg, (int)x.gateup->ld, x.gu_rows(), x.n, x.top, x.ff, x.ff_shared,
-                    x.scale, x.limit, x.limit_shared, x.glu, x.glu_shared, x.mid_p(), x.active(), n_rows};
+  const FewGateUp p{(const uint16_t*)x.gateup->data, sg, (int)x.gateup->ld, x.gu_rows(), routing(x), x.ff, x.ff_shared,
+                    x.limit, x.limit_shared, x.glu, x.glu_shared, x.mid_p(), x.active(), n_rows};
   FewEntry* list = (FewEntry*)b.few;
-  if (NB > 1) hipLaunchKernelGGL(experts_few_kernel, dim3(1), dim3(64 * EXPERTS_FEW), 0, st, b.z, x.correction, x.n, x.top, x.scale, n_rows, b.wgt, list, b.n_tiles);
+  if (NB > 1) hipLaunchKernelGGL(experts_few_kernel, dim3(1), dim3(64 * EXPERTS_FEW), 0, st, z, ldz, p.q, n_rows, b.wgt, list, b.n_tiles);
   const int entries = NB == 1 ? x.top : std::min(x.n, n_rows * x.top);
-  hipLaunchKernelGGL((experts_gateup_kernel<AT, NB>), dim3((std::max(x.ff, x.ff_shared) + 7) / 8, entries + (sg ? 1 : 0)), dim3(256), 0, st, p, b.z, x.correction, b.wgt, list, b.n_tiles, h, ldh, b.sel, (AT*)b.mid);
+  hipLaunchKernelGGL((experts_gateup_kernel<AT, NB>), dim3((std::max(x.ff, x.ff_shared) + 7) / 8, entries + (sg ? 1 : 0)), dim3(256), 0, st, p, z, b.wgt, list, b.n_tiles, h, ldh, b.sel, (AT*)b.mid);
   const int lds = x.s_down ? (int)x.s_down->ld : 0;
   const dim3 outs((width + 7) / 8, NB == 1 ? 1 : entries + (sd ? 1 : 0));
   if constexpr (NB == 1)
@@ -370,23 +393,27 @@ static void run_few(const NetExperts& x, int width, const AT* h, int64_t ldh, in
 }
 
 template <typename AT>
-static int run(const NetExperts& x, int width, int act_t, const AT* h, int64_t ldh, int n_rows, const ExpertBuf& b, const LinEpi& res)
+static int run(const NetExperts& x, int width, int act_t, const AT* h, int64_t ldh, int n_rows, const float* z, int64_t ldz, const ExpertBuf& b, const LinEpi& res)
 {
   auto st = ctx().stream;
   int rc;
   if (n_rows <= EXPERTS_FEW) {
-    LinEpi e; e.y = b.z; e.ldy = x.n;
-    if ((rc = launch_lin(x.router, act_t, h, ldh, n_rows, e))) return rc;
-    if (n_rows == 1) run_few<AT, 1>(x, width, h, ldh, n_rows, b, res);
-    else if (n_rows == 2) run_few<AT, 2>(x, width, h, ldh, n_rows, b, res);
-    else if (n_rows <= 4) run_few<AT, 4>(x, width, h, ldh, n_rows, b, res);
-    else run_few<AT, 8>(x, width, h, ldh, n_rows, b, res);
+    if (!z) {
+      LinEpi e; e.y = b.z; e.ldy = x.n;
+      if ((rc = launch_lin(x.router, act_t, h, ldh, n_rows, e))) return rc;
+      z = b.z; ldz = x.n;
+    }
+    if (n_rows == 1) run_few<AT, 1>(x, width, h, ldh, n_rows, z, ldz, b, res);
+    else if (n_rows == 2) run_few<AT, 2>(x, width, h, ldh, n_rows, z, ldz, b, res);
+    else if (n_rows <= 4) run_few<AT, 4>(x, width, h, ldh, n_rows, z, ldz, b, res);
+    else run_few<AT, 8>(x, width, h, ldh, n_rows, z, ldz, b, res);
     CAI_HIP(hipGetLastError());
     return CAI_OK;
   }
 #define ROUTE(ET) hipLaunchKernelGGL((experts_route_kernel<AT, ET>), dim3((n_rows + 15) / 16), dim3(64 * ROUTE_WAVES), (ROUTE_WAVES * 16 * ET * 16 + 16 * x.n) * sizeof(float), st, \
-                                     (const uint16_t*)x.router->data, (int)x.router->ld, h, ldh, x.correction, x.n, x.top, x.scale, n_rows, b.sel, b.wgt)
-  if (x.n <= 16) ROUTE(1); else ROUTE(2);
+                                     (const uint16_t*)x.router->data, (int)x.router->ld, h, ldh, routing(x), n_rows, b.sel, b.wgt)
+  if (z) hipLaunchKernelGGL(experts_pick_kernel, dim3((n_rows + 3) / 4), dim3(256), 0, st, z, ldz, routing(x), n_rows, b.sel, b.wgt);
+  else if (x.n <= 16) ROUTE(1); else ROUTE(2);
 #undef ROUTE
   const int tile = n_rows * x.top >= x.n * 96 ? BANK_TILE_MAX : BANK_TILE;       // (by the mean number of rows of an expert)
   hipLaunchKernelGGL(experts_order_kernel, dim3(1), dim3(1024), 0, st, b.sel, x.n, n_rows * x.top, tile, b.order, b.tiles, b.n_tiles);
@@ -405,10 +432,11 @@ static int run(const NetExperts& x, int width, int act_t, const AT* h, int64_t l
   return CAI_OK;
 }
 
-int experts_run(const NetExperts& x, int width, int act_t, const void* h, int64_t ldh, int n_rows, const ExpertBuf& b, const LinEpi& res)
+int experts_run(const NetExperts& x, int width, int act_t, const void* h, int64_t ldh, int n_rows, const float* z, int64_t ldz, const ExpertBuf& b, const LinEpi& res)
 {
+  CAI_REQUIRE(z || x.router, "experts: neither logits nor a router");
   CAI_REQUIRE(x.n >= 1 && x.n <= EXPERTS_MAX && x.top >= 1 && x.top <= std::min(x.n, EXPERTS_TOP), "experts: %d of %d", x.top, x.n);
-  return act_t == ACT_T_BF16 ? run<bf16_t>(x, width, act_t, (const bf16_t*)h, ldh, n_rows, b, res) : run<float>(x, width, act_t, (const float*)h, ldh, n_rows, b, res);
+  return act_t == ACT_T_BF16 ? run<bf16_t>(x, width, act_t, (const bf16_t*)h, ldh, n_rows, z, ldz, b, res) : run<float>(x, width, act_t, (const float*)h, ldh, n_rows, z, ldz, b, res);
 }
 
 }  // namespace cai

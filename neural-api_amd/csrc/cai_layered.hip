@@ -20,7 +20,7 @@ int SeqPool::alloc(int n_seq_, int max_tokens, int act_t_)
 {
   n_seq = n_seq_; act_t = act_t_;
   keep = 0;
-  for (auto& a : attn) keep = std::max(keep, a.d.window);
+  for (auto& d : readers) keep = std::max(keep, d.window);
   n_pages = attn.empty() ? 0 : (max_tokens + PAGE_TOKENS - 1) / PAGE_TOKENS;
   seq.assign(n_seq, Seq());
   const size_t es = act_t == ACT_T_BF16 ? 2 : 4;
@@ -76,7 +76,7 @@ void SeqPool::trim(int s)
   if (!n_pages) return;
   Seq& q = seq[s];
   int oldest = q.len;                                                 // the oldest key the next token sees
-  for (auto& a : attn) oldest = std::min(oldest, a.d.first_key(q.len));
+  for (auto& d : readers) oldest = std::min(oldest, d.first_key(q.len));
   const int first = oldest / PAGE_TOKENS;
   for (; q.first_page < std::min(first, q.end_page); q.first_page++) free_pages.push_back(table[(size_t)s * n_pages + q.first_page % n_pages]);
 }
@@ -149,7 +149,7 @@ __global__ __launch_bounds__(256) void net_embed_kernel(const uint16_t* e, const
     const float v = __builtin_bit_cast(float, (uint32_t)row[i] << 16);
     x[t * width + i] = v;
     if (x0) x0[t * width + i] = v;
-    h[t * ldh + i] = (AT)dyt(next, v, i);
+    if (h) h[t * ldh + i] = (AT)dyt(next, v, i);
     if (cat) cat[t * ldc + i] = (AT)v;
   }
 }
@@ -195,6 +195,29 @@ __global__ __launch_bounds__(1024) void net_join_kernel(const float* yl, const f
   for (int i = tid + 4096; i < width; i += 1024) put(i, a[i], b[i], x[t * width + i], gl[i], gr[i]);
 }
 
+// RMS norm of rows of the stream (of those listed in `rows`, or all) with one gain or two; a work-group a row.
+template <typename AT>
+__global__ __launch_bounds__(256) void net_rms_kernel(const float* x, const int32_t* rows, const int width, const float eps, const float* g1, AT* h1, const float* g2, AT* h2, const int64_t ldh)
+{
+  __shared__ float red[4];
+  const int64_t t = blockIdx.x;
+  const int tid = threadIdx.x;
+  const float* v = x + (rows ? rows[t] : t) * width;
+  float s = 0.0f;
+#pragma unroll 8
+  for (int i = tid; i < width; i += 256) s = fmaf(v[i], v[i], s);
+  for (int o = 32; o; o >>= 1) s += __shfl_xor(s, o);
+  if ((tid & 63) == 0) red[tid >> 6] = s;
+  __syncthreads();
+  const float inv = 1.0f / sqrtf((red[0] + red[1] + red[2] + red[3]) / (float)width + eps);
+#pragma unroll 4
+  for (int i = tid; i < ldh; i += 256) {   // (zeros behind the width)
+    const float n = i < width ? v[i] * inv : 0.0f;
+    h1[t * ldh + i] = (AT)(i < width ? n * g1[i] : 0.0f);
+    if (h2) h2[t * ldh + i] = (AT)(i < width ? n * g2[i] : 0.0f);
+  }
+}
+
 template <typename AT>
 __global__ __launch_bounds__(256) void net_gather_kernel(const AT* h, const int32_t* rows, const int64_t ld, AT* out)
 {
@@ -226,7 +249,8 @@ struct LayeredNet {
   // widths over all layers
   int wp = 0, ld_proj = 0, ld_mid = 0, ld_att = 0, ld_attl = 0, ld_q = 0, ld_ra = 0, ld_rg = 0;
   int w_q = 0, w_k = 0, w_v = 0, w_g = 0, w_b = 0, w_za = 0, w_zg = 0, w_hd = 0, w_qt = 0, w_qk = 0, w_gt1 = 0;
-  int ld_cat = 0, ld_ys = 0;
+  int ld_cat = 0, ld_ys = 0, ld_g2 = 0, ld_h2 = 0;
+  size_t part_floats = 0;
   int64_t w_cb = 0, w_sx = 0, w_sb = 0, w_sdt = 0, w_sy = 0;                       // state-space scratch, elements per row (cb: per chunk)
   int64_t w_ez = 0, w_ep = 0, w_emid = 0, w_emid_s = 0, w_etiles = 0;              // experts: scores, pairs, activations of a row's pairs, of the shared expert, most tiles of experts
   bool has_parallel = false, looped = false;
@@ -234,6 +258,7 @@ struct LayeredNet {
   float *x = nullptr, *x0 = nullptr, *proj = nullptr, *yl = nullptr, *yr = nullptr, *part = nullptr, *logits = nullptr;
   void *h = nullptr, *mid = nullptr, *att = nullptr, *attl = nullptr, *qbuf = nullptr, *ra = nullptr, *rgb = nullptr, *hw = nullptr;
   void* cat = nullptr;                     // [stream; embedding] in front of a pass
+  void* h2 = nullptr; float* g2 = nullptr; // layers beside: the feed-forward's input, its gate logits and the router's
   DeltaBuf db{};
   SsdBuf sb{};
   ExpertBuf eb{};
@@ -242,7 +267,7 @@ struct LayeredNet {
   int32_t* d_dec = nullptr;                // fixed row arrays of captured steps: tok, pos, slot, first, last [DEC_ROWS each], ent [4 DEC_ROWS], gen_idx
   int32_t* h_dec = nullptr;
   int32_t* d_gen = nullptr; int gen_cap = 0;
-  std::map<int, hipGraphExec_t> graphs;
+  std::map<std::pair<int, int>, hipGraphExec_t> graphs;   // (steps and rows, reach)
   bool use_graph = true;
   std::vector<int> row_of;                 // logits row of the k-th wanted row of the last step
   bool rows_gathered = false;
@@ -263,12 +288,12 @@ static void drop_graphs(LayeredNet* n)
 
 static void free_rows(LayeredNet* n)
 {
-  void* p[] = {n->x, n->x0, n->proj, n->yl, n->yr, n->part, n->h, n->mid, n->att, n->attl, n->qbuf, n->ra, n->rgb, n->db.q, n->db.k, n->db.v, n->db.g, n->db.beta, n->db.o, n->db.za, n->db.zg, n->db.w, n->db.qt, n->db.qk, n->db.gt, n->cat,
+  void* p[] = {n->x, n->x0, n->proj, n->yl, n->yr, n->part, n->h, n->mid, n->att, n->attl, n->qbuf, n->ra, n->rgb, n->db.q, n->db.k, n->db.v, n->db.g, n->db.beta, n->db.o, n->db.za, n->db.zg, n->db.w, n->db.qt, n->db.qk, n->db.gt, n->cat, n->h2, n->g2,
                n->sb.x, n->sb.B, n->sb.C, n->sb.dt, n->sb.cb, n->sb.bt, n->sb.fac, n->sb.y, n->eb.z, n->eb.wgt, n->eb.y, n->eb.ys, n->eb.sel, n->eb.order, n->eb.tiles, n->eb.n_tiles, n->eb.few, n->eb.mid, n->eb.mid_s};
   for (void* q : p) if (q) (void)hipFree(q);
   n->x = n->x0 = n->proj = n->yl = n->yr = n->part = nullptr;
   n->h = n->mid = n->att = n->attl = n->qbuf = n->ra = n->rgb = nullptr;
-  n->cat = nullptr;
+  n->cat = n->h2 = nullptr; n->g2 = nullptr;
   n->db = DeltaBuf{}; n->sb = SsdBuf{}; n->eb = ExpertBuf{};
   n->cap = 0;
 }
@@ -291,7 +316,8 @@ static int ensure_rows(LayeredNet* n, int rows)
   size_t part = 0;
   // (with bfloat16 activations only steps without a prompt portion take the row form)
   const int part_rows = n->act_t == ACT_T_F32 ? (int)R : std::min((int)R, ATTN_PROMPT_MIN * n->max_seq);
-  for (auto& a : n->pool.attn) part = std::max(part, attn_paged_part_floats(a.d, part_rows));
+  for (auto& d : n->pool.readers) part = std::max(part, attn_paged_part_floats(d, part_rows));
+  n->part_floats = part;
   int rc;
   if ((rc = get((void**)&n->x, R * w * 4)) || (rc = get((void**)&n->x0, n->looped ? R * w * 4 : 0)) || (rc = get((void**)&n->proj, R * n->ld_proj * 4)) ||
       (rc = get((void**)&n->yl, n->has_parallel ? R * w * 4 : 0)) || (rc = get((void**)&n->yr, n->has_parallel ? R * w * 4 : 0)) || (rc = get((void**)&n->part, part * 4)) ||
@@ -302,7 +328,7 @@ static int ensure_rows(LayeredNet* n, int rows)
       (rc = get((void**)&n->db.za, R * n->w_za * 4)) || (rc = get((void**)&n->db.zg, R * n->w_zg * 4)) ||
       (rc = get((void**)&n->db.w, RS * n->w_hd * 4)) || (rc = get((void**)&n->db.qt, RS * n->w_qt * 4)) || (rc = get((void**)&n->db.qk, RS * n->w_qk * 4)) ||
       (rc = get((void**)&n->db.gt, std::max(RS * n->w_gt1, (R / DELTA_CHUNK + n->max_seq + 1) * n->w_qt + 4) * 4)) ||
-      (rc = get(&n->cat, R * n->ld_cat * n->es)) ||
+      (rc = get(&n->cat, R * n->ld_cat * n->es)) || (rc = get(&n->h2, R * n->ld_h2 * n->es)) || (rc = get((void**)&n->g2, R * n->ld_g2 * 4)) ||
       (rc = get((void**)&n->sb.x, (R + SSD_CHUNK) * n->w_sx * 4)) || (rc = get((void**)&n->sb.B, R * n->w_sb * 4)) || (rc = get((void**)&n->sb.C, (R + SSD_CHUNK) * n->w_sb * 4)) ||
       (rc = get((void**)&n->sb.dt, R * n->w_sdt * 4)) || (rc = get((void**)&n->sb.cb, (R / SSD_CHUNK + n->max_seq + 1) * n->w_cb * 4)) || (rc = get((void**)&n->sb.y, R * n->w_sy * 4)) ||
       (rc = get((void**)&n->sb.bt, (R / SSD_CHUNK + n->max_seq + 1) * n->w_sb * SSD_CHUNK * 4)) || (rc = get((void**)&n->sb.fac, (R / SSD_CHUNK + n->max_seq + 1) * n->w_sdt * SSD_FACTORS * 4)) ||
@@ -341,6 +367,7 @@ int net_create(NetSpec&& spec, int max_tokens, int max_seq, int act_t, LayeredNe
   n->act_t = act_t; n->es = act_t == ACT_T_BF16 ? 2 : 4; n->max_seq = max_seq;
   NetSpec& s = n->s;
   const int L = (int)s.layers.size();
+  std::vector<int> last_run(L, -1);        // a layer's latest run with pages of its own
   auto add_run = [&](int l, bool first, int pass) {
     NetRun r{l, first && !s.loop_in && pass > 0, first && s.loop_in, -1, -1};
     NetLayer& y = s.layers[l];
@@ -349,7 +376,9 @@ int net_create(NetSpec&& spec, int max_tokens, int max_seq, int act_t, LayeredNe
       AttnDims& d = y.attn.d;
       d.span = std::min(d.window, (max_tokens + PAGE_TOKENS - 1) / PAGE_TOKENS * PAGE_TOKENS);
       if (!d.chunked) d.window = d.span;
-      r.attn_run = (int)n->pool.attn.size(); n->pool.attn.push_back({d});
+      if (y.kv_from < 0) { r.attn_run = last_run[l] = (int)n->pool.attn.size(); n->pool.attn.push_back({d}); }
+      else r.attn_run = last_run[y.kv_from];
+      n->pool.readers.push_back(d);
     }
     if (y.has_delta() || y.kind == MIX_SSD) {
       const DeltaDims& d = y.delta.d; const SsdDims& m = y.ssd.d;
@@ -380,7 +409,8 @@ int net_create(NetSpec&& spec, int max_tokens, int max_seq, int act_t, LayeredNe
       if (d.rank_a) { up(n->ld_ra, pad_to(d.rank_a, LIN_PAD)); up(n->w_za, d.channel_decay ? d.heads * d.dim : d.heads); }
       if (d.rank_g) { up(n->ld_rg, pad_to(d.rank_g, LIN_PAD)); up(n->w_zg, d.heads * d.vdim); }
     }
-    if (y.gateup) up(n->ld_mid, pad_to(y.ff, LIN_PAD));
+    if (y.down) up(n->ld_mid, pad_to(y.ff, LIN_PAD));
+    if (y.in2) { up(n->ld_g2, pad_to(s.width + y.experts.n, 4)); n->ld_h2 = n->wp; }
     if (y.has_attn()) { up(n->ld_attl, pad_to(y.attn.d.heads * y.attn.d.vdim, LIN_PAD)); up(n->ld_q, y.attn.d.heads * y.attn.d.dim_p); }
     if (y.kind == MIX_PARALLEL) n->has_parallel = true;
     if (y.kind == MIX_SSD) {
@@ -430,6 +460,50 @@ void net_destroy(LayeredNet* n)
 static_assert(ATTN_TILE == SSD_CHUNK, "one list of tiles serves the prompt attention and the state-space walk");
 struct StepLists { const int32_t *tiles = nullptr, *tile0 = nullptr; int n_tiles = 0; bool tall = false; const int32_t* chunks = nullptr; int n_chunks = 0; const int32_t* chunk0 = nullptr; };
 
+template <typename AT>
+static void rms_rows_t(LayeredNet* n, const int32_t* rows, int n_rows, const float* g1, void* h1, const float* g2, void* h2)
+{
+  hipLaunchKernelGGL(net_rms_kernel<AT>, dim3(n_rows), dim3(256), 0, ctx().stream, n->x, rows, n->s.width, n->s.eps, g1, (AT*)h1, g2, (AT*)h2, (int64_t)n->wp);
+}
+static void rms_rows(LayeredNet* n, const int32_t* rows, int n_rows, const float* g1, void* h1, const float* g2 = nullptr, void* h2 = nullptr)
+{
+  if (n->act_t == ACT_T_BF16) rms_rows_t<bf16_t>(n, rows, n_rows, g1, h1, g2, h2);
+  else rms_rows_t<float>(n, rows, n_rows, g1, h1, g2, h2);
+}
+
+static int enqueue_attention(LayeredNet* n, const NetRun& run, const NetLayer& y, const StepRows& r, bool single, const StepLists& lists)
+{
+  const NetAttn& A = y.attn;
+  const int at = n->act_t;
+  const AttnIn ain{n->proj, n->ld_proj, A.oq, A.ok, A.ov, A.og, A.qn, A.kn};
+  const KvView kv = n->pool.view(run.attn_run);
+  int rc;
+  if (!single && (rc = attn_paged_prep(A.d, kv, at, ain, r, n->qbuf))) return rc;
+  if (!single && lists.tall && attn_paged_prompt_ok(A.d, at)) return attn_paged_prompt(A.d, kv, ain, n->qbuf, r, lists.tiles, lists.n_tiles, n->attl, n->ld_attl);
+  return attn_paged_rows(A.d, kv, at, n->qbuf, r, n->attl, n->ld_attl, n->part, n->part_floats, single, ain);
+}
+
+// A layer whose feed-forward works beside its mixer: x += scale1 gate1 mixer(norm1(x)) + scale2 gate2 ff(norm2(x)).
+static int enqueue_beside(LayeredNet* n, const NetRun& run, const NetLayer& y, const StepRows& r, bool single, const StepLists& lists)
+{
+  const int R = r.n_rows, w = n->s.width, at = n->act_t;
+  int rc;
+  rms_rows(n, nullptr, R, y.rms1, n->h, y.rms2, y.has_mlp() ? n->h2 : nullptr);
+  LinEpi a, b;
+  a.y = n->proj; a.ldy = n->ld_proj; a.bias = y.in_b;
+  b.y = n->g2; b.ldy = n->ld_g2; b.bias = y.in2_b;
+  if (y.down) { b.mode = EPI_SPLIT; b.split = w; b.act = LIN_RELU_SQUARED; b.h = n->mid; b.ldh = n->ld_mid; }
+  if ((rc = launch_lin(y.in, at, n->h, n->wp, R, a)) || (y.in2 && (rc = launch_lin(y.in2, at, n->h2, n->wp, R, b)))) return rc;
+  if ((rc = enqueue_attention(n, run, y, r, single, lists))) return rc;
+  LinEpi m, f;
+  m.mode = f.mode = EPI_RESIDUAL; m.y = f.y = n->x; m.ldy = f.ldy = w;
+  m.mult = y.scale1; m.gate = n->proj; m.ldg = n->ld_proj;
+  f.mult = y.scale2; f.gate = n->g2; f.ldg = n->ld_g2;
+  if ((rc = launch_lin(y.attn.out, at, n->attl, n->ld_attl, R, m))) return rc;
+  if (y.experts.n) return experts_run(y.experts, w, at, n->h2, n->wp, R, n->g2 + w, n->ld_g2, n->eb, f);
+  return y.down ? launch_lin(y.down, at, n->mid, n->ld_mid, R, f) : CAI_OK;
+}
+
 // One step over the rows of `r`.  single: every entry is one row (the decode kernels).  want: device list of the rows whose
 // logits are produced (null: all rows, in order).
 static int enqueue_net(LayeredNet* n, const StepRows& r, bool single, const StepLists& lists, const int32_t* want, int n_want)
@@ -446,13 +520,18 @@ static int enqueue_net(LayeredNet* n, const StepRows& r, bool single, const Step
     e.next = i < n->runs.size() ? norm1_of(i) : s.final_norm; e.h = n->h; e.ldh = n->wp;
     if (i < n->runs.size() && n->runs[i].again) { e.add0 = n->x0; e.ld0 = w; }
   };
-  LinEpi first; lead_to(0, first);
+  LinEpi first;
+  if (!s.rms_final) lead_to(0, first);
 #define EMBED(T) hipLaunchKernelGGL(net_embed_kernel<T>, eg, dim3(256), 0, st, (const uint16_t*)s.embed->data, (int)s.embed->ld, r.tok, w, n->x, n->x0, (T*)first.h, first.ldh, first.next, s.loop_in ? (T*)n->cat + w : nullptr, (int64_t)n->ld_cat)
   if (at == ACT_T_BF16) EMBED(bf16_t); else EMBED(float);
 #undef EMBED
   for (size_t i = 0; i < n->runs.size(); i++) {
     const NetRun& run = n->runs[i];
     const NetLayer& y = s.layers[run.layer];
+    if (y.beside) {
+      if ((rc = enqueue_beside(n, run, y, r, single, lists))) return rc;
+      continue;
+    }
     if (run.enter) {
       LinEpi e; e.mode = EPI_RESIDUAL; e.fresh = true; e.y = n->x; e.ldy = w; e.h = n->h; e.ldh = n->wp; e.next = y.norm1;
       if ((rc = launch_lin(s.loop_in, at, n->cat, n->ld_cat, R, e))) return rc;
@@ -489,15 +568,7 @@ static int enqueue_net(LayeredNet* n, const StepRows& r, bool single, const Step
       else if (!(rc = ssd_prep(M.d, sin, M.w, ss, r, n->sb))) rc = ssd_walk(M.d, M.w, ss, r, n->sb, lists.tiles, lists.n_tiles, lists.tile0);
       if (rc || (rc = ssd_finish(M.d, sin, M.w, ss, r, n->sb, single, at, n->att, n->ld_att))) return rc;
     }
-    if (y.has_attn()) {
-      const NetAttn& A = y.attn;
-      const AttnIn ain{n->proj, n->ld_proj, A.oq, A.ok, A.ov, A.og, A.qn, A.kn};
-      const KvView kv = n->pool.view(run.attn_run);
-      if (!single && (rc = attn_paged_prep(A.d, kv, at, ain, r, n->qbuf))) return rc;
-      if (!single && lists.tall && attn_paged_prompt_ok(A.d, at)) rc = attn_paged_prompt(A.d, kv, ain, n->qbuf, r, lists.tiles, lists.n_tiles, n->attl, n->ld_attl);
-      else rc = attn_paged_rows(A.d, kv, at, n->qbuf, r, n->attl, n->ld_attl, n->part, single, ain);
-      if (rc) return rc;
-    }
+    if (y.has_attn() && (rc = enqueue_attention(n, run, y, r, single, lists))) return rc;
     if (y.kind == MIX_PARALLEL) {
       LinEpi el, er; el.y = n->yl; er.y = n->yr; el.ldy = er.ldy = w;
       if ((rc = launch_lin(y.attn.out, at, n->attl, n->ld_attl, R, el)) || (rc = launch_lin(y.delta.out, at, n->att, n->ld_att, R, er))) return rc;
@@ -513,7 +584,7 @@ static int enqueue_net(LayeredNet* n, const StepRows& r, bool single, const Step
     res.post = y.norm2b;
     lead_to(i + 1, res);
     if (y.experts.n) {
-      if ((rc = experts_run(y.experts, w, at, n->h, n->wp, R, n->eb, res))) return rc;
+      if ((rc = experts_run(y.experts, w, at, n->h, n->wp, R, nullptr, 0, n->eb, res))) return rc;
       continue;
     }
     LinEpi g; g.mode = EPI_GLU; g.h = n->mid; g.ldh = n->ld_mid; g.glu = y.glu;
@@ -521,12 +592,15 @@ static int enqueue_net(LayeredNet* n, const StepRows& r, bool single, const Step
   }
   if (n_want > 0) {
     const void* hs = n->h;
-    if (want) {
+    if (s.rms_final) {
+      if (want) hs = n->hw;
+      rms_rows(n, want, n_want, s.rms_final, (void*)hs);
+    } else if (want) {
       if (at == ACT_T_BF16) hipLaunchKernelGGL(net_gather_kernel<bf16_t>, dim3(n_want), dim3(256), 0, st, (const bf16_t*)n->h, want, (int64_t)n->wp, (bf16_t*)n->hw);
       else hipLaunchKernelGGL(net_gather_kernel<float>, dim3(n_want), dim3(256), 0, st, (const float*)n->h, want, (int64_t)n->wp, (float*)n->hw);
       hs = n->hw;
     }
-    LinEpi e; e.y = n->logits; e.ldy = s.vocab;
+    LinEpi e; e.y = n->logits; e.ldy = s.vocab; e.scale = s.logit_scale;
     if ((rc = launch_lin(s.head, at, hs, n->wp, n_want, e))) return rc;
     launch_argmax(n->logits, s.vocab, n_want, n->best, n->am_v, n->am_i);
   }
@@ -534,17 +608,22 @@ static int enqueue_net(LayeredNet* n, const StepRows& r, bool single, const Step
   return CAI_OK;
 }
 
-static StepRows dec_rows(const LayeredNet* n, int R)
+static StepRows dec_rows(const LayeredNet* n, int R, int reach)
 {
   int32_t* d = n->d_dec;
-  return StepRows{d, d + DEC_ROWS, d + 2 * DEC_ROWS, d + 3 * DEC_ROWS, d + 4 * DEC_ROWS, d + 5 * DEC_ROWS, R, R};
+  return StepRows{d, d + DEC_ROWS, d + 2 * DEC_ROWS, d + 3 * DEC_ROWS, d + 4 * DEC_ROWS, d + 5 * DEC_ROWS, R, R, reach};
 }
 
-// `steps` captured steps of R single rows, with the greedy hand-over after each when gen is set (R = 1)
-static int run_captured(LayeredNet* n, int R, int steps, bool gen)
+// `steps` captured steps of R single rows, with the greedy hand-over after each when gen is set (R = 1).  No position reaches `end`:
+// launches over the keys are sized by the next power of two (or by the widest window), so that a sequence captures a few times while
+// it grows.
+static int run_captured(LayeredNet* n, int R, int steps, bool gen, int end)
 {
   auto st = ctx().stream;
-  const StepRows r = dec_rows(n, R);
+  int reach = 256;
+  while (reach < end && reach < n->pool.keep) reach *= 2;
+  if (reach >= n->pool.keep) reach = std::max(n->pool.keep, 1);
+  const StepRows r = dec_rows(n, R, reach);
   auto body = [&]() -> int {
     for (int i = 0; i < steps; i++) {
       const int rc = enqueue_net(n, r, true, StepLists(), nullptr, R);
@@ -554,7 +633,7 @@ static int run_captured(LayeredNet* n, int R, int steps, bool gen)
     return CAI_OK;
   };
   if (!n->use_graph) return body();
-  hipGraphExec_t& ge = n->graphs[(gen ? 1000 : 0) + steps * 16 + R];
+  hipGraphExec_t& ge = n->graphs[{(gen ? 1000 : 0) + steps * 16 + R, reach}];
   if (!ge) {
     hipGraph_t g = nullptr;
     CAI_HIP(hipStreamBeginCapture(st, hipStreamCaptureModeThreadLocal));
@@ -600,19 +679,23 @@ int net_step(LayeredNet* n, int n_ent, const int32_t* seq, const int32_t* count,
   n->row_of.clear();
   if (single && R <= DEC_ROWS) {
     int32_t* hd = n->h_dec;
+    int end = 0;
     for (int e = 0; e < R; e++) {
       const int pos = n->pool.seq[seq[e]].len;
+      end = std::max(end, pos + 1);
       hd[e] = tokens[e]; hd[DEC_ROWS + e] = pos; hd[2 * DEC_ROWS + e] = seq[e]; hd[3 * DEC_ROWS + e] = e; hd[4 * DEC_ROWS + e] = e;
       int32_t* en = hd + 5 * DEC_ROWS + 4 * e; en[0] = seq[e]; en[1] = e; en[2] = 1; en[3] = pos;
     }
     CAI_HIP(hipMemcpyAsync(n->d_dec, hd, 9 * DEC_ROWS * sizeof(int32_t), hipMemcpyHostToDevice, st));
-    if ((rc = run_captured(n, R, 1, false))) return rc;
+    if ((rc = run_captured(n, R, 1, false, end))) return rc;
     n->row_of = wrows; n->rows_gathered = false;
   } else {
     // rows, entries, tiles of the prompt attention kernel, wanted rows
     std::vector<int32_t> tiles, tile0, chunks, chunk0;
     bool tall = false, chunked = false;
+    int end = 0;
     for (int e = 0; e < n_ent; e++) {
+      end = std::max(end, n->pool.seq[seq[e]].len + count[e]);
       tall = tall || count[e] >= ATTN_PROMPT_MIN; chunked = chunked || count[e] >= DELTA_CHUNK_MIN;
       chunk0.push_back((int)chunks.size() / 2); tile0.push_back((int)tiles.size() / 2);
       for (int t = 0; t < count[e]; t += ATTN_TILE) { tiles.push_back(e); tiles.push_back(t); }
@@ -644,7 +727,7 @@ int net_step(LayeredNet* n, int n_ent, const int32_t* seq, const int32_t* count,
     std::copy(wrows.begin(), wrows.end(), ht);
     CAI_HIP(hipMemcpyAsync(n->d_rows, hr, need * sizeof(int32_t), hipMemcpyHostToDevice, st));
     const int32_t* d = n->d_rows;
-    const StepRows r{d, d + R, d + 2 * R, d + 3 * R, d + 4 * R, d + 5 * R, R, n_ent};
+    const StepRows r{d, d + R, d + 2 * R, d + 3 * R, d + 4 * R, d + 5 * R, R, n_ent, end};
     const int32_t* dt = d + 5 * R + 4 * n_ent, *dt0 = dt + tiles.size(), *dc = dt0 + tile0.size(), *dc0 = dc + chunks.size();
     StepLists lists;
     lists.tiles = dt; lists.n_tiles = (int)tiles.size() / 2; lists.tile0 = dt0; lists.tall = tall;
@@ -690,7 +773,7 @@ int net_generate(LayeredNet* n, int seq, int32_t first, int n_tokens, int32_t* o
     if (rc || (rc = n->pool.upload_table())) return rc;
     for (int k = 0; k < m;) {
       const int steps = m - k >= GEN_STEPS ? GEN_STEPS : 1;
-      if ((rc = run_captured(n, 1, steps, true))) return rc;
+      if ((rc = run_captured(n, 1, steps, true, q.len + k + steps))) return rc;
       k += steps;
     }
     q.len += m; i += m;
@@ -747,7 +830,7 @@ int64_t net_weight_bytes(const LayeredNet* n)
   for (const NetRun& r : n->runs) {
     const NetLayer& y = n->s.layers[r.layer];
     const NetExperts& x = y.experts;
-    b += qb(y.in) + qb(y.delta.out) + qb(y.attn.out) + qb(y.ssd.out) + qb(y.delta.w.a2) + qb(y.delta.w.g2) + qb(y.gateup) + qb(y.down) + 8 * (int64_t)n->s.width * 4;
+    b += qb(y.in) + qb(y.delta.out) + qb(y.attn.out) + qb(y.ssd.out) + qb(y.delta.w.a2) + qb(y.delta.w.g2) + qb(y.gateup) + qb(y.down) + qb(y.in2) + 8 * (int64_t)n->s.width * 4;
     if (r.enter) b += qb(n->s.loop_in);
     if (x.n) b += qb(x.router) + qb(x.s_gateup) + qb(x.s_down) + (qb(x.gateup) + qb(x.down)) / x.n * x.top;   // (of one token)
   }

@@ -26,16 +26,20 @@ struct Dyt { const float* w = nullptr; const float* b = nullptr; float alpha = 0
 __device__ __forceinline__ float dyt(const Dyt& t, float x, int i) { return t.w ? tanhf(t.alpha * x) * t.w[i] + t.b[i] : x; }
 
 // What a linear layer does with its finished sums.
-enum { EPI_STORE = 0, EPI_GLU = 1, EPI_RESIDUAL = 2 };
+enum { EPI_STORE = 0, EPI_GLU = 1, EPI_RESIDUAL = 2, EPI_SPLIT = 3 };
+constexpr int LIN_RELU_SQUARED = 100;       // an activation of layered decoders only, beside the CAI_ACT_ ones: max(v, 0)^2
 // Gated pairs: relu(g) u;  silu(g) u;  gelu(g) u, tanh form;  with g = min(gate, limit) and u = clamp(up, -limit, limit):
 // g sigmoid(1.702 g) (u + 1)
 enum { GLU_RELU = 0, GLU_SILU = 1, GLU_GELU_TANH = 2, GLU_CLAMPED = 3 };
 struct LinEpi {
   int mode = EPI_STORE;
-  float* y = nullptr; int64_t ldy = 0;              // STORE: result; RESIDUAL: the residual stream, updated in place
-  void* h = nullptr; int64_t ldh = 0;               // GLU: act(gate) * up; RESIDUAL: input of the next sublayer (null: none)
+  float* y = nullptr; int64_t ldy = 0;              // STORE: result; RESIDUAL: the residual stream, updated in place; SPLIT: the first results
+  void* h = nullptr; int64_t ldh = 0;               // GLU: act(gate) * up; RESIDUAL: input of the next sublayer (null: none); SPLIT: the others
   const float* add0 = nullptr; int64_t ld0 = 0;     // RESIDUAL: added to the stream after the sum (start of a repeated pass)
-  const float* bias = nullptr; int act = CAI_ACT_NONE;   // STORE: act(sum + bias); RESIDUAL: the sum includes it
+  const float* bias = nullptr; int act = CAI_ACT_NONE;   // STORE: act(scale sum + bias); RESIDUAL: the sum includes it
+  float scale = 1.0f;
+  int split = 0;                                    // SPLIT: results [0, split) are sum + bias in y, the others act(sum + bias) in h
+  const float* mult = nullptr; const float* gate = nullptr; int64_t ldg = 0;   // RESIDUAL: the sum is first multiplied by mult[n] sigmoid(gate[t][n]) (null: not)
   int glu = GLU_RELU; float limit = 0.0f;
   bool fresh = false;                               // RESIDUAL: x = post(sum) instead of x += post(sum)
   Dyt post, next;                                   // RESIDUAL: x += post(sum) [+ add0]; h = next(x)
@@ -65,6 +69,7 @@ struct StepRows {
   const int32_t *tok, *pos, *slot, *first, *last;   // [n_rows] device
   const int32_t* ent;                               // [n_ent][4] device: slot, row0, n, pos0
   int n_rows, n_ent;
+  int reach;                                        // no position is this or more: what launches over the keys are sized by
 };
 
 // ------------------------------------------------------------------------------------------
@@ -81,6 +86,11 @@ struct AttnDims {
   int chunked;                             // window is the size of fixed blocks of positions: a token sees its own block up to itself
   int rot; const double* turns;            // the first rot dimensions turn, i with i + rot / 2, by turns[i] full turns a position (0: none)
   int span;                                // most keys a token sees
+  int whole_norm;                          // queries and keys are normed over all their heads at once instead of per head
+  float temp; int temp_every;              // queries are multiplied by 1 + temp ln(floor((pos + 1) / temp_every) + 1) (temp_every 0: not)
+  // Sigmoid weights instead of a soft-max: the weight of a key `far` positions back is sigmoid(score - r1 ln(1 + r2 far) + bias), with
+  // numbers per head, and nothing is normalised over the keys.
+  int sigmoid; const float *r1, *r2, *bias;
   __host__ __device__ int first_key(int pos) const { return chunked ? pos / window * window : pos >= window ? pos - window + 1 : 0; }
 };
 struct DeltaDims {
@@ -100,6 +110,7 @@ struct SsdDims {
   __host__ __device__ int np() const { return (state + 63) & ~63; }    // strides of the prompt buffers (zero filled)
   __host__ __device__ int xp() const { return (vdim + 15) & ~15; }
 };
+constexpr int ATTN_EVERY_KEY = 1 << 30;     // a window that holds every earlier key
 struct KvView {                            // what a kernel needs to reach one attention run's pages
   void* base; int64_t page_elems;          // K [kv_head][PAGE_TOKENS][dim_p] then V [kv_head][PAGE_TOKENS][vdim_p]
   const int32_t* table; int ring;          // [slot][ring]
@@ -110,6 +121,7 @@ struct SeqPool {
   struct AttnRun { AttnDims d; void* base = nullptr; int64_t page_elems = 0, v_off = 0; };
   struct StateRun { int64_t s_elems = 0, h_elems = 0; float* S = nullptr; float* hist = nullptr; };   // state and convolution inputs of one sequence
   std::vector<AttnRun> attn; std::vector<StateRun> state;
+  std::vector<AttnDims> readers;                           // the masks of all attention runs, those that read another run's pages too
   int32_t* d_table = nullptr; std::vector<int32_t> table; bool table_dirty = false;
   std::vector<int> free_pages;
   struct Seq { int len = 0; int first_page = 0, end_page = 0; };   // live pages [first_page, end_page)
@@ -127,13 +139,14 @@ struct SeqPool {
 };
 
 // ---- grouped attention over pages, in a sliding window or in fixed blocks (cai_attn_paged.hip) ----
-// rows of proj: q at column oq ([heads][dim]), k at ok, v at ov.  Queries and keys are RMS-normed per head over dim with a
-// shared gain before the rotation and the score (gain null: not).  og >= 0: the heads' outputs are multiplied by the sigmoid of
-// the columns from og on ([heads][vdim]).
+// rows of proj: q at column oq ([heads][dim]), k at ok, v at ov.  ok < 0: the pages hold these tokens' keys and values already (an
+// earlier run's).  Queries and keys are RMS-normed before the rotation and the score, per head over dim with a shared gain or, with
+// whole_norm, over all heads with gains [heads][dim] and [kv_heads][dim] (gain null: not).  og >= 0: the heads' outputs are multiplied
+// by the sigmoid of the columns from og on ([heads][vdim]).
 struct AttnIn { const float* proj; int64_t ldp; int oq, ok, ov, og; const float *qn, *kn; };
 int attn_paged_prep(const AttnDims& d, const KvView& kv, int act_t, const AttnIn& in, const StepRows& r, void* qbuf);     // norms + append; qbuf [row][heads][dim_p]
-int attn_paged_rows(const AttnDims& d, const KvView& kv, int act_t, const void* qbuf, const StepRows& r, void* out, int64_t ldo, float* part, bool single, const AttnIn& in);
-size_t attn_paged_part_floats(const AttnDims& d, int n_rows);
+int attn_paged_rows(const AttnDims& d, const KvView& kv, int act_t, const void* qbuf, const StepRows& r, void* out, int64_t ldo, float* part, size_t part_floats, bool single, const AttnIn& in);
+size_t attn_paged_part_floats(const AttnDims& d, int n_rows);   // what n_rows at the longest reach want (many rows share less, in turns)
 bool attn_paged_prompt_ok(const AttnDims& d, int act_t);
 int attn_paged_prompt(const AttnDims& d, const KvView& kv, const AttnIn& in, const void* qbuf, const StepRows& r, const int32_t* tiles, int n_tiles, void* out, int64_t ldo);
 constexpr int ATTN_PROMPT_MIN = 16;        // portions from here on make a step take the prompt kernel
@@ -173,11 +186,15 @@ int ssd_finish(const SsdDims& d, const SsdIn& in, const SsdW& w, const SeqPool::
 
 // ---- mixtures of experts over bfloat16 weights (cai_experts.hip) ----
 // Soft-max scores over all experts; the `top` largest of score + correction are chosen; their weights are the scores over their sum,
-// times scale.  A shared expert may run for every token beside them.
+// times scale.  ROUTE_AMONG: the `top` largest logits are chosen, and the soft-max is over these alone (times scale).  A shared expert
+// may run for every token beside them.
+enum { ROUTE_ALL = 0, ROUTE_AMONG = 1 };
 struct NetExperts {
+  int route = ROUTE_ALL;
   int n = 0, top = 0, ff = 0, ff_shared = 0, glu = GLU_CLAMPED, glu_shared = GLU_CLAMPED;   // ff_shared 0: no shared expert
   float scale = 1.0f, limit = 0.0f, limit_shared = 0.0f;
-  cai_qw_s *router = nullptr, *gateup = nullptr, *down = nullptr, *s_gateup = nullptr, *s_down = nullptr;   // gateup, down: banks
+  cai_qw_s *router = nullptr;              // null: the logits are made elsewhere
+  cai_qw_s *gateup = nullptr, *down = nullptr, *s_gateup = nullptr, *s_down = nullptr;   // gateup, down: banks
   const float* correction = nullptr;       // [n], may be null
   int gu_rows() const { return pad_to(ff, 16) * 2; }
   int mid_p() const { return pad_to(ff, LIN_PAD); }
@@ -191,7 +208,8 @@ constexpr int EXPERTS_FEW_WORDS = 2 + EXPERTS_FEW / 2;   // words of a listed ex
 struct ExpertBuf {
   float *z, *wgt, *y, *ys; int32_t *sel, *order, *tiles, *n_tiles, *few; void *mid, *mid_s;
 };
-int experts_run(const NetExperts& x, int width, int act_t, const void* h, int64_t ldh, int n_rows, const ExpertBuf& b, const LinEpi& res);   // res: the residual update
+// z: the rows' logits, ldz apart (null: made here); res: the residual update
+int experts_run(const NetExperts& x, int width, int act_t, const void* h, int64_t ldh, int n_rows, const float* z, int64_t ldz, const ExpertBuf& b, const LinEpi& res);
 
 // ------------------------------------------------------------------------------------------
 // The layered decoder (cai_layered.hip): layers of different kinds, some run several times.
@@ -209,9 +227,17 @@ struct NetLayer {
   Dyt norm1, norm1b, norm2, norm2b;
   cai_qw_s *gateup = nullptr, *down = nullptr; int ff = 0, glu = GLU_RELU;   // gateup null: no dense feed-forward
   NetExperts experts;                      // n > 0: the feed-forward is a mixture
+  // Beside: the feed-forward works beside the mixer on the same stream, each behind an RMS norm of its own, and both results join the
+  // stream times a scale per element and the sigmoid of a matrix over the sublayer's input.
+  bool beside = false;
+  const float *rms1 = nullptr, *rms2 = nullptr, *scale1 = nullptr, *scale2 = nullptr;
+  // (`in` begins with the matrix of the mixer's gate logits)  every matrix over the feed-forward's input: its gate logits, then up
+  // (squared ReLU; ff rows) or the router
+  cai_qw_s* in2 = nullptr; const float* in2_b = nullptr;
+  int kv_from = -1;                        // attention over an earlier layer's keys and values
   bool has_delta() const { return kind == MIX_DELTA || kind == MIX_PARALLEL; }
   bool has_attn() const { return kind == MIX_ATTN || kind == MIX_PARALLEL; }
-  bool has_mlp() const { return gateup || experts.n > 0; }
+  bool has_mlp() const { return gateup || in2 || experts.n > 0; }
 };
 // again: the embedding output is added before this run; enter: the stream is replaced by loop_in [stream; embedding output] before it
 struct NetRun { int layer; bool again, enter; int attn_run, state_run; };
@@ -221,6 +247,8 @@ struct NetSpec {                           // filled by a loader
   cai_qw_s *embed = nullptr, *head = nullptr;
   cai_qw_s* loop_in = nullptr;             // in front of every pass of the repeated stretch (null: the embedding output is added from the second pass on)
   Dyt final_norm;
+  const float* rms_final = nullptr;        // gain of an RMS norm in its place (layers beside)
+  float logit_scale = 1.0f;
   std::vector<NetLayer> layers;
   int loop_start = 0, loop_stop = 0, loop_times = 1;
   std::vector<cai_qw_s*> weights;          // owned

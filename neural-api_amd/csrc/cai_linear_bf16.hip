@@ -251,19 +251,36 @@ __global__ __launch_bounds__(64 * WM * WN) void gemm_bf16(const uint16_t* __rest
     for (int j = 0; j < TN; j++) {
       const int n = n0 + wn + j * 16 + fc * 4;
       if (n >= n_rows) continue;
-      if (n + 3 < n_rows && (e.ldy & 3) == 0 && (e.ldh & 3) == 0 && (e.ld0 & 3) == 0) {
+      if (n + 3 < n_rows && (e.ldy & 3) == 0 && (e.ldh & 3) == 0 && (e.ld0 & 3) == 0 && (e.ldg & 3) == 0 && (e.split & 3) == 0) {
         f32x4* yp = reinterpret_cast<f32x4*>(e.y + (int64_t)t * e.ldy + n);
         f32x4 v = acc[j][i];
         if (e.mode == EPI_STORE) {
-          if (e.bias || e.act != CAI_ACT_NONE) {
+          if (e.bias || e.act != CAI_ACT_NONE || e.scale != 1.0f) {
 #pragma unroll
-            for (int q = 0; q < 4; q++) v[q] = act_apply(e.bias ? v[q] + e.bias[n + q] : v[q], e.act);
+            for (int q = 0; q < 4; q++) v[q] = lin_act(e.bias ? e.scale * v[q] + e.bias[n + q] : e.scale * v[q], e.act);
           }
           *yp = v;
+        } else if (e.mode == EPI_SPLIT) {
+          if (e.bias) v += f32x4{e.bias[n], e.bias[n + 1], e.bias[n + 2], e.bias[n + 3]};
+          if (n < e.split) *yp = v;
+          else {
+            const int o = n - e.split;
+#pragma unroll
+            for (int q = 0; q < 4; q++) v[q] = lin_act(v[q], e.act);
+            if constexpr (sizeof(AT) == 2)
+              *reinterpret_cast<uint2*>(reinterpret_cast<uint16_t*>(e.h) + (int64_t)t * e.ldh + o) = make_uint2(bf16_bits(v[0]) | (uint32_t)bf16_bits(v[1]) << 16, bf16_bits(v[2]) | (uint32_t)bf16_bits(v[3]) << 16);
+            else *reinterpret_cast<f32x4*>(reinterpret_cast<float*>(e.h) + (int64_t)t * e.ldh + o) = v;
+          }
         } else {
           f32x4 x = {0.0f, 0.0f, 0.0f, 0.0f};
           if (!e.fresh) x = *yp;
           if (e.bias) v += f32x4{e.bias[n], e.bias[n + 1], e.bias[n + 2], e.bias[n + 3]};
+          if (e.mult || e.gate) {
+            f32x4 g = {0.0f, 0.0f, 0.0f, 0.0f};
+            if (e.gate) g = *reinterpret_cast<const f32x4*>(e.gate + (int64_t)t * e.ldg + n);
+#pragma unroll
+            for (int q = 0; q < 4; q++) { v[q] *= e.mult ? e.mult[n + q] : 1.0f; if (e.gate) v[q] /= 1.0f + expf(-g[q]); }
+          }
 #pragma unroll
           for (int q = 0; q < 4; q++) x[q] += dyt(e.post, v[q], n + q);
           if (e.add0) x += *reinterpret_cast<const f32x4*>(e.add0 + (int64_t)t * e.ld0 + n);

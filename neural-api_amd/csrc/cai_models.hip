@@ -182,14 +182,23 @@ struct Builder {
     }
     return stack(parts, width, &order);
   }
-  const Json* layer_list(const Json& cfg)          // sizes every layered design has, and its list of layers
+  // the experts' matrices, one after the other
+  void banks(const std::string& pre, int n, int ff, int width, NetExperts& x)
+  {
+    std::vector<std::string> names; std::vector<std::pair<std::string, int64_t>> down;
+    for (int i = 0; i < n; i++) { names.push_back(pre + "e" + std::to_string(i) + "."); down.push_back({names.back() + "down", width}); }
+    x.gateup = gated(names, ff, width);
+    x.down = stack(down, ff);
+  }
+  // sizes every layered design has, and its list of layers; may_loop: a stretch of layers may run several times
+  const Json* layer_list(const Json& cfg, bool may_loop)
   {
     s.width = integer(&cfg, "width", ""); s.vocab = integer(&cfg, "vocab", "", 1, 1 << 28);
     s.eps = number(cfg.get("norm"), "eps", "norm.");
     const Json* layers = cfg.get("layers");
     if (!layers || layers->kind != Json::ARR || layers->arr.empty()) { fail("\"layers\" is missing or empty"); return nullptr; }
     const int L = (int)layers->arr.size();
-    const Json* loop = cfg.get("loop");
+    const Json* loop = may_loop ? cfg.get("loop") : nullptr;
     if (loop && loop->kind != Json::NUL) {
       s.loop_start = integer(loop, "start", "loop.", 0, L); s.loop_stop = integer(loop, "stop", "loop.", 0, L); s.loop_times = integer(loop, "times", "loop.", 1, 4096);
       if (!rc && s.loop_stop < s.loop_start) fail("loop.stop lies before loop.start");
@@ -197,7 +206,6 @@ struct Builder {
     if (rc) return nullptr;
     s.embed = stack({{"embed", s.vocab}}, s.width);
     s.head = stack({{"head", s.vocab}}, s.width);
-    s.final_norm = dyt_norm("final.norm", s.width);
     return rc ? nullptr : layers;
   }
   std::string word(const Json* o, const char* key) { const Json* v = o ? o->get(key) : nullptr; return v && v->kind == Json::STR ? v->str : std::string(); }
@@ -261,8 +269,9 @@ void attn_block(Builder& b, const Json* c, const std::string& where, const std::
 void build_samanex(Builder& b, const Json& cfg)
 {
   NetSpec& s = b.s;
-  const Json* layers = b.layer_list(cfg);
+  const Json* layers = b.layer_list(cfg, true);
   if (!layers) return;
+  s.final_norm = b.dyt_norm("final.norm", s.width);
   const int L = (int)layers->arr.size(), w = s.width;
   for (int l = 0; l < L && !b.rc; l++) {
     const Json& c = layers->arr[l];
@@ -364,10 +373,7 @@ void experts_block(Builder& b, const Json* c, const std::string& where, const st
   x.glu = x.glu_shared = GLU_CLAMPED;
   x.router = b.stack({{pre + "router", n}}, width);
   x.correction = b.vec(pre + "correction", {n});
-  std::vector<std::string> names; std::vector<std::pair<std::string, int64_t>> down;
-  for (int i = 0; i < n; i++) { names.push_back(pre + "e" + std::to_string(i) + "."); down.push_back({names.back() + "down", width}); }
-  x.gateup = b.gated(names, x.ff, width);
-  x.down = b.stack(down, x.ff);
+  b.banks(pre, n, x.ff, width, x);
   if (sh && sh->kind != Json::NUL) {
     x.ff_shared = b.integer(sh, "ff", where + "shared."); x.limit_shared = b.number(sh, "limit", where + "shared.");
     if (b.rc) return;
@@ -380,9 +386,10 @@ void experts_block(Builder& b, const Json* c, const std::string& where, const st
 void build_kiruvik(Builder& b, const Json& cfg)
 {
   NetSpec& s = b.s;
-  const Json* layers = b.layer_list(cfg);
+  const Json* layers = b.layer_list(cfg, true);
   const float mult = b.number(&cfg, "residual_mult", "");
   if (!layers || b.rc) return;
+  s.final_norm = b.dyt_norm("final.norm", s.width);
   const int L = (int)layers->arr.size(), w = s.width;
   if (s.loop_stop > s.loop_start) s.loop_in = b.stack({{"loop.in", w}}, 2 * w);
   for (int l = 0; l < L && !b.rc; l++) {
@@ -412,8 +419,95 @@ void build_kiruvik(Builder& b, const Json& cfg)
   }
 }
 
+// ------------------------------------------------------------------------------------------
+// Gamanex: attention with sigmoid weights over every earlier key, the feed-forward (squared ReLU, or a mixture of experts) beside it on
+// the same stream, both gated by a matrix over their own input.  A layer may attend over an earlier layer's keys and values.
+// ------------------------------------------------------------------------------------------
+void sigmoid_attention(Builder& b, const Json* c, const std::string& where, const std::string& p, int width, int layer, NetLayer& y)
+{
+  NetAttn& A = y.attn; AttnDims& d = A.d;
+  const std::string pre = p + "mix.";
+  d.heads = b.integer(c, "heads", where, 1, 65535); d.kv_heads = b.integer(c, "kv_heads", where, 1, 65535);
+  d.dim = b.integer(c, "dim", where, 1, 256); d.vdim = b.integer(c, "vdim", where, 1, 256);
+  d.scale = b.number(c, "scale", where); d.eps = b.s.eps; d.window = ATTN_EVERY_KEY;
+  const Json *temp = c ? c->get("q_temp") : nullptr, *from = c ? c->get("kv_from") : nullptr;
+  if (temp && temp->kind != Json::NUL) { d.temp = b.number(temp, "coef", where + "q_temp."); d.temp_every = b.integer(temp, "every", where + "q_temp.", 1, 1 << 30); }
+  d.dim_p = pad_to(d.dim, 8); d.vdim_p = pad_to(d.vdim, 8); d.whole_norm = 1; d.sigmoid = 1;
+  if (b.rc) return;
+  if (d.heads % d.kv_heads) { b.fail(where + "heads is not a multiple of " + where + "kv_heads"); return; }
+  if (from && from->kind != Json::NUL) {
+    y.kv_from = b.integer(c, "kv_from", where, 0, 1 << 24);
+    if (b.rc) return;
+    if (y.kv_from >= layer || b.s.layers[y.kv_from].kv_from >= 0) { b.fail(where + "kv_from is not an earlier layer with keys and values of its own"); return; }
+    const AttnDims& o = b.s.layers[y.kv_from].attn.d;
+    if (o.heads != d.heads || o.kv_heads != d.kv_heads || o.dim != d.dim || o.vdim != d.vdim) { b.fail(where + "kv_from is a layer of other head counts or sizes"); return; }
+  }
+  const bool own = y.kv_from < 0;
+  const int qw = d.heads * d.dim, kw = d.kv_heads * d.dim, vw = d.kv_heads * d.vdim;
+  std::vector<std::pair<std::string, int64_t>> parts = {{p + "rg1", width}, {pre + "q", qw}};
+  A.oq = width; A.ok = A.ov = A.og = -1;
+  if (own) { A.ok = width + qw; A.ov = A.ok + kw; parts.push_back({pre + "k", kw}); parts.push_back({pre + "v", vw}); }
+  y.in = b.stack(parts, width);
+  std::vector<float> bias;
+  if (!b.floats(p + "rg1.b", {width}, bias)) return;
+  bias.resize((size_t)width + qw + (own ? kw + vw : 0), 0.0f);   // (the projections have none)
+  y.in_b = b.upload(bias);
+  A.qn = b.vec(pre + "q.norm", {qw});
+  if (own) A.kn = b.vec(pre + "k.norm", {kw});
+  d.r1 = b.vec(pre + "r1", {d.heads}); d.r2 = b.vec(pre + "r2", {d.heads}); d.bias = b.vec(pre + "pb", {d.heads});
+  A.out = b.stack({{pre + "o", width}}, (int64_t)d.heads * d.vdim);
+}
+
+void build_gamanex(Builder& b, const Json& cfg)
+{
+  NetSpec& s = b.s;
+  const Json* layers = b.layer_list(cfg, false);
+  if (!layers) return;
+  s.logit_scale = b.number(&cfg, "logit_scale", "");
+  const int L = (int)layers->arr.size(), w = s.width;
+  s.rms_final = b.vec("final.norm", {w});
+  for (int l = 0; l < L && !b.rc; l++) {
+    const Json& c = layers->arr[l];
+    const std::string p = "l" + std::to_string(l) + ".", where = "layers[" + std::to_string(l) + "].";
+    const Json* mlp = c.get("mlp");
+    NetLayer y;
+    y.beside = true; y.kind = MIX_ATTN;
+    if (b.word(&c, "type") != "attention") { b.fail("\"" + where + "type\" is not attention"); return; }
+    sigmoid_attention(b, c.get("mixer"), where + "mixer.", p, w, l, y);
+    y.rms1 = b.vec(p + "norm1", {w}); y.scale1 = b.vec(p + "ls1", {w});
+    if (b.rc) return;
+    if (mlp && mlp->kind == Json::OBJ) {
+      const std::string kind = b.word(mlp, "kind"), m = p + "mlp.", at = where + "mlp.";
+      std::vector<float> bias, part;
+      if (!b.floats(p + "rg2.b", {w}, bias)) return;
+      if (kind == "dense") {
+        y.ff = b.integer(mlp, "ff", at);
+        if (b.rc) return;
+        y.in2 = b.stack({{p + "rg2", w}, {m + "up", y.ff}}, w);
+        y.down = b.stack({{m + "down", w}}, y.ff);
+        bias.resize((size_t)w + y.ff, 0.0f);
+      } else if (kind == "moe") {
+        NetExperts& x = y.experts;
+        const Json *r = mlp->get("router"), *e = mlp->get("expert");
+        const int n = b.integer(r, "experts", at + "router.", 1, EXPERTS_MAX);
+        x.top = b.integer(r, "top", at + "router.", 1, std::min(n, EXPERTS_TOP)); x.ff = b.integer(e, "ff", at + "expert.");
+        if (b.rc) return;
+        x.route = ROUTE_AMONG; x.glu = GLU_SILU;
+        y.in2 = b.stack({{p + "rg2", w}, {m + "router", n}}, w);
+        if (!b.floats(m + "router.b", {n}, part)) return;
+        bias.insert(bias.end(), part.begin(), part.end());
+        b.banks(m, n, x.ff, w, x);
+        x.n = n;
+      } else { b.fail("\"" + at + "kind\" is not one of dense, moe"); return; }
+      y.in2_b = b.upload(bias);
+      y.rms2 = b.vec(p + "norm2", {w}); y.scale2 = b.vec(p + "ls2", {w});
+    } else if (mlp && mlp->kind != Json::NUL) b.fail("\"" + where + "mlp\" is neither an object nor null");
+    s.layers.push_back(y);
+  }
+}
+
 struct Arch { const char* name; void (*build)(Builder&, const Json&); };
-const Arch ARCHS[] = {{"Samanex", build_samanex}, {"Kiruvik", build_kiruvik}};
+const Arch ARCHS[] = {{"Samanex", build_samanex}, {"Kiruvik", build_kiruvik}, {"Gamanex", build_gamanex}};
 
 bool is_dir(const char* path) { struct stat sb; return stat(path, &sb) == 0 && S_ISDIR(sb.st_mode); }
 

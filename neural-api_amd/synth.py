@@ -234,10 +234,21 @@ def kiruvik_config(width, ff, heads, kv_heads, dim, n_layers, vocab, block, conv
     return dict(architecture="Kiruvik", width=width, vocab=vocab, layers=layers, norm=dict(eps=1e-6), residual_mult=0.8, loop=dict(start=0, stop=n_layers, times=1))
 
 
+def gamanex_config(width, ff, heads, kv_heads, dim, n_layers, vocab, experts=32, top=4):
+    """A Gamanex configuration of real-model proportions: every second layer reads the keys and values of the one before it; dense
+    feed-forwards (two matrices, three halves of the width a gated one would have) and mixtures (of as many active rows) in turn."""
+    att = dict(heads=heads, kv_heads=max(1, kv_heads // 2), dim=dim, vdim=dim, scale=dim ** -0.5, q_temp=dict(coef=0.1, every=256))
+    moe = dict(kind="moe", expert=dict(ff=ff // top), router=dict(experts=experts, top=top))
+    layers = [dict(type="attention", mixer=dict(att, kv_from=i - 1) if i % 2 else att, mlp=moe if i % 2 else dict(kind="dense", ff=ff * 3 // 2)) for i in range(n_layers)]
+    return dict(architecture="Gamanex", width=width, vocab=vocab, layers=layers, norm=dict(eps=1e-6), logit_scale=0.5)
+
+
 def layered_shapes(cfg, rank=128):
     """name -> (shape, standard deviation, mean) of every tensor of a layered model"""
     if cfg["architecture"] == "Kiruvik":
         return kiruvik_shapes(cfg)
+    if cfg["architecture"] == "Gamanex":
+        return gamanex_shapes(cfg)
     w, out = cfg["width"], {}
 
     def lin(name, rows, cols):
@@ -315,6 +326,36 @@ def kiruvik_shapes(cfg):
                 for e in range(f["router"]["experts"]):
                     glu(p + "mlp.e%d." % e, f["expert"]["ff"])
                 glu(p + "mlp.shared.", f["shared"]["ff"])
+    return out
+
+
+def gamanex_shapes(cfg):
+    w, out = cfg["width"], {}
+
+    def lin(name, rows, cols):
+        out[name] = ((rows, cols), cols ** -0.5, 0.0)
+
+    def vec(name, n, std, mean):
+        out[name] = ((n,), std, mean)
+
+    out["embed"] = ((cfg["vocab"], w), 1.0, 0.0)
+    lin("head", cfg["vocab"], w); vec("final.norm", w, 0.1, 1.0)
+    for i, L in enumerate(cfg["layers"]):
+        p, m, f = "l%d." % i, L["mixer"], L["mlp"]
+        lin(p + "mix.q", m["heads"] * m["dim"], w); vec(p + "mix.q.norm", m["heads"] * m["dim"], 0.1, 1.0)
+        if m.get("kv_from") is None:
+            lin(p + "mix.k", m["kv_heads"] * m["dim"], w); lin(p + "mix.v", m["kv_heads"] * m["vdim"], w); vec(p + "mix.k.norm", m["kv_heads"] * m["dim"], 0.1, 1.0)
+        vec(p + "mix.r1", m["heads"], 0.1, 0.5); vec(p + "mix.r2", m["heads"], 0.1, 0.5); vec(p + "mix.pb", m["heads"], 0.5, -4.0)
+        lin(p + "mix.o", w, m["heads"] * m["vdim"])
+        for k in "12" if f else "1":
+            vec(p + "norm" + k, w, 0.1, 1.0); vec(p + "ls" + k, w, 0.1, 0.5); lin(p + "rg" + k, w, w); vec(p + "rg" + k + ".b", w, 0.1, 0.0)
+        if f and f["kind"] == "dense":
+            lin(p + "mlp.up", f["ff"], w); lin(p + "mlp.down", w, f["ff"])
+        elif f:
+            lin(p + "mlp.router", f["router"]["experts"], w); vec(p + "mlp.router.b", f["router"]["experts"], 0.01, 0.0)
+            for e in range(f["router"]["experts"]):
+                x = p + "mlp.e%d." % e
+                lin(x + "gate", f["expert"]["ff"], w); lin(x + "up", f["expert"]["ff"], w); lin(x + "down", w, f["expert"]["ff"])
     return out
 
 

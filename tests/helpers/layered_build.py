@@ -112,10 +112,77 @@ def steady_choice(w):
             w[n] = 4.0 * np.random.default_rng(len(w[n])).permutation(len(w[n]))
 
 
+# ---------------------------------------------------------------- Gamanex
+def sig(heads=4, kv_heads=2, dim=24, vdim=40, scale=0.21, coef=0.4, every=7, kv_from=None):
+    m = dict(heads=heads, kv_heads=kv_heads, dim=dim, vdim=vdim, scale=scale, q_temp=dict(coef=coef, every=every))
+    return m if kv_from is None else dict(m, kv_from=kv_from)
+
+
+def gmoe(experts=6, top=2, ff=20):
+    return dict(kind="moe", expert=dict(ff=ff), router=dict(experts=experts, top=top))
+
+
+def glayer(mixer, mlp=None):
+    """mlp: a width (dense), a mixture, or None"""
+    return dict(type="attention", mixer=mixer, mlp=dict(kind="dense", ff=mlp) if isinstance(mlp, int) else mlp)
+
+
+def gconfig(layers, width=72, vocab=131, eps=1e-5, logit_scale=0.7):
+    return dict(architecture="Gamanex", width=width, vocab=vocab, layers=layers, norm=dict(eps=eps), logit_scale=logit_scale)
+
+
+def gamanex_weights(cfg, seed=0):
+    rng = np.random.default_rng(seed)
+    w, width = {}, cfg["width"]
+
+    def lin(name, rows, cols, gain=1.0):
+        w[name] = rng.standard_normal((rows, cols)) * gain / np.sqrt(cols)
+
+    def vec(name, shape, mean=0.0, spread=0.2):
+        w[name] = mean + spread * rng.standard_normal(shape)
+
+    vec("embed", (cfg["vocab"], width), 0.0, 1.0)
+    lin("head", cfg["vocab"], width, 2.0)
+    vec("final.norm", width, 1.0)
+    for i, L in enumerate(cfg["layers"]):
+        p, m, f = "l%d." % i, L["mixer"], L["mlp"]
+        a = p + "mix."
+        qw, kw = m["heads"] * m["dim"], m["kv_heads"] * m["dim"]
+        lin(a + "q", qw, width); vec(a + "q.norm", qw, 1.2, 0.4)
+        if m.get("kv_from") is None:
+            lin(a + "k", kw, width); lin(a + "v", m["kv_heads"] * m["vdim"], width); vec(a + "k.norm", kw, 1.1, 0.4)
+        w[a + "r1"] = rng.uniform(0.1, 1.2, m["heads"]); w[a + "r2"] = rng.uniform(0.05, 2.0, m["heads"])
+        vec(a + "pb", m["heads"], -1.5, 1.0)
+        lin(a + "o", width, m["heads"] * m["vdim"])
+        for k in ("1", "2") if f else ("1",):
+            vec(p + "norm" + k, width, 1.0); vec(p + "ls" + k, width, 0.8, 0.4)
+            lin(p + "rg" + k, width, width, 1.5); vec(p + "rg" + k + ".b", width, 0.3, 0.5)
+        if f and f["kind"] == "dense":
+            lin(p + "mlp.up", f["ff"], width); lin(p + "mlp.down", width, f["ff"])
+        elif f:
+            lin(p + "mlp.router", f["router"]["experts"], width, 2.0); vec(p + "mlp.router.b", f["router"]["experts"], 0.0, 0.5)
+            for e in range(f["router"]["experts"]):
+                x = p + "mlp.e%d." % e
+                lin(x + "gate", f["expert"]["ff"], width, 1.5); lin(x + "up", f["expert"]["ff"], width, 1.5); lin(x + "down", width, f["expert"]["ff"])
+    return w
+
+
+def steady_experts(cfg):
+    """edit: logits whose bias alone decides which experts run, so that rounding cannot change the choice"""
+    def edit(w):
+        for i, L in enumerate(cfg["layers"]):
+            if L["mlp"] and L["mlp"]["kind"] == "moe":
+                n, top = L["mlp"]["router"]["experts"], L["mlp"]["router"]["top"]
+                w["l%d.mlp.router.b" % i][np.random.default_rng(i).permutation(n)[:top]] += 14.0
+    return edit
+
+
 def weights(cfg, seed=0, rank_a=7, rank_g=11):
     """name -> float array before rounding"""
     if cfg["architecture"] == "Kiruvik":
         return kiruvik_weights(cfg, seed)
+    if cfg["architecture"] == "Gamanex":
+        return gamanex_weights(cfg, seed)
     rng = np.random.default_rng(seed)
     w, width = {}, cfg["width"]
 

@@ -232,6 +232,70 @@ def expert_mixture(w, pre, c, h):
     return y
 
 
+# ---------------------------------------------------------------- mechanisms of Gamanex
+def sigmoid_attention(q, k, v, scale, r1, r2, bias):
+    """q [T, H, d], k [T, G, d], v [T, G, dv].  Query i weighs every key j <= i by the sigmoid of its score, nothing is normalised over
+    the keys.  The score loses r1 ln(1 + r2 (i - j)) with the distance and gains a number per head."""
+    T, H, _ = q.shape
+    G = k.shape[1]
+    i, j = np.arange(T)[:, None], np.arange(T)[None, :]
+    far = np.maximum(i - j, 0)
+    out = np.zeros((T, H, v.shape[2]))
+    for h in range(H):
+        g = h // (H // G)
+        s = (q[:, h] @ k[:, g].T) * scale - r1[h] * np.log(1.0 + r2[h] * far) + bias[h]
+        out[:, h] = np.where(j <= i, sigmoid(s), 0.0) @ v[:, g]
+    return out
+
+
+def query_temperature(positions, coef, every):
+    """factor of a query at a position: grows with the logarithm of how many times `every` positions have passed"""
+    return 1.0 + coef * np.log(np.floor((positions + 1) / every) + 1.0)
+
+
+def sigmoid_attention_mixer(w, pre, c, h, eps, kept, layer):
+    """kept: keys and values of earlier layers by layer number; a layer with 'kv_from' reads them there"""
+    T = h.shape[0]
+    H, G, d, dv = c["heads"], c["kv_heads"], c["dim"], c["vdim"]
+    q = rms_norm(linear(w[pre + "q"], h), eps) * w[pre + "q.norm"]
+    q = q * query_temperature(np.arange(T), c["q_temp"]["coef"], c["q_temp"]["every"])[:, None]
+    if c.get("kv_from") is not None:
+        k, v = kept[c["kv_from"]]
+    else:
+        k = (rms_norm(linear(w[pre + "k"], h), eps) * w[pre + "k.norm"]).reshape(T, G, d)
+        v = linear(w[pre + "v"], h).reshape(T, G, dv)
+        kept[layer] = k, v
+    o = sigmoid_attention(q.reshape(T, H, d), k, v, c["scale"], w[pre + "r1"], w[pre + "r2"], w[pre + "pb"])
+    return linear(w[pre + "o"], o.reshape(T, H * dv))
+
+
+def squared_relu_mlp(w, pre, h):
+    return linear(w[pre + "down"], np.maximum(linear(w[pre + "up"], h), 0.0) ** 2)
+
+
+def silu_expert(w, pre, h):
+    return linear(w[pre + "down"], silu(linear(w[pre + "gate"], h)) * linear(w[pre + "up"], h))
+
+
+def route_among_chosen(z, top):
+    """[T, experts] weights: the `top` largest logits, soft-max over these alone"""
+    out = np.zeros_like(z)
+    for t in range(z.shape[0]):
+        chosen = np.argsort(-z[t], kind="stable")[:top]
+        out[t, chosen] = softmax_rows(z[t, chosen][None])[0]
+    return out
+
+
+def silu_expert_mixture(w, pre, c, h):
+    wt = route_among_chosen(linear(w[pre + "router"], h) + w[pre + "router.b"], c["router"]["top"])
+    return sum(wt[:, e:e + 1] * silu_expert(w, pre + "e%d." % e, h) for e in range(c["router"]["experts"]))
+
+
+def sublayer_gate(w, name, h):
+    """what a sublayer's result is multiplied by before it joins the stream, from the sublayer's own input"""
+    return sigmoid(linear(w[name], h) + w[name + ".b"])
+
+
 # ---------------------------------------------------------------- the models
 def run_order(cfg):
     """(layer, first layer of a repeated pass) for every layer run"""
@@ -247,6 +311,8 @@ def forward(cfg, w, tokens, layers_out=None):
     """logits [T, vocab] of a whole prompt"""
     if cfg["architecture"] == "Kiruvik":
         return kiruvik_forward(cfg, w, tokens, layers_out)
+    if cfg["architecture"] == "Gamanex":
+        return gamanex_forward(cfg, w, tokens, layers_out)
     eps = cfg["norm"]["eps"]
     norm = lambda name, x: dynamic_tanh(x, w[name + ".alpha"], w[name], w[name + ".b"])
     x = w["embed"][np.asarray(tokens)]
@@ -289,3 +355,20 @@ def kiruvik_forward(cfg, w, tokens, layers_out=None):
         if layers_out is not None:
             layers_out.append(x.copy())
     return linear(w["head"], norm("final.norm", x))
+
+
+def gamanex_forward(cfg, w, tokens, layers_out=None):
+    eps, kept = cfg["norm"]["eps"], {}
+    x = w["embed"][np.asarray(tokens)]
+    for i, L in enumerate(cfg["layers"]):
+        p = "l%d." % i
+        h = rms_norm(x, eps) * w[p + "norm1"]
+        y = sigmoid_attention_mixer(w, p + "mix.", L["mixer"], h, eps, kept, i) * w[p + "ls1"] * sublayer_gate(w, p + "rg1", h)
+        if L.get("mlp"):
+            h = rms_norm(x, eps) * w[p + "norm2"]
+            f = squared_relu_mlp(w, p + "mlp.", h) if L["mlp"]["kind"] == "dense" else silu_expert_mixture(w, p + "mlp.", L["mlp"], h)
+            y = y + f * w[p + "ls2"] * sublayer_gate(w, p + "rg2", h)
+        x = x + y
+        if layers_out is not None:
+            layers_out.append(x.copy())
+    return linear(w["head"], rms_norm(x, eps) * w["final.norm"]) * cfg["logit_scale"]

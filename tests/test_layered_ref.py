@@ -147,6 +147,57 @@ def test_kiruvik_oracle_is_sensitive_to_what_it_checks():
         assert np.abs(R.forward(cfg, other, tok) - base).max() > 1e-2, name
 
 
+# ---------------------------------------------------------------- Gamanex's mechanisms
+def test_sigmoid_attention_weighs_each_key_for_itself():
+    rng = np.random.default_rng(11)
+    T, r1, r2, b = 7, np.array([0.5, 0.0, 1.3, 0.2]), np.array([0.3, 1.0, 2.0, 0.7]), np.array([-1.0, 0.5, 0.0, -2.0])
+    q, k, v = rng.standard_normal((T, 4, 6)), rng.standard_normal((T, 2, 6)), rng.standard_normal((T, 2, 5))
+    o = R.sigmoid_attention(q, k, v, 0.3, r1, r2, b)
+    for i in range(T):
+        for h in range(4):
+            want = sum(v[j, h // 2] / (1 + np.exp(-(0.3 * k[j, h // 2] @ q[i, h] + b[h])) * (1 + r2[h] * (i - j)) ** r1[h]) for j in range(i + 1))
+            assert np.allclose(o[i, h], want)
+    # nothing is shared between the keys: another key more changes the sum by its own part alone
+    far = R.sigmoid_attention(q[:, :, :], np.concatenate([k[:-1], k[-1:] * 9]), v, 0.3, r1, r2, b)
+    assert np.allclose(far[:-1], o[:-1]) and not np.allclose(far[-1], o[-1])
+
+
+def test_query_temperature_steps_with_the_position():
+    t = R.query_temperature(np.arange(12), 0.5, 4)
+    assert np.allclose(t[:3], 1.0) and np.allclose(t[3:7], 1 + 0.5 * np.log(2)) and np.allclose(t[7:11], 1 + 0.5 * np.log(3)) and np.isclose(t[11], 1 + 0.5 * np.log(4))
+    assert np.allclose(R.query_temperature(np.arange(3), 1.0, 1), 1 + np.log([2, 3, 4]))
+
+
+def test_routing_among_the_chosen():
+    z = np.array([[1.0, 3.0, -2.0, 2.0]])
+    e = np.exp([3.0, 2.0])
+    assert np.allclose(R.route_among_chosen(z, 2), [[0, e[0] / e.sum(), 0, e[1] / e.sum()]])
+    assert np.allclose(R.route_among_chosen(z, 1), [[0, 1, 0, 0]]) and np.allclose(R.route_among_chosen(z, 4), R.softmax_rows(z))
+
+
+def test_gamanex_oracle_is_sensitive_to_what_it_checks():
+    """every constant and every small tensor, a far token, another layer's keys: each moves the logits well beyond the tests' tolerances"""
+    cfg = B.gconfig([B.glayer(B.sig(), 40), B.glayer(B.sig(heads=6, kv_heads=3, dim=10), B.gmoe()), B.glayer(B.sig(kv_from=0, every=5, coef=0.7), B.gmoe(top=3)), B.glayer(B.sig())])
+    w = {n: B.to_bf16(a)[1].reshape(np.shape(a)) for n, a in B.weights(cfg, 5).items()}
+    tok = np.random.default_rng(6).integers(0, cfg["vocab"], 40)
+    base = R.forward(cfg, w, tok)
+    at = lambda c, i: c["layers"][i]
+    for change in (lambda c: at(c, 0)["mixer"].update(scale=0.25), lambda c: at(c, 2)["mixer"]["q_temp"].update(coef=0.8), lambda c: at(c, 0)["mixer"]["q_temp"].update(every=8),
+                   lambda c: c["norm"].update(eps=0.1), lambda c: c.update(logit_scale=0.75), lambda c: at(c, 1)["mlp"]["router"].update(top=3)):
+        other = json.loads(json.dumps(cfg)); change(other)
+        assert np.abs(R.forward(other, w, tok) - base).max() > 1e-2
+    for name in w:
+        if not name.startswith("l1.mlp.e") and not name.startswith("l2.mlp.e"):
+            other = dict(w); other[name] = w[name] * 0.5
+            assert np.abs(R.forward(cfg, other, tok) - base).max() > 1e-2 or name in ("l0.mix.k", "l1.mix.k", "l3.mix.k", "l0.mix.q", "l1.mix.q", "l2.mix.q", "l3.mix.q"), name   # (a norm takes these back)
+    other = dict(w); other["embed"] = w["embed"].copy(); other["embed"][tok[0]] += 1.0
+    first_only = tok.copy(); first_only[1:][first_only[1:] == tok[0]] = (tok[0] + 1) % cfg["vocab"]
+    assert np.abs(R.forward(cfg, other, first_only)[-1] - R.forward(cfg, w, first_only)[-1]).max() > 1e-2
+    own = json.loads(json.dumps(cfg)); del own["layers"][2]["mixer"]["kv_from"]
+    ow = dict(w, **{"l2.mix." + n: w["l3.mix." + n] for n in ("k", "v", "k.norm")})
+    assert np.abs(R.forward(own, ow, tok) - base).max() > 1e-2
+
+
 @pytest.mark.parametrize("text, reason", [("{", "malformed"), ("[]", ""), ('{"architecture": "Nobody"}', "Samanex"), ("{}", "Samanex"),
                                           ('{"architecture": "Samanex"} x', "after"), ('{"architecture": "\\ud800"}', "malformed")])
 def test_registry_refuses_what_it_does_not_know(tmp_path, text, reason):
