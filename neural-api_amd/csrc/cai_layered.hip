@@ -496,7 +496,7 @@ static int enqueue_beside(LayeredNet* n, const NetRun& run, const NetLayer& y, c
   if ((rc = launch_lin(y.in, at, n->h, n->wp, R, a)) || (y.in2 && (rc = launch_lin(y.in2, at, n->h2, n->wp, R, b)))) return rc;
   if ((rc = enqueue_attention(n, run, y, r, single, lists))) return rc;
   LinEpi m, f;
-  m.mode = f.mode = EPI_RESIDUAL; m.y = f.y = n->x; m.ldy = f.ldy = w;
+  m.mode = f.mode = EPI_JOIN; m.y = f.y = n->x; m.ldy = f.ldy = w;
   m.mult = y.scale1; m.gate = n->proj; m.ldg = n->ld_proj;
   f.mult = y.scale2; f.gate = n->g2; f.ldg = n->ld_g2;
   if ((rc = launch_lin(y.attn.out, at, n->attl, n->ld_attl, R, m))) return rc;

@@ -26,20 +26,20 @@ struct Dyt { const float* w = nullptr; const float* b = nullptr; float alpha = 0
 __device__ __forceinline__ float dyt(const Dyt& t, float x, int i) { return t.w ? tanhf(t.alpha * x) * t.w[i] + t.b[i] : x; }
 
 // What a linear layer does with its finished sums.
-enum { EPI_STORE = 0, EPI_GLU = 1, EPI_RESIDUAL = 2, EPI_SPLIT = 3 };
+enum { EPI_STORE = 0, EPI_GLU = 1, EPI_RESIDUAL = 2, EPI_SPLIT = 3, EPI_JOIN = 4 };
 constexpr int LIN_RELU_SQUARED = 100;       // an activation of layered decoders only, beside the CAI_ACT_ ones: max(v, 0)^2
 // Gated pairs: relu(g) u;  silu(g) u;  gelu(g) u, tanh form;  with g = min(gate, limit) and u = clamp(up, -limit, limit):
 // g sigmoid(1.702 g) (u + 1)
 enum { GLU_RELU = 0, GLU_SILU = 1, GLU_GELU_TANH = 2, GLU_CLAMPED = 3 };
 struct LinEpi {
   int mode = EPI_STORE;
-  float* y = nullptr; int64_t ldy = 0;              // STORE: result; RESIDUAL: the residual stream, updated in place; SPLIT: the first results
+  float* y = nullptr; int64_t ldy = 0;              // STORE: result; RESIDUAL, JOIN: the residual stream, updated in place; SPLIT: the first results
   void* h = nullptr; int64_t ldh = 0;               // GLU: act(gate) * up; RESIDUAL: input of the next sublayer (null: none); SPLIT: the others
   const float* add0 = nullptr; int64_t ld0 = 0;     // RESIDUAL: added to the stream after the sum (start of a repeated pass)
   const float* bias = nullptr; int act = CAI_ACT_NONE;   // STORE: act(scale sum + bias); RESIDUAL: the sum includes it
   float scale = 1.0f;
   int split = 0;                                    // SPLIT: results [0, split) are sum + bias in y, the others act(sum + bias) in h
-  const float* mult = nullptr; const float* gate = nullptr; int64_t ldg = 0;   // RESIDUAL: the sum is first multiplied by mult[n] sigmoid(gate[t][n]) (null: not)
+  const float* mult = nullptr; const float* gate = nullptr; int64_t ldg = 0;   // JOIN: y += mult[n] sigmoid(gate[t][n]) (sum + bias)
   int glu = GLU_RELU; float limit = 0.0f;
   bool fresh = false;                               // RESIDUAL: x = post(sum) instead of x += post(sum)
   Dyt post, next;                                   // RESIDUAL: x += post(sum) [+ add0]; h = next(x)

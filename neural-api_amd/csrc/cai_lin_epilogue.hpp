@@ -22,9 +22,7 @@ __device__ __forceinline__ float lin_act(float v, int act)
 // factor of a sublayer's result before it joins the stream
 __device__ __forceinline__ float join_factor(const LinEpi& e, int n, int64_t t)
 {
-  float f = e.mult ? e.mult[n] : 1.0f;
-  if (e.gate) f /= 1.0f + expf(-e.gate[t * e.ldg + n]);
-  return f;
+  return e.mult[n] / (1.0f + expf(-e.gate[t * e.ldg + n]));
 }
 
 template <typename AT> __device__ __forceinline__ void put_act(void* p, int64_t i, float v)
@@ -33,24 +31,73 @@ template <typename AT> __device__ __forceinline__ void put_act(void* p, int64_t 
   else reinterpret_cast<float*>(p)[i] = v;
 }
 
-// one finished sum of STORE / RESIDUAL / SPLIT
-template <typename AT> __device__ __forceinline__ void epi_one(const LinEpi& e, int n, int t, float v)
+// one finished sum of any mode but GLU
+template <typename AT, int MODE> __device__ __forceinline__ void epi_as(const LinEpi& e, int n, int64_t t, float v)
 {
-  if (e.mode == EPI_STORE) {
-    v *= e.scale;
-    if (e.bias) v += e.bias[n];
-    e.y[t * e.ldy + n] = lin_act(v, e.act);
-  } else if (e.mode == EPI_SPLIT) {
-    if (e.bias) v += e.bias[n];
-    if (n < e.split) e.y[t * e.ldy + n] = v;
+  if constexpr (MODE == EPI_STORE) v *= e.scale;
+  if (e.bias) v += e.bias[n];
+  float* y = e.y + t * e.ldy + n;
+  if constexpr (MODE == EPI_STORE) *y = lin_act(v, e.act);
+  else if constexpr (MODE == EPI_SPLIT) {
+    if (n < e.split) *y = v;
     else put_act<AT>(e.h, t * e.ldh + n - e.split, lin_act(v, e.act));
-  } else {
-    if (e.bias) v += e.bias[n];
-    if (e.mult || e.gate) v *= join_factor(e, n, t);
-    float x = (e.fresh ? 0.0f : e.y[t * e.ldy + n]) + dyt(e.post, v, n);
+  } else if constexpr (MODE == EPI_JOIN) *y += v * join_factor(e, n, t);
+  else {
+    float x = (e.fresh ? 0.0f : *y) + dyt(e.post, v, n);
     if (e.add0) x += e.add0[t * e.ld0 + n];
-    e.y[t * e.ldy + n] = x;
+    *y = x;
     if (e.h) put_act<AT>(e.h, t * e.ldh + n, dyt(e.next, x, n));
+  }
+}
+template <typename AT> __device__ __forceinline__ void epi_one(const LinEpi& e, int n, int64_t t, float v)
+{
+  if (e.mode == EPI_STORE) epi_as<AT, EPI_STORE>(e, n, t, v);
+  else if (e.mode == EPI_SPLIT) epi_as<AT, EPI_SPLIT>(e, n, t, v);
+  else if (e.mode == EPI_JOIN) epi_as<AT, EPI_JOIN>(e, n, t, v);
+  else epi_as<AT, EPI_RESIDUAL>(e, n, t, v);
+}
+
+// four consecutive ones, every stride and `split` a multiple of four
+template <typename AT> __device__ __forceinline__ void put_four(void* p, int64_t i, f32x4 v)
+{
+  if constexpr (sizeof(AT) == 2)
+    *reinterpret_cast<uint2*>(reinterpret_cast<uint16_t*>(p) + i) = make_uint2(bf16_bits(v[0]) | (uint32_t)bf16_bits(v[1]) << 16, bf16_bits(v[2]) | (uint32_t)bf16_bits(v[3]) << 16);
+  else *reinterpret_cast<f32x4*>(reinterpret_cast<float*>(p) + i) = v;
+}
+template <typename AT, int MODE> __device__ __forceinline__ void epi_four(const LinEpi& e, int n, int64_t t, f32x4 v)
+{
+  if constexpr (MODE == EPI_STORE) v *= e.scale;
+  if (e.bias) v += f32x4{e.bias[n], e.bias[n + 1], e.bias[n + 2], e.bias[n + 3]};
+  f32x4* yp = reinterpret_cast<f32x4*>(e.y + t * e.ldy + n);
+  if constexpr (MODE == EPI_STORE) {
+    if (e.act != CAI_ACT_NONE) {
+#pragma unroll
+      for (int q = 0; q < 4; q++) v[q] = lin_act(v[q], e.act);
+    }
+    *yp = v;
+  } else if constexpr (MODE == EPI_SPLIT) {
+    if (n < e.split) { *yp = v; return; }
+#pragma unroll
+    for (int q = 0; q < 4; q++) v[q] = lin_act(v[q], e.act);
+    put_four<AT>(e.h, t * e.ldh + n - e.split, v);
+  } else if constexpr (MODE == EPI_JOIN) {
+    const f32x4 g = *reinterpret_cast<const f32x4*>(e.gate + t * e.ldg + n);
+    f32x4 x = *yp;
+#pragma unroll
+    for (int q = 0; q < 4; q++) x[q] += v[q] * (e.mult[n + q] / (1.0f + expf(-g[q])));
+    *yp = x;
+  } else {
+    f32x4 x = {0.0f, 0.0f, 0.0f, 0.0f};
+    if (!e.fresh) x = *yp;
+#pragma unroll
+    for (int q = 0; q < 4; q++) x[q] += dyt(e.post, v[q], n + q);
+    if (e.add0) x += *reinterpret_cast<const f32x4*>(e.add0 + t * e.ld0 + n);
+    *yp = x;
+    if (e.h) {
+#pragma unroll
+      for (int q = 0; q < 4; q++) v[q] = dyt(e.next, x[q], n + q);
+      put_four<AT>(e.h, t * e.ldh + n, v);
+    }
   }
 }
 

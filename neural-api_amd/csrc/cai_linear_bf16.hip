@@ -127,7 +127,7 @@ __global__ __launch_bounds__(64 * GV_WAVES) void gemv_bf16(const uint16_t* __res
 // Both operand tiles are 128 bytes deep per row (64 bfloat16 or 32 floats), double buffered in LDS; the 16-byte chunks of a row
 // are stored at chunk ^ (row & 7), which makes the fragment reads conflict-free.
 // ------------------------------------------------------------------------------------------
-template <typename AT, int BM, int BN, int WM, int WN, bool BANK>
+template <typename AT, int BM, int BN, int WM, int WN, bool BANK, int MODE>   // MODE: e.mode (one epilogue a kernel: with all of them the accumulators would leave their registers)
 __global__ __launch_bounds__(64 * WM * WN) void gemm_bf16(const uint16_t* __restrict__ W, const AT* __restrict__ X, int n_rows, int ldw, int64_t ldx, int n_tok, int tiles_m, int n_tiles, LinEpi e, BankList l)
 {
   constexpr int NT = 64 * WM * WN;
@@ -226,9 +226,9 @@ __global__ __launch_bounds__(64 * WM * WN) void gemm_bf16(const uint16_t* __rest
     float scale = 1.0f;
     if constexpr (BANK) {
       const int at = l.order[t];
-      if (e.mode == EPI_GLU) scale = l.scale[at]; else t = at;
+      if (MODE == EPI_GLU) scale = l.scale[at]; else t = at;
     }
-    if (e.mode == EPI_GLU) {
+    if constexpr (MODE == EPI_GLU) {
 #pragma unroll
       for (int j = 0; j < TN; j += 2) {
         const int n = n0 + wn + j * 16;                // block of 16 gate rows; its up rows are the next fragment
@@ -241,61 +241,19 @@ __global__ __launch_bounds__(64 * WM * WN) void gemm_bf16(const uint16_t* __rest
 #pragma unroll
           for (int q = 0; q < 4; q++) v[q] *= scale;
         }
-        if constexpr (sizeof(AT) == 2)
-          *reinterpret_cast<uint2*>(reinterpret_cast<uint16_t*>(e.h) + (int64_t)t * e.ldh + o) = make_uint2(bf16_bits(v[0]) | (uint32_t)bf16_bits(v[1]) << 16, bf16_bits(v[2]) | (uint32_t)bf16_bits(v[3]) << 16);
-        else *reinterpret_cast<f32x4*>(reinterpret_cast<float*>(e.h) + (int64_t)t * e.ldh + o) = f32x4{v[0], v[1], v[2], v[3]};
+        put_four<AT>(e.h, (int64_t)t * e.ldh + o, f32x4{v[0], v[1], v[2], v[3]});
       }
       continue;
     }
+    const bool whole = (e.ldy & 3) == 0 && (e.ldh & 3) == 0 && (e.ld0 & 3) == 0 && (e.ldg & 3) == 0 && (e.split & 3) == 0;
 #pragma unroll
     for (int j = 0; j < TN; j++) {
       const int n = n0 + wn + j * 16 + fc * 4;
       if (n >= n_rows) continue;
-      if (n + 3 < n_rows && (e.ldy & 3) == 0 && (e.ldh & 3) == 0 && (e.ld0 & 3) == 0 && (e.ldg & 3) == 0 && (e.split & 3) == 0) {
-        f32x4* yp = reinterpret_cast<f32x4*>(e.y + (int64_t)t * e.ldy + n);
-        f32x4 v = acc[j][i];
-        if (e.mode == EPI_STORE) {
-          if (e.bias || e.act != CAI_ACT_NONE || e.scale != 1.0f) {
+      if (n + 3 < n_rows && whole) epi_four<AT, MODE>(e, n, t, acc[j][i]);
+      else {
 #pragma unroll
-            for (int q = 0; q < 4; q++) v[q] = lin_act(e.bias ? e.scale * v[q] + e.bias[n + q] : e.scale * v[q], e.act);
-          }
-          *yp = v;
-        } else if (e.mode == EPI_SPLIT) {
-          if (e.bias) v += f32x4{e.bias[n], e.bias[n + 1], e.bias[n + 2], e.bias[n + 3]};
-          if (n < e.split) *yp = v;
-          else {
-            const int o = n - e.split;
-#pragma unroll
-            for (int q = 0; q < 4; q++) v[q] = lin_act(v[q], e.act);
-            if constexpr (sizeof(AT) == 2)
-              *reinterpret_cast<uint2*>(reinterpret_cast<uint16_t*>(e.h) + (int64_t)t * e.ldh + o) = make_uint2(bf16_bits(v[0]) | (uint32_t)bf16_bits(v[1]) << 16, bf16_bits(v[2]) | (uint32_t)bf16_bits(v[3]) << 16);
-            else *reinterpret_cast<f32x4*>(reinterpret_cast<float*>(e.h) + (int64_t)t * e.ldh + o) = v;
-          }
-        } else {
-          f32x4 x = {0.0f, 0.0f, 0.0f, 0.0f};
-          if (!e.fresh) x = *yp;
-          if (e.bias) v += f32x4{e.bias[n], e.bias[n + 1], e.bias[n + 2], e.bias[n + 3]};
-          if (e.mult || e.gate) {
-            f32x4 g = {0.0f, 0.0f, 0.0f, 0.0f};
-            if (e.gate) g = *reinterpret_cast<const f32x4*>(e.gate + (int64_t)t * e.ldg + n);
-#pragma unroll
-            for (int q = 0; q < 4; q++) { v[q] *= e.mult ? e.mult[n + q] : 1.0f; if (e.gate) v[q] /= 1.0f + expf(-g[q]); }
-          }
-#pragma unroll
-          for (int q = 0; q < 4; q++) x[q] += dyt(e.post, v[q], n + q);
-          if (e.add0) x += *reinterpret_cast<const f32x4*>(e.add0 + (int64_t)t * e.ld0 + n);
-          *yp = x;
-          if (e.h) {
-#pragma unroll
-            for (int q = 0; q < 4; q++) v[q] = dyt(e.next, x[q], n + q);
-            if constexpr (sizeof(AT) == 2)
-              *reinterpret_cast<uint2*>(reinterpret_cast<uint16_t*>(e.h) + (int64_t)t * e.ldh + n) = make_uint2(bf16_bits(v[0]) | (uint32_t)bf16_bits(v[1]) << 16, bf16_bits(v[2]) | (uint32_t)bf16_bits(v[3]) << 16);
-            else *reinterpret_cast<f32x4*>(reinterpret_cast<float*>(e.h) + (int64_t)t * e.ldh + n) = v;
-          }
-        }
-      } else {
-#pragma unroll
-        for (int q = 0; q < 4; q++) if (n + q < n_rows) epi_one<AT>(e, n + q, t, acc[j][i][q]);
+        for (int q = 0; q < 4; q++) if (n + q < n_rows) epi_as<AT, MODE>(e, n + q, t, acc[j][i][q]);
       }
     }
   }
@@ -305,16 +263,20 @@ template <typename AT, int BM, int BN, int WM, int WN>
 static void run_gemm(const cai_qw_s* w, const AT* x, int64_t ldx, int n_tok, const LinEpi& e)
 {
   const int tm = (n_tok + BM - 1) / BM, tn = ((int)w->rows + BN - 1) / BN;
-  hipLaunchKernelGGL((gemm_bf16<AT, BM, BN, WM, WN, false>), dim3(tm * tn), dim3(64 * WM * WN), 0, ctx().stream,
-                     (const uint16_t*)w->data, x, (int)w->rows, (int)w->ld, ldx, n_tok, tm, tm * tn, e, BankList{});
+#define GEMM(MODE) case MODE: hipLaunchKernelGGL((gemm_bf16<AT, BM, BN, WM, WN, false, MODE>), dim3(tm * tn), dim3(64 * WM * WN), 0, ctx().stream, \
+                              (const uint16_t*)w->data, x, (int)w->rows, (int)w->ld, ldx, n_tok, tm, tm * tn, e, BankList{}); break
+  switch (e.mode) { GEMM(EPI_STORE); GEMM(EPI_GLU); GEMM(EPI_RESIDUAL); GEMM(EPI_SPLIT); GEMM(EPI_JOIN); }
+#undef GEMM
 }
 
 template <typename AT, int BM, int BN>
 static void run_bank(const cai_qw_s* w, int mat_rows, const AT* x, int64_t ldx, const BankList& l, const LinEpi& e)
 {
   const int tm = l.max_tiles, tn = (mat_rows + BN - 1) / BN;
-  hipLaunchKernelGGL((gemm_bf16<AT, BM, BN, 2, 2, true>), dim3(tm * tn), dim3(256), 0, ctx().stream,
-                     (const uint16_t*)w->data, x, mat_rows, (int)w->ld, ldx, 0, tm, tm * tn, e, l);
+#define GEMM(MODE) case MODE: hipLaunchKernelGGL((gemm_bf16<AT, BM, BN, 2, 2, true, MODE>), dim3(tm * tn), dim3(256), 0, ctx().stream, \
+                              (const uint16_t*)w->data, x, mat_rows, (int)w->ld, ldx, 0, tm, tm * tn, e, l); break
+  switch (e.mode) { GEMM(EPI_STORE); GEMM(EPI_GLU); }
+#undef GEMM
 }
 
 int launch_lin_bank(const cai_qw_s* w, int mat_rows, int act_t, const void* x, int64_t ldx, const BankList& l, const LinEpi& e)
