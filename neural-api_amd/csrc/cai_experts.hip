@@ -187,10 +187,12 @@ __global__ __launch_bounds__(256) void experts_gateup_kernel(const FewGateUp p, 
   }
 }
 
-// The output product of one row: a wave makes two outputs over all choices, then the residual update.
+// The output product of one row: a wave makes two outputs over all choices, then the residual update.  wo: the product beside (null:
+// none).
+struct BesideArg { const uint16_t* w = nullptr; const void* x = nullptr; int ld = 0; int64_t ldx = 0; LinEpi e; };
 template <typename AT>
 __global__ __launch_bounds__(256) void experts_down_kernel(const uint16_t* w, const uint16_t* ws, const int ldw, const int lds, const int top, const int width, const int n_experts,
-                                                           const int32_t* sel, const AT* mid, const LinEpi e)
+                                                           const int32_t* sel, const AT* mid, const LinEpi e, const BesideArg o)
 {
   const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6);
   const int o0 = (blockIdx.x * 4 + wave) * 2;
@@ -198,6 +200,7 @@ __global__ __launch_bounds__(256) void experts_down_kernel(const uint16_t* w, co
   const int o1 = min(o0 + 1, width - 1);
   float acc[2] = {0.0f, 0.0f};
   const AT* x = mid;
+  float b0 = 0.0f, b1 = 0.0f;
   auto slot = [&](const uint16_t* m, int ld) {
     const uint16_t *a = m + (int64_t)o0 * ld, *b = m + (int64_t)o1 * ld;
 #pragma unroll 2
@@ -207,17 +210,28 @@ __global__ __launch_bounds__(256) void experts_down_kernel(const uint16_t* w, co
     }
     x += ld;
   };
+  if (o.w) {
+    x = reinterpret_cast<const AT*>(o.x);
+    slot(o.w, o.ld);
+    b0 = lanes_total(acc[0]); b1 = lanes_total(acc[1]);
+    acc[0] = acc[1] = 0.0f;
+    x = mid;
+  }
 #pragma unroll 4
   for (int s = 0; s < top; s++) slot(w + (int64_t)min(max(sel[s], 0), n_experts - 1) * width * ldw, ldw);
   if (ws) slot(ws, lds);
   const float y0 = lanes_total(acc[0]), y1 = lanes_total(acc[1]);
-  if (lane < 2 && o0 + lane < width) epi_one<AT>(e, o0 + lane, 0, lane ? y1 : y0);
+  if (lane < 2 && o0 + lane < width) {
+    if (o.w) join_two(o.e, lane ? b1 : b0, e, lane ? y1 : y0, o0 + lane, 0);
+    else epi_one<AT>(e, o0 + lane, 0, lane ? y1 : y0);
+  }
 }
 
 // That of several rows, an entry at a time (blockIdx as in the gate and up kernel): outputs of every choice, summed by experts_sum_kernel.
+// The product beside takes the place of the shared expert: ws over rows xs, lxs apart.
 template <typename AT, int NB>
 __global__ __launch_bounds__(256) void experts_out_kernel(const uint16_t* w, const uint16_t* ws, const int ldw, const int lds, const int top, const int active, const int width, const int n_rows,
-                                                          const FewEntry* list, const int32_t* n_list, const AT* mid, float* y, float* ys)
+                                                          const FewEntry* list, const int32_t* n_list, const AT* mid, float* y, float* ys, const AT* xs, const int64_t lxs)
 {
   const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), entry = blockIdx.y;
   const bool shared = ws && entry == (int)gridDim.y - 1;
@@ -232,7 +246,7 @@ __global__ __launch_bounds__(256) void experts_out_kernel(const uint16_t* w, con
 #pragma unroll
   for (int b = 0; b < NB; b++) {
     row[b] = b >= nb ? 0 : shared ? b : list[entry].row[b]; slot[b] = b >= nb ? 0 : shared ? top : list[entry].slot[b];
-    x[b] = mid + (int64_t)row[b] * active + slot[b] * ldw;
+    x[b] = shared && xs ? xs + row[b] * lxs : mid + (int64_t)row[b] * active + slot[b] * ldw;
     acc[b][0] = acc[b][1] = 0.0f;
   }
   for (int k = lane * 8; k < ld; k += 512) {
@@ -359,20 +373,23 @@ __global__ __launch_bounds__(1024) void experts_order_kernel(const int32_t* sel,
 }
 
 template <typename AT>
-__global__ __launch_bounds__(256) void experts_sum_kernel(const float* y, const float* ys, const int top, const int width, const LinEpi e)
+__global__ __launch_bounds__(256) void experts_sum_kernel(const float* y, const float* ys, const int top, const int width, const LinEpi e, const LinEpi beside)
 {
   const int64_t row = blockIdx.y;
   for (int i = blockIdx.x * 256 + threadIdx.x; i < width; i += gridDim.x * 256) {
-    float s = ys ? ys[row * width + i] : 0.0f;
+    const float s0 = ys ? ys[row * width + i] : 0.0f;
+    float s = beside.y ? 0.0f : s0;
+#pragma unroll 4
     for (int k = 0; k < top; k++) s += y[(row * top + k) * width + i];
-    epi_one<AT>(e, i, (int)row, s);
+    if (beside.y) join_two(beside, s0, e, s, i, row);
+    else epi_one<AT>(e, i, (int)row, s);
   }
 }
 
 static Routing routing(const NetExperts& x) { return Routing{x.correction, x.n, x.top, x.route == ROUTE_AMONG, x.scale}; }
 
 template <typename AT, int NB>
-static void run_few(const NetExperts& x, int width, const AT* h, int64_t ldh, int n_rows, const float* z, int64_t ldz, const ExpertBuf& b, const LinEpi& res)
+static void run_few(const NetExperts& x, int width, const AT* h, int64_t ldh, int n_rows, const float* z, int64_t ldz, const ExpertBuf& b, const LinEpi& res, const BesideLin* beside)
 {
   auto st = ctx().stream;
   const uint16_t *sg = x.s_gateup ? (const uint16_t*)x.s_gateup->data : nullptr, *sd = x.s_down ? (const uint16_t*)x.s_down->data : nullptr;
@@ -382,18 +399,21 @@ static void run_few(const NetExperts& x, int width, const AT* h, int64_t ldh, in
   if (NB > 1) hipLaunchKernelGGL(experts_few_kernel, dim3(1), dim3(64 * EXPERTS_FEW), 0, st, z, ldz, p.q, n_rows, b.wgt, list, b.n_tiles);
   const int entries = NB == 1 ? x.top : std::min(x.n, n_rows * x.top);
   hipLaunchKernelGGL((experts_gateup_kernel<AT, NB>), dim3((std::max(x.ff, x.ff_shared) + 7) / 8, entries + (sg ? 1 : 0)), dim3(256), 0, st, p, z, b.wgt, list, b.n_tiles, h, ldh, b.sel, (AT*)b.mid);
+  BesideArg o;
+  if (beside) { o.w = (const uint16_t*)beside->w->data; o.x = beside->x; o.ld = (int)beside->w->ld; o.ldx = beside->ldx; o.e = beside->e; }
   const int lds = x.s_down ? (int)x.s_down->ld : 0;
-  const dim3 outs((width + 7) / 8, NB == 1 ? 1 : entries + (sd ? 1 : 0));
+  const dim3 outs((width + 7) / 8, NB == 1 ? 1 : entries + (sd || beside ? 1 : 0));
   if constexpr (NB == 1)
-    hipLaunchKernelGGL(experts_down_kernel<AT>, outs, dim3(256), 0, st, (const uint16_t*)x.down->data, sd, (int)x.down->ld, lds, x.top, width, x.n, b.sel, (const AT*)b.mid, res);
+    hipLaunchKernelGGL(experts_down_kernel<AT>, outs, dim3(256), 0, st, (const uint16_t*)x.down->data, sd, (int)x.down->ld, lds, x.top, width, x.n, b.sel, (const AT*)b.mid, res, o);
   else {
-    hipLaunchKernelGGL((experts_out_kernel<AT, NB>), outs, dim3(256), 0, st, (const uint16_t*)x.down->data, sd, (int)x.down->ld, lds, x.top, x.active(), width, n_rows, list, b.n_tiles, (const AT*)b.mid, b.y, b.ys);
-    hipLaunchKernelGGL(experts_sum_kernel<AT>, dim3(std::min((width + 255) / 256, 32), n_rows), dim3(256), 0, st, b.y, sd ? b.ys : nullptr, x.top, width, res);
+    hipLaunchKernelGGL((experts_out_kernel<AT, NB>), outs, dim3(256), 0, st, (const uint16_t*)x.down->data, beside ? o.w : sd, (int)x.down->ld, beside ? o.ld : lds, x.top, x.active(), width, n_rows, list, b.n_tiles, (const AT*)b.mid, b.y, b.ys,
+                       (const AT*)o.x, o.ldx);
+    hipLaunchKernelGGL(experts_sum_kernel<AT>, dim3(std::min((width + 255) / 256, 32), n_rows), dim3(256), 0, st, b.y, sd || beside ? b.ys : nullptr, x.top, width, res, o.e);
   }
 }
 
 template <typename AT>
-static int run(const NetExperts& x, int width, int act_t, const AT* h, int64_t ldh, int n_rows, const float* z, int64_t ldz, const ExpertBuf& b, const LinEpi& res)
+static int run(const NetExperts& x, int width, int act_t, const AT* h, int64_t ldh, int n_rows, const float* z, int64_t ldz, const ExpertBuf& b, const LinEpi& res, const BesideLin* beside)
 {
   auto st = ctx().stream;
   int rc;
@@ -403,10 +423,10 @@ static int run(const NetExperts& x, int width, int act_t, const AT* h, int64_t l
       if ((rc = launch_lin(x.router, act_t, h, ldh, n_rows, e))) return rc;
       z = b.z; ldz = x.n;
     }
-    if (n_rows == 1) run_few<AT, 1>(x, width, h, ldh, n_rows, z, ldz, b, res);
-    else if (n_rows == 2) run_few<AT, 2>(x, width, h, ldh, n_rows, z, ldz, b, res);
-    else if (n_rows <= 4) run_few<AT, 4>(x, width, h, ldh, n_rows, z, ldz, b, res);
-    else run_few<AT, 8>(x, width, h, ldh, n_rows, z, ldz, b, res);
+    if (n_rows == 1) run_few<AT, 1>(x, width, h, ldh, n_rows, z, ldz, b, res, beside);
+    else if (n_rows == 2) run_few<AT, 2>(x, width, h, ldh, n_rows, z, ldz, b, res, beside);
+    else if (n_rows <= 4) run_few<AT, 4>(x, width, h, ldh, n_rows, z, ldz, b, res, beside);
+    else run_few<AT, 8>(x, width, h, ldh, n_rows, z, ldz, b, res, beside);
     CAI_HIP(hipGetLastError());
     return CAI_OK;
   }
@@ -427,16 +447,17 @@ static int run(const NetExperts& x, int width, int act_t, const AT* h, int64_t l
     LinEpi s; s.y = b.ys; s.ldy = width;
     if ((rc = launch_lin(x.s_down, act_t, b.mid_s, x.shared_p(), n_rows, s))) return rc;
   }
-  hipLaunchKernelGGL(experts_sum_kernel<AT>, dim3(std::min((width + 255) / 256, 32), n_rows), dim3(256), 0, st, b.y, x.ff_shared ? b.ys : nullptr, x.top, width, res);
+  hipLaunchKernelGGL(experts_sum_kernel<AT>, dim3(std::min((width + 255) / 256, 32), n_rows), dim3(256), 0, st, b.y, x.ff_shared ? b.ys : nullptr, x.top, width, res, LinEpi());
   CAI_HIP(hipGetLastError());
   return CAI_OK;
 }
 
-int experts_run(const NetExperts& x, int width, int act_t, const void* h, int64_t ldh, int n_rows, const float* z, int64_t ldz, const ExpertBuf& b, const LinEpi& res)
+int experts_run(const NetExperts& x, int width, int act_t, const void* h, int64_t ldh, int n_rows, const float* z, int64_t ldz, const ExpertBuf& b, const LinEpi& res, const BesideLin* beside)
 {
+  CAI_REQUIRE(!beside || (n_rows <= EXPERTS_FEW && !x.ff_shared && beside->w->rows == width && beside->e.mode == EPI_JOIN && res.mode == EPI_JOIN), "experts: a product of another kind beside them");
   CAI_REQUIRE(z || x.router, "experts: neither logits nor a router");
   CAI_REQUIRE(x.n >= 1 && x.n <= EXPERTS_MAX && x.top >= 1 && x.top <= std::min(x.n, EXPERTS_TOP), "experts: %d of %d", x.top, x.n);
-  return act_t == ACT_T_BF16 ? run<bf16_t>(x, width, act_t, (const bf16_t*)h, ldh, n_rows, z, ldz, b, res) : run<float>(x, width, act_t, (const float*)h, ldh, n_rows, z, ldz, b, res);
+  return act_t == ACT_T_BF16 ? run<bf16_t>(x, width, act_t, (const bf16_t*)h, ldh, n_rows, z, ldz, b, res, beside) : run<float>(x, width, act_t, (const float*)h, ldh, n_rows, z, ldz, b, res, beside);
 }
 
 }  // namespace cai

@@ -421,7 +421,7 @@ int net_create(NetSpec&& spec, int max_tokens, int max_seq, int act_t, LayeredNe
     if (y.experts.n) {
       const NetExperts& x = y.experts;
       up(n->w_ez, x.n); up(n->w_ep, x.top); up(n->w_etiles, x.n); up(n->w_emid, std::max(x.active(), x.top * x.mid_p())); up(n->w_emid_s, x.shared_p());
-      if (x.ff_shared) up(n->ld_ys, s.width);
+      if (x.ff_shared || y.beside) up(n->ld_ys, s.width);
     }
   }
   const char* ng = getenv("CAIHIP_NO_GRAPH");
@@ -487,20 +487,29 @@ static int enqueue_attention(LayeredNet* n, const NetRun& run, const NetLayer& y
 static int enqueue_beside(LayeredNet* n, const NetRun& run, const NetLayer& y, const StepRows& r, bool single, const StepLists& lists)
 {
   const int R = r.n_rows, w = n->s.width, at = n->act_t;
+  const bool few = R <= LIN_FEW;
   int rc;
-  rms_rows(n, nullptr, R, y.rms1, n->h, y.rms2, y.has_mlp() ? n->h2 : nullptr);
   LinEpi a, b;
   a.y = n->proj; a.ldy = n->ld_proj; a.bias = y.in_b;
   b.y = n->g2; b.ldy = n->ld_g2; b.bias = y.in2_b;
   if (y.down) { b.mode = EPI_SPLIT; b.split = w; b.act = LIN_RELU_SQUARED; b.h = n->mid; b.ldh = n->ld_mid; }
-  if ((rc = launch_lin(y.in, at, n->h, n->wp, R, a)) || (y.in2 && (rc = launch_lin(y.in2, at, n->h2, n->wp, R, b)))) return rc;
+  if (few) {                               // both norms inside one launch of both stacks of matrices
+    const RmsLin first{y.in, y.rms1, a}, second{y.in2, y.rms2, b, y.experts.n ? n->h2 : nullptr, n->wp};
+    if ((rc = launch_lin_rms(at, n->x, w, n->s.eps, R, first, y.in2 ? &second : nullptr))) return rc;
+  } else {
+    rms_rows(n, nullptr, R, y.rms1, n->h, y.rms2, y.has_mlp() ? n->h2 : nullptr);
+    if ((rc = launch_lin(y.in, at, n->h, n->wp, R, a)) || (y.in2 && (rc = launch_lin(y.in2, at, n->h2, n->wp, R, b)))) return rc;
+  }
   if ((rc = enqueue_attention(n, run, y, r, single, lists))) return rc;
   LinEpi m, f;
   m.mode = f.mode = EPI_JOIN; m.y = f.y = n->x; m.ldy = f.ldy = w;
   m.mult = y.scale1; m.gate = n->proj; m.ldg = n->ld_proj;
   f.mult = y.scale2; f.gate = n->g2; f.ldg = n->ld_g2;
+  const BesideLin o{y.attn.out, n->attl, n->ld_attl, m};
+  if (few && y.experts.n) return experts_run(y.experts, w, at, n->h2, n->wp, R, n->g2 + w, n->ld_g2, n->eb, f, &o);
+  if (few && y.down) return launch_lin_pair(at, R, y.attn.out, n->attl, n->ld_attl, m, y.down, n->mid, n->ld_mid, f);
   if ((rc = launch_lin(y.attn.out, at, n->attl, n->ld_attl, R, m))) return rc;
-  if (y.experts.n) return experts_run(y.experts, w, at, n->h2, n->wp, R, n->g2 + w, n->ld_g2, n->eb, f);
+  if (y.experts.n) return experts_run(y.experts, w, at, n->h2, n->wp, R, n->g2 + w, n->ld_g2, n->eb, f, nullptr);
   return y.down ? launch_lin(y.down, at, n->mid, n->ld_mid, R, f) : CAI_OK;
 }
 
@@ -584,7 +593,7 @@ static int enqueue_net(LayeredNet* n, const StepRows& r, bool single, const Step
     res.post = y.norm2b;
     lead_to(i + 1, res);
     if (y.experts.n) {
-      if ((rc = experts_run(y.experts, w, at, n->h, n->wp, R, nullptr, 0, n->eb, res))) return rc;
+      if ((rc = experts_run(y.experts, w, at, n->h, n->wp, R, nullptr, 0, n->eb, res, nullptr))) return rc;
       continue;
     }
     LinEpi g; g.mode = EPI_GLU; g.h = n->mid; g.ldh = n->ld_mid; g.glu = y.glu;
@@ -592,7 +601,11 @@ static int enqueue_net(LayeredNet* n, const StepRows& r, bool single, const Step
   }
   if (n_want > 0) {
     const void* hs = n->h;
-    if (s.rms_final) {
+    LinEpi e; e.y = n->logits; e.ldy = s.vocab; e.scale = s.logit_scale;
+    if (s.rms_final && !want && n_want <= LIN_FEW) {
+      if ((rc = launch_lin_rms(at, n->x, w, s.eps, n_want, RmsLin{s.head, s.rms_final, e, n->h, n->wp}, nullptr))) return rc;
+      hs = nullptr;
+    } else if (s.rms_final) {
       if (want) hs = n->hw;
       rms_rows(n, want, n_want, s.rms_final, (void*)hs);
     } else if (want) {
@@ -600,8 +613,7 @@ static int enqueue_net(LayeredNet* n, const StepRows& r, bool single, const Step
       else hipLaunchKernelGGL(net_gather_kernel<float>, dim3(n_want), dim3(256), 0, st, (const float*)n->h, want, (int64_t)n->wp, (float*)n->hw);
       hs = n->hw;
     }
-    LinEpi e; e.y = n->logits; e.ldy = s.vocab; e.scale = s.logit_scale;
-    if ((rc = launch_lin(s.head, at, hs, n->wp, n_want, e))) return rc;
+    if (hs && (rc = launch_lin(s.head, at, hs, n->wp, n_want, e))) return rc;
     launch_argmax(n->logits, s.vocab, n_want, n->best, n->am_v, n->am_i);
   }
   CAI_HIP(hipGetLastError());

@@ -49,7 +49,14 @@ __host__ __device__ inline int glu_row(int j, int up) { return (j >> 4) * 32 + u
 
 // y = W x for n_tok activation rows x[t][ldx] (zero padded to LIN_PAD columns, element type act_t); W is a CAI_BF16 matrix.
 int launch_lin(const cai_qw_s* w, int act_t, const void* x, int64_t ldx, int n_tok, const LinEpi& e);
-// The same over a bank of equal matrices stacked in w (mat_rows rows each): work lists of (matrix, first place, places) over an order
+constexpr int LIN_FEW = 8;                  // up to so many rows take the streaming kernel
+// Up to LIN_FEW rows of the float stream x[t][width] through an RMS norm and a matrix, with one launch also through a second norm and
+// matrix (null: none).  normed: where the normed rows themselves go, ldn apart and zero padded (null: nowhere; both ldn alike).
+struct RmsLin { const cai_qw_s* w; const float* gain; LinEpi e; void* normed = nullptr; int64_t ldn = 0; };
+int launch_lin_rms(int act_t, const float* x, int width, float eps, int n_tok, const RmsLin& a, const RmsLin* b);
+// Up to LIN_FEW rows of two products with the same outputs that both join one stream.
+int launch_lin_pair(int act_t, int n_tok, const cai_qw_s* w, const void* x, int64_t ldx, const LinEpi& e, const cai_qw_s* w2, const void* x2, int64_t ldx2, const LinEpi& e2);
+// launch_lin over a bank of equal matrices stacked in w (mat_rows rows each): work lists of (matrix, first place, places) over an order
 // of activation rows.  Place p reads activation row order[p] / div (div 0: row p) and writes row p of e.h, scaled by
 // scale[order[p]] (GLU), or row order[p] of e.y (STORE).
 constexpr int BANK_TILE = 64, BANK_TILE_MAX = 128;      // most places of a list entry: one of the two
@@ -208,8 +215,10 @@ constexpr int EXPERTS_FEW_WORDS = 2 + EXPERTS_FEW / 2;   // words of a listed ex
 struct ExpertBuf {
   float *z, *wgt, *y, *ys; int32_t *sel, *order, *tiles, *n_tiles, *few; void *mid, *mid_s;
 };
-// z: the rows' logits, ldz apart (null: made here); res: the residual update
-int experts_run(const NetExperts& x, int width, int act_t, const void* h, int64_t ldh, int n_rows, const float* z, int64_t ldz, const ExpertBuf& b, const LinEpi& res);
+// z: the rows' logits, ldz apart (null: made here); res: the residual update.  beside: a product with the same outputs that joins the
+// stream with them, for up to EXPERTS_FEW rows and no shared expert (null: none).
+struct BesideLin { const cai_qw_s* w; const void* x; int64_t ldx; LinEpi e; };
+int experts_run(const NetExperts& x, int width, int act_t, const void* h, int64_t ldh, int n_rows, const float* z, int64_t ldz, const ExpertBuf& b, const LinEpi& res, const BesideLin* beside);
 
 // ------------------------------------------------------------------------------------------
 // The layered decoder (cai_layered.hip): layers of different kinds, some run several times.

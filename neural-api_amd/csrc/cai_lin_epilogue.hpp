@@ -25,6 +25,14 @@ __device__ __forceinline__ float join_factor(const LinEpi& e, int n, int64_t t)
   return e.mult[n] / (1.0f + expf(-e.gate[t * e.ldg + n]));
 }
 
+// two finished sums of the same output, both joined
+__device__ __forceinline__ void join_two(const LinEpi& a, float va, const LinEpi& b, float vb, int n, int64_t t)
+{
+  if (a.bias) va += a.bias[n];
+  if (b.bias) vb += b.bias[n];
+  a.y[t * a.ldy + n] += va * join_factor(a, n, t) + vb * join_factor(b, n, t);
+}
+
 template <typename AT> __device__ __forceinline__ void put_act(void* p, int64_t i, float v)
 {
   if constexpr (sizeof(AT) == 2) reinterpret_cast<uint16_t*>(p)[i] = bf16_bits(v);
