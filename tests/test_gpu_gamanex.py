@@ -217,6 +217,29 @@ def test_decoding_together_agrees_with_each_request_alone(cai, models, rows, dt)
     dec.close()
 
 
+@pytest.fixture(scope="module")
+def wide(tmp_path_factory):
+    """wider than the streaming products stage at once for eight rows, rows split between waves, a width that is no multiple of the padding"""
+    cfg = B.gconfig([B.glayer(B.sig(heads=4, kv_heads=2, dim=130, vdim=136), 2600), B.glayer(B.sig(heads=4, kv_heads=2, dim=130, vdim=136, kv_from=0), B.gmoe(experts=4, top=2, ff=300))], width=2100, vocab=50)
+    return Model(tmp_path_factory.mktemp("wide"), cfg, seed=2, edit=B.steady_experts(cfg))
+
+
+@DT
+@pytest.mark.parametrize("rows", [1, 2, 3, 4, 5, 6, 7, 8, 9])
+def test_wide_layers_in_small_batches(cai, wide, rows, dt):
+    reqs = [wide.tokens(4 + b, 500 + b) for b in range(rows)]
+    dec = wide.open(cai, 64 * rows, rows, dt)
+    got = [[] for _ in reqs]
+    for k in range(2):                            # one token each, twice
+        lg = dec.step_batch([(b, reqs[b][k:k + 1], [0]) for b in range(rows)])[1]
+        for b in range(rows):
+            got[b].append(lg[b:b + 1])
+    for b in range(rows):                         # the rest in a portion of one to eight tokens
+        got[b].append(dec.step_batch([(b, reqs[b][2:], range(len(reqs[b]) - 2))])[1])
+        check(np.concatenate(got[b]), wide.ref(reqs[b]), dt)
+    dec.close()
+
+
 def test_batches_agree_with_each_request_alone_to_rounding(cai, models):
     m = models["f32"]
     reqs = [m.tokens(n, 60 + n) for n in (21, 90, 2, 1)]
