@@ -3,8 +3,10 @@
 // and the step function.  A step is any mixture of prompt portions and single tokens of different sequences; a step of single
 // tokens only is captured once per width as a graph and replayed.
 //
-// The residual stream is float.  A sublayer's epilogue adds its result and already leaves the next sublayer's normed input, so
-// between two mixers with a dense feed-forward there are three products and nothing else.
+// The residual stream is float.  Behind Dynamic Tanh a sublayer's epilogue adds its result and already leaves the next sublayer's
+// normed input, so between two mixers with a dense feed-forward there are three products and nothing else.  Layers whose feed-forward
+// works beside the mixer have RMS norms: a small step takes both norms into the one launch of the layer's input matrices and joins
+// both results in one other launch; a prompt norms the rows first.
 #include "cai_layered.hpp"
 
 #include <algorithm>

@@ -5,7 +5,8 @@
 // 32-bit sums) or float; with float activations the weights are widened exactly and every product and sum is 32-bit (the
 // 16x16x4 float form of the matrix cores).  What follows the product runs in its epilogue on the 32-bit sums: bias and
 // activation, act(gate) * up of a gated pair, or the residual update with the Dynamic Tanh before and after it - that norm
-// has no statistics, so a sublayer needs no launch besides its products and its mixer.  The matrix-core kernel also runs over a
+// has no statistics, so a sublayer needs no launch besides its products and its mixer - or a result's scaled and gated joining.  The
+// streaming kernel takes the float stream through an RMS norm itself, and runs two products in one launch.  The matrix-core kernel also runs over a
 // bank of equal matrices with a list of activation rows for each (mixtures of experts).
 #include "cai_lin_epilogue.hpp"
 
