@@ -1,7 +1,7 @@
 // Grouped-query attention over a paged key/value pool, in a sliding window or in fixed blocks of positions: key and value widths of
 // their own, optional RMS norm of queries and keys (per head or over all heads at once), optional rotation of the first dimensions of
 // a head, optional growth of the queries with the position, an explicit score scale, an optional sigmoid gate on the heads' outputs.
-// The weights are a soft-max over the keys or, each key for itself, a sigmoid of the score with a logarithmic loss over the distance.
+// The weights are a soft-max over the keys (a sink, a number without a key, may join its normaliser) or, each key for itself, a sigmoid of the score with a logarithmic loss over the distance.
 // A run may read the pages that an earlier run has filled.
 //
 // Two forms: one work-group per (row, key/value head, slice of keys) for decoded tokens, short portions and the all-32-bit mode,
@@ -238,7 +238,7 @@ __global__ __launch_bounds__(256) void attn_rows_kernel(const AttnDims d, const 
     for (int i = 0; i < SLICE / 64; i++) { v[i] = expf(v[i] - m); s += v[i]; sc[hh][lane + 64 * i] = v[i]; }
 #pragma unroll
     for (int o = 32; o; o >>= 1) s += __shfl_xor(s, o);
-    if (lane == 0) { smax[hh] = m; ssum[hh] = s; }
+    if (lane == 0) { smax[hh] = m; ssum[hh] = d.sink && n_sl == 1 ? s + expf(d.sink[h0 + hh] - m) : s; }
   }
   __syncthreads();
   // weighted values: CB lanes along the columns (eight each), the rest of the work-group along the keys
@@ -316,6 +316,7 @@ __global__ __launch_bounds__(256) void attn_rows_merge_kernel(const AttnDims d, 
     m = fmaxf(fmaxf(sm[0], sm[1]), fmaxf(sm[2], sm[3]));
     for (int s = tid; s < used; s += 256) l += p[s * st + d.vdim_p + 1] * expf(p[s * st + d.vdim_p] - m);
     for (int o = 32; o; o >>= 1) l += __shfl_xor(l, o);
+    if (d.sink && tid == 0) l += expf(d.sink[h] - m);    // (counts once, whatever the number of slices)
     if ((tid & 63) == 0) sl[tid >> 6] = l;
   }
   float acc = 0.0f;
@@ -343,8 +344,8 @@ __global__ __launch_bounds__(256) void attn_rows_merge_kernel(const AttnDims d, 
 // O^T = V^T P^T as they are: key slot (lane group g, j) of a 32-key step is key 4 g + j of its first 16 keys for j < 4 and
 // 4 g + j - 4 of its second 16 otherwise, and V^T is read from LDS in that order.
 // ------------------------------------------------------------------------------------------
-template <int KQ, int VQ, bool SIG>        // key width in 32s, value width in 16s; sigmoid weights
-__global__ __launch_bounds__(256) void attn_prompt_paged_kernel(const AttnDims d, const KvView kv, const AttnIn in, const bf16_t* qbuf, const StepRows r, const int32_t* tiles, bf16_t* out, const int64_t ldo)
+template <int KQ, int VQ, bool SIG, bool FLAT>   // key width in 32s, value width in 16s; sigmoid weights; keys and values in rows (FlatKv)
+__global__ __launch_bounds__(256) void attn_prompt_paged_kernel(const AttnDims d, const KvView kv, const FlatKv flat, const AttnIn in, const bf16_t* qbuf, const StepRows r, const int32_t* tiles, bf16_t* out, const int64_t ldo)
 {
   constexpr int KST = KQ * 32 + 8, VST = PAGE_TOKENS + 4;
   __shared__ __align__(16) uint16_t sk[PAGE_TOKENS * KST];
@@ -386,9 +387,25 @@ __global__ __launch_bounds__(256) void attn_prompt_paged_kernel(const AttnDims d
   auto vtok = [](int e) { return ((e & 7) + (e / (VQ * 2 * 8)) * 8) * 2; };
   auto vcol = [](int e) { return (e >> 3) % (VQ * 2) * 8; };
   int page_no = kv.table[slot * kv.ring + first % kv.ring];
+  const bf16_t* flat_rows = FLAT ? reinterpret_cast<const bf16_t*>(flat.base) + (int64_t)flat.row0[tiles[2 * tile]] * flat.ld + (int64_t)g * flat.head : nullptr;
   auto fetch = [&](int pg) {
     const bf16_t* page = reinterpret_cast<const bf16_t*>(kv.base) + (int64_t)page_no * kv.page_elems;
     page_no = kv.table[slot * kv.ring + min(pg + 1, last) % kv.ring];      // (the next page's number, a page ahead)
+    if constexpr (FLAT) {
+      const bf16_t* rows = flat_rows + (int64_t)pg * PAGE_TOKENS * flat.ld;
+#pragma unroll
+      for (int i = 0; i < KC; i++) {
+        const int e = tid + 256 * i, t = e / (KQ * 4), c = e % (KQ * 4) * 8;
+        rk[i] = *reinterpret_cast<const u32x4*>(c < flat.split || c >= d.dim_p ? rows + (unsigned)(t * (int)flat.ld + (c < flat.split ? c : 0)) : page + (unsigned)(t * flat.page_row + flat.shared + c - flat.split));
+      }
+#pragma unroll
+      for (int i = 0; i < VC; i++) {
+        const int t = vtok(tid + 256 * i), c = vcol(tid + 256 * i);
+        const bf16_t* vp = rows + (unsigned)(t * (int)flat.ld + flat.v_off + (c < d.vdim_p ? c : 0));
+        rv[i][0] = *reinterpret_cast<const u32x4*>(vp); rv[i][1] = *reinterpret_cast<const u32x4*>(vp + flat.ld);
+      }
+      return;
+    }
 #pragma unroll
     for (int i = 0; i < KC; i++) {
       const int e = tid + 256 * i, t = e / (KQ * 4), c = e % (KQ * 4) * 8;
@@ -503,6 +520,7 @@ __global__ __launch_bounds__(256) void attn_prompt_paged_kernel(const AttnDims d
     }
   }
   l += __shfl_xor(l, 16); l += __shfl_xor(l, 32);
+  if (!SIG && d.sink) l += __builtin_amdgcn_exp2f(d.sink[h] * 1.44269504088896340736f - m);
   if (qi < n) {
     const float inv = SIG ? 1.0f : 1.0f / l;
 #pragma unroll
@@ -574,12 +592,26 @@ bool attn_paged_prompt_ok(const AttnDims& d, int act_t) { return act_t == ACT_T_
 int attn_paged_prompt(const AttnDims& d, const KvView& kv, const AttnIn& in, const void* qbuf, const StepRows& r, const int32_t* tiles, int n_tiles, void* out, int64_t ldo)
 {
   const dim3 grid(n_tiles, d.heads), blk(256);
-#define PROMPT_S(K, V, S) hipLaunchKernelGGL((attn_prompt_paged_kernel<K, V, S>), grid, blk, 0, ctx().stream, d, kv, in, (const bf16_t*)qbuf, r, tiles, (bf16_t*)out, ldo)
-#define PROMPT(K, V) do { if (d.sigmoid) PROMPT_S(K, V, true); else PROMPT_S(K, V, false); } while (0)
-#define PROMPT_V(K) do { if (d.vdim <= 64) PROMPT(K, 4); else if (d.vdim <= 128) PROMPT(K, 8); else PROMPT(K, 16); } while (0)
-  if (d.dim <= 64) PROMPT_V(2); else if (d.dim <= 128) PROMPT_V(4); else PROMPT_V(8);
+#define PROMPT_S(K, V, S, F) hipLaunchKernelGGL((attn_prompt_paged_kernel<K, V, S, F>), grid, blk, 0, ctx().stream, d, kv, f, in, (const bf16_t*)qbuf, r, tiles, (bf16_t*)out, ldo)
+#define PROMPT_V(K, P) do { if (d.vdim <= 64) P(K, 4); else if (d.vdim <= 128) P(K, 8); else P(K, 16); } while (0)
+#define PROMPT_K(P) do { if (d.dim <= 64) PROMPT_V(2, P); else if (d.dim <= 128) PROMPT_V(4, P); else PROMPT_V(8, P); } while (0)
+#define PAGED(K, V) do { if (d.sigmoid) PROMPT_S(K, V, true, false); else PROMPT_S(K, V, false, false); } while (0)
+  const FlatKv f;
+  PROMPT_K(PAGED);
+#undef PAGED
+  CAI_HIP(hipGetLastError());
+  return CAI_OK;
+}
+
+int attn_flat_prompt(const AttnDims& d, const KvView& kv, const FlatKv& f, const AttnIn& in, const void* qbuf, const StepRows& r, const int32_t* tiles, int n_tiles, void* out, int64_t ldo)
+{
+  CAI_REQUIRE(!d.sigmoid && f.base && f.row0 && f.split % 8 == 0 && f.shared % 8 == 0 && f.ld % 8 == 0 && f.ld < (1 << 24), "attention over rows: %d shared columns from %d, rows of %lld", f.shared, f.split, (long long)f.ld);
+  const dim3 grid(n_tiles, d.heads), blk(256);
+#define FLAT(K, V) PROMPT_S(K, V, false, true)
+  PROMPT_K(FLAT);
+#undef FLAT
+#undef PROMPT_K
 #undef PROMPT_V
-#undef PROMPT
 #undef PROMPT_S
   CAI_HIP(hipGetLastError());
   return CAI_OK;

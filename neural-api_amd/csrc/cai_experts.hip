@@ -2,7 +2,7 @@
 //
 // The experts' gated matrices lie one after the other in one bank, and so do their output matrices.  A chosen expert's weight
 // multiplies its gated activations, which the output product is linear in, so that the sum over a row's experts is one long product.
-// Everything about the routing is 32-bit.
+// Experts without a gate have one matrix and an activation in the gated one's place.  Everything about the routing is 32-bit.
 #include "cai_lin_epilogue.hpp"
 
 #include <algorithm>
@@ -34,7 +34,13 @@ __device__ __forceinline__ float lanes_total(float v)
 }
 
 // How a row's experts are chosen and weighted.
-struct Routing { const float* correction; int n, top, among; float scale; };
+struct Routing { const float* correction; int n, top, route; float scale; int groups, keep, per_group; };
+
+__device__ __forceinline__ float route_sigmoid(float z)
+{
+  if (z >= 0.0f) return 1.0f / (1.0f + expf(-z));
+  const float s = expf(z); return s / (1.0f + s);
+}
 
 // One row's experts, by one wave: lane k < top ends with the k-th choice and its weight.  Equal choice scores: the lower index.
 __device__ __forceinline__ void route_row(const float* z, const Routing& q, const int lane, int& expert, float& weight)
@@ -45,16 +51,42 @@ __device__ __forceinline__ void route_row(const float* z, const Routing& q, cons
   float s[PER], c[PER], m = -INFINITY, sum = 0.0f;
 #pragma unroll
   for (int i = 0; i < PER; i++) { const int e = lane + 64 * i; s[i] = e < n ? z[e] : -INFINITY; c[i] = e < n && correction ? correction[e] : 0.0f; m = fmaxf(m, s[i]); }
-  m = wave_max(m);
-  if (!q.among) {
+  const bool sigmoid = q.route == ROUTE_SIGMOID;
+  uint64_t kept = ~0ull;                   // groups that take part
+  const int per_group = q.per_group;
+  if (sigmoid) {
+#pragma unroll
+    for (int i = 0; i < PER; i++) if (64 * i < n) s[i] = route_sigmoid(s[i]);
+    if (q.keep < q.groups) {               // a lane a group: its two largest choice scores
+      float a = -INFINITY, b = -INFINITY;
+      if (lane < q.groups)
+#pragma unroll 4
+        for (int i = 0; i < per_group; i++) {
+          const int e = lane * per_group + i;
+          const float v = route_sigmoid(z[e]) + (correction ? correction[e] : 0.0f);
+          b = fmaxf(b, fminf(a, v)); a = fmaxf(a, v);
+        }
+      float score = lane >= q.groups ? -INFINITY : per_group > 1 ? a + b : a;
+      kept = 0;
+      for (int k = 0; k < q.keep; k++) {
+        const float most = wave_max(score);
+        const int g = wave_min(score == most && !(kept >> lane & 1) ? lane : 63);
+        kept |= 1ull << g;
+        if (lane == g) score = -INFINITY;
+      }
+    }
+  } else m = wave_max(m);
+  if (q.route == ROUTE_ALL) {
 #pragma unroll
     for (int i = 0; i < PER; i++) if (64 * i < n) { s[i] = expf(s[i] - m); sum += s[i]; }
     sum = lanes_total(sum);
   }
 #pragma unroll
   for (int i = 0; i < PER; i++) {
-    if (64 * i < n && !q.among) s[i] /= sum;
-    c[i] = lane + 64 * i < n ? s[i] + c[i] : -INFINITY;
+    if (64 * i < n && q.route == ROUTE_ALL) s[i] /= sum;
+    bool in = lane + 64 * i < n;
+    if (64 * i < n && sigmoid) in = in && (kept >> ((lane + 64 * i) / per_group & 63) & 1);
+    c[i] = in ? s[i] + c[i] : -INFINITY;
   }
   expert = 0; weight = 0.0f;
   float total = 0.0f;
@@ -65,13 +97,13 @@ __device__ __forceinline__ void route_row(const float* z, const Routing& q, cons
     const float most = wave_max(bv);
     be = wave_min(bv == most ? be : n - 1);
     bs = __builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, bs), be & 63));
-    if (q.among) bs = expf(bs - m);        // (m is the largest logit, the first choice)
+    if (q.route == ROUTE_AMONG) bs = expf(bs - m);       // (m is the largest logit, the first choice)
     total += bs;
     if (lane == k) { expert = be; weight = bs; }
 #pragma unroll
     for (int i = 0; i < PER; i++) if (lane + 64 * i == be) c[i] = -INFINITY;
   }
-  weight = weight / (total + 1e-20f) * q.scale;
+  weight = sigmoid ? weight * q.scale : weight / (total + 1e-20f) * q.scale;
 }
 
 // eight activations times eight weights
@@ -93,11 +125,12 @@ template <typename AT> __device__ __forceinline__ float dot8(const AT* x, const 
 // Up to EXPERTS_FEW rows.  The gate and up kernel takes blockIdx x = outputs, y = entry; a wave makes two outputs of every row of its
 // entry, so that a matrix is read once however many rows chose it.  The entries of one row are its choices, and every wave routes the
 // row itself; for more rows a launch before it routes them and lists the experts that were chosen.  The last entry is the shared one.
+// Experts that are not gated: four outputs a wave.
 // ------------------------------------------------------------------------------------------
 struct FewEntry { int32_t expert, n_rows; uint8_t row[EXPERTS_FEW], slot[EXPERTS_FEW]; };
 static_assert(sizeof(FewEntry) == EXPERTS_FEW_WORDS * 4, "size of a listed expert");
 struct FewGateUp {
-  const uint16_t *w, *ws; int ldw, gu_rows; Routing q; int ff, ff_s; float limit, limit_s; int glu, glu_s; int mid_p, active; int n_rows;
+  const uint16_t *w, *ws; int ldw, gu_rows; Routing q; int ff, ff_s; float limit, limit_s; int glu, glu_s; int mid_p, active; int n_rows; int act;
 };
 
 __global__ __launch_bounds__(64 * EXPERTS_FEW) void experts_few_kernel(const float* z, const int64_t ldz, const Routing q, const int n_rows, float* wgt, FewEntry* list, int32_t* n_list)
@@ -130,13 +163,14 @@ __global__ __launch_bounds__(64 * EXPERTS_FEW) void experts_few_kernel(const flo
   if (tid == 0) *n_list = total;
 }
 
-template <typename AT, int NB>
+template <typename AT, int NB, bool GATED>
 __global__ __launch_bounds__(256) void experts_gateup_kernel(const FewGateUp p, const float* z, const float* wgt, const FewEntry* list, const int32_t* n_list, const AT* h, const int64_t ldh, int32_t* sel, AT* mid)
 {
   constexpr int UNROLL = NB == 1 ? 2 : 1;
   const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), entry = blockIdx.y;
   const bool shared = p.ws && entry == (int)gridDim.y - 1;
-  const int ff = shared ? p.ff_s : p.ff, j0 = (blockIdx.x * 4 + wave) * 2;
+  constexpr int OUT = GATED ? 2 : 4;
+  const int ff = shared ? p.ff_s : p.ff, j0 = (blockIdx.x * 4 + wave) * OUT;
   if (j0 >= ff) return;
   const uint16_t* W = p.ws;
   float weight = 1.0f;
@@ -153,7 +187,9 @@ __global__ __launch_bounds__(256) void experts_gateup_kernel(const FewGateUp p, 
     }
   }
   const int j1 = min(j0 + 1, ff - 1);
-  const uint16_t* wr[4] = {W + (int64_t)glu_row(j0, 0) * p.ldw, W + (int64_t)glu_row(j0, 1) * p.ldw, W + (int64_t)glu_row(j1, 0) * p.ldw, W + (int64_t)glu_row(j1, 1) * p.ldw};
+  const uint16_t* wr[4];
+#pragma unroll
+  for (int i = 0; i < 4; i++) wr[i] = W + (int64_t)(GATED ? glu_row(i < 2 ? j0 : j1, i & 1) : min(j0 + i, ff - 1)) * p.ldw;
   const AT* x[NB];
 #pragma unroll
   for (int b = 0; b < NB; b++) x[b] = h + (int64_t)(NB == 1 || b >= nb ? 0 : shared ? b : list[entry].row[b]) * ldh;
@@ -181,7 +217,10 @@ __global__ __launch_bounds__(256) void experts_gateup_kernel(const FewGateUp p, 
     for (int i = 0; i < 4; i++) acc[b][i] = lanes_total(acc[b][i]);
     const int row = NB == 1 ? 0 : shared ? b : list[entry].row[b], slot = NB == 1 ? entry : shared ? p.q.top : list[entry].slot[b];
     if (NB > 1) weight = shared ? 1.0f : wgt[row * p.q.top + slot];
-    if (lane < 2 && j0 + lane < ff)
+    if constexpr (!GATED) {
+      if (lane < 4 && j0 + lane < ff)
+        put_act<AT>(mid, (int64_t)row * p.active + slot * p.mid_p + j0 + lane, lin_act(lane & 2 ? (lane & 1 ? acc[b][3] : acc[b][2]) : lane & 1 ? acc[b][1] : acc[b][0], p.act, 0.0f) * weight);
+    } else if (lane < 2 && j0 + lane < ff)
       put_act<AT>(mid, (int64_t)row * p.active + slot * p.mid_p + j0 + lane,
                   glu_pair(shared ? p.glu_s : p.glu, shared ? p.limit_s : p.limit, lane ? acc[b][2] : acc[b][0], lane ? acc[b][3] : acc[b][1]) * weight);
   }
@@ -386,7 +425,7 @@ __global__ __launch_bounds__(256) void experts_sum_kernel(const float* y, const 
   }
 }
 
-static Routing routing(const NetExperts& x) { return Routing{x.correction, x.n, x.top, x.route == ROUTE_AMONG, x.scale}; }
+static Routing routing(const NetExperts& x) { return Routing{x.correction, x.n, x.top, x.route, x.scale, x.groups, x.keep, x.n / x.groups}; }
 
 template <typename AT, int NB>
 static void run_few(const NetExperts& x, int width, const AT* h, int64_t ldh, int n_rows, const float* z, int64_t ldz, const ExpertBuf& b, const LinEpi& res, const BesideLin* beside)
@@ -394,21 +433,26 @@ static void run_few(const NetExperts& x, int width, const AT* h, int64_t ldh, in
   auto st = ctx().stream;
   const uint16_t *sg = x.s_gateup ? (const uint16_t*)x.s_gateup->data : nullptr, *sd = x.s_down ? (const uint16_t*)x.s_down->data : nullptr;
   const FewGateUp p{(const uint16_t*)x.gateup->data, sg, (int)x.gateup->ld, x.gu_rows(), routing(x), x.ff, x.ff_shared,
-                    x.limit, x.limit_shared, x.glu, x.glu_shared, x.mid_p(), x.active(), n_rows};
+                    x.limit, x.limit_shared, x.glu, x.glu_shared, x.mid_p(), x.active(), n_rows, x.act};
   FewEntry* list = (FewEntry*)b.few;
   if (NB > 1) hipLaunchKernelGGL(experts_few_kernel, dim3(1), dim3(64 * EXPERTS_FEW), 0, st, z, ldz, p.q, n_rows, b.wgt, list, b.n_tiles);
   const int entries = NB == 1 ? x.top : std::min(x.n, n_rows * x.top);
-  hipLaunchKernelGGL((experts_gateup_kernel<AT, NB>), dim3((std::max(x.ff, x.ff_shared) + 7) / 8, entries + (sg ? 1 : 0)), dim3(256), 0, st, p, z, b.wgt, list, b.n_tiles, h, ldh, b.sel, (AT*)b.mid);
+  if (x.gated) hipLaunchKernelGGL((experts_gateup_kernel<AT, NB, true>), dim3((std::max(x.ff, x.ff_shared) + 7) / 8, entries + (sg ? 1 : 0)), dim3(256), 0, st, p, z, b.wgt, list, b.n_tiles, h, ldh, b.sel, (AT*)b.mid);
+  else hipLaunchKernelGGL((experts_gateup_kernel<AT, NB, false>), dim3((x.ff + 15) / 16, entries), dim3(256), 0, st, p, z, b.wgt, list, b.n_tiles, h, ldh, b.sel, (AT*)b.mid);
   BesideArg o;
   if (beside) { o.w = (const uint16_t*)beside->w->data; o.x = beside->x; o.ld = (int)beside->w->ld; o.ldx = beside->ldx; o.e = beside->e; }
   const int lds = x.s_down ? (int)x.s_down->ld : 0;
   const dim3 outs((width + 7) / 8, NB == 1 ? 1 : entries + (sd || beside ? 1 : 0));
   if constexpr (NB == 1)
-    hipLaunchKernelGGL(experts_down_kernel<AT>, outs, dim3(256), 0, st, (const uint16_t*)x.down->data, sd, (int)x.down->ld, lds, x.top, width, x.n, b.sel, (const AT*)b.mid, res, o);
+  {
+    LinEpi e = res;
+    if (!e.y) { e.y = b.y; e.ldy = width; }
+    hipLaunchKernelGGL(experts_down_kernel<AT>, outs, dim3(256), 0, st, (const uint16_t*)x.down->data, sd, (int)x.down->ld, lds, x.top, width, x.n, b.sel, (const AT*)b.mid, e, o);
+  }
   else {
     hipLaunchKernelGGL((experts_out_kernel<AT, NB>), outs, dim3(256), 0, st, (const uint16_t*)x.down->data, beside ? o.w : sd, (int)x.down->ld, beside ? o.ld : lds, x.top, x.active(), width, n_rows, list, b.n_tiles, (const AT*)b.mid, b.y, b.ys,
                        (const AT*)o.x, o.ldx);
-    hipLaunchKernelGGL(experts_sum_kernel<AT>, dim3(std::min((width + 255) / 256, 32), n_rows), dim3(256), 0, st, b.y, sd || beside ? b.ys : nullptr, x.top, width, res, o.e);
+    if (res.y) hipLaunchKernelGGL(experts_sum_kernel<AT>, dim3(std::min((width + 255) / 256, 32), n_rows), dim3(256), 0, st, b.y, sd || beside ? b.ys : nullptr, x.top, width, res, o.e);
   }
 }
 
@@ -438,7 +482,7 @@ static int run(const NetExperts& x, int width, int act_t, const AT* h, int64_t l
   const int tile = n_rows * x.top >= x.n * 96 ? BANK_TILE_MAX : BANK_TILE;       // (by the mean number of rows of an expert)
   hipLaunchKernelGGL(experts_order_kernel, dim3(1), dim3(1024), 0, st, b.sel, x.n, n_rows * x.top, tile, b.order, b.tiles, b.n_tiles);
   BankList l{b.tiles, b.n_tiles, b.order, b.wgt, x.top, tile, x.max_tiles(n_rows, tile)};
-  { LinEpi e; e.mode = EPI_GLU; e.h = b.mid; e.ldh = x.mid_p(); e.glu = x.glu; e.limit = x.limit; if ((rc = launch_lin_bank(x.gateup, x.gu_rows(), act_t, h, ldh, l, e))) return rc; }
+  { LinEpi e; e.mode = x.gated ? EPI_GLU : EPI_SPLIT; e.h = b.mid; e.ldh = x.mid_p(); e.glu = x.glu; e.limit = x.limit; e.act = x.act; if ((rc = launch_lin_bank(x.gateup, x.gu_rows(), act_t, h, ldh, l, e))) return rc; }
   l.div = 0;
   { LinEpi e; e.y = b.y; e.ldy = width; if ((rc = launch_lin_bank(x.down, width, act_t, b.mid, x.mid_p(), l, e))) return rc; }
   if (x.ff_shared) {
@@ -447,7 +491,7 @@ static int run(const NetExperts& x, int width, int act_t, const AT* h, int64_t l
     LinEpi s; s.y = b.ys; s.ldy = width;
     if ((rc = launch_lin(x.s_down, act_t, b.mid_s, x.shared_p(), n_rows, s))) return rc;
   }
-  hipLaunchKernelGGL(experts_sum_kernel<AT>, dim3(std::min((width + 255) / 256, 32), n_rows), dim3(256), 0, st, b.y, x.ff_shared ? b.ys : nullptr, x.top, width, res, LinEpi());
+  if (res.y) hipLaunchKernelGGL(experts_sum_kernel<AT>, dim3(std::min((width + 255) / 256, 32), n_rows), dim3(256), 0, st, b.y, x.ff_shared ? b.ys : nullptr, x.top, width, res, LinEpi());
   CAI_HIP(hipGetLastError());
   return CAI_OK;
 }
@@ -455,6 +499,9 @@ static int run(const NetExperts& x, int width, int act_t, const AT* h, int64_t l
 int experts_run(const NetExperts& x, int width, int act_t, const void* h, int64_t ldh, int n_rows, const float* z, int64_t ldz, const ExpertBuf& b, const LinEpi& res, const BesideLin* beside)
 {
   CAI_REQUIRE(!beside || (n_rows <= EXPERTS_FEW && !x.ff_shared && beside->w->rows == width && beside->e.mode == EPI_JOIN && res.mode == EPI_JOIN), "experts: a product of another kind beside them");
+  CAI_REQUIRE(x.gated || !x.ff_shared, "experts: a shared one beside experts without a gate");
+  CAI_REQUIRE(res.y || (res.mode == EPI_STORE && !x.ff_shared && !beside), "experts: outputs left apart with something beside them");
+  CAI_REQUIRE(x.groups >= 1 && x.groups <= EXPERTS_GROUPS && x.n % x.groups == 0 && x.keep >= 1 && x.keep <= x.groups, "experts: %d of %d groups of %d", x.keep, x.groups, x.n);
   CAI_REQUIRE(z || x.router, "experts: neither logits nor a router");
   CAI_REQUIRE(x.n >= 1 && x.n <= EXPERTS_MAX && x.top >= 1 && x.top <= std::min(x.n, EXPERTS_TOP), "experts: %d of %d", x.top, x.n);
   return act_t == ACT_T_BF16 ? run<bf16_t>(x, width, act_t, (const bf16_t*)h, ldh, n_rows, z, ldz, b, res, beside) : run<float>(x, width, act_t, (const float*)h, ldh, n_rows, z, ldz, b, res, beside);

@@ -6,7 +6,8 @@
 // The residual stream is float.  Behind Dynamic Tanh a sublayer's epilogue adds its result and already leaves the next sublayer's
 // normed input, so between two mixers with a dense feed-forward there are three products and nothing else.  Layers whose feed-forward
 // works beside the mixer have RMS norms: a small step takes both norms into the one launch of the layer's input matrices and joins
-// both results in one other launch; a prompt norms the rows first.
+// both results in one other launch; a prompt norms the rows first.  Sublayers that stand in RMS norms (a sandwich) leave their result in
+// 32-bit, and one launch a row does everything between it and the next sublayer's input (cai_stream.hip).
 #include "cai_layered.hpp"
 
 #include <algorithm>
@@ -34,10 +35,11 @@ int SeqPool::alloc(int n_seq_, int max_tokens, int act_t_)
     CAI_HIP(hipMemsetAsync(a.base, 0, (size_t)n_pages * a.page_elems * es, s));
   }
   for (auto& d : state) {
-    CAI_HIP(hipMalloc((void**)&d.S, (size_t)n_seq * d.s_elems * 4));
-    CAI_HIP(hipMalloc((void**)&d.hist, (size_t)n_seq * d.h_elems * 4));
-    CAI_HIP(hipMemsetAsync(d.S, 0, (size_t)n_seq * d.s_elems * 4, s));
-    CAI_HIP(hipMemsetAsync(d.hist, 0, (size_t)n_seq * d.h_elems * 4, s));
+    for (auto& part : {std::make_pair(&d.S, d.s_elems), std::make_pair(&d.hist, d.h_elems)}) {
+      if (!part.second) continue;
+      CAI_HIP(hipMalloc((void**)part.first, (size_t)n_seq * part.second * 4));
+      CAI_HIP(hipMemsetAsync(*part.first, 0, (size_t)n_seq * part.second * 4, s));
+    }
   }
   if (n_pages) {
     table.assign((size_t)n_seq * n_pages, 0);
@@ -126,8 +128,8 @@ int SeqPool::fork(int src, int dst)
     table_dirty = true;
   }
   for (auto& r : state) {
-    CAI_HIP(hipMemcpyAsync(r.S + dst * r.s_elems, r.S + src * r.s_elems, (size_t)r.s_elems * 4, hipMemcpyDeviceToDevice, s));
-    CAI_HIP(hipMemcpyAsync(r.hist + dst * r.h_elems, r.hist + src * r.h_elems, (size_t)r.h_elems * 4, hipMemcpyDeviceToDevice, s));
+    if (r.s_elems) CAI_HIP(hipMemcpyAsync(r.S + dst * r.s_elems, r.S + src * r.s_elems, (size_t)r.s_elems * 4, hipMemcpyDeviceToDevice, s));
+    if (r.h_elems) CAI_HIP(hipMemcpyAsync(r.hist + dst * r.h_elems, r.hist + src * r.h_elems, (size_t)r.h_elems * 4, hipMemcpyDeviceToDevice, s));
   }
   b.len = a.len;
   return CAI_OK;
@@ -255,12 +257,17 @@ struct LayeredNet {
   size_t part_floats = 0;
   int64_t w_cb = 0, w_sx = 0, w_sb = 0, w_sdt = 0, w_sy = 0;                       // state-space scratch, elements per row (cb: per chunk)
   int64_t w_ez = 0, w_ep = 0, w_emid = 0, w_emid_s = 0, w_etiles = 0;              // experts: scores, pairs, activations of a row's pairs, of the shared expert, most tiles of experts
-  bool has_parallel = false, looped = false;
+  int ld_ql = 0, ld_qr = 0, ld_lat = 0; int64_t w_qa = 0; bool has_latent = false;   // latent attention: queries' latent, queries, latents, queries in the latent's space
+  bool has_parallel = false, has_sandwich = false, looped = false;
   int cap = 0, logit_cap = 0;
   float *x = nullptr, *x0 = nullptr, *proj = nullptr, *yl = nullptr, *yr = nullptr, *part = nullptr, *logits = nullptr;
   void *h = nullptr, *mid = nullptr, *att = nullptr, *attl = nullptr, *qbuf = nullptr, *ra = nullptr, *rgb = nullptr, *hw = nullptr;
   void* cat = nullptr;                     // [stream; embedding] in front of a pass
   void* h2 = nullptr; float* g2 = nullptr; // layers beside: the feed-forward's input, its gate logits and the router's
+  float *kept = nullptr, *inv = nullptr;   // sandwiches: embedding output and layer results [layers + 1][rows][width]; reciprocal roots
+  void *ql = nullptr; float *qraw = nullptr, *qabs = nullptr;
+  int64_t w_flat = 0, flat_cap = 0;        // keys and values of the expanded form, elements per row; rows there are
+  void *lat = nullptr, *flat = nullptr;
   DeltaBuf db{};
   SsdBuf sb{};
   ExpertBuf eb{};
@@ -290,12 +297,12 @@ static void drop_graphs(LayeredNet* n)
 
 static void free_rows(LayeredNet* n)
 {
-  void* p[] = {n->x, n->x0, n->proj, n->yl, n->yr, n->part, n->h, n->mid, n->att, n->attl, n->qbuf, n->ra, n->rgb, n->db.q, n->db.k, n->db.v, n->db.g, n->db.beta, n->db.o, n->db.za, n->db.zg, n->db.w, n->db.qt, n->db.qk, n->db.gt, n->cat, n->h2, n->g2,
+  void* p[] = {n->x, n->x0, n->proj, n->yl, n->yr, n->part, n->h, n->mid, n->att, n->attl, n->qbuf, n->ra, n->rgb, n->db.q, n->db.k, n->db.v, n->db.g, n->db.beta, n->db.o, n->db.za, n->db.zg, n->db.w, n->db.qt, n->db.qk, n->db.gt, n->cat, n->h2, n->g2, n->kept, n->inv, n->ql, n->qraw, n->qabs,
                n->sb.x, n->sb.B, n->sb.C, n->sb.dt, n->sb.cb, n->sb.bt, n->sb.fac, n->sb.y, n->eb.z, n->eb.wgt, n->eb.y, n->eb.ys, n->eb.sel, n->eb.order, n->eb.tiles, n->eb.n_tiles, n->eb.few, n->eb.mid, n->eb.mid_s};
   for (void* q : p) if (q) (void)hipFree(q);
   n->x = n->x0 = n->proj = n->yl = n->yr = n->part = nullptr;
   n->h = n->mid = n->att = n->attl = n->qbuf = n->ra = n->rgb = nullptr;
-  n->cat = n->h2 = nullptr; n->g2 = nullptr;
+  n->cat = n->h2 = n->ql = nullptr; n->g2 = n->kept = n->inv = n->qraw = n->qabs = nullptr;
   n->db = DeltaBuf{}; n->sb = SsdBuf{}; n->eb = ExpertBuf{};
   n->cap = 0;
 }
@@ -319,10 +326,11 @@ static int ensure_rows(LayeredNet* n, int rows)
   // (with bfloat16 activations only steps without a prompt portion take the row form)
   const int part_rows = n->act_t == ACT_T_F32 ? (int)R : std::min((int)R, ATTN_PROMPT_MIN * n->max_seq);
   for (auto& d : n->pool.readers) part = std::max(part, attn_paged_part_floats(d, part_rows));
+  for (auto& y : n->s.layers) if (y.kind == MIX_LATENT) part = std::max(part, latent_part_floats(y.latent.d, n->act_t == ACT_T_F32 ? (int)R : std::min((int)R, LATENT_EXPAND_MIN * n->max_seq)));
   n->part_floats = part;
   int rc;
-  if ((rc = get((void**)&n->x, R * w * 4)) || (rc = get((void**)&n->x0, n->looped ? R * w * 4 : 0)) || (rc = get((void**)&n->proj, R * n->ld_proj * 4)) ||
-      (rc = get((void**)&n->yl, n->has_parallel ? R * w * 4 : 0)) || (rc = get((void**)&n->yr, n->has_parallel ? R * w * 4 : 0)) || (rc = get((void**)&n->part, part * 4)) ||
+  if ((rc = get((void**)&n->x, R * w * 4)) || (rc = get((void**)&n->x0, n->looped ? R * w * 4 : 0)) || (rc = get((void**)&n->proj, RS * n->ld_proj * 4)) ||
+      (rc = get((void**)&n->yl, n->has_parallel || n->has_sandwich ? R * w * 4 : 0)) || (rc = get((void**)&n->yr, n->has_parallel ? R * w * 4 : 0)) || (rc = get((void**)&n->part, part * 4)) ||
       (rc = get(&n->h, R * n->wp * n->es)) || (rc = get(&n->mid, R * n->ld_mid * n->es)) || (rc = get(&n->att, R * n->ld_att * n->es)) ||
       (rc = get(&n->attl, R * n->ld_attl * n->es)) || (rc = get(&n->qbuf, R * n->ld_q * n->es)) || (rc = get(&n->ra, R * n->ld_ra * n->es)) || (rc = get(&n->rgb, R * n->ld_rg * n->es)) ||
       (rc = get((void**)&n->db.q, RS * n->w_q * 4)) || (rc = get((void**)&n->db.k, RS * n->w_k * 4)) || (rc = get((void**)&n->db.v, RS * n->w_v * 4)) ||
@@ -331,6 +339,8 @@ static int ensure_rows(LayeredNet* n, int rows)
       (rc = get((void**)&n->db.w, RS * n->w_hd * 4)) || (rc = get((void**)&n->db.qt, RS * n->w_qt * 4)) || (rc = get((void**)&n->db.qk, RS * n->w_qk * 4)) ||
       (rc = get((void**)&n->db.gt, std::max(RS * n->w_gt1, (R / DELTA_CHUNK + n->max_seq + 1) * n->w_qt + 4) * 4)) ||
       (rc = get(&n->cat, R * n->ld_cat * n->es)) || (rc = get(&n->h2, R * n->ld_h2 * n->es)) || (rc = get((void**)&n->g2, R * n->ld_g2 * 4)) ||
+      (rc = get((void**)&n->kept, n->has_sandwich ? (n->s.layers.size() + 1) * R * w * 4 : 0)) || (rc = get((void**)&n->inv, n->has_sandwich ? R * 4 : 0)) ||
+      (rc = get(&n->ql, R * n->ld_ql * n->es)) || (rc = get((void**)&n->qraw, R * n->ld_qr * 4)) || (rc = get((void**)&n->qabs, R * n->w_qa * 4)) ||
       (rc = get((void**)&n->sb.x, (R + SSD_CHUNK) * n->w_sx * 4)) || (rc = get((void**)&n->sb.B, R * n->w_sb * 4)) || (rc = get((void**)&n->sb.C, (R + SSD_CHUNK) * n->w_sb * 4)) ||
       (rc = get((void**)&n->sb.dt, R * n->w_sdt * 4)) || (rc = get((void**)&n->sb.cb, (R / SSD_CHUNK + n->max_seq + 1) * n->w_cb * 4)) || (rc = get((void**)&n->sb.y, R * n->w_sy * 4)) ||
       (rc = get((void**)&n->sb.bt, (R / SSD_CHUNK + n->max_seq + 1) * n->w_sb * SSD_CHUNK * 4)) || (rc = get((void**)&n->sb.fac, (R / SSD_CHUNK + n->max_seq + 1) * n->w_sdt * SSD_FACTORS * 4)) ||
@@ -340,6 +350,21 @@ static int ensure_rows(LayeredNet* n, int rows)
       (rc = get(&n->eb.mid, R * n->w_emid * n->es)) || (rc = get(&n->eb.mid_s, R * n->w_emid_s * n->es))) return rc;
   CAI_HIP(hipStreamSynchronize(ctx().stream));
   n->cap = (int)R;
+  return CAI_OK;
+}
+
+// rows of whole pages for the expanded form of latent attention (and a page of slack that the last tile may read)
+static int ensure_flat(LayeredNet* n, int64_t rows)
+{
+  if (n->flat_cap >= rows) return CAI_OK;
+  CAI_HIP(hipStreamSynchronize(ctx().stream));
+  for (void** p : {&n->lat, &n->flat}) { if (*p) (void)hipFree(*p); *p = nullptr; }
+  n->flat_cap = 0;
+  const int64_t R = rows + rows / 2 + PAGE_TOKENS;
+  CAI_HIP(hipMalloc(&n->lat, (size_t)R * n->ld_lat * 2));
+  CAI_HIP(hipMalloc(&n->flat, (size_t)R * n->w_flat * 2));
+  CAI_HIP(hipMemsetAsync(n->flat, 0, (size_t)R * n->w_flat * 2, ctx().stream));
+  n->flat_cap = R - PAGE_TOKENS;
   return CAI_OK;
 }
 
@@ -371,21 +396,28 @@ int net_create(NetSpec&& spec, int max_tokens, int max_seq, int act_t, LayeredNe
   const int L = (int)s.layers.size();
   std::vector<int> last_run(L, -1);        // a layer's latest run with pages of its own
   auto add_run = [&](int l, bool first, int pass) {
-    NetRun r{l, first && !s.loop_in && pass > 0, first && s.loop_in, -1, -1};
+    NetRun r{l, first && !s.loop_in && pass > 0, first && s.loop_in, -1, -1, -1};
     NetLayer& y = s.layers[l];
-    if (y.has_attn()) {
+    if (y.has_pages()) {
       // (a sequence longer than the pool exists only if every window is shorter than it: a wider window sees the same keys cut down)
       AttnDims& d = y.attn.d;
       d.span = std::min(d.window, (max_tokens + PAGE_TOKENS - 1) / PAGE_TOKENS * PAGE_TOKENS);
       if (!d.chunked) d.window = d.span;
+      y.latent.d.span = d.span;
       if (y.kv_from < 0) { r.attn_run = last_run[l] = (int)n->pool.attn.size(); n->pool.attn.push_back({d}); }
       else r.attn_run = last_run[y.kv_from];
       n->pool.readers.push_back(d);
     }
-    if (y.has_delta() || y.kind == MIX_SSD) {
-      const DeltaDims& d = y.delta.d; const SsdDims& m = y.ssd.d;
+    if (y.conv.w) {
       SeqPool::StateRun st;
-      if (y.kind == MIX_SSD) { st.s_elems = (int64_t)m.heads * m.state * m.vdim_p(); st.h_elems = (int64_t)m.taps * m.channels(); }
+      st.h_elems = (int64_t)y.conv.taps * s.width;
+      r.conv_run = (int)n->pool.state.size(); n->pool.state.push_back(st);
+    }
+    if (y.has_state()) {
+      const DeltaDims& d = y.delta.d; const SsdDims& m = y.ssd.d; const GlaDims& a = y.gla.d;
+      SeqPool::StateRun st;
+      if (y.kind == MIX_GLA) st.s_elems = (int64_t)a.heads * a.dim * a.vdim_p();
+      else if (y.kind == MIX_SSD) { st.s_elems = (int64_t)m.heads * m.state * m.vdim_p(); st.h_elems = (int64_t)m.taps * m.channels(); }
       else { st.s_elems = (int64_t)d.heads * d.dim * d.vdim_p(); st.h_elems = (int64_t)d.taps * d.channels(); }
       r.state_run = (int)n->pool.state.size(); n->pool.state.push_back(st);
     }
@@ -415,6 +447,19 @@ int net_create(NetSpec&& spec, int max_tokens, int max_seq, int act_t, LayeredNe
     if (y.in2) { up(n->ld_g2, pad_to(s.width + y.experts.n, 4)); n->ld_h2 = n->wp; }
     if (y.has_attn()) { up(n->ld_attl, pad_to(y.attn.d.heads * y.attn.d.vdim, LIN_PAD)); up(n->ld_q, y.attn.d.heads * y.attn.d.dim_p); }
     if (y.kind == MIX_PARALLEL) n->has_parallel = true;
+    if (y.sandwich) n->has_sandwich = true;
+    if (y.kind == MIX_LATENT) {
+      const LatentDims& d = y.latent.d;
+      n->has_latent = true;
+      up(n->ld_attl, pad_to(d.heads * d.vdim, LIN_PAD)); up(n->ld_q, d.heads * d.key_e());
+      up(n->ld_ql, pad_to(d.q_rank, LIN_PAD)); up(n->ld_qr, pad_to(d.heads * (d.dim + d.rot_dim), 4)); up(n->w_qa, d.heads * d.lat_p());
+      up(n->ld_lat, pad_to(d.kv_rank, LIN_PAD)); up(n->w_flat, d.heads * d.head_e());
+    }
+    if (y.kind == MIX_GLA) {
+      const GlaDims& d = y.gla.d;
+      up(n->ld_att, pad_to(d.heads * d.vdim, LIN_PAD));
+      up(n->w_v, d.heads * d.vdim); up(n->w_g, d.heads * d.dim); up(n->w_qt, d.heads * d.dim); up(n->w_qk, d.heads * DELTA_CHUNK);
+    }
     if (y.kind == MIX_SSD) {
       const SsdDims& d = y.ssd.d;
       up(n->ld_att, pad_to(d.inner(), LIN_PAD));
@@ -447,7 +492,7 @@ void net_destroy(LayeredNet* n)
   if (ctx().ready) (void)hipStreamSynchronize(ctx().stream);
   drop_graphs(n);
   free_rows(n);
-  void* p[] = {n->logits, n->hw, n->am_v, n->am_i, n->best, n->d_rows, n->d_dec, n->d_gen};
+  void* p[] = {n->logits, n->hw, n->am_v, n->am_i, n->best, n->d_rows, n->d_dec, n->d_gen, n->lat, n->flat};
   for (void* q : p) if (q) (void)hipFree(q);
   if (n->h_rows) (void)hipHostFree(n->h_rows);
   if (n->h_dec) (void)hipHostFree(n->h_dec);
@@ -457,10 +502,16 @@ void net_destroy(LayeredNet* n)
 }
 
 // Work lists of a step with prompt portions (device pointers): tiles of 64 rows and of DELTA_CHUNK rows (entry, first row in it), and
-// the first tile of each entry.  tall: some portion is long enough for the prompt attention kernel; chunks null: none is long enough
+// the first tile of each entry.  tall: some portion is long enough for the prompt attention kernel; chunked: some portion is long enough
 // for the chunked delta rule.
 static_assert(ATTN_TILE == SSD_CHUNK, "one list of tiles serves the prompt attention and the state-space walk");
-struct StepLists { const int32_t *tiles = nullptr, *tile0 = nullptr; int n_tiles = 0; bool tall = false; const int32_t* chunks = nullptr; int n_chunks = 0; const int32_t* chunk0 = nullptr; };
+// pages, row0, wide, short_rows: of nets with latent attention - the pages of the entries long enough for its expanded form (slot, page),
+// the first row of every such entry there, their tiles, and the rows of the other entries.
+struct StepLists {
+  const int32_t *tiles = nullptr, *tile0 = nullptr; int n_tiles = 0; bool tall = false;
+  const int32_t* chunks = nullptr; int n_chunks = 0; const int32_t* chunk0 = nullptr; bool chunked = false;
+  const int32_t *pages = nullptr, *row0 = nullptr, *wide = nullptr, *short_rows = nullptr; int n_pages = 0, n_wide = 0, n_short = 0;
+};
 
 template <typename AT>
 static void rms_rows_t(LayeredNet* n, const int32_t* rows, int n_rows, const float* g1, void* h1, const float* g2, void* h2)
@@ -497,7 +548,7 @@ static int enqueue_beside(LayeredNet* n, const NetRun& run, const NetLayer& y, c
   if (y.down) { b.mode = EPI_SPLIT; b.split = w; b.act = LIN_RELU_SQUARED; b.h = n->mid; b.ldh = n->ld_mid; }
   if (few) {                               // both norms inside one launch of both stacks of matrices
     const RmsLin first{y.in, y.rms1, a}, second{y.in2, y.rms2, b, y.experts.n ? n->h2 : nullptr, n->wp};
-    if ((rc = launch_lin_rms(at, n->x, w, n->s.eps, R, first, y.in2 ? &second : nullptr))) return rc;
+    if ((rc = launch_lin_rms(at, n->x, w, w, n->s.eps, R, first, y.in2 ? &second : nullptr))) return rc;
   } else {
     rms_rows(n, nullptr, R, y.rms1, n->h, y.rms2, y.has_mlp() ? n->h2 : nullptr);
     if ((rc = launch_lin(y.in, at, n->h, n->wp, R, a)) || (y.in2 && (rc = launch_lin(y.in2, at, n->h2, n->wp, R, b)))) return rc;
@@ -515,6 +566,123 @@ static int enqueue_beside(LayeredNet* n, const NetRun& run, const NetLayer& y, c
   return y.down ? launch_lin(y.down, at, n->mid, n->ld_mid, R, f) : CAI_OK;
 }
 
+static int enqueue_latent(LayeredNet* n, const NetRun& run, const NetLayer& y, const StepRows& r, bool single, const StepLists& lists)
+{
+  const NetLatent& L = y.latent;
+  const LatentDims& d = L.d;
+  const int at = n->act_t, R = r.n_rows;
+  const LatentIn in{n->proj, n->ld_proj, L.oq, L.okv, L.og, L.qn, L.kvn, n->qraw, n->ld_qr};
+  const KvView kv = n->pool.view(run.attn_run);
+  const bool few = R <= LIN_FEW;
+  int rc;
+  if (!single && (rc = latent_append(d, kv, at, in, r, few ? nullptr : n->ql, n->ld_ql))) return rc;
+  LinEpi e; e.y = n->qraw; e.ldy = n->ld_qr;
+  if (few) rc = launch_lin_rms(at, n->proj + L.oq, n->ld_proj, d.q_rank, d.eps, R, RmsLin{L.uq, L.qn, e}, nullptr);
+  else rc = launch_lin(L.uq, at, n->ql, n->ld_ql, R, e);
+  if (rc) return rc;
+  const bool wide = lists.n_wide > 0 && latent_expand_ok(d, at);
+  if (!wide || lists.n_short) {
+    const int32_t* rows = wide ? lists.short_rows : nullptr;
+    if ((rc = latent_rows(d, kv, at, in, L.up, r, rows, wide ? lists.n_short : R, single, n->qabs, n->part, n->part_floats, n->attl, n->ld_attl))) return rc;
+  }
+  if (!wide) return CAI_OK;
+  // the expanded form: keys and values of all positions of the longer entries
+  AttnDims a{};
+  a.heads = a.kv_heads = d.heads; a.dim = a.dim_p = d.key_e(); a.vdim = d.vdim; a.vdim_p = d.vdim_e(); a.window = y.attn.d.window; a.span = d.span; a.scale = d.scale;
+  const int64_t ldf = (int64_t)d.heads * d.head_e(), ldc = L.up->ld;
+  const FlatKv f{n->flat, ldf, d.head_e(), d.dim_e(), d.dim_e(), d.lat_p(), d.lat_c(), lists.row0};
+  const AttnIn ain{n->proj, n->ld_proj, 0, -1, -1, L.og, nullptr, nullptr};
+  LinEpi x; x.mode = EPI_SPLIT; x.split = 0; x.h = n->flat; x.ldh = ldf;
+  if ((rc = latent_queries(d, in, r, n->qbuf)) || (rc = latent_gather(d, kv, lists.pages, lists.n_pages, n->lat, ldc)) ||
+      (rc = launch_lin(L.up, at, n->lat, ldc, lists.n_pages * PAGE_TOKENS, x))) return rc;
+  return attn_flat_prompt(a, kv, f, ain, n->qbuf, r, lists.wide, lists.n_wide, n->attl, n->ld_attl);
+}
+
+// Norm (and convolution) in front of run i's mixer, or in front of the logits.
+static void sandwich_lead(LayeredNet* n, size_t i, StreamStep& s)
+{
+  if (i >= n->runs.size()) { s.next = n->s.rms_final; return; }
+  const NetLayer& y = n->s.layers[n->runs[i].layer];
+  s.next = y.rms1; s.conv = y.conv;
+  if (y.conv.w) { const SeqPool::StateRun& c = n->pool.state[n->runs[i].conv_run]; s.ring = c.hist; s.ring_elems = c.h_elems; }
+}
+static int sandwich_stream(LayeredNet* n, const StreamStep& s, const StepRows& r, bool single)
+{
+  const int rc = launch_stream(s, n->act_t, r, single);
+  return rc || single || !s.conv.w ? rc : launch_input_conv(s, n->act_t, r);
+}
+static StreamStep sandwich_step(LayeredNet* n)
+{
+  StreamStep s;
+  s.x = n->x; s.width = n->s.width; s.eps = n->s.eps; s.h = n->h; s.ldh = n->wp; s.inv = n->inv;
+  return s;
+}
+
+// A layer whose sublayers stand in RMS norms; its mixer's input is in h already.
+static int enqueue_sandwich(LayeredNet* n, size_t i, const StepRows& r, bool single, const StepLists& lists)
+{
+  const NetRun& run = n->runs[i];
+  const NetLayer& y = n->s.layers[run.layer];
+  const int R = r.n_rows, w = n->s.width, at = n->act_t;
+  int rc;
+  { LinEpi e; e.y = n->proj; e.ldy = n->ld_proj; e.bias = y.in_b; if ((rc = launch_lin(y.in, at, n->h, n->wp, R, e))) return rc; }
+  const cai_qw_s* out = y.attn.out; const void* heads = n->attl; int ldo = n->ld_attl;
+  if (y.kind == MIX_LATENT) { out = y.latent.out; rc = enqueue_latent(n, run, y, r, single, lists); }
+  else if (y.kind == MIX_GLA) {
+    const NetGla& G = y.gla;
+    const GlaIn gin{n->proj, n->ld_proj, G.oq, G.of, G.ov};
+    const SeqPool::StateRun& st = n->pool.state[run.state_run];
+    out = G.out; heads = n->att; ldo = n->ld_att;
+    rc = single ? gla_single(G.d, gin, G.w, st, r, at, n->att, ldo) : gla_chunked(G.d, gin, G.w, st, r, n->db, lists.chunks, lists.n_chunks, lists.chunk0, at, n->att, ldo);
+  } else rc = enqueue_attention(n, run, y, r, single, lists);
+  if (rc) return rc;
+  { LinEpi e; e.y = n->yl; e.ldy = w; if ((rc = launch_lin(out, at, heads, ldo, R, e))) return rc; }
+  StreamStep s = sandwich_step(n);
+  s.y = n->yl; s.post = y.rms1b;
+  if (y.conv.w && !single) { const SeqPool::StateRun& c = n->pool.state[run.conv_run]; s.keep_ring = c.hist; s.keep_elems = c.h_elems; s.keep_gain = y.rms1; s.keep_taps = y.conv.taps; }
+  if (y.has_mlp()) {
+    s.next = y.rms2;
+    if ((rc = launch_stream(s, at, r, single))) return rc;
+    LinEpi apart;
+    if ((rc = experts_run(y.experts, w, at, n->h, n->wp, R, nullptr, 0, n->eb, apart, nullptr))) return rc;
+    s = sandwich_step(n);
+    s.y = n->eb.y; s.parts = experts_parts(y.experts, R); s.post = y.rms2b;
+  }
+  s.kept = n->kept; s.kept_stride = (int64_t)n->cap * w; s.n_kept = (int)i + 1; s.avg = y.depth;
+  sandwich_lead(n, i + 1, s);
+  return sandwich_stream(n, s, r, single);
+}
+
+// Logits of the wanted rows (null: all), and their greedy choices.  A sandwich's last stream step has normed the rows already.
+static int enqueue_logits(LayeredNet* n, const int32_t* want, int n_want)
+{
+  if (n_want > 0) {
+    const NetSpec& s = n->s;
+    const int w = s.width, at = n->act_t;
+    const bool norm = s.rms_final && !n->has_sandwich;
+    auto st = ctx().stream;
+    const void* hs = n->h;
+    int rc;
+    LinEpi e; e.y = n->logits; e.ldy = s.vocab; e.scale = s.logit_scale;
+    if (s.logit_cap > 0.0f) { e.act = LIN_SOFT_CAP; e.limit = s.logit_cap; }
+    if (norm && !want && n_want <= LIN_FEW) {
+      if ((rc = launch_lin_rms(at, n->x, w, w, s.eps, n_want, RmsLin{s.head, s.rms_final, e, n->h, n->wp}, nullptr))) return rc;
+      hs = nullptr;
+    } else if (norm) {
+      if (want) hs = n->hw;
+      rms_rows(n, want, n_want, s.rms_final, (void*)hs);
+    } else if (want) {
+      if (at == ACT_T_BF16) hipLaunchKernelGGL(net_gather_kernel<bf16_t>, dim3(n_want), dim3(256), 0, st, (const bf16_t*)n->h, want, (int64_t)n->wp, (bf16_t*)n->hw);
+      else hipLaunchKernelGGL(net_gather_kernel<float>, dim3(n_want), dim3(256), 0, st, (const float*)n->h, want, (int64_t)n->wp, (float*)n->hw);
+      hs = n->hw;
+    }
+    if (hs && (rc = launch_lin(s.head, at, hs, n->wp, n_want, e))) return rc;
+    launch_argmax(n->logits, s.vocab, n_want, n->best, n->am_v, n->am_i);
+  }
+  CAI_HIP(hipGetLastError());
+  return CAI_OK;
+}
+
 // One step over the rows of `r`.  single: every entry is one row (the decode kernels).  want: device list of the rows whose
 // logits are produced (null: all rows, in order).
 static int enqueue_net(LayeredNet* n, const StepRows& r, bool single, const StepLists& lists, const int32_t* want, int n_want)
@@ -525,6 +693,14 @@ static int enqueue_net(LayeredNet* n, const StepRows& r, bool single, const Step
   int rc;
   auto norm1_of = [&](size_t i) -> const Dyt& { return s.layers[n->runs[i].layer].norm1; };
   const dim3 eg((unsigned)std::min((w + 255) / 256, 32), R);
+  if (n->has_sandwich) {
+    StreamStep e = sandwich_step(n);
+    e.embed = s.embed; e.embed_scale = s.embed_scale; e.kept = n->kept; e.kept_stride = (int64_t)n->cap * w;
+    sandwich_lead(n, 0, e);
+    if ((rc = sandwich_stream(n, e, r, single))) return rc;
+    for (size_t i = 0; i < n->runs.size(); i++) if ((rc = enqueue_sandwich(n, i, r, single, lists))) return rc;
+    return enqueue_logits(n, want, n_want);
+  }
   // where the stream goes after the last sublayer before run i: the norm of what follows, or as it is in front of loop_in
   auto lead_to = [&](size_t i, LinEpi& e) {
     if (i < n->runs.size() && n->runs[i].enter) { e.next = Dyt(); e.h = n->cat; e.ldh = n->ld_cat; return; }
@@ -567,7 +743,7 @@ static int enqueue_net(LayeredNet* n, const StepRows& r, bool single, const Step
           if ((rc = launch_pack_rows(n->proj, n->ld_proj, D.og, D.d.rank_g, R, at, n->rgb, n->ld_rg)) || (rc = launch_lin(D.w.g2, at, n->rgb, n->ld_rg, R, e))) return rc;
         }
         if ((rc = delta_prep(D.d, din, D.w, ds, r, n->db)) ||
-            (rc = lists.chunks ? delta_chunked(D.d, ds, r, n->db, lists.chunks, lists.n_chunks, lists.chunk0) : delta_scan(D.d, ds, r, n->db)) ||
+            (rc = lists.chunked ? delta_chunked(D.d, ds, r, n->db, lists.chunks, lists.n_chunks, lists.chunk0) : delta_scan(D.d, ds, r, n->db)) ||
             (rc = delta_finish(D.d, din, D.w, ds, r, n->db, at, n->att, n->ld_att))) return rc;
       }
     }
@@ -601,25 +777,7 @@ static int enqueue_net(LayeredNet* n, const StepRows& r, bool single, const Step
     LinEpi g; g.mode = EPI_GLU; g.h = n->mid; g.ldh = n->ld_mid; g.glu = y.glu;
     if ((rc = launch_lin(y.gateup, at, n->h, n->wp, R, g)) || (rc = launch_lin(y.down, at, n->mid, n->ld_mid, R, res))) return rc;
   }
-  if (n_want > 0) {
-    const void* hs = n->h;
-    LinEpi e; e.y = n->logits; e.ldy = s.vocab; e.scale = s.logit_scale;
-    if (s.rms_final && !want && n_want <= LIN_FEW) {
-      if ((rc = launch_lin_rms(at, n->x, w, s.eps, n_want, RmsLin{s.head, s.rms_final, e, n->h, n->wp}, nullptr))) return rc;
-      hs = nullptr;
-    } else if (s.rms_final) {
-      if (want) hs = n->hw;
-      rms_rows(n, want, n_want, s.rms_final, (void*)hs);
-    } else if (want) {
-      if (at == ACT_T_BF16) hipLaunchKernelGGL(net_gather_kernel<bf16_t>, dim3(n_want), dim3(256), 0, st, (const bf16_t*)n->h, want, (int64_t)n->wp, (bf16_t*)n->hw);
-      else hipLaunchKernelGGL(net_gather_kernel<float>, dim3(n_want), dim3(256), 0, st, (const float*)n->h, want, (int64_t)n->wp, (float*)n->hw);
-      hs = n->hw;
-    }
-    if (hs && (rc = launch_lin(s.head, at, hs, n->wp, n_want, e))) return rc;
-    launch_argmax(n->logits, s.vocab, n_want, n->best, n->am_v, n->am_i);
-  }
-  CAI_HIP(hipGetLastError());
-  return CAI_OK;
+  return enqueue_logits(n, want, n_want);
 }
 
 static StepRows dec_rows(const LayeredNet* n, int R, int reach)
@@ -705,7 +863,7 @@ int net_step(LayeredNet* n, int n_ent, const int32_t* seq, const int32_t* count,
     n->row_of = wrows; n->rows_gathered = false;
   } else {
     // rows, entries, tiles of the prompt attention kernel, wanted rows
-    std::vector<int32_t> tiles, tile0, chunks, chunk0;
+    std::vector<int32_t> tiles, tile0, chunks, chunk0, pages, row0, wide, short_rows;
     bool tall = false, chunked = false;
     int end = 0;
     for (int e = 0; e < n_ent; e++) {
@@ -715,7 +873,15 @@ int net_step(LayeredNet* n, int n_ent, const int32_t* seq, const int32_t* count,
       for (int t = 0; t < count[e]; t += ATTN_TILE) { tiles.push_back(e); tiles.push_back(t); }
       for (int t = 0; t < count[e]; t += DELTA_CHUNK) { chunks.push_back(e); chunks.push_back(t); }
     }
-    const size_t need = (size_t)5 * R + 4 * n_ent + tiles.size() + tile0.size() + chunks.size() + chunk0.size() + W;
+    for (int e = 0, i = 0; n->has_latent && e < n_ent; i += count[e++]) {
+      row0.push_back((int)pages.size() / 2 * PAGE_TOKENS);
+      if (count[e] < LATENT_EXPAND_MIN) { for (int t = 0; t < count[e]; t++) short_rows.push_back(i + t); continue; }
+      for (int p = 0; p * PAGE_TOKENS < n->pool.seq[seq[e]].len + count[e]; p++) { pages.push_back(seq[e]); pages.push_back(p); }
+      for (int t = 0; t < count[e]; t += ATTN_TILE) { wide.push_back(e); wide.push_back(t); }
+    }
+    std::vector<const std::vector<int32_t>*> parts = {&tiles, &tile0, &chunks, &chunk0, &pages, &row0, &wide, &short_rows, &wrows};
+    size_t need = (size_t)5 * R + 4 * n_ent;
+    for (auto* v : parts) need += v->size();
     if (n->rows_cap < need) {
       CAI_HIP(hipStreamSynchronize(st));
       if (n->d_rows) (void)hipFree(n->d_rows);
@@ -725,7 +891,7 @@ int net_step(LayeredNet* n, int n_ent, const int32_t* seq, const int32_t* count,
       CAI_HIP(hipHostMalloc((void**)&n->h_rows, need * 2 * sizeof(int32_t), hipHostMallocDefault));
       n->rows_cap = need * 2;
     }
-    if ((rc = ensure_rows(n, R)) || (rc = ensure_logits(n, std::max(W, 1)))) return rc;
+    if ((rc = ensure_rows(n, R)) || (rc = ensure_logits(n, std::max(W, 1))) || (pages.size() && n->act_t == ACT_T_BF16 && (rc = ensure_flat(n, (int64_t)pages.size() / 2 * PAGE_TOKENS)))) return rc;
     int32_t* hr = n->h_rows;
     int32_t* ent = hr + 5 * R;
     for (int e = 0, i = 0; e < n_ent; e++) {
@@ -734,19 +900,18 @@ int net_step(LayeredNet* n, int n_ent, const int32_t* seq, const int32_t* count,
       for (int t = 0; t < count[e]; t++, i++) { hr[i] = tokens[i]; hr[R + i] = pos0 + t; hr[2 * R + i] = seq[e]; hr[3 * R + i] = r0; hr[4 * R + i] = r0 + count[e] - 1; }
     }
     int32_t* ht = ent + 4 * n_ent;
-    ht = std::copy(tiles.begin(), tiles.end(), ht);
-    ht = std::copy(tile0.begin(), tile0.end(), ht);
-    ht = std::copy(chunks.begin(), chunks.end(), ht);
-    ht = std::copy(chunk0.begin(), chunk0.end(), ht);
-    std::copy(wrows.begin(), wrows.end(), ht);
+    for (auto* v : parts) ht = std::copy(v->begin(), v->end(), ht);
     CAI_HIP(hipMemcpyAsync(n->d_rows, hr, need * sizeof(int32_t), hipMemcpyHostToDevice, st));
     const int32_t* d = n->d_rows;
     const StepRows r{d, d + R, d + 2 * R, d + 3 * R, d + 4 * R, d + 5 * R, R, n_ent, end};
-    const int32_t* dt = d + 5 * R + 4 * n_ent, *dt0 = dt + tiles.size(), *dc = dt0 + tile0.size(), *dc0 = dc + chunks.size();
+    const int32_t* at = d + 5 * R + 4 * n_ent;
+    auto next = [&](const std::vector<int32_t>& v) { const int32_t* p = at; at += v.size(); return p; };
     StepLists lists;
-    lists.tiles = dt; lists.n_tiles = (int)tiles.size() / 2; lists.tile0 = dt0; lists.tall = tall;
-    if (chunked) { lists.chunks = dc; lists.n_chunks = (int)chunks.size() / 2; lists.chunk0 = dc0; }
-    if ((rc = enqueue_net(n, r, false, lists, dc0 + chunk0.size(), W))) return rc;
+    lists.tiles = next(tiles); lists.n_tiles = (int)tiles.size() / 2; lists.tile0 = next(tile0); lists.tall = tall;
+    lists.chunks = next(chunks); lists.n_chunks = (int)chunks.size() / 2; lists.chunk0 = next(chunk0); lists.chunked = chunked;
+    lists.pages = next(pages); lists.n_pages = (int)pages.size() / 2; lists.row0 = next(row0);
+    lists.wide = next(wide); lists.n_wide = (int)wide.size() / 2; lists.short_rows = next(short_rows); lists.n_short = (int)short_rows.size();
+    if ((rc = enqueue_net(n, r, false, lists, next(wrows), W))) return rc;
     for (int k = 0; k < W; k++) n->row_of.push_back(k);
     n->rows_gathered = true;
   }
@@ -844,7 +1009,7 @@ int64_t net_weight_bytes(const LayeredNet* n)
   for (const NetRun& r : n->runs) {
     const NetLayer& y = n->s.layers[r.layer];
     const NetExperts& x = y.experts;
-    b += qb(y.in) + qb(y.delta.out) + qb(y.attn.out) + qb(y.ssd.out) + qb(y.delta.w.a2) + qb(y.delta.w.g2) + qb(y.gateup) + qb(y.down) + qb(y.in2) + 8 * (int64_t)n->s.width * 4;
+    b += qb(y.in) + qb(y.delta.out) + qb(y.latent.uq) + qb(y.latent.up) + qb(y.latent.out) + qb(y.gla.out) + qb(y.attn.out) + qb(y.ssd.out) + qb(y.delta.w.a2) + qb(y.delta.w.g2) + qb(y.gateup) + qb(y.down) + qb(y.in2) + 8 * (int64_t)n->s.width * 4;
     if (r.enter) b += qb(n->s.loop_in);
     if (x.n) b += qb(x.router) + qb(x.s_gateup) + qb(x.s_down) + (qb(x.gateup) + qb(x.down)) / x.n * x.top;   // (of one token)
   }
@@ -877,9 +1042,9 @@ template <typename F> static int snap_walk(LayeredNet* n, int seq, F f)
       off += sz;
     }
   for (auto& d : n->pool.state) {
-    if ((rc = f((char*)(d.S + seq * d.s_elems), (size_t)d.s_elems * 4, off))) return rc;
+    if (d.s_elems && (rc = f((char*)(d.S + seq * d.s_elems), (size_t)d.s_elems * 4, off))) return rc;
     off += d.s_elems * 4;
-    if ((rc = f((char*)(d.hist + seq * d.h_elems), (size_t)d.h_elems * 4, off))) return rc;
+    if (d.h_elems && (rc = f((char*)(d.hist + seq * d.h_elems), (size_t)d.h_elems * 4, off))) return rc;
     off += d.h_elems * 4;
   }
   return CAI_OK;

@@ -14,8 +14,9 @@ __device__ __forceinline__ float glu_pair(int kind, float limit, float g, float 
   return g / (1.0f + expf(-1.702f * g)) * (u + 1.0f);
 }
 
-__device__ __forceinline__ float lin_act(float v, int act)
+__device__ __forceinline__ float lin_act(float v, int act, float limit)
 {
+  if (act == LIN_SOFT_CAP) return limit * tanhf(v / limit);
   if (act == LIN_RELU_SQUARED) { v = fmaxf(v, 0.0f); return v * v; }
   return act_apply(v, act);
 }
@@ -45,10 +46,10 @@ template <typename AT, int MODE> __device__ __forceinline__ void epi_as(const Li
   if constexpr (MODE == EPI_STORE) v *= e.scale;
   if (e.bias) v += e.bias[n];
   float* y = e.y + t * e.ldy + n;
-  if constexpr (MODE == EPI_STORE) *y = lin_act(v, e.act);
+  if constexpr (MODE == EPI_STORE) *y = lin_act(v, e.act, e.limit);
   else if constexpr (MODE == EPI_SPLIT) {
     if (n < e.split) *y = v;
-    else put_act<AT>(e.h, t * e.ldh + n - e.split, lin_act(v, e.act));
+    else put_act<AT>(e.h, t * e.ldh + n - e.split, lin_act(v, e.act, e.limit));
   } else if constexpr (MODE == EPI_JOIN) *y += v * join_factor(e, n, t);
   else {
     float x = (e.fresh ? 0.0f : *y) + dyt(e.post, v, n);
@@ -80,13 +81,13 @@ template <typename AT, int MODE> __device__ __forceinline__ void epi_four(const 
   if constexpr (MODE == EPI_STORE) {
     if (e.act != CAI_ACT_NONE) {
 #pragma unroll
-      for (int q = 0; q < 4; q++) v[q] = lin_act(v[q], e.act);
+      for (int q = 0; q < 4; q++) v[q] = lin_act(v[q], e.act, e.limit);
     }
     *yp = v;
   } else if constexpr (MODE == EPI_SPLIT) {
     if (n < e.split) { *yp = v; return; }
 #pragma unroll
-    for (int q = 0; q < 4; q++) v[q] = lin_act(v[q], e.act);
+    for (int q = 0; q < 4; q++) v[q] = lin_act(v[q], e.act, e.limit);
     put_four<AT>(e.h, t * e.ldh + n - e.split, v);
   } else if constexpr (MODE == EPI_JOIN) {
     const f32x4 g = *reinterpret_cast<const f32x4*>(e.gate + t * e.ldg + n);

@@ -6,7 +6,7 @@
 // 16x16x4 float form of the matrix cores).  What follows the product runs in its epilogue on the 32-bit sums: bias and
 // activation, act(gate) * up of a gated pair, or the residual update with the Dynamic Tanh before and after it - that norm
 // has no statistics, so a sublayer needs no launch besides its products and its mixer - or a result's scaled and gated joining.  The
-// streaming kernel takes the float stream through an RMS norm itself, and runs two products in one launch.  The matrix-core kernel also runs over a
+// streaming kernel takes float rows (the stream's) through an RMS norm itself, and runs two products in one launch.  The matrix-core kernel also runs over a
 // bank of equal matrices with a list of activation rows for each (mixtures of experts).
 #include "cai_lin_epilogue.hpp"
 
@@ -294,7 +294,7 @@ __global__ __launch_bounds__(64 * WM * WN) void gemm_bf16(const uint16_t* __rest
     float scale = 1.0f;
     if constexpr (BANK) {
       const int at = l.order[t];
-      if (MODE == EPI_GLU) scale = l.scale[at]; else t = at;
+      if (MODE == EPI_GLU || MODE == EPI_SPLIT) scale = l.scale[at]; else t = at;
     }
     if constexpr (MODE == EPI_GLU) {
 #pragma unroll
@@ -310,6 +310,18 @@ __global__ __launch_bounds__(64 * WM * WN) void gemm_bf16(const uint16_t* __rest
           for (int q = 0; q < 4; q++) v[q] *= scale;
         }
         put_four<AT>(e.h, (int64_t)t * e.ldh + o, f32x4{v[0], v[1], v[2], v[3]});
+      }
+      continue;
+    }
+    if constexpr (BANK && MODE == EPI_SPLIT) {           // (split 0, rows in whole fours)
+#pragma unroll
+      for (int j = 0; j < TN; j++) {
+        const int n = n0 + wn + j * 16 + fc * 4;
+        if (n >= n_rows) continue;
+        f32x4 v = acc[j][i];
+#pragma unroll
+        for (int q = 0; q < 4; q++) v[q] = lin_act(v[q], e.act, e.limit) * scale;
+        put_four<AT>(e.h, (int64_t)t * e.ldh + n, v);
       }
       continue;
     }
@@ -343,14 +355,14 @@ static void run_bank(const cai_qw_s* w, int mat_rows, const AT* x, int64_t ldx, 
   const int tm = l.max_tiles, tn = (mat_rows + BN - 1) / BN;
 #define GEMM(MODE) case MODE: hipLaunchKernelGGL((gemm_bf16<AT, BM, BN, 2, 2, true, MODE>), dim3(tm * tn), dim3(256), 0, ctx().stream, \
                               (const uint16_t*)w->data, x, mat_rows, (int)w->ld, ldx, 0, tm, tm * tn, e, l); break
-  switch (e.mode) { GEMM(EPI_STORE); GEMM(EPI_GLU); }
+  switch (e.mode) { GEMM(EPI_STORE); GEMM(EPI_GLU); GEMM(EPI_SPLIT); }
 #undef GEMM
 }
 
 int launch_lin_bank(const cai_qw_s* w, int mat_rows, int act_t, const void* x, int64_t ldx, const BankList& l, const LinEpi& e)
 {
   CAI_REQUIRE(w->qtype == CAI_BF16 && mat_rows >= 1 && w->rows % mat_rows == 0 && ldx >= w->ld && l.max_tiles >= 1, "bf16 bank: matrices of %d rows of %lld, activation rows of %lld", mat_rows, (long long)w->rows, (long long)ldx);
-  CAI_REQUIRE(e.mode == EPI_STORE || (e.mode == EPI_GLU && mat_rows % 32 == 0), "bf16 bank: a gated matrix needs whole blocks of 32 rows");
+  CAI_REQUIRE(e.mode == EPI_STORE || (e.mode == EPI_GLU && mat_rows % 32 == 0) || (e.mode == EPI_SPLIT && e.split == 0 && !e.bias && mat_rows % 4 == 0 && e.ldh % 4 == 0), "bf16 bank: a gated matrix needs whole blocks of 32 rows, another one of 4");
   CAI_REQUIRE(l.tile == BANK_TILE || l.tile == BANK_TILE_MAX, "bf16 bank: runs of %d places", l.tile);
   if (act_t == ACT_T_BF16) {
     if (l.tile == BANK_TILE_MAX) run_bank<bf16_t, BANK_TILE_MAX, 128>(w, mat_rows, (const bf16_t*)x, ldx, l, e);
@@ -418,7 +430,7 @@ static int run_lin(const cai_qw_s* w, const AT* x, int64_t ldx, int n_tok, const
   return CAI_OK;
 }
 
-int launch_lin_rms(int act_t, const float* x, int width, float eps, int n_tok, const RmsLin& a, const RmsLin* b)
+int launch_lin_rms(int act_t, const float* x, int64_t ldx, int width, float eps, int n_tok, const RmsLin& a, const RmsLin* b)
 {
   CAI_REQUIRE(n_tok >= 1 && n_tok <= LIN_FEW && a.w->cols == width && (!b || b->w->cols == width), "normed bf16 products: %d rows of %d columns", n_tok, width);
   auto mode_ok = [](const LinEpi& e) { return e.mode == EPI_STORE || e.mode == EPI_SPLIT; };
@@ -433,8 +445,8 @@ int launch_lin_rms(int act_t, const float* x, int width, float eps, int n_tok, c
     if (b->normed) q.ldn = b->ldn;
     blocks += gv_blocks((int)b->w->rows, s, false);
   }
-  if (act_t == ACT_T_BF16) run_gemv_rows<bf16_t, GV_RMS>(n_tok, a.w, x, width, a.e, s, blocks, gv_turns(a.w), q);
-  else run_gemv_rows<float, GV_RMS>(n_tok, a.w, x, width, a.e, s, blocks, gv_turns(a.w), q);
+  if (act_t == ACT_T_BF16) run_gemv_rows<bf16_t, GV_RMS>(n_tok, a.w, x, ldx, a.e, s, blocks, gv_turns(a.w), q);
+  else run_gemv_rows<float, GV_RMS>(n_tok, a.w, x, ldx, a.e, s, blocks, gv_turns(a.w), q);
   CAI_HIP(hipGetLastError());
   return CAI_OK;
 }

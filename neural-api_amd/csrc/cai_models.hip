@@ -182,16 +182,48 @@ struct Builder {
     }
     return stack(parts, width, &order);
   }
+  // matrices of equal shape one after the other, each padded to whole blocks of 16 rows with zeros
+  cai_qw_s* padded_bank(const std::vector<std::string>& names, int rows, int width)
+  {
+    std::vector<std::pair<std::string, int64_t>> parts;
+    std::vector<int> order((size_t)pad_to(rows, 16) * names.size(), -1);
+    for (size_t e = 0; e < names.size(); e++) {
+      parts.push_back({names[e], rows});
+      for (int j = 0; j < rows; j++) order[e * pad_to(rows, 16) + j] = (int)e * rows + j;
+    }
+    return stack(parts, width, &order);
+  }
   // the experts' matrices, one after the other
   void banks(const std::string& pre, int n, int ff, int width, NetExperts& x)
   {
     std::vector<std::string> names; std::vector<std::pair<std::string, int64_t>> down;
     for (int i = 0; i < n; i++) { names.push_back(pre + "e" + std::to_string(i) + "."); down.push_back({names.back() + "down", width}); }
-    x.gateup = gated(names, ff, width);
+    if (x.gated) x.gateup = gated(names, ff, width);
+    else { for (auto& s : names) s += "up"; x.gateup = padded_bank(names, ff, width); }
     x.down = stack(down, ff);
   }
-  // sizes every layered design has, and its list of layers; may_loop: a stretch of layers may run several times
-  const Json* layer_list(const Json& cfg, bool may_loop)
+  // a rotation's rates: turns a position of each pair of the first `dims` dimensions, base^(-2i/dims) radians divided by `linear`.  yarn:
+  // pairs that make less than `slow` turns over `original` positions are divided by `factor`, those that make more than `fast` are not,
+  // with a ramp in between (slow and fast turned into pair numbers, rounded outwards)
+  struct Yarn { double factor, original, fast, slow; };
+  const double* rates(int dims, double base, double linear, const Yarn* y)
+  {
+    std::vector<double> turns((size_t)dims / 2);
+    double lo = 0.0, hi = 0.0;
+    if (y) {
+      auto pair = [&](double t) { return dims * log(y->original / (2.0 * M_PI * t)) / (2.0 * log(base)); };
+      lo = std::max(floor(pair(y->fast)), 0.0); hi = std::min(ceil(pair(y->slow)), dims - 1.0);
+    }
+    for (int i = 0; i < dims / 2; i++) {
+      const double f = pow(base, -2.0 * i / dims) / (2.0 * M_PI) / linear;
+      const double ramp = y ? std::min(std::max((i - lo) / std::max(hi - lo, 0.001), 0.0), 1.0) : 0.0;
+      turns[i] = y ? f / y->factor * ramp + f * (1.0 - ramp) : f;
+    }
+    return dims ? upload(turns) : nullptr;
+  }
+  // sizes every layered design has, and its list of layers; may_loop: a stretch of layers may run several times; tied: the embedding
+  // table is the matrix of the logits too
+  const Json* layer_list(const Json& cfg, bool may_loop, bool tied = false)
   {
     s.width = integer(&cfg, "width", ""); s.vocab = integer(&cfg, "vocab", "", 1, 1 << 28);
     s.eps = number(cfg.get("norm"), "eps", "norm.");
@@ -205,7 +237,7 @@ struct Builder {
     }
     if (rc) return nullptr;
     s.embed = stack({{"embed", s.vocab}}, s.width);
-    s.head = stack({{"head", s.vocab}}, s.width);
+    s.head = tied ? s.embed : stack({{"head", s.vocab}}, s.width);
     return rc ? nullptr : layers;
   }
   std::string word(const Json* o, const char* key) { const Json* v = o ? o->get(key) : nullptr; return v && v->kind == Json::STR ? v->str : std::string(); }
@@ -324,11 +356,7 @@ void block_attention(Builder& b, const Json* c, const std::string& where, const 
   if (b.rc) return;
   if (d.heads % d.kv_heads) { b.fail(where + "heads is not a multiple of " + where + "kv_heads"); return; }
   if (d.rot % 2 || !(base > 0.0f)) { b.fail(where + "rot needs an even number of dims and a base above zero"); return; }
-  if (d.rot) {
-    std::vector<double> turns((size_t)d.rot / 2);
-    for (int i = 0; i < d.rot / 2; i++) turns[i] = pow((double)rot->get("base")->num, -2.0 * i / d.rot) / (2.0 * M_PI);
-    d.turns = b.upload(turns);
-  }
+  d.turns = b.rates(d.rot, rot->get("base")->num, 1.0, nullptr);
   const int qw = d.heads * d.dim, kw = d.kv_heads * d.dim, vw = d.kv_heads * d.vdim, ow = d.heads * d.vdim;
   A.oq = 0; A.ok = qw; A.ov = qw + kw; A.og = qw + kw + vw;
   y.in = b.stack({{pre + "q", qw}, {pre + "k", kw}, {pre + "v", vw}, {pre + "g", ow}}, width);
@@ -506,8 +534,152 @@ void build_gamanex(Builder& b, const Json& cfg)
   }
 }
 
+// ------------------------------------------------------------------------------------------
+// Zenorax: latent attention, attention whose values are its keys, and linear attention with forget gates; mixtures of experts without
+// gates, routed by sigmoids within groups; every sublayer between RMS norms, a convolution over time in front of every mixer, and a
+// weighted sum of the results of all layers so far behind every layer.
+// ------------------------------------------------------------------------------------------
+bool rotation(Builder& b, const Json* rot, const std::string& where, int most, int& dims, double& base)
+{
+  dims = b.integer(rot, "dims", where, 0, most);
+  b.number(rot, "base", where);
+  if (b.rc) return false;
+  base = rot->get("base")->num;
+  if (dims % 2 || !(base > 0.0) || base == 1.0) return b.fail(where + "dims is odd, or " + where + "base no base of powers");
+  return true;
+}
+const Json* present(const Json* o, const char* key) { const Json* v = o ? o->get(key) : nullptr; return v && v->kind != Json::NUL ? v : nullptr; }
+
+void latent_attention(Builder& b, const Json* c, const std::string& where, const std::string& pre, int width, NetLayer& y)
+{
+  NetLatent& L = y.latent; LatentDims& d = L.d;
+  d.heads = b.integer(c, "heads", where, 1, 65534); d.dim = b.integer(c, "dim", where, 1, 256); d.rot_dim = b.integer(c, "rot_dim", where, 0, 256);
+  d.vdim = b.integer(c, "vdim", where, 1, 1024); d.q_rank = b.integer(c, "q_rank", where); d.kv_rank = b.integer(c, "kv_rank", where, 1, 768);
+  d.scale = b.number(c, "scale", where); d.eps = b.s.eps; d.amp = 1.0f;
+  const Json* rot = c ? c->get("rot") : nullptr;
+  double base = 0.0;
+  if (b.rc || !rotation(b, rot, where + "rot.", d.rot_dim, d.rot, base)) return;
+  if (const Json* sc = present(rot, "scaling")) {
+    for (const char* k : {"factor", "original", "fast", "slow"}) b.number(sc, k, where + "rot.scaling.");
+    if (b.rc) return;
+    const Builder::Yarn yarn{sc->get("factor")->num, sc->get("original")->num, sc->get("fast")->num, sc->get("slow")->num};
+    if (!(yarn.factor > 0.0 && yarn.original > 0.0 && yarn.fast > 0.0 && yarn.slow > 0.0)) { b.fail(where + "rot.scaling has a number that is not above zero"); return; }
+    d.turns = b.rates(d.rot, base, 1.0, &yarn);
+    d.amp = (float)(0.1 * log(yarn.factor) + 1.0);
+  } else d.turns = b.rates(d.rot, base, 1.0, nullptr);
+  const int ow = d.heads * d.vdim;
+  L.oq = 0; L.okv = d.q_rank; L.og = L.okv + d.kv_rank + d.rot_dim;
+  y.in = b.stack({{pre + "dq", d.q_rank}, {pre + "dkv", d.kv_rank + d.rot_dim}, {pre + "g", ow}}, width);
+  L.qn = b.vec(pre + "dq.norm", {d.q_rank}); L.kvn = b.vec(pre + "dkv.norm", {d.kv_rank});
+  L.uq = b.stack({{pre + "uq", (int64_t)d.heads * (d.dim + d.rot_dim)}}, d.q_rank);
+  // per head the rows of uk, then those of uv, each padded to eight
+  std::vector<int> order((size_t)d.heads * d.head_e(), -1);
+  for (int h = 0; h < d.heads; h++) {
+    for (int i = 0; i < d.dim; i++) order[(size_t)h * d.head_e() + i] = h * d.dim + i;
+    for (int i = 0; i < d.vdim; i++) order[(size_t)h * d.head_e() + d.dim_e() + i] = d.heads * d.dim + h * d.vdim + i;
+  }
+  L.up = b.stack({{pre + "uk", (int64_t)d.heads * d.dim}, {pre + "uv", ow}}, d.kv_rank, &order);
+  L.out = b.stack({{pre + "o", width}}, ow);
+  AttnDims& a = y.attn.d;                  // (the pages: one row of latent and turned part a token)
+  a.heads = d.heads; a.kv_heads = 1; a.dim = a.dim_p = d.lat_p(); a.window = ATTN_EVERY_KEY;
+}
+
+// Queries and keys are normed behind the rotation; it leaves a head's length as it is, so the norm in front of it, with a gain of ones, is
+// the same.
+void key_value_attention(Builder& b, const Json* c, const std::string& where, const std::string& pre, int width, NetLayer& y)
+{
+  NetAttn& A = y.attn; AttnDims& d = A.d;
+  d.heads = b.integer(c, "heads", where, 1, 65535); d.kv_heads = b.integer(c, "kv_heads", where, 1, 65535);
+  d.dim = b.integer(c, "dim", where, 1, 256); d.vdim = b.integer(c, "vdim", where, 1, 256);
+  d.scale = b.number(c, "scale", where); d.eps = b.s.eps; d.window = ATTN_EVERY_KEY;
+  d.dim_p = pad_to(d.dim, 8); d.vdim_p = pad_to(d.vdim, 8);
+  const Json* rot = c ? c->get("rot") : nullptr;
+  double base = 0.0, linear = 1.0;
+  if (b.rc || !rotation(b, rot, where + "rot.", d.dim, d.rot, base)) return;
+  if (const Json* sc = present(rot, "scaling")) {
+    b.number(sc, "factor", where + "rot.scaling.");
+    if (b.rc) return;
+    linear = sc->get("factor")->num;
+    if (!(linear > 0.0)) { b.fail(where + "rot.scaling.factor is not above zero"); return; }
+  }
+  if (d.heads % d.kv_heads) { b.fail(where + "heads is not a multiple of " + where + "kv_heads"); return; }
+  if (d.vdim != d.dim) { b.fail(where + "vdim is not " + where + "dim, but the values are the keys"); return; }
+  d.turns = b.rates(d.rot, base, linear, nullptr);
+  const int qw = d.heads * d.dim;
+  A.oq = 0; A.ok = A.ov = qw; A.og = -1;
+  y.in = b.stack({{pre + "q", qw}, {pre + "k", (int64_t)d.kv_heads * d.dim}}, width);
+  A.qn = A.kn = b.upload(std::vector<float>(d.dim, 1.0f));
+  d.sink = b.vec(pre + "sink", {d.heads});
+  A.out = b.stack({{pre + "o", width}}, qw);
+}
+
+void forget_gate_attention(Builder& b, const Json* c, const std::string& where, const std::string& pre, int width, NetLayer& y)
+{
+  NetGla& G = y.gla; GlaDims& d = G.d;
+  d.heads = b.integer(c, "heads", where, 1, 65535); d.dim = b.integer(c, "dim", where, 1, 256); d.vdim = b.integer(c, "vdim", where, 1, 256);
+  d.eps = b.s.eps;
+  if (b.rc) return;
+  const int gw = d.heads * d.dim, vw = d.heads * d.vdim;
+  G.oq = 0; G.of = gw; G.ov = 2 * gw;
+  y.in = b.stack({{pre + "q", gw}, {pre + "f", gw}, {pre + "v", vw}}, width);
+  G.w.bias = b.vec(pre + "f.b", {gw}); G.w.lower = b.vec(pre + "lower", {gw}); G.w.norm = b.vec(pre + "norm", {d.vdim});
+  G.out = b.stack({{pre + "o", width}}, vw);
+}
+
+void grouped_experts(Builder& b, const Json* c, const std::string& where, const std::string& pre, int width, NetExperts& x)
+{
+  const Json *r = c->get("router"), *g = r ? r->get("groups") : nullptr;
+  const int n = b.integer(r, "experts", where + "router.", 1, EXPERTS_MAX);
+  x.top = b.integer(r, "top", where + "router.", 1, std::min(n, EXPERTS_TOP)); x.ff = b.integer(c->get("expert"), "ff", where + "expert.");
+  x.groups = b.integer(g, "count", where + "router.groups.", 1, std::min(n, EXPERTS_GROUPS)); x.keep = b.integer(g, "keep", where + "router.groups.", 1, x.groups);
+  if (b.rc) return;
+  if (n % x.groups || x.top > n / x.groups * x.keep) { b.fail(where + "router.groups: " + std::to_string(x.top) + " of " + std::to_string(n) + " experts from " + std::to_string(x.keep) + " of " + std::to_string(x.groups) + " groups"); return; }
+  x.route = ROUTE_SIGMOID; x.gated = false; x.act = LIN_RELU_SQUARED;
+  x.router = b.stack({{pre + "router", n}}, width);
+  x.correction = b.vec(pre + "correction", {n});
+  b.banks(pre, n, x.ff, width, x);
+  x.n = n;
+}
+
+void build_zenorax(Builder& b, const Json& cfg)
+{
+  NetSpec& s = b.s;
+  const Json* layers = b.layer_list(cfg, false, true);
+  if (!layers) return;
+  s.embed_scale = b.number(cfg.get("embedding"), "scale", "embedding."); s.logit_cap = b.number(&cfg, "logit_softcap", "");
+  const int taps = b.integer(cfg.get("canon"), "taps", "canon.", 1, 64);
+  if (!b.rc && !(s.logit_cap > 0.0f)) b.fail("\"logit_softcap\" is not above zero");
+  const int L = (int)layers->arr.size(), w = s.width;
+  s.rms_final = b.vec("final.norm", {w});
+  for (int l = 0; l < L && !b.rc; l++) {
+    const Json& c = layers->arr[l];
+    const std::string p = "l" + std::to_string(l) + ".", where = "layers[" + std::to_string(l) + "].", type = b.word(&c, "type");
+    const Json *mix = c.get("mixer"), *mlp = c.get("mlp");
+    NetLayer y;
+    y.sandwich = true;
+    if (type == "latent_attention") { y.kind = MIX_LATENT; latent_attention(b, mix, where + "mixer.", p + "mix.", w, y); }
+    else if (type == "attention") { y.kind = MIX_ATTN; key_value_attention(b, mix, where + "mixer.", p + "mix.", w, y); }
+    else if (type == "hgrn2") { y.kind = MIX_GLA; forget_gate_attention(b, mix, where + "mixer.", p + "mix.", w, y); }
+    else b.fail("\"" + where + "type\" is not one of latent_attention, attention, hgrn2");
+    if (b.rc) return;
+    y.rms1 = b.vec(p + "norm1", {w}); y.rms1b = b.vec(p + "norm1b", {w}); y.depth = b.vec(p + "dwa", {l + 2});
+    std::vector<float> cw;
+    if (!b.floats(p + "canon1", {w, taps}, cw)) return;
+    std::vector<float> by_tap(cw.size());
+    for (int i = 0; i < w; i++) for (int j = 0; j < taps; j++) by_tap[(size_t)j * w + i] = cw[(size_t)i * taps + j];
+    y.conv.taps = taps; y.conv.w = b.upload(by_tap);
+    if (mlp && mlp->kind == Json::OBJ) {
+      if (b.word(mlp, "kind") != "moe") { b.fail("\"" + where + "mlp.kind\" is not moe"); return; }
+      grouped_experts(b, mlp, where + "mlp.", p + "mlp.", w, y.experts);
+      if (b.rc) return;
+      y.rms2 = b.vec(p + "norm2", {w}); y.rms2b = b.vec(p + "norm2b", {w});
+    } else if (mlp && mlp->kind != Json::NUL) b.fail("\"" + where + "mlp\" is neither an object nor null");
+    s.layers.push_back(y);
+  }
+}
+
 struct Arch { const char* name; void (*build)(Builder&, const Json&); };
-const Arch ARCHS[] = {{"Samanex", build_samanex}, {"Kiruvik", build_kiruvik}, {"Gamanex", build_gamanex}};
+const Arch ARCHS[] = {{"Samanex", build_samanex}, {"Kiruvik", build_kiruvik}, {"Gamanex", build_gamanex}, {"Zenorax", build_zenorax}};
 
 bool is_dir(const char* path) { struct stat sb; return stat(path, &sb) == 0 && S_ISDIR(sb.st_mode); }
 

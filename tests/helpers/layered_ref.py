@@ -296,6 +296,123 @@ def sublayer_gate(w, name, h):
     return sigmoid(linear(w[name], h) + w[name + ".b"])
 
 
+# ---------------------------------------------------------------- mechanisms of Zenorax
+def turn_rates(dims, base, linear=1.0, yarn=None):
+    """radians a position of every pair of a rotation over `dims` dimensions, and what cosine and sine are multiplied by.  linear: all
+    slowed down alike.  yarn: the slow pairs are slowed down by its factor, the fast ones not, a ramp in between."""
+    i = np.arange(dims // 2)
+    f = base ** (-2.0 * i / dims) / linear
+    if not yarn:
+        return f, 1.0
+    pair = lambda turns: dims * np.log(yarn["original"] / (2 * np.pi * turns)) / (2 * np.log(base))
+    lo, hi = max(np.floor(pair(yarn["fast"])), 0), min(np.ceil(pair(yarn["slow"])), dims - 1)
+    ramp = np.clip((i - lo) / max(hi - lo, 0.001), 0, 1)
+    return f / yarn["factor"] * ramp + f * (1 - ramp), 0.1 * np.log(yarn["factor"]) + 1
+
+
+def rotate_pairs(x, rates, amp=1.0, neighbours=False, pos0=0):
+    """x [T, heads, d]: pair i turns by position * rates[i] and grows by amp; a pair is dimensions 2i and 2i + 1 (neighbours) or i and
+    i + len(rates); dimensions past 2 len(rates) stay"""
+    n = len(rates)
+    out = x.copy()
+    for i in range(n):
+        a = ((pos0 + np.arange(x.shape[0])) * rates[i])[:, None]
+        p, q = (2 * i, 2 * i + 1) if neighbours else (i, i + n)
+        u, v = x[:, :, p], x[:, :, q]
+        out[:, :, p] = amp * (u * np.cos(a) - v * np.sin(a))
+        out[:, :, q] = amp * (v * np.cos(a) + u * np.sin(a))
+    return out
+
+
+def causal_attention(q, k, v, scale, sink=None):
+    """q [T, H, d], k [T, G, d], v [T, G, dv]; soft-max over every key up to the query.  sink [H]: the denominator holds one more term,
+    the exponential of a number per head that has no key"""
+    T, H, _ = q.shape
+    G = k.shape[1]
+    seen = np.arange(T)[None, :] <= np.arange(T)[:, None]
+    out = np.zeros((T, H, v.shape[2]))
+    for h in range(H):
+        g = h // (H // G)
+        s = np.where(seen, (q[:, h] @ k[:, g].T) * scale, -np.inf)
+        m = s.max(-1, keepdims=True) if sink is None else np.maximum(s.max(-1, keepdims=True), sink[h])
+        e = np.exp(s - m)
+        den = e.sum(-1, keepdims=True) + (0.0 if sink is None else np.exp(sink[h] - m))
+        out[:, h] = (e / den) @ v[:, g]
+    return out
+
+
+def latent_attention_mixer(w, pre, c, h, eps):
+    """queries through a latent of their own; keys (the part that does not turn) and values made from one shared latent; one key part that
+    turns, shared by all heads; a sigmoid gate on the heads"""
+    T, H, d, dr, dv, r = h.shape[0], c["heads"], c["dim"], c["rot_dim"], c["vdim"], c["kv_rank"]
+    rates, amp = turn_rates(c["rot"]["dims"], c["rot"]["base"], yarn=c["rot"].get("scaling"))
+    q = linear(w[pre + "uq"], rms_norm(linear(w[pre + "dq"], h), eps) * w[pre + "dq.norm"]).reshape(T, H, d + dr)
+    kv = linear(w[pre + "dkv"], h)
+    lat = rms_norm(kv[:, :r], eps) * w[pre + "dkv.norm"]
+    turned = rotate_pairs(kv[:, None, r:], rates, amp, True)
+    q = np.concatenate([q[:, :, :d], rotate_pairs(q[:, :, d:], rates, amp, True)], axis=2)
+    k = np.concatenate([linear(w[pre + "uk"], lat).reshape(T, H, d), np.repeat(turned, H, axis=1)], axis=2)
+    o = causal_attention(q, k, linear(w[pre + "uv"], lat).reshape(T, H, dv), c["scale"]).reshape(T, H * dv)
+    return linear(w[pre + "o"], o * sigmoid(linear(w[pre + "g"], h)))
+
+
+def key_value_attention_mixer(w, pre, c, h, eps):
+    """the values are the keys as projected; queries and keys turn, then are normed per head without a gain"""
+    T, H, G, d = h.shape[0], c["heads"], c["kv_heads"], c["dim"]
+    scaling = c["rot"].get("scaling")
+    rates, _ = turn_rates(c["rot"]["dims"], c["rot"]["base"], linear=scaling["factor"] if scaling else 1.0)
+    q, k = linear(w[pre + "q"], h).reshape(T, H, d), linear(w[pre + "k"], h).reshape(T, G, d)
+    o = causal_attention(rms_norm(rotate_pairs(q, rates), eps), rms_norm(rotate_pairs(k, rates), eps), k, c["scale"], w[pre + "sink"])
+    return linear(w[pre + "o"], o.reshape(T, H * d))
+
+
+def forget_gate_recurrence(q, f, v):
+    """q, f [T, H, d]; v [T, H, dv].  S [H, d, dv] starts at zero: its rows are forgotten by f, what f forgets is written, q reads"""
+    T, H, d = q.shape
+    S = np.zeros((H, d, v.shape[2]))
+    out = np.zeros(v.shape)
+    for t in range(T):
+        for i in range(H):
+            S[i] = f[t, i][:, None] * S[i] + np.outer(1.0 - f[t, i], v[t, i])
+            out[t, i] = S[i].T @ q[t, i]
+    return out
+
+
+def forget_gate_mixer(w, pre, c, h, eps):
+    T, H, d, dv = h.shape[0], c["heads"], c["dim"], c["vdim"]
+    q, v = silu(linear(w[pre + "q"], h)).reshape(T, H, d), linear(w[pre + "v"], h).reshape(T, H, dv)
+    low = w[pre + "lower"]
+    f = (low + (1.0 - low) * sigmoid(linear(w[pre + "f"], h) + w[pre + "f.b"])).reshape(T, H, d)
+    o = rms_norm(forget_gate_recurrence(q, f, v), eps) * w[pre + "norm"]
+    return linear(w[pre + "o"], o.reshape(T, H * dv))
+
+
+def route_groups(z, correction, top, count, keep):
+    """[T, experts] weights, zero where not chosen: sigmoid scores; with the correction added, the `keep` groups whose two best add up to
+    most, then the `top` best of these groups; weighted by the scores alone"""
+    s = sigmoid(z)
+    n = z.shape[1]
+    out = np.zeros_like(s)
+    for t in range(z.shape[0]):
+        c = (s[t] + correction).reshape(count, n // count)
+        best = np.argsort(-np.sort(c, axis=1)[:, -2:].sum(1), kind="stable")[:keep]
+        masked = np.full(c.shape, -np.inf)
+        masked[best] = c[best]
+        chosen = np.argsort(-masked.reshape(-1), kind="stable")[:top]
+        out[t, chosen] = s[t, chosen]
+    return out
+
+
+def grouped_expert_mixture(w, pre, c, h):
+    r = c["router"]
+    wt = route_groups(linear(w[pre + "router"], h), w[pre + "correction"], r["top"], r["groups"]["count"], r["groups"]["keep"])
+    return sum(wt[:, e:e + 1] * squared_relu_mlp(w, pre + "e%d." % e, h) for e in range(r["experts"]))
+
+
+def soft_cap(z, cap):
+    return cap * np.tanh(z / cap)
+
+
 # ---------------------------------------------------------------- the models
 def run_order(cfg):
     """(layer, first layer of a repeated pass) for every layer run"""
@@ -313,6 +430,8 @@ def forward(cfg, w, tokens, layers_out=None):
         return kiruvik_forward(cfg, w, tokens, layers_out)
     if cfg["architecture"] == "Gamanex":
         return gamanex_forward(cfg, w, tokens, layers_out)
+    if cfg["architecture"] == "Zenorax":
+        return zenorax_forward(cfg, w, tokens, layers_out)
     eps = cfg["norm"]["eps"]
     norm = lambda name, x: dynamic_tanh(x, w[name + ".alpha"], w[name], w[name + ".b"])
     x = w["embed"][np.asarray(tokens)]
@@ -372,3 +491,25 @@ def gamanex_forward(cfg, w, tokens, layers_out=None):
         if layers_out is not None:
             layers_out.append(x.copy())
     return linear(w["head"], rms_norm(x, eps) * w["final.norm"]) * cfg["logit_scale"]
+
+
+ZENORAX_MIXERS = dict(latent_attention=latent_attention_mixer, attention=key_value_attention_mixer, hgrn2=forget_gate_mixer)
+
+
+def zenorax_forward(cfg, w, tokens, layers_out=None):
+    eps = cfg["norm"]["eps"]
+    norm = lambda name, z: rms_norm(z, eps) * w[name]
+    x = w["embed"][np.asarray(tokens)] * cfg["embedding"]["scale"]
+    kept = [x]
+    for i, L in enumerate(cfg["layers"]):
+        p = "l%d." % i
+        h = norm(p + "norm1", x)
+        h = h + causal_conv(h, w[p + "canon1"])
+        x = x + norm(p + "norm1b", ZENORAX_MIXERS[L["type"]](w, p + "mix.", L["mixer"], h, eps))
+        if L.get("mlp"):
+            x = x + norm(p + "norm2b", grouped_expert_mixture(w, p + "mlp.", L["mlp"], norm(p + "norm2", x)))
+        kept.append(x)
+        x = sum(a * z for a, z in zip(w[p + "dwa"], kept))
+        if layers_out is not None:
+            layers_out.append(x.copy())
+    return soft_cap(linear(w["embed"], norm("final.norm", x)), cfg["logit_softcap"])
