@@ -290,12 +290,10 @@ __global__ __launch_bounds__(256) void latent_merge_kernel(const LatentDims d, c
   __syncthreads();
   const int l16 = tid & 15, per = (d.vdim + gridDim.z - 1) / gridDim.z, v1 = min(d.vdim, (int)(blockIdx.z + 1) * per);
   const uint16_t* m0 = up + ((int64_t)h * d.head_e() + d.dim_e()) * ldu;
-#pragma unroll 2
   for (int v0 = blockIdx.z * per; v0 < v1; v0 += 16) {
     const int v = v0 + (tid >> 4);
     const uint16_t* mr = m0 + (int64_t)min(v, v1 - 1) * ldu;
     float s = 0.0f;
-#pragma unroll 4
     for (int c = l16 * 8; c < lc; c += 128) {
       float x[8];
       load_eight(reinterpret_cast<const bf16_t*>(mr + c), x);

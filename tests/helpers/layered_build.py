@@ -177,12 +177,93 @@ def steady_experts(cfg):
     return edit
 
 
+# ---------------------------------------------------------------- Zenorax
+def lat(heads=4, dim=20, rot_dim=12, vdim=28, kv_rank=36, q_rank=44, scale=0.2, rot=None, base=300.0, yarn=(4.0, 400, 8.0, 1.0)):
+    """yarn: factor, original, fast, slow, or None"""
+    r = dict(base=base, dims=rot_dim if rot is None else rot)
+    if yarn:
+        r["scaling"] = dict(zip(("factor", "original", "fast", "slow"), yarn))
+    return dict(heads=heads, dim=dim, rot_dim=rot_dim, vdim=vdim, kv_rank=kv_rank, q_rank=q_rank, scale=scale, rot=r)
+
+
+def keyval(heads=4, kv_heads=2, dim=24, scale=0.3, rot=16, base=200.0, factor=1.7):
+    r = dict(base=base, dims=rot)
+    if factor:
+        r["scaling"] = dict(factor=factor)
+    return dict(heads=heads, kv_heads=kv_heads, dim=dim, vdim=dim, scale=scale, rot=r)
+
+
+def forget(heads=3, dim=20, vdim=28):
+    return dict(heads=heads, dim=dim, vdim=vdim)
+
+
+def zmoe(experts=8, top=3, ff=20, count=4, keep=2):
+    return dict(kind="moe", expert=dict(ff=ff), router=dict(experts=experts, top=top, groups=dict(count=count, keep=keep)))
+
+
+def zlayer(mixer, mlp=None):
+    return dict(type="latent_attention" if "kv_rank" in mixer else "attention" if "rot" in mixer else "hgrn2", mixer=mixer, mlp=mlp)
+
+
+def zconfig(layers, width=72, vocab=131, eps=1e-5, taps=3, scale=1.9, cap=9.0):
+    return dict(architecture="Zenorax", width=width, vocab=vocab, layers=layers, norm=dict(eps=eps), canon=dict(taps=taps), embedding=dict(scale=scale), logit_softcap=cap)
+
+
+def steady_groups(w):
+    """as steady_choice, for a choice of groups in front of it: no two pairs of corrections have the same sum"""
+    for n in w:
+        if n.endswith(".correction"):
+            w[n] = 4.0 * 2.0 ** np.random.default_rng(len(w[n])).permutation(len(w[n]))
+
+
+def zenorax_weights(cfg, seed=0):
+    rng = np.random.default_rng(seed)
+    w, width = {}, cfg["width"]
+
+    def lin(name, rows, cols, gain=1.0):
+        w[name] = rng.standard_normal((rows, cols)) * gain / np.sqrt(cols)
+
+    def vec(name, shape, mean=0.0, spread=0.2):
+        w[name] = mean + spread * rng.standard_normal(shape)
+
+    vec("embed", (cfg["vocab"], width), 0.0, 0.7)
+    vec("final.norm", width, 1.0)
+    for i, L in enumerate(cfg["layers"]):
+        p, m, f = "l%d." % i, L["mixer"], L["mlp"]
+        a = p + "mix."
+        for n in ("norm1", "norm1b") + (("norm2", "norm2b") if f else ()):
+            vec(p + n, width, 1.0)
+        vec(p + "canon1", (width, cfg["canon"]["taps"]), 0.1, 0.4)
+        vec(p + "dwa", i + 2, 0.2, 0.3); w[p + "dwa"][-1] += 0.8
+        if L["type"] == "latent_attention":
+            H = m["heads"]
+            lin(a + "dq", m["q_rank"], width); vec(a + "dq.norm", m["q_rank"], 1.2)
+            lin(a + "uq", H * (m["dim"] + m["rot_dim"]), m["q_rank"], 1.3)
+            lin(a + "dkv", m["kv_rank"] + m["rot_dim"], width, 1.4); vec(a + "dkv.norm", m["kv_rank"], 1.1)
+            lin(a + "uk", H * m["dim"], m["kv_rank"], 1.3); lin(a + "uv", H * m["vdim"], m["kv_rank"])
+            lin(a + "g", H * m["vdim"], width, 1.5); lin(a + "o", width, H * m["vdim"])
+        elif L["type"] == "attention":
+            lin(a + "q", m["heads"] * m["dim"], width); lin(a + "k", m["kv_heads"] * m["dim"], width)
+            vec(a + "sink", m["heads"], 1.0, 1.0); lin(a + "o", width, m["heads"] * m["dim"])
+        else:
+            n = m["heads"] * m["dim"]
+            lin(a + "q", n, width, 1.5); lin(a + "f", n, width, 1.5); lin(a + "v", m["heads"] * m["vdim"], width)
+            vec(a + "f.b", n, 1.0, 1.0); w[a + "lower"] = rng.uniform(0.0, 0.9, n); vec(a + "norm", m["vdim"], 1.0); lin(a + "o", width, m["heads"] * m["vdim"])
+        if f:
+            lin(p + "mlp.router", f["router"]["experts"], width, 2.0); vec(p + "mlp.correction", f["router"]["experts"], 0.0, 0.2)
+            for e in range(f["router"]["experts"]):
+                lin(p + "mlp.e%d.up" % e, f["expert"]["ff"], width, 1.5); lin(p + "mlp.e%d.down" % e, width, f["expert"]["ff"])
+    return w
+
+
 def weights(cfg, seed=0, rank_a=7, rank_g=11):
     """name -> float array before rounding"""
     if cfg["architecture"] == "Kiruvik":
         return kiruvik_weights(cfg, seed)
     if cfg["architecture"] == "Gamanex":
         return gamanex_weights(cfg, seed)
+    if cfg["architecture"] == "Zenorax":
+        return zenorax_weights(cfg, seed)
     rng = np.random.default_rng(seed)
     w, width = {}, cfg["width"]
 

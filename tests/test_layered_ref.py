@@ -198,6 +198,91 @@ def test_gamanex_oracle_is_sensitive_to_what_it_checks():
     assert np.abs(R.forward(own, ow, tok) - base).max() > 1e-2
 
 
+# ---------------------------------------------------------------- Zenorax's mechanisms
+def test_turn_rates_slow_down_the_slow_pairs():
+    f, amp = R.turn_rates(16, 100.0)
+    assert np.allclose(f, 100.0 ** (-np.arange(8) / 8)) and amp == 1.0
+    assert np.allclose(R.turn_rates(16, 100.0, linear=2.5)[0], f / 2.5)
+    g, amp = R.turn_rates(16, 100.0, yarn=dict(factor=4.0, original=200, fast=10.0, slow=2.0))
+    turns = 200 * f / (2 * np.pi)                       # over the original length
+    assert np.allclose(g[turns > 14], f[turns > 14]) and np.allclose(g[turns < 1.5], f[turns < 1.5] / 4) and np.isclose(amp, 1 + 0.1 * np.log(4))
+    between = (g < f * 0.999) & (g > f / 4 * 1.001)
+    assert between.any() and not between[0] and not between[-1] and np.all(np.diff(g / f) <= 1e-12)
+
+
+def test_rotation_of_neighbours_and_halves():
+    rng = np.random.default_rng(4)
+    x, y, rates = rng.standard_normal((1, 1, 12)), rng.standard_normal((1, 1, 12)), np.array([1.0, 0.3, 0.05])
+    for near in (False, True):
+        rot = lambda z, p: R.rotate_pairs(z, rates, 1.5, near, p)
+        assert np.allclose(rot(x, 0)[..., :6], 1.5 * x[..., :6]) and np.allclose(rot(x, 9)[..., 6:], x[..., 6:])
+        assert np.isclose((rot(x, 7) * rot(y, 3)).sum(), (rot(x, 104) * rot(y, 100)).sum())
+        z = np.zeros((1, 1, 12)); z[0, 0, 2 if near else 1] = 1.0
+        assert np.allclose(rot(z, 5)[0, 0, [2, 3] if near else [1, 4]], 1.5 * np.array([np.cos(1.5), np.sin(1.5)]))
+    assert np.allclose(R.rotate_pairs(x, R.turn_rates(8, 50.0)[0], pos0=7), R.rotate_half(x, 50.0, 8, 7))
+
+
+def test_sink_takes_its_share_of_the_weights():
+    rng = np.random.default_rng(8)
+    T, sink = 6, np.array([2.0, -3.0, 40.0, -60.0])
+    q, k, v = rng.standard_normal((T, 4, 6)), rng.standard_normal((T, 2, 6)), rng.standard_normal((T, 2, 5))
+    o, bare = R.causal_attention(q, k, v, 0.3, sink), R.causal_attention(q, k, v, 0.3)
+    for i in range(T):
+        for h in range(4):
+            s = np.exp(0.3 * k[:i + 1, h // 2] @ q[i, h])
+            assert np.allclose(o[i, h], s @ v[:i + 1, h // 2] / (s.sum() + np.exp(sink[h]))) and np.allclose(bare[i, h], s @ v[:i + 1, h // 2] / s.sum())
+
+
+def test_forget_gates_write_what_they_forget():
+    rng = np.random.default_rng(9)
+    T, d, dv = 6, 4, 3
+    q, f, v = rng.standard_normal((T, 1, d)), rng.uniform(0, 1, (T, 1, d)), rng.standard_normal((T, 1, dv))
+    o = R.forget_gate_recurrence(q, f, v)
+    for t in range(T):
+        want = sum(q[t, 0, c] * f[s + 1:t + 1, 0, c].prod() * (1 - f[s, 0, c]) * v[s, 0] for s in range(t + 1) for c in range(d))
+        assert np.allclose(o[t, 0], want)
+    one = np.repeat(v[:1], T, axis=0)                   # a constant input: every row of the state tends to it
+    assert np.allclose(R.forget_gate_recurrence(q, 0 * f, one), q.sum(-1, keepdims=True) * one)
+
+
+def test_routing_within_the_best_groups():
+    z = np.array([[2.0, -1.0, 1.5, 1.4, 0.0, 0.1]])
+    s = 1 / (1 + np.exp(-z[0]))
+    pick = lambda *e: [[s[i] if i in e else 0.0 for i in range(6)]]
+    none = np.zeros(6)
+    assert np.allclose(R.route_groups(z, none, 2, 3, 1), pick(2, 3))           # two good ones beat the best with a bad neighbour
+    assert np.allclose(R.route_groups(z, none, 2, 3, 3), pick(0, 2)) and np.allclose(R.route_groups(z, none, 2, 1, 1), pick(0, 2))
+    assert np.allclose(R.route_groups(z, none, 3, 3, 2), pick(0, 2, 3))
+    assert np.allclose(R.route_groups(z, np.array([0, 0, -1.0, -1.0, 0, 0]), 1, 3, 1), pick(0))
+    low = np.full(6, -5.0); low[4] = -4.0; low[5] = -4.9                       # negative choice scores: left out is less than any of them
+    assert np.allclose(R.route_groups(z, low, 2, 3, 1), pick(4, 5))
+    assert np.allclose(R.route_groups(z, none, 2, 6, 2), pick(0, 2))           # groups of one
+    assert np.allclose(R.soft_cap(np.array([0.01, 1e3, -1e3]), 5.0), [0.01, 5.0, -5.0], atol=1e-6)
+
+
+def test_zenorax_oracle_is_sensitive_to_what_it_checks():
+    """every constant and every small tensor, a far token: each moves the logits well beyond the tests' tolerances"""
+    cfg = B.zconfig([B.zlayer(B.lat(), B.zmoe()), B.zlayer(B.keyval(), B.zmoe(keep=3)), B.zlayer(B.forget(), B.zmoe(top=2)), B.zlayer(B.lat(heads=2, yarn=None))])
+    w = {n: B.to_bf16(a)[1].reshape(np.shape(a)) for n, a in B.weights(cfg, 5).items()}
+    tok = np.random.default_rng(6).integers(0, cfg["vocab"], 40)
+    base = R.forward(cfg, w, tok)
+    at = lambda c, i: c["layers"][i]
+    mix = lambda i, **kw: lambda c: at(c, i)["mixer"].update(**kw)
+    rot = lambda i, **kw: lambda c: at(c, i)["mixer"]["rot"].update(**kw)
+    yarn = lambda **kw: lambda c: at(c, 0)["mixer"]["rot"]["scaling"].update(**kw)
+    for change in (mix(0, scale=0.25), mix(1, scale=0.4), rot(0, base=100.0), rot(1, base=20.0), rot(1, dims=8), yarn(factor=8.0), yarn(original=1200), yarn(fast=20.0), yarn(slow=4.0),
+                   lambda c: at(c, 1)["mixer"]["rot"]["scaling"].update(factor=3.0), lambda c: at(c, 1)["mixer"]["rot"].pop("scaling"), lambda c: c["norm"].update(eps=0.1),
+                   lambda c: c["embedding"].update(scale=1.0), lambda c: c.update(logit_softcap=7.0), lambda c: at(c, 0)["mlp"]["router"].update(top=2),
+                   lambda c: at(c, 0)["mlp"]["router"]["groups"].update(keep=1 + 2), lambda c: at(c, 0)["mlp"]["router"]["groups"].update(count=2, keep=1)):
+        other = json.loads(json.dumps(cfg)); change(other)
+        assert np.abs(R.forward(other, w, tok) - base).max() > 1e-2
+    for name in w:
+        if ".mlp.e" not in name:
+            other = dict(w, **{name: w[name].copy()}); other[name][::2] *= 0.3          # (every second row: a norm takes a common factor back)
+            assert np.abs(R.forward(cfg, other, tok) - base).max() > 1e-2, name
+    assert np.abs(R.forward(cfg, w, tok[1:])[-1] - base[-1]).max() > 1e-2
+
+
 @pytest.mark.parametrize("text, reason", [("{", "malformed"), ("[]", ""), ('{"architecture": "Nobody"}', "Samanex"), ("{}", "Samanex"),
                                           ('{"architecture": "Samanex"} x', "after"), ('{"architecture": "\\ud800"}', "malformed")])
 def test_registry_refuses_what_it_does_not_know(tmp_path, text, reason):
