@@ -315,12 +315,12 @@ def layered_bench(cai, synth, torch, only, size, what, prompt_len, batch):
     for name, z in LAYERED_SIZES.items():
         if size and size != name:
             continue
-        for kind in ("gamanex", "kiruvik_attention", "kiruvik", "samanex", "llama"):
+        for kind in ("zenorax", "gamanex", "kiruvik_attention", "kiruvik", "samanex", "llama"):
             if only and only != kind:
                 continue
             rng = np.random.default_rng(1)
             if kind != "llama":
-                cfg = (synth.gamanex_config(**z) if kind == "gamanex" else synth.layered_config(window=1024, **z) if kind == "samanex" else
+                cfg = (synth.zenorax_config(**z) if kind == "zenorax" else synth.gamanex_config(**z) if kind == "gamanex" else synth.layered_config(window=1024, **z) if kind == "samanex" else
                        synth.kiruvik_config(block=4096, every=1, **z) if kind == "kiruvik_attention" else synth.kiruvik_config(block=1024, **z))
                 with tempfile.TemporaryDirectory() as td:
                     synth.write_layered_folder(td, cfg, 1)
@@ -396,8 +396,8 @@ def main():
     ap.add_argument("--gemm-sweep", action="store_true", help="isolated prompt-product sweep: Q8_0 / Q4_0 / Q4_K / Q5_K / Q6_K, four shapes, 64..2048 tokens (cai_qgemm, device pointers)")
     ap.add_argument("--step-timeline", action="store_true", help="device-side timeline of one captured batch-1 step (cai_decoder_timeline): per kernel class the gap to the previous launch, dispatch skew, staging, loop and tail times from wall-clock stamps taken inside the kernels")
     ap.add_argument("--copy-calibration", action="store_true", help="only run the 1 GiB device copy kernel 5 times (reference for traffic counters)")
-    ap.add_argument("--layered", action="store_true", help="layered decoders (Gamanex, Kiruvik once with attention in every layer over all keys and once as it is, Samanex; bfloat16) at two sizes with random weights beside the Llama-type decoder of the same width, feed-forward, heads and depth (Q8_0 body, half-precision cache): prompt and decode throughput, one JSON line per measurement")
-    ap.add_argument("--layered-only", choices=["", "gamanex", "kiruvik_attention", "kiruvik", "samanex", "llama"], default="", help="with --layered: measure one of them (for profiles)")
+    ap.add_argument("--layered", action="store_true", help="layered decoders (Zenorax, Gamanex, Kiruvik once with attention in every layer over all keys and once as it is, Samanex; bfloat16) at two sizes with random weights beside the Llama-type decoder of the same width, feed-forward, heads and depth (Q8_0 body, half-precision cache): prompt and decode throughput, one JSON line per measurement")
+    ap.add_argument("--layered-only", choices=["", "zenorax", "gamanex", "kiruvik_attention", "kiruvik", "samanex", "llama"], default="", help="with --layered: measure one of them (for profiles)")
     ap.add_argument("--layered-size", choices=["", "w2048", "w4096"], default="", help="with --layered: measure one size")
     ap.add_argument("--layered-what", choices=["", "prompt", "decode"], default="", help="with --layered: prompts only (of --prompt tokens, if given) or decoding only (of --batch sequences)")
     args = ap.parse_args()

@@ -594,7 +594,7 @@ int attn_paged_prompt(const AttnDims& d, const KvView& kv, const AttnIn& in, con
   const dim3 grid(n_tiles, d.heads), blk(256);
 #define PROMPT_S(K, V, S, F) hipLaunchKernelGGL((attn_prompt_paged_kernel<K, V, S, F>), grid, blk, 0, ctx().stream, d, kv, f, in, (const bf16_t*)qbuf, r, tiles, (bf16_t*)out, ldo)
 #define PROMPT_V(K, P) do { if (d.vdim <= 64) P(K, 4); else if (d.vdim <= 128) P(K, 8); else P(K, 16); } while (0)
-#define PROMPT_K(P) do { if (d.dim <= 64) PROMPT_V(2, P); else if (d.dim <= 128) PROMPT_V(4, P); else PROMPT_V(8, P); } while (0)
+#define PROMPT_K(P) do { if (d.dim <= 64) PROMPT_V(2, P); else if (d.dim <= 128) PROMPT_V(4, P); else if (d.dim <= 192) PROMPT_V(6, P); else PROMPT_V(8, P); } while (0)
 #define PAGED(K, V) do { if (d.sigmoid) PROMPT_S(K, V, true, false); else PROMPT_S(K, V, false, false); } while (0)
   const FlatKv f;
   PROMPT_K(PAGED);

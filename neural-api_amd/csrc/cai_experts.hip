@@ -42,7 +42,22 @@ __device__ __forceinline__ float route_sigmoid(float z)
   const float s = expf(z); return s / (1.0f + s);
 }
 
-// One row's experts, by one wave: lane k < top ends with the k-th choice and its weight.  Equal choice scores: the lower index.
+// how many of the first n lanes hold more, or as much in front of this lane
+__device__ __forceinline__ int lane_rank(float v, int n, int lane)
+{
+  int rank = 0;
+  for (int j0 = 0; j0 < n; j0 += 8)
+#pragma unroll
+    for (int u = 0; u < 8; u++) {          // (n is 64 at most; lanes past it do not count)
+      const int j = j0 + u;
+      const float o = __builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, v), j));
+      rank += j < n && (o > v || (o == v && j < lane));
+    }
+  return rank;
+}
+
+// One row's experts (SIG: by ROUTE_SIGMOID), by one wave: lane k < top ends with the k-th choice and its weight.  Equal choice scores: the lower index.
+template <bool SIG>
 __device__ __forceinline__ void route_row(const float* z, const Routing& q, const int lane, int& expert, float& weight)
 {
   const float* correction = q.correction;
@@ -51,42 +66,46 @@ __device__ __forceinline__ void route_row(const float* z, const Routing& q, cons
   float s[PER], c[PER], m = -INFINITY, sum = 0.0f;
 #pragma unroll
   for (int i = 0; i < PER; i++) { const int e = lane + 64 * i; s[i] = e < n ? z[e] : -INFINITY; c[i] = e < n && correction ? correction[e] : 0.0f; m = fmaxf(m, s[i]); }
-  const bool sigmoid = q.route == ROUTE_SIGMOID;
   uint64_t kept = ~0ull;                   // groups that take part
   const int per_group = q.per_group;
-  if (sigmoid) {
+  if constexpr (SIG) {
 #pragma unroll
     for (int i = 0; i < PER; i++) if (64 * i < n) s[i] = route_sigmoid(s[i]);
-    if (q.keep < q.groups) {               // a lane a group: its two largest choice scores
+    if (q.keep < q.groups) {               // a lane a group: its two largest choice scores, and how many groups are better
       float a = -INFINITY, b = -INFINITY;
-      if (lane < q.groups)
+      auto meet = [&](float v) { b = fmaxf(b, fminf(a, v)); a = fmaxf(a, v); };
+      if (n <= 64) {
+        const float v = s[0] + c[0];
+        for (int i0 = 0; i0 < per_group; i0 += 4)
+#pragma unroll
+          for (int i = i0; i < i0 + 4; i++) { const float o = __shfl(v, (lane * per_group + i) & 63); meet(i < per_group ? o : -INFINITY); }
+      } else if (lane < q.groups)
 #pragma unroll 4
         for (int i = 0; i < per_group; i++) {
           const int e = lane * per_group + i;
-          const float v = route_sigmoid(z[e]) + (correction ? correction[e] : 0.0f);
-          b = fmaxf(b, fminf(a, v)); a = fmaxf(a, v);
+          meet(route_sigmoid(z[e]) + (correction ? correction[e] : 0.0f));
         }
-      float score = lane >= q.groups ? -INFINITY : per_group > 1 ? a + b : a;
-      kept = 0;
-      for (int k = 0; k < q.keep; k++) {
-        const float most = wave_max(score);
-        const int g = wave_min(score == most && !(kept >> lane & 1) ? lane : 63);
-        kept |= 1ull << g;
-        if (lane == g) score = -INFINITY;
-      }
+      const float score = per_group > 1 ? a + b : a;
+      kept = __ballot(lane < q.groups && lane_rank(score, q.groups, lane) < q.keep);
     }
   } else m = wave_max(m);
-  if (q.route == ROUTE_ALL) {
+  if (!SIG && q.route == ROUTE_ALL) {
 #pragma unroll
     for (int i = 0; i < PER; i++) if (64 * i < n) { s[i] = expf(s[i] - m); sum += s[i]; }
     sum = lanes_total(sum);
   }
 #pragma unroll
   for (int i = 0; i < PER; i++) {
-    if (64 * i < n && q.route == ROUTE_ALL) s[i] /= sum;
+    if (!SIG && 64 * i < n && q.route == ROUTE_ALL) s[i] /= sum;
     bool in = lane + 64 * i < n;
-    if (64 * i < n && sigmoid) in = in && (kept >> ((lane + 64 * i) / per_group & 63) & 1);
+    if (SIG && 64 * i < n) in = in && (kept >> ((lane + 64 * i) / per_group & 63) & 1);
     c[i] = in ? s[i] + c[i] : -INFINITY;
+  }
+  if (SIG && n <= 64) {                    // a lane an expert: each goes to the lane of its rank
+    const int to = (lane < n ? lane_rank(c[0], n, lane) : lane) * 4;
+    expert = min(max(__builtin_amdgcn_ds_permute(to, lane), 0), n - 1);
+    weight = __builtin_bit_cast(float, __builtin_amdgcn_ds_permute(to, __builtin_bit_cast(int, s[0]))) * q.scale;
+    return;
   }
   expert = 0; weight = 0.0f;
   float total = 0.0f;
@@ -97,13 +116,13 @@ __device__ __forceinline__ void route_row(const float* z, const Routing& q, cons
     const float most = wave_max(bv);
     be = wave_min(bv == most ? be : n - 1);
     bs = __builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, bs), be & 63));
-    if (q.route == ROUTE_AMONG) bs = expf(bs - m);       // (m is the largest logit, the first choice)
+    if (!SIG && q.route == ROUTE_AMONG) bs = expf(bs - m);       // (m is the largest logit, the first choice)
     total += bs;
     if (lane == k) { expert = be; weight = bs; }
 #pragma unroll
     for (int i = 0; i < PER; i++) if (lane + 64 * i == be) c[i] = -INFINITY;
   }
-  weight = sigmoid ? weight * q.scale : weight / (total + 1e-20f) * q.scale;
+  weight = SIG ? weight * q.scale : weight / (total + 1e-20f) * q.scale;
 }
 
 // eight activations times eight weights
@@ -133,6 +152,7 @@ struct FewGateUp {
   const uint16_t *w, *ws; int ldw, gu_rows; Routing q; int ff, ff_s; float limit, limit_s; int glu, glu_s; int mid_p, active; int n_rows; int act;
 };
 
+template <bool SIG>
 __global__ __launch_bounds__(64 * EXPERTS_FEW) void experts_few_kernel(const float* z, const int64_t ldz, const Routing q, const int n_rows, float* wgt, FewEntry* list, int32_t* n_list)
 {
   const int n = q.n, top = q.top;
@@ -143,7 +163,7 @@ __global__ __launch_bounds__(64 * EXPERTS_FEW) void experts_few_kernel(const flo
   __syncthreads();
   if (wave < n_rows) {
     int e; float w;
-    route_row(z + wave * ldz, q, lane, e, w);
+    route_row<SIG>(z + wave * ldz, q, lane, e, w);
     if (lane < top) { wgt[wave * top + lane] = w; slot_of[wave][e] = (int8_t)lane; }
   }
   __syncthreads();
@@ -163,7 +183,7 @@ __global__ __launch_bounds__(64 * EXPERTS_FEW) void experts_few_kernel(const flo
   if (tid == 0) *n_list = total;
 }
 
-template <typename AT, int NB, bool GATED>
+template <typename AT, int NB, bool GATED, bool SIG>       // (SIG counts for one row only)
 __global__ __launch_bounds__(256) void experts_gateup_kernel(const FewGateUp p, const float* z, const float* wgt, const FewEntry* list, const int32_t* n_list, const AT* h, const int64_t ldh, int32_t* sel, AT* mid)
 {
   constexpr int UNROLL = NB == 1 ? 2 : 1;
@@ -178,7 +198,7 @@ __global__ __launch_bounds__(256) void experts_gateup_kernel(const FewGateUp p, 
   if (!shared) {
     if constexpr (NB == 1) {
       int e; float wt;
-      route_row(z, p.q, lane, e, wt);
+      route_row<SIG>(z, p.q, lane, e, wt);
       if (j0 == 0 && lane == entry) sel[entry] = e;
       W = p.w + (int64_t)__shfl(e, entry) * p.gu_rows * p.ldw; weight = __shfl(wt, entry);
     } else {
@@ -311,7 +331,7 @@ __global__ __launch_bounds__(256) void experts_out_kernel(const uint16_t* w, con
 // Router scores of 16 rows and their choices: sixteen waves share the width, 16 ET experts at a time; the matrix cores multiply as in the
 // other products (bfloat16, or exactly widened weights in 32-bit), the sums meet in LDS.
 constexpr int ROUTE_WAVES = 16;
-template <typename AT, int ET>
+template <typename AT, int ET, bool SIG>
 __global__ __launch_bounds__(64 * ROUTE_WAVES) void experts_route_kernel(const uint16_t* W, const int ldw, const AT* h, const int64_t ldh, const Routing q, const int n_rows, int32_t* sel, float* wgt)
 {
   const int n = q.n, top = q.top;
@@ -367,19 +387,20 @@ __global__ __launch_bounds__(64 * ROUTE_WAVES) void experts_route_kernel(const u
   __syncthreads();
   for (int r = wave; r < 16 && r0 + r < n_rows; r += ROUTE_WAVES) {
     int e; float w;
-    route_row(z + r * n, q, lane, e, w);
+    route_row<SIG>(z + r * n, q, lane, e, w);
     if (lane < top) { sel[(int64_t)(r0 + r) * top + lane] = e; wgt[(int64_t)(r0 + r) * top + lane] = w; }
   }
 }
 
 // choices of rows whose logits are there already, a wave a row
+template <bool SIG>
 __global__ __launch_bounds__(256) void experts_pick_kernel(const float* z, const int64_t ldz, const Routing q, const int n_rows, int32_t* sel, float* wgt)
 {
   const int lane = threadIdx.x & 63;
   const int64_t row = blockIdx.x * 4 + (threadIdx.x >> 6);
   if (row >= n_rows) return;
   int e; float w;
-  route_row(z + row * ldz, q, lane, e, w);
+  route_row<SIG>(z + row * ldz, q, lane, e, w);
   if (lane < q.top) { sel[row * q.top + lane] = e; wgt[row * q.top + lane] = w; }
 }
 
@@ -435,10 +456,14 @@ static void run_few(const NetExperts& x, int width, const AT* h, int64_t ldh, in
   const FewGateUp p{(const uint16_t*)x.gateup->data, sg, (int)x.gateup->ld, x.gu_rows(), routing(x), x.ff, x.ff_shared,
                     x.limit, x.limit_shared, x.glu, x.glu_shared, x.mid_p(), x.active(), n_rows, x.act};
   FewEntry* list = (FewEntry*)b.few;
-  if (NB > 1) hipLaunchKernelGGL(experts_few_kernel, dim3(1), dim3(64 * EXPERTS_FEW), 0, st, z, ldz, p.q, n_rows, b.wgt, list, b.n_tiles);
+  const bool sig = x.route == ROUTE_SIGMOID;
+  if (NB > 1) hipLaunchKernelGGL(sig ? experts_few_kernel<true> : experts_few_kernel<false>, dim3(1), dim3(64 * EXPERTS_FEW), 0, st, z, ldz, p.q, n_rows, b.wgt, list, b.n_tiles);
   const int entries = NB == 1 ? x.top : std::min(x.n, n_rows * x.top);
-  if (x.gated) hipLaunchKernelGGL((experts_gateup_kernel<AT, NB, true>), dim3((std::max(x.ff, x.ff_shared) + 7) / 8, entries + (sg ? 1 : 0)), dim3(256), 0, st, p, z, b.wgt, list, b.n_tiles, h, ldh, b.sel, (AT*)b.mid);
-  else hipLaunchKernelGGL((experts_gateup_kernel<AT, NB, false>), dim3((x.ff + 15) / 16, entries), dim3(256), 0, st, p, z, b.wgt, list, b.n_tiles, h, ldh, b.sel, (AT*)b.mid);
+  const dim3 mids(x.gated ? (std::max(x.ff, x.ff_shared) + 7) / 8 : (x.ff + 15) / 16, entries + (sg ? 1 : 0));
+#define GATEUP(G, S) hipLaunchKernelGGL((experts_gateup_kernel<AT, NB, G, S>), mids, dim3(256), 0, st, p, z, b.wgt, list, b.n_tiles, h, ldh, b.sel, (AT*)b.mid)
+  if (NB == 1 && sig) { if (x.gated) GATEUP(true, NB == 1); else GATEUP(false, NB == 1); }
+  else if (x.gated) GATEUP(true, false); else GATEUP(false, false);
+#undef GATEUP
   BesideArg o;
   if (beside) { o.w = (const uint16_t*)beside->w->data; o.x = beside->x; o.ld = (int)beside->w->ld; o.ldx = beside->ldx; o.e = beside->e; }
   const int lds = x.s_down ? (int)x.s_down->ld : 0;
@@ -474,10 +499,12 @@ static int run(const NetExperts& x, int width, int act_t, const AT* h, int64_t l
     CAI_HIP(hipGetLastError());
     return CAI_OK;
   }
-#define ROUTE(ET) hipLaunchKernelGGL((experts_route_kernel<AT, ET>), dim3((n_rows + 15) / 16), dim3(64 * ROUTE_WAVES), (ROUTE_WAVES * 16 * ET * 16 + 16 * x.n) * sizeof(float), st, \
-                                     (const uint16_t*)x.router->data, (int)x.router->ld, h, ldh, routing(x), n_rows, b.sel, b.wgt)
-  if (z) hipLaunchKernelGGL(experts_pick_kernel, dim3((n_rows + 3) / 4), dim3(256), 0, st, z, ldz, routing(x), n_rows, b.sel, b.wgt);
-  else if (x.n <= 16) ROUTE(1); else ROUTE(2);
+  const bool sig = x.route == ROUTE_SIGMOID;
+#define ROUTE(ET, S) hipLaunchKernelGGL((experts_route_kernel<AT, ET, S>), dim3((n_rows + 15) / 16), dim3(64 * ROUTE_WAVES), (ROUTE_WAVES * 16 * ET * 16 + 16 * x.n) * sizeof(float), st, \
+                                        (const uint16_t*)x.router->data, (int)x.router->ld, h, ldh, routing(x), n_rows, b.sel, b.wgt)
+  if (z) hipLaunchKernelGGL(sig ? experts_pick_kernel<true> : experts_pick_kernel<false>, dim3((n_rows + 3) / 4), dim3(256), 0, st, z, ldz, routing(x), n_rows, b.sel, b.wgt);
+  else if (x.n <= 16) { if (sig) ROUTE(1, true); else ROUTE(1, false); }
+  else if (sig) ROUTE(2, true); else ROUTE(2, false);
 #undef ROUTE
   const int tile = n_rows * x.top >= x.n * 96 ? BANK_TILE_MAX : BANK_TILE;       // (by the mean number of rows of an expert)
   hipLaunchKernelGGL(experts_order_kernel, dim3(1), dim3(1024), 0, st, b.sel, x.n, n_rows * x.top, tile, b.order, b.tiles, b.n_tiles);

@@ -392,7 +392,8 @@ static int run_latent_rows(const LatentDims& d, const KvView& kv, const LatentIn
     const float* qa = qabs + (int64_t)z0 * d.heads * lp;
     if (ht == 4) hipLaunchKernelGGL((latent_rows_kernel<T, 4>), dim3(ns, (d.heads + 3) / 4, m), dim3(256), (size_t)4 * lp * 4, st, d, kv, q, list, qa, part);
     else hipLaunchKernelGGL((latent_rows_kernel<T, 8>), dim3(ns, (d.heads + 7) / 8, m), dim3(256), (size_t)8 * lp * 4, st, d, kv, q, list, qa, part);
-    const int split = d.heads * m >= ctx().n_cu / 2 ? 1 : d.vdim > 64 ? 4 : 2;
+    int split = 1;                         // parts of a head's values, until every CU has two work-groups
+    while (split < 8 && d.heads * m * split < 2 * ctx().n_cu && d.vdim / (2 * split) >= 16) split *= 2;
     hipLaunchKernelGGL(latent_merge_kernel<T>, dim3(d.heads, m, split), dim3(256), (size_t)pad_to(d.lat_c(), 128) * 4, st, d, a, (const uint16_t*)up->data, (int)up->ld, q, list, ns, part, o, ldo);
   }
   CAI_HIP(hipGetLastError());

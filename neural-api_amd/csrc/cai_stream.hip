@@ -64,34 +64,45 @@ __global__ __launch_bounds__(THREADS) void stream_kernel(const StreamArg a, cons
 #pragma unroll
     for (int u = 0; u < PER; u++) if (col(u) < w) *reinterpret_cast<T*>(ring + col(u)) = x[u] * inv * at(s.keep_gain + col(u));
   }
-  if (s.y) {
-    T y[PER];
-    float q = 0.0f;
+  // everything the row needs is requested before the first meeting of the work-group
+  T y[PER], past[PER], next[PER], looked[PER];           // past: of the average; looked: what the convolution sees of earlier inputs
+  const int taps = s.conv.taps;
+  const bool conv = SINGLE && s.conv.w;
+  const int pos = conv ? r.pos[row] : 0;
+  float* ring = conv ? s.ring + r.slot[row] * s.ring_elems : nullptr;
+  float q = 0.0f;
 #pragma unroll
-    for (int u = 0; u < PER; u++) {
-      const int c = col(u) < w ? col(u) : 0;
+  for (int u = 0; u < PER; u++) {
+    const int c = col(u) < w ? col(u) : 0;
+    y[u] = past[u] = next[u] = looked[u] = T{};
+    if (s.y) {
       const float* p = s.y + row * s.parts * w + c;
       y[u] = at(p);
 #pragma unroll 4
       for (int k = 1; k < s.parts; k++) y[u] += at(p + (int64_t)k * w);
-      if (col(u) < w) q += X::square(y[u]);
     }
+    if (s.kept && s.avg) {
+      const float* k = s.kept + row * w + c;
+#pragma unroll 4
+      for (int j = 0; j < s.n_kept; j++) past[u] += at(k + j * s.kept_stride) * s.avg[j];
+    }
+    if (s.next) next[u] = at(s.next + c);
+    if (conv)
+      for (int j = 1; j < taps && j <= pos; j++) looked[u] += at(ring + (int64_t)((pos - j) % taps) * w + c) * at(s.conv.w + (int64_t)(taps - 1 - j) * w + c);
+  }
+  if (s.y) {
+    T post[PER];
+#pragma unroll
+    for (int u = 0; u < PER; u++) { post[u] = at(s.post + (col(u) < w ? col(u) : 0)); if (col(u) < w) q += X::square(y[u]); }
     const float inv = 1.0f / sqrtf(group_total<THREADS>(q, red[0]) / (float)w + s.eps);
 #pragma unroll
-    for (int u = 0; u < PER; u++) x[u] += y[u] * inv * at(s.post + (col(u) < w ? col(u) : 0));
+    for (int u = 0; u < PER; u++) x[u] += y[u] * inv * post[u];
   }
   if (s.kept) {
 #pragma unroll
     for (int u = 0; u < PER; u++) {
-      const int c = col(u) < w ? col(u) : 0;
-      const float* k = s.kept + row * w + c;
-      if (col(u) < w) *reinterpret_cast<T*>(s.kept + s.n_kept * s.kept_stride + row * w + c) = x[u];
-      if (s.avg) {
-        T m = x[u] * s.avg[s.n_kept];
-#pragma unroll 4
-        for (int j = 0; j < s.n_kept; j++) m += at(k + j * s.kept_stride) * s.avg[j];
-        x[u] = m;
-      }
+      if (col(u) < w) *reinterpret_cast<T*>(s.kept + s.n_kept * s.kept_stride + row * w + col(u)) = x[u];
+      if (s.avg) x[u] = past[u] + x[u] * s.avg[s.n_kept];
     }
   }
   if (s.y || a.e || s.kept) {
@@ -99,7 +110,7 @@ __global__ __launch_bounds__(THREADS) void stream_kernel(const StreamArg a, cons
     for (int u = 0; u < PER; u++) if (col(u) < w) *reinterpret_cast<T*>(xr + col(u)) = x[u];
   }
   if (!s.next) return;
-  float q = 0.0f;
+  q = 0.0f;
 #pragma unroll
   for (int u = 0; u < PER; u++) if (col(u) < w) q += X::square(x[u]);
   const float inv = 1.0f / sqrtf(group_total<THREADS>(q, red[1]) / (float)w + s.eps);
@@ -107,17 +118,14 @@ __global__ __launch_bounds__(THREADS) void stream_kernel(const StreamArg a, cons
     if (tid == 0) s.inv[row] = inv;
     return;
   }
-  const int taps = s.conv.taps, pos = s.conv.w ? r.pos[row] : 0;
-  float* ring = s.conv.w ? s.ring + r.slot[row] * s.ring_elems : nullptr;
 #pragma unroll
   for (int u = 0; u < PER; u++) {
     const int c = col(u);
     if (c >= w) continue;
-    const T n = x[u] * inv * at(s.next + c);
+    const T n = x[u] * inv * next[u];
     T h = n;
-    if (SINGLE && s.conv.w) {
-      h += n * at(s.conv.w + (int64_t)(taps - 1) * w + c);
-      for (int j = 1; j < taps && j <= pos; j++) h += at(ring + (int64_t)((pos - j) % taps) * w + c) * at(s.conv.w + (int64_t)(taps - 1 - j) * w + c);
+    if (conv) {
+      h += n * at(s.conv.w + (int64_t)(taps - 1) * w + c) + looked[u];
       *reinterpret_cast<T*>(ring + (int64_t)(pos % taps) * w + c) = n;
     }
     X::template put<AT>(s.h, row * s.ldh + c, h);

@@ -243,12 +243,27 @@ def gamanex_config(width, ff, heads, kv_heads, dim, n_layers, vocab, experts=32,
     return dict(architecture="Gamanex", width=width, vocab=vocab, layers=layers, norm=dict(eps=1e-6), logit_scale=0.5)
 
 
+def zenorax_config(width, ff, heads, kv_heads, dim, n_layers, vocab, experts=32, top=8, taps=4):
+    """A Zenorax configuration of real-model proportions: latent attention, attention with keys as values and forget-gate layers in turn,
+    each with a mixture of `top` of `experts` experts (of as many active weights as a gated feed-forward of width `ff`)."""
+    lat = dict(heads=heads, dim=dim, rot_dim=dim // 2, vdim=dim, kv_rank=4 * dim, q_rank=width * 3 // 8, scale=(1.5 * dim) ** -0.5,
+               rot=dict(base=1e4, dims=dim // 2, scaling=dict(factor=8.0, original=4096, fast=32.0, slow=1.0)))
+    att = dict(heads=heads, kv_heads=max(1, kv_heads // 2), dim=dim, vdim=dim, scale=dim ** -0.5, rot=dict(base=1e4, dims=dim, scaling=dict(factor=2.0)))
+    rec = dict(heads=width // dim, dim=dim, vdim=dim)
+    moe = dict(kind="moe", expert=dict(ff=ff * 3 // (2 * top)), router=dict(experts=experts, top=top, groups=dict(count=8, keep=4)))
+    kinds = (("latent_attention", lat), ("attention", att), ("hgrn2", rec))
+    layers = [dict(type=kinds[i % 3][0], mixer=kinds[i % 3][1], mlp=moe) for i in range(n_layers)]
+    return dict(architecture="Zenorax", width=width, vocab=vocab, layers=layers, norm=dict(eps=1e-6), canon=dict(taps=taps), embedding=dict(scale=width ** 0.5), logit_softcap=30.0)
+
+
 def layered_shapes(cfg, rank=128):
     """name -> (shape, standard deviation, mean) of every tensor of a layered model"""
     if cfg["architecture"] == "Kiruvik":
         return kiruvik_shapes(cfg)
     if cfg["architecture"] == "Gamanex":
         return gamanex_shapes(cfg)
+    if cfg["architecture"] == "Zenorax":
+        return zenorax_shapes(cfg)
     w, out = cfg["width"], {}
 
     def lin(name, rows, cols):
@@ -359,12 +374,47 @@ def gamanex_shapes(cfg):
     return out
 
 
+def zenorax_shapes(cfg):
+    w, out = cfg["width"], {}
+
+    def lin(name, rows, cols):
+        out[name] = ((rows, cols), cols ** -0.5, 0.0)
+
+    def vec(name, n, std, mean):
+        out[name] = ((n,), std, mean)
+
+    out["embed"] = ((cfg["vocab"], w), w ** -0.5, 0.0)
+    vec("final.norm", w, 0.1, 1.0)
+    for i, L in enumerate(cfg["layers"]):
+        p, m, f = "l%d." % i, L["mixer"], L["mlp"]
+        a = p + "mix."
+        for n in ("norm1", "norm1b") + (("norm2", "norm2b") if f else ()):
+            vec(p + n, w, 0.1, 1.0)
+        out[p + "canon1"] = ((w, cfg["canon"]["taps"]), 0.2, 0.1); vec(p + "dwa", i + 2, 0.05, 1.0 / (i + 2))
+        if L["type"] == "latent_attention":
+            lin(a + "dq", m["q_rank"], w); vec(a + "dq.norm", m["q_rank"], 0.1, 1.0); lin(a + "uq", m["heads"] * (m["dim"] + m["rot_dim"]), m["q_rank"])
+            lin(a + "dkv", m["kv_rank"] + m["rot_dim"], w); vec(a + "dkv.norm", m["kv_rank"], 0.1, 1.0)
+            lin(a + "uk", m["heads"] * m["dim"], m["kv_rank"]); lin(a + "uv", m["heads"] * m["vdim"], m["kv_rank"])
+            lin(a + "g", m["heads"] * m["vdim"], w); lin(a + "o", w, m["heads"] * m["vdim"])
+        elif L["type"] == "attention":
+            lin(a + "q", m["heads"] * m["dim"], w); lin(a + "k", m["kv_heads"] * m["dim"], w); vec(a + "sink", m["heads"], 0.5, 0.0); lin(a + "o", w, m["heads"] * m["dim"])
+        else:
+            n = m["heads"] * m["dim"]
+            lin(a + "q", n, w); lin(a + "f", n, w); lin(a + "v", m["heads"] * m["vdim"], w)
+            vec(a + "f.b", n, 1.0, 2.0); vec(a + "lower", n, 0.05, 0.5); vec(a + "norm", m["vdim"], 0.1, 1.0); lin(a + "o", w, m["heads"] * m["vdim"])
+        if f:
+            lin(p + "mlp.router", f["router"]["experts"], w); vec(p + "mlp.correction", f["router"]["experts"], 0.01, 0.0)
+            for e in range(f["router"]["experts"]):
+                lin(p + "mlp.e%d.up" % e, f["expert"]["ff"], w); lin(p + "mlp.e%d.down" % e, w, f["expert"]["ff"])
+    return out
+
+
 def layered_active_weights(cfg):
     """linear weights one token of a prompt meets, the vocabulary left out"""
     import numpy as np
     total = 0
     for name, (shape, _, _) in layered_shapes(cfg).items():
-        if len(shape) != 2 or name in ("embed", "head") or name.endswith("conv"):
+        if len(shape) != 2 or name in ("embed", "head") or name.endswith(("conv", "canon1")):
             continue
         n = int(np.prod(shape))
         part = name.split(".")
