@@ -20,6 +20,20 @@ __device__ __forceinline__ float lin_act(float v, int act, float limit)
   if (act == LIN_RELU_SQUARED) { v = fmaxf(v, 0.0f); return v * v; }
   return act_apply(v, act);
 }
+// four of them; the kinds the products of a layer have cost no more than a branch, and one loop holds the others (64 copies of those in a
+// kernel's epilogue, each visited once, would wait for instructions longer than the product takes)
+__device__ __forceinline__ f32x4 lin_act_four(f32x4 v, int act, float limit)
+{
+  if (act == CAI_ACT_NONE) return v;
+  if (act == LIN_RELU_SQUARED) {
+#pragma unroll
+    for (int q = 0; q < 4; q++) { const float p = fmaxf(v[q], 0.0f); v[q] = p * p; }
+    return v;
+  }
+#pragma unroll 1
+  for (int q = 0; q < 4; q++) v = f32x4{v[1], v[2], v[3], lin_act(v[0], act, limit)};
+  return v;
+}
 // factor of a sublayer's result before it joins the stream
 __device__ __forceinline__ float join_factor(const LinEpi& e, int n, int64_t t)
 {
@@ -79,16 +93,10 @@ template <typename AT, int MODE> __device__ __forceinline__ void epi_four(const 
   if (e.bias) v += f32x4{e.bias[n], e.bias[n + 1], e.bias[n + 2], e.bias[n + 3]};
   f32x4* yp = reinterpret_cast<f32x4*>(e.y + t * e.ldy + n);
   if constexpr (MODE == EPI_STORE) {
-    if (e.act != CAI_ACT_NONE) {
-#pragma unroll
-      for (int q = 0; q < 4; q++) v[q] = lin_act(v[q], e.act, e.limit);
-    }
-    *yp = v;
+    *yp = lin_act_four(v, e.act, e.limit);
   } else if constexpr (MODE == EPI_SPLIT) {
     if (n < e.split) { *yp = v; return; }
-#pragma unroll
-    for (int q = 0; q < 4; q++) v[q] = lin_act(v[q], e.act, e.limit);
-    put_four<AT>(e.h, t * e.ldh + n - e.split, v);
+    put_four<AT>(e.h, t * e.ldh + n - e.split, lin_act_four(v, e.act, e.limit));
   } else if constexpr (MODE == EPI_JOIN) {
     const f32x4 g = *reinterpret_cast<const f32x4*>(e.gate + t * e.ldg + n);
     f32x4 x = *yp;

@@ -318,10 +318,7 @@ __global__ __launch_bounds__(64 * WM * WN) void gemm_bf16(const uint16_t* __rest
       for (int j = 0; j < TN; j++) {
         const int n = n0 + wn + j * 16 + fc * 4;
         if (n >= n_rows) continue;
-        f32x4 v = acc[j][i];
-#pragma unroll
-        for (int q = 0; q < 4; q++) v[q] = lin_act(v[q], e.act, e.limit) * scale;
-        put_four<AT>(e.h, (int64_t)t * e.ldh + n, v);
+        put_four<AT>(e.h, (int64_t)t * e.ldh + n, lin_act_four(acc[j][i], e.act, e.limit) * scale);
       }
       continue;
     }
