@@ -395,7 +395,7 @@ int cai_gguf_load_qw(cai_gguf_t g, const char* name, const char* bias_name, cai_
  * is the identity). */
 int cai_decoder_load_gguf(const char* path, int max_ctx, int max_batch, int kv_dtype, cai_decoder_t* out);
 /* Model registry: `path` is a folder with config.json and model.safetensors, loaded by the builder registered under the
- * configuration's "architecture" (Samanex, Kiruvik, Gamanex), or a GGUF file (cai_decoder_load_gguf).  max_tokens is the size of the cache pool:
+ * configuration's "architecture" (Samanex, Kiruvik, Gamanex, Zenorax), or a GGUF file (cai_decoder_load_gguf).  max_tokens is the size of the cache pool:
  * the tokens all live sequences may hold together, each count rounded up to whole pages of 64 (a GGUF decoder keeps max_tokens
  * rows for every sequence); max_seq the sequences (state slots).  dtype: CAI_DTYPE_BF16 or CAI_DTYPE_F32. */
 int cai_decoder_load(const char* path, int max_tokens, int max_seq, int dtype, cai_decoder_t* out);
